@@ -1,0 +1,325 @@
+// Attention over the paged latent cache (gfx950): every head's keys and values are linear images of one cached row per
+// token, [c (R, padded to Rp) | rotated key part (padded to rp)], so with the up-projections folded into the query and
+// applied to the output the cache is read once for all heads: score = q_abs . c + q_rot . k_rot, out = sum p c.
+//
+// latent_attn_kernel (bf16): workgroup = (token, split of the keys, 16 heads), 4 waves. KT-key tiles of the cache rows
+// arrive by LDS-DMA into two buffers (16-byte chunks swizzled by the key on the DMA source); each wave forms S^T of 16
+// keys (A = cache rows, B = the queries, held in registers), the waves exchange row maxima and the bf16 weights through
+// LDS, and each wave owns a quarter of the output columns: O^T += C^T P^T with C^T fragments from transposed LDS reads
+// of the same tile. Softmax in base 2, all of it f32.
+// latent_attn_f32_kernel: the f32 form, one workgroup per (token, head).
+#include "../kernels/lds_dma.h"
+
+namespace nls_latent {
+using nls_dma::glds16;
+using nls_dma::lds_addr;
+
+typedef short s16x4 __attribute__((ext_vector_type(4)));
+typedef short s16x8 __attribute__((ext_vector_type(8)));
+
+struct LA {
+  const void* q;            // [T][H][Dp]
+  const void* cache;        // [slots][Dp]
+  void* out;                // [T][H][Rp]
+  float* part_o;            // [T][H][ns][Rp]
+  float* part_ml;           // [T][H][ns][2]
+  const int* bt;            // block tables
+  const int* tok_seq;
+  const int* ctx_len;       // keys of each token (0: padded row)
+  int bts, bs, T, H, ns, Rp, rp;
+  float scale;
+};
+
+DEVI void bar_lgkm() {
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  __builtin_amdgcn_s_barrier();
+  asm volatile("" ::: "memory");
+}
+
+constexpr int NBT = 1024;    // block-table entries of the split kept in LDS
+
+template <int NT, int RT, int KT>
+__global__ __launch_bounds__(256, 1) void latent_attn_kernel(LA p) {
+  constexpr int Rp = 64 * NT, Dp = Rp + 64 * RT;
+  constexpr int CPR = Dp / 8;                  // 16-byte chunks per row
+  constexpr int TB = KT * Dp * 2;              // bytes per tile
+  constexpr int ND = TB / 4096;                // DMA instructions per wave per tile
+  constexpr int NK = Dp / 32;                  // k-steps of a score
+  constexpr int PS = KT + 8;                   // P row stride
+  static_assert(TB % 4096 == 0, "tile");
+  extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+  __bf16* P = reinterpret_cast<__bf16*>(lds + 2 * TB);                 // [16][PS]
+  float* mx = reinterpret_cast<float*>(lds + 2 * TB + 16 * PS * 2);    // [4][16]
+  int* btl = reinterpret_cast<int*>(mx + 64);                          // [NBT]
+
+  const int HB = (p.H + 15) >> 4;
+  const int ts = ((int)blockIdx.x / (8 * HB)) * 8 + (blockIdx.x & 7);
+  const int hb = ((int)blockIdx.x >> 3) % HB;
+  if (ts >= p.T * p.ns) return;
+  const int t = ts / p.ns, split = ts % p.ns;
+  const int ctx = p.ctx_len[t];
+  const int chunk = ((ctx + p.ns - 1) / p.ns + KT - 1) / KT * KT;
+  const int k0 = split * chunk, k1 = min(ctx, k0 + chunk);
+  const int lane = threadIdx.x & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int r = lane & 15, g = lane >> 4;
+  const int head = hb * 16 + r;
+  const __bf16* cache = reinterpret_cast<const __bf16*>(p.cache);
+  const int* bt = p.bt + (size_t)p.tok_seq[t] * p.bts;
+
+  f32x4 o[NT];
+#pragma unroll
+  for (int c = 0; c < NT; ++c) o[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m = -INFINITY, l = 0.f;
+
+  if (k0 < k1) {
+    const int b0 = k0 / p.bs, nb = (k1 - 1) / p.bs - b0 + 1;
+    for (int i = threadIdx.x; i < min(nb, NBT); i += 256) btl[i] = bt[b0 + i];
+    u32x4 qf[NK];
+    const __bf16* qr = reinterpret_cast<const __bf16*>(p.q) + ((size_t)t * p.H + min(head, p.H - 1)) * Dp;
+#pragma unroll
+    for (int kk = 0; kk < NK; ++kk) qf[kk] = ld16(qr + kk * 32 + 8 * g);
+    __syncthreads();
+    const float sl2 = p.scale * 1.4426950408889634f;
+    const uint32_t base = __builtin_amdgcn_readfirstlane(lds_addr(lds));
+    auto dma = [&](int j) __attribute__((always_inline)) {
+      const uint32_t dst = base + (uint32_t)(j & 1) * TB + (uint32_t)(ND * wave) * 1024u;
+#pragma unroll
+      for (int i = 0; i < ND; ++i) {
+        const int ci = (ND * wave + i) * 64 + lane;
+        const int row = ci / CPR, pc = ci - row * CPR;
+        const int key = min(k0 + j * KT + row, k1 - 1);
+        const int bi = key / p.bs - b0;
+        const int blk = bi < NBT ? btl[bi] : bt[b0 + bi];
+        glds16(cache + ((size_t)blk * p.bs + key % p.bs) * Dp + (pc ^ (row & 7)) * 8, dst + i * 1024);
+      }
+    };
+    const int nt = (k1 - k0 + KT - 1) / KT;
+    dma(0);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    bar_lgkm();
+    for (int j = 0; j < nt; ++j) {
+      const uint8_t* cb = lds + (j & 1) * TB;
+      if (j + 1 < nt) dma(j + 1);              // that buffer was last read in tile j - 1
+      f32x4 s = f32x4{-INFINITY, -INFINITY, -INFINITY, -INFINITY};
+      float tm = -INFINITY;
+      if (KT == 64 || wave < KT / 16) {
+        s = f32x4{0.f, 0.f, 0.f, 0.f};
+        const int row = 16 * wave + r;
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk) {
+          const bf16x8 a = *reinterpret_cast<const bf16x8*>(cb + row * (2 * Dp) + (((4 * kk + g) ^ (row & 7)) << 4));
+          s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, __builtin_bit_cast(bf16x8, qf[kk]), s, 0, 0, 0);
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          s[i] = k0 + j * KT + 16 * wave + 4 * g + i < k1 ? s[i] * sl2 : -INFINITY;
+          tm = fmaxf(tm, s[i]);
+        }
+        tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+        tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+      }
+      if (g == 0) mx[wave * 16 + r] = tm;
+      bar_lgkm();
+      const float mn = fmaxf(fmaxf(fmaxf(mx[r], mx[16 + r]), fmaxf(mx[32 + r], mx[48 + r])), m);
+      const float alpha = m == -INFINITY ? 0.f : exp2f(m - mn);
+      if (KT == 64 || wave < KT / 16) {
+        typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+        bf4 pb;
+        float ps = 0.f;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float e = s[i] == -INFINITY ? 0.f : exp2f(s[i] - mn);
+          ps += e;
+          pb[i] = (__bf16)e;
+        }
+        l = l * alpha + ps;                    // this lane's keys; lanes and waves are summed at the end
+        *reinterpret_cast<bf4*>(P + r * PS + 16 * wave + 4 * g) = pb;
+      }
+      m = mn;
+      bar_lgkm();
+      const int qq = r >> 2, pp = r & 3;
+#pragma unroll
+      for (int u = 0; u < KT / 32; ++u) {
+        const uint2 p0 = *reinterpret_cast<const uint2*>(P + r * PS + 32 * u + 4 * g);
+        const uint2 p1 = *reinterpret_cast<const uint2*>(P + r * PS + 32 * u + 16 + 4 * g);
+        const bf16x8 pf = __builtin_bit_cast(bf16x8, u32x4{p0.x, p0.y, p1.x, p1.y});
+        const int ra = 32 * u + 4 * g + qq, rb = ra + 16;
+#pragma unroll
+        for (int c = 0; c < NT; ++c) {
+          const int ch = 2 * (wave * NT + c) + (pp >> 1);
+          const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+              (__attribute__((address_space(3))) s16x4*)(cb + ra * (2 * Dp) + ((ch ^ (ra & 7)) << 4) + 8 * (pp & 1)));
+          const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+              (__attribute__((address_space(3))) s16x4*)(cb + rb * (2 * Dp) + ((ch ^ (rb & 7)) << 4) + 8 * (pp & 1)));
+          const s16x8 a8 = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
+          const f32x4 acc = u == 0 ? o[c] * alpha : o[c];
+          o[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a8), pf, acc, 0, 0, 0);
+        }
+      }
+      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      bar_lgkm();
+    }
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    if (g == 0) mx[wave * 16 + r] = l;
+    bar_lgkm();
+    l = mx[r] + mx[16 + r] + mx[32 + r] + mx[48 + r];
+  }
+  if (head >= p.H) return;
+  if (p.ns == 1) {
+    const float inv = l > 0.f ? 1.f / l : 0.f;
+    typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+    __bf16* y = reinterpret_cast<__bf16*>(p.out) + ((size_t)t * p.H + head) * Rp + wave * NT * 16 + 4 * g;
+#pragma unroll
+    for (int c = 0; c < NT; ++c)
+      *reinterpret_cast<bf4*>(y + 16 * c) =
+          bf4{(__bf16)(o[c][0] * inv), (__bf16)(o[c][1] * inv), (__bf16)(o[c][2] * inv), (__bf16)(o[c][3] * inv)};
+    return;
+  }
+  const size_t pi = ((size_t)t * p.H + head) * p.ns + split;
+#pragma unroll
+  for (int c = 0; c < NT; ++c)
+    *reinterpret_cast<f32x4*>(p.part_o + pi * Rp + wave * NT * 16 + 16 * c + 4 * g) = o[c];
+  if (wave == 0 && g == 0) {
+    p.part_ml[2 * pi] = m;
+    p.part_ml[2 * pi + 1] = l;
+  }
+}
+
+__global__ __launch_bounds__(256) void latent_merge_kernel(LA p) {
+  const size_t th = blockIdx.x;
+  const float* ml = p.part_ml + th * p.ns * 2;
+  float M = -INFINITY, L = 0.f;
+  for (int s = 0; s < p.ns; ++s) M = fmaxf(M, ml[2 * s]);
+  if (M == -INFINITY) M = 0.f;
+  for (int s = 0; s < p.ns; ++s) L += ml[2 * s + 1] * exp2f(ml[2 * s] - M);
+  const float inv = L > 0.f ? 1.f / L : 0.f;
+  const float* po = p.part_o + th * p.ns * p.Rp;
+  __bf16* y = reinterpret_cast<__bf16*>(p.out) + th * p.Rp;
+  for (int i = threadIdx.x; i < p.Rp; i += 256) {
+    float a = 0.f;
+    for (int s = 0; s < p.ns; ++s) a += po[(size_t)s * p.Rp + i] * exp2f(ml[2 * s] - M);
+    y[i] = (__bf16)(a * inv);
+  }
+}
+
+constexpr int NC = 4;         // output columns per thread: Rp <= 1024
+
+__global__ __launch_bounds__(256) void latent_attn_f32_kernel(LA p) {
+  __shared__ __attribute__((aligned(16))) float q[2048], sc[64];
+  const int t = blockIdx.x, h = blockIdx.y, Dp = p.Rp + p.rp;
+  const int ctx = p.ctx_len[t];
+  const int* bt = p.bt + (size_t)p.tok_seq[t] * p.bts;
+  const float* cache = reinterpret_cast<const float*>(p.cache);
+  const float* qr = reinterpret_cast<const float*>(p.q) + ((size_t)t * p.H + h) * Dp;
+  for (int i = threadIdx.x; i < Dp; i += 256) q[i] = qr[i];
+  __syncthreads();
+  const int key = threadIdx.x >> 2, part = threadIdx.x & 3;
+  float m = -INFINITY, l = 0.f, acc[NC] = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < ctx; k0 += 64) {
+    const int k = k0 + key;
+    float s = 0.f;
+    if (k < ctx) {
+      const float* c = cache + ((size_t)bt[k / p.bs] * p.bs + k % p.bs) * Dp;
+      for (int d = part * 4; d < Dp; d += 16) {
+        const f32x4 a = *reinterpret_cast<const f32x4*>(c + d), b = *reinterpret_cast<const f32x4*>(q + d);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) s = fmaf(a[e], b[e], s);
+      }
+    }
+    s += __shfl_xor(s, 1, 64);
+    s += __shfl_xor(s, 2, 64);
+    if (part == 0) sc[key] = k < ctx ? s * p.scale : -INFINITY;
+    __syncthreads();
+    float mn = m;
+    for (int i = 0; i < 64; ++i) mn = fmaxf(mn, sc[i]);
+    const float alpha = m == -INFINITY ? 0.f : expf(m - mn);
+    l *= alpha;
+#pragma unroll
+    for (int i = 0; i < NC; ++i) acc[i] *= alpha;
+    m = mn;
+    const int n = min(64, ctx - k0);
+    for (int i = 0; i < n; ++i) {
+      const float e = expf(sc[i] - mn);
+      l += e;
+      const int kk = k0 + i;
+      const float* c = cache + ((size_t)bt[kk / p.bs] * p.bs + kk % p.bs) * Dp;
+#pragma unroll
+      for (int q4 = 0; q4 < NC; ++q4) {
+        const int col = threadIdx.x + 256 * q4;
+        if (col < p.Rp) acc[q4] = fmaf(e, c[col], acc[q4]);
+      }
+    }
+    __syncthreads();
+  }
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  float* y = reinterpret_cast<float*>(p.out) + ((size_t)t * p.H + h) * p.Rp;
+#pragma unroll
+  for (int q4 = 0; q4 < NC; ++q4) {
+    const int col = threadIdx.x + 256 * q4;
+    if (col < p.Rp) y[col] = acc[q4] * inv;
+  }
+}
+
+template <int NT, int RT>
+int launch_t(const LA& p, hipStream_t st) {
+  constexpr int KT = NT + RT > 9 ? 32 : 64;
+  constexpr int LDS = 2 * KT * 128 * (NT + RT) + 16 * (KT + 8) * 2 + 256 + NBT * 4;
+  static_assert(LDS <= 160 * 1024, "LDS");
+  static bool attr = false;
+  if (!attr) {
+    if (hipFuncSetAttribute((const void*)latent_attn_kernel<NT, RT, KT>, hipFuncAttributeMaxDynamicSharedMemorySize,
+                            LDS) != hipSuccess)
+      return -1;
+    attr = true;
+  }
+  const int HB = (p.H + 15) / 16, n = (p.T * p.ns + 7) / 8 * 8 * HB;
+  hipLaunchKernelGGL((latent_attn_kernel<NT, RT, KT>), dim3(n), dim3(256), LDS, st, p);
+  int rc = (int)hipGetLastError();
+  if (rc == 0 && p.ns > 1) {
+    hipLaunchKernelGGL(latent_merge_kernel, dim3(p.T * p.H), dim3(256), 0, st, p);
+    rc = (int)hipGetLastError();
+  }
+  return rc;
+}
+
+template <int NT>
+int launch_r(const LA& p, hipStream_t st) {
+  if (p.rp == 64) return launch_t<NT, 1>(p, st);
+  if (p.rp == 128) return launch_t<NT, 2>(p, st);
+  return -1;
+}
+
+}  // namespace nls_latent
+
+extern "C" {
+
+// Rp: latent width padded to 64 * {1, 2, 3, 4, 6, 8, 12, 16}; rp: rotated width padded to 64 or 128 (multiples of 4 in
+// f32 launches); cache rows and queries are Rp + rp wide, zero in the padding.
+int nls_latent_attn(const void* q, const void* cache, void* out, float* part_o, float* part_ml, const int* bt, int bts,
+                    int bs, const int* tok_seq, const int* ctx_len, int T, int H, int ns, int Rp, int rp, float scale,
+                    int f32, void* stream) {
+  using namespace nls_latent;
+  if (T < 1 || H < 1 || ns < 1 || bs < 1 || (ns > 1 && (!part_o || !part_ml))) return -1;
+  LA p{q, cache, out, part_o, part_ml, bt, tok_seq, ctx_len, bts, bs, T, H, ns, Rp, rp, scale};
+  hipStream_t st = (hipStream_t)stream;
+  if (f32) {
+    if (Rp > 256 * NC || Rp + rp > 2048 || (Rp & 3) || (rp & 3) || H > 65535) return -1;
+    hipLaunchKernelGGL(latent_attn_f32_kernel, dim3(T, H), dim3(256), 0, st, p);
+    return (int)hipGetLastError();
+  }
+  switch (Rp / 64 * (Rp % 64 == 0)) {
+    case 1: return launch_r<1>(p, st);
+    case 2: return launch_r<2>(p, st);
+    case 3: return launch_r<3>(p, st);
+    case 4: return launch_r<4>(p, st);
+    case 6: return launch_r<6>(p, st);
+    case 8: return launch_r<8>(p, st);
+    case 12: return launch_r<12>(p, st);
+    case 16: return launch_r<16>(p, st);
+  }
+  return -1;
+}
+
+}  // extern "C"

@@ -1,0 +1,412 @@
+// Row kernels of the config-driven decoder stacks (models/stack.py): embedding, output norms with the residual add,
+// routed-expert combine, latent-attention row preparation, expert routing. The residual stream is f32; `xb` is its
+// bf16 rounding, the operand of the next projections (f32 launches use the residual itself: xb null).
+#include "../kernels/common.h"
+
+namespace nls_stack {
+
+DEVI float wsum(float v) {
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);
+  return v;
+}
+
+// sum over the workgroup's NW waves; sh: NW floats, reusable on return
+template <int NW>
+DEVI float bsum(float v, float* sh) {
+  v = wsum(v);
+  if ((threadIdx.x & 63) == 0) sh[threadIdx.x >> 6] = v;
+  __syncthreads();
+  float t = 0.f;
+#pragma unroll
+  for (int i = 0; i < NW; ++i) t += sh[i];
+  __syncthreads();
+  return t;
+}
+
+template <typename T> DEVI float ldv(const T* p, long i) { return (float)p[i]; }
+template <typename T> DEVI void stv(T* p, long i, float v) { p[i] = (T)v; }
+
+// ---- x[t] = table[id], id from the host or (use_prev) the previous step's next_ids
+__global__ __launch_bounds__(256) void embed_kernel(int* __restrict__ ids, const int* __restrict__ next_ids,
+                                                    const int* __restrict__ use_prev, const __bf16* __restrict__ tab,
+                                                    int V, int D, float* __restrict__ x, __bf16* __restrict__ xb,
+                                                    long ldx) {
+  const int t = blockIdx.x;
+  int id = ids[t];
+  if (use_prev && use_prev[t]) id = next_ids[t];
+  id = min(max(id, 0), V - 1);
+  __syncthreads();
+  if (threadIdx.x == 0 && use_prev) ids[t] = id;
+  for (int i = threadIdx.x; i < D; i += 256) {
+    const __bf16 v = tab[(size_t)id * D + i];
+    x[(size_t)t * ldx + i] = (float)v;
+    if (xb) xb[(size_t)t * ldx + i] = v;
+  }
+}
+
+// ---- x[t] += LayerNorm(y) * w; y = one row, or (topk) sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t], the shared
+// expert). Optional second LayerNorm (the model's last norm) of the new x into `on` instead of xb.
+// Each of the 256 threads keeps its <= 8 float4 of the row in registers up to D = 8192; wider rows take the LDS copy.
+struct NormAdd {
+  const float* y;
+  const float* topw;
+  const float* w;
+  float* x;
+  __bf16* xb;
+  const float* ow;      // optional output norm weight
+  void* on;             // its output, activation type
+  long ldy, ldx, ldo;
+  long sh0;             // first shared-expert row, -1: none
+  int D, topk, f32;
+  float eps;
+};
+
+template <int NV>
+__global__ __launch_bounds__(256) void norm_add_kernel(NormAdd p) {
+  __shared__ float sh[4];
+  const int t = blockIdx.x, D = p.D;
+  float v[4 * NV], xr[4 * NV];
+  float s = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = (threadIdx.x + j * 256) * 4 + e;
+      float a = 0.f, b = 0.f;
+      if (i < D) {
+        b = p.x[(size_t)t * p.ldx + i];
+        if (p.topk) {
+          for (int k = 0; k < p.topk; ++k)
+            a += p.topw[t * p.topk + k] * p.y[((size_t)t * p.topk + k) * p.ldy + i];
+          if (p.sh0 >= 0) a += p.y[(size_t)(p.sh0 + t) * p.ldy + i];
+        } else {
+          a = p.y[(size_t)t * p.ldy + i];
+        }
+      }
+      v[4 * j + e] = a;
+      xr[4 * j + e] = b;
+      s += a;
+    }
+  }
+  const float mean = bsum<4>(s, sh) / (float)D;
+  s = 0.f;
+#pragma unroll
+  for (int j = 0; j < 4 * NV; ++j) {
+    const int i = (threadIdx.x + (j >> 2) * 256) * 4 + (j & 3);
+    const float d = i < D ? v[j] - mean : 0.f;
+    v[j] = d;
+    s += d * d;
+  }
+  const float inv = 1.f / sqrtf(bsum<4>(s, sh) / (float)D + p.eps);
+  s = 0.f;
+#pragma unroll
+  for (int j = 0; j < 4 * NV; ++j) {
+    const int i = (threadIdx.x + (j >> 2) * 256) * 4 + (j & 3);
+    if (i < D) {
+      const float o = xr[j] + v[j] * inv * p.w[i];
+      xr[j] = o;
+      s += o;
+      p.x[(size_t)t * p.ldx + i] = o;
+      if (p.xb) p.xb[(size_t)t * p.ldx + i] = (__bf16)o;
+    }
+  }
+  if (!p.ow) return;
+  const float m2 = bsum<4>(s, sh) / (float)D;
+  s = 0.f;
+#pragma unroll
+  for (int j = 0; j < 4 * NV; ++j) {
+    const int i = (threadIdx.x + (j >> 2) * 256) * 4 + (j & 3);
+    const float d = i < D ? xr[j] - m2 : 0.f;
+    s += d * d;
+  }
+  const float inv2 = 1.f / sqrtf(bsum<4>(s, sh) / (float)D + p.eps);
+#pragma unroll
+  for (int j = 0; j < 4 * NV; ++j) {
+    const int i = (threadIdx.x + (j >> 2) * 256) * 4 + (j & 3);
+    if (i < D) {
+      const float o = (xr[j] - m2) * inv2 * p.ow[i];
+      if (p.f32) reinterpret_cast<float*>(p.on)[(size_t)t * p.ldo + i] = o;
+      else reinterpret_cast<__bf16*>(p.on)[(size_t)t * p.ldo + i] = (__bf16)o;
+    }
+  }
+}
+
+// ---- out[i] = LayerNorm(x[rows ? rows[i] : i]) * w
+__global__ __launch_bounds__(256) void layer_norm_kernel(const float* __restrict__ x, long ldx,
+                                                         const int* __restrict__ rows, const float* __restrict__ w,
+                                                         void* __restrict__ out, long ldo, int D, float eps, int f32) {
+  __shared__ float sh[4];
+  const float* xr = x + (size_t)(rows ? rows[blockIdx.x] : (int)blockIdx.x) * ldx;
+  float s = 0.f;
+  for (int i = threadIdx.x; i < D; i += 256) s += xr[i];
+  const float mean = bsum<4>(s, sh) / (float)D;
+  s = 0.f;
+  for (int i = threadIdx.x; i < D; i += 256) s += (xr[i] - mean) * (xr[i] - mean);
+  const float inv = 1.f / sqrtf(bsum<4>(s, sh) / (float)D + eps);
+  for (int i = threadIdx.x; i < D; i += 256) {
+    const float o = (xr[i] - mean) * inv * w[i];
+    if (f32) reinterpret_cast<float*>(out)[(size_t)blockIdx.x * ldo + i] = o;
+    else reinterpret_cast<__bf16*>(out)[(size_t)blockIdx.x * ldo + i] = (__bf16)o;
+  }
+}
+
+// ---- latent attention rows: cq = RMSNorm(dq) * wq -> activation; c = RMSNorm(dkv[:R]) * wc and the rotated key part
+// rope(dkv[R:]) -> the paged cache row of the token ([c | zeros to Rp | k_rot | zeros]; slot < 0: not stored)
+template <typename T>
+__global__ __launch_bounds__(256) void latent_rows_kernel(const float* __restrict__ dq, long lddq, int Q,
+                                                          const float* __restrict__ wq, T* __restrict__ cq, long ldcq,
+                                                          const float* __restrict__ dkv, long lddkv, int R, int Rp,
+                                                          int rot, const float* __restrict__ wc,
+                                                          const float* __restrict__ cs, const int* __restrict__ pos,
+                                                          const int* __restrict__ slot, T* __restrict__ cache,
+                                                          long ldc, float eps) {
+  __shared__ float sh[4];
+  const int t = blockIdx.x;
+  const float* a = dq + (size_t)t * lddq;
+  float s = 0.f;
+  for (int i = threadIdx.x; i < Q; i += 256) s += a[i] * a[i];
+  const float iq = 1.f / sqrtf(bsum<4>(s, sh) / (float)Q + eps);
+  for (int i = threadIdx.x; i < Q; i += 256) stv(cq + (size_t)t * ldcq, i, a[i] * iq * wq[i]);
+  if (!dkv) return;
+  const float* b = dkv + (size_t)t * lddkv;
+  s = 0.f;
+  for (int i = threadIdx.x; i < R; i += 256) s += b[i] * b[i];
+  const float ic = 1.f / sqrtf(bsum<4>(s, sh) / (float)R + eps);
+  const int sl = slot[t];
+  if (sl < 0) return;
+  T* c = cache + (size_t)sl * ldc;
+  for (int i = threadIdx.x; i < R; i += 256) stv(c, i, b[i] * ic * wc[i]);
+  const float* f = cs + (size_t)pos[t] * rot;
+  for (int i = threadIdx.x; i < rot / 2; i += 256) {
+    const float u = b[R + 2 * i], v = b[R + 2 * i + 1];
+    stv(c, Rp + 2 * i, u * f[2 * i] - v * f[2 * i + 1]);
+    stv(c, Rp + 2 * i + 1, v * f[2 * i] + u * f[2 * i + 1]);
+  }
+}
+
+// ---- expert choice of one token: sigmoid scores, the `keep` groups with the largest sum of their two best scores, the
+// `topk` best experts of those; weight = score * scale. Ties go to the lowest index. One wave per token; scores in LDS.
+DEVI void pick_experts(const float* __restrict__ z, int E, int topk, int groups, int keep, float scale, int lane,
+                       float* sc, float* gs, float* __restrict__ topw, int* __restrict__ sel) {
+  for (int e = lane; e < E; e += 64) {
+    const float s = 1.f / (1.f + expf(-z[e]));
+    sc[e] = s == s ? s : -1.f;
+  }
+  __builtin_amdgcn_wave_barrier();
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  const int per = E / groups;
+  for (int g = lane; g < groups; g += 64) {
+    float a = -2.f, b = -2.f;
+    for (int i = 0; i < per; ++i) {
+      const float s = sc[g * per + i];
+      if (s > a) { b = a; a = s; }
+      else if (s > b) b = s;
+    }
+    gs[g] = per > 1 ? a + b : a;
+  }
+  __builtin_amdgcn_wave_barrier();
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  // group g is kept when fewer than `keep` groups beat it
+  for (int g = lane; g < groups; g += 64) {
+    int better = 0;
+    for (int h = 0; h < groups; ++h) better += gs[h] > gs[g] || (gs[h] == gs[g] && h < g);
+    if (better >= keep)
+      for (int i = 0; i < per; ++i) sc[g * per + i] = -3.f;
+  }
+  __builtin_amdgcn_wave_barrier();
+  asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  for (int j = 0; j < topk; ++j) {
+    float bv = -4.f;
+    int be = 0x7fffffff;
+    for (int e = lane; e < E; e += 64)
+      if (sc[e] > bv) { bv = sc[e]; be = e; }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(bv, o, 64);
+      const int oe = __shfl_xor(be, o, 64);
+      if (ov > bv || (ov == bv && oe < be)) { bv = ov; be = oe; }
+    }
+    if (lane == 0) {
+      topw[j] = bv * scale;
+      sel[j] = be;
+    }
+    if (lane == (be & 63)) sc[be] = -4.f;
+    __builtin_amdgcn_wave_barrier();
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+  }
+}
+
+constexpr int ME = 512;       // experts per layer
+constexpr int PW = 8;         // waves that choose experts in moe_plan_kernel<true>
+
+__global__ __launch_bounds__(64) void moe_pick_kernel(const float* __restrict__ z, long ldz, int E, int topk,
+                                                      int groups, int keep, float scale, float* __restrict__ topw,
+                                                      int* __restrict__ sel) {
+  __shared__ float sc[ME], gs[ME];
+  const int t = blockIdx.x;
+  pick_experts(z + (size_t)t * ldz, E, topk, groups, keep, scale, threadIdx.x, sc, gs, topw + (size_t)t * topk,
+               sel + (size_t)t * topk);
+}
+
+// ---- routed-entry lists of one step: entries (token t, choice j) = t * topk + j grouped by expert (entry order within
+// an expert is arbitrary: rows do not interact), and the (expert, <= bm entries) tiles of the grouped products.
+// One workgroup. PICK: also choose the experts (small steps: one launch less).
+template <bool PICK>
+__global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict__ z, long ldz, int T, int E, int topk,
+                                                        int groups, int keep, float scale, float* __restrict__ topw,
+                                                        int* __restrict__ sel, int bm, int* __restrict__ rows,
+                                                        int* __restrict__ tiles, int* __restrict__ ntiles, int maxtiles) {
+  __shared__ int cnt[ME], off[ME], pos[ME];
+  __shared__ float sc[PICK ? PW : 1][PICK ? ME : 1], gs[PICK ? PW : 1][PICK ? ME : 1];
+  const int n = T * topk;
+  if constexpr (PICK) {
+    const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    for (int t = w; w < PW && t < T; t += PW)
+      pick_experts(z + (size_t)t * ldz, E, topk, groups, keep, scale, lane, sc[w], gs[w], topw + (size_t)t * topk,
+                   sel + (size_t)t * topk);
+    __threadfence_block();
+  }
+  for (int e = threadIdx.x; e < E; e += 1024) cnt[e] = 0;
+  __syncthreads();
+  for (int i = threadIdx.x; i < n; i += 1024) atomicAdd(&cnt[min(max(sel[i], 0), E - 1)], 1);
+  __syncthreads();
+  if (threadIdx.x < 64) {
+    // one wave: exclusive prefix sums of counts and tile counts, 64 experts at a time
+    int o = 0, to = 0;
+    for (int e0 = 0; e0 < E; e0 += 64) {
+      const int e = e0 + threadIdx.x;
+      const int c = e < E ? cnt[e] : 0;
+      const int nt = (c + bm - 1) / bm;
+      int a = c, b = nt;
+#pragma unroll
+      for (int s = 1; s < 64; s <<= 1) {
+        const int ua = __shfl_up(a, s, 64), ub = __shfl_up(b, s, 64);
+        if (threadIdx.x >= s) { a += ua; b += ub; }
+      }
+      if (e < E) {
+        off[e] = o + a - c;
+        pos[e] = 0;
+        for (int i = 0; i < nt; ++i) {
+          const int ti = to + b - nt + i;
+          if (ti < maxtiles) {
+            tiles[4 * ti] = e;
+            tiles[4 * ti + 1] = o + a - c + i * bm;
+            tiles[4 * ti + 2] = min(bm, c - i * bm);
+            tiles[4 * ti + 3] = 0;
+          }
+        }
+      }
+      o += __shfl(a, 63, 64);
+      to += __shfl(b, 63, 64);
+    }
+    if (threadIdx.x == 0) *ntiles = min(to, maxtiles);
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < n; i += 1024) {
+    const int e = min(max(sel[i], 0), E - 1);
+    rows[off[e] + atomicAdd(&pos[e], 1)] = i;
+  }
+}
+
+// ---- greedy pick: lowest index of the row's largest logit
+__global__ __launch_bounds__(1024) void argmax_kernel(const float* __restrict__ z, long ldz, int V,
+                                                      int* __restrict__ out) {
+  __shared__ float bv[16];
+  __shared__ int bi[16];
+  const float* r = z + (size_t)blockIdx.x * ldz;
+  float v = -INFINITY;
+  int ix = 0x7fffffff;
+  for (int i = threadIdx.x; i < V; i += 1024) {
+    const float a = r[i];
+    if (a > v || ix == 0x7fffffff) { v = a; ix = i; }
+  }
+  auto take = [&](float ov, int oi) {
+    if (ov > v || (ov == v && oi < ix)) { v = ov; ix = oi; }
+  };
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    const float ov = __shfl_xor(v, o, 64);
+    const int oi = __shfl_xor(ix, o, 64);
+    take(ov, oi);
+  }
+  if ((threadIdx.x & 63) == 0) { bv[threadIdx.x >> 6] = v; bi[threadIdx.x >> 6] = ix; }
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    for (int w = 1; w < 16; ++w) take(bv[w], bi[w]);
+    out[blockIdx.x] = ix < V ? ix : 0;
+  }
+}
+
+}  // namespace nls_stack
+
+extern "C" {
+using namespace nls_stack;
+
+int nls_stack_embed(int* ids, const int* next_ids, const int* use_prev, const void* tab, int V, int D, float* x,
+                    void* xb, long ldx, int T, void* stream) {
+  if (T < 1 || D < 1 || V < 1) return -1;
+  hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, ids, next_ids, use_prev,
+                     (const __bf16*)tab, V, D, x, (__bf16*)xb, ldx);
+  return (int)hipGetLastError();
+}
+
+int nls_norm_add(const float* y, long ldy, const float* topw, int topk, long sh0, const float* w, float* x, void* xb,
+                 long ldx, const float* ow, void* on, long ldo, int D, int T, float eps, int f32, void* stream) {
+  if (T < 1 || D < 1 || D > 16384) return -1;
+  NormAdd p{y, topw, w, x, (__bf16*)xb, ow, on, ldy, ldx, ldo, sh0, D, topk, f32, eps};
+  hipStream_t st = (hipStream_t)stream;
+  if (D <= 1024) hipLaunchKernelGGL(norm_add_kernel<1>, dim3(T), dim3(256), 0, st, p);
+  else if (D <= 2048) hipLaunchKernelGGL(norm_add_kernel<2>, dim3(T), dim3(256), 0, st, p);
+  else if (D <= 4096) hipLaunchKernelGGL(norm_add_kernel<4>, dim3(T), dim3(256), 0, st, p);
+  else if (D <= 8192) hipLaunchKernelGGL(norm_add_kernel<8>, dim3(T), dim3(256), 0, st, p);
+  else hipLaunchKernelGGL(norm_add_kernel<16>, dim3(T), dim3(256), 0, st, p);
+  return (int)hipGetLastError();
+}
+
+int nls_layer_norm(const float* x, long ldx, const int* rows, const float* w, void* out, long ldo, int D, int n,
+                   float eps, int f32, void* stream) {
+  if (n < 1 || D < 1) return -1;
+  hipLaunchKernelGGL(layer_norm_kernel, dim3(n), dim3(256), 0, (hipStream_t)stream, x, ldx, rows, w, out, ldo, D, eps,
+                     f32);
+  return (int)hipGetLastError();
+}
+
+int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq, long ldcq, const float* dkv,
+                    long lddkv, int R, int Rp, int rot, const float* wc, const float* cs, const int* pos,
+                    const int* slot, void* cache, long ldc, int T, float eps, int f32, void* stream) {
+  if (T < 1 || Q < 1 || (dkv && (R < 1 || (rot & 1) || Rp + rot > ldc))) return -1;
+  if (f32)
+    hipLaunchKernelGGL(latent_rows_kernel<float>, dim3(T), dim3(256), 0, (hipStream_t)stream, dq, lddq, Q, wq,
+                       (float*)cq, ldcq, dkv, lddkv, R, Rp, rot, wc, cs, pos, slot, (float*)cache, ldc, eps);
+  else
+    hipLaunchKernelGGL(latent_rows_kernel<__bf16>, dim3(T), dim3(256), 0, (hipStream_t)stream, dq, lddq, Q, wq,
+                       (__bf16*)cq, ldcq, dkv, lddkv, R, Rp, rot, wc, cs, pos, slot, (__bf16*)cache, ldc, eps);
+  return (int)hipGetLastError();
+}
+
+int nls_stack_argmax(const float* z, long ldz, int V, int* out, int n, void* stream) {
+  if (n < 1 || V < 1) return -1;
+  hipLaunchKernelGGL(argmax_kernel, dim3(n), dim3(1024), 0, (hipStream_t)stream, z, ldz, V, out);
+  return (int)hipGetLastError();
+}
+
+// rows: int [T * topk]; tiles: int [maxtiles][4], maxtiles >= min(T * topk, E + T * topk / bm)
+int nls_moe_plan(const float* z, long ldz, int T, int E, int topk, int groups, int keep, float scale, float* topw,
+                 int* sel, int bm, int* rows, int* tiles, int* ntiles, int maxtiles, void* stream) {
+  if (T < 1 || E < 1 || E > ME || topk < 1 || topk > E || groups < 1 || E % groups || keep < 1 || bm < 1 ||
+      (long)min(keep, groups) * (E / groups) < topk || maxtiles < 1)
+    return -1;
+  hipStream_t st = (hipStream_t)stream;
+  if (T <= 32) {
+    hipLaunchKernelGGL(moe_plan_kernel<true>, dim3(1), dim3(1024), 0, st, z, ldz, T, E, topk, groups, keep, scale, topw,
+                       sel, bm, rows, tiles, ntiles, maxtiles);
+    return (int)hipGetLastError();
+  }
+  hipLaunchKernelGGL(moe_pick_kernel, dim3(T), dim3(64), 0, st, z, ldz, E, topk, groups, keep, scale, topw, sel);
+  hipLaunchKernelGGL(moe_plan_kernel<false>, dim3(1), dim3(1024), 0, st, z, ldz, T, E, topk, groups, keep, scale, topw,
+                     sel, bm, rows, tiles, ntiles, maxtiles);
+  return (int)hipGetLastError();
+}
+
+}  // extern "C"

@@ -1,0 +1,240 @@
+// Gated linear recurrence with a per-channel decay ("wkv" time mixing), gfx950.
+//
+// Per head, with keys i and values j (state S [dim][dim], f32):
+//   o_t[j] = sum_i r_t[i] (S[i][j] + u[i] k_t[i] v_t[j]);   S[i][j] = w_t[i] S[i][j] + k_t[i] v_t[j]
+//
+// The scan is sequential in the tokens of a run, so a position's result does not depend on how its sequence was cut
+// into steps. Parallelism is (run, head, 32 value columns) x lanes: a wave owns 8 value columns, lane = 8 key parts x 8
+// columns, each lane DP / 8 state values in registers; the key sum closes with three lane exchanges. Tokens are staged
+// in LDS in chunks of CH as f32, the next chunk's loads in flight while the current one runs.
+//
+// A run = (first row, tokens, state slot, first position): consecutive rows of one sequence. A run at position 0
+// starts from a zero state, any other from its slot; slot < 0 or 0 tokens: nothing to do (padded decode rows).
+#include "../kernels/common.h"
+
+namespace nls_wkv {
+
+template <typename T> DEVI float ld1(const T* p) { return (float)*p; }
+
+// ---- token shift: m_s[t] = h[t] + (h[t - 1] - h[t]) * mu_s for NS mixes; h = the f32 residual row. The row before
+// a run's first is the slot's previous token (zeros at position 0).
+constexpr int NS = 5;
+struct Mix {
+  const float* x;
+  const float* mu;      // [NS][D]
+  const float* prev;    // [slots][prev stride]
+  void* out;            // [NS][rows cap][ldo]
+  const int* runs;      // [nruns][4]
+  const int* tok_seq;   // row -> run
+  long ldx, ldp, ldo, mstride;
+  int D, f32;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void shift_mix_kernel(Mix p) {
+  const int t = blockIdx.x;
+  const int* run = p.runs + 4 * p.tok_seq[t];
+  const int t0 = run[0], n = run[1], slot = run[2], pos0 = run[3];
+  if (slot < 0 || t < t0 || t >= t0 + n) return;
+  const float* h = p.x + (size_t)t * p.ldx;
+  const float* q = t > t0 ? h - p.ldx : (pos0 > 0 ? p.prev + (size_t)slot * p.ldp : nullptr);
+  T* o = reinterpret_cast<T*>(p.out) + (size_t)t * p.ldo;
+  for (int i = threadIdx.x; i < p.D; i += 256) {
+    const float a = h[i], d = (q ? q[i] : 0.f) - a;
+#pragma unroll
+    for (int s = 0; s < NS; ++s) o[s * p.mstride + i] = (T)(a + d * p.mu[s * p.D + i]);
+  }
+}
+
+struct Scan {
+  const void *r, *k, *v;   // activation type, [rows][ld]
+  const float* w;          // decays in (0, 1), f32 [rows][ldw]
+  const float* u;          // [H * D]
+  float* o;                // f32 [rows][ldo]
+  float* state;            // [slots][sstride]: [H][D][D]
+  const float* x;          // residual rows: the run's last becomes the slot's previous token
+  float* prev;
+  const int* runs;
+  long ld, ldw, ldo, sstride, ldx, ldp;
+  int H, D, width;
+};
+
+// DP: key channels padded to a multiple of 32 (zeros past D)
+template <typename T, int DP>
+__global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
+  constexpr int CH = DP <= 64 ? 16 : 8;          // tokens per staged chunk
+  constexpr int R = DP / 8;                      // state rows per lane
+  constexpr int LR = DP + 4;                     // LDS row stride
+  constexpr int NV = (CH * DP + 255) / 256;      // staged values per thread and operand
+  __shared__ __attribute__((aligned(16))) float rs[CH][LR], ks[CH][LR], ws[CH][LR];
+  __shared__ float vs[CH][32], ruk[CH];
+  const int* run = p.runs + 4 * blockIdx.y;
+  const int t0 = run[0], n = run[1], slot = run[2], pos0 = run[3];
+  if (slot < 0 || n < 1) return;
+  const int D = p.D;
+  const int ncb = (D + 31) / 32;
+  const int head = blockIdx.x / ncb, c0 = (blockIdx.x % ncb) * 32;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int part = lane >> 3, col = wave * 8 + (lane & 7);
+  const int j = c0 + col;
+  const size_t hb = (size_t)head * D;
+  const T* rp = (const T*)p.r + hb;
+  const T* kp = (const T*)p.k + hb;
+  const T* vp = (const T*)p.v + hb;
+  const float* wp = p.w + hb;
+  float* st = p.state + (size_t)slot * p.sstride + hb * D;
+
+  float S[R];
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int row = part * R + i;
+    S[i] = (pos0 > 0 && row < D && j < D) ? st[(size_t)row * D + j] : 0.f;
+  }
+  float fr[NV], fk[NV], fw[NV], fv[(CH * 32 + 255) / 256];
+  auto fetch = [&](int base) __attribute__((always_inline)) {
+#pragma unroll
+    for (int q = 0; q < NV; ++q) {
+      const int e = threadIdx.x + q * 256, tt = e / DP, i = e % DP;
+      const bool in = tt < CH && base + tt < n && i < D;
+      const size_t row = (size_t)(t0 + min(base + tt, n - 1));
+      fr[q] = in ? ld1(rp + row * p.ld + i) : 0.f;
+      fk[q] = in ? ld1(kp + row * p.ld + i) : 0.f;
+      fw[q] = in ? wp[row * p.ldw + i] : 0.f;
+    }
+#pragma unroll
+    for (int q = 0; q < (CH * 32 + 255) / 256; ++q) {
+      const int e = threadIdx.x + q * 256, tt = e / 32, i = c0 + (e & 31);
+      const bool in = tt < CH && base + tt < n && i < D;
+      fv[q] = in ? ld1(vp + (size_t)(t0 + min(base + tt, n - 1)) * p.ld + i) : 0.f;
+    }
+  };
+  fetch(0);
+  for (int base = 0; base < n; base += CH) {
+    __syncthreads();
+#pragma unroll
+    for (int q = 0; q < NV; ++q) {
+      const int e = threadIdx.x + q * 256, tt = e / DP, i = e % DP;
+      if (tt < CH) {
+        rs[tt][i] = fr[q];
+        ks[tt][i] = fk[q];
+        ws[tt][i] = fw[q];
+      }
+    }
+#pragma unroll
+    for (int q = 0; q < (CH * 32 + 255) / 256; ++q) {
+      const int e = threadIdx.x + q * 256;
+      if (e < CH * 32) vs[e / 32][e & 31] = fv[q];
+    }
+    __syncthreads();
+    if (base + CH < n) fetch(base + CH);
+    // sum_i r u k of every staged token: 16 lanes each
+    {
+      const int tt = threadIdx.x >> 4, l = threadIdx.x & 15;
+      float a = 0.f;
+      if (tt < CH)
+        for (int i = l; i < D; i += 16) a += rs[tt][i] * p.u[hb + i] * ks[tt][i];
+#pragma unroll
+      for (int s = 8; s > 0; s >>= 1) a += __shfl_xor(a, s, 64);
+      if (tt < CH && l == 0) ruk[tt] = a;
+    }
+    __syncthreads();
+    const int m = min(CH, n - base);
+    for (int tt = 0; tt < m; ++tt) {
+      const float v = vs[tt][col];
+      float o = 0.f;
+#pragma unroll
+      for (int i4 = 0; i4 < R; i4 += 4) {
+        const f32x4 r4 = *reinterpret_cast<const f32x4*>(&rs[tt][part * R + i4]);
+        const f32x4 k4 = *reinterpret_cast<const f32x4*>(&ks[tt][part * R + i4]);
+        const f32x4 w4 = *reinterpret_cast<const f32x4*>(&ws[tt][part * R + i4]);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          o = fmaf(r4[e], S[i4 + e], o);
+          S[i4 + e] = fmaf(w4[e], S[i4 + e], k4[e] * v);
+        }
+      }
+      o += __shfl_xor(o, 8, 64);
+      o += __shfl_xor(o, 16, 64);
+      o += __shfl_xor(o, 32, 64);
+      if (part == 0 && j < D) p.o[(size_t)(t0 + base + tt) * p.ldo + hb + j] = o + ruk[tt] * v;
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int row = part * R + i;
+    if (row < D && j < D) st[(size_t)row * D + j] = S[i];
+  }
+  // the run's last row is the next step's previous token (this layer's shift_mix, which reads it, came before)
+  const int G = gridDim.x;
+  for (int i = blockIdx.x * 256 + threadIdx.x; i < p.width; i += G * 256)
+    p.prev[(size_t)slot * p.ldp + i] = p.x[(size_t)(t0 + n - 1) * p.ldx + i];
+}
+
+// ---- out = (o / rms(o) per head) * norm * gate
+template <typename T>
+__global__ __launch_bounds__(256) void wkv_out_kernel(const float* __restrict__ o, long ldo,
+                                                      const float* __restrict__ norm, const T* __restrict__ gate,
+                                                      long ldg, T* __restrict__ out, long ld, int H, int D, float eps) {
+  const int t = blockIdx.x, lane = threadIdx.x & 63;
+  for (int h = blockIdx.y * 4 + (threadIdx.x >> 6); h < H; h += gridDim.y * 4) {
+    const float* p = o + (size_t)t * ldo + (size_t)h * D;
+    float s = 0.f;
+    for (int i = lane; i < D; i += 64) s += p[i] * p[i];
+#pragma unroll
+    for (int q = 32; q > 0; q >>= 1) s += __shfl_xor(s, q, 64);
+    const float inv = 1.f / sqrtf(s / (float)D + eps);
+    for (int i = lane; i < D; i += 64) {
+      const int c = h * D + i;
+      out[(size_t)t * ld + c] = (T)(p[i] * inv * norm[c] * (float)gate[(size_t)t * ldg + c]);
+    }
+  }
+}
+
+template <typename T>
+int scan_t(const Scan& p, int nruns, hipStream_t st) {
+  const dim3 grid(p.H * ((p.D + 31) / 32), nruns);
+  if (p.D <= 32) hipLaunchKernelGGL((wkv_scan_kernel<T, 32>), grid, dim3(256), 0, st, p);
+  else if (p.D <= 64) hipLaunchKernelGGL((wkv_scan_kernel<T, 64>), grid, dim3(256), 0, st, p);
+  else if (p.D <= 128) hipLaunchKernelGGL((wkv_scan_kernel<T, 128>), grid, dim3(256), 0, st, p);
+  else if (p.D <= 256) hipLaunchKernelGGL((wkv_scan_kernel<T, 256>), grid, dim3(256), 0, st, p);
+  else return -1;
+  return (int)hipGetLastError();
+}
+
+}  // namespace nls_wkv
+
+extern "C" {
+using namespace nls_wkv;
+
+int nls_shift_mix(const float* x, long ldx, const float* mu, const float* prev, long ldp, void* out, long ldo,
+                  long mstride, const int* runs, const int* tok_seq, int D, int T, int f32, void* stream) {
+  if (T < 1 || D < 1) return -1;
+  Mix p{x, mu, prev, out, runs, tok_seq, ldx, ldp, ldo, mstride, D, f32};
+  if (f32) hipLaunchKernelGGL(shift_mix_kernel<float>, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
+  else hipLaunchKernelGGL(shift_mix_kernel<__bf16>, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
+  return (int)hipGetLastError();
+}
+
+int nls_wkv_scan(const void* r, const void* k, const void* v, long ld, const float* w, long ldw, const float* u,
+                 float* o, long ldo, float* state, long sstride, const float* x, long ldx, float* prev, long ldp,
+                 int width, const int* runs, int nruns, int H, int D, int f32, void* stream) {
+  if (nruns < 1 || H < 1 || D < 1) return -1;
+  Scan p{r, k, v, w, u, o, state, x, prev, runs, ld, ldw, ldo, sstride, ldx, ldp, H, D, width};
+  return f32 ? scan_t<float>(p, nruns, (hipStream_t)stream) : scan_t<__bf16>(p, nruns, (hipStream_t)stream);
+}
+
+int nls_wkv_out(const float* o, long ldo, const float* norm, const void* gate, long ldg, void* out, long ld, int H,
+                int D, int T, float eps, int f32, void* stream) {
+  if (T < 1 || H < 1 || D < 1) return -1;
+  const int gy = T >= 256 ? 1 : min((H + 3) / 4, 64);
+  const dim3 grid(T, gy);
+  if (f32)
+    hipLaunchKernelGGL(wkv_out_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, o, ldo, norm,
+                       (const float*)gate, ldg, (float*)out, ld, H, D, eps);
+  else
+    hipLaunchKernelGGL(wkv_out_kernel<__bf16>, grid, dim3(256), 0, (hipStream_t)stream, o, ldo, norm,
+                       (const __bf16*)gate, ldg, (__bf16*)out, ld, H, D, eps);
+  return (int)hipGetLastError();
+}
+
+}  // extern "C"

@@ -1,6 +1,8 @@
 """Build the native parts in-tree (no JIT cache, no site-packages):
 
 * `_kernels.so`  -- gfx950 HIP kernels (hipcc --offload-arch=gfx950)
+* `_stack.so`    -- gfx950 HIP kernels of the config-driven decoder stacks (models/stack.py), a library of its own so
+                    that a stack model can be built and run without the quantised GEMM families
 * `_natscore.*.so` -- C++ NATS wire core (client + embedded server + JetStream object store), pybind11
 
     python -m nats_llm_studio_amd.build [--force]
@@ -60,8 +62,20 @@ def kernel_sources():
     return srcs, srcs + sorted(glob.glob(os.path.join(CSRC, "kernels", "*.h")))
 
 
+def stack_sources():
+    srcs = sorted(glob.glob(os.path.join(CSRC, "stack", "*.hip")))
+    hdrs = sorted(glob.glob(os.path.join(CSRC, "stack", "*.h")))
+    return srcs, srcs + hdrs + [os.path.join(CSRC, "kernels", h) for h in ("common.h", "lds_dma.h")]
+
+
+# no packed FP32 instructions (v_pk_add / mul / fma_f32): hipcc -O3 forms them from ordinary float code, and some of
+# their forms are not reliable on this hardware. Device pass only; the host pass warns that it does not know the feature.
+NO_PACKED_F32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+
+
 def kernel_flags(defines=()):
-    return [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-munsafe-fp-atomics", *[f"-D{d}" for d in defines]]
+    return [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-munsafe-fp-atomics", *NO_PACKED_F32,
+            *[f"-D{d}" for d in defines]]
 
 
 def _run(cmd):
@@ -69,19 +83,14 @@ def _run(cmd):
     subprocess.check_call(cmd)
 
 
-def build_kernels(force: bool = False, defines=(), tag: str = "") -> str:
-    """Compile each .hip translation unit to an object in parallel, then link one .so.
-    `defines` + `tag`: an A/B variant library `_kernels_<tag>.so` (e.g. tools/gemm_ab.py), built in
-    its own object directory; the default build is `_kernels.so`."""
-    out = os.path.join(PKG, f"_kernels_{tag}.so" if tag else "_kernels.so")
-    srcs, deps = kernel_sources()
-    flags = kernel_flags(defines)
+def _build_hip_lib(out: str, sources, bdir: str, flags, force: bool) -> str:
+    """Compile each .hip translation unit to an object in parallel, then link one .so."""
+    srcs, deps = sources
     if force or _stale(out, deps, flags):
         from concurrent.futures import ThreadPoolExecutor
         hipcc = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
-        bdir = os.path.join(ROOT, "build", f"kernels_{tag}" if tag else "kernels")
         os.makedirs(bdir, exist_ok=True)
-        hdrs = sorted(glob.glob(os.path.join(CSRC, "kernels", "*.h")))
+        hdrs = [d for d in deps if d.endswith(".h")]
         objs = [os.path.join(bdir, os.path.basename(s) + ".o") for s in srcs]
         jobs = [(s, o) for s, o in zip(srcs, objs) if force or _stale(o, [s] + hdrs, flags)]
 
@@ -98,11 +107,30 @@ def build_kernels(force: bool = False, defines=(), tag: str = "") -> str:
     return out
 
 
+def build_kernels(force: bool = False, defines=(), tag: str = "") -> str:
+    """`defines` + `tag`: an A/B variant library `_kernels_<tag>.so` (e.g. tools/gemm_ab.py), built in
+    its own object directory; the default build is `_kernels.so`."""
+    out = os.path.join(PKG, f"_kernels_{tag}.so" if tag else "_kernels.so")
+    bdir = os.path.join(ROOT, "build", f"kernels_{tag}" if tag else "kernels")
+    return _build_hip_lib(out, kernel_sources(), bdir, kernel_flags(defines), force)
+
+
+def build_stack(force: bool = False) -> str:
+    return _build_hip_lib(os.path.join(PKG, "_stack.so"), stack_sources(), os.path.join(ROOT, "build", "stack"),
+                          kernel_flags(), force)
+
+
 def kernels_current(out: str = None) -> bool:
     """True when the in-tree `_kernels.so` was built from exactly the current kernel sources."""
     out = out or os.path.join(PKG, "_kernels.so")
     srcs, deps = kernel_sources()
     return os.path.exists(out) and read_stamp(out) == source_hash(deps, kernel_flags())
+
+
+def stack_current(out: str = None) -> bool:
+    """True when the in-tree `_stack.so` was built from exactly the current sources."""
+    out = out or os.path.join(PKG, "_stack.so")
+    return os.path.exists(out) and read_stamp(out) == source_hash(stack_sources()[1], kernel_flags())
 
 
 def natscore_path() -> str:
@@ -174,7 +202,7 @@ def build_diag(force: bool = False):
     hipcc = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
     for src in sorted(glob.glob(os.path.join(CSRC, "diag", "*.hip"))):
         out = os.path.join(ROOT, "tools", "diag", "_" + os.path.basename(src)[:-4] + ".so")
-        flags = [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-shared"]
+        flags = [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-shared", *NO_PACKED_F32]
         if force or _stale(out, [src], flags):
             tmp = out + ".tmp"
             _run([hipcc, *flags, src, "-o", tmp])
@@ -186,6 +214,7 @@ def build_diag(force: bool = False):
 
 def build_all(force: bool = False):
     k = build_kernels(force)
+    build_stack(force)
     n = build_natscore(force)
     build_tokcore(force)
     build_tool(force=force)

@@ -31,7 +31,6 @@ import numpy as np
 import torch
 
 from .. import ops
-from ..models.llama import LlamaModel
 from .sampling import HIST, SamplingParams, sample_rows, sample_rows_dev, sample_rows_gpu, uniform01
 
 BUCKETS = (1, 2, 4, 8, 16, 32, 48, 64, 96, 128, 192, 256, 384, 512, 640, 768, 1024)
@@ -170,10 +169,25 @@ class BlockAllocator:
         return len(self.free) + len(self.lru)
 
 
+class StateSlots:
+    """Slots of the per-sequence recurrent states (StackModel.state_pool): one per admitted sequence, handed back when it
+    finishes or is preempted. Slots are not cleared: a sequence's first run starts from a zero state."""
+
+    def __init__(self, n: int):
+        self.n = n
+        self.free: Deque[int] = deque(range(n))
+
+    def alloc(self) -> Optional[int]:
+        return self.free.popleft() if self.free else None
+
+    def release(self, slot: int):
+        self.free.append(slot)
+
+
 class _Seq:
     __slots__ = ("req", "fut", "tokens", "n_prompt", "n_prefilled", "blocks", "t_submit", "t_admit", "t_first",
                  "t_done", "gen", "max_new", "done", "text_cache", "row", "n_fed", "keys", "n_cached", "n_target",
-                 "preempted")
+                 "preempted", "state_slot")
 
     def __init__(self, req: GenRequest, fut: Future):
         self.req = req
@@ -184,6 +198,7 @@ class _Seq:
         self.preempted = 0
         self.n_prefilled = 0
         self.blocks: List[int] = []
+        self.state_slot = -1            # recurrent models: this sequence's state slot
         self.t_submit = time.monotonic()
         self.t_admit = None
         self.t_first = None
@@ -203,10 +218,11 @@ class _Seq:
 
 
 class Engine:
-    def __init__(self, model: LlamaModel, tokenizer=None, max_batch: int = 64, block_size: int = 16,
+    def __init__(self, model, tokenizer=None, max_batch: int = 64, block_size: int = 16,
                  num_blocks: Optional[int] = None, max_prefill_tokens: int = 2048, use_graphs: bool = True,
                  ctx: Optional[int] = None, kv_mem_fraction: float = 0.5, eos_ids: Seq[int] = (),
-                 prefill_attn: bool = True, async_decode: bool = True, prefix_cache: bool = True):
+                 prefill_attn: bool = True, async_decode: bool = True, prefix_cache: bool = True,
+                 max_logit_rows: int = 0):
         self.model = model
         self.tok = tokenizer
         self.cfg = model.cfg
@@ -233,9 +249,7 @@ class Engine:
                 # left) could not hold every row of a full batch at full context -- the copies buy ~10 % of
                 # large-batch step time, a squeezed pool costs admissions (Llama-3-70B at 512 x 480 tokens:
                 # 79 GB of KV, no copies; Llama-3-8B: 31 GB, copies kept)
-                esz = torch.finfo(getattr(model, "kv_dtype", torch.bfloat16)).bits // 8
-                kv_need = (self.max_batch * self.ctx * 2 * self.cfg.n_layer * model.Hkv * model.D * esz
-                           if num_blocks is None else 0)
+                kv_need = self.max_batch * self.ctx * model.kv_token_bytes if num_blocks is None else 0
                 budget = max(0, min(int(0.60 * free), int(free - kv_need / max(kv_mem_fraction, 1e-3))))
                 frac = model.dense_decode_fraction(self.max_batch) if hasattr(model, "dense_decode_fraction") else 1.0
                 if frac < 0.5:
@@ -254,18 +268,22 @@ class Engine:
             num_blocks = self.max_batch * self.max_blocks
             num_blocks += num_blocks // 99 + 1
             if self.dev.type == "cuda":
-                esz = torch.finfo(getattr(model, "kv_dtype", torch.bfloat16)).bits // 8
-                per_block = 2 * self.cfg.n_layer * block_size * model.Hkv * model.D * esz
+                per_block = block_size * model.kv_token_bytes
                 free, _ = torch.cuda.mem_get_info(self.dev)
-                num_blocks = int(min(num_blocks, kv_mem_fraction * free // per_block))
+                if per_block:
+                    num_blocks = int(min(num_blocks, kv_mem_fraction * free // per_block))
         self.tp = model.comm if model.shard.size > 1 else None
         self.rank = model.shard.rank
         if self.tp is not None:                # every shard must hold the same KV block pool
             num_blocks = self.tp.min_int(num_blocks)
         self.num_blocks = num_blocks
         self.kc, self.vc = model.kv_cache(num_blocks, block_size)
-        self.kv_pool_bytes = 2 * self.kc.numel() * self.kc.element_size()
-        self.alloc = BlockAllocator(num_blocks, cache=prefix_cache)
+        self.kv_pool_bytes = num_blocks * block_size * model.kv_token_bytes
+        # recurrent models: one state slot per live sequence. A cached prompt prefix would need the states at its end
+        # as well, so these models prefill every prompt from its first token.
+        self.slots = StateSlots(self.max_batch) if model.recurrent else None
+        self.state = model.state_pool(self.max_batch) if model.recurrent else None
+        self.alloc = BlockAllocator(num_blocks, cache=prefix_cache and not model.recurrent)
         # admission keeps this many blocks free for the running sequences to grow into (fewer
         # preemptions right after a burst of admissions); NLS_KV_RESERVE=full restores worst-case
         # reservation of prompt + max_tokens at admission (no growth, no preemption)
@@ -285,7 +303,11 @@ class Engine:
         self.max_prefill = max_prefill_tokens
         self.prefill_attn = prefill_attn      # MFMA flash-prefill attention (else per-token decode kernel)
         self.db = model.step_buffers(self.max_batch, self.max_batch, self.max_blocks)
-        self.pb = model.step_buffers(max_prefill_tokens, self.max_batch, self.max_blocks)
+        # logit rows of one prefill forward: one per sequence ending in it; feeds may want more (max_logit_rows)
+        self.max_logit_rows = max(self.max_batch, max_logit_rows)
+        kw = {"logit_rows": self.max_logit_rows} if max_logit_rows > self.max_batch else {}
+        self.pb = model.step_buffers(max_prefill_tokens, self.max_batch, self.max_blocks, **kw)
+        self._fed: Dict[object, _Seq] = {}
         pin = self.dev.type == "cuda"
         # decode metadata / next-token host buffers are double-buffered (async decode: step N+1 is
         # prepared and launched while step N's copies may still be in flight)
@@ -451,7 +473,7 @@ class Engine:
         self.shutdown()
         self.graphs.clear()
         self.pf_graphs.clear()
-        self.kc = self.vc = None
+        self.kc = self.vc = self.state = None
         self.db = self.pb = None
         self.model = None
         if self.dev.type == "cuda":
@@ -551,12 +573,14 @@ class Engine:
                 if self.running and self.counters["steps"] < self._pressure_until:
                     reserve = max(reserve, len(self.running))
                 blocks = None
-                if need - len(hit) + reserve <= self.alloc.n_free:
+                if need - len(hit) + reserve <= self.alloc.n_free and (self.slots is None or self.slots.free):
                     blocks = self.alloc.alloc(need - len(hit))
                 if blocks is None:
                     self.alloc.release(hit)
                     break
                 s.blocks = hit + blocks
+                if self.slots is not None:
+                    s.state_slot = self.slots.alloc()
                 s.n_prefilled = s.n_cached = len(hit) * self.bs
                 self.alloc.hits += s.n_cached
                 s.t_admit = time.monotonic()
@@ -564,6 +588,15 @@ class Engine:
                 self.running.append(s)
                 if growth is not None:
                     growth += max(0, self._expected_blocks(s) - len(s.blocks))
+
+    def _release_memory(self, s: _Seq):
+        """Hand back the cache blocks and the state slot of s."""
+        if s.blocks:
+            self.alloc.release(s.blocks)
+            s.blocks = []
+        if s.state_slot >= 0:
+            self.slots.release(s.state_slot)
+            s.state_slot = -1
 
     def _slot(self, s: _Seq, p: int) -> int:
         return s.blocks[p // self.bs] * self.bs + p % self.bs
@@ -576,23 +609,28 @@ class Engine:
             ev.synchronize()
         self.h_meta_p = self.h_meta_p2[self._pfk]
 
-    def _prefill(self):
-        self._next_prefill_buf()
-        b, pad = self.pb, self.pb.pad
+    def _tables(self, meta: torch.Tensor, pad: int):
+        """The block tables [max_batch, max_blocks] and (recurrent models) the runs table [max_batch, 4] of a host
+        metadata buffer."""
+        h, n = meta.numpy(), self.max_batch * self.max_blocks
+        o = _NSEG * pad
+        bt = h[o:o + n].reshape(self.max_batch, self.max_blocks)
+        if self.slots is None:
+            return bt, None
+        return bt, h[o + n:o + n + 4 * self.max_batch].reshape(self.max_batch, 4)
+
+    def _fill_rows(self, parts) -> int:
+        """Stage one batch of rows in the current prefill metadata buffer: parts = [(sequence, first position, tokens)],
+        one run of consecutive rows each. Returns the row count."""
+        pad = self.pb.pad
         h = self.h_meta_p.numpy()
         ids, pos, slot, tseq, ctxl = (h[i * pad:(i + 1) * pad] for i in range(5))
         h[5 * pad:6 * pad] = 0                              # use_prev: prefill feeds host ids
-        bt = h[_NSEG * pad:].reshape(self.max_batch, self.max_blocks)
-        budget = self.max_prefill
+        bt, runs = self._tables(self.h_meta_p, pad)
         T = 0
-        rows, finishing = [], []
-        batch = [s for s in self.running if s.n_prefilled < s.n_target]
-        for si, s in enumerate(batch):
-            if budget <= 0:
-                break
-            n = min(budget, s.n_target - s.n_prefilled)
-            p0 = s.n_prefilled
-            ids[T:T + n] = s.tokens[p0:p0 + n]
+        for si, (s, p0, toks) in enumerate(parts):
+            n = len(toks)
+            ids[T:T + n] = toks
             pr = np.arange(p0, p0 + n)
             pos[T:T + n] = pr
             blk = np.asarray(s.blocks, dtype=np.int64)
@@ -600,6 +638,24 @@ class Engine:
             tseq[T:T + n] = si
             ctxl[T:T + n] = pr + 1
             bt[si, :len(s.blocks)] = s.blocks
+            if runs is not None:
+                runs[si] = (T, n, s.state_slot, p0)
+            T += n
+        return T
+
+    def _prefill(self):
+        self._next_prefill_buf()
+        b, pad = self.pb, self.pb.pad
+        budget = self.max_prefill
+        parts, rows, finishing = [], [], []
+        T = 0
+        batch = [s for s in self.running if s.n_prefilled < s.n_target]
+        for s in batch:
+            if budget <= 0:
+                break
+            n = min(budget, s.n_target - s.n_prefilled)
+            p0 = s.n_prefilled
+            parts.append((s, p0, s.tokens[p0:p0 + n]))
             s.n_prefilled += n
             T += n
             budget -= n
@@ -607,17 +663,123 @@ class Engine:
                 rows.append(T - 1)
                 finishing.append(s)
                 self.alloc.register(s.blocks[:len(s.keys)], s.keys)
+        self._fill_rows(parts)
         nrows = max(1, len(rows))
         need = any(not s.req.params.greedy for s in finishing)
         self._cand_mode = need and self._cand_ok(finishing)
         self._ctrl(_OP_PREFILL, T, nrows, need, rows + [0] * (nrows - len(rows)), len(batch), self.h_meta_p, pad)
-        self._exec_prefill(T, rows + [0] * (nrows - len(rows)), need)
+        self._exec_prefill(T, rows + [0] * (nrows - len(rows)), need, len(parts))
         self.counters["prefill_tokens"] += T
         if finishing:
             if self.dev.type == "cuda" and self.tp is None and _ASYNC_FIRST:
                 self._pick_async(finishing, b)
             else:
                 self._first_tokens(finishing, self._pick(finishing, b, list(range(len(finishing)))))
+
+    # ------------------------------------------------------------------ teacher-forced feeding
+    # A feed hands the engine the tokens of live requests instead of sampling them (trace replay, scoring): the same
+    # block pool, state slots, step metadata, step functions and graphs as generation. One feed step is one batch:
+    # portions of prompts beside single decoded tokens run together as a row batch, a step of single tokens only is a
+    # decode step. Not to be mixed with submitted requests.
+    def feed(self, entries) -> List[torch.Tensor]:
+        """entries: [(id, tokens, want)]: the next tokens of request `id` (admitted at its first entry) and the places
+        among them whose logits are wanted. Returns one CPU f32 tensor [len(want), vocab] per entry."""
+        if self.tp is not None:
+            raise NotImplementedError("feed: single-GPU engines only")
+        if self.running or self.waiting:
+            raise RuntimeError("feed: the engine is generating")
+        if len(set(e[0] for e in entries)) != len(entries):
+            raise ValueError("feed: one entry per request and step")
+        seqs = []
+        for rid, toks, want in entries:
+            s = self._fed.get(rid)
+            if s is None:
+                if len(self._fed) >= self.max_batch:
+                    raise RuntimeError(f"feed: more than {self.max_batch} live requests")
+                s = _Seq(GenRequest([], request_id=str(rid)), Future())
+                if self.slots is not None:
+                    s.state_slot = self.slots.alloc()
+                self._fed[rid] = s
+            if not len(toks):
+                raise ValueError("feed: an entry without tokens")
+            if any(not 0 <= int(t) < self.cfg.vocab for t in toks):
+                raise ValueError("feed: token outside the vocabulary")
+            if any(not 0 <= int(w) < len(toks) for w in want):
+                raise ValueError("feed: wanted place outside the entry")
+            n = s.n_fed + len(toks)
+            if n > self.ctx:
+                raise ValueError(f"feed: {n} tokens exceed the context length ({self.ctx})")
+            more = math.ceil(n / self.bs) - len(s.blocks)
+            if more > 0:
+                blocks = self.alloc.alloc(more)
+                if blocks is None:
+                    raise RuntimeError("feed: the cache pool is full")
+                s.blocks += blocks
+                if s.row >= 0:
+                    for hm in self.h_meta_d2:
+                        self._tables(hm, self.db.pad)[0][s.row, :len(s.blocks)] = s.blocks
+            seqs.append(s)
+        out = [torch.zeros(len(e[2]), self.cfg.vocab) for e in entries]
+        if all(len(e[1]) == 1 and s.n_fed > 0 for e, s in zip(entries, seqs)):
+            self._feed_decode(seqs, entries, out)
+        else:
+            self._feed_rows(seqs, entries, out)
+        return out
+
+    def _feed_decode(self, seqs, entries, out):
+        for s, e in zip(seqs, entries):
+            s.tokens.append(int(e[1][0]))
+            if s.row < 0:
+                self._assign_row(s)
+        need = any(len(e[2]) for e in entries)
+        (snap, k) = self._launch(seqs, set(), need)
+        if self.dev.type == "cuda":
+            self._ev[k].synchronize()
+        if need:
+            lg = self.db.logits[[r for r, _ in snap]].float().cpu()
+            for i, e in enumerate(entries):
+                out[i][:] = lg[i]
+
+    def _feed_rows(self, seqs, entries, out):
+        """Row batches of at most max_prefill rows and max_logit_rows wanted rows (one batch unless the step is larger)."""
+        work = [(i, s, [int(t) for t in e[1]], sorted((int(w), j) for j, w in enumerate(e[2])))
+                for i, (s, e) in enumerate(zip(seqs, entries))]
+        done = [0] * len(work)
+        while any(done[i] < len(toks) for i, _, toks, _ in work):
+            parts, rows, dest, T = [], [], [], 0
+            for i, s, toks, want in work:
+                n = min(len(toks) - done[i], self.max_prefill - T)
+                w = [(p, j) for p, j in want if done[i] <= p < done[i] + n]
+                room = self.max_logit_rows - len(rows)
+                if len(w) > room:                          # stop ahead of the first wanted row that does not fit
+                    n = w[room][0] - done[i]
+                    w = w[:room]
+                if n <= 0:
+                    continue
+                parts.append((s, s.n_fed, toks[done[i]:done[i] + n]))
+                rows += [T + p - done[i] for p, _ in w]
+                dest += [(i, j) for _, j in w]
+                s.tokens += toks[done[i]:done[i] + n]
+                s.n_fed += n
+                done[i] += n
+                T += n
+            self._next_prefill_buf()
+            self._fill_rows(parts)
+            self._exec_prefill(T, rows or [0], True, len(parts))
+            self.counters["prefill_tokens"] += T
+            if rows:
+                lg = self.pb.logits[:len(rows)].float().cpu()
+                for r, (i, j) in enumerate(dest):
+                    out[i][j] = lg[r]
+            elif self.dev.type == "cuda":
+                torch.cuda.current_stream(self.dev).synchronize()
+
+    def feed_end(self, rid):
+        """The request is finished: its blocks, state slot and decode row are free again."""
+        s = self._fed.pop(rid)
+        s.done = True
+        self._release_memory(s)
+        self._release_rows()
 
     def _first_tokens(self, seqs: List[_Seq], toks: List[int]):
         now = time.monotonic()
@@ -667,16 +829,16 @@ class Engine:
         if not hasattr(self, "_pf_pin"):
             cuda = self.dev.type == "cuda"
             nq = (self.max_prefill + 15) // 16 + self.max_batch
-            self._pf_pin = [(torch.zeros(self.max_batch, dtype=torch.int32, pin_memory=cuda),
+            self._pf_pin = [(torch.zeros(self.max_logit_rows, dtype=torch.int32, pin_memory=cuda),
                              torch.zeros(nq, 4, dtype=torch.int32, pin_memory=cuda)) for _ in range(2)]
-            self._pf_dev = (torch.zeros(self.max_batch, dtype=torch.int32, device=self.dev),
+            self._pf_dev = (torch.zeros(self.max_logit_rows, dtype=torch.int32, device=self.dev),
                             torch.zeros(nq, 4, dtype=torch.int32, device=self.dev))
 
     def _pf_graph_key(self, T: int, rows: List[int], qb, need_logits: bool):
         """The prefill graph of this chunk, if any: single GPU, one contiguous run of <= 64 tokens of one
         sequence (one query block, one logit row) -- the shape of a chat request's prompt."""
         if not (self.use_graphs and _PREFILL_GRAPHS and self.tp is None and qb is not None and len(qb) == 1
-                and len(rows) == 1 and self.model.cfg.n_expert == 0):
+                and len(rows) == 1 and self.model.cfg.n_expert == 0 and self.model.prefill_graphs):
             return None
         for Tb in self.PREFILL_GRAPH_T:
             if T <= Tb <= self.max_prefill:
@@ -685,7 +847,7 @@ class Engine:
 
     def _pf_forward(self, Tb: int, need_logits: bool):
         ld, qd = self._pf_dev
-        return self.model.forward(self.pb, self.kc, self.vc, Tb, self.bs, LlamaModel.attn_splits(Tb, self.model.Hkv),
+        return self.model.forward(self.pb, self.kc, self.vc, Tb, self.bs, self.model.n_splits(Tb),
                                   logit_rows=ld[:1], n_logits=1, qblocks=qd[:1], nqb=1, need_logits=need_logits)
 
     def _capture_prefill(self, key):
@@ -697,7 +859,7 @@ class Engine:
         torch.cuda.synchronize(self.dev)
         self.pf_graphs[key] = g
 
-    def _exec_prefill(self, T: int, rows: List[int], need_logits: bool):
+    def _exec_prefill(self, T: int, rows: List[int], need_logits: bool, nruns: int = 0):
         b = self.pb
         cuda = self.dev.type == "cuda"
         pad = b.pad
@@ -740,10 +902,13 @@ class Engine:
                 n = self._pf_forward(*key)
                 self._capture_prefill(key)
         else:
-            n = self.model.forward(b, self.kc, self.vc, T, self.bs, LlamaModel.attn_splits(T, self.model.Hkv),
+            n = self.model.forward(b, self.kc, self.vc, T, self.bs, self.model.n_splits(T),
                                    logit_rows=lr, n_logits=len(rows), qblocks=qbt, nqb=0 if qbt is None else len(qb),
-                                   need_logits=need_logits)
+                                   need_logits=need_logits, **self._state_args(nruns))
         self._gather(b, n, need_logits)
+
+    def _state_args(self, nruns: int) -> dict:
+        return {"state": self.state, "nruns": nruns} if self.slots is not None else {}
 
     CAND = 128           # TP sampling: candidates per rank and row
     PREFILL_CHUNKS = int(os.environ.get("NLS_PREFILL_CHUNKS", "4"))   # prefill chunks per step (backlog)
@@ -853,7 +1018,7 @@ class Engine:
             if op == _OP_STOP:
                 return
             if op == _OP_CAPTURE:
-                self._capture(T, LlamaModel.attn_splits(T, self.model.Hkv), dsamp=bool(dsamp))
+                self._capture(T, self.model.n_splits(T), dsamp=bool(dsamp))
                 continue
             if op == _OP_RESET:
                 if _TP_TRACE:
@@ -966,7 +1131,7 @@ class Engine:
         s.n_fed = len(s.tokens) - 1
         nb = len(s.blocks)
         for hm in self.h_meta_d2:
-            bt = hm.numpy()[_NSEG * self.db.pad:].reshape(self.max_batch, self.max_blocks)
+            bt = self._tables(hm, self.db.pad)[0]
             bt[r, :nb] = s.blocks
             bt[r, nb:] = 0
         if self.device_sampling:
@@ -1032,7 +1197,7 @@ class Engine:
         pad = self.db.pad
         h = self.h_meta_d2[k].numpy()
         ids, pos, slot, tseq, ctxl, usep = (h[i * pad:(i + 1) * pad] for i in range(_NSEG))
-        bt = h[_NSEG * pad:].reshape(self.max_batch, self.max_blocks)
+        bt, runs = self._tables(self.h_meta_d2[k], pad)
         top = max(s.row for s in launch) + 1
         Bp = self._bucket(top)
         ids[:Bp] = 0
@@ -1049,6 +1214,12 @@ class Engine:
         pos[rows] = p
         ctxl[rows] = p + 1
         slot[rows] = bt[rows, p // self.bs] * self.bs + p % self.bs
+        if runs is not None:                # every row is a run of one token; padded rows have no slot
+            runs[:Bp] = (0, 0, -1, 0)
+            runs[rows, 0] = rows
+            runs[rows, 1] = 1
+            runs[rows, 2] = [s.state_slot for s in launch]
+            runs[rows, 3] = p
         return Bp
 
     def _launch(self, launch: List[_Seq], prev: set, need: bool = False, dsamp: bool = False):
@@ -1163,15 +1334,14 @@ class Engine:
             s.blocks.append(b[0])
             if s.row >= 0:
                 for hm in self.h_meta_d2:
-                    hm.numpy()[_NSEG * self.db.pad:].reshape(self.max_batch, self.max_blocks)[s.row, len(s.blocks) - 1] = b[0]
+                    self._tables(hm, self.db.pad)[0][s.row, len(s.blocks) - 1] = b[0]
         return seqs
 
     def _preempt(self, s: _Seq):
         """Recompute preemption (no step in flight): free the sequence's blocks and decode row and put it
         back at the head of the queue; it is re-prefilled from prompt + generated tokens (the prefix cache
         usually still holds its prompt blocks) and its stream continues where it stopped."""
-        self.alloc.release(s.blocks)
-        s.blocks = []
+        self._release_memory(s)
         if s.row >= 0:
             self.rows[s.row] = None
             s.row = -1
@@ -1265,7 +1435,7 @@ class Engine:
 
     def _step_forward(self, Bp: int, ns: int, need_logits: bool, dsamp: bool):
         self.model.forward(self.db, self.kc, self.vc, Bp, self.bs, ns, feed_prev=True,
-                           need_logits=need_logits or dsamp)
+                           need_logits=need_logits or dsamp, **self._state_args(Bp))
         if dsamp:
             b = self.db
             if self.tp is None:
@@ -1279,7 +1449,7 @@ class Engine:
                                    b.ctx_len, self.d_hist, b.next_ids)
 
     def _run_decode(self, Bp: int, need_logits: bool = False, dsamp: bool = False):
-        ns = LlamaModel.attn_splits(Bp, self.model.Hkv)
+        ns = self.model.n_splits(Bp)
         if not self.use_graphs:
             self._step_forward(Bp, ns, need_logits, dsamp)
             return
@@ -1328,7 +1498,7 @@ class Engine:
         block over the whole bucket at position 0 of sequence 0 (its reads land in valid blocks, the outputs are
         discarded)."""
         if not (self.use_graphs and _PREFILL_GRAPHS and self.tp is None and self.model.cfg.n_expert == 0
-                and self.prefill_attn):
+                and self.prefill_attn and self.model.prefill_graphs):
             return
         self._pf_buffers()
         b, pad = self.pb, self.pb.pad
@@ -1360,17 +1530,20 @@ class Engine:
         h = self.h_meta_d2[0].numpy()
         h[:_NSEG * pad] = 0
         h[2 * pad:3 * pad] = -1
+        runs = self._tables(self.h_meta_d2[0], pad)[1]
+        if runs is not None:
+            runs[:] = (0, 0, -1, 0)
         self.db.meta.copy_(self.h_meta_d2[0])
         for Bp in buckets or [k for k in BUCKETS if k <= self.max_batch]:
             if (Bp, False) not in self.graphs:
                 self._ctrl(_OP_CAPTURE, Bp, 0, False, [], 0, None, 0)
-                self._capture(Bp, LlamaModel.attn_splits(Bp, self.model.Hkv))
+                self._capture(Bp, self.model.n_splits(Bp))
             # the in-graph sampling variant too (on every rank): captured lazily, it stalls the first sampled
             # burst at every bucket (an eager step + capture + two device syncs each, ~0.2-0.4 s over a
             # 512-request ramp). Padded rows have ctx 0 and every row's params are greedy here: no history writes.
             if self.device_sampling and (Bp, False, True) not in self.graphs:
                 self._ctrl(_OP_CAPTURE, Bp, 0, False, [], 0, None, 0, dsamp=True)
-                self._capture(Bp, LlamaModel.attn_splits(Bp, self.model.Hkv), dsamp=True)
+                self._capture(Bp, self.model.n_splits(Bp), dsamp=True)
 
     # ------------------------------------------------------------------ completion
     def _append(self, s: _Seq, t: int):
@@ -1421,9 +1594,7 @@ class Engine:
         s.t_done = time.monotonic()
         if finish in ("stop", "length") and s.max_new > 0:     # admission's expected-growth estimate
             self.gen_ratio += 0.1 * (min(1.0, (len(s.tokens) - s.n_prompt) / s.max_new) - self.gen_ratio)
-        if s.blocks:
-            self.alloc.release(s.blocks)
-            s.blocks = []
+        self._release_memory(s)
         gen = s.generated
         text = ""
         if self.tok is not None:

@@ -369,6 +369,15 @@ class LlamaModel:
         return added
 
     # ------------------------------------------------------------------ buffers
+    format = "gguf"
+    recurrent = False             # no per-sequence state beside the paged KV cache
+    prefill_graphs = True
+
+    @property
+    def kv_token_bytes(self) -> int:
+        """Cache bytes of one token over all layers (this shard)."""
+        return 2 * self.cfg.n_layer * self.Hkv * self.D * (torch.finfo(self.kv_dtype).bits // 8)
+
     @property
     def kv_dtype(self) -> torch.dtype:
         """Paged KV cache element type: NLS_KV_DTYPE=bf16 (default) | fp8 (OCP e4m3, half the bytes)."""
@@ -438,6 +447,9 @@ class LlamaModel:
                 yexp=torch.zeros(pad * k, cfg.d_model, dtype=torch.float32, device=dev),
             )
         return b
+
+    def n_splits(self, T: int) -> int:
+        return self.attn_splits(T, self.Hkv)
 
     @staticmethod
     def attn_splits(T: int, Hkv: int) -> int:

@@ -1,0 +1,397 @@
+"""Decoder stacks assembled from a config: a list of layers, each a mixer plus an optional feed-forward.
+
+A mixer or feed-forward is a class that loads its weights, adds its step buffers, and runs on the rows of a step; the
+per-token cache rows (paged) and the per-sequence states (slots) of all layers belong to the engine, which sees them as
+`kv_cache` / `state_pool`. Everything runs on the HIP kernels of csrc/stack (ops/stack.py): bf16 operands with an f32
+residual, or `dtype=torch.float32` for 32-bit throughout.
+
+Rows of a step are runs of consecutive tokens of one sequence (whole prompts, portions of any size, single decoded
+tokens), all in one batch:
+  runs     [sequences][4]: first row, rows, state slot, first position   (recurrent layers)
+  slot / tok_seq / ctx_len / block_tables                                (paged cache, as in models/llama.py)
+"""
+from __future__ import annotations
+
+import os
+from dataclasses import dataclass, field
+from typing import Dict, List, Optional
+
+import torch
+
+from ..ops import stack as K
+from ..ops import rope_table
+from ..safetensors_io import SafetensorsReader
+from .llama import ShardSpec
+from .stack_config import StackConfig
+
+_SPLIT_WG = 256          # target workgroups of a decode attention launch (one per CU)
+_SPLIT_CAP = 64
+
+
+@dataclass
+class StackBuffers:
+    """Device buffers of one step of up to `cap` tokens (static for hipGraph capture). Linear-layer inputs have rows of
+    ops.stack.act_ld columns whose padding stays zero."""
+    cap: int
+    pad: int
+    meta: torch.Tensor
+    ids: torch.Tensor
+    pos: torch.Tensor
+    slot: torch.Tensor
+    tok_seq: torch.Tensor
+    ctx_len: torch.Tensor
+    use_prev: torch.Tensor
+    block_tables: torch.Tensor
+    runs: torch.Tensor
+    x: torch.Tensor                     # f32 residual
+    xb: Optional[torch.Tensor]          # its bf16 rounding (None: 32-bit model, the residual itself is the operand)
+    y: torch.Tensor                     # f32 sublayer output
+    hn: torch.Tensor                    # normed rows of the head
+    logits: torch.Tensor
+    next_ids: torch.Tensor
+    shared: Dict[tuple, torch.Tensor] = field(default_factory=dict)    # scratch shared between layers
+    launches: Dict[tuple, object] = field(default_factory=dict)
+
+    @property
+    def act(self) -> torch.Tensor:
+        return self.x if self.xb is None else self.xb
+
+
+class _Part:
+    """A mixer or feed-forward of layer i: weights `w(name)` are '<layer>.<mix|mlp>.<name>'."""
+
+    def __init__(self, model: "StackModel", i: int, cfg, prefix: str):
+        self.m, self.i, self.cfg, self.prefix = model, i, cfg, prefix
+
+    def t(self, name: str) -> torch.Tensor:
+        return self.m.reader.tensor(self.prefix + name)
+
+    def vec(self, name: str) -> torch.Tensor:
+        return self.t(name).to(device=self.m.device, dtype=torch.float32).reshape(-1).contiguous()
+
+    def lin(self, w, shape=None) -> K.PackedLinear:
+        w = self.t(w) if isinstance(w, str) else w
+        if shape is not None and tuple(w.shape) != tuple(shape):
+            raise ValueError(f"{self.prefix}: a weight of shape {tuple(w.shape)}, expected {tuple(shape)}")
+        p = K.PackedLinear(w, self.m.f32, self.m.device)
+        self.m.weight_bytes += p.nbytes
+        return p
+
+    def scratch(self, b: StackBuffers, name: str, rows: int, cols: int, dtype=None) -> torch.Tensor:
+        """A zeroed [rows, cols] buffer shared by every layer that asks for this name and shape (same layout: what one
+        layer leaves in the padding columns is what the next would)."""
+        key = (name, rows, cols, dtype or self.m.dtype)
+        if key not in b.shared:
+            b.shared[key] = torch.zeros(rows, cols, dtype=dtype or self.m.dtype, device=self.m.device)
+        return b.shared[key]
+
+
+class WkvMixer(_Part):
+    """Token-shift mixes -> r | k | v | gate | decay projections -> gated linear recurrence with a per-channel decay
+    -> per-head RMS norm, norm weight and gate -> output projection."""
+    SHIFTS = ("r", "k", "v", "g", "w")
+
+    def __init__(self, model, i, cfg, prefix):
+        super().__init__(model, i, cfg, prefix)
+        d, HD = model.cfg.d_model, cfg.heads * cfg.dim
+        if cfg.dim > 256:
+            raise ValueError(f"wkv head dim {cfg.dim} > 256")
+        self.mu = torch.stack([self.vec("mu." + s) for s in self.SHIFTS]).contiguous()
+        self.r, self.k, self.v, self.g = (self.lin(n, (HD, d)) for n in ("r", "k", "v", "g"))
+        self.w1, self.w2, self.o = self.lin("w1"), self.lin("w2"), self.lin("o", (d, HD))
+        self.w0, self.u, self.norm = self.vec("w0"), self.vec("u"), self.vec("norm")
+
+    def state_shapes(self):
+        c = self.cfg
+        return {"S": c.heads * c.dim * c.dim, "prev": self.m.cfg.d_model}
+
+    def bind(self, b: StackBuffers) -> dict:
+        d, HD, P = self.m.cfg.d_model, self.cfg.heads * self.cfg.dim, b.pad
+        mix = self.scratch(b, "wkv.mix", len(self.SHIFTS) * P, K.act_ld(d)).view(len(self.SHIFTS), P, -1)
+        ld = K.act_ld(HD)
+        r, k, v, g, out = (self.scratch(b, "wkv." + n, P, ld) for n in ("r", "k", "v", "g", "out"))
+        low = self.scratch(b, "wkv.low", P, K.act_ld(self.w1.N))
+        w, o = (self.scratch(b, "wkv." + n, P, ld, torch.float32) for n in ("w", "o"))
+        return dict(
+            mix=mix, r=r, k=k, v=v, g=g, w=w, o=o, out=out,
+            proj=K.LinLaunch([K.Seg(self.r, mix[0], r), K.Seg(self.k, mix[1], k), K.Seg(self.v, mix[2], v),
+                              K.Seg(self.g, mix[3], g, "silu"), K.Seg(self.w1, mix[4], low, "tanh")]),
+            decay=K.LinLaunch([K.Seg(self.w2, low, w, "decay", bias=self.w0)]),
+            o_proj=K.LinLaunch([K.Seg(self.o, out, b.y)]))
+
+    def run(self, b: StackBuffers, e: dict, cache, state, step: "_Step"):
+        c, st, T = self.cfg, step.st, step.T
+        S, prev = state["S"], state["prev"]
+        K.shift_mix(b.x, self.mu, prev, e["mix"], b.runs, b.tok_seq, T, st)
+        e["proj"].run(T, st)
+        e["decay"].run(T, st)
+        K.wkv_scan(e["r"], e["k"], e["v"], e["w"], self.u, e["o"], S, b.x, prev, b.runs, step.nruns, c.heads, c.dim, st)
+        K.wkv_out(e["o"], self.norm, e["g"], e["out"], c.heads, c.dim, T, self.m.cfg.eps, st)
+        e["o_proj"].run(T, st)
+
+
+class LatentMixer(_Part):
+    """Latent attention. The cache holds, per token, the normed latent and one rotated key part shared by all heads; a
+    layer with kv_from reads an earlier layer's rows. The key up-projection is folded into the query and the value
+    up-projection applied to the attended latent, so every head attends over the same cached rows."""
+
+    def __init__(self, model, i, cfg, prefix):
+        super().__init__(model, i, cfg, prefix)
+        c, d = cfg, model.cfg.d_model
+        H, D, RD, VD, R, Q = c.heads, c.dim, c.rot_dim, c.vdim, c.kv_rank, c.q_rank
+        self.Rp, self.rp = K.latent_pad(R), K.rot_pad(RD)
+        self.Dp = self.Rp + self.rp
+        self.Dq = K.act_ld(D)                              # unrotated query columns per head
+        self.RD4 = K.pad_to(RD, 4)
+        self.dq, self.dqn = self.lin("dq", (Q, d)), self.vec("dq.norm")
+        self.owner = c.kv_from is None
+        if self.owner:
+            self.dkv, self.dkvn = self.lin("dkv", (R + RD, d)), self.vec("dkv.norm")
+        uq = self.t("uq").to(model.device).view(H, D + RD, Q)
+        zero = uq.new_zeros
+        self.uqn = self.lin(torch.cat([uq[:, :D], zero(H, self.Dq - D, Q)], 1).reshape(H * self.Dq, Q))
+        self.uqr = self.lin(torch.cat([uq[:, D:], zero(H, self.RD4 - RD, Q)], 1).reshape(H * self.RD4, Q))
+        self.uk = self.lin(self.t("uk").to(model.device).view(H, D, R).transpose(1, 2).contiguous())   # [H][R][D]
+        self.uv = self.lin(self.t("uv").to(model.device).view(H, VD, R))                               # [H][VD][R]
+        self.g, self.o = self.lin("g", (H, d)), self.lin("o", (d, H * VD))
+        self.cs = model.rope(c.rot_base, RD)
+
+    @property
+    def cache_width(self) -> int:
+        return self.Dp if self.owner else 0
+
+    def bind(self, b: StackBuffers) -> dict:
+        c, P = self.cfg, b.pad
+        H, f = c.heads, torch.float32
+        dq = self.scratch(b, "lat.dq", P, c.q_rank, f)
+        dkv = self.scratch(b, "lat.dkv", P, c.kv_rank + c.rot_dim, f) if self.owner else None
+        gate = self.scratch(b, "lat.gate", P, H, f)
+        cq = self.scratch(b, "lat.cq", P, K.act_ld(c.q_rank))
+        qn = self.scratch(b, "lat.qn", P, H * self.Dq)
+        # (columns between the written parts stay zero: the buffer is shared only between equal layouts)
+        q = self.scratch(b, f"lat.q{c.kv_rank}.{c.rot_dim}", P, H * self.Dp)
+        lat = self.scratch(b, f"lat.o{c.kv_rank}", P, H * self.Rp)
+        ao = self.scratch(b, "lat.ao", P, K.act_ld(H * c.vdim))
+        hb = (H + 15) // 16
+        n = (_SPLIT_WG // hb + 1) * H
+        po = self.scratch(b, "lat.po", 1, n * self.Rp, f)
+        pm = self.scratch(b, "lat.pm", 1, n * 2, f)
+        down = [K.Seg(self.dq, b.act, dq), K.Seg(self.g, b.act, gate, "sigmoid")]
+        if self.owner:
+            down.append(K.Seg(self.dkv, b.act, dkv))
+        return dict(
+            dq=dq, dkv=dkv, cq=cq, q=q, lat=lat, part=(po, pm), hb=hb,
+            down=K.LinLaunch(down),
+            up=K.LinLaunch([K.Seg(self.uqn, cq, qn),
+                            K.Seg(self.uqr, cq, q, "rope", ycol=self.Rp, block=(self.RD4, self.Dp),
+                                  rope=(self.cs, b.pos, c.rot_dim // 2))]),
+            absorb=K.LinLaunch([K.Seg(self.uk, qn, q, xgs=self.Dq, ygs=self.Dp)]),
+            value=K.LinLaunch([K.Seg(self.uv, lat, ao, "gate", xgs=self.Rp, ygs=c.vdim, gate=gate)]),
+            o_proj=K.LinLaunch([K.Seg(self.o, ao, b.y)]))
+
+    def run(self, b: StackBuffers, e: dict, cache, state, step: "_Step"):
+        c, st, T = self.cfg, step.st, step.T
+        rows = cache[self.i if self.owner else c.kv_from]
+        e["down"].run(T, st)
+        K.latent_rows(e["dq"], self.dqn, e["cq"], e["dkv"], self.dkvn if self.owner else None, c.kv_rank, self.Rp,
+                      c.rot_dim, self.cs, b.pos, b.slot, rows if self.owner else None, T, self.m.cfg.eps, st)
+        e["up"].run(T, st)
+        e["absorb"].run(T, st)
+        ns = 1 if self.m.f32 else max(1, min(_SPLIT_CAP, _SPLIT_WG // (T * e["hb"])))
+        K.latent_attention(e["q"], rows, e["lat"], e["part"], b.block_tables, step.block_size, b.tok_seq, b.ctx_len, T,
+                           c.heads, ns, self.Rp, self.rp, c.scale, st)
+        e["value"].run(T, st)
+        e["o_proj"].run(T, st)
+
+
+class MoeFeedForward(_Part):
+    """Routed experts (two matrices, squared-relu) chosen by group-limited sigmoid scores, plus a shared expert. Leaves
+    the experts' output rows in `ye`; the caller's output norm combines them."""
+
+    def __init__(self, model, i, cfg, prefix):
+        super().__init__(model, i, cfg, prefix)
+        d, E = model.cfg.d_model, cfg.experts
+        self.router = self.lin("router", (E, d))
+        self.up = self.lin(torch.stack([self.t(f"e{j}.up") for j in range(E)]), (E, cfg.ff, d))
+        self.down = self.lin(torch.stack([self.t(f"e{j}.down") for j in range(E)]), (E, d, cfg.ff))
+        if cfg.shared_ff:
+            self.sup, self.sdown = self.lin("shared.up", (cfg.shared_ff, d)), self.lin("shared.down", (d, cfg.shared_ff))
+
+    def bind(self, b: StackBuffers) -> dict:
+        c, P = self.cfg, b.pad
+        k = c.top
+        act = self.m.cfg.design.expert_act
+        key = ("plan", c.experts, k, c.groups, c.keep, c.scale)
+        plan = b.launches.get(key)
+        if plan is None:
+            plan = b.launches[key] = K.MoePlan(P, c.experts, k, c.groups, c.keep, c.scale, self.m.device)
+        z = self.scratch(b, "moe.z", P, c.experts, torch.float32)
+        h = self.scratch(b, "moe.h", P * k, K.act_ld(c.ff))
+        ye = self.scratch(b, "moe.y", P * (k + 1), self.m.cfg.d_model, torch.float32)
+        first = [K.Seg(self.router, b.act, z)]
+        down = [K.Seg(self.down, h, ye, routed=(plan.rows, 1))]
+        if c.shared_ff:
+            hs = self.scratch(b, "moe.hs", P, K.act_ld(c.shared_ff))
+            first.append(K.Seg(self.sup, b.act, hs, act))
+            down.append(K.Seg(self.sdown, hs, ye, yrow=P * k))
+        return dict(plan=plan, z=z, ye=ye, first=K.LinLaunch(first), shared_row0=P * k if c.shared_ff else -1,
+                    up=K.LinLaunch([K.Seg(self.up, b.act, h, act, routed=(plan.rows, k))], plan),
+                    down=K.LinLaunch(down, plan))
+
+    def run(self, b: StackBuffers, e: dict, step: "_Step"):
+        T, st = step.T, step.st
+        e["first"].run(T, st)
+        e["plan"].run(e["z"], T, st)
+        e["up"].run(T, st)
+        e["down"].run(T, st)
+
+
+MIXERS = {"wkv": WkvMixer, "latent_attention": LatentMixer}
+FEED_FORWARDS = {"moe": MoeFeedForward}
+
+
+@dataclass
+class _Step:
+    T: int
+    nruns: int
+    block_size: int
+    st: int
+
+
+class StackModel:
+    """What the engine drives: step buffers, paged cache rows, state slots and `forward`."""
+
+    format = "safetensors"
+    prefill_graphs = False        # (the captured single-prompt prefill of the GGUF families)
+
+    def __init__(self, path: str, device="cuda:0", dtype: torch.dtype = torch.bfloat16, shard: ShardSpec = ShardSpec(),
+                 comm=None, ctx: Optional[int] = None):
+        self.device = torch.device(device)
+        if self.device.type != "cuda":
+            raise RuntimeError("stack models run on the GPU kernels only")
+        if shard.size > 1:
+            raise NotImplementedError("tensor / expert parallelism is not supported for stack models")
+        if dtype not in (torch.bfloat16, torch.float32):
+            raise ValueError("stack models run in bfloat16 or float32")
+        K.lib()
+        self.path, self.dtype, self.f32 = path, dtype, dtype == torch.float32
+        self.shard, self.comm, self.ep = shard, comm, False
+        self.reader = r = SafetensorsReader(os.path.join(path, "model.safetensors"))
+        self.cfg = cfg = StackConfig.from_dir(path, lambda n: r.shape(n) if n in r else None)
+        if ctx is not None:
+            cfg.ctx = int(ctx)
+        if cfg.d_model > 16384:
+            raise ValueError("stack models take widths up to 16384")
+        if max([L.mlp.experts for L in cfg.layers if L.mlp is not None], default=0) > 512:
+            raise ValueError("stack models take up to 512 experts")
+        self.weight_bytes = 0
+        self._rope = {}
+        dev = self.device
+        vec = lambda n: r.tensor(n).to(device=dev, dtype=torch.float32).contiguous()      # noqa: E731
+        self.embed = r.tensor("embed").to(device=dev, dtype=torch.bfloat16).contiguous()
+        self.weight_bytes += self.embed.numel() * 2
+        self.layers = []
+        for i, L in enumerate(cfg.layers):
+            p = f"l{i}."
+            mix = MIXERS[L.mixer.kind](self, i, L.mixer, p + "mix.")
+            mlp = FEED_FORWARDS[L.mlp.kind](self, i, L.mlp, p + "mlp.") if L.mlp is not None else None
+            self.layers.append((mix, vec(p + "norm1"), mlp, vec(p + "norm2") if mlp is not None else None))
+        self.final_norm = vec("final.norm")
+        self.head = K.PackedLinear(r.tensor("head"), self.f32, dev)
+        self.weight_bytes += self.head.nbytes
+        self.vocab_lo, self.vocab_hi = 0, cfg.vocab
+
+    # ---- what the engine asks
+    @property
+    def recurrent(self) -> bool:
+        return self.cfg.recurrent
+
+    @property
+    def kv_token_bytes(self) -> int:
+        return sum(m.cache_width for m, *_ in self.layers if isinstance(m, LatentMixer)) * self.dtype.itemsize
+
+    def n_splits(self, T: int) -> int:
+        return 1                      # (each latent layer sizes its own splits, LatentMixer.run)
+
+    def rope(self, base: float, dims: int) -> torch.Tensor:
+        key = (base, dims)
+        if key not in self._rope:
+            self._rope[key] = rope_table(self.cfg.ctx, dims, base, self.device)
+        return self._rope[key]
+
+    def kv_cache(self, num_blocks: int, block_size: int = 16):
+        """Paged rows of the layers that own a cache: {layer: [slots, width]}."""
+        return {m.i: torch.zeros(num_blocks * block_size, m.cache_width, dtype=self.dtype, device=self.device)
+                for m, *_ in self.layers if isinstance(m, LatentMixer) and m.owner}, None
+
+    def state_pool(self, slots: int):
+        """Per-sequence states, f32: {layer: {name: [slots, n]}}. A sequence's first run (position 0) ignores what its
+        slot holds, so a reused slot needs no clearing."""
+        return {m.i: {k: torch.zeros(slots, n, dtype=torch.float32, device=self.device)
+                      for k, n in m.state_shapes().items()}
+                for m, *_ in self.layers if hasattr(m, "state_shapes")}
+
+    def step_buffers(self, cap: int, max_seqs: int, max_blocks: int, logit_rows: Optional[int] = None) -> StackBuffers:
+        """Step metadata is ONE int32 tensor, as in LlamaModel.step_buffers, with the runs table behind the block tables:
+        [ids | pos | slot | tok_seq | ctx_len | use_prev | block_tables | runs]."""
+        cfg, dev = self.cfg, self.device
+        pad = K.pad_to(cap, 64)
+        nb = max_seqs * max_blocks
+        meta = torch.zeros(6 * pad + nb + 4 * max_seqs, dtype=torch.int32, device=dev)
+        seg = [meta[i * pad:(i + 1) * pad] for i in range(6)]
+        f = dict(dtype=torch.float32, device=dev)
+        ld = K.act_ld(cfg.d_model)
+        nl = min(pad, max(64, max_seqs, logit_rows or 0))
+        b = StackBuffers(
+            cap=cap, pad=pad, meta=meta, ids=seg[0], pos=seg[1], slot=seg[2], tok_seq=seg[3], ctx_len=seg[4],
+            use_prev=seg[5], block_tables=meta[6 * pad:6 * pad + nb].view(max_seqs, max_blocks),
+            runs=meta[6 * pad + nb:].view(max_seqs, 4),
+            x=torch.zeros(pad, ld, **f), xb=None if self.f32 else torch.zeros(pad, ld, dtype=self.dtype, device=dev),
+            y=torch.zeros(pad, cfg.d_model, **f), hn=torch.zeros(pad, ld, dtype=self.dtype, device=dev),
+            logits=torch.zeros(nl, cfg.vocab, **f), next_ids=torch.zeros(pad, dtype=torch.int32, device=dev))
+        b.slot.fill_(-1)
+        b.runs[:, 2] = -1
+        for i, (mix, _, mlp, _) in enumerate(self.layers):
+            b.launches[i, "mix"] = mix.bind(b)
+            if mlp is not None:
+                b.launches[i, "mlp"] = mlp.bind(b)
+        b.launches["head"] = K.LinLaunch([K.Seg(self.head, b.hn, b.logits)])
+        return b
+
+    # ---- forward
+    @torch.no_grad()
+    def forward(self, b: StackBuffers, kc, vc, T: int, block_size: int, n_split: int = 1,
+                logit_rows: Optional[torch.Tensor] = None, n_logits: Optional[int] = None, qblocks=None, nqb: int = 0,
+                feed_prev: bool = False, need_logits: bool = True, state=None, nruns: Optional[int] = None,
+                taps: Optional[list] = None):
+        """One step of T rows: logits (of `logit_rows`, or of every row) in b.logits[:n], their greedy ids in
+        b.next_ids[:n]. `taps` (a list) receives the residual after every layer."""
+        if T < 1 or T > b.pad:
+            raise ValueError(f"step of {T} rows, buffers hold {b.pad}")
+        cfg = self.cfg
+        st = K.stream(self.device)
+        step = _Step(T, T if nruns is None else nruns, block_size, st)
+        K.embed(b.ids, self.embed, b.x, b.xb, T, st, prev=(b.next_ids, b.use_prev) if feed_prev else None)
+        last = len(self.layers) - 1
+        direct = logit_rows is None
+        for i, (mix, norm1, mlp, norm2) in enumerate(self.layers):
+            fin = dict(out_norm=self.final_norm, out=b.hn) if direct and i == last else {}
+            mix.run(b, b.launches[i, "mix"], kc, state.get(i) if state else None, step)
+            K.norm_add(b.y, norm1, b.x, b.xb, T, cfg.eps, st, **(fin if mlp is None else {}))
+            if mlp is not None:
+                e = b.launches[i, "mlp"]
+                mlp.run(b, e, step)
+                K.norm_add(e["ye"], norm2, b.x, b.xb, T, cfg.eps, st, plan=e["plan"], shared_row0=e["shared_row0"], **fin)
+            if taps is not None:
+                taps.append(b.x[:T, :cfg.d_model].clone())
+        n = T
+        if not direct:
+            n = int(n_logits)
+            if n == 0:
+                return 0
+            K.layer_norm(b.x, logit_rows, self.final_norm, b.hn, n, cfg.eps, st)
+        if n > b.logits.shape[0]:
+            raise ValueError(f"{n} logit rows, buffers hold {b.logits.shape[0]}")
+        b.launches["head"].run(n, st)
+        K.argmax(b.logits, n, b.next_ids, st)
+        return n

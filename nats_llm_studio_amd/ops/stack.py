@@ -1,0 +1,341 @@
+"""Device ops of the config-driven decoder stacks: ctypes bindings of `_stack.so` (csrc/stack/*.hip, gfx950).
+
+GPU tensors only: there is no eager form of these ops, a missing library raises. Operands are bf16 (f32 accumulation,
+f32 norms / routing / softmax / recurrences) or, for 32-bit models, f32 throughout (f32 MFMA)."""
+from __future__ import annotations
+
+import ctypes
+import os
+from typing import List, Optional
+
+import torch
+
+_PKG = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+LIB_PATH = os.environ.get("NLS_STACK_SO") or os.path.join(_PKG, "_stack.so")
+
+P, I, L, F = ctypes.c_void_p, ctypes.c_int, ctypes.c_long, ctypes.c_float
+SEGS = 6
+EPI = {"none": 0, "silu": 1, "tanh": 2, "sigmoid": 3, "relu2": 4, "decay": 5, "gate": 6, "rope": 7}
+NO_BLOCK = 1 << 30       # LinSeg.cb: output columns are not blocked
+
+
+class LinSeg(ctypes.Structure):
+    """csrc/stack/lin.h LinSeg."""
+    _fields_ = [("w", P), ("x", P), ("y", P), ("bias", P), ("gate", P), ("cs", P), ("pos", P), ("rows", P), ("xmap", P),
+                ("wstride", L), ("ldx", L), ("ldy", L), ("xgs", L), ("ygs", L),
+                ("N", I), ("nsub", I), ("M", I), ("ng", I), ("epi", I), ("yact", I), ("cb", I), ("cstep", I),
+                ("xdiv", I), ("ldg", I), ("half", I), ("pad0", I)]
+
+
+class LinArgs(ctypes.Structure):
+    _fields_ = [("s", LinSeg * SEGS), ("tiles", P), ("ntiles", P), ("nseg", I), ("maxtiles", I),
+                ("begin", I * (SEGS + 1)), ("nmt", I * SEGS)]
+
+
+_SIGS = {
+    "nls_lin_args_size": [],
+    "nls_lin_small": [P, I, I, I, P],
+    "nls_lin_gemm": [P, I, I, P],
+    "nls_stack_embed": [P, P, P, P, I, I, P, P, L, I, P],
+    "nls_norm_add": [P, L, P, I, L, P, P, P, L, P, P, L, I, I, F, I, P],
+    "nls_layer_norm": [P, L, P, P, P, L, I, I, F, I, P],
+    "nls_latent_rows": [P, L, I, P, P, L, P, L, I, I, I, P, P, P, P, P, L, I, F, I, P],
+    "nls_stack_argmax": [P, L, I, P, I, P],
+    "nls_moe_plan": [P, L, I, I, I, I, I, F, P, P, I, P, P, P, I, P],
+    "nls_shift_mix": [P, L, P, P, L, P, L, L, P, P, I, I, I, P],
+    "nls_wkv_scan": [P, P, P, L, P, L, P, P, L, P, L, P, L, P, L, I, P, I, I, I, I, P],
+    "nls_wkv_out": [P, L, P, P, L, P, L, I, I, I, F, I, P],
+    "nls_latent_attn": [P, P, P, P, P, P, I, I, P, P, I, I, I, I, I, F, I, P],
+}
+
+_lib = None
+
+
+def lib():
+    global _lib
+    if _lib is None:
+        if not os.path.exists(LIB_PATH):
+            raise RuntimeError(f"HIP kernel library missing: {LIB_PATH} (run `python -m nats_llm_studio_amd.build`)")
+        lb = ctypes.CDLL(LIB_PATH)
+        for name, args in _SIGS.items():
+            fn = getattr(lb, name)
+            fn.argtypes = args
+            fn.restype = I
+        if lb.nls_lin_args_size() != ctypes.sizeof(LinArgs):
+            raise RuntimeError("stale _stack.so: LinArgs layout mismatch (rebuild the kernels)")
+        _lib = lb
+    return _lib
+
+
+def _check(rc: int, name: str):
+    if rc != 0:
+        raise RuntimeError(f"{name} failed with code {rc}")
+
+
+def _p(t: Optional[torch.Tensor]):
+    return None if t is None else t.data_ptr()
+
+
+def stream(dev) -> int:
+    return torch.cuda.current_stream(dev).cuda_stream
+
+
+def pad_to(n: int, m: int) -> int:
+    return (n + m - 1) // m * m
+
+
+def act_ld(n: int) -> int:
+    """Row stride of an activation that feeds a linear layer of n inputs: the packed weights' padded K."""
+    return pad_to(n, 64)
+
+
+# ---------------------------------------------------------------------------
+# Linear layers
+# ---------------------------------------------------------------------------
+
+class PackedLinear:
+    """[groups, N, K] weights in the packed layout of csrc/stack/lin.h (1 KiB sub-tiles in MFMA fragment order), bf16
+    or f32. A plain matrix is one group; experts and per-head products are stacked groups."""
+
+    def __init__(self, w: torch.Tensor, f32: bool, device):
+        if w.dim() == 2:
+            w = w[None]
+        G, N, K = w.shape
+        self.groups, self.N, self.K, self.f32 = G, N, K, f32
+        dt, ks, el = (torch.float32, 16, 4) if f32 else (torch.bfloat16, 32, 8)
+        Np, Kp = pad_to(N, 16), act_ld(K)
+        self.nsub = Kp // ks
+        self.data = torch.empty(G, Np * Kp, dtype=dt, device=device)
+        step = max(1, (1 << 28) // (Np * Kp))               # groups per conversion pass
+        for g0 in range(0, G, step):
+            a = w[g0:g0 + step].to(device=device, dtype=dt)
+            a = torch.nn.functional.pad(a, (0, Kp - K, 0, Np - N))
+            a = a.view(-1, Np // 16, 16, Kp // ks, 4, el).permute(0, 1, 3, 4, 2, 5)
+            self.data[g0:g0 + step] = a.reshape(-1, Np * Kp)
+        self.wstride = Np * Kp * dt.itemsize
+
+    @property
+    def nbytes(self) -> int:
+        return self.data.numel() * self.data.element_size()
+
+
+class Seg:
+    """One segment of a LinLaunch. y / x: 2-D buffers (row stride = their stride(0)); ycol / xcol: first column.
+    xgs / ygs: column step per group. block = (cb, cstep): output column n -> (n / cb) * cstep + n % cb.
+    routed = (entry list, xdiv): the rows are routed entries (x row = entry / xdiv, y row = entry).
+    rope = (table, pos, pairs)."""
+
+    def __init__(self, w: PackedLinear, x: torch.Tensor, y: torch.Tensor, epi: str = "none", ycol: int = 0,
+                 xcol: int = 0, xgs: int = 0, ygs: int = 0, block=None, bias=None, gate=None, routed=None, rope=None,
+                 yrow: int = 0):
+        if x.stride(1) != 1 or y.stride(1) != 1:
+            raise ValueError("row-major operands")
+        if xcol + (0 if routed else (w.groups - 1) * xgs) + act_ld(w.K) > x.stride(0):
+            raise ValueError(f"x rows ({x.stride(0)}) do not cover the padded K of {w.K} inputs")
+        if x.dtype != w.data.dtype:
+            raise TypeError(f"activations must be {w.data.dtype}, got {x.dtype}")
+        if (xcol * x.element_size()) % 16 or (x.stride(0) * x.element_size()) % 16 or (xgs * x.element_size()) % 16:
+            raise ValueError("activation rows must be 16-byte aligned")
+        self.w, self.y, self.x = w, y, x
+        self.rows_cap = min(x.shape[0] * (routed[1] if routed else 1), y.shape[0] - yrow)
+        s = self.s = LinSeg()
+        s.w = w.data.data_ptr()
+        s.x = x.data_ptr() + xcol * x.element_size()
+        s.y = y.data_ptr() + (yrow * y.stride(0) + ycol) * y.element_size()
+        s.bias, s.gate = _p(bias), _p(gate)
+        s.ldg = gate.stride(0) if gate is not None else 0
+        s.wstride, s.ldx, s.ldy, s.xgs, s.ygs = w.wstride, x.stride(0), y.stride(0), xgs, ygs
+        s.N, s.nsub, s.ng, s.epi = w.N, w.nsub, w.groups, EPI[epi]
+        s.yact = int(y.dtype != torch.float32)
+        s.cb, s.cstep = block if block else (NO_BLOCK, 0)
+        s.xdiv = 1
+        if routed:
+            s.rows, s.xdiv = routed[0].data_ptr(), routed[1]
+        if rope:
+            s.cs, s.pos, s.half = rope[0].data_ptr(), rope[1].data_ptr(), rope[2]
+        self.keep = (bias, gate, routed, rope)
+
+
+GEMM_TILES = ((64, 64), (128, 64), (128, 128), (256, 128), (256, 256))     # (weight rows, rows) of lin_gemm's cfg
+
+
+class LinLaunch:
+    """A launch of up to SEGS independent linear layers, bound to its buffers once (only the row count and the launch
+    config change from step to step)."""
+
+    def __init__(self, segs: List[Seg], plan: "MoePlan" = None):
+        self.segs, self.plan = segs, plan
+        self.f32 = int(segs[0].w.f32)
+        self.a = LinArgs()
+        for i, s in enumerate(segs):
+            self.a.s[i] = s.s
+        self.a.nseg = len(segs)
+        if plan is not None:
+            self.a.tiles, self.a.ntiles = plan.tiles.data_ptr(), plan.ntiles.data_ptr()
+        self._cfg = {}
+
+    def _tiles(self, bn: int, bm: int, M: int) -> int:
+        n = 0
+        for s in self.segs:
+            nt = (s.w.N + bn - 1) // bn
+            n += nt * (min(self.a.maxtiles, self._routed_tiles(bm, M)) if s.s.rows else s.w.groups * ((M + bm - 1) // bm))
+        return n
+
+    def _routed_tiles(self, bm: int, M: int) -> int:
+        return self.plan.expect_tiles(M, bm)
+
+    def config(self, M: int):
+        """(gemm?, a, b): few-row kernel with a 16-row tiles and b waves, or GEMM config a."""
+        bm = self.plan.bm(M) if self.plan is not None else None
+        if bm is not None and bm <= 32 or bm is None and M <= 64:
+            mt = (bm or pad_to(M, 16)) // 16
+            mt = 1 if mt <= 1 else (2 if mt == 2 else 4)
+            n = self._tiles(16, 16 * mt, M)
+            ns = max(s.w.nsub for s in self.segs)
+            nw = 4 if n >= 1536 or ns <= 16 else (8 if n >= 512 or mt > 1 or ns <= 64 else 16)
+            return False, mt, nw
+        for c in (4, 3, 2, 1, 0):
+            bn, b = GEMM_TILES[c]
+            if bm is not None and b != bm:
+                continue
+            if c in (0,) or self._tiles(bn, b, M) >= 224:
+                return True, c, 0
+        return True, (2 if bm == 128 else 0), 0
+
+    def run(self, M: int, st: int, M_of: Optional[dict] = None):
+        if self.plan is not None:
+            self.a.maxtiles = self.plan.max_tiles(M)
+        for i, s in enumerate(self.segs):
+            if (M * self.plan.top if s.s.rows else M) > s.rows_cap:
+                raise ValueError(f"linear launch: {M} rows but the buffers hold {s.rows_cap}")
+            self.a.s[i].M = M
+        cfg = self._cfg.get(M)
+        if cfg is None:
+            if len(self._cfg) > 4096:
+                self._cfg.clear()
+            cfg = self._cfg[M] = self.config(M)
+        if cfg[0]:
+            _check(lib().nls_lin_gemm(ctypes.byref(self.a), self.f32, cfg[1], st), "nls_lin_gemm")
+        else:
+            _check(lib().nls_lin_small(ctypes.byref(self.a), self.f32, cfg[1], cfg[2], st), "nls_lin_small")
+
+
+class MoePlan:
+    """Expert choice and routed-entry lists of one step (csrc/stack/stack_ops.hip moe_plan_kernel), shared by the layers
+    of a step. Scores: sigmoid of the router logits; the `keep` best of `groups` groups stay eligible; a chosen expert's
+    weight is score * scale."""
+
+    def __init__(self, cap: int, experts: int, top: int, groups: int, keep: int, scale: float, device):
+        self.experts, self.top, self.groups, self.keep, self.scale = experts, top, groups, keep, scale
+        i32 = dict(dtype=torch.int32, device=device)
+        self.topw = torch.zeros(cap * top, dtype=torch.float32, device=device)
+        self.sel = torch.zeros(cap * top, **i32)
+        self.rows = torch.zeros(cap * top, **i32)
+        self.tiles = torch.zeros(self.max_tiles(cap, 16), 4, **i32)
+        self.ntiles = torch.zeros(4, **i32)
+
+    def bm(self, T: int) -> int:
+        """Rows per tile of the expert products at T tokens."""
+        avg = T * self.top / self.experts
+        return 16 if avg <= 12 else (32 if avg <= 24 else (64 if avg <= 96 else 128))
+
+    def max_tiles(self, T: int, bm: Optional[int] = None) -> int:
+        bm = bm or self.bm(T)
+        n = T * self.top
+        return max(1, min(n, self.experts + n // bm))
+
+    def expect_tiles(self, T: int, bm: int) -> int:
+        n = T * self.top
+        return max(1, min(n, self.experts), n // bm)
+
+    def run(self, z: torch.Tensor, T: int, st: int):
+        _check(lib().nls_moe_plan(z.data_ptr(), z.stride(0), T, self.experts, self.top, self.groups, self.keep,
+                                  self.scale, self.topw.data_ptr(), self.sel.data_ptr(), self.bm(T),
+                                  self.rows.data_ptr(), self.tiles.data_ptr(), self.ntiles.data_ptr(),
+                                  self.max_tiles(T), st), "nls_moe_plan")
+
+
+# ---------------------------------------------------------------------------
+# Row kernels
+# ---------------------------------------------------------------------------
+
+def embed(ids, table: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor], T: int, st: int, prev=None):
+    nx, up = prev if prev is not None else (None, None)
+    _check(lib().nls_stack_embed(ids.data_ptr(), _p(nx), _p(up), table.data_ptr(), table.shape[0], table.shape[1],
+                                 x.data_ptr(), _p(xb), x.stride(0), T, st), "nls_stack_embed")
+
+
+def norm_add(y: torch.Tensor, w: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor], T: int, eps: float, st: int,
+             plan: Optional[MoePlan] = None, shared_row0: int = -1, out_norm: Optional[torch.Tensor] = None,
+             out: Optional[torch.Tensor] = None):
+    """x[:T] += LayerNorm(y) * w (xb: its bf16 rounding). With `plan`, y holds the routed experts' rows (token-major) and
+    from row `shared_row0` on the shared expert's, combined first. out = LayerNorm(x) * out_norm (the model's last norm)."""
+    _check(lib().nls_norm_add(y.data_ptr(), y.stride(0), _p(plan.topw) if plan else None, plan.top if plan else 0,
+                              shared_row0, w.data_ptr(), x.data_ptr(), _p(xb), x.stride(0), _p(out_norm), _p(out),
+                              out.stride(0) if out is not None else 0, w.numel(), T, eps,
+                              int(out is not None and out.dtype == torch.float32), st), "nls_norm_add")
+
+
+def layer_norm(x: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor, out: torch.Tensor, n: int, eps: float,
+               st: int):
+    _check(lib().nls_layer_norm(x.data_ptr(), x.stride(0), _p(rows), w.data_ptr(), out.data_ptr(), out.stride(0),
+                                w.numel(), n, eps, int(out.dtype == torch.float32), st), "nls_layer_norm")
+
+
+def argmax(logits: torch.Tensor, n: int, out: torch.Tensor, st: int):
+    _check(lib().nls_stack_argmax(logits.data_ptr(), logits.stride(0), logits.shape[1], out.data_ptr(), n, st),
+           "nls_stack_argmax")
+
+
+def latent_rows(dq, wq, cq, dkv, wc, R: int, Rp: int, rot: int, cs, pos, slot, cache, T: int, eps: float, st: int):
+    """cq = RMSNorm(dq) * wq; with `dkv`: the tokens' cache rows [RMSNorm(dkv[:R]) * wc | rotated dkv[R:]]."""
+    _check(lib().nls_latent_rows(dq.data_ptr(), dq.stride(0), wq.numel(), wq.data_ptr(), cq.data_ptr(), cq.stride(0),
+                                 _p(dkv), dkv.stride(0) if dkv is not None else 0, R, Rp, rot, _p(wc), cs.data_ptr(),
+                                 pos.data_ptr(), slot.data_ptr(), _p(cache), cache.stride(0) if cache is not None else 0,
+                                 T, eps, int(cq.dtype == torch.float32), st), "nls_latent_rows")
+
+
+LATENT_TILES = (1, 2, 3, 4, 6, 8, 12, 16)     # padded latent widths / 64 the attention kernels are built for
+
+
+def latent_pad(R: int) -> int:
+    for n in LATENT_TILES:
+        if R <= 64 * n:
+            return 64 * n
+    raise ValueError(f"latent width {R} > {64 * LATENT_TILES[-1]}")
+
+
+def rot_pad(rot: int) -> int:
+    if rot > 128:
+        raise ValueError(f"rotated width {rot} > 128")
+    return 64 if rot <= 64 else 128
+
+
+def latent_attention(q, cache, out, part, block_tables, block_size: int, tok_seq, ctx_len, T: int, H: int, ns: int,
+                     Rp: int, rp: int, scale: float, st: int):
+    po, pm = part if part is not None else (None, None)
+    if ns > 1 and (po.numel() < T * H * ns * Rp or pm.numel() < T * H * ns * 2):
+        raise ValueError("latent_attention: split workspace too small")
+    _check(lib().nls_latent_attn(q.data_ptr(), cache.data_ptr(), out.data_ptr(), _p(po), _p(pm), block_tables.data_ptr(),
+                                 block_tables.stride(0), block_size, tok_seq.data_ptr(), ctx_len.data_ptr(), T, H, ns,
+                                 Rp, rp, scale, int(q.dtype == torch.float32), st), "nls_latent_attn")
+
+
+def shift_mix(x, mu, prev, out: torch.Tensor, runs, tok_seq, T: int, st: int):
+    """out [mixes, rows, ld]: x + (previous token's x - x) * mu[s]; `prev` [slots, D] precedes each run's first row."""
+    _check(lib().nls_shift_mix(x.data_ptr(), x.stride(0), mu.data_ptr(), prev.data_ptr(), prev.stride(0), out.data_ptr(),
+                               out.stride(1), out.stride(0), runs.data_ptr(), tok_seq.data_ptr(), mu.shape[1], T,
+                               int(out.dtype == torch.float32), st), "nls_shift_mix")
+
+
+def wkv_scan(r, k, v, w, u, o, state, x, prev, runs, nruns: int, H: int, D: int, st: int):
+    """The recurrence over each run's tokens; state [slots, H * D * D] and prev [slots, width] are carried on."""
+    _check(lib().nls_wkv_scan(r.data_ptr(), k.data_ptr(), v.data_ptr(), r.stride(0), w.data_ptr(), w.stride(0),
+                              u.data_ptr(), o.data_ptr(), o.stride(0), state.data_ptr(), state.stride(0), x.data_ptr(),
+                              x.stride(0), prev.data_ptr(), prev.stride(0), prev.shape[1], runs.data_ptr(), nruns, H, D,
+                              int(r.dtype == torch.float32), st), "nls_wkv_scan")
+
+
+def wkv_out(o, norm, gate, out, H: int, D: int, T: int, eps: float, st: int):
+    _check(lib().nls_wkv_out(o.data_ptr(), o.stride(0), norm.data_ptr(), gate.data_ptr(), gate.stride(0), out.data_ptr(),
+                             out.stride(0), H, D, T, eps, int(out.dtype == torch.float32), st), "nls_wkv_out")
