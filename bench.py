@@ -69,6 +69,9 @@ def parse(argv=None):
     ap.add_argument("--tp-leg-concurrency", type=int, default=64)
     ap.add_argument("--tp-leg-timeout", type=float, default=480.0,
                     help="seconds before the TP leg is abandoned (bounds what it adds to an N-GPU run)")
+    ap.add_argument("--stack", default=None, choices=("prefill", "decode", "all"),
+                    help="instead of the headline workload: the config-driven stack design (Sekolorn) at sizes of real "
+                         "layers beside a Mixtral-shaped model of the GGUF families at equal size (bench_stack.py)")
     ap.add_argument("--step-breakdown", action="store_true",
                     help="report host time vs time blocked on the previous step's tokens (diagnostic)")
     a = ap.parse_args(argv)

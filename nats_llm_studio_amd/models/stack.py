@@ -19,7 +19,7 @@ from typing import Dict, List, Optional
 import torch
 
 from ..ops import stack as K
-from ..ops import rope_table
+from ..ops import prefill_blocks, rope_table
 from ..safetensors_io import SafetensorsReader
 from .llama import ShardSpec
 from .stack_config import StackConfig
@@ -357,6 +357,12 @@ class StackModel:
                 b.launches[i, "mlp"] = mlp.bind(b)
         b.launches["head"] = K.LinLaunch([K.Seg(self.head, b.hn, b.logits)])
         return b
+
+    def attention_blocks(self, b: StackBuffers, T: int) -> dict:
+        """The forward arguments that describe a row batch's attention blocks, from its staged metadata (the engine builds
+        them on the host: ops.prefill_blocks)."""
+        qb = prefill_blocks(b.tok_seq[:T].cpu().numpy(), b.pos[:T].cpu().numpy(), T)
+        return dict(qblocks=torch.from_numpy(qb).to(self.device), nqb=len(qb))
 
     # ---- forward
     @torch.no_grad()

@@ -11,6 +11,11 @@ from dataclasses import dataclass, field
 from typing import List, Optional
 
 
+def default_ctx() -> int:
+    """Context length of a stack model: the designs set no limit, the position and block tables are sized by this one."""
+    return int(os.environ.get("NLS_STACK_CTX", "32768"))
+
+
 @dataclass(frozen=True)
 class Design:
     """What every model of a design has in common."""
@@ -75,7 +80,7 @@ class StackConfig:
     vocab: int
     eps: float
     layers: List[LayerConfig] = field(default_factory=list)
-    ctx: int = 32768                   # the design itself has no limit; sizes the position tables and block tables
+    ctx: int = 32768
 
     @property
     def n_layer(self) -> int:
@@ -113,7 +118,7 @@ class StackConfig:
 
         norm = cfg.get("norm") or {}
         out = cls(arch=arch, design=design, d_model=size(cfg, "width", "embed", 1), vocab=size(cfg, "vocab", "embed"),
-                  eps=float(norm["eps"]), ctx=int(os.environ.get("NLS_STACK_CTX", "32768")))
+                  eps=float(norm["eps"]), ctx=default_ctx())
         for i, L in enumerate(cfg["layers"]):
             t, m, p = L["type"], L["mixer"], f"l{i}."
             if t not in design.mixers:

@@ -44,8 +44,9 @@ def chat_response(model_id: str, entry: Optional[ModelEntry], text: str, prompt_
                   "generation_time": round(gen_time, 6), "stop_reason": stop_reason},
         "model_info": {"arch": arch or (entry.arch if entry else ""),
                        "quant": quant or (entry.quantization if entry else ""),
-                       "format": "gguf", "context_length": ctx},
-        "runtime": {"name": "nats-llm-studio-amd", "version": __version__, "supported_formats": ["gguf"]},
+                       "format": entry.format if entry else "gguf", "context_length": ctx},
+        "runtime": {"name": "nats-llm-studio-amd", "version": __version__,
+                    "supported_formats": ["gguf", "safetensors"]},
     }
 
 
@@ -107,7 +108,7 @@ class StubBackend:
 
 
 class EngineBackend:
-    """GGUF models served by the HIP engine; JIT-loaded, LRU-evicted.
+    """GGUF and stack (config.json + safetensors) models served by the HIP engine; JIT-loaded, LRU-evicted.
 
     Loading never holds the registry lock: a model is built outside it (concurrent chats for the
     same model wait on one per-model future), so `list_models` / `health` / chats of loaded models
@@ -145,19 +146,23 @@ class EngineBackend:
         self._ids = tuple(self._loaded)
 
     def build_state(self, entry: ModelEntry, shard=None, comm=None, start: bool = True) -> dict:
-        """GGUF -> device model + tokenizer + chat template + engine (one TP shard if `shard`)."""
+        """Checkpoint -> device model + tokenizer + chat template + engine (one TP shard if `shard`)."""
         from ..engine.engine import Engine
-        from ..gguf.reader import GGUFReader
-        from ..models.llama import LlamaModel, ShardSpec
+        from ..models.registry import load_model
         from ..tokenizer.bpe import tokenizer_from_metadata
         from ..tokenizer.chat_template import ChatTemplate, default_template
         t0 = time.time()
-        reader = GGUFReader(entry.path)
-        md = reader.metadata
-        model = LlamaModel(reader, self.device(), shard or ShardSpec(), comm)
-        tok = tokenizer_from_metadata(md)
-        tmpl = md.get("tokenizer.chat_template") or default_template(model.cfg.arch,
-                                                                     md.get("tokenizer.ggml.model", "gpt2"))
+        import torch
+        model = load_model(entry.path, self.device(), shard, comm, dtype=getattr(torch, self.cfg.dtype),
+                           ctx=self.cfg.max_ctx or None)
+        if model.format == "gguf":
+            md = model.reader.metadata
+            tok = tokenizer_from_metadata(md)
+            tmpl = md.get("tokenizer.chat_template") or default_template(model.cfg.arch,
+                                                                         md.get("tokenizer.ggml.model", "gpt2"))
+        else:
+            from ..tokenizer import ids
+            tok, tmpl = ids.IdTokenizer(model.cfg.vocab), ids.TEMPLATE
         bos = tok.tokens[tok.bos_id] if tok.bos_id is not None else ""
         eos = tok.tokens[tok.eos_id] if tok.eos_id is not None else ""
         # EP: prefill chunks stay within the IPC row exchange's token budget (larger ones take the all-to-all)

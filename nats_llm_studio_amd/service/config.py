@@ -44,7 +44,8 @@ class WorkerConfig:
     device: str = "auto"               # auto | cuda:N | cpu
     tp: int = 1                        # tensor-parallel ranks (launch with torchrun, one process per GPU)
     ep: bool = False                   # MoE: expert-parallel instead of TP-sharded experts
-    model: str = ""                    # model to preload (registry id or .gguf path; required when tp > 1)
+    model: str = ""                    # model to preload (registry id, .gguf path or model folder; required when tp > 1)
+    dtype: str = "bfloat16"            # config.json models: bfloat16, or float32 throughout
     max_batch: int = 64
     max_ctx: int = 0                   # 0 = model context length
     kv_mem_fraction: float = 0.5
@@ -122,6 +123,7 @@ class WorkerConfig:
         if seed_file and not c.nats_nkey_seed:
             with open(os.path.expanduser(seed_file)) as f:
                 c.nats_nkey_seed = f.read().strip()
+        c.dtype = e.get("STACK_DTYPE", c.dtype)
         c.nats_creds = e.get("NATS_CREDS", c.nats_creds)
         yes = ("1", "true", "yes")
         c.nats_tls = e.get("NATS_TLS", "0").lower() in yes
@@ -144,6 +146,8 @@ class WorkerConfig:
         ap.add_argument("--backend", default=c.backend, choices=["engine", "stub", "http"])
         ap.add_argument("--lmstudio-base-url", default=c.lmstudio_base_url)
         ap.add_argument("--model", default=c.model)
+        ap.add_argument("--dtype", default=c.dtype, choices=["bfloat16", "float32"],
+                        help="number format of config.json (safetensors) models")
         ap.add_argument("--ep", action="store_true", default=c.ep)
         ap.add_argument("--device", default=c.device)
         ap.add_argument("--tp", type=int, default=c.tp)

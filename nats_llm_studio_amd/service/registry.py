@@ -1,4 +1,5 @@
-"""Local model registry over the LM Studio on-disk tree `<MODELS_DIR>/<publisher>/<model>/*.gguf`.
+"""Local model registry over the LM Studio on-disk tree `<MODELS_DIR>/<publisher>/<model>/*.gguf`, and, beside them,
+model folders with config.json + model.safetensors of a design in models/stack_config.py.
 
 Replaces LM Studio's `GET /api/v0/models` and `GET /api/v0/models/{id}` that the reference
 calls (`/root/reference/nats_llm_studio.go:61-85`, `:136-156`). Entries are read from the
@@ -19,6 +20,8 @@ from dataclasses import dataclass, field
 from typing import Dict, List, Optional
 
 from ..gguf.reader import read_metadata
+from ..models.registry import stack_arch
+from ..models.stack_config import default_ctx, is_stack_dir
 
 
 @dataclass
@@ -26,12 +29,13 @@ class ModelEntry:
     id: str
     publisher: str
     model_dir: str            # directory name under the publisher
-    path: str                 # .gguf file
+    path: str                 # .gguf file (format "safetensors": the model folder)
     dir: str                  # absolute model directory
     arch: str = "unknown"
     quantization: str = "unknown"
     max_context_length: int = 0
     size_bytes: int = 0
+    format: str = "gguf"
     aliases: List[str] = field(default_factory=list)
 
     def to_api(self, loaded: bool) -> dict:
@@ -41,7 +45,7 @@ class ModelEntry:
             "type": "llm",
             "publisher": self.publisher,
             "arch": self.arch,
-            "compatibility_type": "gguf",
+            "compatibility_type": self.format,
             "quantization": self.quantization,
             "state": "loaded" if loaded else "not-loaded",
             "max_context_length": self.max_context_length,
@@ -90,6 +94,12 @@ class Registry:
                         entries[e.id] = e
                         for a in e.aliases:
                             alias.setdefault(a.lower(), e.id)
+                    if not ggufs:
+                        e = self._stack_entry(pub, mdir, d)
+                        if e is not None:
+                            entries[e.id] = e
+                            for a in e.aliases:
+                                alias.setdefault(a.lower(), e.id)
         for e in getattr(self, "_extra", {}).values():       # added entries survive re-scans
             entries.setdefault(e.id, e)
             for a in [e.id] + list(e.aliases):
@@ -130,6 +140,23 @@ class Registry:
             aliases=[mid, f"{pub}/{mdir}", f"{pub}/{mid}", mdir, stem, f"{pub}/{mdir}/{fname}", f"{pub}/{stem}"],
         )
         return e
+
+    @staticmethod
+    def _stack_entry(pub, mdir, d) -> Optional[ModelEntry]:
+        """A model folder (config.json + model.safetensors) of a supported design."""
+        if not is_stack_dir(d):
+            return None
+        arch = stack_arch(d)
+        if arch is None:
+            return None
+        try:
+            size = sum(os.path.getsize(os.path.join(d, f)) for f in ("config.json", "model.safetensors"))
+        except OSError:
+            return None
+        mid = model_id_for(mdir)
+        return ModelEntry(id=mid, publisher=pub, model_dir=mdir, path=d, dir=d, arch=arch, quantization="BF16",
+                          max_context_length=default_ctx(), size_bytes=size, format="safetensors",
+                          aliases=[mid, f"{pub}/{mdir}", f"{pub}/{mid}", mdir])
 
     def add(self, e: ModelEntry):
         """Register an entry that does not live under models_dir (e.g. a preloaded model)."""

@@ -25,6 +25,10 @@ class PullError(Exception):
         self.output = output
 
 
+# objects that make up a model: a GGUF file, or a folder of config.json + model.safetensors
+MODEL_FILES = (".gguf", "/model.safetensors", "/config.json")
+
+
 def _match(identifier: str, name: str) -> bool:
     ident = identifier.strip("/").lower()
     n = name.lower()
@@ -84,7 +88,7 @@ class ModelStore:
         except Exception as e:
             left(0.25)
             raise PullError(f"failed to list bucket '{self.bucket}': {e}", "")
-        matches = [o for o in objs if _match(identifier, o["name"]) and o["name"].lower().endswith(".gguf")]
+        matches = [o for o in objs if _match(identifier, o["name"]) and o["name"].lower().endswith(MODEL_FILES)]
         if not matches:
             raise PullError(f"model '{identifier}' not found in bucket '{self.bucket}'",
                             f"no objects matching {identifier!r} in bucket {self.bucket!r}")

@@ -31,6 +31,9 @@ def _resolve_model(cfg):
     reg = Registry(cfg.models_dir)
     reg.scan()
     ent = reg.resolve(cfg.model) if cfg.model else None
+    if ent is None and cfg.model and os.path.isdir(cfg.model):
+        d = os.path.abspath(cfg.model)
+        ent = Registry._stack_entry("local", os.path.basename(d), d)
     if ent is None and cfg.model and os.path.isfile(cfg.model):
         d = os.path.dirname(os.path.abspath(cfg.model))
         ent = ModelEntry(id=os.path.splitext(os.path.basename(cfg.model))[0].lower(), publisher="local",

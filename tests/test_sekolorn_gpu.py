@@ -1,0 +1,588 @@
+"""Sekolorn on the GPU kernels against the plain implementation (sekolorn_oracle): each mechanism alone, then whole models
+through the engine's feeds, scheduler and graphs."""
+import math
+
+import pytest
+import torch
+
+import sekolorn_models as S
+import sekolorn_oracle as O
+
+pytestmark = pytest.mark.gpu
+# Whole models: largest row error (sekolorn_models.error) in f32. In bf16 an expert choice can still be a close call, and a
+# squared relu whose units are all nearly off leaves the norm after it mostly rounding, so there the bound holds for nine
+# rows of ten; f32 runs the same kernels' f32 forms and holds for all.
+F32, BF16 = 2e-4, 0.06
+DT = {"f32": torch.float32, "bf16": torch.bfloat16}
+TOL = {"f32": 3e-5, "bf16": 1.5e-2}
+
+
+@pytest.fixture(scope="module")
+def K(gpu):
+    from nats_llm_studio_amd.ops import stack
+    stack.lib()
+    return stack
+
+
+def rnd(*shape, seed=0, scale=1.0):
+    return torch.randn(*shape, generator=torch.Generator().manual_seed(seed), dtype=torch.float64) * scale
+
+
+def relerr(got, want):
+    return float((got.double().cpu() - want).abs().max() / (want.abs().max() + 1e-30))
+
+
+def act(t, ld, dt, rows=None):
+    """t [n, k] as an activation buffer of `ld` columns, padding zero."""
+    b = torch.zeros(rows or t.shape[0], ld, dtype=dt, device="cuda")
+    b[:t.shape[0], :t.shape[1]] = t.to(dt)
+    return b
+
+
+def st():
+    return torch.cuda.current_stream().cuda_stream
+
+
+# ---------------------------------------------------------------- linear layers
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("M", [1, 2, 17, 33, 64, 65, 200, 700])
+@pytest.mark.parametrize("N,Kd", [(5, 16), (96, 70), (200, 256), (520, 130)])
+def test_linear(K, dt, M, N, Kd):
+    d = DT[dt]
+    w, x = rnd(N, Kd, seed=1).to(d), rnd(M, Kd, seed=2).to(d)
+    ref = x.double() @ w.double().T / math.sqrt(Kd)
+    w = (w / math.sqrt(Kd)).to(d)
+    ref = x.double() @ w.double().T
+    p = K.PackedLinear(w, dt == "f32", "cuda")
+    y = torch.full((M, N + 3), 7.0, device="cuda")
+    xa = act(x, K.act_ld(Kd), d)
+    K.LinLaunch([K.Seg(p, xa, y, ycol=2)]).run(M, st())
+    assert relerr(y[:, 2:2 + N], ref) < 2e-6 * math.sqrt(Kd)
+    assert (y[:, :2] == 7).all() and (y[:, 2 + N:] == 7).all()
+
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("cfg", [(True, c, 0) for c in range(5)] + [(False, 1, 4), (False, 1, 8), (False, 1, 16), (False, 2, 4),
+                                                                   (False, 2, 8), (False, 4, 4), (False, 4, 8)])
+def test_linear_every_tile(K, dt, cfg):
+    """Every launch shape gives the same product, also where tiles end past the matrix and K has one step."""
+    d = DT[dt]
+    for M, N, Kd in ((70, 330, 200), (1, 16, 64), (300, 40, 1000)):
+        w, x = (rnd(N, Kd, seed=3) / math.sqrt(Kd)).to(d), rnd(M, Kd, seed=4).to(d)
+        y = torch.zeros(M, N, device="cuda")
+        L = K.LinLaunch([K.Seg(K.PackedLinear(w, dt == "f32", "cuda"), act(x, K.act_ld(Kd), d), y)])
+        L.config = lambda M, c=cfg: c
+        L.run(M, st())
+        assert relerr(y, x.double() @ w.double().T) < 2e-6 * math.sqrt(Kd)
+
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("M", [3, 150])
+def test_linear_epilogues_in_one_launch(K, dt, M):
+    d = DT[dt]
+    Kd, N = 72, 50
+    x = rnd(M, Kd, seed=5).to(d)
+    ws = [(rnd(N, Kd, seed=10 + i) / math.sqrt(Kd) * 2).to(d) for i in range(6)]
+    z = [x.double() @ w.double().T for w in ws]
+    bias = rnd(N, seed=6).float()
+    pos = torch.randint(0, 40, (M,), dtype=torch.int32)
+    from nats_llm_studio_amd.ops import rope_table
+    cs = rope_table(64, 20, 50.0, "cuda")
+    # rope: 2 blocks of 24 columns, 20 of them rotated, written 32 apart
+    want_r = z[5][:, :48].reshape(M, 2, 24)
+    want_r = torch.cat([O.rotate(want_r[..., :20], pos.long(), 50.0, 20), want_r[..., 20:]], -1)
+    ys = [torch.zeros(M, N, dtype=d if i < 4 else torch.float32, device="cuda") for i in range(5)]
+    yr = torch.zeros(M, 64, device="cuda")
+    xa = act(x, K.act_ld(Kd), d)
+    P = lambda w: K.PackedLinear(w, dt == "f32", "cuda")      # noqa: E731
+    names = ("silu", "tanh", "sigmoid", "relu2", "decay")
+    segs = [K.Seg(P(ws[i]), xa, ys[i], n, bias=bias.cuda() if n == "decay" else None) for i, n in enumerate(names)]
+    segs.append(K.Seg(P(ws[5][:48]), xa, yr, "rope", block=(24, 32), rope=(cs, pos.cuda(), 10)))
+    K.LinLaunch(segs).run(M, st())
+    want = [z[0] * torch.sigmoid(z[0]), torch.tanh(z[1]), torch.sigmoid(z[2]), torch.relu(z[3]) ** 2,
+            torch.exp(-torch.exp(z[4] + bias.double()))]
+    for n, y, w in zip(names, ys, want):
+        assert relerr(y, w) < (5e-3 if y.dtype == torch.bfloat16 else 2e-5), n
+    assert relerr(yr.view(M, 2, 32)[..., :24], want_r) < 2e-5 and (yr.view(M, 2, 32)[..., 24:] == 0).all()
+
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("M", [2, 90])
+def test_linear_groups_and_gate(K, dt, M):
+    """Per-head products: groups step through the input and output columns; the gate is per row and head."""
+    d, G, N, Kd = DT[dt], 5, 20, 40
+    w, x, gate = (rnd(G, N, Kd, seed=7) / math.sqrt(Kd)).to(d), rnd(M, G, Kd, seed=8).to(d), rnd(M, G, seed=9).float()
+    xb = torch.zeros(M, G, 64, dtype=d, device="cuda")
+    xb[..., :Kd] = x
+    xb[..., Kd:] = 3.0                                     # what the zero-padded weights must hide
+    y = torch.zeros(M, G * N, device="cuda")
+    K.LinLaunch([K.Seg(K.PackedLinear(w, dt == "f32", "cuda"), xb.view(M, -1), y, "gate", xgs=64, ygs=N,
+                       gate=gate.cuda())]).run(M, st())
+    want = torch.einsum("mgk,gnk->mgn", x.double(), w.double()) * gate.double()[:, :, None]
+    assert relerr(y.view(M, G, N), want) < 1e-5
+
+
+# ---------------------------------------------------------------- norms, routing, experts
+
+@pytest.mark.parametrize("D", [37, 256, 1030, 4100])
+def test_norm_add(K, D):
+    T, eps = 5, 1e-2
+    y, x, w, ow = rnd(T, D, seed=1), rnd(T, D, seed=2, scale=3), rnd(D, seed=3), rnd(D, seed=4)
+    ld = K.act_ld(D)
+    xd = act(x, ld, torch.float32)
+    xb = torch.zeros(T, ld, dtype=torch.bfloat16, device="cuda")
+    on = torch.zeros(T, ld, dtype=torch.bfloat16, device="cuda")
+    K.norm_add(y.float().cuda(), w.float().cuda(), xd, xb, T, eps, st(), out_norm=ow.float().cuda(), out=on)
+    want = x + O.layer_norm(y, w, eps)
+    assert relerr(xd[:, :D], want) < 1e-5 and relerr(xb[:, :D], want) < 5e-3
+    assert relerr(on[:, :D], O.layer_norm(want, ow, eps)) < 5e-3
+    assert (xd[:, D:] == 0).all() and (xb[:, D:] == 0).all() and (on[:, D:] == 0).all()
+    rows = torch.tensor([3, 0], dtype=torch.int32, device="cuda")
+    K.layer_norm(xd, rows, ow.float().cuda(), on, 2, eps, st())
+    assert relerr(on[:2, :D], O.layer_norm(want[[3, 0]], ow, eps)) < 5e-3
+
+
+@pytest.mark.parametrize("E,top,groups,keep", [(12, 3, 3, 2), (16, 2, 4, 1), (5, 2, 1, 1), (1, 1, 1, 1), (6, 3, 6, 4),
+                                               (64, 6, 8, 3), (200, 8, 4, 2), (512, 10, 16, 5)])
+@pytest.mark.parametrize("T", [1, 3, 32, 33, 150])
+def test_expert_choice_and_lists(K, E, top, groups, keep, T):
+    z = rnd(T, E, seed=E + T, scale=2.0)
+    if groups > 1:
+        z[0, 0] = 9.0                 # the best expert alone in a weak group: the group may lose
+        z[0, 1:E // groups] = -9.0
+    p = K.MoePlan(T + 9, E, top, groups, keep, 1.7, "cuda")
+    p.run(z.float().cuda(), T, st())
+    sel, tw = p.sel[:T * top].view(T, top).cpu(), p.topw[:T * top].view(T, top).cpu()
+    for t in range(T):
+        want = O.route(z[t].float().double(), top, 1.7, groups, keep)
+        assert sel[t].tolist() == [e for e, _ in want], t
+        assert torch.allclose(tw[t].double(), torch.stack([w for _, w in want]), atol=1e-6)
+    n, tiles, rows = int(p.ntiles[0]), p.tiles.cpu(), p.rows.cpu()
+    assert n <= p.max_tiles(T)
+    seen = []
+    for e, o, c, _ in tiles[:n].tolist():
+        assert 1 <= c <= p.bm(T)
+        ent = rows[o:o + c].tolist()
+        assert all(int(sel.view(-1)[i]) == e for i in ent)
+        seen += ent
+    assert sorted(seen) == list(range(T * top))
+
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("name,i", [("uneven", 0), ("uneven", 1), ("uneven", 3), ("ones", 0), ("ones", 1), ("wide", 0), ("wide", 1)])
+@pytest.mark.parametrize("T", [1, 7, 40, 230])
+def test_moe_layer(K, tmp_path, dt, name, i, T):
+    cfg = S.CONFIGS[name]
+    W = S.make_weights(cfg)
+    m = load(tmp_path, cfg, W, dt)
+    b = m.step_buffers(T, 1, 16)
+    x = rnd(T, cfg["width"], seed=T).to(torch.bfloat16)
+    b.act[:T, :cfg["width"]] = x.to(b.act.dtype)
+    mlp, e = m.layers[i][2], b.launches[i, "mlp"]
+    from nats_llm_studio_amd.models.stack import _Step
+    mlp.run(b, e, _Step(T, 1, 16, st()))
+    one = torch.ones(cfg["width"], device="cuda")
+    b.x.zero_()
+    K.norm_add(e["ye"], one, b.x, None, T, 1e-6, st(), plan=e["plan"], shared_row0=e["shared_row0"])
+    want = O.moe(x.double(), {k: v.double() for k, v in W.items()}, f"l{i}.mlp.", cfg["layers"][i]["mlp"])
+    assert relerr(b.x[:T, :cfg["width"]], O.layer_norm(want, 1.0, 1e-6)) < TOL[dt] * 2
+
+
+# ---------------------------------------------------------------- the recurrence
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("H,D", [(1, 16), (3, 20), (2, 64), (2, 33), (1, 128), (1, 200)])
+def test_wkv_scan(K, dt, H, D):
+    """Runs of two sequences in one launch, cut at 2, 3 and 16 tokens, slots given out of order: the plain recurrence, and
+    bit for bit the same as one whole run."""
+    d, n, HD = DT[dt], 70, H * D
+    ld = K.act_ld(HD)
+    r, k, v = (rnd(2, n, HD, seed=s).to(d) for s in (1, 2, 3))
+    w, u = torch.sigmoid(rnd(2, n, HD, seed=4, scale=3)).float(), rnd(HD, seed=5).float()
+    w[0, 20:40, :HD // 2] = 0.0                             # a state that is wiped out
+    w[1, :, 0] = 1.0                                        # one that never decays
+    x = rnd(2, n, 8, seed=6).float()
+
+    def run(cuts):
+        S0 = torch.full((4, HD * D), 9.0, device="cuda")    # slots start dirty
+        prev = torch.zeros(4, 8, device="cuda")
+        out = torch.zeros(2, n, HD)
+        for a, b in zip((0,) + cuts, cuts + (n,)):
+            m = b - a
+            buf = lambda t, dd: act(torch.cat([t[0, a:b], t[1, a:b]]).double(), ld, dd)     # noqa: E731
+            runs = torch.tensor([[0, m, 3, a], [m, m, 1, a], [0, 0, -1, 0]], dtype=torch.int32, device="cuda")
+            o = torch.zeros(2 * m, ld, device="cuda")
+            K.wkv_scan(buf(r, d), buf(k, d), buf(v, d), buf(w, torch.float32), u.cuda(), o, S0,
+                       torch.cat([x[0, a:b], x[1, a:b]]).cuda(), prev, runs, 3, H, D, st())
+            out[0, a:b], out[1, a:b] = o[:m, :HD].cpu(), o[m:, :HD].cpu()
+        assert torch.equal(prev[3].cpu(), x[0, -1]) and torch.equal(prev[1].cpu(), x[1, -1]) and (S0[0] == 9).all()
+        return out, S0
+    whole, Sw = run(())
+    for q, slot in ((0, 3), (1, 1)):
+        o, Sx = O.wkv_scan(*(t[q].double().view(n, H, D) for t in (r, k, v, w)), u.double().view(H, D))
+        assert relerr(whole[q].view(n, H, D), o) < 1e-5
+        assert relerr(Sw[slot].view(H, D, D), Sx) < 1e-5
+    for cuts in ((2, 4, 7), (16, 32, 48), (15, 17, 69)):
+        o, Sc = run(cuts)
+        assert torch.equal(o, whole) and torch.equal(Sc, Sw)
+
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("name,i", [("uneven", 1), ("uneven", 3), ("ones", 0), ("wide", 0)])
+def test_wkv_mixer(K, tmp_path, dt, name, i):
+    cfg = S.CONFIGS[name]
+    W, d, n = S.make_weights(cfg), cfg["width"], 41
+    m = load(tmp_path, cfg, W, dt)
+    b = m.step_buffers(64, 2, 16)
+    mix, state = m.layers[i][0], m.state_pool(3)[i]
+    for t in state.values():
+        t.fill_(5.0)
+    x = rnd(n, d, seed=2).to(torch.bfloat16)
+    from nats_llm_studio_amd.models.stack import _Step
+    out = []
+    for a, c in ((0, 2), (2, 20), (20, 21), (21, n)):
+        T = c - a
+        b.x[:T, :d] = x[a:c].float()
+        b.runs[0] = torch.tensor([0, T, 2, a])
+        b.tok_seq.zero_()
+        mix.run(b, b.launches[i, "mix"], None, state, _Step(T, 1, 16, st()))
+        out.append(b.y[:T].cpu())
+    want, _ = O.wkv_mixer(x.double(), {k: v.double() for k, v in W.items()}, f"l{i}.mix.", cfg["layers"][i]["mixer"],
+                          cfg["norm"]["eps"])
+    assert relerr(torch.cat(out), want) < TOL[dt]
+
+
+# ---------------------------------------------------------------- latent attention
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("H,R,rot", [(1, 8, 2), (5, 40, 12), (17, 192, 64), (3, 264, 70), (16, 512, 64), (2, 700, 128)])
+def test_latent_attention(K, dt, H, R, rot):
+    """Contexts around the page and tile edges, with and without splits of the keys; a key whose score stands out sits at a
+    page's or tile's edge, first, or last."""
+    d, bs = DT[dt], 16
+    Rp, rp = K.latent_pad(R), K.rot_pad(rot)
+    Dp = Rp + rp
+    ctxs = [1, 2, 15, 16, 17, 63, 64, 65, 128, 200, 331]
+    nb = 24
+    T = len(ctxs)
+    perm = torch.randperm(T * nb, generator=torch.Generator().manual_seed(5))
+    bt = perm.view(T, nb).int()
+    cache = torch.zeros(T * nb * bs, Dp, dtype=d)
+    q = torch.zeros(T, H, Dp, dtype=d)
+    q[..., :R], q[..., Rp:Rp + rot] = rnd(T, H, R, seed=1).to(d), rnd(T, H, rot, seed=2).to(d)
+    scale = 0.7 / math.sqrt(R + rot)
+    want = torch.zeros(T, H, R, dtype=torch.float64)
+    for t, n in enumerate(ctxs):
+        c = torch.zeros(n, Dp, dtype=d)
+        c[:, :R], c[:, Rp:Rp + rot] = rnd(n, R, seed=10 + t).to(d), rnd(n, rot, seed=40 + t).to(d)
+        spike = [0, n - 1, min(15, n - 1), min(16, n - 1), min(63, n - 1), min(64, n - 1)][t % 6]
+        qs = q[t, t % H].double()
+        c[spike] = (qs * 12.0 / (scale * (qs @ qs))).to(d)
+        for p in range(n):
+            cache[int(bt[t, p // bs]) * bs + p % bs] = c[p]
+        s = q[t].double() @ c.double().T * scale
+        want[t] = torch.softmax(s, -1) @ c[:, :R].double()
+    cache, q, bt = cache.cuda(), q.view(T, -1).cuda(), bt.cuda()
+    rows = torch.arange(T, dtype=torch.int32, device="cuda")
+    ctx = torch.tensor(ctxs, dtype=torch.int32, device="cuda")
+    for ns in (1, 3, 16) if dt == "bf16" else (1,):
+        out = torch.full((T, H * Rp), 7.0, dtype=d, device="cuda")
+        part = (torch.zeros(T * H * ns * Rp, device="cuda"), torch.zeros(T * H * ns * 2, device="cuda"))
+        K.latent_attention(q, cache, out, part, bt, bs, rows, ctx, T, H, ns, Rp, rp, scale, st())
+        out = out.view(T, H, Rp)
+        for t in range(T):
+            assert relerr(out[t, :, :R], want[t]) < TOL[dt], (ns, ctxs[t])
+        assert (out[..., R:] == 0).all()
+    # a padded row (no keys) leaves zeros
+    ctx[3] = 0
+    K.latent_attention(q, cache, out.view(T, -1), part, bt, bs, rows, ctx, T, H, 1, Rp, rp, scale, st())
+    assert (out[3] == 0).all()
+
+
+def run_rows(m, b, kc, state, parts, bs=16):
+    """One forward of [(seq row, slot, blocks, first position, tokens)] with every row's logits; CPU logits per part."""
+    T = 0
+    b.slot.fill_(-1)
+    dev = b.ids.device
+    for r, (slot, blocks, p0, toks) in enumerate(parts):
+        n = len(toks)
+        pos = torch.arange(p0, p0 + n)
+        blk = torch.tensor(blocks)
+        b.ids[T:T + n] = torch.tensor(toks, dtype=torch.int32)
+        b.pos[T:T + n] = pos.int()
+        b.slot[T:T + n] = (blk[pos // bs] * bs + pos % bs).int()
+        b.tok_seq[T:T + n] = r
+        b.ctx_len[T:T + n] = (pos + 1).int()
+        b.block_tables[r, :len(blocks)] = blk.int()
+        b.runs[r] = torch.tensor([T, n, slot, p0])
+        T += n
+    qb = m.attention_blocks(b, T)
+    rows = torch.arange(T, dtype=torch.int32, device=dev)
+    m.forward(b, kc, None, T, bs, logit_rows=rows, n_logits=T, state=state, nruns=len(parts), **qb)
+    lg = b.logits[:T].cpu()
+    out, o = [], 0
+    for _, _, _, toks in parts:
+        out.append(lg[o:o + len(toks)])
+        o += len(toks)
+    return out
+
+
+def load(tmp_path, cfg, W, dt, ctx=1024):
+    from nats_llm_studio_amd.models.registry import load_model
+    return load_model(S.write_model(str(tmp_path / "model"), cfg, W), "cuda:0", dtype=DT[dt], ctx=ctx)
+
+
+def close(got, want, dt):
+    return S.error(got, want) < F32 if dt == "f32" else S.error(got, want, 0.9) < BF16
+
+
+# ---------------------------------------------------------------- whole models
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("name", S.CONFIGS)
+def test_prompt_layers(gpu, tmp_path, dt, name):
+    """The residual after every layer, and the logits, of a prompt."""
+    cfg = S.CONFIGS[name]
+    W, n = S.make_weights(cfg), 75
+    m = load(tmp_path, cfg, W, dt)
+    toks = S.tokens(n, cfg["vocab"])
+    want_l = []
+    want = O.forward(cfg, W, toks, layers=want_l)
+    b = m.step_buffers(128, 2, 16, logit_rows=128)
+    kc, _ = m.kv_cache(12, 16)
+    taps = []
+    orig = m.forward
+    m.forward = lambda *a, **k: orig(*a, taps=taps, **k)
+    (got,) = run_rows(m, b, kc, m.state_pool(2), [(1, [7, 2, 9, 4, 0], 0, toks)])
+    for t, w in zip(taps, want_l):
+        assert close(t.cpu(), w, dt)
+    assert close(got, want, dt)
+
+
+def engine(m, dt, **kw):
+    from nats_llm_studio_amd.engine.engine import Engine
+    kw = dict(dict(max_batch=4, num_blocks=64, max_prefill_tokens=512, max_logit_rows=512, ctx=512), **kw)
+    return Engine(m, None, **kw)
+
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("name", ["uneven", "wide", "ones"])
+def test_feed_schedules(gpu, tmp_path, dt, name):
+    """One sequence whole, token by token, and in portions of several sizes; three unequal ones mixed, in reused pages and
+    slots: always the plain implementation's logits."""
+    cfg = S.CONFIGS[name]
+    W = S.make_weights(cfg)
+    m = load(tmp_path, cfg, W, dt)
+    eng = engine(m, dt)
+    toks = S.tokens(150, cfg["vocab"])
+    want = O.forward(cfg, W, toks)
+    (got,) = eng.feed([("w", toks, list(range(150)))])
+    assert close(got, want, dt)
+    eng.feed_end("w")
+    whole = got
+    for name_, cuts in (("pairs", [2] * 20 + [1] * 10 + [100]), ("decode", [60] + [1] * 90), ("odd", [1, 2, 13, 16, 17, 31, 33, 37]),
+                        ("edges", [15, 1, 1, 47, 1, 63, 22])):
+        assert sum(cuts) == 150
+        o, rows = 0, []
+        for c in cuts:
+            (r,) = eng.feed([(name_, toks[o:o + c], list(range(c)))])
+            rows.append(r)
+            o += c
+        eng.feed_end(name_)
+        assert close(torch.cat(rows), want, dt), name_
+        assert close(torch.cat(rows), whole.double(), dt), name_
+    # mixed batches: (id, tokens) per step; "b" rests, "c" comes when "a" is gone
+    seqs = {k: S.tokens(n, cfg["vocab"], 7 + i) for i, (k, n) in enumerate((("a", 90), ("b", 70), ("c", 120), ("d", 9)))}
+    plan = [{"a": 64, "b": 1}, {"a": 2, "b": 40}, {"a": 1, "d": 5}, {"a": 1, "b": 1, "d": 1}, {"a": 1, "b": 1, "d": 1},
+            {"a": 21, "b": 2, "d": 2}, {"b": 1, "c": 33}, {"b": 24, "c": 2}, {"c": 1}, {"c": 84}]
+    at = {k: 0 for k in seqs}
+    got = {k: [] for k in seqs}
+    for stp in plan:
+        ent = []
+        for k, n in stp.items():
+            ent.append((k, seqs[k][at[k]:at[k] + n], list(range(n))))
+            at[k] += n
+        for (k, _, _), r in zip(ent, eng.feed(ent)):
+            got[k].append(r)
+        for k in stp:
+            if at[k] == len(seqs[k]):
+                eng.feed_end(k)
+    for k, t in seqs.items():
+        assert at[k] == len(t)
+        assert close(torch.cat(got[k]), O.forward(cfg, W, t), dt), k
+    assert eng.alloc.n_free == eng.num_blocks and len(eng.slots.free) == 4
+    assert eng.counters["graph_replays"] > 20
+
+
+@pytest.mark.parametrize("dt", DT)
+def test_batch_independence(gpu, tmp_path, dt):
+    """A prompt's logits next to others, and in other pages and slots, are those it has alone, beyond rounding."""
+    cfg = S.CONFIGS["uneven"]
+    m = load(tmp_path, cfg, S.make_weights(cfg), dt)
+    b = m.step_buffers(512, 4, 16, logit_rows=512)
+    kc, _ = m.kv_cache(40, 16)
+    state = m.state_pool(4)
+    ps = [S.tokens(n, cfg["vocab"], n) for n in (3, 81, 130, 2)]
+    blk = [[0], [3, 1, 9, 30, 31, 5], list(range(10, 19)), [39]]
+    alone = [run_rows(m, b, kc, state, [(0, list(range(20, 30)), 0, p)])[0] for p in ps]
+    for order in ((0, 1, 2, 3), (2, 3, 1, 0)):
+        got = run_rows(m, b, kc, state, [(3 - i, blk[i], 0, ps[i]) for i in order])
+        for i, g in zip(order, got):
+            assert close(g, alone[i].double(), dt)
+
+
+@pytest.mark.parametrize("dt", DT)
+def test_far_key(gpu, tmp_path, dt):
+    """Attention finds one early key among hundreds: its removal from the context shows, in a prompt and when decoding."""
+    cfg = S.config([S.layer(S.mixer_latent(heads=4, dim=16, rot=8, kv_rank=64, scale=0.7), None),
+                    S.layer(S.mixer_latent(heads=4, dim=16, rot=8, kv_rank=64, scale=0.7, kv_from=0), None)], width=64, vocab=99)
+    W = S.make_weights(cfg)
+    # position-free matching: queries and keys of equal tokens agree, token 98 and 97 share a strong direction
+    W["embed"][97] = W["embed"][98] = (W["embed"][98] * 3).to(torch.bfloat16)
+    m = load(tmp_path, cfg, W, dt)
+    n = 400
+    toks = [t % 97 for t in S.tokens(n, 97, 3)]
+    toks[17], toks[-1], toks[-40] = 97, 98, 98
+    want = O.forward(cfg, W, toks)
+    other = O.forward(cfg, W, toks[:17] + [5] + toks[18:])
+    assert S.error(want[[-1]], other[[-1]]) > 0.1
+    eng = engine(m, dt)
+    (g,) = eng.feed([("p", toks, [n - 40, n - 1])])
+    assert close(g, want[[n - 40, n - 1]], dt)
+    eng.feed_end("p")
+    (g,) = eng.feed([("q", toks[:n - 40], [])])
+    rows = [eng.feed([("q", [t], [0])])[0] for t in toks[n - 40:]]
+    assert close(torch.cat(rows), want[n - 40:], dt)
+
+
+def greedy(cfg, W, prompt, n):
+    seq = list(prompt)
+    for _ in range(n):
+        seq.append(int(O.forward(cfg, W, seq)[-1].argmax()))
+    return seq[len(prompt):]
+
+
+@pytest.mark.parametrize("blocks,graphs", [(64, True), (64, False), (7, True)])
+def test_generation(gpu, tmp_path, blocks, graphs):
+    """Greedy generation of six requests over three decode rows, with and without graphs, and over a pool so small that
+    sequences are preempted and prefilled again."""
+    from nats_llm_studio_amd.engine.engine import GenRequest
+    from nats_llm_studio_amd.engine.sampling import SamplingParams
+    cfg = S.CONFIGS["uneven"]
+    W = S.make_weights(cfg)
+    m = load(tmp_path, cfg, W, "f32")
+    eng = engine(m, "f32", max_batch=3, num_blocks=blocks, max_prefill_tokens=40, use_graphs=graphs, max_logit_rows=0)
+    eng.gen_ratio = 0.0                  # admit on the prompts alone
+    if graphs:
+        eng.capture_all()
+    reqs = [(S.tokens(6 + 11 * i, cfg["vocab"], 20 + i), 24 - 2 * i) for i in range(6)]
+    futs = [eng.submit(GenRequest(p, SamplingParams(max_tokens=n, ignore_eos=True))) for p, n in reqs]
+    for _ in range(1000):
+        if all(f.done() for f in futs):
+            break
+        eng.step()
+    for (p, n), f in zip(reqs, futs):
+        assert f.result().token_ids == greedy(cfg, W, p, n)
+    assert len(eng.slots.free) == 3
+    assert blocks == 64 or eng.counters["preemptions"] > 0
+    assert not graphs or eng.counters["graph_replays"] > 0
+
+
+def test_generation_bf16(gpu, tmp_path):
+    """bf16 greedy tokens are the plain implementation's, or nearly as likely."""
+    from nats_llm_studio_amd.engine.sampling import SamplingParams
+    cfg = S.CONFIGS["wide"]
+    W = S.make_weights(cfg)
+    eng = engine(load(tmp_path, cfg, W, "bf16"), "bf16", max_logit_rows=0)
+    p = S.tokens(60, cfg["vocab"], 5)
+    r = eng.generate(p, SamplingParams(max_tokens=30, ignore_eos=True))
+    lg = O.forward(cfg, W, p + r.token_ids)[len(p) - 1:-1]
+    gap = lg.max(-1).values - lg[torch.arange(30), torch.tensor(r.token_ids)]
+    assert float((gap / lg.std() < 0.1).double().mean()) > 0.8
+
+
+def test_seeded_sampling(gpu, tmp_path):
+    """A seeded sampled request draws the same tokens alone and beside greedy ones."""
+    from nats_llm_studio_amd.engine.engine import GenRequest
+    from nats_llm_studio_amd.engine.sampling import SamplingParams
+    cfg = S.CONFIGS["uneven"]
+    eng = engine(load(tmp_path, cfg, S.make_weights(cfg), "f32"), "f32", max_logit_rows=0)
+    p = S.tokens(60, cfg["vocab"], 5)
+    sp = SamplingParams(max_tokens=12, ignore_eos=True, temperature=0.9, top_k=30, seed=11)
+    alone = eng.generate(p, sp).token_ids
+    futs = [eng.submit(GenRequest(p, sp))] + [eng.submit(GenRequest(S.tokens(9, 200, i), SamplingParams(
+        max_tokens=15, ignore_eos=True))) for i in range(3)]
+    while not all(f.done() for f in futs):
+        eng.step()
+    assert futs[0].result().token_ids == alone and len(set(alone)) > 3
+
+
+@pytest.mark.parametrize("dt", DT)
+def test_long_decoding_and_graph_replays(gpu, tmp_path, dt):
+    """A few hundred decoded tokens through the captured graph, every replay checked."""
+    cfg = S.CONFIGS["ones"]
+    W = S.make_weights(cfg)
+    eng = engine(load(tmp_path, cfg, W, dt), dt)
+    toks = S.tokens(320, cfg["vocab"], 4)
+    want = O.forward(cfg, W, toks)
+    eng.feed([("x", toks[:20], [])])
+    rows = [eng.feed([("x", [t], [0])])[0] for t in toks[20:]]
+    assert close(torch.cat(rows), want[20:], dt)
+    assert eng.counters["graph_replays"] > 250
+
+
+def test_trace_runner(gpu, tmp_path):
+    """The trace runner as a user starts it: steps on standard input, files of logits, one line per step."""
+    import json
+    import os
+    import subprocess
+    import sys
+    import numpy as np
+    cfg = S.CONFIGS["uneven"]
+    W = S.make_weights(cfg)
+    d = S.write_model(str(tmp_path / "m"), cfg, W)
+    toks = S.tokens(50, cfg["vocab"], 9)
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    steps = [{"step": 0, "entries": [{"id": "q", "tokens": toks[:40], "want": [39, 0]}], "end": []},
+             {"step": 1, "entries": [{"id": "q", "tokens": toks[40:41], "want": []}, {"id": "r", "tokens": toks[:2], "want": [1]}],
+              "end": ["r"]},
+             {"step": 2, "entries": [{"id": "q", "tokens": toks[41:], "want": [8]}], "end": ["q"]}]
+    p = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", d, "--dtype", "float32", "--out",
+                        str(tmp_path), "--max-tokens", "128"], input="\n".join(map(json.dumps, steps)) + "\n", text=True,
+                       capture_output=True, timeout=110)
+    assert p.returncode == 0, p.stderr[-2000:]
+    assert [x for x in p.stdout.splitlines() if x.startswith("done")] == ["done 0", "done 1", "done 2"]
+    want = O.forward(cfg, W, toks)
+    for n, rows in ((0, want[[39, 0]]), (1, want[[1]]), (2, want[[49]])):
+        g = torch.from_numpy(np.fromfile(str(tmp_path / f"{n}.f32"), dtype="<f4")).view(-1, cfg["vocab"])
+        assert g.shape == rows.shape and S.error(g, rows) < F32
+    assert not os.path.exists(str(tmp_path / "3.f32"))
+
+
+def test_chat_service(gpu, tmp_path):
+    """A chat request over the worker's engine backend: listing, load by folder, generation, reply."""
+    import threading
+    from nats_llm_studio_amd.service.backends import EngineBackend
+    from nats_llm_studio_amd.service.config import WorkerConfig
+    from nats_llm_studio_amd.service.registry import Registry
+    cfg = S.CONFIGS["uneven"]
+    W = S.make_weights(cfg)
+    S.write_model(str(tmp_path / "pub" / "seko"), cfg, W)
+    reg = Registry(str(tmp_path))
+    reg.scan()
+    be = EngineBackend(WorkerConfig(models_dir=str(tmp_path), device="cuda:0", max_batch=4, max_ctx=256, dtype="float32",
+                                    max_prefill_tokens=256))
+    got, ev = [], threading.Event()
+
+    def done(status, body, *a):
+        got.append((status, body))
+        ev.set()
+    be.chat("seko", reg.resolve("seko"), {"messages": [{"role": "user", "content": "5 17 3 99"}], "max_tokens": 6,
+                                          "ignore_eos": True}, done)
+    assert ev.wait(100)
+    status, body = got[0]
+    assert status == 200, body
+    assert body["model_info"]["arch"] == "Sekolorn" and body["model_info"]["format"] == "safetensors"
+    assert [int(t) for t in body["choices"][0]["message"]["content"].split()] == greedy(cfg, W, [5, 17, 3, 99], 6)
+    assert be.unload("seko")
