@@ -71,7 +71,10 @@ def parse(argv=None):
                     help="seconds before the TP leg is abandoned (bounds what it adds to an N-GPU run)")
     ap.add_argument("--stack", default=None, choices=("prefill", "decode", "all"),
                     help="instead of the headline workload: the config-driven stack design (Sekolorn) at sizes of real "
-                         "layers beside a Mixtral-shaped model of the GGUF families at equal size (bench_stack.py)")
+                         "layers beside a Mixtral-shaped model of the GGUF families at equal size (nats_llm_studio_amd/bench_stack.py)")
+    ap.add_argument("--stack-sizes", default="2k,4k,4k-fine", help="with --stack: sizes to run")
+    ap.add_argument("--stack-only", default=None, choices=("sekolorn", "closest"), help="with --stack: one of the two models")
+    ap.add_argument("--stack-case", default=None, help="with --stack: one BATCHxPROMPT case")
     ap.add_argument("--step-breakdown", action="store_true",
                     help="report host time vs time blocked on the previous step's tokens (diagnostic)")
     a = ap.parse_args(argv)
@@ -101,6 +104,9 @@ def spawn(args, argv) -> int:
 def main(argv=None):
     argv = list(sys.argv[1:] if argv is None else argv)
     args = parse(argv)
+    if args.stack:
+        from nats_llm_studio_amd import bench_stack
+        return bench_stack.run(args)
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         return spawn(args, argv)
     world = int(os.environ.get("WORLD_SIZE", "1"))

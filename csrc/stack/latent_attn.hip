@@ -2,11 +2,12 @@
 // token, [c (R, padded to Rp) | rotated key part (padded to rp)], so with the up-projections folded into the query and
 // applied to the output the cache is read once for all heads: score = q_abs . c + q_rot . k_rot, out = sum p c.
 //
-// latent_attn_kernel (bf16): workgroup = (token, split of the keys, 16 heads), 4 waves. KT-key tiles of the cache rows
-// arrive by LDS-DMA into two buffers (16-byte chunks swizzled by the key on the DMA source); each wave forms S^T of 16
-// keys (A = cache rows, B = the queries, held in registers), the waves exchange row maxima and the bf16 weights through
-// LDS, and each wave owns a quarter of the output columns: O^T += C^T P^T with C^T fragments from transposed LDS reads
-// of the same tile. Softmax in base 2, all of it f32.
+// latent_attn_kernel (bf16): workgroup = (token, split of the keys, NHB blocks of 16 heads), 4 waves per head block.
+// KT-key tiles of the cache rows arrive by LDS-DMA into two buffers (16-byte chunks swizzled by the key on the DMA
+// source), once for all head blocks; each wave forms S^T of 16 keys (A = cache rows, B = its block's queries, held in
+// registers), the four waves of a block exchange row maxima and the bf16 weights through LDS, and each owns a quarter of
+// the output columns: O^T += C^T P^T with C^T fragments from transposed LDS reads of the same tile. Softmax in base 2, all
+// of it f32.
 // latent_attn_f32_kernel: the f32 form, one workgroup per (token, head).
 #include "../kernels/lds_dma.h"
 
@@ -26,7 +27,7 @@ struct LA {
   const int* bt;            // block tables
   const int* tok_seq;
   const int* ctx_len;       // keys of each token (0: padded row)
-  int bts, bs, T, H, ns, Rp, rp;
+  int bts, bs, T, H, ns, Rp, rp, bshift;
   float scale;
 };
 
@@ -38,21 +39,24 @@ DEVI void bar_lgkm() {
 
 constexpr int NBT = 1024;    // block-table entries of the split kept in LDS
 
-template <int NT, int RT, int KT>
-__global__ __launch_bounds__(256, 1) void latent_attn_kernel(LA p) {
+template <int NT, int RT, int KT, int NHB>
+__global__ __launch_bounds__(256 * NHB, 1) void latent_attn_kernel(LA p) {
   constexpr int Rp = 64 * NT, Dp = Rp + 64 * RT;
   constexpr int CPR = Dp / 8;                  // 16-byte chunks per row
   constexpr int TB = KT * Dp * 2;              // bytes per tile
-  constexpr int ND = TB / 4096;                // DMA instructions per wave per tile
+  constexpr int NDT = TB / 1024;               // DMA instructions per tile
+  constexpr int ND = (NDT + 4 * NHB - 1) / (4 * NHB);   // ... per wave (the last ones may be idle)
   constexpr int NK = Dp / 32;                  // k-steps of a score
   constexpr int PS = KT + 8;                   // P row stride
-  static_assert(TB % 4096 == 0, "tile");
+  static_assert(TB % 1024 == 0, "tile");
   extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-  __bf16* P = reinterpret_cast<__bf16*>(lds + 2 * TB);                 // [16][PS]
-  float* mx = reinterpret_cast<float*>(lds + 2 * TB + 16 * PS * 2);    // [4][16]
-  int* btl = reinterpret_cast<int*>(mx + 64);                          // [NBT]
+  const int wv = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int wave = wv & 3, hsub = wv >> 2;     // wave of its head block; head block of the workgroup
+  __bf16* P = reinterpret_cast<__bf16*>(lds + 2 * TB) + hsub * 16 * PS;                  // [NHB][16][PS]
+  float* mx = reinterpret_cast<float*>(lds + 2 * TB + NHB * 16 * PS * 2) + hsub * 64;    // [NHB][4][16]
+  int* btl = reinterpret_cast<int*>(lds + 2 * TB + NHB * (16 * PS * 2 + 256));           // [NBT]
 
-  const int HB = (p.H + 15) >> 4;
+  const int HB = (p.H + 16 * NHB - 1) / (16 * NHB);
   const int ts = ((int)blockIdx.x / (8 * HB)) * 8 + (blockIdx.x & 7);
   const int hb = ((int)blockIdx.x >> 3) % HB;
   if (ts >= p.T * p.ns) return;
@@ -61,9 +65,8 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LA p) {
   const int chunk = ((ctx + p.ns - 1) / p.ns + KT - 1) / KT * KT;
   const int k0 = split * chunk, k1 = min(ctx, k0 + chunk);
   const int lane = threadIdx.x & 63;
-  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int r = lane & 15, g = lane >> 4;
-  const int head = hb * 16 + r;
+  const int head = (hb * NHB + hsub) * 16 + r;
   const __bf16* cache = reinterpret_cast<const __bf16*>(p.cache);
   const int* bt = p.bt + (size_t)p.tok_seq[t] * p.bts;
 
@@ -73,8 +76,8 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LA p) {
   float m = -INFINITY, l = 0.f;
 
   if (k0 < k1) {
-    const int b0 = k0 / p.bs, nb = (k1 - 1) / p.bs - b0 + 1;
-    for (int i = threadIdx.x; i < min(nb, NBT); i += 256) btl[i] = bt[b0 + i];
+    const int b0 = k0 >> p.bshift, nb = ((k1 - 1) >> p.bshift) - b0 + 1, bmask = p.bs - 1;
+    for (int i = threadIdx.x; i < min(nb, NBT); i += 256 * NHB) btl[i] = bt[b0 + i];
     u32x4 qf[NK];
     const __bf16* qr = reinterpret_cast<const __bf16*>(p.q) + ((size_t)t * p.H + min(head, p.H - 1)) * Dp;
 #pragma unroll
@@ -83,15 +86,16 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LA p) {
     const float sl2 = p.scale * 1.4426950408889634f;
     const uint32_t base = __builtin_amdgcn_readfirstlane(lds_addr(lds));
     auto dma = [&](int j) __attribute__((always_inline)) {
-      const uint32_t dst = base + (uint32_t)(j & 1) * TB + (uint32_t)(ND * wave) * 1024u;
+      const uint32_t dst = base + (uint32_t)(j & 1) * TB + (uint32_t)(ND * wv) * 1024u;
 #pragma unroll
       for (int i = 0; i < ND; ++i) {
-        const int ci = (ND * wave + i) * 64 + lane;
+        if (NDT % (4 * NHB) != 0 && ND * wv + i >= NDT) break;
+        const int ci = (ND * wv + i) * 64 + lane;
         const int row = ci / CPR, pc = ci - row * CPR;
         const int key = min(k0 + j * KT + row, k1 - 1);
-        const int bi = key / p.bs - b0;
+        const int bi = (key >> p.bshift) - b0;
         const int blk = bi < NBT ? btl[bi] : bt[b0 + bi];
-        glds16(cache + ((size_t)blk * p.bs + key % p.bs) * Dp + (pc ^ (row & 7)) * 8, dst + i * 1024);
+        glds16(cache + (((size_t)blk << p.bshift) + (key & bmask)) * Dp + (pc ^ (row & 7)) * 8, dst + i * 1024);
       }
     };
     const int nt = (k1 - k0 + KT - 1) / KT;
@@ -104,13 +108,14 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LA p) {
       f32x4 s = f32x4{-INFINITY, -INFINITY, -INFINITY, -INFINITY};
       float tm = -INFINITY;
       if (KT == 64 || wave < KT / 16) {
-        s = f32x4{0.f, 0.f, 0.f, 0.f};
+        f32x4 s2[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};     // two chains of dependent products
         const int row = 16 * wave + r;
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) {
           const bf16x8 a = *reinterpret_cast<const bf16x8*>(cb + row * (2 * Dp) + (((4 * kk + g) ^ (row & 7)) << 4));
-          s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, __builtin_bit_cast(bf16x8, qf[kk]), s, 0, 0, 0);
+          s2[kk & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, __builtin_bit_cast(bf16x8, qf[kk]), s2[kk & 1], 0, 0, 0);
         }
+        s = s2[0] + s2[1];
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           s[i] = k0 + j * KT + 16 * wave + 4 * g + i < k1 ? s[i] * sl2 : -INFINITY;
@@ -178,6 +183,7 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LA p) {
     return;
   }
   const size_t pi = ((size_t)t * p.H + head) * p.ns + split;
+  if (k0 < k1)                                 // (an empty split weighs nothing: only its (m, l) is read)
 #pragma unroll
   for (int c = 0; c < NT; ++c)
     *reinterpret_cast<f32x4*>(p.part_o + pi * Rp + wave * NT * 16 + 16 * c + 4 * g) = o[c];
@@ -187,20 +193,38 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(LA p) {
   }
 }
 
+// splits of one (token, head), 64 output columns: 16 lanes x 4 columns, 16 groups of splits
 __global__ __launch_bounds__(256) void latent_merge_kernel(LA p) {
+  __shared__ float w[64];
+  __shared__ f32x4 red[16][16];
   const size_t th = blockIdx.x;
   const float* ml = p.part_ml + th * p.ns * 2;
-  float M = -INFINITY, L = 0.f;
-  for (int s = 0; s < p.ns; ++s) M = fmaxf(M, ml[2 * s]);
-  if (M == -INFINITY) M = 0.f;
-  for (int s = 0; s < p.ns; ++s) L += ml[2 * s + 1] * exp2f(ml[2 * s] - M);
-  const float inv = L > 0.f ? 1.f / L : 0.f;
-  const float* po = p.part_o + th * p.ns * p.Rp;
-  __bf16* y = reinterpret_cast<__bf16*>(p.out) + th * p.Rp;
-  for (int i = threadIdx.x; i < p.Rp; i += 256) {
-    float a = 0.f;
-    for (int s = 0; s < p.ns; ++s) a += po[(size_t)s * p.Rp + i] * exp2f(ml[2 * s] - M);
-    y[i] = (__bf16)(a * inv);
+  const int lane = threadIdx.x & 63;
+  if (threadIdx.x < 64) {
+    const float m = lane < p.ns ? ml[2 * lane] : -INFINITY, l = lane < p.ns ? ml[2 * lane + 1] : 0.f;
+    float M = m;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) M = fmaxf(M, __shfl_xor(M, o, 64));
+    const float e = m == -INFINITY ? 0.f : exp2f(m - M);
+    float L = l * e;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) L += __shfl_xor(L, o, 64);
+    w[lane] = L > 0.f ? e / L : 0.f;
+  }
+  __syncthreads();
+  const int c = threadIdx.x & 15, g = threadIdx.x >> 4;
+  const float* po = p.part_o + th * p.ns * p.Rp + blockIdx.y * 64 + 4 * c;
+  f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int s = g; s < p.ns; s += 16)
+    if (w[s] != 0.f) a += *reinterpret_cast<const f32x4*>(po + (size_t)s * p.Rp) * w[s];
+  red[g][c] = a;
+  __syncthreads();
+  if (g == 0) {
+#pragma unroll
+    for (int i = 1; i < 16; ++i) a += red[i][c];
+    typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+    *reinterpret_cast<bf4*>(reinterpret_cast<__bf16*>(p.out) + th * p.Rp + blockIdx.y * 64 + 4 * c) =
+        bf4{(__bf16)a[0], (__bf16)a[1], (__bf16)a[2], (__bf16)a[3]};
   }
 }
 
@@ -262,23 +286,23 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(LA p) {
   }
 }
 
-template <int NT, int RT>
+template <int NT, int RT, int NHB>
 int launch_t(const LA& p, hipStream_t st) {
   constexpr int KT = NT + RT > 9 ? 32 : 64;
-  constexpr int LDS = 2 * KT * 128 * (NT + RT) + 16 * (KT + 8) * 2 + 256 + NBT * 4;
+  constexpr int LDS = 2 * KT * 128 * (NT + RT) + NHB * (16 * (KT + 8) * 2 + 256) + NBT * 4;
   static_assert(LDS <= 160 * 1024, "LDS");
   static bool attr = false;
   if (!attr) {
-    if (hipFuncSetAttribute((const void*)latent_attn_kernel<NT, RT, KT>, hipFuncAttributeMaxDynamicSharedMemorySize,
-                            LDS) != hipSuccess)
+    if (hipFuncSetAttribute((const void*)latent_attn_kernel<NT, RT, KT, NHB>,
+                            hipFuncAttributeMaxDynamicSharedMemorySize, LDS) != hipSuccess)
       return -1;
     attr = true;
   }
-  const int HB = (p.H + 15) / 16, n = (p.T * p.ns + 7) / 8 * 8 * HB;
-  hipLaunchKernelGGL((latent_attn_kernel<NT, RT, KT>), dim3(n), dim3(256), LDS, st, p);
+  const int HB = (p.H + 16 * NHB - 1) / (16 * NHB), n = (p.T * p.ns + 7) / 8 * 8 * HB;
+  hipLaunchKernelGGL((latent_attn_kernel<NT, RT, KT, NHB>), dim3(n), dim3(256 * NHB), LDS, st, p);
   int rc = (int)hipGetLastError();
   if (rc == 0 && p.ns > 1) {
-    hipLaunchKernelGGL(latent_merge_kernel, dim3(p.T * p.H), dim3(256), 0, st, p);
+    hipLaunchKernelGGL(latent_merge_kernel, dim3(p.T * p.H, p.Rp / 64), dim3(256), 0, st, p);
     rc = (int)hipGetLastError();
   }
   return rc;
@@ -286,8 +310,10 @@ int launch_t(const LA& p, hipStream_t st) {
 
 template <int NT>
 int launch_r(const LA& p, hipStream_t st) {
-  if (p.rp == 64) return launch_t<NT, 1>(p, st);
-  if (p.rp == 128) return launch_t<NT, 2>(p, st);
+  // 17 .. 32 heads (and pairs of 16-head blocks beyond) share a workgroup's tiles
+  constexpr int PAIR = NT < 16 ? 2 : 1;        // (the widest latents would spill)
+  if (p.rp == 64) return p.H > 16 ? launch_t<NT, 1, PAIR>(p, st) : launch_t<NT, 1, 1>(p, st);
+  if (p.rp == 128) return p.H > 16 ? launch_t<NT, 2, PAIR>(p, st) : launch_t<NT, 2, 1>(p, st);
   return -1;
 }
 
@@ -301,8 +327,10 @@ int nls_latent_attn(const void* q, const void* cache, void* out, float* part_o, 
                     int bs, const int* tok_seq, const int* ctx_len, int T, int H, int ns, int Rp, int rp, float scale,
                     int f32, void* stream) {
   using namespace nls_latent;
-  if (T < 1 || H < 1 || ns < 1 || bs < 1 || (ns > 1 && (!part_o || !part_ml))) return -1;
-  LA p{q, cache, out, part_o, part_ml, bt, tok_seq, ctx_len, bts, bs, T, H, ns, Rp, rp, scale};
+  if (T < 1 || H < 1 || ns < 1 || ns > 64 || bs < 1 || (bs & (bs - 1)) || (ns > 1 && (!part_o || !part_ml))) return -1;
+  int bshift = 0;
+  while ((1 << bshift) < bs) ++bshift;
+  LA p{q, cache, out, part_o, part_ml, bt, tok_seq, ctx_len, bts, bs, T, H, ns, Rp, rp, bshift, scale};
   hipStream_t st = (hipStream_t)stream;
   if (f32) {
     if (Rp > 256 * NC || Rp + rp > 2048 || (Rp & 3) || (rp & 3) || H > 65535) return -1;

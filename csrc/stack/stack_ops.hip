@@ -38,16 +38,28 @@ __global__ __launch_bounds__(256) void embed_kernel(int* __restrict__ ids, const
   id = min(max(id, 0), V - 1);
   __syncthreads();
   if (threadIdx.x == 0 && use_prev) ids[t] = id;
+  const __bf16* row = tab + (size_t)id * D;
+  if ((D & 7) == 0) {
+    for (int i = threadIdx.x * 8; i < D; i += 2048) {
+      const u32x4 v = ld16(row + i);
+      const bf16x8 b = __builtin_bit_cast(bf16x8, v);
+      float* o = x + (size_t)t * ldx + i;
+      *reinterpret_cast<f32x4*>(o) = f32x4{(float)b[0], (float)b[1], (float)b[2], (float)b[3]};
+      *reinterpret_cast<f32x4*>(o + 4) = f32x4{(float)b[4], (float)b[5], (float)b[6], (float)b[7]};
+      if (xb) *reinterpret_cast<u32x4*>(xb + (size_t)t * ldx + i) = v;
+    }
+    return;
+  }
   for (int i = threadIdx.x; i < D; i += 256) {
-    const __bf16 v = tab[(size_t)id * D + i];
+    const __bf16 v = row[i];
     x[(size_t)t * ldx + i] = (float)v;
     if (xb) xb[(size_t)t * ldx + i] = v;
   }
 }
 
 // ---- x[t] += LayerNorm(y) * w; y = one row, or (topk) sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t], the shared
-// expert). Optional second LayerNorm (the model's last norm) of the new x into `on` instead of xb.
-// Each of the 256 threads keeps its <= 8 float4 of the row in registers up to D = 8192; wider rows take the LDS copy.
+// expert); y null: x is only read. Optional second LayerNorm (the model's last norm) of the new x into `on`.
+// A workgroup per row (`rows`: gathered), 4 consecutive columns x NV per thread in registers.
 struct NormAdd {
   const float* y;
   const float* topw;
@@ -56,99 +68,135 @@ struct NormAdd {
   __bf16* xb;
   const float* ow;      // optional output norm weight
   void* on;             // its output, activation type
+  const int* rows;      // optional: row i of the launch is row rows[i] of x
   long ldy, ldx, ldo;
   long sh0;             // first shared-expert row, -1: none
   int D, topk, f32;
   float eps;
 };
 
-template <int NV>
-__global__ __launch_bounds__(256) void norm_add_kernel(NormAdd p) {
-  __shared__ float sh[4];
-  const int t = blockIdx.x, D = p.D;
-  float v[4 * NV], xr[4 * NV];
+// 4 consecutive values, columns i .. i + 3 of a row of D (VEC: D and the row strides are multiples of 4)
+template <bool VEC>
+DEVI f32x4 row4(const float* p, int i, int D) {
+  f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
+  if (VEC) {
+    if (i < D) v = *reinterpret_cast<const f32x4*>(p + i);
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (i + e < D) v[e] = p[i + e];
+  }
+  return v;
+}
+template <bool VEC>
+DEVI void put4(float* p, int i, int D, const f32x4& v) {
+  if (VEC) {
+    if (i < D) *reinterpret_cast<f32x4*>(p + i) = v;
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (i + e < D) p[i + e] = v[e];
+  }
+}
+template <bool VEC>
+DEVI void put4(__bf16* p, int i, int D, const f32x4& v) {
+  typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+  const bf4 b = {(__bf16)v[0], (__bf16)v[1], (__bf16)v[2], (__bf16)v[3]};
+  if (VEC) {
+    if (i < D) *reinterpret_cast<bf4*>(p + i) = b;
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (i + e < D) p[i + e] = b[e];
+  }
+}
+// (v - mean) / sqrt(var + eps) over the row's D columns
+template <int NV, int NTH>
+DEVI void normalise(f32x4 (&v)[NV], int D, float eps, float* sh) {
   float s = 0.f;
 #pragma unroll
-  for (int j = 0; j < NV; ++j) {
+  for (int j = 0; j < NV; ++j) s += (v[j][0] + v[j][1]) + (v[j][2] + v[j][3]);
+  const float mean = bsum<NTH / 64>(s, sh) / (float)D;
+  s = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j)
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
-      const int i = (threadIdx.x + j * 256) * 4 + e;
-      float a = 0.f, b = 0.f;
-      if (i < D) {
-        b = p.x[(size_t)t * p.ldx + i];
-        if (p.topk) {
-          for (int k = 0; k < p.topk; ++k)
-            a += p.topw[t * p.topk + k] * p.y[((size_t)t * p.topk + k) * p.ldy + i];
-          if (p.sh0 >= 0) a += p.y[(size_t)(p.sh0 + t) * p.ldy + i];
-        } else {
-          a = p.y[(size_t)t * p.ldy + i];
-        }
-      }
-      v[4 * j + e] = a;
-      xr[4 * j + e] = b;
-      s += a;
+      const float d = (int)(threadIdx.x + j * NTH) * 4 + e < D ? v[j][e] - mean : 0.f;
+      v[j][e] = d;
+      s += d * d;
     }
-  }
-  const float mean = bsum<4>(s, sh) / (float)D;
-  s = 0.f;
+  const float inv = 1.f / sqrtf(bsum<NTH / 64>(s, sh) / (float)D + eps);
 #pragma unroll
-  for (int j = 0; j < 4 * NV; ++j) {
-    const int i = (threadIdx.x + (j >> 2) * 256) * 4 + (j & 3);
-    const float d = i < D ? v[j] - mean : 0.f;
-    v[j] = d;
-    s += d * d;
-  }
-  const float inv = 1.f / sqrtf(bsum<4>(s, sh) / (float)D + p.eps);
-  s = 0.f;
+  for (int j = 0; j < NV; ++j) v[j] *= inv;
+}
+
+template <int NV, int NTH, bool VEC>
+__global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
+  __shared__ float sh[NTH / 64];
+  const int t = p.rows ? p.rows[blockIdx.x] : (int)blockIdx.x, D = p.D;
+  float* xr = p.x + (size_t)t * p.ldx;
+  f32x4 v[NV], x[NV], w[NV];
 #pragma unroll
-  for (int j = 0; j < 4 * NV; ++j) {
-    const int i = (threadIdx.x + (j >> 2) * 256) * 4 + (j & 3);
-    if (i < D) {
-      const float o = xr[j] + v[j] * inv * p.w[i];
-      xr[j] = o;
-      s += o;
-      p.x[(size_t)t * p.ldx + i] = o;
-      if (p.xb) p.xb[(size_t)t * p.ldx + i] = (__bf16)o;
+  for (int j = 0; j < NV; ++j) x[j] = row4<VEC>(xr, (threadIdx.x + j * NTH) * 4, D);
+  if (p.y) {
+#pragma unroll
+    for (int j = 0; j < NV; ++j) w[j] = row4<VEC>(p.w, (threadIdx.x + j * NTH) * 4, D);
+    if (p.topk) {
+#pragma unroll
+      for (int j = 0; j < NV; ++j)
+        v[j] = p.sh0 >= 0 ? row4<VEC>(p.y + (size_t)(p.sh0 + t) * p.ldy, (threadIdx.x + j * NTH) * 4, D)
+                          : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+      for (int k = 0; k < p.topk; ++k) {
+        const float wk = p.topw[(size_t)t * p.topk + k];
+        const float* yr = p.y + ((size_t)t * p.topk + k) * p.ldy;
+#pragma unroll
+        for (int j = 0; j < NV; ++j) v[j] += row4<VEC>(yr, (threadIdx.x + j * NTH) * 4, D) * wk;
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < NV; ++j) v[j] = row4<VEC>(p.y + (size_t)t * p.ldy, (threadIdx.x + j * NTH) * 4, D);
+    }
+    normalise<NV, NTH>(v, D, p.eps, sh);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int i = (threadIdx.x + j * NTH) * 4;
+      x[j] += v[j] * w[j];
+      put4<VEC>(xr, i, D, x[j]);
+      if (p.xb) put4<VEC>(p.xb + (size_t)t * p.ldx, i, D, x[j]);
     }
   }
   if (!p.ow) return;
-  const float m2 = bsum<4>(s, sh) / (float)D;
-  s = 0.f;
 #pragma unroll
-  for (int j = 0; j < 4 * NV; ++j) {
-    const int i = (threadIdx.x + (j >> 2) * 256) * 4 + (j & 3);
-    const float d = i < D ? xr[j] - m2 : 0.f;
-    s += d * d;
-  }
-  const float inv2 = 1.f / sqrtf(bsum<4>(s, sh) / (float)D + p.eps);
+  for (int j = 0; j < NV; ++j) w[j] = row4<VEC>(p.ow, (threadIdx.x + j * NTH) * 4, D);
+  normalise<NV, NTH>(x, D, p.eps, sh);
 #pragma unroll
-  for (int j = 0; j < 4 * NV; ++j) {
-    const int i = (threadIdx.x + (j >> 2) * 256) * 4 + (j & 3);
-    if (i < D) {
-      const float o = (xr[j] - m2) * inv2 * p.ow[i];
-      if (p.f32) reinterpret_cast<float*>(p.on)[(size_t)t * p.ldo + i] = o;
-      else reinterpret_cast<__bf16*>(p.on)[(size_t)t * p.ldo + i] = (__bf16)o;
-    }
+  for (int j = 0; j < NV; ++j) {
+    const int i = (threadIdx.x + j * NTH) * 4;
+    if (p.f32) put4<VEC>(reinterpret_cast<float*>(p.on) + (size_t)blockIdx.x * p.ldo, i, D, x[j] * w[j]);
+    else put4<VEC>(reinterpret_cast<__bf16*>(p.on) + (size_t)blockIdx.x * p.ldo, i, D, x[j] * w[j]);
   }
 }
 
-// ---- out[i] = LayerNorm(x[rows ? rows[i] : i]) * w
-__global__ __launch_bounds__(256) void layer_norm_kernel(const float* __restrict__ x, long ldx,
-                                                         const int* __restrict__ rows, const float* __restrict__ w,
-                                                         void* __restrict__ out, long ldo, int D, float eps, int f32) {
-  __shared__ float sh[4];
-  const float* xr = x + (size_t)(rows ? rows[blockIdx.x] : (int)blockIdx.x) * ldx;
-  float s = 0.f;
-  for (int i = threadIdx.x; i < D; i += 256) s += xr[i];
-  const float mean = bsum<4>(s, sh) / (float)D;
-  s = 0.f;
-  for (int i = threadIdx.x; i < D; i += 256) s += (xr[i] - mean) * (xr[i] - mean);
-  const float inv = 1.f / sqrtf(bsum<4>(s, sh) / (float)D + eps);
-  for (int i = threadIdx.x; i < D; i += 256) {
-    const float o = (xr[i] - mean) * inv * w[i];
-    if (f32) reinterpret_cast<float*>(out)[(size_t)blockIdx.x * ldo + i] = o;
-    else reinterpret_cast<__bf16*>(out)[(size_t)blockIdx.x * ldo + i] = (__bf16)o;
+template <bool VEC>
+int norm_add_v(const NormAdd& p, int n, hipStream_t st) {
+#define NLS_NA(LIM, NV, NTH) \
+  if (p.D <= LIM) { \
+    hipLaunchKernelGGL((norm_add_kernel<NV, NTH, VEC>), dim3(n), dim3(NTH), 0, st, p); \
+    return (int)hipGetLastError(); \
   }
+  NLS_NA(1024, 1, 256) NLS_NA(2048, 2, 256)
+  if (n <= 64) { NLS_NA(4096, 1, 1024) NLS_NA(8192, 2, 1024) }      // few rows: shorter per-thread chains
+  NLS_NA(4096, 4, 256) NLS_NA(8192, 4, 512) NLS_NA(16384, 4, 1024)
+#undef NLS_NA
+  return -1;
+}
+
+inline int norm_add(const NormAdd& p, int n, hipStream_t st) {
+  if (n < 1 || p.D < 1) return -1;
+  const bool vec = !(p.D & 3) && !(p.ldx & 3) && !(p.ldy & 3) && !(p.ldo & 3);
+  return vec ? norm_add_v<true>(p, n, st) : norm_add_v<false>(p, n, st);
 }
 
 // ---- latent attention rows: cq = RMSNorm(dq) * wq -> activation; c = RMSNorm(dkv[:R]) * wc and the rotated key part
@@ -317,7 +365,16 @@ __global__ __launch_bounds__(1024) void argmax_kernel(const float* __restrict__ 
   const float* r = z + (size_t)blockIdx.x * ldz;
   float v = -INFINITY;
   int ix = 0x7fffffff;
-  for (int i = threadIdx.x; i < V; i += 1024) {
+  int i = threadIdx.x;
+  for (; i + 7 * 1024 < V; i += 8 * 1024) {      // 8 loads in flight
+    float a[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) a[j] = r[i + j * 1024];
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      if (a[j] > v || ix == 0x7fffffff) { v = a[j]; ix = i + j * 1024; }
+  }
+  for (; i < V; i += 1024) {
     const float a = r[i];
     if (a > v || ix == 0x7fffffff) { v = a; ix = i; }
   }
@@ -353,23 +410,16 @@ int nls_stack_embed(int* ids, const int* next_ids, const int* use_prev, const vo
 
 int nls_norm_add(const float* y, long ldy, const float* topw, int topk, long sh0, const float* w, float* x, void* xb,
                  long ldx, const float* ow, void* on, long ldo, int D, int T, float eps, int f32, void* stream) {
-  if (T < 1 || D < 1 || D > 16384) return -1;
-  NormAdd p{y, topw, w, x, (__bf16*)xb, ow, on, ldy, ldx, ldo, sh0, D, topk, f32, eps};
-  hipStream_t st = (hipStream_t)stream;
-  if (D <= 1024) hipLaunchKernelGGL(norm_add_kernel<1>, dim3(T), dim3(256), 0, st, p);
-  else if (D <= 2048) hipLaunchKernelGGL(norm_add_kernel<2>, dim3(T), dim3(256), 0, st, p);
-  else if (D <= 4096) hipLaunchKernelGGL(norm_add_kernel<4>, dim3(T), dim3(256), 0, st, p);
-  else if (D <= 8192) hipLaunchKernelGGL(norm_add_kernel<8>, dim3(T), dim3(256), 0, st, p);
-  else hipLaunchKernelGGL(norm_add_kernel<16>, dim3(T), dim3(256), 0, st, p);
-  return (int)hipGetLastError();
+  if (!y || !w) return -1;
+  return norm_add(NormAdd{y, topw, w, x, (__bf16*)xb, ow, on, nullptr, ldy, ldx, ldo, sh0, D, topk, f32, eps}, T,
+                  (hipStream_t)stream);
 }
 
+// out[i] = LayerNorm(x[rows ? rows[i] : i]) * w
 int nls_layer_norm(const float* x, long ldx, const int* rows, const float* w, void* out, long ldo, int D, int n,
                    float eps, int f32, void* stream) {
-  if (n < 1 || D < 1) return -1;
-  hipLaunchKernelGGL(layer_norm_kernel, dim3(n), dim3(256), 0, (hipStream_t)stream, x, ldx, rows, w, out, ldo, D, eps,
-                     f32);
-  return (int)hipGetLastError();
+  return norm_add(NormAdd{nullptr, nullptr, nullptr, const_cast<float*>(x), nullptr, w, out, rows, 0, ldx, ldo, -1, D, 0,
+                          f32, eps}, n, (hipStream_t)stream);
 }
 
 int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq, long ldcq, const float* dkv,

@@ -4,9 +4,11 @@
 //   o_t[j] = sum_i r_t[i] (S[i][j] + u[i] k_t[i] v_t[j]);   S[i][j] = w_t[i] S[i][j] + k_t[i] v_t[j]
 //
 // The scan is sequential in the tokens of a run, so a position's result does not depend on how its sequence was cut
-// into steps. Parallelism is (run, head, 32 value columns) x lanes: a wave owns 8 value columns, lane = 8 key parts x 8
-// columns, each lane DP / 8 state values in registers; the key sum closes with three lane exchanges. Tokens are staged
-// in LDS in chunks of CH as f32, the next chunk's loads in flight while the current one runs.
+// into steps. Parallelism is (run, head, 32 value columns) x lanes: a wave owns 8 value columns, lane = 8 columns x 8 key
+// parts, each lane DP / 8 state values in registers; the key sum closes with three in-row lane exchanges (DPP). Tokens are
+// staged in LDS in chunks of CH as f32, the next chunk's loads in flight while the current one runs.
+// A step of single tokens (decode) streams each head's state once with 16-byte accesses and ends with the head's norm and
+// gate (wkv_step_kernel).
 //
 // A run = (first row, tokens, state slot, first position): consecutive rows of one sequence. A run at position 0
 // starts from a zero state, any other from its slot; slot < 0 or 0 tokens: nothing to do (padded decode rows).
@@ -39,12 +41,20 @@ __global__ __launch_bounds__(256) void shift_mix_kernel(Mix p) {
   const float* h = p.x + (size_t)t * p.ldx;
   const float* q = t > t0 ? h - p.ldx : (pos0 > 0 ? p.prev + (size_t)slot * p.ldp : nullptr);
   T* o = reinterpret_cast<T*>(p.out) + (size_t)t * p.ldo;
-  for (int i = threadIdx.x; i < p.D; i += 256) {
+  for (int i = blockIdx.y * 256 + threadIdx.x; i < p.D; i += gridDim.y * 256) {
     const float a = h[i], d = (q ? q[i] : 0.f) - a;
 #pragma unroll
     for (int s = 0; s < NS; ++s) o[s * p.mstride + i] = (T)(a + d * p.mu[s * p.D + i]);
   }
 }
+
+// sum over the 8 lanes of a group (lane & 7)
+template <int C>
+DEVI float dpp_add(float v) {
+  const int x = __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), C, 0xf, 0xf, true);
+  return v + __builtin_bit_cast(float, x);
+}
+DEVI float sum8(float v) { return dpp_add<0x141>(dpp_add<0x4E>(dpp_add<0xB1>(v))); }   // quad swaps, then half-row mirror
 
 struct Scan {
   const void *r, *k, *v;   // activation type, [rows][ld]
@@ -62,7 +72,7 @@ struct Scan {
 // DP: key channels padded to a multiple of 32 (zeros past D)
 template <typename T, int DP>
 __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
-  constexpr int CH = DP <= 64 ? 16 : 8;          // tokens per staged chunk
+  constexpr int CH = DP <= 64 ? 32 : (DP <= 128 ? 16 : 8);   // tokens per staged chunk
   constexpr int R = DP / 8;                      // state rows per lane
   constexpr int LR = DP + 4;                     // LDS row stride
   constexpr int NV = (CH * DP + 255) / 256;      // staged values per thread and operand
@@ -75,7 +85,7 @@ __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
   const int ncb = (D + 31) / 32;
   const int head = blockIdx.x / ncb, c0 = (blockIdx.x % ncb) * 32;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int part = lane >> 3, col = wave * 8 + (lane & 7);
+  const int part = lane & 7, col = wave * 8 + (lane >> 3);
   const int j = c0 + col;
   const size_t hb = (size_t)head * D;
   const T* rp = (const T*)p.r + hb;
@@ -128,8 +138,9 @@ __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
     __syncthreads();
     if (base + CH < n) fetch(base + CH);
     // sum_i r u k of every staged token: 16 lanes each
-    {
-      const int tt = threadIdx.x >> 4, l = threadIdx.x & 15;
+#pragma unroll
+    for (int t8 = 0; t8 < CH; t8 += 16) {
+      const int tt = t8 + (threadIdx.x >> 4), l = threadIdx.x & 15;
       float a = 0.f;
       if (tt < CH)
         for (int i = l; i < D; i += 16) a += rs[tt][i] * p.u[hb + i] * ks[tt][i];
@@ -138,8 +149,7 @@ __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
       if (tt < CH && l == 0) ruk[tt] = a;
     }
     __syncthreads();
-    const int m = min(CH, n - base);
-    for (int tt = 0; tt < m; ++tt) {
+    auto token = [&](int tt) __attribute__((always_inline)) {
       const float v = vs[tt][col];
       float o = 0.f;
 #pragma unroll
@@ -153,11 +163,18 @@ __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
           S[i4 + e] = fmaf(w4[e], S[i4 + e], k4[e] * v);
         }
       }
-      o += __shfl_xor(o, 8, 64);
-      o += __shfl_xor(o, 16, 64);
-      o += __shfl_xor(o, 32, 64);
+      o = sum8(o);
       if (part == 0 && j < D) p.o[(size_t)(t0 + base + tt) * p.ldo + hb + j] = o + ruk[tt] * v;
+    };
+    const int m = min(CH, n - base);
+    int tt = 0;
+    for (; tt + 4 <= m; tt += 4) {           // the LDS reads of later tokens overlap the sums of earlier ones
+      token(tt);
+      token(tt + 1);
+      token(tt + 2);
+      token(tt + 3);
     }
+    for (; tt < m; ++tt) token(tt);
   }
 #pragma unroll
   for (int i = 0; i < R; ++i) {
@@ -168,6 +185,66 @@ __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
   const int G = gridDim.x;
   for (int i = blockIdx.x * 256 + threadIdx.x; i < p.width; i += G * 256)
     p.prev[(size_t)slot * p.ldp + i] = p.x[(size_t)(t0 + n - 1) * p.ldx + i];
+}
+
+// ---- one token per run: the state of (run, head) is read and written once, 4 value columns per thread; then
+// out = (o / rms(o)) * norm * gate. D is a multiple of 4.
+template <typename T>
+__global__ __launch_bounds__(256) void wkv_step_kernel(Scan p, const float* __restrict__ norm, const T* __restrict__ gate,
+                                                       long ldg, T* __restrict__ out, long ldout, float eps) {
+  __shared__ __attribute__((aligned(16))) float rs[256], ks[256], ws[256], vs[256], red[1024 + 256];
+  __shared__ float part[8];
+  const int* run = p.runs + 4 * blockIdx.y;
+  const int t = run[0], n = run[1], slot = run[2], pos0 = run[3];
+  if (slot < 0 || n != 1) return;
+  const int D = p.D, head = blockIdx.x, tid = threadIdx.x;
+  const size_t hb = (size_t)head * D;
+  const int C4 = D >> 2, G = 256 / C4, c = (tid % C4) * 4, g = tid / C4;
+  float* st = p.state + (size_t)slot * p.sstride + hb * D;
+  float ruk = 0.f;
+  if (tid < D) {
+    const float r = ld1((const T*)p.r + (size_t)t * p.ld + hb + tid), k = ld1((const T*)p.k + (size_t)t * p.ld + hb + tid);
+    rs[tid] = r;
+    ks[tid] = k;
+    ws[tid] = p.w[(size_t)t * p.ldw + hb + tid];
+    vs[tid] = ld1((const T*)p.v + (size_t)t * p.ld + hb + tid);
+    ruk = r * p.u[hb + tid] * k;
+  }
+#pragma unroll
+  for (int q = 32; q > 0; q >>= 1) ruk += __shfl_xor(ruk, q, 64);
+  if ((tid & 63) == 0) part[tid >> 6] = ruk;
+  __syncthreads();
+  ruk = part[0] + part[1] + part[2] + part[3];
+  if (g < G) {
+    const f32x4 v = *reinterpret_cast<const f32x4*>(vs + c);
+    f32x4 o = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int i = g; i < D; i += G) {
+      float* sp = st + (size_t)i * D + c;
+      const f32x4 s = pos0 > 0 ? *reinterpret_cast<const f32x4*>(sp) : f32x4{0.f, 0.f, 0.f, 0.f};
+      o += s * rs[i];
+      *reinterpret_cast<f32x4*>(sp) = s * ws[i] + v * ks[i];
+    }
+    *reinterpret_cast<f32x4*>(red + g * D + c) = o;
+  }
+  __syncthreads();
+  float o = 0.f, ss = 0.f;
+  if (tid < D) {
+    for (int i = 0; i < G; ++i) o += red[i * D + tid];
+    o += ruk * vs[tid];
+    ss = o * o;
+  }
+#pragma unroll
+  for (int q = 32; q > 0; q >>= 1) ss += __shfl_xor(ss, q, 64);
+  if ((tid & 63) == 0) part[4 + (tid >> 6)] = ss;
+  __syncthreads();
+  ss = part[4] + part[5] + part[6] + part[7];
+  if (tid < D) {
+    const float inv = 1.f / sqrtf(ss / (float)D + eps);
+    out[(size_t)t * ldout + hb + tid] = (T)(o * inv * norm[hb + tid] * (float)gate[(size_t)t * ldg + hb + tid]);
+  }
+  for (int i = blockIdx.x * 256 + tid; i < p.width; i += gridDim.x * 256)
+    p.prev[(size_t)slot * p.ldp + i] = p.x[(size_t)t * p.ldx + i];
 }
 
 // ---- out = (o / rms(o) per head) * norm * gate
@@ -210,8 +287,9 @@ int nls_shift_mix(const float* x, long ldx, const float* mu, const float* prev, 
                   long mstride, const int* runs, const int* tok_seq, int D, int T, int f32, void* stream) {
   if (T < 1 || D < 1) return -1;
   Mix p{x, mu, prev, out, runs, tok_seq, ldx, ldp, ldo, mstride, D, f32};
-  if (f32) hipLaunchKernelGGL(shift_mix_kernel<float>, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
-  else hipLaunchKernelGGL(shift_mix_kernel<__bf16>, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
+  const dim3 grid(T, T >= 256 ? 1 : min((D + 255) / 256, 16));
+  if (f32) hipLaunchKernelGGL(shift_mix_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, p);
+  else hipLaunchKernelGGL(shift_mix_kernel<__bf16>, grid, dim3(256), 0, (hipStream_t)stream, p);
   return (int)hipGetLastError();
 }
 
@@ -221,6 +299,23 @@ int nls_wkv_scan(const void* r, const void* k, const void* v, long ld, const flo
   if (nruns < 1 || H < 1 || D < 1) return -1;
   Scan p{r, k, v, w, u, o, state, x, prev, runs, ld, ldw, ldo, sstride, ldx, ldp, H, D, width};
   return f32 ? scan_t<float>(p, nruns, (hipStream_t)stream) : scan_t<__bf16>(p, nruns, (hipStream_t)stream);
+}
+
+// every run has one token (or none); D a multiple of 4
+int nls_wkv_step(const void* r, const void* k, const void* v, long ld, const float* w, long ldw, const float* u,
+                 float* state, long sstride, const float* x, long ldx, float* prev, long ldp, int width, const int* runs,
+                 int nruns, const float* norm, const void* gate, long ldg, void* out, long ldout, int H, int D, float eps,
+                 int f32, void* stream) {
+  if (nruns < 1 || H < 1 || D < 4 || D > 256 || (D & 3) || (sstride & 3)) return -1;
+  Scan p{r, k, v, w, u, nullptr, state, x, prev, runs, ld, ldw, 0, sstride, ldx, ldp, H, D, width};
+  const dim3 grid(H, nruns);
+  if (f32)
+    hipLaunchKernelGGL(wkv_step_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, p, norm, (const float*)gate, ldg,
+                       (float*)out, ldout, eps);
+  else
+    hipLaunchKernelGGL(wkv_step_kernel<__bf16>, grid, dim3(256), 0, (hipStream_t)stream, p, norm, (const __bf16*)gate, ldg,
+                       (__bf16*)out, ldout, eps);
+  return (int)hipGetLastError();
 }
 
 int nls_wkv_out(const float* o, long ldo, const float* norm, const void* gate, long ldg, void* out, long ld, int H,

@@ -829,10 +829,11 @@ class Engine:
         if not hasattr(self, "_pf_pin"):
             cuda = self.dev.type == "cuda"
             nq = (self.max_prefill + 15) // 16 + self.max_batch
+            bw = getattr(self.model, "block_width", 4)
             self._pf_pin = [(torch.zeros(self.max_logit_rows, dtype=torch.int32, pin_memory=cuda),
-                             torch.zeros(nq, 4, dtype=torch.int32, pin_memory=cuda)) for _ in range(2)]
+                             torch.zeros(nq, bw, dtype=torch.int32, pin_memory=cuda)) for _ in range(2)]
             self._pf_dev = (torch.zeros(self.max_logit_rows, dtype=torch.int32, device=self.dev),
-                            torch.zeros(nq, 4, dtype=torch.int32, device=self.dev))
+                            torch.zeros(nq, bw, dtype=torch.int32, device=self.dev))
 
     def _pf_graph_key(self, T: int, rows: List[int], qb, need_logits: bool):
         """The prefill graph of this chunk, if any: single GPU, one contiguous run of <= 64 tokens of one
@@ -864,7 +865,13 @@ class Engine:
         cuda = self.dev.type == "cuda"
         pad = b.pad
         h = self.h_meta_p.numpy()
-        qb = ops.prefill_blocks(h[3 * pad:4 * pad], h[pad:2 * pad], T) if self.prefill_attn else None
+        info = {}
+        if hasattr(self.model, "row_blocks"):
+            qb, ri = self.model.row_blocks(h[3 * pad:4 * pad], h[pad:2 * pad], T) if self.prefill_attn else (None, None)
+            if ri is not None:
+                info = {"row_info": ri}
+        else:
+            qb = ops.prefill_blocks(h[3 * pad:4 * pad], h[pad:2 * pad], T) if self.prefill_attn else None
         key = self._pf_graph_key(T, rows, qb, need_logits)
         if key is not None:
             # rows T .. Tb-1 of the token bucket: no KV writes (slot -1), position 0 (the RoPE table), no attention
@@ -904,7 +911,7 @@ class Engine:
         else:
             n = self.model.forward(b, self.kc, self.vc, T, self.bs, self.model.n_splits(T),
                                    logit_rows=lr, n_logits=len(rows), qblocks=qbt, nqb=0 if qbt is None else len(qb),
-                                   need_logits=need_logits, **self._state_args(nruns))
+                                   need_logits=need_logits, **info, **self._state_args(nruns))
         self._gather(b, n, need_logits)
 
     def _state_args(self, nruns: int) -> dict:

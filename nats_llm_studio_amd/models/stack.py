@@ -16,10 +16,11 @@ import os
 from dataclasses import dataclass, field
 from typing import Dict, List, Optional
 
+import numpy as np
 import torch
 
 from ..ops import stack as K
-from ..ops import prefill_blocks, rope_table
+from ..ops import rope_table
 from ..safetensors_io import SafetensorsReader
 from .llama import ShardSpec
 from .stack_config import StackConfig
@@ -125,6 +126,11 @@ class WkvMixer(_Part):
         K.shift_mix(b.x, self.mu, prev, e["mix"], b.runs, b.tok_seq, T, st)
         e["proj"].run(T, st)
         e["decay"].run(T, st)
+        if T == step.nruns and c.dim % 4 == 0:          # single tokens only
+            K.wkv_step(e["r"], e["k"], e["v"], e["w"], self.u, S, b.x, prev, b.runs, T, self.norm, e["g"], e["out"], c.heads,
+                       c.dim, self.m.cfg.eps, st)
+            e["o_proj"].run(T, st)
+            return
         K.wkv_scan(e["r"], e["k"], e["v"], e["w"], self.u, e["o"], S, b.x, prev, b.runs, step.nruns, c.heads, c.dim, st)
         K.wkv_out(e["o"], self.norm, e["g"], e["out"], c.heads, c.dim, T, self.m.cfg.eps, st)
         e["o_proj"].run(T, st)
@@ -133,7 +139,8 @@ class WkvMixer(_Part):
 class LatentMixer(_Part):
     """Latent attention. The cache holds, per token, the normed latent and one rotated key part shared by all heads; a
     layer with kv_from reads an earlier layer's rows. The key up-projection is folded into the query and the value
-    up-projection applied to the attended latent, so every head attends over the same cached rows."""
+    up-projection applied to the attended latent, so every head attends over the same cached rows. Long runs (prompt
+    chunks) instead expand their context's keys and values once and attend per head (`plan` of the step)."""
 
     def __init__(self, model, i, cfg, prefix):
         super().__init__(model, i, cfg, prefix)
@@ -151,6 +158,13 @@ class LatentMixer(_Part):
         zero = uq.new_zeros
         self.uqn = self.lin(torch.cat([uq[:, :D], zero(H, self.Dq - D, Q)], 1).reshape(H * self.Dq, Q))
         self.uqr = self.lin(torch.cat([uq[:, D:], zero(H, self.RD4 - RD, Q)], 1).reshape(H * self.RD4, Q))
+        # expanded form: per-head keys / values of prompt contexts
+        self.xk, self.xr, self.xv = (K.expand_width(*a) for a in (("key", D), ("rot", RD), ("value", VD)))
+        self.expand = not model.f32 and None not in (self.xk, self.xr, self.xv)
+        if self.expand:
+            uk, uv = self.t("uk").to(model.device).view(H, D, R), self.t("uv").to(model.device).view(H, VD, R)
+            self.xuk = self.lin(torch.cat([uk, zero(H, self.xk - D, R)], 1).reshape(H * self.xk, R))
+            self.xuv = self.lin(torch.cat([uv, zero(H, self.xv - VD, R)], 1).reshape(H * self.xv, R))
         self.uk = self.lin(self.t("uk").to(model.device).view(H, D, R).transpose(1, 2).contiguous())   # [H][R][D]
         self.uv = self.lin(self.t("uv").to(model.device).view(H, VD, R))                               # [H][VD][R]
         self.g, self.o = self.lin("g", (H, d)), self.lin("o", (d, H * VD))
@@ -180,7 +194,7 @@ class LatentMixer(_Part):
         if self.owner:
             down.append(K.Seg(self.dkv, b.act, dkv))
         return dict(
-            dq=dq, dkv=dkv, cq=cq, q=q, lat=lat, part=(po, pm), hb=hb,
+            dq=dq, dkv=dkv, cq=cq, q=q, qn=qn, gate=gate, ao=ao, lat=lat, part=(po, pm), hb=hb,
             down=K.LinLaunch(down),
             up=K.LinLaunch([K.Seg(self.uqn, cq, qn),
                             K.Seg(self.uqr, cq, q, "rope", ycol=self.Rp, block=(self.RD4, self.Dp),
@@ -196,12 +210,31 @@ class LatentMixer(_Part):
         K.latent_rows(e["dq"], self.dqn, e["cq"], e["dkv"], self.dkvn if self.owner else None, c.kv_rank, self.Rp,
                       c.rot_dim, self.cs, b.pos, b.slot, rows if self.owner else None, T, self.m.cfg.eps, st)
         e["up"].run(T, st)
-        e["absorb"].run(T, st)
-        ns = 1 if self.m.f32 else max(1, min(_SPLIT_CAP, _SPLIT_WG // (T * e["hb"])))
-        K.latent_attention(e["q"], rows, e["lat"], e["part"], b.block_tables, step.block_size, b.tok_seq, b.ctx_len, T,
-                           c.heads, ns, self.Rp, self.rp, c.scale, st)
-        e["value"].run(T, st)
+        plan = step.plan
+        if plan is None or plan.rest:
+            # latent-space attention of the rows outside the expanded runs (the others have no keys here)
+            e["absorb"].run(T, st)
+            ns = 1 if self.m.f32 else max(1, min(_SPLIT_CAP, _SPLIT_WG // (T * e["hb"])))
+            K.latent_attention(e["q"], rows, e["lat"], e["part"], b.block_tables, step.block_size, b.tok_seq,
+                               b.ctx_len if plan is None else plan.actx, T, c.heads, ns, self.Rp, self.rp, c.scale, st)
+            e["value"].run(T, st)
+        if plan is not None:
+            kx, vx, lin = self._expansion(b, e, rows, plan)
+            lin.run(plan.nx, st)
+            K.latent_prefill(e["qn"], self.Dq, e["q"], self.Rp, self.Dp, kx, vx, rows, plan.xmap, plan.blocks, plan.nblocks,
+                             plan.waves, e["gate"], e["ao"], c.heads, self.xk, self.xr, self.xv, c.vdim, c.scale, st)
         e["o_proj"].run(T, st)
+
+    def _expansion(self, b: StackBuffers, e: dict, rows, plan):
+        """Scratch for the expanded keys / values (shared by the layers, grown on demand) and the launch that fills it."""
+        H = self.cfg.heads
+        kx = self.m.grown(b, "lat.kx", plan.nx, H * self.xk)
+        vx = self.m.grown(b, "lat.vx", plan.nx, H * self.xv)
+        key = (kx.data_ptr(), vx.data_ptr(), rows.data_ptr(), plan.xmap.data_ptr())
+        if e.get("expand_key") != key:
+            e["expand_key"] = key
+            e["expand"] = K.LinLaunch([K.Seg(self.xuk, rows, kx, xmap=plan.xmap), K.Seg(self.xuv, rows, vx, xmap=plan.xmap)])
+        return kx, vx, e["expand"]
 
 
 class MoeFeedForward(_Part):
@@ -251,11 +284,30 @@ FEED_FORWARDS = {"moe": MoeFeedForward}
 
 
 @dataclass
+class _ExpandPlan:
+    """The runs of a step whose attention expands keys and values: `nx` context rows, query blocks of 32 * waves rows."""
+    nx: int
+    xmap: torch.Tensor          # [nx] cache slots of the runs' contexts
+    blocks: torch.Tensor        # [nblocks][8]
+    nblocks: int
+    waves: int
+    rest: bool                  # some rows attend in the latent space
+    actx: Optional[torch.Tensor]
+
+
+@dataclass
 class _Step:
     T: int
     nruns: int
     block_size: int
     st: int
+    plan: Optional[_ExpandPlan] = None
+
+
+# runs of at least this many rows expand (below, the latent-space attention's extra products cost less than the expansion
+# of the context), as long as their contexts fit the scratch
+_EXPAND_RUN = int(os.environ.get("NLS_EXPAND_RUN", "32"))
+_EXPAND_BYTES = int(os.environ.get("NLS_EXPAND_BYTES", str(4 << 30)))
 
 
 class StackModel:
@@ -358,18 +410,69 @@ class StackModel:
         b.launches["head"] = K.LinLaunch([K.Seg(self.head, b.hn, b.logits)])
         return b
 
+    # ---- prompt attention: which runs expand their context
+    block_width = K.BLOCK_INTS
+
+    def row_blocks(self, tok_seq, pos, T: int):
+        """Host side of a row batch's expansion plan, from its staged metadata: (int32 [spans + blocks][8], info), or
+        (None, None) when every row attends in the latent space. Rows of the table: spans (first row, rows, sequence, first
+        position, first expanded row, context, 0, 0), then query blocks (the same, per 32 * waves rows), longest context
+        first."""
+        lat = [m for m, *_ in self.layers if isinstance(m, LatentMixer)]
+        if not lat or not all(m.expand for m in lat):
+            return None, None
+        ts, ps = np.asarray(tok_seq[:T]), np.asarray(pos[:T])
+        cut = np.flatnonzero(ts[1:] != ts[:-1]) + 1
+        width = max(m.cfg.heads * (m.xk + m.xv) for m in lat) * 2
+        spans, nx, rows = [], 0, 0
+        for a, e in zip(np.concatenate([[0], cut]), np.concatenate([cut, [T]])):
+            n, p0 = int(e - a), int(ps[a])
+            if n < _EXPAND_RUN or (nx + p0 + n) * width > _EXPAND_BYTES:
+                continue
+            spans.append((int(a), n, int(ts[a]), p0, nx, p0 + n, 0, 0))
+            nx += p0 + n
+            rows += n
+        if not spans:
+            return None, None
+        H = max(m.cfg.heads for m in lat)
+        waves = 8 if H * sum(-(-s[1] // 256) for s in spans) >= 256 else 4
+        q = 32 * waves
+        blocks = [(s[0] + o, min(q, s[1] - o), s[2], s[3] + o, s[4], 0, 0, 0) for s in spans for o in range(0, s[1], q)]
+        blocks.sort(key=lambda v: -(v[3] + v[1]))
+        info = dict(nspans=len(spans), nblocks=len(blocks), nx=nx, maxctx=max(s[5] for s in spans), waves=waves,
+                    rest=rows < T)
+        return np.asarray(spans + blocks, dtype=np.int32), info
+
     def attention_blocks(self, b: StackBuffers, T: int) -> dict:
-        """The forward arguments that describe a row batch's attention blocks, from its staged metadata (the engine builds
-        them on the host: ops.prefill_blocks)."""
-        qb = prefill_blocks(b.tok_seq[:T].cpu().numpy(), b.pos[:T].cpu().numpy(), T)
-        return dict(qblocks=torch.from_numpy(qb).to(self.device), nqb=len(qb))
+        """row_blocks as forward arguments, from a row batch already staged on the device."""
+        qb, info = self.row_blocks(b.tok_seq[:T].cpu().numpy(), b.pos[:T].cpu().numpy(), T)
+        return {} if qb is None else dict(qblocks=torch.from_numpy(qb).to(self.device), nqb=len(qb), row_info=info)
+
+    def grown(self, b: StackBuffers, name: str, rows: int, cols: int, dtype=None) -> torch.Tensor:
+        """A [>= rows, cols] scratch that grows (eager row batches only: captured graphs never use it)."""
+        key = ("grown", name, cols)
+        t = b.shared.get(key)
+        if t is None or t.shape[0] < rows:
+            b.shared[key] = None
+            t = b.shared[key] = torch.zeros(K.pad_to(rows, 1024), cols, dtype=dtype or self.dtype, device=self.device)
+        return t
+
+    def _expand_plan(self, b: StackBuffers, qblocks, info: dict, T: int, block_size: int, st: int) -> _ExpandPlan:
+        ns = info["nspans"]
+        xmap = self.grown(b, "lat.xmap", info["nx"], 1, torch.int32).view(-1)
+        actx = None
+        if info["rest"]:
+            actx = self.grown(b, "lat.actx", b.pad, 1, torch.int32).view(-1)
+            actx[:T].copy_(b.ctx_len[:T])
+        K.expand_plan(qblocks, ns, info["maxctx"], b.block_tables, block_size, xmap, actx, st)
+        return _ExpandPlan(info["nx"], xmap, qblocks[ns:], info["nblocks"], info["waves"], info["rest"], actx)
 
     # ---- forward
     @torch.no_grad()
     def forward(self, b: StackBuffers, kc, vc, T: int, block_size: int, n_split: int = 1,
                 logit_rows: Optional[torch.Tensor] = None, n_logits: Optional[int] = None, qblocks=None, nqb: int = 0,
                 feed_prev: bool = False, need_logits: bool = True, state=None, nruns: Optional[int] = None,
-                taps: Optional[list] = None):
+                row_info: Optional[dict] = None, taps: Optional[list] = None):
         """One step of T rows: logits (of `logit_rows`, or of every row) in b.logits[:n], their greedy ids in
         b.next_ids[:n]. `taps` (a list) receives the residual after every layer."""
         if T < 1 or T > b.pad:
@@ -377,6 +480,8 @@ class StackModel:
         cfg = self.cfg
         st = K.stream(self.device)
         step = _Step(T, T if nruns is None else nruns, block_size, st)
+        if row_info is not None and qblocks is not None:
+            step.plan = self._expand_plan(b, qblocks, row_info, T, block_size, st)
         K.embed(b.ids, self.embed, b.x, b.xb, T, st, prev=(b.next_ids, b.use_prev) if feed_prev else None)
         last = len(self.layers) - 1
         direct = logit_rows is None

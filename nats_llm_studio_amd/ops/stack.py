@@ -45,6 +45,9 @@ _SIGS = {
     "nls_shift_mix": [P, L, P, P, L, P, L, L, P, P, I, I, I, P],
     "nls_wkv_scan": [P, P, P, L, P, L, P, P, L, P, L, P, L, P, L, I, P, I, I, I, I, P],
     "nls_wkv_out": [P, L, P, P, L, P, L, I, I, I, F, I, P],
+    "nls_wkv_step": [P, P, P, L, P, L, P, P, L, P, L, P, L, I, P, I, P, P, L, P, L, I, I, F, I, P],
+    "nls_expand_plan": [P, I, I, P, I, I, P, P, P],
+    "nls_latent_prefill": [P, L, I, P, L, I, P, P, P, L, P, P, I, P, I, P, L, I, I, I, I, I, I, F, P],
     "nls_latent_attn": [P, P, P, P, P, P, I, I, P, P, I, I, I, I, I, F, I, P],
 }
 
@@ -127,7 +130,7 @@ class Seg:
 
     def __init__(self, w: PackedLinear, x: torch.Tensor, y: torch.Tensor, epi: str = "none", ycol: int = 0,
                  xcol: int = 0, xgs: int = 0, ygs: int = 0, block=None, bias=None, gate=None, routed=None, rope=None,
-                 yrow: int = 0):
+                 yrow: int = 0, xmap: Optional[torch.Tensor] = None):
         if x.stride(1) != 1 or y.stride(1) != 1:
             raise ValueError("row-major operands")
         if xcol + (0 if routed else (w.groups - 1) * xgs) + act_ld(w.K) > x.stride(0):
@@ -138,6 +141,8 @@ class Seg:
             raise ValueError("activation rows must be 16-byte aligned")
         self.w, self.y, self.x = w, y, x
         self.rows_cap = min(x.shape[0] * (routed[1] if routed else 1), y.shape[0] - yrow)
+        if xmap is not None:               # x row of row m: xmap[m] (the caller keeps the entries inside x)
+            self.rows_cap = min(xmap.numel(), y.shape[0] - yrow)
         s = self.s = LinSeg()
         s.w = w.data.data_ptr()
         s.x = x.data_ptr() + xcol * x.element_size()
@@ -153,7 +158,8 @@ class Seg:
             s.rows, s.xdiv = routed[0].data_ptr(), routed[1]
         if rope:
             s.cs, s.pos, s.half = rope[0].data_ptr(), rope[1].data_ptr(), rope[2]
-        self.keep = (bias, gate, routed, rope)
+        s.xmap = _p(xmap)
+        self.keep = (bias, gate, routed, rope, xmap)
 
 
 GEMM_TILES = ((64, 64), (128, 64), (128, 128), (256, 128), (256, 256))     # (weight rows, rows) of lin_gemm's cfg
@@ -194,6 +200,8 @@ class LinLaunch:
             ns = max(s.w.nsub for s in self.segs)
             nw = 4 if n >= 1536 or ns <= 16 else (8 if n >= 512 or mt > 1 or ns <= 64 else 16)
             return False, mt, nw
+        if bm is None and self._tiles(64, 64, M) < 96 and self._tiles(16, 16, M) <= 1024:
+            return False, 1, 16           # few outputs (routers): split K over a workgroup's waves instead
         for c in (4, 3, 2, 1, 0):
             bn, b = GEMM_TILES[c]
             if bm is not None and b != bm:
@@ -321,6 +329,30 @@ def latent_attention(q, cache, out, part, block_tables, block_size: int, tok_seq
                                  Rp, rp, scale, int(q.dtype == torch.float32), st), "nls_latent_attn")
 
 
+BLOCK_INTS = 8           # int32 words per span / query block of the row plan (StackModel.row_blocks)
+EXPAND_UNITS = {"key": (32, 64, 128), "rot": (32, 64), "value": (32, 64, 128)}      # per-head widths of latent_prefill
+
+
+def expand_width(kind: str, n: int) -> Optional[int]:
+    return next((w for w in EXPAND_UNITS[kind] if n <= w), None)
+
+
+def expand_plan(spans, nspans: int, maxctx: int, block_tables, block_size: int, xmap, actx, st: int):
+    """xmap: cache slots of the spans' contexts; actx (optional): key counts of the rows, cleared inside the spans."""
+    _check(lib().nls_expand_plan(spans.data_ptr(), nspans, maxctx, block_tables.data_ptr(), block_tables.stride(0),
+                                 block_size, xmap.data_ptr(), _p(actx), st), "nls_expand_plan")
+
+
+def latent_prefill(qn, qns: int, q, Rp: int, qrs: int, kx, vx, cache, xmap, blocks, nblocks: int, waves: int, gate, out,
+                   H: int, dku: int, dr: int, dv: int, vdim: int, scale: float, st: int):
+    """Causal attention of query blocks over expanded keys / values; the rotated parts sit at column Rp of q and cache."""
+    _check(lib().nls_latent_prefill(qn.data_ptr(), qn.stride(0), qns, q.data_ptr() + Rp * q.element_size(), q.stride(0), qrs,
+                                    kx.data_ptr(), vx.data_ptr(), cache.data_ptr() + Rp * cache.element_size(),
+                                    cache.stride(0), xmap.data_ptr(), blocks.data_ptr(), nblocks, gate.data_ptr(),
+                                    gate.stride(0), out.data_ptr(), out.stride(0), H, dku, dr, dv, vdim, waves, scale, st),
+           "nls_latent_prefill")
+
+
 def shift_mix(x, mu, prev, out: torch.Tensor, runs, tok_seq, T: int, st: int):
     """out [mixes, rows, ld]: x + (previous token's x - x) * mu[s]; `prev` [slots, D] precedes each run's first row."""
     _check(lib().nls_shift_mix(x.data_ptr(), x.stride(0), mu.data_ptr(), prev.data_ptr(), prev.stride(0), out.data_ptr(),
@@ -334,6 +366,15 @@ def wkv_scan(r, k, v, w, u, o, state, x, prev, runs, nruns: int, H: int, D: int,
                               u.data_ptr(), o.data_ptr(), o.stride(0), state.data_ptr(), state.stride(0), x.data_ptr(),
                               x.stride(0), prev.data_ptr(), prev.stride(0), prev.shape[1], runs.data_ptr(), nruns, H, D,
                               int(r.dtype == torch.float32), st), "nls_wkv_scan")
+
+
+def wkv_step(r, k, v, w, u, state, x, prev, runs, nruns: int, norm, gate, out, H: int, D: int, eps: float, st: int):
+    """wkv_scan and wkv_out of runs of one token each."""
+    _check(lib().nls_wkv_step(r.data_ptr(), k.data_ptr(), v.data_ptr(), r.stride(0), w.data_ptr(), w.stride(0), u.data_ptr(),
+                              state.data_ptr(), state.stride(0), x.data_ptr(), x.stride(0), prev.data_ptr(),
+                              prev.stride(0), prev.shape[1], runs.data_ptr(), nruns, norm.data_ptr(), gate.data_ptr(),
+                              gate.stride(0), out.data_ptr(), out.stride(0), H, D, eps, int(out.dtype == torch.float32),
+                              st), "nls_wkv_step")
 
 
 def wkv_out(o, norm, gate, out, H: int, D: int, T: int, eps: float, st: int):
