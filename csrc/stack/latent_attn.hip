@@ -4,7 +4,8 @@
 //
 // latent_attn_kernel (bf16): workgroup = (token, split of the keys, NHB blocks of 16 heads), 4 waves per head block.
 // KT-key tiles of the cache rows arrive by LDS-DMA into two buffers (16-byte chunks swizzled by the key on the DMA
-// source), once for all head blocks; each wave forms S^T of 16 keys (A = cache rows, B = its block's queries, held in
+// source), once for all head blocks; a 32-key half is refilled as soon as it is consumed, so loads of the next two tiles
+// stay in flight. Each wave forms S^T of 16 keys (A = cache rows, B = its block's queries, held in
 // registers), the four waves of a block exchange row maxima and the bf16 weights through LDS, and each owns a quarter of
 // the output columns: O^T += C^T P^T with C^T fragments from transposed LDS reads of the same tile. Softmax in base 2, all
 // of it f32.
@@ -37,18 +38,37 @@ DEVI void bar_lgkm() {
   asm volatile("" ::: "memory");
 }
 
-constexpr int NBT = 1024;    // block-table entries of the split kept in LDS
+// chunk permutation of a cache row in LDS: 16 consecutive rows of one chunk land on distinct banks (a row is an odd or even
+// multiple of 128 bytes)
+template <int Dp>
+DEVI int row_swz(int row) {
+  return (Dp / 64) & 1 ? (row >> 1) & 7 : row & 15;
+}
+
+constexpr int NBT = 1024;    // block-table entries of one split, kept in LDS
+
+template <int N>
+DEVI void wait_vm() {
+  asm volatile("s_waitcnt vmcnt(%0)" ::"i"(N) : "memory");
+}
+// everything but one tile's own DMA instructions of this wave has landed
+template <int ND, int NH, int NHB>
+DEVI void wait_tile(int hsub) {
+  if (NHB == 1) wait_vm<ND * NH>();
+  else if (hsub < NH) wait_vm<ND>();
+  else wait_vm<0>();
+}
 
 template <int NT, int RT, int KT, int NHB>
 __global__ __launch_bounds__(256 * NHB, 1) void latent_attn_kernel(LA p) {
   constexpr int Rp = 64 * NT, Dp = Rp + 64 * RT;
   constexpr int CPR = Dp / 8;                  // 16-byte chunks per row
   constexpr int TB = KT * Dp * 2;              // bytes per tile
-  constexpr int NDT = TB / 1024;               // DMA instructions per tile
-  constexpr int ND = (NDT + 4 * NHB - 1) / (4 * NHB);   // ... per wave (the last ones may be idle)
+  constexpr int NH = KT / 32;                  // 32-key halves per tile
+  constexpr int ND = Dp / 64;                  // DMA instructions per half and issuing wave (four waves issue a half)
   constexpr int NK = Dp / 32;                  // k-steps of a score
   constexpr int PS = KT + 8;                   // P row stride
-  static_assert(TB % 1024 == 0, "tile");
+  constexpr int PR = (Dp / 64) & 1 ? 8 : 16;   // chunks a row's permutation ranges over
   extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
   const int wv = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int wave = wv & 3, hsub = wv >> 2;     // wave of its head block; head block of the workgroup
@@ -76,94 +96,126 @@ __global__ __launch_bounds__(256 * NHB, 1) void latent_attn_kernel(LA p) {
   float m = -INFINITY, l = 0.f;
 
   if (k0 < k1) {
-    const int b0 = k0 >> p.bshift, nb = ((k1 - 1) >> p.bshift) - b0 + 1, bmask = p.bs - 1;
-    for (int i = threadIdx.x; i < min(nb, NBT); i += 256 * NHB) btl[i] = bt[b0 + i];
     u32x4 qf[NK];
     const __bf16* qr = reinterpret_cast<const __bf16*>(p.q) + ((size_t)t * p.H + min(head, p.H - 1)) * Dp;
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) qf[kk] = ld16(qr + kk * 32 + 8 * g);
-    __syncthreads();
     const float sl2 = p.scale * 1.4426950408889634f;
     const uint32_t base = __builtin_amdgcn_readfirstlane(lds_addr(lds));
-    auto dma = [&](int j) __attribute__((always_inline)) {
-      const uint32_t dst = base + (uint32_t)(j & 1) * TB + (uint32_t)(ND * wv) * 1024u;
+    const int bmask = p.bs - 1;
+    // keys [w0, w1) per pass: as many as the block-table window in LDS holds
+    for (int w0 = k0; w0 < k1; w0 += NBT << p.bshift) {
+      const int w1 = min(k1, w0 + (NBT << p.bshift));
+      const int b0 = w0 >> p.bshift, nb = ((w1 - 1) >> p.bshift) - b0 + 1;
+      __syncthreads();
+      for (int i = threadIdx.x; i < min(nb, NBT); i += 256 * NHB) btl[i] = bt[b0 + i];
+      __syncthreads();
+      // half u (32 keys) of tile j -> its place in buffer j & 1; issued by the four waves of head block u % NHB
+      auto dma = [&](int j, int u) __attribute__((always_inline)) {
+        if (NHB > 1 && hsub != u % NHB) return;
+        const uint32_t dst = base + (uint32_t)(j & 1) * TB + (uint32_t)u * (32 * Dp * 2) + (uint32_t)(ND * wave) * 1024u;
+        // every source address first (their block lookups overlap), then the copies
+        const __bf16* src[ND];
 #pragma unroll
-      for (int i = 0; i < ND; ++i) {
-        if (NDT % (4 * NHB) != 0 && ND * wv + i >= NDT) break;
-        const int ci = (ND * wv + i) * 64 + lane;
-        const int row = ci / CPR, pc = ci - row * CPR;
-        const int key = min(k0 + j * KT + row, k1 - 1);
-        const int bi = (key >> p.bshift) - b0;
-        const int blk = bi < NBT ? btl[bi] : bt[b0 + bi];
-        glds16(cache + (((size_t)blk << p.bshift) + (key & bmask)) * Dp + (pc ^ (row & 7)) * 8, dst + i * 1024);
-      }
-    };
-    const int nt = (k1 - k0 + KT - 1) / KT;
-    dma(0);
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    bar_lgkm();
-    for (int j = 0; j < nt; ++j) {
-      const uint8_t* cb = lds + (j & 1) * TB;
-      if (j + 1 < nt) dma(j + 1);              // that buffer was last read in tile j - 1
-      f32x4 s = f32x4{-INFINITY, -INFINITY, -INFINITY, -INFINITY};
-      float tm = -INFINITY;
-      if (KT == 64 || wave < KT / 16) {
-        f32x4 s2[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};     // two chains of dependent products
-        const int row = 16 * wave + r;
-#pragma unroll
-        for (int kk = 0; kk < NK; ++kk) {
-          const bf16x8 a = *reinterpret_cast<const bf16x8*>(cb + row * (2 * Dp) + (((4 * kk + g) ^ (row & 7)) << 4));
-          s2[kk & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, __builtin_bit_cast(bf16x8, qf[kk]), s2[kk & 1], 0, 0, 0);
+        for (int i = 0; i < ND; ++i) {
+          const int ci = (ND * wave + i) * 64 + lane;
+          const int row = ci / CPR, pc = ci - row * CPR;
+          const int key = min(w0 + j * KT + 32 * u + row, w1 - 1);
+          src[i] = cache + (uint32_t)((pc ^ row_swz<Dp>(row)) * 8) +
+                   (((size_t)btl[min((key >> p.bshift) - b0, NBT - 1)] << p.bshift) + (key & bmask)) * Dp;
         }
-        s = s2[0] + s2[1];
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          s[i] = k0 + j * KT + 16 * wave + 4 * g + i < k1 ? s[i] * sl2 : -INFINITY;
-          tm = fmaxf(tm, s[i]);
-        }
-        tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
-        tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
+        for (int i = 0; i < ND; ++i) glds16(src[i], dst + i * 1024);
+      };
+      const int nt = (w1 - w0 + KT - 1) / KT;
+#pragma unroll
+      for (int u = 0; u < NH; ++u) dma(0, u);
+      if (nt > 1) {
+#pragma unroll
+        for (int u = 0; u < NH; ++u) dma(1, u);
+        wait_tile<ND, NH, NHB>(hsub);
+      } else {
+        wait_vm<0>();
       }
-      if (g == 0) mx[wave * 16 + r] = tm;
       bar_lgkm();
-      const float mn = fmaxf(fmaxf(fmaxf(mx[r], mx[16 + r]), fmaxf(mx[32 + r], mx[48 + r])), m);
-      const float alpha = m == -INFINITY ? 0.f : exp2f(m - mn);
-      if (KT == 64 || wave < KT / 16) {
-        typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
-        bf4 pb;
-        float ps = 0.f;
+      for (int j = 0; j < nt; ++j) {
+        const uint8_t* cb = lds + (j & 1) * TB;
+        f32x4 s = f32x4{-INFINITY, -INFINITY, -INFINITY, -INFINITY};
+        float tm = -INFINITY;
+        if (KT == 64 || wave < KT / 16) {
+          f32x4 s2[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};     // two chains of dependent products
+          const uint8_t* kr = cb + (16 * wave + r) * (2 * Dp);
+          const int sw = row_swz<Dp>(r);                                            // (16 rows: one period)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const float e = s[i] == -INFINITY ? 0.f : exp2f(s[i] - mn);
-          ps += e;
-          pb[i] = (__bf16)e;
+          for (int kk = 0; kk < NK; ++kk) {
+            const int hi = 4 * kk & ~(PR - 1);
+            const bf16x8 a = *reinterpret_cast<const bf16x8*>(kr + (hi << 4) + (((((4 * kk) & (PR - 1)) + g) ^ sw) << 4));
+            s2[kk & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, __builtin_bit_cast(bf16x8, qf[kk]), s2[kk & 1], 0, 0, 0);
+          }
+          s = s2[0] + s2[1];
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            s[i] = w0 + j * KT + 16 * wave + 4 * g + i < w1 ? s[i] * sl2 : -INFINITY;
+            tm = fmaxf(tm, s[i]);
+          }
+          tm = fmaxf(tm, __shfl_xor(tm, 16, 64));
+          tm = fmaxf(tm, __shfl_xor(tm, 32, 64));
         }
-        l = l * alpha + ps;                    // this lane's keys; lanes and waves are summed at the end
-        *reinterpret_cast<bf4*>(P + r * PS + 16 * wave + 4 * g) = pb;
-      }
-      m = mn;
-      bar_lgkm();
-      const int qq = r >> 2, pp = r & 3;
+        if (g == 0) mx[wave * 16 + r] = tm;
+        bar_lgkm();
+        const float mn = fmaxf(fmaxf(fmaxf(mx[r], mx[16 + r]), fmaxf(mx[32 + r], mx[48 + r])), m);
+        const float alpha = m == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(m - mn);
+        if (KT == 64 || wave < KT / 16) {
+          typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+          bf4 pb;
+          float ps = 0.f;
 #pragma unroll
-      for (int u = 0; u < KT / 32; ++u) {
-        const uint2 p0 = *reinterpret_cast<const uint2*>(P + r * PS + 32 * u + 4 * g);
-        const uint2 p1 = *reinterpret_cast<const uint2*>(P + r * PS + 32 * u + 16 + 4 * g);
-        const bf16x8 pf = __builtin_bit_cast(bf16x8, u32x4{p0.x, p0.y, p1.x, p1.y});
-        const int ra = 32 * u + 4 * g + qq, rb = ra + 16;
-#pragma unroll
-        for (int c = 0; c < NT; ++c) {
-          const int ch = 2 * (wave * NT + c) + (pp >> 1);
-          const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-              (__attribute__((address_space(3))) s16x4*)(cb + ra * (2 * Dp) + ((ch ^ (ra & 7)) << 4) + 8 * (pp & 1)));
-          const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-              (__attribute__((address_space(3))) s16x4*)(cb + rb * (2 * Dp) + ((ch ^ (rb & 7)) << 4) + 8 * (pp & 1)));
-          const s16x8 a8 = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
-          const f32x4 acc = u == 0 ? o[c] * alpha : o[c];
-          o[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a8), pf, acc, 0, 0, 0);
+          for (int i = 0; i < 4; ++i) {
+            const float e = s[i] == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(s[i] - mn);
+            ps += e;
+            pb[i] = (__bf16)e;
+          }
+          l = l * alpha + ps;                    // this lane's keys; lanes and waves are summed at the end
+          *reinterpret_cast<bf4*>(P + r * PS + 16 * wave + 4 * g) = pb;
         }
+        m = mn;
+        bar_lgkm();
+        const int qq = r >> 2, pp = r & 3;
+#pragma unroll
+        for (int u = 0; u < KT / 32; ++u) {
+          const uint2 p0 = *reinterpret_cast<const uint2*>(P + r * PS + 32 * u + 4 * g);
+          const uint2 p1 = *reinterpret_cast<const uint2*>(P + r * PS + 32 * u + 16 + 4 * g);
+          const bf16x8 pf = __builtin_bit_cast(bf16x8, u32x4{p0.x, p0.y, p1.x, p1.y});
+          const uint8_t* vr = cb + (4 * g + qq) * (2 * Dp) + 8 * (pp & 1);
+          const int sw = row_swz<Dp>(4 * g + qq);                                   // same for the rows 16, 32, .. below
+#pragma unroll
+          for (int c = 0; c < NT; ++c) {
+            int off;
+            if constexpr (2 * NT % PR == 0) {
+              const int hi = 2 * c & ~(PR - 1);
+              off = ((2 * wave * NT + hi) << 4) + (((((2 * c) & (PR - 1)) + (pp >> 1)) ^ sw) << 4);
+            } else {
+              off = ((2 * (wave * NT + c) + (pp >> 1)) ^ sw) << 4;
+            }
+            const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+                (__attribute__((address_space(3))) s16x4*)(vr + off + 32 * u * (2 * Dp)));
+            const s16x4 hi4 = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+                (__attribute__((address_space(3))) s16x4*)(vr + off + (32 * u + 16) * (2 * Dp)));
+            const s16x8 a8 = __builtin_shufflevector(lo, hi4, 0, 1, 2, 3, 4, 5, 6, 7);
+            const f32x4 acc = u == 0 ? o[c] * alpha : o[c];
+            o[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a8), pf, acc, 0, 0, 0);
+          }
+          // the half is free once every wave is done with it: refill it with tile j + 2's
+          if (u + 1 < NH) {
+            bar_lgkm();
+            if (j + 2 < nt) dma(j + 2, u);
+          }
+        }
+        if (j + 2 < nt && NH > 1 && (NHB == 1 || hsub == 0)) wait_vm<ND>();       // tile j + 1 landed, that refill in flight
+        else wait_vm<0>();
+        bar_lgkm();
+        if (j + 2 < nt) dma(j + 2, NH - 1);
       }
-      asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-      bar_lgkm();
     }
     l += __shfl_xor(l, 16, 64);
     l += __shfl_xor(l, 32, 64);

@@ -4,9 +4,9 @@
 //   o_t[j] = sum_i r_t[i] (S[i][j] + u[i] k_t[i] v_t[j]);   S[i][j] = w_t[i] S[i][j] + k_t[i] v_t[j]
 //
 // The scan is sequential in the tokens of a run, so a position's result does not depend on how its sequence was cut
-// into steps. Parallelism is (run, head, 32 value columns) x lanes: a wave owns 8 value columns, lane = 8 columns x 8 key
-// parts, each lane DP / 8 state values in registers; the key sum closes with three in-row lane exchanges (DPP). Tokens are
-// staged in LDS in chunks of CH as f32, the next chunk's loads in flight while the current one runs.
+// into steps. Parallelism is (run, head, value columns) x lanes: a lane holds DP / PARTS key rows of CPL value columns in
+// registers, PARTS neighbouring lanes cover the keys and close the sum with in-row lane exchanges (DPP). Few runs take
+// many key parts (short per-token chains on all CUs). Tokens are staged in LDS in chunks of CH as f32, the next chunk's loads in flight while the current one runs.
 // A step of single tokens (decode) streams each head's state once with 16-byte accesses and ends with the head's norm and
 // gate (wkv_step_kernel).
 //
@@ -48,13 +48,17 @@ __global__ __launch_bounds__(256) void shift_mix_kernel(Mix p) {
   }
 }
 
-// sum over the 8 lanes of a group (lane & 7)
 template <int C>
 DEVI float dpp_add(float v) {
   const int x = __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), C, 0xf, 0xf, true);
   return v + __builtin_bit_cast(float, x);
 }
-DEVI float sum8(float v) { return dpp_add<0x141>(dpp_add<0x4E>(dpp_add<0xB1>(v))); }   // quad swaps, then half-row mirror
+// sum over aligned groups of 8 or 16 lanes: quad swaps, half-row mirror, row mirror
+template <int PARTS>
+DEVI float sum_parts(float v) {
+  v = dpp_add<0x141>(dpp_add<0x4E>(dpp_add<0xB1>(v)));
+  return PARTS == 16 ? dpp_add<0x140>(v) : v;
+}
 
 struct Scan {
   const void *r, *k, *v;   // activation type, [rows][ld]
@@ -70,22 +74,23 @@ struct Scan {
 };
 
 // DP: key channels padded to a multiple of 32 (zeros past D)
-template <typename T, int DP>
+template <typename T, int DP, int PARTS, int CPL>
 __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
+  constexpr int WC = 256 / PARTS * CPL;          // value columns per workgroup
   constexpr int CH = DP <= 64 ? 32 : (DP <= 128 ? 16 : 8);   // tokens per staged chunk
-  constexpr int R = DP / 8;                      // state rows per lane
+  constexpr int R = DP / PARTS;                  // state rows per lane
   constexpr int LR = DP + 4;                     // LDS row stride
   constexpr int NV = (CH * DP + 255) / 256;      // staged values per thread and operand
   __shared__ __attribute__((aligned(16))) float rs[CH][LR], ks[CH][LR], ws[CH][LR];
-  __shared__ float vs[CH][32], ruk[CH];
+  __shared__ __attribute__((aligned(16))) float vs[CH][WC], ruk[CH];
   const int* run = p.runs + 4 * blockIdx.y;
   const int t0 = run[0], n = run[1], slot = run[2], pos0 = run[3];
   if (slot < 0 || n < 1) return;
   const int D = p.D;
-  const int ncb = (D + 31) / 32;
-  const int head = blockIdx.x / ncb, c0 = (blockIdx.x % ncb) * 32;
+  const int ncb = (D + WC - 1) / WC;
+  const int head = blockIdx.x / ncb, c0 = (blockIdx.x % ncb) * WC;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int part = lane & 7, col = wave * 8 + (lane >> 3);
+  const int part = lane & (PARTS - 1), col = (wave * (64 / PARTS) + lane / PARTS) * CPL;
   const int j = c0 + col;
   const size_t hb = (size_t)head * D;
   const T* rp = (const T*)p.r + hb;
@@ -94,13 +99,21 @@ __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
   const float* wp = p.w + hb;
   float* st = p.state + (size_t)slot * p.sstride + hb * D;
 
-  float S[R];
+  float S[CPL][R];
 #pragma unroll
-  for (int i = 0; i < R; ++i) {
-    const int row = part * R + i;
-    S[i] = (pos0 > 0 && row < D && j < D) ? st[(size_t)row * D + j] : 0.f;
+  for (int i = 0; i < R; ++i)
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) {
+      const int row = part * R + i;
+      S[c][i] = (pos0 > 0 && row < D && j + c < D) ? st[(size_t)row * D + j + c] : 0.f;
+    }
+  float ur[DP / 16];                             // u of the bonus sums' columns
+#pragma unroll
+  for (int q = 0; q < DP / 16; ++q) {
+    const int i = (threadIdx.x & 15) + 16 * q;
+    ur[q] = i < D ? p.u[hb + i] : 0.f;
   }
-  float fr[NV], fk[NV], fw[NV], fv[(CH * 32 + 255) / 256];
+  float fr[NV], fk[NV], fw[NV], fv[(CH * WC + 255) / 256];
   auto fetch = [&](int base) __attribute__((always_inline)) {
 #pragma unroll
     for (int q = 0; q < NV; ++q) {
@@ -112,8 +125,8 @@ __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
       fw[q] = in ? wp[row * p.ldw + i] : 0.f;
     }
 #pragma unroll
-    for (int q = 0; q < (CH * 32 + 255) / 256; ++q) {
-      const int e = threadIdx.x + q * 256, tt = e / 32, i = c0 + (e & 31);
+    for (int q = 0; q < (CH * WC + 255) / 256; ++q) {
+      const int e = threadIdx.x + q * 256, tt = e / WC, i = c0 + (e & (WC - 1));
       const bool in = tt < CH && base + tt < n && i < D;
       fv[q] = in ? ld1(vp + (size_t)(t0 + min(base + tt, n - 1)) * p.ld + i) : 0.f;
     }
@@ -131,9 +144,9 @@ __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
       }
     }
 #pragma unroll
-    for (int q = 0; q < (CH * 32 + 255) / 256; ++q) {
+    for (int q = 0; q < (CH * WC + 255) / 256; ++q) {
       const int e = threadIdx.x + q * 256;
-      if (e < CH * 32) vs[e / 32][e & 31] = fv[q];
+      if (e < CH * WC) vs[e / WC][e & (WC - 1)] = fv[q];
     }
     __syncthreads();
     if (base + CH < n) fetch(base + CH);
@@ -143,44 +156,82 @@ __global__ __launch_bounds__(256) void wkv_scan_kernel(Scan p) {
       const int tt = t8 + (threadIdx.x >> 4), l = threadIdx.x & 15;
       float a = 0.f;
       if (tt < CH)
-        for (int i = l; i < D; i += 16) a += rs[tt][i] * p.u[hb + i] * ks[tt][i];
+#pragma unroll
+        for (int q = 0; q < DP / 16; ++q) a += rs[tt][l + 16 * q] * ur[q] * ks[tt][l + 16 * q];
 #pragma unroll
       for (int s = 8; s > 0; s >>= 1) a += __shfl_xor(a, s, 64);
       if (tt < CH && l == 0) ruk[tt] = a;
     }
     __syncthreads();
-    auto token = [&](int tt) __attribute__((always_inline)) {
-      const float v = vs[tt][col];
-      float o = 0.f;
+    // 8 tokens at a time, the next token's operands on their way while one is summed; lane part q keeps token q's output
+    const int m = min(CH, n - base);
+    f32x4 r4[2][R / 4], k4[2][R / 4], w4[2][R / 4];
+    float v1[2][CPL];
+    auto get = [&](int tt, int b) __attribute__((always_inline)) {
 #pragma unroll
-      for (int i4 = 0; i4 < R; i4 += 4) {
-        const f32x4 r4 = *reinterpret_cast<const f32x4*>(&rs[tt][part * R + i4]);
-        const f32x4 k4 = *reinterpret_cast<const f32x4*>(&ks[tt][part * R + i4]);
-        const f32x4 w4 = *reinterpret_cast<const f32x4*>(&ws[tt][part * R + i4]);
+      for (int q = 0; q < R / 4; ++q) {
+        r4[b][q] = *reinterpret_cast<const f32x4*>(&rs[tt][part * R + 4 * q]);
+        k4[b][q] = *reinterpret_cast<const f32x4*>(&ks[tt][part * R + 4 * q]);
+        w4[b][q] = *reinterpret_cast<const f32x4*>(&ws[tt][part * R + 4 * q]);
+      }
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          o = fmaf(r4[e], S[i4 + e], o);
-          S[i4 + e] = fmaf(w4[e], S[i4 + e], k4[e] * v);
+      for (int c = 0; c < CPL; ++c) v1[b][c] = vs[tt][col + c];
+    };
+    auto token = [&](int b, float (&o)[CPL]) __attribute__((always_inline)) {
+#pragma unroll
+      for (int c = 0; c < CPL; ++c) {
+        float o0 = 0.f, o1 = 0.f;
+#pragma unroll
+        for (int i4 = 0; i4 < R / 4; ++i4)
+#pragma unroll
+          for (int e = 0; e < 4; e += 2) {
+            const int i = 4 * i4 + e;
+            o0 = fmaf(r4[b][i4][e], S[c][i], o0);
+            o1 = fmaf(r4[b][i4][e + 1], S[c][i + 1], o1);
+            S[c][i] = fmaf(w4[b][i4][e], S[c][i], k4[b][i4][e] * v1[b][c]);
+            S[c][i + 1] = fmaf(w4[b][i4][e + 1], S[c][i + 1], k4[b][i4][e + 1] * v1[b][c]);
+          }
+        o[c] = sum_parts<PARTS>(o0 + o1);
+      }
+    };
+    get(0, 0);
+    for (int t8 = 0; t8 < m; t8 += 8) {
+      float mine[CPL], o[CPL];
+#pragma unroll
+      for (int c = 0; c < CPL; ++c) mine[c] = 0.f;
+      const int last = m - 1 - t8, tt = t8 + (part & 7);
+      const float rk = ruk[tt];
+      if (last >= 7) {
+#pragma unroll
+        for (int q = 0; q < 8; ++q) {
+          get(min(t8 + q + 1, CH - 1), (q & 1) ^ 1);
+          token(q & 1, o);
+#pragma unroll
+          for (int c = 0; c < CPL; ++c) mine[c] = part == q ? o[c] : mine[c];
+        }
+      } else {
+#pragma unroll
+        for (int q = 0; q < 8; ++q) {
+          get(min(t8 + q + 1, CH - 1), (q & 1) ^ 1);
+          if (q > last) continue;              // (uniform)
+          token(q & 1, o);
+#pragma unroll
+          for (int c = 0; c < CPL; ++c) mine[c] = part == q ? o[c] : mine[c];
         }
       }
-      o = sum8(o);
-      if (part == 0 && j < D) p.o[(size_t)(t0 + base + tt) * p.ldo + hb + j] = o + ruk[tt] * v;
-    };
-    const int m = min(CH, n - base);
-    int tt = 0;
-    for (; tt + 4 <= m; tt += 4) {           // the LDS reads of later tokens overlap the sums of earlier ones
-      token(tt);
-      token(tt + 1);
-      token(tt + 2);
-      token(tt + 3);
+      if (part < 8 && part <= last)
+#pragma unroll
+        for (int c = 0; c < CPL; ++c)
+          if (j + c < D) p.o[(size_t)(t0 + base + tt) * p.ldo + hb + j + c] = fmaf(rk, vs[tt][col + c], mine[c]);
     }
-    for (; tt < m; ++tt) token(tt);
   }
 #pragma unroll
-  for (int i = 0; i < R; ++i) {
-    const int row = part * R + i;
-    if (row < D && j < D) st[(size_t)row * D + j] = S[i];
-  }
+  for (int i = 0; i < R; ++i)
+#pragma unroll
+    for (int c = 0; c < CPL; ++c) {
+      const int row = part * R + i;
+      if (row < D && j + c < D) st[(size_t)row * D + j + c] = S[c][i];
+    }
   // the run's last row is the next step's previous token (this layer's shift_mix, which reads it, came before)
   const int G = gridDim.x;
   for (int i = blockIdx.x * 256 + threadIdx.x; i < p.width; i += G * 256)
@@ -267,15 +318,23 @@ __global__ __launch_bounds__(256) void wkv_out_kernel(const float* __restrict__ 
   }
 }
 
+template <typename T, int DP>
+int scan_d(const Scan& p, int nruns, hipStream_t st) {
+  auto grid = [&](int wc) { return dim3(p.H * ((p.D + wc - 1) / wc), nruns); };
+  if (DP < 64 || p.H * nruns * ((p.D + 31) / 32) >= 256)
+    hipLaunchKernelGGL((wkv_scan_kernel<T, DP, 8, 1>), grid(32), dim3(256), 0, st, p);
+  else
+    hipLaunchKernelGGL((wkv_scan_kernel<T, DP, DP < 64 ? 8 : 16, 1>), grid(16), dim3(256), 0, st, p);
+  return (int)hipGetLastError();
+}
+
 template <typename T>
 int scan_t(const Scan& p, int nruns, hipStream_t st) {
-  const dim3 grid(p.H * ((p.D + 31) / 32), nruns);
-  if (p.D <= 32) hipLaunchKernelGGL((wkv_scan_kernel<T, 32>), grid, dim3(256), 0, st, p);
-  else if (p.D <= 64) hipLaunchKernelGGL((wkv_scan_kernel<T, 64>), grid, dim3(256), 0, st, p);
-  else if (p.D <= 128) hipLaunchKernelGGL((wkv_scan_kernel<T, 128>), grid, dim3(256), 0, st, p);
-  else if (p.D <= 256) hipLaunchKernelGGL((wkv_scan_kernel<T, 256>), grid, dim3(256), 0, st, p);
-  else return -1;
-  return (int)hipGetLastError();
+  if (p.D <= 32) return scan_d<T, 32>(p, nruns, st);
+  if (p.D <= 64) return scan_d<T, 64>(p, nruns, st);
+  if (p.D <= 128) return scan_d<T, 128>(p, nruns, st);
+  if (p.D <= 256) return scan_d<T, 256>(p, nruns, st);
+  return -1;
 }
 
 }  // namespace nls_wkv

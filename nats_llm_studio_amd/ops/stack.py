@@ -165,6 +165,9 @@ class Seg:
 GEMM_TILES = ((64, 64), (128, 64), (128, 128), (256, 128), (256, 256))     # (weight rows, rows) of lin_gemm's cfg
 
 
+GEMM_RATE = {4: 1.0, 3: 0.95, 2: 0.75, 1: 0.55, 0: 0.4}      # relative multiply rates of the tiles
+
+
 class LinLaunch:
     """A launch of up to SEGS independent linear layers, bound to its buffers once (only the row count and the launch
     config change from step to step)."""
@@ -202,6 +205,11 @@ class LinLaunch:
             return False, mt, nw
         if bm is None and self._tiles(64, 64, M) < 96 and self._tiles(16, 16, M) <= 1024:
             return False, 1, 16           # few outputs (routers): split K over a workgroup's waves instead
+        if bm is None and M > 512:
+            # compute-bound: rounds of 256 workgroups times a tile's cost (the small tiles run two to a CU)
+            cost = {c: -(-self._tiles(*GEMM_TILES[c], M) // 256) * GEMM_TILES[c][0] * GEMM_TILES[c][1] / GEMM_RATE[c]
+                    for c in GEMM_RATE}
+            return True, min(cost, key=cost.get), 0
         for c in (4, 3, 2, 1, 0):
             bn, b = GEMM_TILES[c]
             if bm is not None and b != bm:
