@@ -6,7 +6,8 @@
 // The scan is sequential in the tokens of a run, so a position's result does not depend on how its sequence was cut
 // into steps. Parallelism is (run, head, value columns) x lanes: a lane holds DP / PARTS key rows of CPL value columns in
 // registers, PARTS neighbouring lanes cover the keys and close the sum with in-row lane exchanges (DPP). Few runs take
-// many key parts (short per-token chains on all CUs). Tokens are staged in LDS in chunks of CH as f32, the next chunk's loads in flight while the current one runs.
+// many key parts (short per-token chains on all CUs). Tokens are staged in LDS in chunks of CH as f32, the next chunk's
+// loads in flight while the current one runs.
 // A step of single tokens (decode) streams each head's state once with 16-byte accesses and ends with the head's norm and
 // gate (wkv_step_kernel).
 //

@@ -34,7 +34,7 @@ class LinArgs(ctypes.Structure):
 
 _SIGS = {
     "nls_lin_args_size": [],
-    "nls_lin_small": [P, I, I, I, P],
+    "nls_lin_small": [P, I, I, I, I, P],
     "nls_lin_gemm": [P, I, I, P],
     "nls_stack_embed": [P, P, P, P, I, I, P, P, L, I, P],
     "nls_norm_add": [P, L, P, I, L, P, P, P, L, P, P, L, I, I, F, I, P],
@@ -194,29 +194,35 @@ class LinLaunch:
         return self.plan.expect_tiles(M, bm)
 
     def config(self, M: int):
-        """(gemm?, a, b): few-row kernel with a 16-row tiles and b waves, or GEMM config a."""
-        bm = self.plan.bm(M) if self.plan is not None else None
-        if bm is not None and bm <= 32 or bm is None and M <= 64:
-            mt = (bm or pad_to(M, 16)) // 16
-            mt = 1 if mt <= 1 else (2 if mt == 2 else 4)
-            n = self._tiles(16, 16 * mt, M)
-            ns = max(s.w.nsub for s in self.segs)
-            nw = 4 if n >= 1536 or ns <= 16 else (8 if n >= 512 or mt > 1 or ns <= 64 else 16)
-            return False, mt, nw
-        if bm is None and self._tiles(64, 64, M) < 96 and self._tiles(16, 16, M) <= 1024:
-            return False, 1, 16           # few outputs (routers): split K over a workgroup's waves instead
-        if bm is None and M > 512:
-            # compute-bound: rounds of 256 workgroups times a tile's cost (the small tiles run two to a CU)
-            cost = {c: -(-self._tiles(*GEMM_TILES[c], M) // 256) * GEMM_TILES[c][0] * GEMM_TILES[c][1] / GEMM_RATE[c]
-                    for c in GEMM_RATE}
-            return True, min(cost, key=cost.get), 0
-        for c in (4, 3, 2, 1, 0):
-            bn, b = GEMM_TILES[c]
-            if bm is not None and b != bm:
-                continue
-            if c in (0,) or self._tiles(bn, b, M) >= 224:
-                return True, c, 0
-        return True, (2 if bm == 128 else 0), 0
+        """(False, mt, nw, rt): few-row kernel with mt activation tiles, nw waves and rt weight tiles per workgroup; or
+        (True, c): GEMM config c."""
+        if self.plan is not None:
+            bm = self.plan.bm(M)
+            if bm == 16:
+                return False, 1, (4 if self._tiles(16, 16, M) >= 1536 else 8), 1
+            if bm == 64:
+                return True, 0
+            return True, (3 if self._tiles(256, 128, M) >= 224 else 2)
+        n16, n64 = self._tiles(16, 16, M), self._tiles(64, 64, M)
+        ns = max(s.w.nsub for s in self.segs)
+        if M <= 16:
+            if M > 8 and n16 >= 1024:
+                return False, 1, 4, 2
+            return False, 1, (4 if ns <= 16 else 8 if n16 >= 320 or ns <= 32 else 16), 1
+        if n16 <= 64:                     # a router's few outputs: split K over a workgroup's waves
+            return False, 1, 16, 1
+        if M <= 64:
+            if n64 >= 250:
+                return True, 0
+            return False, 2, (4 if ns <= 16 else 8), (2 if M > 32 or n16 >= 640 else 1)
+        if n64 < 96 and n16 <= 1024:
+            return False, 1, 16, 1
+        if M <= 512:
+            return True, (3 if self._tiles(256, 128, M) >= 120 else 0)
+        # compute-bound: rounds of 256 workgroups times a tile's cost (the small tiles run two to a CU)
+        cost = {c: -(-self._tiles(*GEMM_TILES[c], M) // 256) * GEMM_TILES[c][0] * GEMM_TILES[c][1] / GEMM_RATE[c]
+                for c in GEMM_RATE}
+        return True, min(cost, key=cost.get)
 
     def run(self, M: int, st: int, M_of: Optional[dict] = None):
         if self.plan is not None:
@@ -233,7 +239,7 @@ class LinLaunch:
         if cfg[0]:
             _check(lib().nls_lin_gemm(ctypes.byref(self.a), self.f32, cfg[1], st), "nls_lin_gemm")
         else:
-            _check(lib().nls_lin_small(ctypes.byref(self.a), self.f32, cfg[1], cfg[2], st), "nls_lin_small")
+            _check(lib().nls_lin_small(ctypes.byref(self.a), self.f32, *cfg[1:], st), "nls_lin_small")
 
 
 class MoePlan:
@@ -253,7 +259,7 @@ class MoePlan:
     def bm(self, T: int) -> int:
         """Rows per tile of the expert products at T tokens."""
         avg = T * self.top / self.experts
-        return 16 if avg <= 12 else (32 if avg <= 24 else (64 if avg <= 96 else 128))
+        return 16 if avg <= 6 else (64 if avg <= 96 else 128)
 
     def max_tiles(self, T: int, bm: Optional[int] = None) -> int:
         bm = bm or self.bm(T)

@@ -63,8 +63,9 @@ def test_linear(K, dt, M, N, Kd):
 
 
 @pytest.mark.parametrize("dt", DT)
-@pytest.mark.parametrize("cfg", [(True, c, 0) for c in range(5)] + [(False, 1, 4), (False, 1, 8), (False, 1, 16), (False, 2, 4),
-                                                                   (False, 2, 8), (False, 4, 4), (False, 4, 8)])
+@pytest.mark.parametrize("cfg", [(True, c) for c in range(5)] + [(False, m, w, r) for m, w, r in (
+    (1, 4, 1), (1, 8, 1), (1, 16, 1), (1, 4, 2), (1, 8, 2), (2, 4, 1), (2, 8, 1), (2, 4, 2), (2, 8, 2), (2, 4, 4), (4, 4, 1),
+    (4, 8, 1), (4, 4, 2), (4, 8, 2), (4, 4, 4))])
 def test_linear_every_tile(K, dt, cfg):
     """Every launch shape gives the same product, also where tiles end past the matrix and K has one step."""
     d = DT[dt]
@@ -298,6 +299,80 @@ def test_latent_attention(K, dt, H, R, rot):
     ctx[3] = 0
     K.latent_attention(q, cache, out.view(T, -1), part, bt, bs, rows, ctx, T, H, 1, Rp, rp, scale, st())
     assert (out[3] == 0).all()
+
+
+LATENT = {"small": S.mixer_latent(), "one": S.mixer_latent(1, 8, 2, 4, 8, 8, base=40.0, scale=1.0),
+          "odd": S.mixer_latent(heads=3, dim=50, rot=34, vdim=37, kv_rank=100, q_rank=70, scale=0.2),
+          "even": S.mixer_latent(heads=20, dim=128, rot=64, vdim=128, kv_rank=512, q_rank=192, base=1e4, scale=0.07)}
+
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("name", LATENT)
+@pytest.mark.parametrize("expand", [32, 1 << 30])
+def test_latent_mixer(gpu, tmp_path, dt, name, expand, monkeypatch):
+    """A latent layer and one that reads its cache, over portions of one sequence (prompt rows expanded to per-head keys, or
+    all in the latent space), next to a second sequence; one key's direction is boosted so that a few rows hang on it."""
+    from nats_llm_studio_amd.models import stack
+    monkeypatch.setattr(stack, "_EXPAND_RUN", expand)
+    mx = LATENT[name]
+    cfg = S.config([S.layer(mx), S.layer({"type": mx["type"], "mixer": dict(mx["mixer"], kv_from=0)})], width=72, vocab=50)
+    W, d, n = S.make_weights(cfg), 72, 330
+    m = load(tmp_path, cfg, W, dt)
+    b = m.step_buffers(512, 2, 32)
+    kc, _ = m.kv_cache(64, 16)
+    x = rnd(n, d, seed=4)
+    for far in (0, 15, 16, 63, 64, 200, 255, 256):           # equal rows: their queries and keys agree whatever the place
+        x[far] = 3 * x[5]
+    x[n - 1] = x[270] = 3 * x[5]
+    x, z = x.to(torch.bfloat16), rnd(n, d, seed=9).to(torch.bfloat16)
+    blk = torch.randperm(42, generator=torch.Generator().manual_seed(1)).view(2, 21)
+    got = {0: [], 1: []}
+    for a, c in ((0, 1), (1, 3), (3, 67), (67, 100), (100, 300), (300, 301), (301, 330)):
+        T = c - a
+        for r, src in ((0, x), (1, z)):
+            o = r * T
+            pos = torch.arange(a, c)
+            b.act[o:o + T, :d] = src[a:c].to(b.act.dtype)
+            b.pos[o:o + T], b.ctx_len[o:o + T], b.tok_seq[o:o + T] = pos.int(), (pos + 1).int(), r
+            b.slot[o:o + T] = (blk[r][pos // 16] * 16 + pos % 16).int()
+            b.block_tables[r, :21] = blk[r].int()
+        info = m.attention_blocks(b, 2 * T)
+        assert bool(info) == (dt == "bf16" and T >= expand)
+        step = stack._Step(2 * T, 2, 16, st())
+        if info:
+            step.plan = m._expand_plan(b, info["qblocks"], info["row_info"], 2 * T, 16, st())
+        for i in (0, 1):
+            m.layers[i][0].run(b, b.launches[i, "mix"], kc, None, step)
+            got[i].append(b.y[:2 * T].clone())
+    Wd, pos = {k: v.double() for k, v in W.items()}, torch.arange(n)
+    for r, src in ((0, x), (1, z)):
+        c, kr = O.latent_rows(src.double(), Wd, "l0.mix.", mx["mixer"], pos, cfg["norm"]["eps"])
+        for i in (0, 1):
+            want = O.latent_mixer(src.double(), Wd, f"l{i}.mix.", mx["mixer"], pos, cfg["norm"]["eps"], c, kr)
+            g = torch.cat([y[r * (len(y) // 2):(r + 1) * (len(y) // 2)] for y in got[i]])
+            assert relerr(g, want) < TOL[dt] * 2, (r, i)
+
+
+def test_expanded_runs_beside_short_ones(gpu, tmp_path):
+    """A batch of expanded prompts, short portions and single tokens, and the plan it makes."""
+    cfg = S.CONFIGS["wide"]
+    W = S.make_weights(cfg)
+    m = load(tmp_path, cfg, W, "bf16")
+    ts = [0] * 300 + [1] + [2] * 31 + [3] * 40
+    ps = list(range(300)) + [77] + list(range(31)) + list(range(100, 140))
+    qb, info = m.row_blocks(ts, ps, len(ts))
+    assert info["nspans"] == 2 and info["nx"] == 300 + 140 and info["maxctx"] == 300 and info["rest"]
+    q = 32 * info["waves"]
+    assert sorted(map(tuple, qb[2:, :5].tolist())) == sorted([(o, min(q, 300 - o), 0, o, 0) for o in range(0, 300, q)]
+                                                             + [(332, 40, 3, 100, 300)])
+    assert m.row_blocks([0, 1], [5, 9], 2) == (None, None)
+    eng = engine(m, "bf16")
+    seqs = {k: S.tokens(n, cfg["vocab"], n) for k, n in (("a", 300), ("b", 78), ("c", 31), ("d", 140))}
+    eng.feed([("b", seqs["b"][:77], []), ("d", seqs["d"][:100], [])])
+    got = eng.feed([("a", seqs["a"], list(range(300))), ("b", seqs["b"][77:], [0]), ("c", seqs["c"], list(range(31))),
+                    ("d", seqs["d"][100:], list(range(40)))])
+    for (k, t), g in zip(seqs.items(), got):
+        assert close(g, O.forward(cfg, W, t)[-len(g):], "bf16"), k
 
 
 def run_rows(m, b, kc, state, parts, bs=16):
