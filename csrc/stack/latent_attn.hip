@@ -82,8 +82,8 @@ __global__ __launch_bounds__(256 * NHB, 1) void latent_attn_kernel(LA p) {
   if (ts >= p.T * p.ns) return;
   const int t = ts / p.ns, split = ts % p.ns;
   const int ctx = p.ctx_len[t];
-  const int chunk = ((ctx + p.ns - 1) / p.ns + KT - 1) / KT * KT;
-  const int k0 = split * chunk, k1 = min(ctx, k0 + chunk);
+  const int tiles = (ctx + KT - 1) / KT;       // dealt to the splits as evenly as whole tiles go
+  const int k0 = tiles * split / p.ns * KT, k1 = min(ctx, tiles * (split + 1) / p.ns * KT);
   const int lane = threadIdx.x & 63;
   const int r = lane & 15, g = lane >> 4;
   const int head = (hb * NHB + hsub) * 16 + r;
@@ -245,6 +245,34 @@ __global__ __launch_bounds__(256 * NHB, 1) void latent_attn_kernel(LA p) {
   }
 }
 
+// few splits: a workgroup per (token, head), 4 columns per thread
+__global__ __launch_bounds__(256) void latent_merge_few_kernel(LA p) {
+  const size_t th = blockIdx.x;
+  const float* ml = p.part_ml + th * p.ns * 2;
+  float M = -INFINITY, L = 0.f, w[8];
+#pragma unroll
+  for (int s = 0; s < 8; ++s) {
+    w[s] = s < p.ns ? ml[2 * s] : -INFINITY;
+    M = fmaxf(M, w[s]);
+  }
+#pragma unroll
+  for (int s = 0; s < 8; ++s) {
+    w[s] = w[s] == -INFINITY ? 0.f : exp2f(w[s] - M);
+    if (s < p.ns) L += ml[2 * s + 1] * w[s];
+  }
+  const float inv = L > 0.f ? 1.f / L : 0.f;
+  for (int c = threadIdx.x * 4; c < p.Rp; c += (int)blockDim.x * 4) {
+    const float* po = p.part_o + th * p.ns * p.Rp + c;
+    f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < 8; ++s)
+      if (w[s] != 0.f) a += *reinterpret_cast<const f32x4*>(po + (size_t)s * p.Rp) * (w[s] * inv);
+    typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+    *reinterpret_cast<bf4*>(reinterpret_cast<__bf16*>(p.out) + th * p.Rp + c) =
+        bf4{(__bf16)a[0], (__bf16)a[1], (__bf16)a[2], (__bf16)a[3]};
+  }
+}
+
 // splits of one (token, head), 64 output columns: 16 lanes x 4 columns, 16 groups of splits
 __global__ __launch_bounds__(256) void latent_merge_kernel(LA p) {
   __shared__ float w[64];
@@ -354,7 +382,10 @@ int launch_t(const LA& p, hipStream_t st) {
   hipLaunchKernelGGL((latent_attn_kernel<NT, RT, KT, NHB>), dim3(n), dim3(256 * NHB), LDS, st, p);
   int rc = (int)hipGetLastError();
   if (rc == 0 && p.ns > 1) {
-    hipLaunchKernelGGL(latent_merge_kernel, dim3(p.T * p.H, p.Rp / 64), dim3(256), 0, st, p);
+    if (p.ns <= 8)
+      hipLaunchKernelGGL(latent_merge_few_kernel, dim3(p.T * p.H), dim3(min(256, p.Rp / 4)), 0, st, p);
+    else
+      hipLaunchKernelGGL(latent_merge_kernel, dim3(p.T * p.H, p.Rp / 64), dim3(256), 0, st, p);
     rc = (int)hipGetLastError();
   }
   return rc;

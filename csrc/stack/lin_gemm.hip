@@ -146,6 +146,7 @@ int gemm_d(LinArgs& a, int cfg, hipStream_t st) {
     case 2: return gemm_t<T, 128, 128, 2, 2, 2>(a, st);
     case 3: return gemm_t<T, 256, 128, 4, 2, 3>(a, st);
     case 4: return gemm_t<T, 256, 256, 4, 2, 2>(a, st);
+    case 5: return gemm_t<T, 64, 64, 2, 2, 8>(a, st);
   }
   return -1;
 }
@@ -154,7 +155,8 @@ int gemm_d(LinArgs& a, int cfg, hipStream_t st) {
 
 extern "C" {
 
-// cfg: tile of the launch (BN x BM): 0 = 64 x 64, 1 = 128 x 64, 2 = 128 x 128, 3 = 256 x 128, 4 = 256 x 256
+// cfg: tile of the launch (BN x BM): 0 = 64 x 64, 1 = 128 x 64, 2 = 128 x 128, 3 = 256 x 128, 4 = 256 x 256,
+// 5 = 64 x 64 with 8 stages in flight (launches of at most one workgroup per CU)
 int nls_lin_gemm(const void* args, int f32, int cfg, void* stream) {
   nls_lin::LinArgs a = *reinterpret_cast<const nls_lin::LinArgs*>(args);
   return f32 ? nls_lin::gemm_d<float>(a, cfg, (hipStream_t)stream)

@@ -162,7 +162,7 @@ class Seg:
         self.keep = (bias, gate, routed, rope, xmap)
 
 
-GEMM_TILES = ((64, 64), (128, 64), (128, 128), (256, 128), (256, 256))     # (weight rows, rows) of lin_gemm's cfg
+GEMM_TILES = ((64, 64), (128, 64), (128, 128), (256, 128), (256, 256), (64, 64))     # (weight rows, rows) of lin_gemm's cfg
 
 
 GEMM_RATE = {4: 1.0, 3: 0.95, 2: 0.75, 1: 0.55, 0: 0.4}      # relative multiply rates of the tiles
@@ -218,7 +218,7 @@ class LinLaunch:
         if n64 < 96 and n16 <= 1024:
             return False, 1, 16, 1
         if M <= 512:
-            return True, (3 if self._tiles(256, 128, M) >= 120 else 0)
+            return True, (3 if self._tiles(256, 128, M) >= 120 else 5 if n64 <= 256 else 0)
         # compute-bound: rounds of 256 workgroups times a tile's cost (the small tiles run two to a CU)
         cost = {c: -(-self._tiles(*GEMM_TILES[c], M) // 256) * GEMM_TILES[c][0] * GEMM_TILES[c][1] / GEMM_RATE[c]
                 for c in GEMM_RATE}

@@ -12,7 +12,7 @@ pytestmark = pytest.mark.gpu
 # Whole models: largest row error (sekolorn_models.error) in f32. In bf16 an expert choice can still be a close call, and a
 # squared relu whose units are all nearly off leaves the norm after it mostly rounding, so there the bound holds for nine
 # rows of ten; f32 runs the same kernels' f32 forms and holds for all.
-F32, BF16 = 2e-4, 0.06
+F32, BF16 = 2e-5, 0.06
 DT = {"f32": torch.float32, "bf16": torch.bfloat16}
 TOL = {"f32": 3e-5, "bf16": 1.5e-2}
 
@@ -63,7 +63,7 @@ def test_linear(K, dt, M, N, Kd):
 
 
 @pytest.mark.parametrize("dt", DT)
-@pytest.mark.parametrize("cfg", [(True, c) for c in range(5)] + [(False, m, w, r) for m, w, r in (
+@pytest.mark.parametrize("cfg", [(True, c) for c in range(6)] + [(False, m, w, r) for m, w, r in (
     (1, 4, 1), (1, 8, 1), (1, 16, 1), (1, 4, 2), (1, 8, 2), (2, 4, 1), (2, 8, 1), (2, 4, 2), (2, 8, 2), (2, 4, 4), (4, 4, 1),
     (4, 8, 1), (4, 4, 2), (4, 8, 2), (4, 4, 4))])
 def test_linear_every_tile(K, dt, cfg):
