@@ -186,7 +186,7 @@ class LatentMixer(_Part):
         q = self.scratch(b, f"lat.q{c.kv_rank}.{c.rot_dim}", P, H * self.Dp)
         lat = self.scratch(b, f"lat.o{c.kv_rank}", P, H * self.Rp)
         ao = self.scratch(b, "lat.ao", P, K.act_ld(H * c.vdim))
-        hb = (H + 15) // 16
+        hb = K.latent_head_groups(H, self.Rp)              # workgroups per (token, split)
         n = (_SPLIT_WG // hb + 1) * H
         po = self.scratch(b, "lat.po", 1, n * self.Rp, f)
         pm = self.scratch(b, "lat.pm", 1, n * 2, f)

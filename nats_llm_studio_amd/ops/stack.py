@@ -184,14 +184,12 @@ class LinLaunch:
         self._cfg = {}
 
     def _tiles(self, bn: int, bm: int, M: int) -> int:
+        """Workgroups of a launch with bn x bm tiles."""
         n = 0
         for s in self.segs:
             nt = (s.w.N + bn - 1) // bn
-            n += nt * (min(self.a.maxtiles, self._routed_tiles(bm, M)) if s.s.rows else s.w.groups * ((M + bm - 1) // bm))
+            n += nt * (self.plan.expect_tiles(M, bm) if s.s.rows else s.w.groups * ((M + bm - 1) // bm))
         return n
-
-    def _routed_tiles(self, bm: int, M: int) -> int:
-        return self.plan.expect_tiles(M, bm)
 
     def config(self, M: int):
         """(False, mt, nw, rt): few-row kernel with mt activation tiles, nw waves and rt weight tiles per workgroup; or
@@ -224,7 +222,7 @@ class LinLaunch:
                 for c in GEMM_RATE}
         return True, min(cost, key=cost.get)
 
-    def run(self, M: int, st: int, M_of: Optional[dict] = None):
+    def run(self, M: int, st: int):
         if self.plan is not None:
             self.a.maxtiles = self.plan.max_tiles(M)
         for i, s in enumerate(self.segs):
@@ -267,6 +265,7 @@ class MoePlan:
         return max(1, min(n, self.experts + n // bm))
 
     def expect_tiles(self, T: int, bm: int) -> int:
+        """About how many tiles T tokens make (launch rules)."""
         n = T * self.top
         return max(1, min(n, self.experts), n // bm)
 
@@ -325,6 +324,11 @@ def latent_pad(R: int) -> int:
         if R <= 64 * n:
             return 64 * n
     raise ValueError(f"latent width {R} > {64 * LATENT_TILES[-1]}")
+
+
+def latent_head_groups(H: int, Rp: int) -> int:
+    """Workgroups a (token, split) of latent_attention takes: 16 heads each, or 32 (csrc/stack/latent_attn.hip launch_r)."""
+    return -(-H // (32 if H > 16 and Rp < 1024 else 16))
 
 
 def rot_pad(rot: int) -> int:
