@@ -9,8 +9,9 @@
 // registers), the four waves of a block exchange row maxima and the bf16 weights through LDS, and each owns a quarter of
 // the output columns: O^T += C^T P^T with C^T fragments from transposed LDS reads of the same tile. Softmax in base 2, all
 // of it f32.
-// latent_attn_f32_kernel: the f32 form, one workgroup per (token, head).
+// 32-bit models: one workgroup per (token, head) (attn_plain.h).
 #include "../kernels/lds_dma.h"
+#include "attn_plain.h"
 
 namespace nls_latent {
 using nls_dma::glds16;
@@ -308,64 +309,6 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(LA p) {
   }
 }
 
-constexpr int NC = 4;         // output columns per thread: Rp <= 1024
-
-__global__ __launch_bounds__(256) void latent_attn_f32_kernel(LA p) {
-  __shared__ __attribute__((aligned(16))) float q[2048], sc[64];
-  const int t = blockIdx.x, h = blockIdx.y, Dp = p.Rp + p.rp;
-  const int ctx = p.ctx_len[t];
-  const int* bt = p.bt + (size_t)p.tok_seq[t] * p.bts;
-  const float* cache = reinterpret_cast<const float*>(p.cache);
-  const float* qr = reinterpret_cast<const float*>(p.q) + ((size_t)t * p.H + h) * Dp;
-  for (int i = threadIdx.x; i < Dp; i += 256) q[i] = qr[i];
-  __syncthreads();
-  const int key = threadIdx.x >> 2, part = threadIdx.x & 3;
-  float m = -INFINITY, l = 0.f, acc[NC] = {0.f, 0.f, 0.f, 0.f};
-  for (int k0 = 0; k0 < ctx; k0 += 64) {
-    const int k = k0 + key;
-    float s = 0.f;
-    if (k < ctx) {
-      const float* c = cache + ((size_t)bt[k / p.bs] * p.bs + k % p.bs) * Dp;
-      for (int d = part * 4; d < Dp; d += 16) {
-        const f32x4 a = *reinterpret_cast<const f32x4*>(c + d), b = *reinterpret_cast<const f32x4*>(q + d);
-#pragma unroll
-        for (int e = 0; e < 4; ++e) s = fmaf(a[e], b[e], s);
-      }
-    }
-    s += __shfl_xor(s, 1, 64);
-    s += __shfl_xor(s, 2, 64);
-    if (part == 0) sc[key] = k < ctx ? s * p.scale : -INFINITY;
-    __syncthreads();
-    float mn = m;
-    for (int i = 0; i < 64; ++i) mn = fmaxf(mn, sc[i]);
-    const float alpha = m == -INFINITY ? 0.f : expf(m - mn);
-    l *= alpha;
-#pragma unroll
-    for (int i = 0; i < NC; ++i) acc[i] *= alpha;
-    m = mn;
-    const int n = min(64, ctx - k0);
-    for (int i = 0; i < n; ++i) {
-      const float e = expf(sc[i] - mn);
-      l += e;
-      const int kk = k0 + i;
-      const float* c = cache + ((size_t)bt[kk / p.bs] * p.bs + kk % p.bs) * Dp;
-#pragma unroll
-      for (int q4 = 0; q4 < NC; ++q4) {
-        const int col = threadIdx.x + 256 * q4;
-        if (col < p.Rp) acc[q4] = fmaf(e, c[col], acc[q4]);
-      }
-    }
-    __syncthreads();
-  }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
-  float* y = reinterpret_cast<float*>(p.out) + ((size_t)t * p.H + h) * p.Rp;
-#pragma unroll
-  for (int q4 = 0; q4 < NC; ++q4) {
-    const int col = threadIdx.x + 256 * q4;
-    if (col < p.Rp) y[col] = acc[q4] * inv;
-  }
-}
-
 template <int NT, int RT, int NHB>
 int launch_t(const LA& p, hipStream_t st) {
   constexpr int KT = NT + RT > 9 ? 32 : 64;
@@ -416,9 +359,10 @@ int nls_latent_attn(const void* q, const void* cache, void* out, float* part_o, 
   LA p{q, cache, out, part_o, part_ml, bt, tok_seq, ctx_len, bts, bs, T, H, ns, Rp, rp, bshift, scale};
   hipStream_t st = (hipStream_t)stream;
   if (f32) {
-    if (Rp > 256 * NC || Rp + rp > 2048 || (Rp & 3) || (rp & 3) || H > 65535) return -1;
-    hipLaunchKernelGGL(latent_attn_f32_kernel, dim3(T, H), dim3(256), 0, st, p);
-    return (int)hipGetLastError();
+    const long Dp = Rp + rp;
+    const nls_plain::PA a{q, cache, cache, out, bt, tok_seq, ctx_len, nullptr, H * Dp, Dp, Dp, 0, (long)H * Rp, Rp, 0,
+                          bts, bs, H, (int)Dp, Rp, scale};
+    return nls_plain::launch<float>(a, T, H, st);
   }
   switch (Rp / 64 * (Rp % 64 == 0)) {
     case 1: return launch_r<1>(p, st);

@@ -25,7 +25,10 @@ enum LinEpi : int {
   LE_DECAY = 5,     // exp(-exp(v + bias[n]))
   LE_GATE = 6,      // v * gate[m * ldg + group]
   LE_ROPE = 7,      // rotate the pairs (n, n + 1), n % cb < 2 * half, with cs[pos[m]]
-};
+  LE_GEGLU = 8,     // gelu_tanh(v[n]) * v[n + 1] -> column n / 2 (gate and up rows of the weights alternate)
+  LE_SIGPOW = 9,    // sigmoid(v + bias[n]) ^ alpha
+  LE_SOFTCAP = 10,  // alpha * tanh(v / alpha)
+};                  // LE_SIGMOID: alpha * sigmoid(v)
 
 struct LinSeg {
   const void* w;        // packed weights of group 0
@@ -45,7 +48,8 @@ struct LinSeg {
   int epi, yact;        // yact: store the activation type (bf16; f32 in f32 launches), else f32
   int cb, cstep;        // output column n -> (n / cb) * cstep + n % cb
   int xdiv, ldg;        // routed: x row = entry / xdiv
-  int half, pad0;
+  int half;
+  float alpha;          // constant of the epilogue
 };
 
 struct LinArgs {
@@ -124,6 +128,8 @@ DEVI void lin_row(const LinSeg& S, const LinTile& t, int i, int& xr, int& yr) {
 }
 
 DEVI float lin_sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
+// z / 2 (1 + tanh(y)) = z sigmoid(2 y), y = sqrt(2 / pi) (z + 0.044715 z^3)
+DEVI float lin_gelu(float z) { return z * lin_sigmoid(1.5957691216057308f * fmaf(0.044715f * z * z, z, z)); }
 
 // epilogue of 4 consecutive output columns n .. n + 3 of one row
 template <typename T>
@@ -141,7 +147,7 @@ DEVI void lin_store4(const LinSeg& S, int grp, int n, int yr, f32x4 v) {
       break;
     case LE_SIGMOID:
 #pragma unroll
-      for (int e = 0; e < 4; ++e) v[e] = lin_sigmoid(v[e]);
+      for (int e = 0; e < 4; ++e) v[e] = S.alpha * lin_sigmoid(v[e]);
       break;
     case LE_RELU2:
 #pragma unroll
@@ -155,6 +161,36 @@ DEVI void lin_store4(const LinSeg& S, int grp, int n, int yr, f32x4 v) {
       for (int e = 0; e < 4; ++e)
         if (n + e < S.N) v[e] = expf(-expf(v[e] + S.bias[n + e]));
       break;
+    case LE_SIGPOW:
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (n + e < S.N) {
+          const float z = v[e] + S.bias[n + e];
+          v[e] = expf(S.alpha * (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))));
+        }
+      break;
+    case LE_SOFTCAP:
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] = S.alpha * tanhf(v[e] / S.alpha);
+      break;
+    case LE_GEGLU: {                    // N is even: both pairs or the first one lie inside
+      const size_t o = (size_t)yr * S.ldy + (size_t)grp * S.ygs + (n >> 1);
+      const float a = lin_gelu(v[0]) * v[1], b = lin_gelu(v[2]) * v[3];
+      if (S.yact && sizeof(T) == 2) {
+        __bf16* y = reinterpret_cast<__bf16*>(S.y) + o;
+        typedef __bf16 bf2 __attribute__((ext_vector_type(2)));
+        if (n + 4 <= S.N && (o & 1) == 0) *reinterpret_cast<bf2*>(y) = bf2{(__bf16)a, (__bf16)b};
+        else {
+          y[0] = (__bf16)a;
+          if (n + 4 <= S.N) y[1] = (__bf16)b;
+        }
+      } else {
+        float* y = reinterpret_cast<float*>(S.y) + o;
+        y[0] = a;
+        if (n + 4 <= S.N) y[1] = b;
+      }
+      return;
+    }
     case LE_GATE: {
       const float gt = S.gate[(size_t)yr * S.ldg + grp];
 #pragma unroll
@@ -207,7 +243,8 @@ inline int lin_count(LinArgs& a, int BN, int BM) {
     if (S.N < 1 || S.nsub < 2 || (S.nsub & 1) || S.ng < 1 || S.cb < 4 || (S.cb & 3) || S.xdiv < 1) return -1;
     if (!S.w || !S.x || !S.y) return -1;
     if (S.epi == LE_ROPE && (!S.cs || !S.pos)) return -1;
-    if (S.epi == LE_DECAY && !S.bias) return -1;
+    if ((S.epi == LE_DECAY || S.epi == LE_SIGPOW) && !S.bias) return -1;
+    if (S.epi == LE_GEGLU && ((S.N & 1) || S.cb < S.N)) return -1;
     if (S.epi == LE_GATE && !S.gate) return -1;
     if (S.rows && (!a.tiles || !a.ntiles || a.maxtiles < 1)) return -1;
     if (!S.rows && S.M < 1) return -1;

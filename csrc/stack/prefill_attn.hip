@@ -1,18 +1,22 @@
-// Prompt attention of latent-attention layers (bf16, gfx950): for runs of many tokens the per-head keys and values are
-// expanded once from the cached latents (a GEMM over the run's context, ops/stack.py) and this kernel is a causal flash
-// attention over them; the rotated key part, shared by all heads, is read from the cache rows themselves. Short runs and
-// decoded tokens attend in the latent space instead (latent_attn.hip).
+// Prompt attention of the config-driven stacks (bf16, gfx950), a causal flash attention in two forms:
+//   latent attention: the per-head keys and values of a run are expanded once from the cached latents (a GEMM over the run's
+//     context, ops/stack.py); the rotated key part, shared by all heads, is read from the cache rows themselves.
+//   grouped-query attention (no rotated part, NKR = 0): keys and values are the paged cache rows; the gs query heads of a key
+//     head are rows beside each other (row = token * gs + head of the group), so any group size fills the MFMA tiles and a
+//     tile staged in LDS serves the whole group.
+// Short runs and decoded tokens attend row by row instead (latent_attn.hip, attn.hip).
 //
-// Workgroup = (head, block of 32 * NWV query tokens of one run), one wave per 32 tokens; every 64-key tile staged in LDS
+// Workgroup = (key head, 32 * NWV rows of a block of one run's tokens), one wave per 32 rows; every 64-key tile staged in LDS
 // serves all of them. Per tile and wave, with v_mfma_f32_32x32x16_bf16:
-//   S^T = K Q^T: lane l owns token l & 31 and, per 32-key block, keys (r & 3) + 8 (r >> 2) + 4 (l >> 5): the row maximum
+//   S^T = K Q^T: lane l owns row l & 31 and, per 32-key block, keys (r & 3) + 8 (r >> 2) + 4 (l >> 5): the row maximum
 //   closes with one lane exchange; P^T goes from those registers straight into O^T += V^T P^T (V^T by transposed LDS
-//   reads in the same key order), so a token's rescale is lane-local and skipped when no maximum grew.
-// The next tile's loads are in flight in registers while a tile computes; one barrier per tile, two LDS buffers. Rows are
-// padded in LDS (K: 16 bytes, V: 64) against bank conflicts. The epilogue applies the head's output gate.
+//   reads in the same key order), so a row's rescale is lane-local and skipped when no maximum grew.
+// The next tile's loads are in flight in registers while a tile computes (its cache slots one tile ahead of that); one
+// barrier per tile, two LDS buffers. Rows are padded in LDS (K: 16 bytes, V: 64) against bank conflicts. The epilogue applies
+// the head's output gate.
 #include "../kernels/common.h"
 
-namespace nls_lpf {
+namespace nls_pfa {
 
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 typedef short s16x4 __attribute__((ext_vector_type(4)));
@@ -29,70 +33,96 @@ __global__ __launch_bounds__(256) void expand_plan_kernel(const int* __restrict_
     for (int i = blockIdx.y * 256 + threadIdx.x; i < s[1]; i += gridDim.y * 256) actx[s[0] + i] = 0;
 }
 
-struct LP {
-  const __bf16* qn;       // unrotated queries [T][ldqn], head stride qns
-  const __bf16* qr;       // rotated queries [T][ldqr], head stride qrs (pointer at the rotated part of head 0)
-  const __bf16* kx;       // expanded keys [context rows][H * DKU]
-  const __bf16* vx;       // expanded values [context rows][H * DV]
-  const __bf16* cache;    // cache rows at their rotated part
-  const int* xmap;
+struct FP {
+  const __bf16* qn;       // queries (latent: their unrotated part) [T][ldqn], head stride qns
+  const __bf16* qr;       // latent: rotated queries [T][ldqr], head stride qrs (pointer at the rotated part of head 0)
+  const __bf16* kx;       // latent: expanded keys [context rows][H * DKU]; grouped: cache rows [slots][ldc], key heads DKU apart
+  const __bf16* vx;       // values likewise (DV)
+  const __bf16* cache;    // latent: cache rows at their rotated part
+  const int* xmap;        // cache slot of every context row
   const int* blocks;      // [n][8]: (first row, rows, sequence, first position, xoff, -, -, -), heaviest first
   const float* gate;      // [T][H]
   __bf16* out;            // [T][ldo], head stride vdim
   long ldqn, ldqr, ldc, ldo;
   int qns, qrs, H, vdim, ldg;
+  int gs, nsub;           // grouped: query heads per key head; workgroups per block and key head
   float scale;
 };
 
 template <int NKU, int NKR, int NDB, int NWV>      // 32-column units: keys unrotated / rotated, values; waves
-__global__ __launch_bounds__(64 * NWV) void latent_prefill_kernel(LP p) {
+__global__ __launch_bounds__(64 * NWV) void flash_prefill_kernel(FP p) {
+  constexpr bool PAGED = NKR == 0;
+  static_assert(!PAGED || NKU == NDB, "grouped form: equal key and value widths");
   constexpr int NT = 64 * NWV, KT = 64;
   constexpr int DKU = 32 * NKU, DR = 32 * NKR, DK = DKU + DR, DV = 32 * NDB;
   constexpr int KROW = DK * 2 + 16, VROW = DV * 2 + (NDB > 1 ? 64 : 0);
   constexpr int TB = KT * (KROW + VROW);
   constexpr int CU = DKU / 8, CR = DR / 8, CV = DV / 8, CPR = CU + CR + CV;   // 16-byte chunks per key
-  constexpr int NLD = (KT * CPR + NT - 1) / NT;
+  constexpr int NLK = (KT * CU + NT - 1) / NT;                               // grouped: chunks per thread of K, and of V
+  constexpr int NLD = PAGED ? 2 * NLK : (KT * CPR + NT - 1) / NT;
   constexpr int NKS = DK / 16;
   extern __shared__ __attribute__((aligned(16))) uint8_t lds[];              // [2][K tile | V tile]
 
-  const int head = blockIdx.x % p.H;
-  const int* blk = p.blocks + 8 * (blockIdx.x / p.H);
+  const int HK = PAGED ? p.H / p.gs : p.H, gs = PAGED ? p.gs : 1;
+  const int kh = blockIdx.x % HK, rest = blockIdx.x / HK;
+  const int row0 = PAGED ? (p.nsub - 1 - rest % p.nsub) * 32 * NWV : 0;      // (later rows see more keys: they go first)
+  const int* blk = p.blocks + 8 * (PAGED ? rest / p.nsub : rest);
   const int t0 = blk[0], ntok = blk[1], pos0 = blk[3], xoff = blk[4];
+  const int nrow = ntok * gs;
+  if (PAGED && row0 >= nrow) return;
   const int tid = threadIdx.x, lane = tid & 63;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int h = lane >> 5, tl = lane & 31;
-  const int tw0 = 32 * wave;
+  const int tw0 = row0 + 32 * wave;
+  const int myrow = min(tw0 + tl, nrow - 1), mytok = myrow / gs, head = PAGED ? kh * gs + myrow - mytok * gs : kh;
   const float sl2 = p.scale * 1.4426950408889634f;
-  const int nkeys = pos0 + ntok, ntile = (nkeys + KT - 1) / KT;
-  const int wlast = pos0 + min(tw0 + 31, ntok - 1);
-  const bool wact = tw0 < ntok;
-  const int qpos = pos0 + tw0 + tl;
+  const int nkeys = pos0 + (min(row0 + 32 * NWV, nrow) - 1) / gs + 1, ntile = (nkeys + KT - 1) / KT;
+  const int wlast = pos0 + min(tw0 + 31, nrow - 1) / gs, wfirst = pos0 + tw0 / gs;
+  const bool wact = tw0 < nrow;
+  const int qpos = pos0 + mytok;
 
   bf16x8 qf[NKS];
   {
-    const size_t row = (size_t)(t0 + min(tw0 + tl, ntok - 1));
+    const size_t row = (size_t)(t0 + mytok);
     const __bf16* a = p.qn + row * p.ldqn + (size_t)head * p.qns + 8 * h;
     const __bf16* b = p.qr + row * p.ldqr + (size_t)head * p.qrs + 8 * h;
 #pragma unroll
     for (int ks = 0; ks < NKS; ++ks)
       qf[ks] = *reinterpret_cast<const bf16x8*>(ks < 2 * NKU ? a + 16 * ks : b + 16 * (ks - 2 * NKU));
   }
+  int sl[PAGED ? NLK : 1];                                      // grouped: cache slots of the next tile's rows
+  auto load_slots = [&](int t) __attribute__((always_inline)) {
+    if constexpr (PAGED) {
+#pragma unroll
+      for (int i = 0; i < NLK; ++i) sl[i] = p.xmap[xoff + min(t * KT + (tid + NT * i) / CU, nkeys - 1)];
+    }
+  };
+  load_slots(0);
 
   u32x4 st[NLD];
   auto load_tile = [&](int t) __attribute__((always_inline)) {
+    if constexpr (PAGED) {
+#pragma unroll
+      for (int i = 0; i < NLK; ++i) {                           // (rows past the last key repeat it: masked below)
+        const size_t o = (size_t)sl[i] * p.ldc + (size_t)kh * DKU + ((tid + NT * i) % CU) * 8;
+        st[i] = ld16(p.kx + o);
+        st[NLK + i] = ld16(p.vx + o);
+      }
+      return;
+    }
 #pragma unroll
     for (int i = 0; i < NLD; ++i) {
       const int e = tid + NT * i;
       u32x4 v = u32x4{0u, 0u, 0u, 0u};
       if (e < KT * CU) {
         const int key = t * KT + e / CU;
-        if (key < nkeys) v = ld16(p.kx + ((size_t)(xoff + key) * p.H + head) * DKU + (e % CU) * 8);
+        if (key < nkeys) v = ld16(p.kx + ((size_t)(xoff + key) * p.H + kh) * DKU + (e % CU) * 8);
       } else if (e < KT * (CU + CR)) {
-        const int f = e - KT * CU, key = t * KT + f / CR;
-        if (key < nkeys) v = ld16(p.cache + (size_t)p.xmap[xoff + key] * p.ldc + (f % CR) * 8);
+        const int f = e - KT * CU, key = t * KT + f / max(CR, 1);
+        if (key < nkeys) v = ld16(p.cache + (size_t)p.xmap[xoff + key] * p.ldc + (f % max(CR, 1)) * 8);
       } else if (e < KT * CPR) {
         const int f = e - KT * (CU + CR), key = t * KT + f / CV;
-        if (key < nkeys) v = ld16(p.vx + ((size_t)(xoff + key) * p.H + head) * DV + (f % CV) * 8);
+        if (key < nkeys) v = ld16(p.vx + ((size_t)(xoff + key) * p.H + kh) * DV + (f % CV) * 8);
       }
       st[i] = v;
     }
@@ -100,12 +130,23 @@ __global__ __launch_bounds__(64 * NWV) void latent_prefill_kernel(LP p) {
   auto store_tile = [&](int buf) __attribute__((always_inline)) {
     uint8_t* kb = lds + buf * TB;
     uint8_t* vb = kb + KT * KROW;
+    if constexpr (PAGED) {
+#pragma unroll
+      for (int i = 0; i < NLK; ++i) {
+        const int e = tid + NT * i;
+        if (KT * CU % NT == 0 || e < KT * CU) {
+          *reinterpret_cast<u32x4*>(kb + (e / CU) * KROW + (e % CU) * 16) = st[i];
+          *reinterpret_cast<u32x4*>(vb + (e / CU) * VROW + (e % CU) * 16) = st[NLK + i];
+        }
+      }
+      return;
+    }
 #pragma unroll
     for (int i = 0; i < NLD; ++i) {
       const int e = tid + NT * i;
       uint8_t* d;
       if (e < KT * CU) d = kb + (e / CU) * KROW + (e % CU) * 16;
-      else if (e < KT * (CU + CR)) d = kb + ((e - KT * CU) / CR) * KROW + DKU * 2 + ((e - KT * CU) % CR) * 16;
+      else if (e < KT * (CU + CR)) d = kb + ((e - KT * CU) / max(CR, 1)) * KROW + DKU * 2 + ((e - KT * CU) % max(CR, 1)) * 16;
       else d = vb + ((e - KT * (CU + CR)) / CV) * VROW + ((e - KT * (CU + CR)) % CV) * 16;
       if (KT * CPR % NT == 0 || e < KT * CPR) *reinterpret_cast<u32x4*>(d) = st[i];
     }
@@ -116,12 +157,16 @@ __global__ __launch_bounds__(64 * NWV) void latent_prefill_kernel(LP p) {
   for (int i = 0; i < NDB; ++i) o[i] = f32x16{};
   float m = -INFINITY, l = 0.f;
   load_tile(0);
+  load_slots(1);
   store_tile(0);
   __syncthreads();
   const int vq = (lane & 15) >> 2, vp = lane & 3, vhalf = (lane >> 4) & 1;
   for (int t = 0; t < ntile; ++t) {
     const int cur = t & 1, k0 = t * KT;
-    if (t + 1 < ntile) load_tile(t + 1);
+    if (t + 1 < ntile) {
+      load_tile(t + 1);
+      load_slots(t + 2);
+    }
     if (wact && k0 <= wlast) {
       const uint8_t* kb = lds + cur * TB;
       const uint8_t* vb = kb + KT * KROW;
@@ -136,7 +181,7 @@ __global__ __launch_bounds__(64 * NWV) void latent_prefill_kernel(LP p) {
                                                          0, 0);
       }
       float mx = -INFINITY;
-      if (k0 + KT - 1 > pos0 + tw0) {
+      if (k0 + KT - 1 > wfirst) {
 #pragma unroll
         for (int u = 0; u < 2; ++u)
 #pragma unroll
@@ -188,11 +233,10 @@ __global__ __launch_bounds__(64 * NWV) void latent_prefill_kernel(LP p) {
     __syncthreads();
   }
   l += __shfl_xor(l, 32, 64);
-  const int tok = tw0 + tl;
-  if (!wact || tok >= ntok) return;
-  // lane holds O[token][32 db + 8 g + 4 h + 0 .. 3] in o[db][4 g ..]
-  const float f = (l > 0.f ? 1.f / l : 0.f) * p.gate[(size_t)(t0 + tok) * p.ldg + head];
-  __bf16* y = p.out + (size_t)(t0 + tok) * p.ldo + (size_t)head * p.vdim;
+  if (tw0 + tl >= nrow) return;
+  // lane holds O[row][32 db + 8 g + 4 h + 0 .. 3] in o[db][4 g ..]
+  const float f = (l > 0.f ? 1.f / l : 0.f) * p.gate[(size_t)(t0 + mytok) * p.ldg + head];
+  __bf16* y = p.out + (size_t)(t0 + mytok) * p.ldo + (size_t)head * p.vdim;
   const bool vec = (p.vdim & 3) == 0;
 #pragma unroll
   for (int db = 0; db < NDB; ++db)
@@ -213,23 +257,24 @@ __global__ __launch_bounds__(64 * NWV) void latent_prefill_kernel(LP p) {
 }
 
 template <int NKU, int NKR, int NDB, int NWV>
-int launch_t(const LP& p, int nblocks, hipStream_t st) {
+int launch_t(const FP& p, int nblocks, hipStream_t st) {
   constexpr int LDS = 2 * 64 * (32 * (NKU + NKR) * 2 + 16 + 32 * NDB * 2 + (NDB > 1 ? 64 : 0));
   static bool attr = false;
   if (!attr) {
-    if (hipFuncSetAttribute((const void*)latent_prefill_kernel<NKU, NKR, NDB, NWV>,
+    if (hipFuncSetAttribute((const void*)flash_prefill_kernel<NKU, NKR, NDB, NWV>,
                             hipFuncAttributeMaxDynamicSharedMemorySize, LDS) != hipSuccess)
       return -1;
     attr = true;
   }
-  hipLaunchKernelGGL((latent_prefill_kernel<NKU, NKR, NDB, NWV>), dim3(nblocks * p.H), dim3(64 * NWV), LDS, st, p);
+  hipLaunchKernelGGL((flash_prefill_kernel<NKU, NKR, NDB, NWV>), dim3(nblocks * (p.H / p.gs) * p.nsub), dim3(64 * NWV), LDS,
+                     st, p);
   return (int)hipGetLastError();
 }
 
-}  // namespace nls_lpf
+}  // namespace nls_pfa
 
 extern "C" {
-using namespace nls_lpf;
+using namespace nls_pfa;
 
 int nls_expand_plan(const int* spans, int nspans, int maxctx, const int* bt, int bts, int bs, int* xmap, int* actx,
                     void* stream) {
@@ -245,8 +290,8 @@ int nls_latent_prefill(const void* qn, long ldqn, int qns, const void* qr, long 
                        const float* gate, int ldg, void* out, long ldo, int H, int dku, int dr, int dv, int vdim,
                        int waves, float scale, void* stream) {
   if (nblocks < 1 || H < 1 || vdim < 1 || vdim > dv) return -1;
-  LP p{(const __bf16*)qn, (const __bf16*)qr, (const __bf16*)kx, (const __bf16*)vx, (const __bf16*)cache, xmap, blocks,
-       gate, (__bf16*)out, ldqn, ldqr, ldc, ldo, qns, qrs, H, vdim, ldg, scale};
+  FP p{(const __bf16*)qn, (const __bf16*)qr, (const __bf16*)kx, (const __bf16*)vx, (const __bf16*)cache, xmap, blocks,
+       gate, (__bf16*)out, ldqn, ldqr, ldc, ldo, qns, qrs, H, vdim, ldg, 1, 1, scale};
   hipStream_t st = (hipStream_t)stream;
 #define NLS_LP(U, R, V) \
   if (dku == 32 * U && dr == 32 * R && dv == 32 * V) \
@@ -256,6 +301,26 @@ int nls_latent_prefill(const void* qn, long ldqn, int qns, const void* qr, long 
 #undef NLS_LPV
 #undef NLS_LP
   return -1;
+}
+
+// Dp: padded head width (32, 64, 128; 256 with 4 waves); k, v: paged [slots][G][Dp]; blocks of up to 32 * waves tokens
+int nls_gqa_prefill(const void* q, long ldq, const void* k, const void* v, const int* xmap, const int* blocks, int nblocks,
+                    const float* gate, int ldg, void* out, long ldo, int H, int G, int Dp, int waves, float scale,
+                    void* stream) {
+  if (nblocks < 1 || G < 1 || H < 1 || H % G || !gate || (ldq & 7) || (ldo & 3)) return -1;
+  FP p{(const __bf16*)q, (const __bf16*)q, (const __bf16*)k, (const __bf16*)v, nullptr, xmap, blocks, gate, (__bf16*)out, ldq, ldq,
+       (long)G * Dp, ldo, Dp, Dp, H, Dp, ldg, H / G, H / G, scale};
+  hipStream_t st = (hipStream_t)stream;
+  // (nsub = H / G workgroups of 32 * waves rows cover a block of 32 * waves tokens)
+  if (waves == 8 && Dp == 256) {
+    p.nsub *= 2;
+    return launch_t<8, 0, 8, 4>(p, nblocks, st);
+  }
+#define NLS_GP(D, N) \
+  if (Dp == D) return waves == 8 ? launch_t<N, 0, N, 8>(p, nblocks, st) : waves == 4 ? launch_t<N, 0, N, 4>(p, nblocks, st) : -1;
+  NLS_GP(32, 1) NLS_GP(64, 2) NLS_GP(128, 4)
+#undef NLS_GP
+  return Dp == 256 && waves == 4 ? launch_t<8, 0, 8, 4>(p, nblocks, st) : -1;
 }
 
 }  // extern "C"

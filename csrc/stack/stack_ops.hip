@@ -1,6 +1,6 @@
-// Row kernels of the config-driven decoder stacks (models/stack.py): embedding, output norms with the residual add,
-// routed-expert combine, latent-attention row preparation, expert routing. The residual stream is f32; `xb` is its
-// bf16 rounding, the operand of the next projections (f32 launches use the residual itself: xb null).
+// Row kernels of the config-driven decoder stacks (models/stack.py): embedding, norms with the residual add,
+// routed-expert combine, attention and latent-attention row preparation, expert routing. The residual stream is f32; `xb`
+// is its bf16 rounding, the operand of the next projections where sublayers read the residual itself (f32 launches: null).
 #include "../kernels/common.h"
 
 namespace nls_stack {
@@ -27,11 +27,11 @@ DEVI float bsum(float v, float* sh) {
 template <typename T> DEVI float ldv(const T* p, long i) { return (float)p[i]; }
 template <typename T> DEVI void stv(T* p, long i, float v) { p[i] = (T)v; }
 
-// ---- x[t] = table[id], id from the host or (use_prev) the previous step's next_ids
+// ---- x[t] = table[id] * scale, id from the host or (use_prev) the previous step's next_ids
 __global__ __launch_bounds__(256) void embed_kernel(int* __restrict__ ids, const int* __restrict__ next_ids,
                                                     const int* __restrict__ use_prev, const __bf16* __restrict__ tab,
-                                                    int V, int D, float* __restrict__ x, __bf16* __restrict__ xb,
-                                                    long ldx) {
+                                                    int V, int D, float scale, float* __restrict__ x,
+                                                    __bf16* __restrict__ xb, long ldx) {
   const int t = blockIdx.x;
   int id = ids[t];
   if (use_prev && use_prev[t]) id = next_ids[t];
@@ -44,21 +44,29 @@ __global__ __launch_bounds__(256) void embed_kernel(int* __restrict__ ids, const
       const u32x4 v = ld16(row + i);
       const bf16x8 b = __builtin_bit_cast(bf16x8, v);
       float* o = x + (size_t)t * ldx + i;
-      *reinterpret_cast<f32x4*>(o) = f32x4{(float)b[0], (float)b[1], (float)b[2], (float)b[3]};
-      *reinterpret_cast<f32x4*>(o + 4) = f32x4{(float)b[4], (float)b[5], (float)b[6], (float)b[7]};
-      if (xb) *reinterpret_cast<u32x4*>(xb + (size_t)t * ldx + i) = v;
+      const f32x4 lo = f32x4{(float)b[0], (float)b[1], (float)b[2], (float)b[3]} * scale;
+      const f32x4 hi = f32x4{(float)b[4], (float)b[5], (float)b[6], (float)b[7]} * scale;
+      *reinterpret_cast<f32x4*>(o) = lo;
+      *reinterpret_cast<f32x4*>(o + 4) = hi;
+      if (xb)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          xb[(size_t)t * ldx + i + e] = (__bf16)lo[e];
+          xb[(size_t)t * ldx + i + 4 + e] = (__bf16)hi[e];
+        }
     }
     return;
   }
   for (int i = threadIdx.x; i < D; i += 256) {
-    const __bf16 v = row[i];
-    x[(size_t)t * ldx + i] = (float)v;
-    if (xb) xb[(size_t)t * ldx + i] = v;
+    const float v = (float)row[i] * scale;
+    x[(size_t)t * ldx + i] = v;
+    if (xb) xb[(size_t)t * ldx + i] = (__bf16)v;
   }
 }
 
-// ---- x[t] += LayerNorm(y) * w; y = one row, or (topk) sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t], the shared
-// expert); y null: x is only read. Optional second LayerNorm (the model's last norm) of the new x into `on`.
+// ---- x[t] += norm(y) * w (w null: x[t] += y); y = one row, or (topk) sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t],
+// the shared expert); y null: x is only read. Optional second norm (the next sublayers' or the model's last one) of the
+// new x into `on`. norm: (v - mean) / sqrt(var + eps), or (rms) v / sqrt(mean(v^2) + eps).
 // A workgroup per row (`rows`: gathered), 4 consecutive columns x NV per thread in registers.
 struct NormAdd {
   const float* y;
@@ -71,7 +79,7 @@ struct NormAdd {
   const int* rows;      // optional: row i of the launch is row rows[i] of x
   long ldy, ldx, ldo;
   long sh0;             // first shared-expert row, -1: none
-  int D, topk, f32;
+  int D, topk, f32, rms;
   float eps;
 };
 
@@ -110,13 +118,15 @@ DEVI void put4(__bf16* p, int i, int D, const f32x4& v) {
       if (i + e < D) p[i + e] = b[e];
   }
 }
-// (v - mean) / sqrt(var + eps) over the row's D columns
+// the norm over the row's D columns (columns past D hold zeros)
 template <int NV, int NTH>
-DEVI void normalise(f32x4 (&v)[NV], int D, float eps, float* sh) {
-  float s = 0.f;
+DEVI void normalise(f32x4 (&v)[NV], int D, float eps, int rms, float* sh) {
+  float s = 0.f, mean = 0.f;
+  if (!rms) {
 #pragma unroll
-  for (int j = 0; j < NV; ++j) s += (v[j][0] + v[j][1]) + (v[j][2] + v[j][3]);
-  const float mean = bsum<NTH / 64>(s, sh) / (float)D;
+    for (int j = 0; j < NV; ++j) s += (v[j][0] + v[j][1]) + (v[j][2] + v[j][3]);
+    mean = bsum<NTH / 64>(s, sh) / (float)D;
+  }
   s = 0.f;
 #pragma unroll
   for (int j = 0; j < NV; ++j)
@@ -141,7 +151,8 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
   for (int j = 0; j < NV; ++j) x[j] = row4<VEC>(xr, (threadIdx.x + j * NTH) * 4, D);
   if (p.y) {
 #pragma unroll
-    for (int j = 0; j < NV; ++j) w[j] = row4<VEC>(p.w, (threadIdx.x + j * NTH) * 4, D);
+    for (int j = 0; j < NV; ++j)
+      w[j] = p.w ? row4<VEC>(p.w, (threadIdx.x + j * NTH) * 4, D) : f32x4{1.f, 1.f, 1.f, 1.f};
     if (p.topk) {
 #pragma unroll
       for (int j = 0; j < NV; ++j)
@@ -158,7 +169,7 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
 #pragma unroll
       for (int j = 0; j < NV; ++j) v[j] = row4<VEC>(p.y + (size_t)t * p.ldy, (threadIdx.x + j * NTH) * 4, D);
     }
-    normalise<NV, NTH>(v, D, p.eps, sh);
+    if (p.w) normalise<NV, NTH>(v, D, p.eps, p.rms, sh);
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int i = (threadIdx.x + j * NTH) * 4;
@@ -170,7 +181,7 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
   if (!p.ow) return;
 #pragma unroll
   for (int j = 0; j < NV; ++j) w[j] = row4<VEC>(p.ow, (threadIdx.x + j * NTH) * 4, D);
-  normalise<NV, NTH>(x, D, p.eps, sh);
+  normalise<NV, NTH>(x, D, p.eps, p.rms, sh);
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int i = (threadIdx.x + j * NTH) * 4;
@@ -231,6 +242,59 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const float* __restric
     stv(c, Rp + 2 * i, u * f[2 * i] - v * f[2 * i + 1]);
     stv(c, Rp + 2 * i + 1, v * f[2 * i] + u * f[2 * i + 1]);
   }
+}
+
+// ---- attention rows: one workgroup per token. q and k are RMS-normed over all their heads together (norm weights optional),
+// rotated on the first `rot` columns of each head (pairs 2i, 2i + 1) and stored in the activation type, heads Dp columns
+// apart: q to `qo`, k and v (unnormed, unrotated) to the token's rows of the paged caches. The columns past D of a head
+// are never written (zero from the start); slot < 0: no cache row.
+struct AttnRows {
+  const float *q, *k, *v;     // projections, f32
+  const float *qn, *kn;       // norm weights (null: no norm)
+  const float* cs;            // [positions][rot / 2][2]
+  const int *pos, *slot;
+  void *qo, *kc, *vc;
+  long ldq, ldqo, ldc;        // row strides: projections, qo, caches
+  int H, G, D, Dp, rot;
+  float eps;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void attn_rows_kernel(AttnRows p) {
+  __shared__ float sh[4];
+  const int t = blockIdx.x, D = p.D, slot = p.slot[t];
+  const float* f = p.cs + (size_t)p.pos[t] * p.rot;
+  auto norm = [&](const float* a, int n) {
+    float s = 0.f;
+    for (int i = threadIdx.x; i < n; i += 256) s += a[i] * a[i];
+    return 1.f / sqrtf(bsum<4>(s, sh) / (float)n + p.eps);
+  };
+  auto put = [&](const float* a, const float* w, float inv, int heads, T* o) {
+    const int D2 = (D + 1) >> 1;
+    for (int e = threadIdx.x; e < heads * D2; e += 256) {
+      const int h = e / D2, c = 2 * (e - h * D2), i = h * D + c;
+      const bool two = c + 1 < D;
+      float u = a[i], v = two ? a[i + 1] : 0.f;
+      if (w) {
+        u = u * inv * w[i];
+        if (two) v = v * inv * w[i + 1];
+      }
+      if (c < p.rot) {
+        const float cc = f[c], ss = f[c + 1], r = u * cc - v * ss;
+        v = v * cc + u * ss;
+        u = r;
+      }
+      o[(size_t)h * p.Dp + c] = (T)u;
+      if (two) o[(size_t)h * p.Dp + c + 1] = (T)v;
+    }
+  };
+  const float *q = p.q + (size_t)t * p.ldq, *k = p.k + (size_t)t * p.ldq, *v = p.v + (size_t)t * p.ldq;
+  put(q, p.qn, p.qn ? norm(q, p.H * D) : 1.f, p.H, (T*)p.qo + (size_t)t * p.ldqo);
+  const float ik = p.kn ? norm(k, p.G * D) : 1.f;
+  if (slot < 0) return;
+  put(k, p.kn, ik, p.G, (T*)p.kc + (size_t)slot * p.ldc);
+  T* vo = (T*)p.vc + (size_t)slot * p.ldc;
+  for (int e = threadIdx.x; e < p.G * D; e += 256) vo[(size_t)(e / D) * p.Dp + e % D] = (T)v[e];
 }
 
 // ---- expert choice of one token: sigmoid scores, the `keep` groups with the largest sum of their two best scores, the
@@ -400,26 +464,26 @@ __global__ __launch_bounds__(1024) void argmax_kernel(const float* __restrict__ 
 extern "C" {
 using namespace nls_stack;
 
-int nls_stack_embed(int* ids, const int* next_ids, const int* use_prev, const void* tab, int V, int D, float* x,
-                    void* xb, long ldx, int T, void* stream) {
+int nls_stack_embed(int* ids, const int* next_ids, const int* use_prev, const void* tab, int V, int D, float scale,
+                    float* x, void* xb, long ldx, int T, void* stream) {
   if (T < 1 || D < 1 || V < 1) return -1;
   hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, ids, next_ids, use_prev,
-                     (const __bf16*)tab, V, D, x, (__bf16*)xb, ldx);
+                     (const __bf16*)tab, V, D, scale, x, (__bf16*)xb, ldx);
   return (int)hipGetLastError();
 }
 
 int nls_norm_add(const float* y, long ldy, const float* topw, int topk, long sh0, const float* w, float* x, void* xb,
-                 long ldx, const float* ow, void* on, long ldo, int D, int T, float eps, int f32, void* stream) {
-  if (!y || !w) return -1;
-  return norm_add(NormAdd{y, topw, w, x, (__bf16*)xb, ow, on, nullptr, ldy, ldx, ldo, sh0, D, topk, f32, eps}, T,
+                 long ldx, const float* ow, void* on, long ldo, int D, int T, float eps, int f32, int rms, void* stream) {
+  if (!y) return -1;
+  return norm_add(NormAdd{y, topw, w, x, (__bf16*)xb, ow, on, nullptr, ldy, ldx, ldo, sh0, D, topk, f32, rms, eps}, T,
                   (hipStream_t)stream);
 }
 
-// out[i] = LayerNorm(x[rows ? rows[i] : i]) * w
-int nls_layer_norm(const float* x, long ldx, const int* rows, const float* w, void* out, long ldo, int D, int n,
-                   float eps, int f32, void* stream) {
+// out[i] = norm(x[rows ? rows[i] : i]) * w
+int nls_row_norm(const float* x, long ldx, const int* rows, const float* w, void* out, long ldo, int D, int n,
+                 float eps, int f32, int rms, void* stream) {
   return norm_add(NormAdd{nullptr, nullptr, nullptr, const_cast<float*>(x), nullptr, w, out, rows, 0, ldx, ldo, -1, D, 0,
-                          f32, eps}, n, (hipStream_t)stream);
+                          f32, rms, eps}, n, (hipStream_t)stream);
 }
 
 int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq, long ldcq, const float* dkv,
@@ -432,6 +496,18 @@ int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq
   else
     hipLaunchKernelGGL(latent_rows_kernel<__bf16>, dim3(T), dim3(256), 0, (hipStream_t)stream, dq, lddq, Q, wq,
                        (__bf16*)cq, ldcq, dkv, lddkv, R, Rp, rot, wc, cs, pos, slot, (__bf16*)cache, ldc, eps);
+  return (int)hipGetLastError();
+}
+
+// heads of D columns, Dp apart in the outputs; rot even, at most D
+int nls_attn_rows(const float* q, const float* k, const float* v, long ldq, const float* qn, const float* kn, const float* cs,
+                  const int* pos, const int* slot, void* qo, long ldqo, void* kc, void* vc, long ldc, int T, int H, int G,
+                  int D, int Dp, int rot, float eps, int f32, void* stream) {
+  if (T < 1 || H < 1 || G < 1 || D < 1 || Dp < D || (rot & 1) || rot < 0 || rot > D || (long)H * Dp > ldqo || (long)G * Dp > ldc)
+    return -1;
+  AttnRows p{q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, ldq, ldqo, ldc, H, G, D, Dp, rot, eps};
+  if (f32) hipLaunchKernelGGL(attn_rows_kernel<float>, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
+  else hipLaunchKernelGGL(attn_rows_kernel<__bf16>, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
   return (int)hipGetLastError();
 }
 

@@ -65,7 +65,7 @@ def kernel_sources():
 def stack_sources():
     srcs = sorted(glob.glob(os.path.join(CSRC, "stack", "*.hip")))
     hdrs = sorted(glob.glob(os.path.join(CSRC, "stack", "*.h")))
-    return srcs, srcs + hdrs + [os.path.join(CSRC, "kernels", h) for h in ("common.h", "lds_dma.h")]
+    return srcs, srcs + hdrs + [os.path.join(CSRC, "kernels", h) for h in ("common.h", "lds_dma.h", "attn_decode.h")]
 
 
 # no packed FP32 instructions (v_pk_add / mul / fma_f32): hipcc -O3 forms them from ordinary float code, and some of

@@ -1,8 +1,8 @@
 """Decoder stacks assembled from a config: a list of layers, each a mixer plus an optional feed-forward.
 
-A mixer or feed-forward is a class that loads its weights, adds its step buffers, and runs on the rows of a step; the
-per-token cache rows (paged) and the per-sequence states (slots) of all layers belong to the engine, which sees them as
-`kv_cache` / `state_pool`. Everything runs on the HIP kernels of csrc/stack (ops/stack.py): bf16 operands with an f32
+A mixer or feed-forward is a class that loads its weights, adds its step buffers, and runs on the rows of a step; a layer
+class (OutputNormLayer, SharedNormLayer) places the norms and joins the sublayers. The per-token cache rows (paged) and the
+per-sequence states (slots) of all layers belong to the engine, which sees them as `kv_cache` / `state_pool`. Everything runs on the HIP kernels of csrc/stack (ops/stack.py): bf16 operands with an f32
 residual, or `dtype=torch.float32` for 32-bit throughout.
 
 Rows of a step are runs of consecutive tokens of one sequence (whole prompts, portions of any size, single decoded
@@ -46,6 +46,7 @@ class StackBuffers:
     runs: torch.Tensor
     x: torch.Tensor                     # f32 residual
     xb: Optional[torch.Tensor]          # its bf16 rounding (None: 32-bit model, the residual itself is the operand)
+    h: Optional[torch.Tensor]           # normed residual that the sublayers read (None: they read the residual)
     y: torch.Tensor                     # f32 sublayer output
     hn: torch.Tensor                    # normed rows of the head
     logits: torch.Tensor
@@ -55,11 +56,23 @@ class StackBuffers:
 
     @property
     def act(self) -> torch.Tensor:
-        return self.x if self.xb is None else self.xb
+        """What the sublayers read."""
+        return self.h if self.h is not None else self.x if self.xb is None else self.xb
 
 
 class _Part:
-    """A mixer or feed-forward of layer i: weights `w(name)` are '<layer>.<mix|mlp>.<name>'."""
+    """A mixer or feed-forward of layer i: weights `w(name)` are '<layer>.<mix|mlp>.<name>'. Layers that use another's weights
+    (weights_of) share its parts: a part keeps nothing of a sequence, its cache and state come with each run."""
+    cache_width = 0               # cache elements per token
+    plan_bytes = 0                # scratch per context token of a planned prompt run
+    plan_run = None               # runs of at least this many tokens take the planned prompt attention (None: never)
+
+    def state_shapes(self) -> Dict[str, int]:
+        return {}
+
+    def new_cache(self, slots: int):
+        """Cache rows of one layer: [slots, width]."""
+        return torch.zeros(slots, self.cache_width, dtype=self.m.dtype, device=self.m.device)
 
     def __init__(self, model: "StackModel", i: int, cfg, prefix: str):
         self.m, self.i, self.cfg, self.prefix = model, i, cfg, prefix
@@ -132,7 +145,7 @@ class WkvMixer(_Part):
             e["o_proj"].run(T, st)
             return
         K.wkv_scan(e["r"], e["k"], e["v"], e["w"], self.u, e["o"], S, b.x, prev, b.runs, step.nruns, c.heads, c.dim, st)
-        K.wkv_out(e["o"], self.norm, e["g"], e["out"], c.heads, c.dim, T, self.m.cfg.eps, st)
+        K.scan_out(e["o"], self.norm, e["g"], e["out"], c.heads, c.dim, T, self.m.cfg.eps, st)
         e["o_proj"].run(T, st)
 
 
@@ -169,10 +182,16 @@ class LatentMixer(_Part):
         self.uv = self.lin(self.t("uv").to(model.device).view(H, VD, R))                               # [H][VD][R]
         self.g, self.o = self.lin("g", (H, d)), self.lin("o", (d, H * VD))
         self.cs = model.rope(c.rot_base, RD)
+        self.attends = True
+        self.plan_bytes = H * (self.xk + self.xv) * 2 if self.expand else 0
 
     @property
     def cache_width(self) -> int:
         return self.Dp if self.owner else 0
+
+    @property
+    def plan_run(self):
+        return _EXPAND_RUN if self.expand else None
 
     def bind(self, b: StackBuffers) -> dict:
         c, P = self.cfg, b.pad
@@ -205,7 +224,7 @@ class LatentMixer(_Part):
 
     def run(self, b: StackBuffers, e: dict, cache, state, step: "_Step"):
         c, st, T = self.cfg, step.st, step.T
-        rows = cache[self.i if self.owner else c.kv_from]
+        rows = cache[step.layer if self.owner else c.kv_from]
         e["down"].run(T, st)
         K.latent_rows(e["dq"], self.dqn, e["cq"], e["dkv"], self.dkvn if self.owner else None, c.kv_rank, self.Rp,
                       c.rot_dim, self.cs, b.pos, b.slot, rows if self.owner else None, T, self.m.cfg.eps, st)
@@ -279,19 +298,280 @@ class MoeFeedForward(_Part):
         e["down"].run(T, st)
 
 
+class _SharedPart(_Part):
+    """A part of a SharedNormLayer: reads the layer's normed input through segments of the layer's one input launch and leaves
+    its operand of the layer's one output product in `out` (columns of a shared buffer). `scale` weights its output; it goes
+    into a 32-bit factor that the operand is multiplied with anyway, so it costs no rounding."""
+    out_width = 0                 # columns of the operand, a multiple of 64
+
+    def __init__(self, model, i, cfg, prefix, scale: float = 1.0):
+        super().__init__(model, i, cfg, prefix)
+        self.scale = scale
+
+    def mat(self, name: str, shape) -> torch.Tensor:
+        w = self.t(name)
+        if tuple(w.shape) != tuple(shape):
+            raise ValueError(f"{self.prefix}{name}: a weight of shape {tuple(w.shape)}, expected {tuple(shape)}")
+        return w.to(self.m.device)
+
+    def vecn(self, name: str, n: int) -> torch.Tensor:
+        v = self.vec(name)
+        if v.numel() != n:
+            raise ValueError(f"{self.prefix}{name}: {v.numel()} values, expected {n}")
+        return v
+
+    def out_weight(self) -> torch.Tensor:
+        """[width of the model, out_width]: the output projection, zero in the operand's padding columns."""
+        raise NotImplementedError
+
+    def bind(self, b: StackBuffers, out: torch.Tensor) -> dict:
+        """Step buffers and launches; "inputs": the segments of the layer's input launch."""
+        raise NotImplementedError
+
+
+class AttentionPart(_SharedPart):
+    """Grouped-query softmax attention: queries and keys optionally RMS-normed over their whole projections, rotary positions
+    on the first columns of each head, values projected on their own or equal to the projected keys, a sigmoid gate per
+    head. The cache holds the finished keys and the values, [2][slots][kv_heads * padded head]."""
+
+    def __init__(self, model, i, cfg, prefix, scale=1.0):
+        super().__init__(model, i, cfg, prefix, scale)
+        c, d, design = cfg, model.cfg.d_model, model.cfg.design
+        H, G, D = c.heads, c.kv_heads, c.dim
+        self.attends = True
+        self.Dp, self.mfma = K.head_pad(D)
+        self.mfma = self.mfma and not model.f32
+        self.own_values = design.attn_values == "projection"
+        names = [("q", H), ("k", G)] + ([("v", G)] if self.own_values else [])
+        self.qkv = self.lin(torch.cat([self.mat(n, (h * D, d)) for n, h in names]))
+        self.qn = self.kn = None
+        if design.attn_qk_norm == "projection":
+            self.qn, self.kn = self.vecn("q.norm", H * D), self.vecn("k.norm", G * D)
+        self.g = self.lin("g", (H, d))
+        self.cs = model.rope(c.rot_base, c.rot_dims)
+        self.cache_width = 2 * G * self.Dp
+        self.out_width = K.act_ld(H * self.Dp)
+        self.groups = K.attn_groups(H, G)
+
+    @property
+    def plan_run(self):
+        return _FLASH_RUN if self.mfma else None
+
+    def new_cache(self, slots):
+        return torch.zeros(2, slots, self.cfg.kv_heads * self.Dp, dtype=self.m.dtype, device=self.m.device)
+
+    def out_weight(self):
+        c, d = self.cfg, self.m.cfg.d_model
+        w = self.mat("o", (d, c.heads * c.dim)).view(d, c.heads, c.dim)
+        w = torch.nn.functional.pad(w, (0, self.Dp - c.dim)).reshape(d, c.heads * self.Dp)
+        return torch.nn.functional.pad(w, (0, self.out_width - w.shape[1]))
+
+    def bind(self, b, out):
+        c, P, f = self.cfg, b.pad, torch.float32
+        H, G, D = c.heads, c.kv_heads, c.dim
+        qkv = self.scratch(b, "attn.qkv", P, self.qkv.N, f)
+        gate = self.scratch(b, "attn.gate", P, H, f)
+        q = self.scratch(b, f"attn.q{D}", P, H * self.Dp)
+        n = _SPLIT_WG // self.groups + 1                  # rows x splits
+        part = (self.scratch(b, "attn.po", 1, n * H * self.Dp, f), self.scratch(b, "attn.pm", 1, n * H * 2, f),
+                self.scratch(b, "attn.cnt", 1, _SPLIT_WG + self.groups, torch.int32))
+        k0 = H * D
+        return dict(q=q, gate=gate, out=out, part=part, qp=qkv, kp=qkv[:, k0:],
+                    vp=qkv[:, k0 + G * D:] if self.own_values else qkv[:, k0:],
+                    inputs=[K.Seg(self.qkv, b.act, qkv), K.Seg(self.g, b.act, gate, "sigmoid", alpha=self.scale)])
+
+    def run(self, b, e, cache, state, step: "_Step"):
+        c, st, T = self.cfg, step.st, step.T
+        kc, vc = cache[0], cache[1]
+        K.attn_rows(e["qp"], e["kp"], e["vp"], self.qn, self.kn, self.cs, b.pos, b.slot, e["q"], kc, vc, T, c.heads,
+                    c.kv_heads, c.dim, self.Dp, c.rot_dims, self.m.cfg.eps, st)
+        plan = step.plan
+        if plan is None or plan.rest:
+            ns = max(1, min(_SPLIT_CAP, _SPLIT_WG // (T * self.groups))) if self.mfma else 1
+            K.gqa_attention(e["q"], kc, vc, e["gate"], e["out"], e["part"], b.block_tables, step.block_size, b.tok_seq,
+                            b.ctx_len if plan is None else plan.actx, T, c.heads, c.kv_heads, self.Dp, self.mfma, ns,
+                            c.scale, st)
+        if plan is not None:
+            K.gqa_prefill(e["q"], kc, vc, plan.xmap, plan.blocks, plan.nblocks, plan.waves, e["gate"], e["out"], c.heads,
+                          c.kv_heads, self.Dp, c.scale, st)
+
+
+class GlaPart(_SharedPart):
+    """Gated linear attention: a recurrent state per head, decayed per key channel by a low-rank gate, read after each
+    token's update; per-head RMS norm, one weight for all heads, silu gate."""
+
+    def __init__(self, model, i, cfg, prefix, scale=1.0):
+        super().__init__(model, i, cfg, prefix, scale)
+        c, d = cfg, model.cfg.d_model
+        H, D, V = c.heads, c.dim, c.vdim
+        if D > 256:
+            raise ValueError(f"gated linear attention: key width {D} > 256")
+        a1 = self.t("a1").to(model.device)
+        # one buffer [q | k | v | zeros | a1]: the low-rank gate input starts at a linear layer's alignment
+        self.low = K.act_ld(H * (2 * D + V))
+        qkv = torch.cat([self.mat("q", (H * D, d)), self.mat("k", (H * D, d)), self.mat("v", (H * V, d))])
+        self.qkva = self.lin(torch.cat([qkv, qkv.new_zeros(self.low - qkv.shape[0], d), a1]))
+        self.ld = self.low + K.act_ld(a1.shape[0])
+        self.a2, self.a2b = self.lin("a2", (H * D, a1.shape[0])), self.vecn("a2.b", H * D)
+        self.g = self.lin("g", (H * V, d))
+        self.norm = (self.vecn("norm", V) * scale).repeat(H).contiguous()
+        self.out_width = K.act_ld(H * V)
+
+    def state_shapes(self):
+        c = self.cfg
+        return {"S": c.heads * c.dim * c.vdim}
+
+    def out_weight(self):
+        c, d = self.cfg, self.m.cfg.d_model
+        return torch.nn.functional.pad(self.mat("o", (d, c.heads * c.vdim)), (0, self.out_width - c.heads * c.vdim))
+
+    def bind(self, b, out):
+        c, P, f = self.cfg, b.pad, torch.float32
+        HD, HV = c.heads * c.dim, c.heads * c.vdim
+        z = self.scratch(b, "gla.qkva", P, self.ld)
+        a, o = self.scratch(b, "gla.a", P, HD, f), self.scratch(b, "gla.o", P, HV, f)
+        g = self.scratch(b, "gla.g", P, HV)
+        return dict(q=z, k=z[:, HD:], v=z[:, 2 * HD:], a=a, o=o, g=g, out=out,
+                    inputs=[K.Seg(self.qkva, b.act, z), K.Seg(self.g, b.act, g, "silu")],
+                    decay=K.LinLaunch([K.Seg(self.a2, z, a, "sigpow", xcol=self.low, bias=self.a2b, alpha=1.0 / c.tau)]))
+
+    def run(self, b, e, cache, state, step: "_Step"):
+        c, st, T, eps = self.cfg, step.st, step.T, self.m.cfg.eps
+        H, D, V, S, qs = c.heads, c.dim, c.vdim, state["S"], c.dim ** -0.5
+        e["decay"].run(T, st)
+        if T == step.nruns and V % 4 == 0 and V <= 1024:      # single tokens only
+            K.gla_step(e["q"], e["k"], e["v"], e["a"], qs, S, b.runs, T, self.norm, e["g"], e["out"], H, D, V, eps, st)
+            return
+        n = step.nruns
+        shape = K.gla_shape(T, n, H, D, V)
+        seg = None
+        if shape[0] > 1:
+            seg = (self.m.grown(b, "gla.seg", n * (shape[0] - 1), H * D * V, torch.float32),
+                   self.m.grown(b, "gla.segw", n * (shape[0] - 1), H * D, torch.float32))
+        K.gla_scan(e["q"], e["k"], e["v"], e["a"], qs, e["o"], S, b.runs, n, H, D, V, shape, seg, st)
+        K.scan_out(e["o"], self.norm, e["g"], e["out"], H, V, T, eps, st)
+
+
+class DensePart(_SharedPart):
+    """Gated dense feed-forward: down(act(gate h) * (up h)), the activation and product in the input launch's epilogue."""
+    EPI = {"gelu_tanh": "geglu"}
+
+    def __init__(self, model, i, cfg, prefix, scale=1.0):
+        super().__init__(model, i, cfg, prefix, scale)
+        d = model.cfg.d_model
+        if scale != 1.0:
+            raise ValueError("the feed-forward's output is not weighted")
+        gate, up = self.mat("gate", (cfg.ff, d)), self.mat("up", (cfg.ff, d))
+        self.gu = self.lin(torch.stack([gate, up], 1).reshape(2 * cfg.ff, d))        # rows alternate
+        self.out_width = K.act_ld(cfg.ff)
+
+    def out_weight(self):
+        ff = self.cfg.ff
+        return torch.nn.functional.pad(self.mat("down", (self.m.cfg.d_model, ff)), (0, self.out_width - ff))
+
+    def bind(self, b, out):
+        return dict(inputs=[K.Seg(self.gu, b.act, out, self.EPI[self.m.cfg.design.glu_act])])
+
+    def run(self, b, e, cache, state, step):
+        pass
+
+
+class OutputNormLayer:
+    """x <- x + norm1(mixer(x)), then x <- x + norm2(feed-forward(x))."""
+
+    def __init__(self, model: "StackModel", i: int, L):
+        p = f"l{i}."
+        self.m = model
+        self.mix = MIXERS[L.mixer.kind](model, i, L.mixer, p + "mix.")
+        self.mlp = FEED_FORWARDS[L.mlp.kind](model, i, L.mlp, p + "mlp.") if L.mlp is not None else None
+        self.norm1 = model.norm_weight(p + "norm1")
+        self.norm2 = model.norm_weight(p + "norm2") if self.mlp is not None else None
+        self.parts = [self.mix]
+
+    def bind(self, b: StackBuffers, key):
+        b.launches[key, "mix"] = self.mix.bind(b)
+        if self.mlp is not None:
+            b.launches[key, "mlp"] = self.mlp.bind(b)
+
+    def new_caches(self, slots):
+        return self.mix.new_cache(slots) if self.mix.cache_width else None
+
+    def run(self, b, key, kc, state, step: "_Step", fin: dict):
+        cfg, st, T = self.m.cfg, step.st, step.T
+        rms = cfg.design.norm == "rms"
+        self.mix.run(b, b.launches[key, "mix"], kc, state, step)
+        K.norm_add(b.y, self.norm1, b.x, b.xb, T, cfg.eps, st, rms=rms, **(fin if self.mlp is None else {}))
+        if self.mlp is not None:
+            e = b.launches[key, "mlp"]
+            self.mlp.run(b, e, step)
+            K.norm_add(e["ye"], self.norm2, b.x, b.xb, T, cfg.eps, st, plan=e["plan"], shared_row0=e["shared_row0"], rms=rms,
+                       **fin)
+
+
+class SharedNormLayer:
+    """h = norm1(x), x <- x + the sum of the sublayers' outputs on h. The sublayers' input projections are one launch (of up
+    to ops.stack.SEGS segments), their output projections one product over the columns of all their operands; the residual
+    add and the next layer's norm are one launch."""
+
+    def __init__(self, model: "StackModel", i: int, L):
+        p = f"l{i}."
+        self.m = model
+        self.norm1 = model.norm_weight(p + "norm1")
+        self.parts = [PARTS[c.kind](model, i, c, p + "mix." + sub, scale) for c, sub, scale in mixer_parts(L.mixer)]
+        if L.mlp is not None:
+            self.parts.append(PARTS[L.mlp.kind](model, i, L.mlp, p + "mlp."))
+        self.o = K.PackedLinear(torch.cat([q.out_weight() for q in self.parts], 1), model.f32, model.device)
+        model.weight_bytes += self.o.nbytes
+
+    def bind(self, b: StackBuffers, key):
+        widths = [q.out_width for q in self.parts]
+        cat = b.shared.get(("cat", sum(widths)))
+        if cat is None:
+            cat = b.shared["cat", sum(widths)] = torch.zeros(b.pad, sum(widths), dtype=self.m.dtype, device=self.m.device)
+        e, c0, segs = [], 0, []
+        for q, w in zip(self.parts, widths):
+            e.append(q.bind(b, cat[:, c0:c0 + w]))
+            segs += e[-1]["inputs"]
+            c0 += w
+        b.launches[key, "parts"] = e
+        b.launches[key, "in"] = [K.LinLaunch(segs[o:o + K.SEGS]) for o in range(0, len(segs), K.SEGS)]
+        b.launches[key, "out"] = K.LinLaunch([K.Seg(self.o, cat, b.y)])
+
+    def new_caches(self, slots):
+        return {j: q.new_cache(slots) for j, q in enumerate(self.parts) if q.cache_width}
+
+    def run(self, b, key, kc, state, step: "_Step", fin: dict):
+        cfg = self.m.cfg
+        for launch in b.launches[key, "in"]:
+            launch.run(step.T, step.st)
+        for j, (q, e) in enumerate(zip(self.parts, b.launches[key, "parts"])):
+            q.run(b, e, kc[step.layer].get(j), state, step)
+        b.launches[key, "out"].run(step.T, step.st)
+        K.norm_add(b.y, None, b.x, None, step.T, cfg.eps, step.st, rms=cfg.design.norm == "rms", **fin)
+
+
+def mixer_parts(c) -> list:
+    """The parts of a mixer on a shared normed input: (config, tensor prefix, weight of the output)."""
+    if c.kind == "parallel":
+        return [(c.left, "left.", c.left_scale), (c.right, "right.", c.right_scale)]
+    return [(c, "", 1.0)]
+
+
 MIXERS = {"wkv": WkvMixer, "latent_attention": LatentMixer}
 FEED_FORWARDS = {"moe": MoeFeedForward}
+PARTS = {"attention": AttentionPart, "gla": GlaPart, "dense": DensePart}
+LAYERS = {"output": OutputNormLayer, "shared": SharedNormLayer}
 
 
 @dataclass
 class _ExpandPlan:
-    """The runs of a step whose attention expands keys and values: `nx` context rows, query blocks of 32 * waves rows."""
+    """The runs of a step that take the prompt attention: `nx` context rows, query blocks of 32 * waves tokens."""
     nx: int
     xmap: torch.Tensor          # [nx] cache slots of the runs' contexts
     blocks: torch.Tensor        # [nblocks][8]
     nblocks: int
     waves: int
-    rest: bool                  # some rows attend in the latent space
+    rest: bool                  # some rows attend row by row
     actx: Optional[torch.Tensor]
 
 
@@ -302,11 +582,14 @@ class _Step:
     block_size: int
     st: int
     plan: Optional[_ExpandPlan] = None
+    layer: int = 0              # the layer that runs: its cache and state (its parts may be another layer's)
 
 
 # runs of at least this many rows expand (below, the latent-space attention's extra products cost less than the expansion
 # of the context), as long as their contexts fit the scratch
 _EXPAND_RUN = int(os.environ.get("NLS_EXPAND_RUN", "32"))
+# runs of at least this many rows take the flash attention of grouped-query layers
+_FLASH_RUN = int(os.environ.get("NLS_FLASH_RUN", "16"))
 _EXPAND_BYTES = int(os.environ.get("NLS_EXPAND_BYTES", str(4 << 30)))
 
 
@@ -334,24 +617,28 @@ class StackModel:
             cfg.ctx = int(ctx)
         if cfg.d_model > 16384:
             raise ValueError("stack models take widths up to 16384")
-        if max([L.mlp.experts for L in cfg.layers if L.mlp is not None], default=0) > 512:
+        if cfg.n_expert > 512:
             raise ValueError("stack models take up to 512 experts")
         self.weight_bytes = 0
         self._rope = {}
         dev = self.device
-        vec = lambda n: r.tensor(n).to(device=dev, dtype=torch.float32).contiguous()      # noqa: E731
         self.embed = r.tensor("embed").to(device=dev, dtype=torch.bfloat16).contiguous()
         self.weight_bytes += self.embed.numel() * 2
-        self.layers = []
-        for i, L in enumerate(cfg.layers):
-            p = f"l{i}."
-            mix = MIXERS[L.mixer.kind](self, i, L.mixer, p + "mix.")
-            mlp = FEED_FORWARDS[L.mlp.kind](self, i, L.mlp, p + "mlp.") if L.mlp is not None else None
-            self.layers.append((mix, vec(p + "norm1"), mlp, vec(p + "norm2") if mlp is not None else None))
-        self.final_norm = vec("final.norm")
+        # one layer object per set of weights; self.owners: the one each layer runs with
+        self.owners = [i if L.weights_of is None else L.weights_of for i, L in enumerate(cfg.layers)]
+        layer = LAYERS[cfg.design.norm_place]
+        own = {i: layer(self, i, cfg.layers[i]) for i in sorted(set(self.owners))}
+        self.layers = [own[o] for o in self.owners]
+        self.final_norm = self.norm_weight("final.norm")
         self.head = K.PackedLinear(r.tensor("head"), self.f32, dev)
         self.weight_bytes += self.head.nbytes
         self.vocab_lo, self.vocab_hi = 0, cfg.vocab
+
+    def norm_weight(self, name: str) -> torch.Tensor:
+        w = self.reader.tensor(name).to(device=self.device, dtype=torch.float32)
+        if w.numel() != self.cfg.d_model:
+            raise ValueError(f"{name}: {w.numel()} values, expected {self.cfg.d_model}")
+        return (w + 1.0 if self.cfg.design.norm_one else w).contiguous()
 
     # ---- what the engine asks
     @property
@@ -360,10 +647,10 @@ class StackModel:
 
     @property
     def kv_token_bytes(self) -> int:
-        return sum(m.cache_width for m, *_ in self.layers if isinstance(m, LatentMixer)) * self.dtype.itemsize
+        return sum(q.cache_width for L in self.layers for q in L.parts) * self.dtype.itemsize
 
     def n_splits(self, T: int) -> int:
-        return 1                      # (each latent layer sizes its own splits, LatentMixer.run)
+        return 1                      # (each attention layer sizes its own splits)
 
     def rope(self, base: float, dims: int) -> torch.Tensor:
         key = (base, dims)
@@ -372,16 +659,16 @@ class StackModel:
         return self._rope[key]
 
     def kv_cache(self, num_blocks: int, block_size: int = 16):
-        """Paged rows of the layers that own a cache: {layer: [slots, width]}."""
-        return {m.i: torch.zeros(num_blocks * block_size, m.cache_width, dtype=self.dtype, device=self.device)
-                for m, *_ in self.layers if isinstance(m, LatentMixer) and m.owner}, None
+        """Paged rows of the layers that own a cache (a layer that shares another's weights has its own): {layer: rows}."""
+        slots = num_blocks * block_size
+        return {i: c for i, c in ((i, L.new_caches(slots)) for i, L in enumerate(self.layers)) if c is not None}, None
 
     def state_pool(self, slots: int):
         """Per-sequence states, f32: {layer: {name: [slots, n]}}. A sequence's first run (position 0) ignores what its
         slot holds, so a reused slot needs no clearing."""
-        return {m.i: {k: torch.zeros(slots, n, dtype=torch.float32, device=self.device)
-                      for k, n in m.state_shapes().items()}
-                for m, *_ in self.layers if hasattr(m, "state_shapes")}
+        out = {i: {k: torch.zeros(slots, n, dtype=torch.float32, device=self.device)
+                   for q in L.parts for k, n in q.state_shapes().items()} for i, L in enumerate(self.layers)}
+        return {i: d for i, d in out.items() if d}
 
     def step_buffers(self, cap: int, max_seqs: int, max_blocks: int, logit_rows: Optional[int] = None) -> StackBuffers:
         """Step metadata is ONE int32 tensor, as in LlamaModel.step_buffers, with the runs table behind the block tables:
@@ -394,47 +681,48 @@ class StackModel:
         f = dict(dtype=torch.float32, device=dev)
         ld = K.act_ld(cfg.d_model)
         nl = min(pad, max(64, max_seqs, logit_rows or 0))
+        shared = cfg.design.norm_place == "shared"
+        act = lambda: torch.zeros(pad, ld, dtype=self.dtype, device=dev)      # noqa: E731
         b = StackBuffers(
             cap=cap, pad=pad, meta=meta, ids=seg[0], pos=seg[1], slot=seg[2], tok_seq=seg[3], ctx_len=seg[4],
             use_prev=seg[5], block_tables=meta[6 * pad:6 * pad + nb].view(max_seqs, max_blocks),
             runs=meta[6 * pad + nb:].view(max_seqs, 4),
-            x=torch.zeros(pad, ld, **f), xb=None if self.f32 else torch.zeros(pad, ld, dtype=self.dtype, device=dev),
-            y=torch.zeros(pad, cfg.d_model, **f), hn=torch.zeros(pad, ld, dtype=self.dtype, device=dev),
+            x=torch.zeros(pad, ld, **f), xb=None if self.f32 or shared else act(), h=act() if shared else None,
+            y=torch.zeros(pad, cfg.d_model, **f), hn=act(),
             logits=torch.zeros(nl, cfg.vocab, **f), next_ids=torch.zeros(pad, dtype=torch.int32, device=dev))
         b.slot.fill_(-1)
         b.runs[:, 2] = -1
-        for i, (mix, _, mlp, _) in enumerate(self.layers):
-            b.launches[i, "mix"] = mix.bind(b)
-            if mlp is not None:
-                b.launches[i, "mlp"] = mlp.bind(b)
-        b.launches["head"] = K.LinLaunch([K.Seg(self.head, b.hn, b.logits)])
+        for o in sorted(set(self.owners)):
+            self.layers[o].bind(b, o)
+        cap_epi = dict(epi="softcap", alpha=cfg.softcap) if cfg.softcap else {}
+        b.launches["head"] = K.LinLaunch([K.Seg(self.head, b.hn, b.logits, **cap_epi)])
         return b
 
-    # ---- prompt attention: which runs expand their context
+    # ---- prompt attention: which runs take it
     block_width = K.BLOCK_INTS
 
     def row_blocks(self, tok_seq, pos, T: int):
-        """Host side of a row batch's expansion plan, from its staged metadata: (int32 [spans + blocks][8], info), or
-        (None, None) when every row attends in the latent space. Rows of the table: spans (first row, rows, sequence, first
-        position, first expanded row, context, 0, 0), then query blocks (the same, per 32 * waves rows), longest context
+        """Host side of a row batch's prompt attention plan, from its staged metadata: (int32 [spans + blocks][8], info), or
+        (None, None) when every row attends on its own. Rows of the table: spans (first row, rows, sequence, first
+        position, first context row, context, 0, 0), then query blocks (the same, per 32 * waves tokens), longest context
         first."""
-        lat = [m for m, *_ in self.layers if isinstance(m, LatentMixer)]
-        if not lat or not all(m.expand for m in lat):
+        att = [q for L in self.layers for q in L.parts if getattr(q, "attends", False)]
+        if not att or any(q.plan_run is None for q in att):
             return None, None
         ts, ps = np.asarray(tok_seq[:T]), np.asarray(pos[:T])
         cut = np.flatnonzero(ts[1:] != ts[:-1]) + 1
-        width = max(m.cfg.heads * (m.xk + m.xv) for m in lat) * 2
+        width, least = max(q.plan_bytes for q in att), max(q.plan_run for q in att)
         spans, nx, rows = [], 0, 0
         for a, e in zip(np.concatenate([[0], cut]), np.concatenate([cut, [T]])):
             n, p0 = int(e - a), int(ps[a])
-            if n < _EXPAND_RUN or (nx + p0 + n) * width > _EXPAND_BYTES:
+            if n < least or (nx + p0 + n) * width > _EXPAND_BYTES:
                 continue
             spans.append((int(a), n, int(ts[a]), p0, nx, p0 + n, 0, 0))
             nx += p0 + n
             rows += n
         if not spans:
             return None, None
-        H = max(m.cfg.heads for m in lat)
+        H = max(q.cfg.heads for q in att)
         waves = 8 if H * sum(-(-s[1] // 256) for s in spans) >= 256 else 4
         q = 32 * waves
         blocks = [(s[0] + o, min(q, s[1] - o), s[2], s[3] + o, s[4], 0, 0, 0) for s in spans for o in range(0, s[1], q)]
@@ -482,17 +770,20 @@ class StackModel:
         step = _Step(T, T if nruns is None else nruns, block_size, st)
         if row_info is not None and qblocks is not None:
             step.plan = self._expand_plan(b, qblocks, row_info, T, block_size, st)
-        K.embed(b.ids, self.embed, b.x, b.xb, T, st, prev=(b.next_ids, b.use_prev) if feed_prev else None)
+        rms = cfg.design.norm == "rms"
+        K.embed(b.ids, self.embed, b.x, b.xb, T, st, prev=(b.next_ids, b.use_prev) if feed_prev else None,
+                scale=cfg.embed_scale)
+        if b.h is not None:
+            K.row_norm(b.x, None, self.layers[0].norm1, b.h, T, cfg.eps, st, rms=rms)
         last = len(self.layers) - 1
         direct = logit_rows is None
-        for i, (mix, norm1, mlp, norm2) in enumerate(self.layers):
-            fin = dict(out_norm=self.final_norm, out=b.hn) if direct and i == last else {}
-            mix.run(b, b.launches[i, "mix"], kc, state.get(i) if state else None, step)
-            K.norm_add(b.y, norm1, b.x, b.xb, T, cfg.eps, st, **(fin if mlp is None else {}))
-            if mlp is not None:
-                e = b.launches[i, "mlp"]
-                mlp.run(b, e, step)
-                K.norm_add(e["ye"], norm2, b.x, b.xb, T, cfg.eps, st, plan=e["plan"], shared_row0=e["shared_row0"], **fin)
+        for i, layer in enumerate(self.layers):
+            if i == last:
+                fin = dict(out_norm=self.final_norm, out=b.hn) if direct else {}
+            else:
+                fin = dict(out_norm=self.layers[i + 1].norm1, out=b.h) if b.h is not None else {}
+            step.layer = i
+            layer.run(b, self.owners[i], kc, state.get(i) if state else None, step, fin)
             if taps is not None:
                 taps.append(b.x[:T, :cfg.d_model].clone())
         n = T
@@ -500,7 +791,7 @@ class StackModel:
             n = int(n_logits)
             if n == 0:
                 return 0
-            K.layer_norm(b.x, logit_rows, self.final_norm, b.hn, n, cfg.eps, st)
+            K.row_norm(b.x, logit_rows, self.final_norm, b.hn, n, cfg.eps, st, rms=rms)
         if n > b.logits.shape[0]:
             raise ValueError(f"{n} logit rows, buffers hold {b.logits.shape[0]}")
         b.launches["head"].run(n, st)

@@ -1,8 +1,8 @@
 """Configuration of the config-driven decoder stacks: a folder with `config.json` and `model.safetensors`.
 
 config.json names the design (`architecture`), the sizes of the model and, layer by layer, the mixer and the
-feed-forward. What a design fixes for all of its models (where the norms sit, the norm's kind, the expert activation,
-how the router scores) is its `Design` entry here; a mechanism takes those constants as parameters."""
+feed-forward. What a design fixes for all of its models (where the norms sit, the norm's kind, activations, how the router
+scores) is its `Design` entry here; a mechanism takes those constants as parameters."""
 from __future__ import annotations
 
 import json
@@ -19,17 +19,23 @@ def default_ctx() -> int:
 @dataclass(frozen=True)
 class Design:
     """What every model of a design has in common."""
-    norm: str = "layer"                # layer: (x - mean) / sqrt(var + eps) * w
+    norm: str = "layer"                # layer: (x - mean) / sqrt(var + eps) * w; rms: x / rms(x) * w
+    norm_one: bool = False             # the norm's weights are stored around zero: factor 1 + w
     norm_place: str = "output"         # output: x + norm(sublayer(x)), the sublayers read x itself
+                                       # shared: h = norm(x), x + mixer(h) + feed-forward(h)
     mixers: tuple = ()
     feed_forwards: tuple = ()
     rotary: str = "interleaved"        # pairs (2i, 2i + 1)
     expert_act: str = "relu2"
     router_score: str = "sigmoid"
+    glu_act: str = "gelu_tanh"         # dense feed-forward: down(act(gate) * up)
+    attn_qk_norm: str = "projection"   # attention: one RMS norm over all heads of the queries, one over the keys'
+    attn_values: str = "keys"          # attention: the values are the projected keys, unnormed and unrotated
 
 
 DESIGNS = {
     "Sekolorn": Design(mixers=("wkv", "latent_attention"), feed_forwards=("moe",)),
+    "Kolodra": Design(norm="rms", norm_one=True, norm_place="shared", mixers=("parallel",), feed_forwards=("dense",)),
 }
 
 
@@ -37,7 +43,7 @@ DESIGNS = {
 class WkvConfig:
     heads: int
     dim: int
-    kind = "wkv"
+    kind, recurrent = "wkv", True
 
 
 @dataclass
@@ -51,7 +57,39 @@ class LatentConfig:
     rot_base: float
     scale: float
     kv_from: Optional[int] = None
-    kind = "latent_attention"
+    kind, recurrent = "latent_attention", False
+
+
+@dataclass
+class AttentionConfig:
+    """Grouped-query softmax attention with partial rotary positions and a gate per head."""
+    heads: int
+    kv_heads: int
+    dim: int                           # of queries, keys and values
+    rot_dims: int
+    rot_base: float
+    scale: float
+    kind, recurrent = "attention", False
+
+
+@dataclass
+class GlaConfig:
+    """Gated linear attention: a state [dim, vdim] per head, decayed per key channel by sigmoid(.)^(1 / tau)."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    kind, recurrent = "gla", True
+
+
+@dataclass
+class ParallelConfig:
+    """Two mixers on the same input, their outputs weighted and added."""
+    left: AttentionConfig
+    right: GlaConfig
+    left_scale: float
+    right_scale: float
+    kind, recurrent = "parallel", True
 
 
 @dataclass
@@ -67,9 +105,17 @@ class MoeConfig:
 
 
 @dataclass
+class DenseConfig:
+    ff: int
+    kind = "dense"
+    experts = top = 0
+
+
+@dataclass
 class LayerConfig:
     mixer: object
-    mlp: Optional[MoeConfig] = None
+    mlp: object = None                 # MoeConfig, DenseConfig or None
+    weights_of: Optional[int] = None   # the layer whose tensors this one uses (resolved: never itself such a layer)
 
 
 @dataclass
@@ -81,6 +127,8 @@ class StackConfig:
     eps: float
     layers: List[LayerConfig] = field(default_factory=list)
     ctx: int = 32768
+    embed_scale: float = 1.0
+    softcap: float = 0.0               # logits: softcap * tanh(logits / softcap); 0: none
 
     @property
     def n_layer(self) -> int:
@@ -97,7 +145,7 @@ class StackConfig:
     @property
     def recurrent(self) -> bool:
         """Some layer carries per-sequence state besides the paged cache."""
-        return any(L.mixer.kind == "wkv" for L in self.layers)
+        return any(L.mixer.recurrent for L in self.layers)
 
     @classmethod
     def from_json(cls, cfg: dict, shape=None) -> "StackConfig":
@@ -118,55 +166,112 @@ class StackConfig:
 
         norm = cfg.get("norm") or {}
         out = cls(arch=arch, design=design, d_model=size(cfg, "width", "embed", 1), vocab=size(cfg, "vocab", "embed"),
-                  eps=float(norm["eps"]), ctx=default_ctx())
+                  eps=float(norm["eps"]), ctx=default_ctx(),
+                  embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
+                  softcap=float(cfg.get("logit_softcap") or 0.0))
+
+        def wkv(i, m, p):
+            u = shape(p + "u")
+            return WkvConfig(int(m["heads"]) if "heads" in m else int(u[0]), int(m["dim"]) if "dim" in m else int(u[1]))
+
+        def latent(i, m, p):
+            H = int(m["heads"]) if "heads" in m else int(shape(p + "g")[0])
+            rd = int(m["rot_dim"]) if "rot_dim" in m else int(m["rot"]["dims"])
+            src = m.get("kv_from")
+            mix = LatentConfig(
+                heads=H, rot_dim=rd, dim=size(m, "dim", p + "uk", 0, H), vdim=size(m, "vdim", p + "uv", 0, H),
+                kv_rank=size(m, "kv_rank", p + "uk", 1), q_rank=size(m, "q_rank", p + "dq"),
+                rot_base=float(m["rot"]["base"]), scale=float(m["scale"]), kv_from=None if src is None else int(src))
+            if rd % 2 or int(m["rot"].get("dims", rd)) != rd:
+                raise ValueError(f"layer {i}: the rotation covers the whole rotated part: rot.dims = rot_dim, even")
+            if mix.kv_from is not None:
+                if not 0 <= mix.kv_from < i:
+                    raise ValueError(f"layer {i}: kv_from {mix.kv_from} is not an earlier layer")
+                o = out.layers[mix.kv_from].mixer
+                if o.kind != "latent_attention" or o.kv_from is not None or (o.kv_rank, o.rot_dim, o.rot_base) != (
+                        mix.kv_rank, mix.rot_dim, mix.rot_base):
+                    raise ValueError(f"layer {i}: kv_from {mix.kv_from} has no matching latent cache of its own")
+            return mix
+
+        def attention(i, m, p):
+            H = size(m, "heads", p + "g")
+            D = size(m, "dim", p + "q", 0, H)
+            G = size(m, "kv_heads", p + "k", 0, D)
+            rot = m.get("rot") or {"dims": 0, "base": 1.0}
+            rd = int(rot.get("dims", D))
+            if H % G:
+                raise ValueError(f"layer {i}: {H} query heads do not divide into {G} key heads")
+            if int(m.get("vdim", D)) != D:
+                raise ValueError(f"layer {i}: the values are the keys: vdim {m['vdim']} must be dim {D}")
+            if rd % 2 or not 0 <= rd <= D:
+                raise ValueError(f"layer {i}: {rd} rotated dimensions of heads of {D}")
+            return AttentionConfig(heads=H, kv_heads=G, dim=D, rot_dims=rd, rot_base=float(rot["base"]), scale=float(m["scale"]))
+
+        def gla(i, m, p):
+            V = size(m, "vdim", p + "norm")
+            H = size(m, "heads", p + "v", 0, V)
+            return GlaConfig(heads=H, dim=size(m, "dim", p + "k", 0, H), vdim=V, tau=float(m["tau"]))
+
+        def parallel(i, m, p):
+            return ParallelConfig(left=attention(i, m["left"], p + "left."), right=gla(i, m["right"], p + "right."),
+                                  left_scale=float(m["left_scale"]), right_scale=float(m["right_scale"]))
+
+        def moe(i, f, p):
+            r = f["router"]
+            g = r.get("groups") or {}
+            E = size(r, "experts", p + "router")
+            mlp = MoeConfig(experts=E, top=int(r["top"]), ff=size(f.get("expert") or {}, "ff", p + "e0.up"),
+                            scale=float(r.get("scale", 1.0)), groups=int(g.get("count", 1)),
+                            keep=int(g.get("keep", g.get("count", 1))))
+            if f.get("shared") is not None:
+                mlp.shared_ff = size(f["shared"], "ff", p + "shared.up")
+            if E % mlp.groups or not 1 <= mlp.keep <= mlp.groups or not 1 <= mlp.top <= mlp.keep * (E // mlp.groups):
+                raise ValueError(f"layer {i}: {E} experts in {mlp.groups} groups, {mlp.keep} kept, cannot give "
+                                 f"{mlp.top} experts")
+            return mlp
+
+        def dense(i, f, p):
+            return DenseConfig(ff=size(f, "ff", p + "gate"))
+
+        mixers = {"wkv": wkv, "latent_attention": latent, "parallel": parallel}
+        feed_forwards = {"moe": moe, "dense": dense}
+        owners = weight_owners(cfg["layers"])
         for i, L in enumerate(cfg["layers"]):
-            t, m, p = L["type"], L["mixer"], f"l{i}."
+            t, p = L["type"], f"l{owners[i]}."
             if t not in design.mixers:
                 raise NotImplementedError(f"{arch}: layer {i}: mixer {t!r} not supported {design.mixers}")
-            if t == "wkv":
-                u = shape(p + "mix.u")
-                mix = WkvConfig(int(m["heads"]) if "heads" in m else int(u[0]),
-                                int(m["dim"]) if "dim" in m else int(u[1]))
-            else:
-                H = int(m["heads"]) if "heads" in m else int(shape(p + "mix.g")[0])
-                rd = int(m["rot_dim"]) if "rot_dim" in m else int(m["rot"]["dims"])
-                src = m.get("kv_from")
-                mix = LatentConfig(
-                    heads=H, rot_dim=rd, dim=size(m, "dim", p + "mix.uk", 0, H), vdim=size(m, "vdim", p + "mix.uv", 0, H),
-                    kv_rank=size(m, "kv_rank", p + "mix.uk", 1), q_rank=size(m, "q_rank", p + "mix.dq"),
-                    rot_base=float(m["rot"]["base"]), scale=float(m["scale"]), kv_from=None if src is None else int(src))
-                if rd % 2 or int(m["rot"].get("dims", rd)) != rd:
-                    raise ValueError(f"layer {i}: the rotation covers the whole rotated part: rot.dims = rot_dim, even")
-                if mix.kv_from is not None:
-                    if not 0 <= mix.kv_from < i:
-                        raise ValueError(f"layer {i}: kv_from {mix.kv_from} is not an earlier layer")
-                    o = out.layers[mix.kv_from].mixer
-                    if o.kind != t or o.kv_from is not None or (o.kv_rank, o.rot_dim, o.rot_base) != (
-                            mix.kv_rank, mix.rot_dim, mix.rot_base):
-                        raise ValueError(f"layer {i}: kv_from {mix.kv_from} has no matching latent cache of its own")
-            mlp = None
-            if L.get("mlp") is not None:
-                f = L["mlp"]
-                if f.get("kind", "moe") not in design.feed_forwards:
-                    raise NotImplementedError(f"{arch}: layer {i}: feed-forward {f.get('kind')!r} not supported")
-                r = f["router"]
-                g = r.get("groups") or {}
-                E = size(r, "experts", p + "mlp.router")
-                mlp = MoeConfig(experts=E, top=int(r["top"]), ff=size(f.get("expert") or {}, "ff", p + "mlp.e0.up"),
-                                scale=float(r.get("scale", 1.0)), groups=int(g.get("count", 1)),
-                                keep=int(g.get("keep", g.get("count", 1))))
-                if f.get("shared") is not None:
-                    mlp.shared_ff = size(f["shared"], "ff", p + "mlp.shared.up")
-                if E % mlp.groups or not 1 <= mlp.keep <= mlp.groups or not 1 <= mlp.top <= mlp.keep * (E // mlp.groups):
-                    raise ValueError(f"layer {i}: {E} experts in {mlp.groups} groups, {mlp.keep} kept, cannot give "
-                                     f"{mlp.top} experts")
-            out.layers.append(LayerConfig(mix, mlp))
+            layer = LayerConfig(mixers[t](i, L["mixer"], p + "mix."), weights_of=None if owners[i] == i else owners[i])
+            f = L.get("mlp")
+            if f is not None:
+                kind = f.get("kind", design.feed_forwards[0])
+                if kind not in design.feed_forwards:
+                    raise NotImplementedError(f"{arch}: layer {i}: feed-forward {kind!r} not supported")
+                layer.mlp = feed_forwards[kind](i, f, p + "mlp.")
+            out.layers.append(layer)
+        for i, L in enumerate(out.layers):
+            o = out.layers[owners[i]]
+            if L.mixer != o.mixer or L.mlp != o.mlp:
+                raise ValueError(f"layer {i}: its entry is not that of layer {owners[i]}, whose weights it uses")
         return out
 
     @classmethod
     def from_dir(cls, path: str, shape=None) -> "StackConfig":
         with open(os.path.join(path, "config.json")) as f:
             return cls.from_json(json.load(f), shape)
+
+
+def weight_owners(layers: List[dict]) -> List[int]:
+    """The layer that holds each layer's tensors (`weights_of`, possibly over several layers)."""
+    out = []
+    for i in range(len(layers)):
+        j, seen = i, {i}
+        while layers[j].get("weights_of") is not None:
+            j = int(layers[j]["weights_of"])
+            if not 0 <= j < len(layers) or j in seen:
+                raise ValueError(f"layer {i}: weights_of {j} names no layer with tensors")
+            seen.add(j)
+        out.append(j)
+    return out
 
 
 def is_stack_dir(path: str) -> bool:

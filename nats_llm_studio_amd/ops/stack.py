@@ -15,7 +15,8 @@ LIB_PATH = os.environ.get("NLS_STACK_SO") or os.path.join(_PKG, "_stack.so")
 
 P, I, L, F = ctypes.c_void_p, ctypes.c_int, ctypes.c_long, ctypes.c_float
 SEGS = 6
-EPI = {"none": 0, "silu": 1, "tanh": 2, "sigmoid": 3, "relu2": 4, "decay": 5, "gate": 6, "rope": 7}
+EPI = {"none": 0, "silu": 1, "tanh": 2, "sigmoid": 3, "relu2": 4, "decay": 5, "gate": 6, "rope": 7,
+       "geglu": 8, "sigpow": 9, "softcap": 10}
 NO_BLOCK = 1 << 30       # LinSeg.cb: output columns are not blocked
 
 
@@ -24,7 +25,7 @@ class LinSeg(ctypes.Structure):
     _fields_ = [("w", P), ("x", P), ("y", P), ("bias", P), ("gate", P), ("cs", P), ("pos", P), ("rows", P), ("xmap", P),
                 ("wstride", L), ("ldx", L), ("ldy", L), ("xgs", L), ("ygs", L),
                 ("N", I), ("nsub", I), ("M", I), ("ng", I), ("epi", I), ("yact", I), ("cb", I), ("cstep", I),
-                ("xdiv", I), ("ldg", I), ("half", I), ("pad0", I)]
+                ("xdiv", I), ("ldg", I), ("half", I), ("alpha", F)]
 
 
 class LinArgs(ctypes.Structure):
@@ -36,15 +37,20 @@ _SIGS = {
     "nls_lin_args_size": [],
     "nls_lin_small": [P, I, I, I, I, P],
     "nls_lin_gemm": [P, I, I, P],
-    "nls_stack_embed": [P, P, P, P, I, I, P, P, L, I, P],
-    "nls_norm_add": [P, L, P, I, L, P, P, P, L, P, P, L, I, I, F, I, P],
-    "nls_layer_norm": [P, L, P, P, P, L, I, I, F, I, P],
+    "nls_stack_embed": [P, P, P, P, I, I, F, P, P, L, I, P],
+    "nls_norm_add": [P, L, P, I, L, P, P, P, L, P, P, L, I, I, F, I, I, P],
+    "nls_row_norm": [P, L, P, P, P, L, I, I, F, I, I, P],
+    "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, F, I, P],
+    "nls_gqa_attn": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, P, L, P, L, P, P, P, I, I, P],
+    "nls_gqa_prefill": [P, L, P, P, P, P, I, P, I, P, L, I, I, I, I, F, P],
+    "nls_gla_scan": [P, P, P, L, P, L, F, P, L, P, L, P, I, I, I, I, I, P, P, I, I, I, P],
+    "nls_gla_step": [P, P, P, L, P, L, F, P, L, P, I, P, P, L, P, L, I, I, I, F, I, P],
     "nls_latent_rows": [P, L, I, P, P, L, P, L, I, I, I, P, P, P, P, P, L, I, F, I, P],
     "nls_stack_argmax": [P, L, I, P, I, P],
     "nls_moe_plan": [P, L, I, I, I, I, I, F, P, P, I, P, P, P, I, P],
     "nls_shift_mix": [P, L, P, P, L, P, L, L, P, P, I, I, I, P],
     "nls_wkv_scan": [P, P, P, L, P, L, P, P, L, P, L, P, L, P, L, I, P, I, I, I, I, P],
-    "nls_wkv_out": [P, L, P, P, L, P, L, I, I, I, F, I, P],
+    "nls_scan_out": [P, L, P, P, L, P, L, I, I, I, F, I, P],
     "nls_wkv_step": [P, P, P, L, P, L, P, P, L, P, L, P, L, I, P, I, P, P, L, P, L, I, I, F, I, P],
     "nls_expand_plan": [P, I, I, P, I, I, P, P, P],
     "nls_latent_prefill": [P, L, I, P, L, I, P, P, P, L, P, P, I, P, I, P, L, I, I, I, I, I, I, F, P],
@@ -126,11 +132,12 @@ class Seg:
     """One segment of a LinLaunch. y / x: 2-D buffers (row stride = their stride(0)); ycol / xcol: first column.
     xgs / ygs: column step per group. block = (cb, cstep): output column n -> (n / cb) * cstep + n % cb.
     routed = (entry list, xdiv): the rows are routed entries (x row = entry / xdiv, y row = entry).
-    rope = (table, pos, pairs)."""
+    rope = (table, pos, pairs). alpha: constant of the epilogue (sigmoid, sigpow, softcap). geglu: the rows of w alternate
+    gate and up, y has half as many columns."""
 
     def __init__(self, w: PackedLinear, x: torch.Tensor, y: torch.Tensor, epi: str = "none", ycol: int = 0,
                  xcol: int = 0, xgs: int = 0, ygs: int = 0, block=None, bias=None, gate=None, routed=None, rope=None,
-                 yrow: int = 0, xmap: Optional[torch.Tensor] = None):
+                 yrow: int = 0, xmap: Optional[torch.Tensor] = None, alpha: float = 1.0):
         if x.stride(1) != 1 or y.stride(1) != 1:
             raise ValueError("row-major operands")
         if xcol + (0 if routed else (w.groups - 1) * xgs) + act_ld(w.K) > x.stride(0):
@@ -159,6 +166,7 @@ class Seg:
         if rope:
             s.cs, s.pos, s.half = rope[0].data_ptr(), rope[1].data_ptr(), rope[2]
         s.xmap = _p(xmap)
+        s.alpha = alpha
         self.keep = (bias, gate, routed, rope, xmap)
 
 
@@ -280,27 +288,31 @@ class MoePlan:
 # Row kernels
 # ---------------------------------------------------------------------------
 
-def embed(ids, table: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor], T: int, st: int, prev=None):
+def embed(ids, table: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor], T: int, st: int, prev=None,
+          scale: float = 1.0):
     nx, up = prev if prev is not None else (None, None)
-    _check(lib().nls_stack_embed(ids.data_ptr(), _p(nx), _p(up), table.data_ptr(), table.shape[0], table.shape[1],
+    _check(lib().nls_stack_embed(ids.data_ptr(), _p(nx), _p(up), table.data_ptr(), table.shape[0], table.shape[1], scale,
                                  x.data_ptr(), _p(xb), x.stride(0), T, st), "nls_stack_embed")
 
 
-def norm_add(y: torch.Tensor, w: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor], T: int, eps: float, st: int,
-             plan: Optional[MoePlan] = None, shared_row0: int = -1, out_norm: Optional[torch.Tensor] = None,
-             out: Optional[torch.Tensor] = None):
-    """x[:T] += LayerNorm(y) * w (xb: its bf16 rounding). With `plan`, y holds the routed experts' rows (token-major) and
-    from row `shared_row0` on the shared expert's, combined first. out = LayerNorm(x) * out_norm (the model's last norm)."""
+def norm_add(y: torch.Tensor, w: Optional[torch.Tensor], x: torch.Tensor, xb: Optional[torch.Tensor], T: int, eps: float,
+             st: int, plan: Optional[MoePlan] = None, shared_row0: int = -1, out_norm: Optional[torch.Tensor] = None,
+             out: Optional[torch.Tensor] = None, rms: bool = False):
+    """x[:T] += norm(y) * w, or += y without w (xb: its bf16 rounding). With `plan`, y holds the routed experts' rows
+    (token-major) and from row `shared_row0` on the shared expert's, combined first. out = norm(x) * out_norm (what the next
+    sublayers read, or the model's last norm). norm: layer norm, or RMS."""
+    D = y.shape[1] if w is None else w.numel()
     _check(lib().nls_norm_add(y.data_ptr(), y.stride(0), _p(plan.topw) if plan else None, plan.top if plan else 0,
-                              shared_row0, w.data_ptr(), x.data_ptr(), _p(xb), x.stride(0), _p(out_norm), _p(out),
-                              out.stride(0) if out is not None else 0, w.numel(), T, eps,
-                              int(out is not None and out.dtype == torch.float32), st), "nls_norm_add")
+                              shared_row0, _p(w), x.data_ptr(), _p(xb), x.stride(0), _p(out_norm), _p(out),
+                              out.stride(0) if out is not None else 0, D, T, eps,
+                              int(out is not None and out.dtype == torch.float32), int(rms), st), "nls_norm_add")
 
 
-def layer_norm(x: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor, out: torch.Tensor, n: int, eps: float,
-               st: int):
-    _check(lib().nls_layer_norm(x.data_ptr(), x.stride(0), _p(rows), w.data_ptr(), out.data_ptr(), out.stride(0),
-                                w.numel(), n, eps, int(out.dtype == torch.float32), st), "nls_layer_norm")
+def row_norm(x: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor, out: torch.Tensor, n: int, eps: float,
+             st: int, rms: bool = False):
+    """out[i] = norm(x[rows[i]]) * w (rows None: row i): layer norm, or RMS."""
+    _check(lib().nls_row_norm(x.data_ptr(), x.stride(0), _p(rows), w.data_ptr(), out.data_ptr(), out.stride(0),
+                              w.numel(), n, eps, int(out.dtype == torch.float32), int(rms), st), "nls_row_norm")
 
 
 def argmax(logits: torch.Tensor, n: int, out: torch.Tensor, st: int):
@@ -395,6 +407,90 @@ def wkv_step(r, k, v, w, u, state, x, prev, runs, nruns: int, norm, gate, out, H
                               st), "nls_wkv_step")
 
 
-def wkv_out(o, norm, gate, out, H: int, D: int, T: int, eps: float, st: int):
-    _check(lib().nls_wkv_out(o.data_ptr(), o.stride(0), norm.data_ptr(), gate.data_ptr(), gate.stride(0), out.data_ptr(),
-                             out.stride(0), H, D, T, eps, int(out.dtype == torch.float32), st), "nls_wkv_out")
+def scan_out(o, norm, gate, out, H: int, D: int, T: int, eps: float, st: int):
+    """out = (o / rms(o) per head of D columns) * norm * gate."""
+    _check(lib().nls_scan_out(o.data_ptr(), o.stride(0), norm.data_ptr(), gate.data_ptr(), gate.stride(0), out.data_ptr(),
+                              out.stride(0), H, D, T, eps, int(out.dtype == torch.float32), st), "nls_scan_out")
+
+
+def gla_shape(T: int, nruns: int, H: int, D: int, V: int):
+    """(segments, lanes per column, columns per lane) of a gla_scan launch: enough workgroups for the chip, segments of at
+    least 128 tokens."""
+    parts = 8 if D <= 64 else 16
+    longest = T - nruns + 1
+    for cpl in (4, 1):
+        wc = 256 // parts * cpl
+        wgs = H * -(-V // wc) * nruns
+        nseg = max(1, min(-(-512 // wgs), longest // 128, 16))
+        if wgs * nseg >= 256 or cpl == 1:
+            return nseg, parts, cpl
+
+
+def gla_scan(q, k, v, a, qscale: float, o, state, runs, nruns: int, H: int, D: int, V: int, shape, seg, st: int):
+    """Gated linear attention over each run's tokens: q, k [rows, H * D], v [rows, H * V] of one buffer (equal strides), decays
+    a; state [slots, H * D * V] is carried on. shape: gla_shape; seg: (end states, decay products) scratch of its segments."""
+    nseg, parts, cpl = shape
+    if nseg > 1 and (seg[0].numel() < nruns * (nseg - 1) * H * D * V or seg[1].numel() < nruns * (nseg - 1) * H * D):
+        raise ValueError("gla_scan: segment scratch too small")
+    s0, s1 = seg if nseg > 1 else (None, None)
+    _check(lib().nls_gla_scan(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), a.data_ptr(), a.stride(0), qscale,
+                              o.data_ptr(), o.stride(0), state.data_ptr(), state.stride(0), runs.data_ptr(), nruns, H, D, V,
+                              nseg, _p(s0), _p(s1), parts, cpl, int(q.dtype == torch.float32), st), "nls_gla_scan")
+
+
+def gla_step(q, k, v, a, qscale: float, state, runs, nruns: int, norm, gate, out, H: int, D: int, V: int, eps: float, st: int):
+    """gla_scan and scan_out of runs of one token each (V a multiple of 4)."""
+    _check(lib().nls_gla_step(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), a.data_ptr(), a.stride(0), qscale,
+                              state.data_ptr(), state.stride(0), runs.data_ptr(), nruns, norm.data_ptr(), gate.data_ptr(),
+                              gate.stride(0), out.data_ptr(), out.stride(0), H, D, V, eps, int(out.dtype == torch.float32),
+                              st), "nls_gla_step")
+
+
+# ---------------------------------------------------------------------------
+# Grouped-query attention
+# ---------------------------------------------------------------------------
+
+HEAD_WIDTHS = (32, 64, 128, 256)      # padded head widths of the MFMA attention kernels
+
+
+def head_pad(D: int):
+    """(padded head width, MFMA kernels): other widths run on the plain kernel, padded for its 16-byte loads."""
+    for w in HEAD_WIDTHS:
+        if D <= w:
+            return w, True
+    if D > 1024:
+        raise ValueError(f"attention head width {D} > 1024")
+    return pad_to(D, 32), False
+
+
+def attn_groups(H: int, G: int) -> int:
+    """Workgroups a (token, split) of gqa_attention takes."""
+    return G * -(-(H // G) // 16)
+
+
+def attn_rows(q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, T: int, H: int, G: int, D: int, Dp: int, rot: int, eps: float, st: int):
+    """Norm over the whole q and k projections (qn, kn: weights or None), rotation of the first `rot` columns of each head,
+    queries to qo, keys and (as projected) values to the tokens' cache rows. q, k, v: f32 with one row stride."""
+    _check(lib().nls_attn_rows(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), _p(qn), _p(kn), cs.data_ptr(),
+                               pos.data_ptr(), slot.data_ptr(), qo.data_ptr(), qo.stride(0), kc.data_ptr(), vc.data_ptr(),
+                               kc.stride(0), T, H, G, D, Dp, rot, eps, int(qo.dtype == torch.float32), st), "nls_attn_rows")
+
+
+def gqa_attention(q, kc, vc, gate, out, part, block_tables, block_size: int, tok_seq, ctx_len, T: int, H: int, G: int, Dp: int,
+                  mfma: bool, ns: int, scale: float, st: int):
+    """Row-by-row attention (decoded tokens, short runs); the head gate is applied to the output. part: (partial outputs,
+    (max, sum) pairs, ticket counters) of `ns` splits."""
+    po, pm, cnt = part
+    if ns > 1 and (po.numel() < T * H * ns * Dp or pm.numel() < T * H * ns * 2 or cnt.numel() < T * attn_groups(H, G)):
+        raise ValueError("gqa_attention: split workspace too small")
+    _check(lib().nls_gqa_attn(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), block_tables.data_ptr(),
+                              block_tables.stride(0), block_size, tok_seq.data_ptr(), ctx_len.data_ptr(), T, H, G, Dp, ns,
+                              scale, gate.data_ptr(), gate.stride(0), out.data_ptr(), out.stride(0), po.data_ptr(),
+                              pm.data_ptr(), cnt.data_ptr(), int(not mfma), int(q.dtype == torch.float32), st), "nls_gqa_attn")
+
+
+def gqa_prefill(q, kc, vc, xmap, blocks, nblocks: int, waves: int, gate, out, H: int, G: int, Dp: int, scale: float, st: int):
+    """Causal attention of query blocks over their sequences' paged keys and values."""
+    _check(lib().nls_gqa_prefill(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), xmap.data_ptr(), blocks.data_ptr(),
+                                 nblocks, gate.data_ptr(), gate.stride(0), out.data_ptr(), out.stride(0), H, G, Dp, waves,
+                                 scale, st), "nls_gqa_prefill")

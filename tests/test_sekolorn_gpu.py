@@ -140,7 +140,7 @@ def test_norm_add(K, D):
     assert relerr(on[:, :D], O.layer_norm(want, ow, eps)) < 5e-3
     assert (xd[:, D:] == 0).all() and (xb[:, D:] == 0).all() and (on[:, D:] == 0).all()
     rows = torch.tensor([3, 0], dtype=torch.int32, device="cuda")
-    K.layer_norm(xd, rows, ow.float().cuda(), on, 2, eps, st())
+    K.row_norm(xd, rows, ow.float().cuda(), on, 2, eps, st())
     assert relerr(on[:2, :D], O.layer_norm(want[[3, 0]], ow, eps)) < 5e-3
 
 
@@ -180,7 +180,7 @@ def test_moe_layer(K, tmp_path, dt, name, i, T):
     b = m.step_buffers(T, 1, 16)
     x = rnd(T, cfg["width"], seed=T).to(torch.bfloat16)
     b.act[:T, :cfg["width"]] = x.to(b.act.dtype)
-    mlp, e = m.layers[i][2], b.launches[i, "mlp"]
+    mlp, e = m.layers[i].mlp, b.launches[i, "mlp"]
     from nats_llm_studio_amd.models.stack import _Step
     mlp.run(b, e, _Step(T, 1, 16, st()))
     one = torch.ones(cfg["width"], device="cuda")
@@ -236,7 +236,7 @@ def test_wkv_mixer(K, tmp_path, dt, name, i):
     W, d, n = S.make_weights(cfg), cfg["width"], 41
     m = load(tmp_path, cfg, W, dt)
     b = m.step_buffers(64, 2, 16)
-    mix, state = m.layers[i][0], m.state_pool(3)[i]
+    mix, state = m.layers[i].mix, m.state_pool(3)[i]
     for t in state.values():
         t.fill_(5.0)
     x = rnd(n, d, seed=2).to(torch.bfloat16)
@@ -342,7 +342,8 @@ def test_latent_mixer(gpu, tmp_path, dt, name, expand, monkeypatch):
         if info:
             step.plan = m._expand_plan(b, info["qblocks"], info["row_info"], 2 * T, 16, st())
         for i in (0, 1):
-            m.layers[i][0].run(b, b.launches[i, "mix"], kc, None, step)
+            step.layer = i
+            m.layers[i].mix.run(b, b.launches[i, "mix"], kc, None, step)
             got[i].append(b.y[:2 * T].clone())
     Wd, pos = {k: v.double() for k, v in W.items()}, torch.arange(n)
     for r, src in ((0, x), (1, z)):
