@@ -70,10 +70,12 @@ def parse(argv=None):
     ap.add_argument("--tp-leg-timeout", type=float, default=480.0,
                     help="seconds before the TP leg is abandoned (bounds what it adds to an N-GPU run)")
     ap.add_argument("--stack", default=None, choices=("prefill", "decode", "all"),
-                    help="instead of the headline workload: the config-driven stack design (Sekolorn) at sizes of real "
-                         "layers beside a Mixtral-shaped model of the GGUF families at equal size (nats_llm_studio_amd/bench_stack.py)")
+                    help="instead of the headline workload: a config-driven stack design at sizes of real layers beside the "
+                         "closest model of the GGUF families at equal size (nats_llm_studio_amd/bench_stack.py)")
+    ap.add_argument("--stack-design", default="sekolorn", choices=("sekolorn", "kolodra"), help="with --stack: the design")
     ap.add_argument("--stack-sizes", default="2k,4k,4k-fine", help="with --stack: sizes to run")
-    ap.add_argument("--stack-only", default=None, choices=("sekolorn", "closest"), help="with --stack: one of the two models")
+    ap.add_argument("--stack-only", default=None, choices=("sekolorn", "kolodra", "closest"),
+                    help="with --stack: one of the two models")
     ap.add_argument("--stack-case", default=None, help="with --stack: one BATCHxPROMPT case")
     ap.add_argument("--step-breakdown", action="store_true",
                     help="report host time vs time blocked on the previous step's tokens (diagnostic)")

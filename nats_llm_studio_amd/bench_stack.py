@@ -1,5 +1,7 @@
-"""`bench.py --stack`: prefill and decode throughput of the Sekolorn design at sizes of real layers, beside the GGUF families'
-closest model (Mixtral: attention + routed experts, F16 weights) with the same width, layers, experts and expert weights.
+"""`bench.py --stack`: prefill and decode throughput of the config-driven stack designs at sizes of real layers, each beside the
+GGUF families' closest model with the same width, layers and weights per layer, F16:
+  sekolorn   Mixtral (attention + routed experts), the same experts
+  kolodra    Llama (grouped-query attention + gated feed-forward), the feed-forward wider by the weights of the second mixer
 
 Both run the engine's own loop: submit, chunked prefill, captured decode steps. Random weights; one JSON line per case."""
 from __future__ import annotations
@@ -11,16 +13,25 @@ from dataclasses import replace
 
 VOCAB = 32000
 
-# name -> (Sekolorn config arguments, closest model's arguments); expert weights: 2 * ff_s = 3 * ff_m
+# design -> size -> (its config arguments, closest model's arguments)
 SIZES = {
-    "2k": dict(width=2048, wkv=(32, 64), latent=dict(heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=768),
-               moe=(8, 2, 6144), mixtral=dict(n_head=16, n_kv_head=4, d_ff=4096)),
-    "4k": dict(width=4096, wkv=(64, 64), latent=dict(heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1536),
-               moe=(8, 2, 6144), mixtral=dict(n_head=32, n_kv_head=8, d_ff=4096)),
-    # many small experts, a shared one, group-limited choice (no GGUF family has this shape)
-    "4k-fine": dict(width=4096, wkv=(64, 64), latent=dict(heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1536),
-                    moe=(64, 6, 1024), groups=(8, 4), shared=1024, mixtral=None),
+    # expert weights: 2 * ff_s = 3 * ff_m
+    "sekolorn": {
+        "2k": dict(width=2048, wkv=(32, 64), latent=dict(heads=16, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=768),
+                   moe=(8, 2, 6144), closest=dict(n_head=16, n_kv_head=4, d_ff=4096)),
+        "4k": dict(width=4096, wkv=(64, 64), latent=dict(heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1536),
+                   moe=(8, 2, 6144), closest=dict(n_head=32, n_kv_head=8, d_ff=4096)),
+        # many small experts, a shared one, group-limited choice (no GGUF family has this shape)
+        "4k-fine": dict(width=4096, wkv=(64, 64), latent=dict(heads=32, dim=128, rot_dim=64, vdim=128, kv_rank=512, q_rank=1536),
+                        moe=(64, 6, 1024), groups=(8, 4), shared=1024, closest=None),
+    },
+    "kolodra": {
+        "2k": dict(width=2048, left=(16, 4, 128), right=(16, 64, 128), ff=5632, closest=dict(n_head=16, n_kv_head=4, d_ff=8192)),
+        "4k": dict(width=4096, left=(32, 8, 128), right=(32, 64, 128), ff=9216, closest=dict(n_head=32, n_kv_head=8, d_ff=14336)),
+    },
 }
+CLOSEST = {"sekolorn": "mixtral-8x7b", "kolodra": "llama-3-8b"}
+DESIGNS = tuple(SIZES)
 
 
 def sekolorn_config(sz: dict) -> dict:
@@ -37,7 +48,81 @@ def sekolorn_config(sz: dict) -> dict:
     return {"architecture": "Sekolorn", "width": sz["width"], "vocab": VOCAB, "norm": {"eps": 1e-5}, "layers": layers}
 
 
-def write_sekolorn(path: str, cfg: dict):
+def kolodra_config(sz: dict) -> dict:
+    H, G, D = sz["left"]
+    RH, RD, RV = sz["right"]
+    mixer = {"left": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "rot": {"base": 10000.0, "dims": D}, "scale": D ** -0.5},
+             "right": {"heads": RH, "dim": RD, "vdim": RV, "tau": 16.0}, "left_scale": 1.0, "right_scale": 1.0}
+    layers = [{"type": "parallel", "mixer": mixer, "mlp": {"kind": "dense", "ff": sz["ff"]}} for _ in range(4)]
+    return {"architecture": "Kolodra", "width": sz["width"], "vocab": VOCAB, "norm": {"eps": 1e-5}, "layers": layers,
+            "embedding": {"scale": 1.0}, "logit_softcap": 30.0}
+
+
+CONFIGS = {"sekolorn": sekolorn_config, "kolodra": kolodra_config}
+
+
+def _sekolorn_layer(p: str, L: dict, d: int, lin, full):
+    m = L["mixer"]
+    full(p + "norm1", 1.0, d)
+    full(p + "norm2", 1.0, d)
+    if L["type"] == "wkv":
+        HD = m["heads"] * m["dim"]
+        for s in "rkvgw":
+            full(p + "mix.mu." + s, 0.5, d)
+        for s in "rkvg":
+            lin(p + "mix." + s, HD, d)
+        lin(p + "mix.w1", 64, d)
+        lin(p + "mix.w2", HD, 64)
+        full(p + "mix.w0", -3.0, HD)
+        full(p + "mix.u", 0.5, m["heads"], m["dim"])
+        full(p + "mix.norm", 1.0, HD)
+        lin(p + "mix.o", d, HD)
+    else:
+        H, D, RD, VD, R, Q = (m[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank"))
+        lin(p + "mix.dq", Q, d)
+        full(p + "mix.dq.norm", 1.0, Q)
+        lin(p + "mix.uq", H * (D + RD), Q)
+        if "kv_from" not in m:
+            lin(p + "mix.dkv", R + RD, d)
+            full(p + "mix.dkv.norm", 1.0, R)
+        lin(p + "mix.uk", H * D, R)
+        lin(p + "mix.uv", H * VD, R)
+        lin(p + "mix.g", H, d)
+        lin(p + "mix.o", d, H * VD)
+    f = L["mlp"]
+    lin(p + "mlp.router", f["router"]["experts"], d)
+    for e in range(f["router"]["experts"]):
+        lin(f"{p}mlp.e{e}.up", f["expert"]["ff"], d)
+        lin(f"{p}mlp.e{e}.down", d, f["expert"]["ff"])
+    if f.get("shared"):
+        lin(p + "mlp.shared.up", f["shared"]["ff"], d)
+        lin(p + "mlp.shared.down", d, f["shared"]["ff"])
+
+
+def _kolodra_layer(p: str, L: dict, d: int, lin, full):
+    a, r, ff = L["mixer"]["left"], L["mixer"]["right"], L["mlp"]["ff"]
+    full(p + "norm1", 0.0, d)
+    q = p + "mix.left."
+    for n, rows in (("q", a["heads"] * a["dim"]), ("k", a["kv_heads"] * a["dim"])):
+        lin(q + n, rows, d)
+        full(q + n + ".norm", 1.0, rows)
+    lin(q + "g", a["heads"], d)
+    lin(q + "o", d, a["heads"] * a["dim"])
+    q, HD, HV = p + "mix.right.", r["heads"] * r["dim"], r["heads"] * r["vdim"]
+    for n, rows in (("q", HD), ("k", HD), ("v", HV), ("g", HV)):
+        lin(q + n, rows, d)
+    lin(q + "a1", 16, d)
+    lin(q + "a2", HD, 16)
+    full(q + "a2.b", 1.0, HD)
+    full(q + "norm", 1.0, r["vdim"])
+    lin(q + "o", d, HV)
+    lin(p + "mlp.gate", ff, d)
+    lin(p + "mlp.up", ff, d)
+    lin(p + "mlp.down", d, ff)
+
+
+def write_stack(path: str, cfg: dict):
+    """A checkpoint folder of `cfg` with random weights."""
     import torch
 
     from .safetensors_io import write_safetensors
@@ -49,72 +134,40 @@ def write_sekolorn(path: str, cfg: dict):
     def lin(name, *shape):
         W[name] = (torch.randn(*shape, generator=g, device=dev) * shape[-1] ** -0.5).to(torch.bfloat16).cpu()
 
-    def one(name, n):
-        W[name] = torch.ones(n, dtype=torch.bfloat16)
+    def full(name, v, *shape):
+        W[name] = torch.full(shape, v, dtype=torch.bfloat16)
     W["embed"] = torch.randn(cfg["vocab"], d, generator=g, device=dev).to(torch.bfloat16).cpu()
+    layer = {"Sekolorn": _sekolorn_layer, "Kolodra": _kolodra_layer}[cfg["architecture"]]
     for i, L in enumerate(cfg["layers"]):
-        p, m = f"l{i}.", L["mixer"]
-        one(p + "norm1", d)
-        one(p + "norm2", d)
-        if L["type"] == "wkv":
-            HD = m["heads"] * m["dim"]
-            for s in "rkvgw":
-                W[p + "mix.mu." + s] = torch.full((d,), 0.5, dtype=torch.bfloat16)
-            for s in "rkvg":
-                lin(p + "mix." + s, HD, d)
-            lin(p + "mix.w1", 64, d)
-            lin(p + "mix.w2", HD, 64)
-            W[p + "mix.w0"] = torch.full((HD,), -3.0, dtype=torch.bfloat16)
-            W[p + "mix.u"] = torch.full((m["heads"], m["dim"]), 0.5, dtype=torch.bfloat16)
-            one(p + "mix.norm", HD)
-            lin(p + "mix.o", d, HD)
-        else:
-            H, D, RD, VD, R, Q = (m[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank", "q_rank"))
-            lin(p + "mix.dq", Q, d)
-            one(p + "mix.dq.norm", Q)
-            lin(p + "mix.uq", H * (D + RD), Q)
-            if "kv_from" not in m:
-                lin(p + "mix.dkv", R + RD, d)
-                one(p + "mix.dkv.norm", R)
-            lin(p + "mix.uk", H * D, R)
-            lin(p + "mix.uv", H * VD, R)
-            lin(p + "mix.g", H, d)
-            lin(p + "mix.o", d, H * VD)
-        f = L["mlp"]
-        lin(p + "mlp.router", f["router"]["experts"], d)
-        for e in range(f["router"]["experts"]):
-            lin(f"{p}mlp.e{e}.up", f["expert"]["ff"], d)
-            lin(f"{p}mlp.e{e}.down", d, f["expert"]["ff"])
-        if f.get("shared"):
-            lin(p + "mlp.shared.up", f["shared"]["ff"], d)
-            lin(p + "mlp.shared.down", d, f["shared"]["ff"])
-    one("final.norm", d)
+        layer(f"l{i}.", L, d, lin, full)
+    full("final.norm", 1.0 if cfg["architecture"] == "Sekolorn" else 0.0, d)
     lin("head", cfg["vocab"], d)
     with open(os.path.join(path, "config.json"), "w") as fh:
         json.dump(cfg, fh)
     write_safetensors(os.path.join(path, "model.safetensors"), W)
 
 
-def load(which: str, size: str, model_dir: str, dev):
+def load(design: str, closest: bool, size: str, model_dir: str, dev):
     from .models.registry import load_model
-    sz = SIZES[size]
+    sz = SIZES[design][size]
     os.makedirs(model_dir, exist_ok=True)
-    if which == "sekolorn":
-        path = os.path.join(model_dir, f"sekolorn-{size}")
+    if not closest:
+        path = os.path.join(model_dir, f"{design}-{size}")
         if not os.path.exists(os.path.join(path, "config.json")):
-            write_sekolorn(path, sekolorn_config(sz))
-    else:
-        from .gguf import synth
-        # F16 experts run on the dense grouped GEMM's row-major copies (the LDS-dequant GEMM takes K-quants only)
-        os.environ.setdefault("NLS_DENSE_WEIGHTS", "1")
-        os.environ.setdefault("NLS_DENSE_EXPERTS", "1")
-        path = os.path.join(model_dir, f"mixtral-{size}.gguf")
-        if not os.path.exists(path):
-            name = f"mixtral-{size}"
-            synth.SPECS[name] = replace(synth.SPECS["mixtral-8x7b"], name=name, n_layer=4, d_model=sz["width"], vocab=VOCAB,
-                                        n_expert=sz["moe"][0], n_expert_used=sz["moe"][1], **sz["mixtral"])
-            synth.write_synthetic_gguf(path, name, "F16", seed=0)
-    return load_model(path, dev, ctx=None if which != "sekolorn" else 8192)
+            write_stack(path, CONFIGS[design](sz))
+        return load_model(path, dev, ctx=8192)
+    from .gguf import synth
+    # F16 weights run on the dense GEMMs' row-major copies (the LDS-dequant GEMM takes K-quants only)
+    os.environ.setdefault("NLS_DENSE_WEIGHTS", "1")
+    os.environ.setdefault("NLS_DENSE_EXPERTS", "1")
+    name = f"{CLOSEST[design].split('-')[0]}-{size}"
+    path = os.path.join(model_dir, f"{name}.gguf")
+    if not os.path.exists(path):
+        moe = dict(n_expert=sz["moe"][0], n_expert_used=sz["moe"][1]) if "moe" in sz else {}
+        synth.SPECS[name] = replace(synth.SPECS[CLOSEST[design]], name=name, n_layer=4, d_model=sz["width"], vocab=VOCAB,
+                                    **moe, **sz["closest"])
+        synth.write_synthetic_gguf(path, name, "F16", seed=0)
+    return load_model(path, dev)
 
 
 def measure(model, B: int, prompt: int, steps: int, warmup: int, repeat: int = 2) -> dict:
@@ -163,19 +216,20 @@ def run(args) -> int:
     cases = CASES["prefill"] + CASES["decode"] if args.stack == "all" else CASES[args.stack]
     if args.stack_case:
         cases = [tuple(int(v) for v in args.stack_case.split("x"))]
-    for size in args.stack_sizes.split(","):
-        for which in ("sekolorn", "closest"):
-            if args.stack_only not in (None, which) or (which == "closest" and SIZES[size]["mixtral"] is None):
+    design, sizes = args.stack_design, SIZES[args.stack_design]
+    for size in [z for z in args.stack_sizes.split(",") if z in sizes]:
+        for which in (design, "closest"):
+            if args.stack_only not in (None, which) or (which == "closest" and sizes[size]["closest"] is None):
                 continue
             t0 = time.time()
-            model = load(which, size, args.model_dir, dev)
+            model = load(design, which == "closest", size, args.model_dir, dev)
             t_load = time.time() - t0
             for B, prompt in cases:
                 steps = 4 if (B, prompt) in CASES["prefill"] and args.stack != "decode" and not args.stack_case else args.steps
                 out = measure(model, B, prompt, min(steps, 100), min(args.warmup, 10))
                 print(json.dumps(dict(bench="stack", model=which, size=size, batch=B, prompt=prompt, layers=4,
                                       weights_gb=round(model.weight_bytes / 1e9, 3), load_s=round(t_load, 1),
-                                      dtype="bf16" if which == "sekolorn" else "fp16", data="synthetic", **out)), flush=True)
+                                      dtype="fp16" if which == "closest" else "bf16", data="synthetic", **out)), flush=True)
             del model
             torch.cuda.empty_cache()
     return 0

@@ -7,13 +7,13 @@ import torch
 
 import sekolorn_models as S
 import sekolorn_oracle as O
+from stack_helpers import DT, act, engine, relerr, rnd, run_rows, st
 
 pytestmark = pytest.mark.gpu
 # Whole models: largest row error (sekolorn_models.error) in f32. In bf16 an expert choice can still be a close call, and a
 # squared relu whose units are all nearly off leaves the norm after it mostly rounding, so there the bound holds for nine
 # rows of ten; f32 runs the same kernels' f32 forms and holds for all.
 F32, BF16 = 2e-5, 0.06
-DT = {"f32": torch.float32, "bf16": torch.bfloat16}
 TOL = {"f32": 3e-5, "bf16": 1.5e-2}
 
 
@@ -22,25 +22,6 @@ def K(gpu):
     from nats_llm_studio_amd.ops import stack
     stack.lib()
     return stack
-
-
-def rnd(*shape, seed=0, scale=1.0):
-    return torch.randn(*shape, generator=torch.Generator().manual_seed(seed), dtype=torch.float64) * scale
-
-
-def relerr(got, want):
-    return float((got.double().cpu() - want).abs().max() / (want.abs().max() + 1e-30))
-
-
-def act(t, ld, dt, rows=None):
-    """t [n, k] as an activation buffer of `ld` columns, padding zero."""
-    b = torch.zeros(rows or t.shape[0], ld, dtype=dt, device="cuda")
-    b[:t.shape[0], :t.shape[1]] = t.to(dt)
-    return b
-
-
-def st():
-    return torch.cuda.current_stream().cuda_stream
 
 
 # ---------------------------------------------------------------- linear layers
@@ -367,41 +348,13 @@ def test_expanded_runs_beside_short_ones(gpu, tmp_path):
     assert sorted(map(tuple, qb[2:, :5].tolist())) == sorted([(o, min(q, 300 - o), 0, o, 0) for o in range(0, 300, q)]
                                                              + [(332, 40, 3, 100, 300)])
     assert m.row_blocks([0, 1], [5, 9], 2) == (None, None)
-    eng = engine(m, "bf16")
+    eng = engine(m)
     seqs = {k: S.tokens(n, cfg["vocab"], n) for k, n in (("a", 300), ("b", 78), ("c", 31), ("d", 140))}
     eng.feed([("b", seqs["b"][:77], []), ("d", seqs["d"][:100], [])])
     got = eng.feed([("a", seqs["a"], list(range(300))), ("b", seqs["b"][77:], [0]), ("c", seqs["c"], list(range(31))),
                     ("d", seqs["d"][100:], list(range(40)))])
     for (k, t), g in zip(seqs.items(), got):
         assert close(g, O.forward(cfg, W, t)[-len(g):], "bf16"), k
-
-
-def run_rows(m, b, kc, state, parts, bs=16):
-    """One forward of [(seq row, slot, blocks, first position, tokens)] with every row's logits; CPU logits per part."""
-    T = 0
-    b.slot.fill_(-1)
-    dev = b.ids.device
-    for r, (slot, blocks, p0, toks) in enumerate(parts):
-        n = len(toks)
-        pos = torch.arange(p0, p0 + n)
-        blk = torch.tensor(blocks)
-        b.ids[T:T + n] = torch.tensor(toks, dtype=torch.int32)
-        b.pos[T:T + n] = pos.int()
-        b.slot[T:T + n] = (blk[pos // bs] * bs + pos % bs).int()
-        b.tok_seq[T:T + n] = r
-        b.ctx_len[T:T + n] = (pos + 1).int()
-        b.block_tables[r, :len(blocks)] = blk.int()
-        b.runs[r] = torch.tensor([T, n, slot, p0])
-        T += n
-    qb = m.attention_blocks(b, T)
-    rows = torch.arange(T, dtype=torch.int32, device=dev)
-    m.forward(b, kc, None, T, bs, logit_rows=rows, n_logits=T, state=state, nruns=len(parts), **qb)
-    lg = b.logits[:T].cpu()
-    out, o = [], 0
-    for _, _, _, toks in parts:
-        out.append(lg[o:o + len(toks)])
-        o += len(toks)
-    return out
 
 
 def load(tmp_path, cfg, W, dt, ctx=1024):
@@ -436,12 +389,6 @@ def test_prompt_layers(gpu, tmp_path, dt, name):
     assert close(got, want, dt)
 
 
-def engine(m, dt, **kw):
-    from nats_llm_studio_amd.engine.engine import Engine
-    kw = dict(dict(max_batch=4, num_blocks=64, max_prefill_tokens=512, max_logit_rows=512, ctx=512), **kw)
-    return Engine(m, None, **kw)
-
-
 @pytest.mark.parametrize("dt", DT)
 @pytest.mark.parametrize("name", ["uneven", "wide", "ones"])
 def test_feed_schedules(gpu, tmp_path, dt, name):
@@ -450,7 +397,7 @@ def test_feed_schedules(gpu, tmp_path, dt, name):
     cfg = S.CONFIGS[name]
     W = S.make_weights(cfg)
     m = load(tmp_path, cfg, W, dt)
-    eng = engine(m, dt)
+    eng = engine(m)
     toks = S.tokens(150, cfg["vocab"])
     want = O.forward(cfg, W, toks)
     (got,) = eng.feed([("w", toks, list(range(150)))])
@@ -523,7 +470,7 @@ def test_far_key(gpu, tmp_path, dt):
     want = O.forward(cfg, W, toks)
     other = O.forward(cfg, W, toks[:17] + [5] + toks[18:])
     assert S.error(want[[-1]], other[[-1]]) > 0.1
-    eng = engine(m, dt)
+    eng = engine(m)
     (g,) = eng.feed([("p", toks, [n - 40, n - 1])])
     assert close(g, want[[n - 40, n - 1]], dt)
     eng.feed_end("p")
@@ -548,7 +495,7 @@ def test_generation(gpu, tmp_path, blocks, graphs):
     cfg = S.CONFIGS["uneven"]
     W = S.make_weights(cfg)
     m = load(tmp_path, cfg, W, "f32")
-    eng = engine(m, "f32", max_batch=3, num_blocks=blocks, max_prefill_tokens=40, use_graphs=graphs, max_logit_rows=0)
+    eng = engine(m, max_batch=3, num_blocks=blocks, max_prefill_tokens=40, use_graphs=graphs, max_logit_rows=0)
     eng.gen_ratio = 0.0                  # admit on the prompts alone
     if graphs:
         eng.capture_all()
@@ -570,7 +517,7 @@ def test_generation_bf16(gpu, tmp_path):
     from nats_llm_studio_amd.engine.sampling import SamplingParams
     cfg = S.CONFIGS["wide"]
     W = S.make_weights(cfg)
-    eng = engine(load(tmp_path, cfg, W, "bf16"), "bf16", max_logit_rows=0)
+    eng = engine(load(tmp_path, cfg, W, "bf16"), max_logit_rows=0)
     p = S.tokens(60, cfg["vocab"], 5)
     r = eng.generate(p, SamplingParams(max_tokens=30, ignore_eos=True))
     lg = O.forward(cfg, W, p + r.token_ids)[len(p) - 1:-1]
@@ -583,7 +530,7 @@ def test_seeded_sampling(gpu, tmp_path):
     from nats_llm_studio_amd.engine.engine import GenRequest
     from nats_llm_studio_amd.engine.sampling import SamplingParams
     cfg = S.CONFIGS["uneven"]
-    eng = engine(load(tmp_path, cfg, S.make_weights(cfg), "f32"), "f32", max_logit_rows=0)
+    eng = engine(load(tmp_path, cfg, S.make_weights(cfg), "f32"), max_logit_rows=0)
     p = S.tokens(60, cfg["vocab"], 5)
     sp = SamplingParams(max_tokens=12, ignore_eos=True, temperature=0.9, top_k=30, seed=11)
     alone = eng.generate(p, sp).token_ids
@@ -599,7 +546,7 @@ def test_long_decoding_and_graph_replays(gpu, tmp_path, dt):
     """A few hundred decoded tokens through the captured graph, every replay checked."""
     cfg = S.CONFIGS["ones"]
     W = S.make_weights(cfg)
-    eng = engine(load(tmp_path, cfg, W, dt), dt)
+    eng = engine(load(tmp_path, cfg, W, dt))
     toks = S.tokens(320, cfg["vocab"], 4)
     want = O.forward(cfg, W, toks)
     eng.feed([("x", toks[:20], [])])
