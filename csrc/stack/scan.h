@@ -1,19 +1,9 @@
-// Gated linear recurrences with a per-channel decay (gfx950): the scan over runs of tokens, the step of single tokens and the
-// per-head output norm, shared by "wkv" time mixing (wkv.hip) and gated linear attention (gla.hip).
+// Gated linear recurrences with a per-channel decay (gfx950): what "wkv" time mixing (wkv.hip) and gated linear attention
+// (gla.hip) share: the step of single tokens and the per-head output norm.
 //
 // Per head, with keys i and values j (state S [D][V], f32):
 //   wkv: o_t[j] = sum_i r_t[i] (S[i][j] + u[i] k_t[i] v_t[j]);   S[i][j] = w_t[i] S[i][j] + k_t[i] v_t[j]
 //   gla: S[i][j] = w_t[i] S[i][j] + k_t[i] v_t[j];               o_t[j] = rs sum_i r_t[i] S[i][j]
-//
-// The scan is sequential in the tokens of a run (or of a segment of it, below), so that a position's result does not depend
-// on how its sequence was cut into steps. Parallelism is (run, head, value columns) x lanes: a lane holds DP / PARTS key rows
-// of CPL value columns in registers, PARTS neighbouring lanes cover the keys and close the sum with in-row lane exchanges
-// (DPP). Few runs take many key parts (short per-token chains on all CUs). Tokens are staged in LDS in chunks of CH as f32,
-// the next chunk's loads in flight while the current one runs.
-// Segments (gla): a long run is cut into `nseg` segments that run in parallel, in two launches. The first runs segment 0 in
-// full and, from a zero state, the end state and the product of decays of every further segment but the last; the second
-// starts each of those and the last from end states chained over the segments before it. Only products with decays in
-// [0, 1] appear, so nothing over- or underflows that would not in the plain recurrence.
 // A step of single tokens (decode) streams each head's state once with 16-byte accesses and ends with the head's norm and
 // gate (step_kernel).
 //
@@ -25,7 +15,6 @@
 namespace nls_scan {
 
 enum Kind : int { WKV = 0, GLA = 1 };
-constexpr int MINSEG = 64;     // fewest tokens of a segment
 
 template <typename T> DEVI float ld1(const T* p) { return (float)*p; }
 
@@ -50,249 +39,10 @@ struct Scan {
   const float* x;          // wkv: residual rows; the run's last becomes the slot's previous token (prev null: no such row)
   float* prev;
   const int* runs;
-  float* seg_s;            // segments: end states [run][nseg - 1][H][D][V] and decay products [run][nseg - 1][H][D]
-  float* seg_w;
   long ld, ldw, ldo, sstride, ldx, ldp;
   int H, D, V, width;
-  int nseg, pass;          // pass 0: the only or first launch, 1: the second
   float rs;                // gla: factor of the output
 };
-
-// DP: key channels padded to a multiple of 32 (zeros past D)
-template <typename T, int KIND, int DP, int PARTS, int CPL>
-__global__ __launch_bounds__(256) void scan_kernel(Scan p) {
-  constexpr int WC = 256 / PARTS * CPL;          // value columns per workgroup
-  constexpr int CH = DP <= 64 ? 32 : (DP <= 128 ? 16 : 8);   // tokens per staged chunk
-  constexpr int R = DP / PARTS;                  // state rows per lane
-  constexpr int LR = DP + 4;                     // LDS row stride
-  constexpr int NV = (CH * DP + 255) / 256;      // staged values per thread and operand
-  __shared__ __attribute__((aligned(16))) float rs[CH][LR], ks[CH][LR], ws[CH][LR];
-  __shared__ __attribute__((aligned(16))) float vs[CH][WC], ruk[KIND == WKV ? CH : 1];
-  const int* run = p.runs + 4 * blockIdx.y;
-  int t0 = run[0], n = run[1];
-  const int slot = run[2], pos0 = run[3];
-  if (slot < 0 || n < 1) return;
-  const int D = p.D, V = p.V;
-  // the segment of this workgroup: rows t0 .. t0 + n - 1
-  const int z = KIND == GLA ? (int)blockIdx.z + p.pass : 0;
-  bool last = true;
-  if (KIND == GLA && p.nseg > 1) {
-    const int sl = max(MINSEG, ((n + p.nseg - 1) / p.nseg + 31) & ~31);
-    if (z * sl >= n) return;
-    last = (z + 1) * sl >= n;
-    if (p.pass == 0 && z > 0 && last) return;
-    t0 += z * sl;
-    n = min(sl, n - z * sl);
-  }
-  const bool local = KIND == GLA && p.pass == 0 && z > 0;       // end state from zero, no outputs
-  const int ncb = (V + WC - 1) / WC;
-  const int head = blockIdx.x / ncb, c0 = (blockIdx.x % ncb) * WC;
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int part = lane & (PARTS - 1), col = (wave * (64 / PARTS) + lane / PARTS) * CPL;
-  const int j = c0 + col;
-  const size_t hb = (size_t)head * D, hv = (size_t)head * V;
-  const T* rp = (const T*)p.r + hb;
-  const T* kp = (const T*)p.k + hb;
-  const T* vp = (const T*)p.v + hv;
-  const float* wp = p.w + hb;
-  float* st = p.state + (size_t)slot * p.sstride + hb * V;
-  const size_t sst = (size_t)p.H * D * V, swt = (size_t)p.H * D;                        // segment records
-  float* sgs = p.seg_s + (size_t)blockIdx.y * (p.nseg - 1) * sst + hb * V;
-  float* sgw = p.seg_w + (size_t)blockIdx.y * (p.nseg - 1) * swt + hb;
-
-  float S[CPL][R], pw[KIND == GLA ? R : 1];
-#pragma unroll
-  for (int i = 0; i < R; ++i)
-#pragma unroll
-    for (int c = 0; c < CPL; ++c) {
-      const int row = part * R + i;
-      const bool in = row < D && j + c < V;
-      if (KIND == GLA && z > 0) {
-        float s = 0.f;
-        if (!local && in) {
-          s = sgs[(size_t)row * V + j + c];
-          for (int q = 1; q < z; ++q) s = fmaf(sgw[q * swt + row], s, sgs[q * sst + (size_t)row * V + j + c]);
-        }
-        S[c][i] = s;
-      } else {
-        S[c][i] = pos0 > 0 && in ? st[(size_t)row * V + j + c] : 0.f;
-      }
-    }
-#pragma unroll
-  for (int i = 0; i < (KIND == GLA ? R : 1); ++i) pw[i] = 1.f;
-  float ur[KIND == WKV ? DP / 16 : 1];           // u of the bonus sums' columns
-  if constexpr (KIND == WKV)
-#pragma unroll
-    for (int q = 0; q < DP / 16; ++q) {
-      const int i = (threadIdx.x & 15) + 16 * q;
-      ur[q] = i < D ? p.u[hb + i] : 0.f;
-    }
-  float fr[NV], fk[NV], fw[NV], fv[(CH * WC + 255) / 256];
-  auto fetch = [&](int base) __attribute__((always_inline)) {
-#pragma unroll
-    for (int q = 0; q < NV; ++q) {
-      const int e = threadIdx.x + q * 256, tt = e / DP, i = e % DP;
-      const bool in = tt < CH && base + tt < n && i < D;
-      const size_t row = (size_t)(t0 + min(base + tt, n - 1));
-      fr[q] = in ? ld1(rp + row * p.ld + i) : 0.f;
-      fk[q] = in ? ld1(kp + row * p.ld + i) : 0.f;
-      fw[q] = in ? wp[row * p.ldw + i] : 0.f;
-    }
-#pragma unroll
-    for (int q = 0; q < (CH * WC + 255) / 256; ++q) {
-      const int e = threadIdx.x + q * 256, tt = e / WC, i = c0 + (e & (WC - 1));
-      const bool in = tt < CH && base + tt < n && i < V;
-      fv[q] = in ? ld1(vp + (size_t)(t0 + min(base + tt, n - 1)) * p.ld + i) : 0.f;
-    }
-  };
-  fetch(0);
-  for (int base = 0; base < n; base += CH) {
-    __syncthreads();
-#pragma unroll
-    for (int q = 0; q < NV; ++q) {
-      const int e = threadIdx.x + q * 256, tt = e / DP, i = e % DP;
-      if (tt < CH) {
-        rs[tt][i] = fr[q];
-        ks[tt][i] = fk[q];
-        ws[tt][i] = fw[q];
-      }
-    }
-#pragma unroll
-    for (int q = 0; q < (CH * WC + 255) / 256; ++q) {
-      const int e = threadIdx.x + q * 256;
-      if (e < CH * WC) vs[e / WC][e & (WC - 1)] = fv[q];
-    }
-    __syncthreads();
-    if (base + CH < n) fetch(base + CH);
-    // wkv: sum_i r u k of every staged token, 16 lanes each
-#pragma unroll
-    for (int t8 = 0; KIND == WKV && t8 < CH; t8 += 16) {
-      const int tt = t8 + (threadIdx.x >> 4), l = threadIdx.x & 15;
-      float a = 0.f;
-      if (tt < CH)
-#pragma unroll
-        for (int q = 0; q < DP / 16; ++q) a += rs[tt][l + 16 * q] * ur[q] * ks[tt][l + 16 * q];
-#pragma unroll
-      for (int s = 8; s > 0; s >>= 1) a += __shfl_xor(a, s, 64);
-      if (tt < CH && l == 0) ruk[tt] = a;
-    }
-    if (KIND == WKV) __syncthreads();
-    // 8 tokens at a time, the next token's operands on their way while one is summed; lane part q keeps token q's output
-    const int m = min(CH, n - base);
-    f32x4 r4[2][R / 4], k4[2][R / 4], w4[2][R / 4];
-    float v1[2][CPL];
-    auto get = [&](int tt, int b) __attribute__((always_inline)) {
-#pragma unroll
-      for (int q = 0; q < R / 4; ++q) {
-        r4[b][q] = *reinterpret_cast<const f32x4*>(&rs[tt][part * R + 4 * q]);
-        k4[b][q] = *reinterpret_cast<const f32x4*>(&ks[tt][part * R + 4 * q]);
-        w4[b][q] = *reinterpret_cast<const f32x4*>(&ws[tt][part * R + 4 * q]);
-      }
-#pragma unroll
-      for (int c = 0; c < CPL; ++c) v1[b][c] = vs[tt][col + c];
-    };
-    auto token = [&](int b, float (&o)[CPL]) __attribute__((always_inline)) {
-      if constexpr (KIND == GLA) {
-#pragma unroll
-        for (int c = 0; c < CPL; ++c) {
-          float o0 = 0.f, o1 = 0.f;
-#pragma unroll
-          for (int i4 = 0; i4 < R / 4; ++i4)
-#pragma unroll
-            for (int e = 0; e < 4; e += 2) {
-              const int i = 4 * i4 + e;
-              S[c][i] = fmaf(w4[b][i4][e], S[c][i], k4[b][i4][e] * v1[b][c]);
-              S[c][i + 1] = fmaf(w4[b][i4][e + 1], S[c][i + 1], k4[b][i4][e + 1] * v1[b][c]);
-              o0 = fmaf(r4[b][i4][e], S[c][i], o0);
-              o1 = fmaf(r4[b][i4][e + 1], S[c][i + 1], o1);
-            }
-          o[c] = sum_parts<PARTS>(o0 + o1);
-        }
-        return;
-      }
-#pragma unroll
-      for (int c = 0; c < CPL; ++c) {
-        float o0 = 0.f, o1 = 0.f;
-#pragma unroll
-        for (int i4 = 0; i4 < R / 4; ++i4)
-#pragma unroll
-          for (int e = 0; e < 4; e += 2) {
-            const int i = 4 * i4 + e;
-            o0 = fmaf(r4[b][i4][e], S[c][i], o0);
-            o1 = fmaf(r4[b][i4][e + 1], S[c][i + 1], o1);
-            S[c][i] = fmaf(w4[b][i4][e], S[c][i], k4[b][i4][e] * v1[b][c]);
-            S[c][i + 1] = fmaf(w4[b][i4][e + 1], S[c][i + 1], k4[b][i4][e + 1] * v1[b][c]);
-          }
-        o[c] = sum_parts<PARTS>(o0 + o1);
-      }
-    };
-    if (local) {
-      // state and decay products only
-      for (int tt = 0; tt < m; ++tt) {
-        get(tt, 0);
-#pragma unroll
-        for (int i = 0; i < R; ++i) {
-          if constexpr (KIND == GLA) pw[i] *= w4[0][i >> 2][i & 3];
-#pragma unroll
-          for (int c = 0; c < CPL; ++c) S[c][i] = fmaf(w4[0][i >> 2][i & 3], S[c][i], k4[0][i >> 2][i & 3] * v1[0][c]);
-        }
-      }
-      continue;
-    }
-    get(0, 0);
-    for (int t8 = 0; t8 < m; t8 += 8) {
-      float mine[CPL], o[CPL];
-#pragma unroll
-      for (int c = 0; c < CPL; ++c) mine[c] = 0.f;
-      const int last = m - 1 - t8, tt = t8 + (part & 7);
-      const float rk = KIND == WKV ? ruk[tt] : 0.f;
-      if (last >= 7) {
-#pragma unroll
-        for (int q = 0; q < 8; ++q) {
-          get(min(t8 + q + 1, CH - 1), (q & 1) ^ 1);
-          token(q & 1, o);
-#pragma unroll
-          for (int c = 0; c < CPL; ++c) mine[c] = part == q ? o[c] : mine[c];
-        }
-      } else {
-#pragma unroll
-        for (int q = 0; q < 8; ++q) {
-          get(min(t8 + q + 1, CH - 1), (q & 1) ^ 1);
-          if (q > last) continue;              // (uniform)
-          token(q & 1, o);
-#pragma unroll
-          for (int c = 0; c < CPL; ++c) mine[c] = part == q ? o[c] : mine[c];
-        }
-      }
-      if (part < 8 && part <= last)
-#pragma unroll
-        for (int c = 0; c < CPL; ++c)
-          if (j + c < V)
-            p.o[(size_t)(t0 + base + tt) * p.ldo + hv + j + c] =
-                KIND == WKV ? fmaf(rk, vs[tt][col + c], mine[c]) : p.rs * mine[c];
-    }
-  }
-  float* dst = last ? st : sgs + z * sst;
-#pragma unroll
-  for (int i = 0; i < R; ++i)
-#pragma unroll
-    for (int c = 0; c < CPL; ++c) {
-      const int row = part * R + i;
-      // (the second launch leaves the records of its segments as they are: others read them)
-      if (row < D && j + c < V && (last || p.pass == 0)) dst[(size_t)row * V + j + c] = S[c][i];
-    }
-  if constexpr (KIND == GLA) {
-    if (local && j == 0)
-#pragma unroll
-      for (int i = 0; i < R; ++i)
-        if (part * R + i < D) sgw[z * swt + part * R + i] = pw[i];
-  }
-  if (KIND != WKV || !p.prev) return;
-  // the run's last row is the next step's previous token (this layer's shift_mix, which reads it, came before)
-  const int G = gridDim.x;
-  for (int i = blockIdx.x * 256 + threadIdx.x; i < p.width; i += G * 256)
-    p.prev[(size_t)slot * p.ldp + i] = p.x[(size_t)(t0 + n - 1) * p.ldx + i];
-}
 
 // ---- one token per run: the state of (run, head) is read and written once, 4 value columns per thread; then
 // out = (o / rms(o)) * norm * gate. V is a multiple of 4, at most 1024; D at most 256.

@@ -429,7 +429,8 @@ class GlaPart(_SharedPart):
         c, P, f = self.cfg, b.pad, torch.float32
         HD, HV = c.heads * c.dim, c.heads * c.vdim
         z = self.scratch(b, "gla.qkva", P, self.ld)
-        a, o = self.scratch(b, "gla.a", P, HD, f), self.scratch(b, "gla.o", P, HV, f)
+        a = self.scratch(b, "gla.a", P, HD, f)
+        o = self.scratch(b, "gla.o", P, HV, f) if c.vdim > 128 else None
         g = self.scratch(b, "gla.g", P, HV)
         return dict(q=z, k=z[:, HD:], v=z[:, 2 * HD:], a=a, o=o, g=g, out=out,
                     inputs=[K.Seg(self.qkva, b.act, z), K.Seg(self.g, b.act, g, "silu")],
@@ -443,13 +444,16 @@ class GlaPart(_SharedPart):
             K.gla_step(e["q"], e["k"], e["v"], e["a"], qs, S, b.runs, T, self.norm, e["g"], e["out"], H, D, V, eps, st)
             return
         n = step.nruns
-        shape = K.gla_shape(T, n, H, D, V)
+        shape = K.gla_shape(T, n, H, V)
         seg = None
         if shape[0] > 1:
-            seg = (self.m.grown(b, "gla.seg", n * (shape[0] - 1), H * D * V, torch.float32),
-                   self.m.grown(b, "gla.segw", n * (shape[0] - 1), H * D, torch.float32))
-        K.gla_scan(e["q"], e["k"], e["v"], e["a"], qs, e["o"], S, b.runs, n, H, D, V, shape, seg, st)
-        K.scan_out(e["o"], self.norm, e["g"], e["out"], H, V, T, eps, st)
+            seg = (self.m.grown(b, "gla.seg", n * shape[0], H * D * V, torch.float32),
+                   self.m.grown(b, "gla.segw", n * shape[0], H * D, torch.float32))
+        fused = V <= 64 * shape[1]
+        K.gla_scan(e["q"], e["k"], e["v"], e["a"], qs, e["o"], self.norm, e["g"], e["out"] if fused else None, S, b.runs, n, H, D,
+                   V, eps, shape, seg, st)
+        if not fused:
+            K.scan_out(e["o"], self.norm, e["g"], e["out"], H, V, T, eps, st)
 
 
 class DensePart(_SharedPart):

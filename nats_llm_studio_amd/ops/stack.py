@@ -43,7 +43,7 @@ _SIGS = {
     "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, F, I, P],
     "nls_gqa_attn": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, P, L, P, L, P, P, P, I, I, P],
     "nls_gqa_prefill": [P, L, P, P, P, P, I, P, I, P, L, I, I, I, I, F, P],
-    "nls_gla_scan": [P, P, P, L, P, L, F, P, L, P, L, P, I, I, I, I, I, P, P, I, I, I, P],
+    "nls_gla_scan": [P, P, P, L, P, L, F, P, L, P, P, L, P, L, F, P, L, P, I, I, I, I, I, P, P, I, I, P],
     "nls_gla_step": [P, P, P, L, P, L, F, P, L, P, I, P, P, L, P, L, I, I, I, F, I, P],
     "nls_latent_rows": [P, L, I, P, P, L, P, L, I, I, I, P, P, P, P, P, L, I, F, I, P],
     "nls_stack_argmax": [P, L, I, P, I, P],
@@ -413,29 +413,30 @@ def scan_out(o, norm, gate, out, H: int, D: int, T: int, eps: float, st: int):
                               out.stride(0), H, D, T, eps, int(out.dtype == torch.float32), st), "nls_scan_out")
 
 
-def gla_shape(T: int, nruns: int, H: int, D: int, V: int):
-    """(segments, lanes per column, columns per lane) of a gla_scan launch: enough workgroups for the chip, segments of at
-    least 128 tokens."""
-    parts = 8 if D <= 64 else 16
-    longest = T - nruns + 1
-    for cpl in (4, 1):
-        wc = 256 // parts * cpl
-        wgs = H * -(-V // wc) * nruns
-        nseg = max(1, min(-(-512 // wgs), longest // 128, 16))
-        if wgs * nseg >= 256 or cpl == 1:
-            return nseg, parts, cpl
+def gla_shape(T: int, nruns: int, H: int, V: int):
+    """(segments, groups of 64 value columns per workgroup) of a gla_scan launch: enough workgroups for the chip, segments of
+    at least 128 tokens."""
+    nt = 1 if V <= 64 else 2
+    wgs = H * -(-V // (64 * nt)) * nruns
+    return max(1, min(-(-512 // wgs), (T - nruns + 1) // 128, 16)), nt
 
 
-def gla_scan(q, k, v, a, qscale: float, o, state, runs, nruns: int, H: int, D: int, V: int, shape, seg, st: int):
+def gla_scan(q, k, v, a, qscale: float, o, norm, gate, out, state, runs, nruns: int, H: int, D: int, V: int, eps: float, shape,
+             seg, st: int):
     """Gated linear attention over each run's tokens: q, k [rows, H * D], v [rows, H * V] of one buffer (equal strides), decays
-    a; state [slots, H * D * V] is carried on. shape: gla_shape; seg: (end states, decay products) scratch of its segments."""
-    nseg, parts, cpl = shape
-    if nseg > 1 and (seg[0].numel() < nruns * (nseg - 1) * H * D * V or seg[1].numel() < nruns * (nseg - 1) * H * D):
+    a; state [slots, H * D * V] is carried on. With `out` (a head's columns fit a workgroup): its norm, `norm` and `gate`
+    applied, else the plain outputs in `o` (scan_out follows). shape: gla_shape; seg: (states, decay products) scratch of its
+    segments."""
+    nseg, nt = shape
+    if nseg > 1 and (seg[0].numel() < nruns * nseg * H * D * V or seg[1].numel() < nruns * nseg * H * D):
         raise ValueError("gla_scan: segment scratch too small")
     s0, s1 = seg if nseg > 1 else (None, None)
+    f = out is not None
     _check(lib().nls_gla_scan(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), a.data_ptr(), a.stride(0), qscale,
-                              o.data_ptr(), o.stride(0), state.data_ptr(), state.stride(0), runs.data_ptr(), nruns, H, D, V,
-                              nseg, _p(s0), _p(s1), parts, cpl, int(q.dtype == torch.float32), st), "nls_gla_scan")
+                              _p(o), o.stride(0) if o is not None else 0, norm.data_ptr() if f else None,
+                              gate.data_ptr() if f else None, gate.stride(0) if f else 0, _p(out), out.stride(0) if f else 0,
+                              eps, state.data_ptr(), state.stride(0), runs.data_ptr(), nruns, H, D, V, nseg, _p(s0), _p(s1), nt,
+                              int(q.dtype == torch.float32), st), "nls_gla_scan")
 
 
 def gla_step(q, k, v, a, qscale: float, state, runs, nruns: int, norm, gate, out, H: int, D: int, V: int, eps: float, st: int):

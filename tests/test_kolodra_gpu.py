@@ -219,13 +219,14 @@ def gla_data(d, H, D, V, n):
 
 @pytest.mark.parametrize("dt", DT)
 @pytest.mark.parametrize("H,D,V", GLA)
-@pytest.mark.parametrize("nseg,cpl", [(1, 1), (1, 4), (2, 4), (5, 1), (16, 4)])
-def test_gla_scan(K, dt, H, D, V, nseg, cpl):
+@pytest.mark.parametrize("nseg,nt", [(1, 1), (1, 2), (2, 2), (5, 1), (16, 2)])
+def test_gla_scan(K, dt, H, D, V, nseg, nt):
     """Two sequences in one launch beside an empty run, cut at 2, 3 and 16 tokens, slots given out of order and dirty, in
-    segments: the plain recurrence; without segments, bit for bit the same however the runs are cut."""
-    d, n, qs = DT[dt], 330, 0.37
+    segments: the plain recurrence however the runs are cut; with the head's norm and gate where a workgroup holds it."""
+    d, n, qs, eps = DT[dt], 330, 0.37, 1e-3
     q, k, v, a = gla_data(d, H, D, V, n)
-    parts, HD, HV = 8 if D <= 64 else 16, H * D, H * V
+    HD, HV, fused = H * D, H * V, V <= 64 * nt
+    norm, g = rnd(HV, seed=7).float(), rnd(2, n, HV, seed=8).to(d)
 
     def run(cuts):
         S0 = torch.full((4, HD * V), 9.0, device="cuda")    # slots start dirty
@@ -237,9 +238,17 @@ def test_gla_scan(K, dt, H, D, V, nseg, cpl):
             z = torch.cat([cat(q), cat(k), cat(v)], 1).cuda()
             runs = torch.tensor([[0, m, 3, x], [m, m, 1, x], [0, 0, -1, 0]], dtype=torch.int32, device="cuda")
             o = torch.zeros(2 * m, HV + 3, device="cuda")
-            K.gla_scan(z, z[:, HD:], z[:, 2 * HD:], cat(a).cuda(), qs, o, S0, runs, 3, H, D, V, (nseg, parts, cpl), seg, st())
+            args = (z, z[:, HD:], z[:, 2 * HD:], cat(a).cuda(), qs, o, norm.cuda(), cat(g).cuda())
+            if fused:
+                y_, S1 = torch.zeros(2 * m, HV + 3, dtype=d, device="cuda"), S0.clone()
+                K.gla_scan(*args, y_, S1, runs, 3, H, D, V, eps, (nseg, nt), seg, st())
+            K.gla_scan(*args, None, S0, runs, 3, H, D, V, eps, (nseg, nt), seg, st())
             out[0, x:y], out[1, x:y] = o[:m, :HV].cpu(), o[m:, :HV].cpu()
             assert (o[:, HV:] == 0).all()
+            if fused:
+                assert torch.equal(S0, S1) and (y_[:, HV:] == 0).all()
+                want = (O.rms(o[:, :HV].cpu().double().view(2 * m, H, V), eps).view(2 * m, HV) * norm.double() * cat(g).double())
+                assert relerr(y_[:, :HV], want) < (2e-5 if dt == "f32" else 5e-3)
         assert (S0[0] == 9).all() and (S0[2] == 9).all()
         return out, S0
     whole, Sw = run(())
@@ -249,10 +258,7 @@ def test_gla_scan(K, dt, H, D, V, nseg, cpl):
         assert relerr(Sw[slot].view(H, D, V), Sx) < 2e-5
     for cuts in ((2, 4, 7, 200), (16, 32, 48, 112, 177), (15, 17, 81, 146, 329)):
         o, Sc = run(cuts)
-        if nseg == 1:
-            assert torch.equal(o, whole) and torch.equal(Sc, Sw)
-        else:
-            assert relerr(o, whole.double()) < 1e-5 and relerr(Sc, Sw.double().cpu()) < 1e-5
+        assert relerr(o, whole.double()) < 2e-5 and relerr(Sc, Sw.double().cpu()) < 2e-5
 
 
 @pytest.mark.parametrize("dt", DT)
@@ -264,12 +270,12 @@ def test_gla_step(K, dt, H, D, V):
     q, k, v, a = gla_data(d, H, D, V, n)
     HD, HV = H * D, H * V
     norm, g = rnd(HV, seed=7).float().cuda(), rnd(2, n, HV, seed=8).to(d)
-    parts = 8 if D <= 64 else 16
     z = torch.cat([torch.cat([q[i], k[i], v[i]], 1) for i in (0, 1)]).cuda()
     o, want = torch.zeros(2 * n, HV, device="cuda"), torch.zeros(2 * n, HV, dtype=d, device="cuda")
     Sw = torch.full((3, HD * V), 9.0, device="cuda")
     runs = torch.tensor([[0, n, 2, 0], [n, n, 0, 0]], dtype=torch.int32, device="cuda")
-    K.gla_scan(z, z[:, HD:], z[:, 2 * HD:], a.view(2 * n, HD).cuda(), qs, o, Sw, runs, 2, H, D, V, (1, parts, 1), None, st())
+    K.gla_scan(z, z[:, HD:], z[:, 2 * HD:], a.view(2 * n, HD).cuda(), qs, o, None, None, None, Sw, runs, 2, H, D, V, eps, (1, 1),
+               None, st())
     K.scan_out(o, norm, g.view(2 * n, HV).cuda(), want, H, V, 2 * n, eps, st())
     ref = O.rms(o.double().cpu().view(2 * n, H, V), eps).view(2 * n, HV) * norm.double().cpu() * g.double().view(2 * n, HV)
     assert relerr(want, ref) < (1e-5 if dt == "f32" else 5e-3)
@@ -428,7 +434,7 @@ def test_long_prompt_segments(gpu, tmp_path, dt):
     W, n = S.make_weights(cfg), 700
     m = load(tmp_path, cfg, W, dt)
     from nats_llm_studio_amd.ops import stack as K
-    assert K.gla_shape(n, 1, 3, 20, 28)[0] > 2 and K.gla_shape(n - 300, 2, 3, 20, 28)[0] > 2
+    assert K.gla_shape(n, 1, 3, 28)[0] > 2 and K.gla_shape(n - 300, 2, 3, 28)[0] > 2
     eng = engine(m, ctx=1024, num_blocks=128, max_prefill_tokens=1024, max_logit_rows=1024)
     toks, other = S.tokens(n + 20, cfg["vocab"], 3), S.tokens(40, cfg["vocab"], 4)
     want = O.forward(cfg, W, toks)
