@@ -402,11 +402,15 @@ int nls_gla_scan(const void* q, const void* k, const void* v, long ld, const flo
   return f32 ? chunk_d<float>(p, nruns, nt, (hipStream_t)stream) : chunk_d<__bf16>(p, nruns, nt, (hipStream_t)stream);
 }
 
-// every run has one token (or none); V a multiple of 4, at most 1024; D at most 256
-int nls_gla_step(const void* q, const void* k, const void* v, long ld, const float* a, long lda, float qscale, float* state,
-                 long sstride, const int* runs, int nruns, const float* norm, const void* gate, long ldg, void* out, long ldout,
-                 int H, int D, int V, float eps, int f32, void* stream) {
-  const Scan p{q, k, v, a, nullptr, nullptr, state, nullptr, nullptr, runs, ld, lda, 0, sstride, 0, 0, H, D, V, 0, qscale};
+// every run has one token (or none); V a multiple of 4, at most 1024; D at most 256. Decays: a, or (a null) from the low-rank
+// gate input `low` (row stride ld, 16-byte aligned rows) with a2 [H * D][rank] in the activation type: sigmoid(a2 low + a2b)^ia
+int nls_gla_step(const void* q, const void* k, const void* v, long ld, const float* a, long lda, const void* low, const void* a2,
+                 const float* a2b, int rank, float ia, float qscale, float* state, long sstride, const int* runs, int nruns,
+                 const float* norm, const void* gate, long ldg, void* out, long ldout, int H, int D, int V, float eps, int f32,
+                 void* stream) {
+  if (!a && (!low || !a2 || !a2b || rank < 1 || ((uintptr_t)low & 15) || ((uintptr_t)a2 & 15) || (ld & 7))) return -1;
+  const Scan p{q, k, v, a, nullptr, nullptr, state, nullptr, nullptr, runs, ld, lda, 0, sstride, 0, 0, H, D, V, 0, qscale,
+               low, a2, a2b, rank, ia};
   return f32 ? step_rows<float, GLA>(p, nruns, norm, gate, ldg, out, ldout, eps, (hipStream_t)stream)
              : step_rows<__bf16, GLA>(p, nruns, norm, gate, ldg, out, ldout, eps, (hipStream_t)stream);
 }

@@ -10,6 +10,8 @@
 // (and finite) up to the padded K. For f32 the four k of a lane are the j-th operands of four 16x16x4 MFMAs: both
 // operands use the same k order, so the sum is over the same products.
 //
+// A segment without an epilogue may split K over `ks` workgroups per tile: each writes an f32 slab of its own (`yks` apart), which
+// the caller's next kernel adds.
 // A launch holds up to LIN_SEGS segments (own x, W, y, epilogue), so independent projections share one grid. A segment
 // may be a batch of `ng` groups (per-head products: column offsets xgs / ygs per group), or routed: its (group, rows)
 // tiles come from a device list written by moe_plan_kernel and its rows from the routed-entry list.
@@ -43,6 +45,7 @@ struct LinSeg {
   long wstride;         // bytes between the groups' packed weights
   long ldx, ldy;        // elements
   long xgs, ygs;        // column offset per group (elements)
+  long yks;             // elements between the slabs of a split K
   int N, nsub;          // output columns; 1 KiB sub-tiles per 16-row tile
   int M, ng;
   int epi, yact;        // yact: store the activation type (bf16; f32 in f32 launches), else f32
@@ -50,6 +53,7 @@ struct LinSeg {
   int xdiv, ldg;        // routed: x row = entry / xdiv
   int half;
   float alpha;          // constant of the epilogue
+  int ks, pad0;         // K splits (identity segments without an epilogue; 1: none)
 };
 
 struct LinArgs {
@@ -79,9 +83,9 @@ template <> struct LT<float> {
   }
 };
 
-// one workgroup's tile: segment, group, first weight row, first row, rows
+// one workgroup's tile: segment, group, split of K, first weight row, first row, rows
 struct LinTile {
-  int seg, grp, n0, m0, cnt;
+  int seg, grp, ks, n0, m0, cnt;
   const int* rows;      // routed: entries of this tile
 };
 
@@ -100,6 +104,7 @@ DEVI bool lin_tile(const LinArgs& a, int id, LinTile& t) {
   const int nnt = (S.N + BN - 1) / BN;
   t.seg = s;
   t.n0 = (q % nnt) * BN;
+  t.ks = 0;
   if (S.rows) {
     if (mi >= *a.ntiles) return false;
     t.grp = a.tiles[4 * mi];
@@ -107,7 +112,9 @@ DEVI bool lin_tile(const LinArgs& a, int id, LinTile& t) {
     t.cnt = a.tiles[4 * mi + 2];
     t.m0 = 0;
   } else {
-    t.grp = q / nnt;
+    q /= nnt;
+    t.grp = S.ng == 1 ? 0 : q % S.ng;
+    t.ks = S.ng == 1 ? q : q / S.ng;
     t.rows = nullptr;
     t.m0 = mi * BM;
     t.cnt = min(BM, S.M - t.m0);
@@ -127,15 +134,24 @@ DEVI void lin_row(const LinSeg& S, const LinTile& t, int i, int& xr, int& yr) {
   }
 }
 
-DEVI float lin_sigmoid(float v) { return 1.f / (1.f + expf(-v)); }
+constexpr float LOG2E = 1.4426950408889634f;
+DEVI float lin_sigmoid(float v) { return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-v * LOG2E)); }
 // z / 2 (1 + tanh(y)) = z sigmoid(2 y), y = sqrt(2 / pi) (z + 0.044715 z^3)
 DEVI float lin_gelu(float z) { return z * lin_sigmoid(1.5957691216057308f * fmaf(0.044715f * z * z, z, z)); }
 
+// sigmoid(z)^a = 2^(-a (max(-z, 0) log2(e) + log2(1 + u))), u = e^-|z|; log2(w) u / (w - 1) with w = fl(1 + u) keeps the
+// digits of a small u
+DEVI float lin_sigpow(float z, float a) {
+  const float u = __builtin_amdgcn_exp2f(-fabsf(z) * LOG2E), w = 1.f + u;
+  const float l = w == 1.f ? u * LOG2E : __builtin_amdgcn_logf(w) * (u * __builtin_amdgcn_rcpf(w - 1.f));
+  return __builtin_amdgcn_exp2f(-a * fmaf(fmaxf(-z, 0.f), LOG2E, l));
+}
+
 // epilogue of 4 consecutive output columns n .. n + 3 of one row
 template <typename T>
-DEVI void lin_store4(const LinSeg& S, int grp, int n, int yr, f32x4 v) {
+DEVI void lin_store4(const LinSeg& S, int grp, int ks, int n, int yr, f32x4 v) {
   if (n >= S.N) return;
-  const int nb = n / S.cb, nr = n - nb * S.cb;
+  const int nb = S.cb < S.N ? n / S.cb : 0, nr = n - nb * S.cb;      // (no division where columns are not blocked)
   switch (S.epi) {
     case LE_SILU:
 #pragma unroll
@@ -164,10 +180,7 @@ DEVI void lin_store4(const LinSeg& S, int grp, int n, int yr, f32x4 v) {
     case LE_SIGPOW:
 #pragma unroll
       for (int e = 0; e < 4; ++e)
-        if (n + e < S.N) {
-          const float z = v[e] + S.bias[n + e];
-          v[e] = expf(S.alpha * (fminf(z, 0.f) - log1pf(expf(-fabsf(z)))));
-        }
+        if (n + e < S.N) v[e] = lin_sigpow(v[e] + S.bias[n + e], S.alpha);
       break;
     case LE_SOFTCAP:
 #pragma unroll
@@ -213,7 +226,7 @@ DEVI void lin_store4(const LinSeg& S, int grp, int n, int yr, f32x4 v) {
     }
     default: break;
   }
-  const size_t o = (size_t)yr * S.ldy + (size_t)grp * S.ygs + (size_t)nb * S.cstep + nr;
+  const size_t o = (size_t)yr * S.ldy + (size_t)grp * S.ygs + (size_t)nb * S.cstep + nr + (size_t)ks * S.yks;
   const bool full = n + 4 <= S.N && (o & 3) == 0;
   if (S.yact && sizeof(T) == 2) {
     __bf16* y = reinterpret_cast<__bf16*>(S.y) + o;
@@ -246,11 +259,12 @@ inline int lin_count(LinArgs& a, int BN, int BM) {
     if ((S.epi == LE_DECAY || S.epi == LE_SIGPOW) && !S.bias) return -1;
     if (S.epi == LE_GEGLU && ((S.N & 1) || S.cb < S.N)) return -1;
     if (S.epi == LE_GATE && !S.gate) return -1;
+    if (S.ks < 1 || S.ks > S.nsub / 2 || (S.ks > 1 && (S.rows || S.yact || S.epi != LE_NONE))) return -1;
     if (S.rows && (!a.tiles || !a.ntiles || a.maxtiles < 1)) return -1;
     if (!S.rows && S.M < 1) return -1;
     a.begin[i] = n;
     a.nmt[i] = S.rows ? a.maxtiles : (S.M + BM - 1) / BM;
-    n += ((S.N + BN - 1) / BN) * a.nmt[i] * (S.rows ? 1 : S.ng);
+    n += ((S.N + BN - 1) / BN) * a.nmt[i] * (S.rows ? 1 : S.ng * S.ks);
   }
   a.begin[a.nseg] = n;
   return n;

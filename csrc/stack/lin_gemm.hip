@@ -45,7 +45,8 @@ __global__ __launch_bounds__(64 * WN * WM) void lin_gemm_kernel(LinArgs a, int n
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int r = lane & 15, g = lane >> 4;
   const int wn = wave / WM, wm = wave % WM;
-  const int nsub = S.nsub, nst = nsub >> 1;
+  const int nsub = S.nsub;
+  const int jb = (nsub >> 1) * t.ks / S.ks, nst = (nsub >> 1) * (t.ks + 1) / S.ks - jb;     // this split's steps
   const int nwt = (S.N + 15) >> 4;
 
   const uint8_t* wbase = (const uint8_t*)S.w + (size_t)t.grp * S.wstride + lane * 16;
@@ -67,7 +68,7 @@ __global__ __launch_bounds__(64 * WN * WM) void lin_gemm_kernel(LinArgs a, int n
   const uint32_t wl = base + (uint32_t)(NW * wave) * 1024u;
   const uint32_t xl = base + G::WST + (uint32_t)(NX * wave) * 1024u;
   auto dma = [&](int j) __attribute__((always_inline)) {     // step j (clamped) -> stage j % NST
-    const int jc = min(j, nst - 1);
+    const int jc = jb + min(j, nst - 1);
     const uint32_t so = (uint32_t)(j % NST) * G::STG;
 #pragma unroll
     for (int i = 0; i < NW; ++i) glds16(wsrc[i] + (size_t)jc * 2048, wl + so + i * 1024);
@@ -117,7 +118,7 @@ __global__ __launch_bounds__(64 * WN * WM) void lin_gemm_kernel(LinArgs a, int n
     int xr, yr;
     lin_row(S, t, row, xr, yr);
 #pragma unroll
-    for (int i = 0; i < NTW; ++i) lin_store4<T>(S, t.grp, t.n0 + 16 * (wn * NTW + i) + 4 * g, yr, acc[i][j]);
+    for (int i = 0; i < NTW; ++i) lin_store4<T>(S, t.grp, t.ks, t.n0 + 16 * (wn * NTW + i) + 4 * g, yr, acc[i][j]);
   }
 }
 

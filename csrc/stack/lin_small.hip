@@ -17,6 +17,7 @@ __global__ __launch_bounds__(64 * NW) void lin_small_kernel(LinArgs a) {
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int r = lane & 15, g = lane >> 4;
   const int nsub = S.nsub, nwt = (S.N + 15) >> 4;
+  const int kb = nsub * t.ks / S.ks, ke = nsub * (t.ks + 1) / S.ks;         // this split's sub-tiles
   const uint8_t* wp[RT];
 #pragma unroll
   for (int q = 0; q < RT; ++q)               // (a tile past the matrix: its last one again, not stored)
@@ -33,8 +34,8 @@ __global__ __launch_bounds__(64 * NW) void lin_small_kernel(LinArgs a) {
   for (int q = 0; q < RT; ++q)
 #pragma unroll
     for (int i = 0; i < MT; ++i) acc[q][i] = f32x4{0.f, 0.f, 0.f, 0.f};
-  int k = wave;
-  for (; k + (U - 1) * NW < nsub; k += U * NW) {
+  int k = kb + wave;
+  for (; k + (U - 1) * NW < ke; k += U * NW) {
     u32x4 w[U][RT], x[U][MT];
 #pragma unroll
     for (int u = 0; u < U; ++u)
@@ -51,7 +52,7 @@ __global__ __launch_bounds__(64 * NW) void lin_small_kernel(LinArgs a) {
 #pragma unroll
         for (int i = 0; i < MT; ++i) acc[q][i] = L::mma(w[u][q], x[u][i], acc[q][i]);
   }
-  for (; k < nsub; k += NW) {
+  for (; k < ke; k += NW) {
 #pragma unroll
     for (int i = 0; i < MT; ++i) {
       const u32x4 x = ld16(xp[i] + (size_t)k * L::KS);
@@ -72,7 +73,7 @@ __global__ __launch_bounds__(64 * NW) void lin_small_kernel(LinArgs a) {
     if (16 * i + r < t.cnt) {
       int xr, yr;
       lin_row(S, t, 16 * i + r, xr, yr);
-      lin_store4<T>(S, t.grp, t.n0 + 16 * q + 4 * g, yr, v);
+      lin_store4<T>(S, t.grp, t.ks, t.n0 + 16 * q + 4 * g, yr, v);
     }
   }
 }

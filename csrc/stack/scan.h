@@ -10,7 +10,7 @@
 // A run = (first row, tokens, state slot, first position): consecutive rows of one sequence. A run at position 0
 // starts from a zero state, any other from its slot; slot < 0 or 0 tokens: nothing to do (padded decode rows).
 #pragma once
-#include "../kernels/common.h"
+#include "lin.h"
 
 namespace nls_scan {
 
@@ -42,6 +42,11 @@ struct Scan {
   long ld, ldw, ldo, sstride, ldx, ldp;
   int H, D, V, width;
   float rs;                // gla: factor of the output
+  // gla step with the decays' last projection: w = sigmoid(a2 low + b)^ia (w above null)
+  const void *low, *a2;    // [rows][ld], [H * D][rank]
+  const float* a2b;
+  int rank;
+  float ia;
 };
 
 // ---- one token per run: the state of (run, head) is read and written once, 4 value columns per thread; then
@@ -63,7 +68,22 @@ __global__ __launch_bounds__(256) void step_kernel(Scan p, const float* __restri
     const float r = ld1((const T*)p.r + (size_t)t * p.ld + hb + tid), k = ld1((const T*)p.k + (size_t)t * p.ld + hb + tid);
     rs[tid] = KIND == GLA ? r * p.rs : r;
     ks[tid] = k;
-    ws[tid] = p.w[(size_t)t * p.ldw + hb + tid];
+    if (KIND == WKV || p.w) {
+      ws[tid] = p.w[(size_t)t * p.ldw + hb + tid];
+    } else {
+      const T *lo = (const T*)p.low + (size_t)t * p.ld, *a2 = (const T*)p.a2 + (hb + tid) * p.rank;
+      float z = p.a2b[hb + tid];
+      int i = 0;
+      if ((p.rank & 7) == 0)                     // (16-byte aligned rows)
+        for (; i < p.rank; i += 8) {
+          typedef T t8 __attribute__((ext_vector_type(8)));
+          const t8 x = *reinterpret_cast<const t8*>(lo + i), y = *reinterpret_cast<const t8*>(a2 + i);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) z = fmaf((float)x[e], (float)y[e], z);
+        }
+      for (; i < p.rank; ++i) z = fmaf((float)lo[i], (float)a2[i], z);
+      ws[tid] = nls_lin::lin_sigpow(z, p.ia);
+    }
     if (KIND == WKV) ruk = r * p.u[hb + tid] * k;
   }
   for (int i = tid; i < V; i += 256) vs[i] = ld1((const T*)p.v + (size_t)t * p.ld + hv + i);

@@ -64,7 +64,7 @@ __global__ __launch_bounds__(256) void embed_kernel(int* __restrict__ ids, const
   }
 }
 
-// ---- x[t] += norm(y) * w (w null: x[t] += y); y = one row, or (topk) sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t],
+// ---- x[t] += norm(y) * w (w null: x[t] += y); y = one row (the sum of `nslab` slabs' rows), or (topk) sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t],
 // the shared expert); y null: x is only read. Optional second norm (the next sublayers' or the model's last one) of the
 // new x into `on`. norm: (v - mean) / sqrt(var + eps), or (rms) v / sqrt(mean(v^2) + eps).
 // A workgroup per row (`rows`: gathered), 4 consecutive columns x NV per thread in registers.
@@ -81,6 +81,8 @@ struct NormAdd {
   long sh0;             // first shared-expert row, -1: none
   int D, topk, f32, rms;
   float eps;
+  int nslab;
+  long slab;            // elements between slabs
 };
 
 // 4 consecutive values, columns i .. i + 3 of a row of D (VEC: D and the row strides are multiples of 4)
@@ -168,6 +170,10 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
     } else {
 #pragma unroll
       for (int j = 0; j < NV; ++j) v[j] = row4<VEC>(p.y + (size_t)t * p.ldy, (threadIdx.x + j * NTH) * 4, D);
+#pragma unroll 4
+      for (int s = 1; s < p.nslab; ++s)
+#pragma unroll
+        for (int j = 0; j < NV; ++j) v[j] += row4<VEC>(p.y + s * p.slab + (size_t)t * p.ldy, (threadIdx.x + j * NTH) * 4, D);
     }
     if (p.w) normalise<NV, NTH>(v, D, p.eps, p.rms, sh);
 #pragma unroll
@@ -295,6 +301,86 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnRows p) {
   put(k, p.kn, ik, p.G, (T*)p.kc + (size_t)slot * p.ldc);
   T* vo = (T*)p.vc + (size_t)slot * p.ldc;
   for (int e = threadIdx.x; e < p.G * D; e += 256) vo[(size_t)(e / D) * p.Dp + e % D] = (T)v[e];
+}
+
+// the same for heads of a multiple of 4 columns: the row's q and k stay in registers, NV groups of 4 columns per thread
+template <typename T, int NV, int NTH>
+__global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
+  __shared__ float sh[2][NTH / 64];
+  typedef T t4 __attribute__((ext_vector_type(4)));
+  const int t = blockIdx.x, D4 = p.D >> 2, nq = p.H * D4, n = nq + p.G * D4, slot = p.slot[t];
+  const float *q = p.q + (size_t)t * p.ldq, *k = p.k + (size_t)t * p.ldq, *v = p.v + (size_t)t * p.ldq;
+  const float* f = p.cs + (size_t)p.pos[t] * p.rot;
+  f32x4 x[NV];
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int e = threadIdx.x + j * NTH;
+    x[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (e < n) x[j] = *reinterpret_cast<const f32x4*>(e < nq ? q + 4 * e : k + 4 * (e - nq));
+    const float s = (x[j][0] * x[j][0] + x[j][1] * x[j][1]) + (x[j][2] * x[j][2] + x[j][3] * x[j][3]);
+    if (e < nq) sq += s;
+    else sk += s;
+  }
+  sq = wsum(sq);
+  sk = wsum(sk);
+  if ((threadIdx.x & 63) == 0) {
+    sh[0][threadIdx.x >> 6] = sq;
+    sh[1][threadIdx.x >> 6] = sk;
+  }
+  __syncthreads();
+  sq = sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < NTH / 64; ++i) {
+    sq += sh[0][i];
+    sk += sh[1][i];
+  }
+  const float iq = 1.f / sqrtf(sq / (float)(4 * nq) + p.eps), ik = 1.f / sqrtf(sk / (float)(4 * (n - nq)) + p.eps);
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int e = threadIdx.x + j * NTH;
+    if (e >= n) continue;
+    const bool isq = e < nq;
+    const int i = isq ? e : e - nq, h = i / D4, c = 4 * (i - h * D4);
+    if (!isq && slot < 0) continue;
+    f32x4 y = x[j];
+    const float* w = isq ? p.qn : p.kn;
+    if (w) y = y * (isq ? iq : ik) * *reinterpret_cast<const f32x4*>(w + 4 * i);
+#pragma unroll
+    for (int u = 0; u < 4; u += 2)
+      if (c + u < p.rot) {
+        const float cc = f[c + u], ss = f[c + u + 1], a = y[u], b = y[u + 1];
+        y[u] = a * cc - b * ss;
+        y[u + 1] = b * cc + a * ss;
+      }
+    const t4 o = {(T)y[0], (T)y[1], (T)y[2], (T)y[3]};
+    if (isq) {
+      *reinterpret_cast<t4*>((T*)p.qo + (size_t)t * p.ldqo + (size_t)h * p.Dp + c) = o;
+    } else {
+      const size_t d = (size_t)slot * p.ldc + (size_t)h * p.Dp + c;
+      *reinterpret_cast<t4*>((T*)p.kc + d) = o;
+      const f32x4 z = p.v == p.k ? x[j] : *reinterpret_cast<const f32x4*>(v + 4 * i);
+      *reinterpret_cast<t4*>((T*)p.vc + d) = t4{(T)z[0], (T)z[1], (T)z[2], (T)z[3]};
+    }
+  }
+}
+
+template <typename T>
+int attn_rows_t(const AttnRows& p, int n, hipStream_t st) {
+  const int cols = (p.H + p.G) * p.D;
+  const bool vec = !(p.D & 3) && !(p.ldq & 3) && !(p.Dp & 3) && !(p.ldqo & 3) && !(p.ldc & 3) &&
+                   !(((uintptr_t)p.q | (uintptr_t)p.k | (uintptr_t)p.v) & 15);
+#define NLS_AR(NV, NTH) \
+  if (vec && cols <= 4 * NV * NTH) { \
+    hipLaunchKernelGGL((attn_rows4_kernel<T, NV, NTH>), dim3(n), dim3(NTH), 0, st, p); \
+    return (int)hipGetLastError(); \
+  }
+  NLS_AR(1, 256)
+  if (n <= 64) { NLS_AR(1, 1024) NLS_AR(2, 1024) }
+  NLS_AR(2, 256) NLS_AR(5, 256) NLS_AR(8, 256) NLS_AR(8, 1024)
+#undef NLS_AR
+  hipLaunchKernelGGL(attn_rows_kernel<T>, dim3(n), dim3(256), 0, st, p);
+  return (int)hipGetLastError();
 }
 
 // ---- expert choice of one token: sigmoid scores, the `keep` groups with the largest sum of their two best scores, the
@@ -473,9 +559,11 @@ int nls_stack_embed(int* ids, const int* next_ids, const int* use_prev, const vo
 }
 
 int nls_norm_add(const float* y, long ldy, const float* topw, int topk, long sh0, const float* w, float* x, void* xb,
-                 long ldx, const float* ow, void* on, long ldo, int D, int T, float eps, int f32, int rms, void* stream) {
-  if (!y) return -1;
-  return norm_add(NormAdd{y, topw, w, x, (__bf16*)xb, ow, on, nullptr, ldy, ldx, ldo, sh0, D, topk, f32, rms, eps}, T,
+                 long ldx, const float* ow, void* on, long ldo, int D, int T, float eps, int f32, int rms, int nslab, long slab,
+                 void* stream) {
+  if (!y || nslab < 1 || (slab & 3)) return -1;
+  return norm_add(NormAdd{y, topw, w, x, (__bf16*)xb, ow, on, nullptr, ldy, ldx, ldo, sh0, D, topk, f32, rms, eps, nslab, slab},
+                  T,
                   (hipStream_t)stream);
 }
 
@@ -483,7 +571,7 @@ int nls_norm_add(const float* y, long ldy, const float* topw, int topk, long sh0
 int nls_row_norm(const float* x, long ldx, const int* rows, const float* w, void* out, long ldo, int D, int n,
                  float eps, int f32, int rms, void* stream) {
   return norm_add(NormAdd{nullptr, nullptr, nullptr, const_cast<float*>(x), nullptr, w, out, rows, 0, ldx, ldo, -1, D, 0,
-                          f32, rms, eps}, n, (hipStream_t)stream);
+                          f32, rms, eps, 1, 0}, n, (hipStream_t)stream);
 }
 
 int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq, long ldcq, const float* dkv,
@@ -506,9 +594,7 @@ int nls_attn_rows(const float* q, const float* k, const float* v, long ldq, cons
   if (T < 1 || H < 1 || G < 1 || D < 1 || Dp < D || (rot & 1) || rot < 0 || rot > D || (long)H * Dp > ldqo || (long)G * Dp > ldc)
     return -1;
   AttnRows p{q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, ldq, ldqo, ldc, H, G, D, Dp, rot, eps};
-  if (f32) hipLaunchKernelGGL(attn_rows_kernel<float>, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
-  else hipLaunchKernelGGL(attn_rows_kernel<__bf16>, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
-  return (int)hipGetLastError();
+  return f32 ? attn_rows_t<float>(p, T, (hipStream_t)stream) : attn_rows_t<__bf16>(p, T, (hipStream_t)stream);
 }
 
 int nls_stack_argmax(const float* z, long ldz, int V, int* out, int n, void* stream) {

@@ -227,7 +227,8 @@ int scan_t(const Scan& p, int nruns, hipStream_t st) {
 
 Scan args(const void* r, const void* k, const void* v, long ld, const float* w, long ldw, const float* u, float* o, long ldo,
           float* state, long sstride, const float* x, long ldx, float* prev, long ldp, int width, const int* runs, int H, int D) {
-  return Scan{r, k, v, w, u, o, state, x, prev, runs, ld, ldw, ldo, sstride, ldx, ldp, H, D, D, width, 1.f};
+  return Scan{r, k, v, w, u, o, state, x, prev, runs, ld, ldw, ldo, sstride, ldx, ldp, H, D, D, width, 1.f, nullptr, nullptr, nullptr, 0,
+              0.f};
 }
 
 }  // namespace nls_wkv

@@ -27,6 +27,7 @@ from .stack_config import StackConfig
 
 _SPLIT_WG = 256          # target workgroups of a decode attention launch (one per CU)
 _SPLIT_CAP = 64
+_SLABS, _SLAB_ROWS = 8, 512      # K splits of an output product, on steps of up to so many rows
 
 
 @dataclass
@@ -47,12 +48,16 @@ class StackBuffers:
     x: torch.Tensor                     # f32 residual
     xb: Optional[torch.Tensor]          # its bf16 rounding (None: 32-bit model, the residual itself is the operand)
     h: Optional[torch.Tensor]           # normed residual that the sublayers read (None: they read the residual)
-    y: torch.Tensor                     # f32 sublayer output
+    y: Optional[torch.Tensor]           # f32 sublayer output (layers with a shared norm: the slabs of their output product)
     hn: torch.Tensor                    # normed rows of the head
     logits: torch.Tensor
     next_ids: torch.Tensor
     shared: Dict[tuple, torch.Tensor] = field(default_factory=dict)    # scratch shared between layers
     launches: Dict[tuple, object] = field(default_factory=dict)
+
+    @property
+    def slab_rows(self) -> int:
+        return min(self.pad, _SLAB_ROWS)
 
     @property
     def act(self) -> torch.Tensor:
@@ -413,6 +418,8 @@ class GlaPart(_SharedPart):
         self.qkva = self.lin(torch.cat([qkv, qkv.new_zeros(self.low - qkv.shape[0], d), a1]))
         self.ld = self.low + K.act_ld(a1.shape[0])
         self.a2, self.a2b = self.lin("a2", (H * D, a1.shape[0])), self.vecn("a2.b", H * D)
+        # decode steps make the decays themselves (a row-major copy of a2) unless the rank is large
+        self.a2r = self.t("a2").to(device=model.device, dtype=model.dtype).contiguous() if a1.shape[0] <= 64 else None
         self.g = self.lin("g", (H * V, d))
         self.norm = (self.vecn("norm", V) * scale).repeat(H).contiguous()
         self.out_width = K.act_ld(H * V)
@@ -432,16 +439,19 @@ class GlaPart(_SharedPart):
         a = self.scratch(b, "gla.a", P, HD, f)
         o = self.scratch(b, "gla.o", P, HV, f) if c.vdim > 128 else None
         g = self.scratch(b, "gla.g", P, HV)
-        return dict(q=z, k=z[:, HD:], v=z[:, 2 * HD:], a=a, o=o, g=g, out=out,
+        return dict(q=z, k=z[:, HD:], v=z[:, 2 * HD:], low=z[:, self.low:], a=a, o=o, g=g, out=out,
                     inputs=[K.Seg(self.qkva, b.act, z), K.Seg(self.g, b.act, g, "silu")],
                     decay=K.LinLaunch([K.Seg(self.a2, z, a, "sigpow", xcol=self.low, bias=self.a2b, alpha=1.0 / c.tau)]))
 
     def run(self, b, e, cache, state, step: "_Step"):
         c, st, T, eps = self.cfg, step.st, step.T, self.m.cfg.eps
         H, D, V, S, qs = c.heads, c.dim, c.vdim, state["S"], c.dim ** -0.5
-        e["decay"].run(T, st)
-        if T == step.nruns and V % 4 == 0 and V <= 1024:      # single tokens only
-            K.gla_step(e["q"], e["k"], e["v"], e["a"], qs, S, b.runs, T, self.norm, e["g"], e["out"], H, D, V, eps, st)
+        single = T == step.nruns and V % 4 == 0 and V <= 1024
+        a = None if single and self.a2r is not None else e["a"]
+        if a is not None:
+            e["decay"].run(T, st)
+        if single:
+            K.gla_step(e["q"], e["k"], e["v"], a, (e["low"], self.a2r, self.a2b, 1.0 / c.tau), qs, S, b.runs, T, self.norm, e["g"], e["out"], H, D, V, eps, st)
             return
         n = step.nruns
         shape = K.gla_shape(T, n, H, V)
@@ -539,7 +549,12 @@ class SharedNormLayer:
             c0 += w
         b.launches[key, "parts"] = e
         b.launches[key, "in"] = [K.LinLaunch(segs[o:o + K.SEGS]) for o in range(0, len(segs), K.SEGS)]
-        b.launches[key, "out"] = K.LinLaunch([K.Seg(self.o, cat, b.y)])
+        # small steps may split K: slabs of up to 512 rows, added by the residual's launch
+        rows = max(b.pad, _SLABS * b.slab_rows)
+        y = b.shared.get("slabs")
+        if y is None:
+            y = b.shared["slabs"] = torch.zeros(rows, self.m.cfg.d_model, dtype=torch.float32, device=self.m.device)
+        b.launches[key, "out"] = K.LinLaunch([K.Seg(self.o, cat, y, slabs=_SLABS, slab_rows=b.slab_rows)])
 
     def new_caches(self, slots):
         return {j: q.new_cache(slots) for j, q in enumerate(self.parts) if q.cache_width}
@@ -550,8 +565,9 @@ class SharedNormLayer:
             launch.run(step.T, step.st)
         for j, (q, e) in enumerate(zip(self.parts, b.launches[key, "parts"])):
             q.run(b, e, kc[step.layer].get(j), state, step)
-        b.launches[key, "out"].run(step.T, step.st)
-        K.norm_add(b.y, None, b.x, None, step.T, cfg.eps, step.st, rms=cfg.design.norm == "rms", **fin)
+        n = b.launches[key, "out"].run(step.T, step.st)
+        K.norm_add(b.shared["slabs"], None, b.x, None, step.T, cfg.eps, step.st, rms=cfg.design.norm == "rms", slabs=n,
+                   slab_rows=b.slab_rows, **fin)
 
 
 def mixer_parts(c) -> list:
@@ -692,7 +708,7 @@ class StackModel:
             use_prev=seg[5], block_tables=meta[6 * pad:6 * pad + nb].view(max_seqs, max_blocks),
             runs=meta[6 * pad + nb:].view(max_seqs, 4),
             x=torch.zeros(pad, ld, **f), xb=None if self.f32 or shared else act(), h=act() if shared else None,
-            y=torch.zeros(pad, cfg.d_model, **f), hn=act(),
+            y=None if shared else torch.zeros(pad, cfg.d_model, **f), hn=act(),
             logits=torch.zeros(nl, cfg.vocab, **f), next_ids=torch.zeros(pad, dtype=torch.int32, device=dev))
         b.slot.fill_(-1)
         b.runs[:, 2] = -1

@@ -23,9 +23,10 @@ NO_BLOCK = 1 << 30       # LinSeg.cb: output columns are not blocked
 class LinSeg(ctypes.Structure):
     """csrc/stack/lin.h LinSeg."""
     _fields_ = [("w", P), ("x", P), ("y", P), ("bias", P), ("gate", P), ("cs", P), ("pos", P), ("rows", P), ("xmap", P),
-                ("wstride", L), ("ldx", L), ("ldy", L), ("xgs", L), ("ygs", L),
+                ("wstride", L), ("ldx", L), ("ldy", L), ("xgs", L), ("ygs", L), ("yks", L),
                 ("N", I), ("nsub", I), ("M", I), ("ng", I), ("epi", I), ("yact", I), ("cb", I), ("cstep", I),
-                ("xdiv", I), ("ldg", I), ("half", I), ("alpha", F)]
+                ("xdiv", I), ("ldg", I), ("half", I), ("alpha", F),
+                ("ks", I), ("pad0", I)]
 
 
 class LinArgs(ctypes.Structure):
@@ -38,13 +39,13 @@ _SIGS = {
     "nls_lin_small": [P, I, I, I, I, P],
     "nls_lin_gemm": [P, I, I, P],
     "nls_stack_embed": [P, P, P, P, I, I, F, P, P, L, I, P],
-    "nls_norm_add": [P, L, P, I, L, P, P, P, L, P, P, L, I, I, F, I, I, P],
+    "nls_norm_add": [P, L, P, I, L, P, P, P, L, P, P, L, I, I, F, I, I, I, L, P],
     "nls_row_norm": [P, L, P, P, P, L, I, I, F, I, I, P],
     "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, F, I, P],
     "nls_gqa_attn": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, P, L, P, L, P, P, P, I, I, P],
     "nls_gqa_prefill": [P, L, P, P, P, P, I, P, I, P, L, I, I, I, I, F, P],
     "nls_gla_scan": [P, P, P, L, P, L, F, P, L, P, P, L, P, L, F, P, L, P, I, I, I, I, I, P, P, I, I, P],
-    "nls_gla_step": [P, P, P, L, P, L, F, P, L, P, I, P, P, L, P, L, I, I, I, F, I, P],
+    "nls_gla_step": [P, P, P, L, P, L, P, P, P, I, F, F, P, L, P, I, P, P, L, P, L, I, I, I, F, I, P],
     "nls_latent_rows": [P, L, I, P, P, L, P, L, I, I, I, P, P, P, P, P, L, I, F, I, P],
     "nls_stack_argmax": [P, L, I, P, I, P],
     "nls_moe_plan": [P, L, I, I, I, I, I, F, P, P, I, P, P, P, I, P],
@@ -133,11 +134,12 @@ class Seg:
     xgs / ygs: column step per group. block = (cb, cstep): output column n -> (n / cb) * cstep + n % cb.
     routed = (entry list, xdiv): the rows are routed entries (x row = entry / xdiv, y row = entry).
     rope = (table, pos, pairs). alpha: constant of the epilogue (sigmoid, sigpow, softcap). geglu: the rows of w alternate
-    gate and up, y has half as many columns."""
+    gate and up, y has half as many columns. slabs: K splits that launches of up to slab_rows rows may use; y holds that many
+    slabs of slab_rows rows, added by the caller (LinLaunch.run returns how many were written)."""
 
     def __init__(self, w: PackedLinear, x: torch.Tensor, y: torch.Tensor, epi: str = "none", ycol: int = 0,
                  xcol: int = 0, xgs: int = 0, ygs: int = 0, block=None, bias=None, gate=None, routed=None, rope=None,
-                 yrow: int = 0, xmap: Optional[torch.Tensor] = None, alpha: float = 1.0):
+                 yrow: int = 0, xmap: Optional[torch.Tensor] = None, alpha: float = 1.0, slabs: int = 1, slab_rows: int = 0):
         if x.stride(1) != 1 or y.stride(1) != 1:
             raise ValueError("row-major operands")
         if xcol + (0 if routed else (w.groups - 1) * xgs) + act_ld(w.K) > x.stride(0):
@@ -167,13 +169,18 @@ class Seg:
             s.cs, s.pos, s.half = rope[0].data_ptr(), rope[1].data_ptr(), rope[2]
         s.xmap = _p(xmap)
         s.alpha = alpha
+        if slabs * slab_rows > y.shape[0]:
+            raise ValueError("y does not hold the slabs")
+        s.ks, self.slabs, self.slab_rows = 1, slabs, slab_rows
+        s.yks = slab_rows * y.stride(0)
         self.keep = (bias, gate, routed, rope, xmap)
 
 
 GEMM_TILES = ((64, 64), (128, 64), (128, 128), (256, 128), (256, 256), (64, 64))     # (weight rows, rows) of lin_gemm's cfg
 
 
-GEMM_RATE = {4: 1.0, 3: 0.95, 2: 0.75, 1: 0.55, 0: 0.4}      # relative multiply rates of the tiles
+# relative multiply rates of the tiles: (up to so many workgroups, below, above); the small tiles run two or more to a CU
+GEMM_RATE = {4: (0, 0.96, 0.96), 3: (0, 1.0, 1.0), 2: (256, 0.47, 0.72), 1: (512, 0.5, 0.63), 0: (1024, 0.45, 0.55)}
 
 
 class LinLaunch:
@@ -221,16 +228,33 @@ class LinLaunch:
             if n64 >= 250:
                 return True, 0
             return False, 2, (4 if ns <= 16 else 8), (2 if M > 32 or n16 >= 640 else 1)
+        if ns <= 4:                       # a step or two of K: all epilogue
+            return True, (0 if M <= 2048 else 1)
         if n64 < 96 and n16 <= 1024:
             return False, 1, 16, 1
         if M <= 512:
             return True, (3 if self._tiles(256, 128, M) >= 120 else 5 if n64 <= 256 else 0)
-        # compute-bound: rounds of 256 workgroups times a tile's cost (the small tiles run two to a CU)
-        cost = {c: -(-self._tiles(*GEMM_TILES[c], M) // 256) * GEMM_TILES[c][0] * GEMM_TILES[c][1] / GEMM_RATE[c]
-                for c in GEMM_RATE}
-        return True, min(cost, key=cost.get)
+        # compute-bound: rounds of 256 workgroups times a tile's cost
+        def cost(c):
+            n, (few, lo, hi) = self._tiles(*GEMM_TILES[c], M), GEMM_RATE[c]
+            return -(-n // 256) * GEMM_TILES[c][0] * GEMM_TILES[c][1] / (lo if n <= few else hi)
+        return True, min(GEMM_RATE, key=cost)
 
-    def run(self, M: int, st: int):
+    def split_config(self, M: int):
+        """(config, K splits) of a launch that may split K: about 512 workgroups of 64 x 64 tiles, or 256 of 256 x 128."""
+        n16 = self._tiles(16, 16, M)
+        if M <= 16:
+            rt = 1 if M <= 8 else 2
+            return (False, 1, 8, rt), -(-512 * rt // (2 * n16)) if M > 8 else -(-512 // n16)
+        if M <= 32:
+            return (False, 2, 4, 4 if n16 >= 256 else 2), 8
+        big, small = self._tiles(256, 128, M), self._tiles(64, 64, M)
+        if M > 128 and big * 8 >= 256:
+            return (True, 3), -(-256 // big)
+        return (True, 0), -(-512 // small)
+
+    def run(self, M: int, st: int) -> int:
+        """Returns the slabs of output rows that were written (1 unless a segment may split K)."""
         if self.plan is not None:
             self.a.maxtiles = self.plan.max_tiles(M)
         for i, s in enumerate(self.segs):
@@ -241,11 +265,20 @@ class LinLaunch:
         if cfg is None:
             if len(self._cfg) > 4096:
                 self._cfg.clear()
-            cfg = self._cfg[M] = self.config(M)
+            s = self.segs[0]
+            if s.slabs > 1 and len(self.segs) == 1 and M <= s.slab_rows and s.w.nsub >= 64:
+                cfg, ks = self.split_config(M)
+                cfg = cfg, max(1, min(ks, s.slabs, s.w.nsub // 16))
+            else:
+                cfg = self.config(M), 1
+            self._cfg[M] = cfg
+        cfg, ks = cfg
+        self.a.s[0].ks = ks
         if cfg[0]:
             _check(lib().nls_lin_gemm(ctypes.byref(self.a), self.f32, cfg[1], st), "nls_lin_gemm")
         else:
             _check(lib().nls_lin_small(ctypes.byref(self.a), self.f32, *cfg[1:], st), "nls_lin_small")
+        return ks
 
 
 class MoePlan:
@@ -297,15 +330,16 @@ def embed(ids, table: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor],
 
 def norm_add(y: torch.Tensor, w: Optional[torch.Tensor], x: torch.Tensor, xb: Optional[torch.Tensor], T: int, eps: float,
              st: int, plan: Optional[MoePlan] = None, shared_row0: int = -1, out_norm: Optional[torch.Tensor] = None,
-             out: Optional[torch.Tensor] = None, rms: bool = False):
-    """x[:T] += norm(y) * w, or += y without w (xb: its bf16 rounding). With `plan`, y holds the routed experts' rows
+             out: Optional[torch.Tensor] = None, rms: bool = False, slabs: int = 1, slab_rows: int = 0):
+    """x[:T] += norm(y) * w, or += y without w (xb: its bf16 rounding); y may be the sum of `slabs` blocks of slab_rows rows. With `plan`, y holds the routed experts' rows
     (token-major) and from row `shared_row0` on the shared expert's, combined first. out = norm(x) * out_norm (what the next
     sublayers read, or the model's last norm). norm: layer norm, or RMS."""
     D = y.shape[1] if w is None else w.numel()
     _check(lib().nls_norm_add(y.data_ptr(), y.stride(0), _p(plan.topw) if plan else None, plan.top if plan else 0,
                               shared_row0, _p(w), x.data_ptr(), _p(xb), x.stride(0), _p(out_norm), _p(out),
                               out.stride(0) if out is not None else 0, D, T, eps,
-                              int(out is not None and out.dtype == torch.float32), int(rms), st), "nls_norm_add")
+                              int(out is not None and out.dtype == torch.float32), int(rms), slabs,
+                              slab_rows * y.stride(0), st), "nls_norm_add")
 
 
 def row_norm(x: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor, out: torch.Tensor, n: int, eps: float,
@@ -439,12 +473,15 @@ def gla_scan(q, k, v, a, qscale: float, o, norm, gate, out, state, runs, nruns: 
                               int(q.dtype == torch.float32), st), "nls_gla_scan")
 
 
-def gla_step(q, k, v, a, qscale: float, state, runs, nruns: int, norm, gate, out, H: int, D: int, V: int, eps: float, st: int):
-    """gla_scan and scan_out of runs of one token each (V a multiple of 4)."""
-    _check(lib().nls_gla_step(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), a.data_ptr(), a.stride(0), qscale,
-                              state.data_ptr(), state.stride(0), runs.data_ptr(), nruns, norm.data_ptr(), gate.data_ptr(),
-                              gate.stride(0), out.data_ptr(), out.stride(0), H, D, V, eps, int(out.dtype == torch.float32),
-                              st), "nls_gla_step")
+def gla_step(q, k, v, a, gate_in, qscale: float, state, runs, nruns: int, norm, gate, out, H: int, D: int, V: int, eps: float,
+             st: int):
+    """gla_scan of runs of one token each (V a multiple of 4), with the norm and gate. Decays `a`, or (None) from gate_in =
+    (low-rank gate input, a2, bias, exponent): sigmoid(a2 low + bias) ^ exponent."""
+    lo, a2, b, ia = gate_in if a is None else (None, None, None, 0.0)
+    _check(lib().nls_gla_step(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), _p(a), a.stride(0) if a is not None else 0,
+                              _p(lo), _p(a2), _p(b), a2.shape[1] if a2 is not None else 0, ia, qscale, state.data_ptr(),
+                              state.stride(0), runs.data_ptr(), nruns, norm.data_ptr(), gate.data_ptr(), gate.stride(0),
+                              out.data_ptr(), out.stride(0), H, D, V, eps, int(out.dtype == torch.float32), st), "nls_gla_step")
 
 
 # ---------------------------------------------------------------------------

@@ -61,6 +61,25 @@ def test_linear_epilogues(K, dt, M, N):
     assert (ys[0][:, 0] == 1).all() and torch.isfinite(ys[0]).all()
 
 
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("M", [1, 5, 13, 30, 64, 100, 256, 300])
+def test_split_products(K, dt, M):
+    """A product whose K is split over workgroups, and the residual add over its slabs."""
+    d, N, Kd, R = DT[dt], 100, 4200, 320
+    w, x, res = (rnd(N, Kd, seed=1) / math.sqrt(Kd)).to(d), rnd(M, Kd, seed=2).to(d), rnd(M, N, seed=3).float()
+    y = torch.full((8 * R, N), 7.0, device="cuda")
+    L = K.LinLaunch([K.Seg(K.PackedLinear(w, dt == "f32", "cuda"), act(x, K.act_ld(Kd), d), y, slabs=8, slab_rows=R)])
+    n = L.run(M, st())
+    assert n > 1
+    xr = act(res, K.act_ld(N), torch.float32)
+    K.norm_add(y, None, xr, None, M, 1e-5, st(), slabs=n, slab_rows=R)
+    want = x.double() @ w.double().T
+    assert relerr(xr[:, :N].cpu().double() - res.double(), want) < 1e-5
+    L._cfg[M] = (L.config(M), 1)                         # not split: the first slab alone
+    y.fill_(7.0)
+    assert L.run(M, st()) == 1 and relerr(y[:M], want) < 1e-5 and (y[R:] == 7).all()
+
+
 @pytest.mark.parametrize("D", [37, 48, 1030, 4100])
 def test_embed_scale_and_rms_norms(K, D):
     T, V, eps, ld = 5, 19, 1e-2, K.act_ld(D)
@@ -286,10 +305,29 @@ def test_gla_step(K, dt, H, D, V):
         gg = torch.stack([g[0, t], g[0, t], g[1, t]]).cuda()
         out = torch.full((3, HV), 7.0, dtype=d, device="cuda")
         runs = torch.tensor([[0, 1, 2, t], [1, 0, -1, 0], [2, 1, 0, t]], dtype=torch.int32, device="cuda")
-        K.gla_step(zz, zz[:, HD:], zz[:, 2 * HD:], aa, qs, S0, runs, 3, norm, gg, out, H, D, V, eps, st())
+        K.gla_step(zz, zz[:, HD:], zz[:, 2 * HD:], aa, None, qs, S0, runs, 3, norm, gg, out, H, D, V, eps, st())
         assert relerr(out[[0, 2]], want[[t, n + t]].double().cpu()) < (3e-5 if dt == "f32" else 8e-3)
         assert (out[1] == 7).all()
     assert relerr(S0[[0, 2]], Sw[[0, 2]].double().cpu()) < 1e-6 and (S0[1] == 9).all()
+
+
+@pytest.mark.parametrize("dt", DT)
+@pytest.mark.parametrize("R", [1, 7, 16, 40])
+def test_gla_step_decays(K, dt, R):
+    """The step that makes its own decays from the low-rank gate input: the state they leave."""
+    d, T, H, D, V = DT[dt], 6, 3, 20, 8
+    HD = H * D
+    a2, b, low = rnd(HD, R, seed=1).to(d), rnd(HD, seed=2, scale=4.0).float(), rnd(T, R, seed=3).to(d)
+    b[0], b[1] = 80.0, -150.0
+    z = torch.zeros(T, 256, dtype=d, device="cuda")                   # keys are zero: the state is its decay
+    z[:, 192:192 + R] = low
+    S0 = torch.ones(T, HD * V, device="cuda")
+    runs = torch.tensor([[t, 1, t, 5] for t in range(T)], dtype=torch.int32, device="cuda")
+    out = torch.zeros(T, H * V, dtype=d, device="cuda")
+    K.gla_step(z, z[:, HD:], z[:, 2 * HD:], None, (z[:, 192:], a2.cuda(), b.cuda(), 1 / 5.0), 1.0, S0, runs, T,
+               torch.ones(H * V, device="cuda"), torch.ones(T, H * V, dtype=d, device="cuda"), out, H, D, V, 1e-5, st())
+    want = O.sigmoid(low.double() @ a2.double().T + b.double()) ** (1 / 5.0)
+    assert relerr(S0.view(T, HD, V), want[:, :, None].expand(T, HD, V)) < 1e-5
 
 
 # ---------------------------------------------------------------- one layer
@@ -335,14 +373,15 @@ def test_layer(gpu, tmp_path, dt, name, i, flash, monkeypatch):
             step.plan = m._expand_plan(b, info["qblocks"], info["row_info"], 2 * T, 16, st())
         K.row_norm(b.x, None, layer.norm1, b.h, 2 * T, cfg["norm"]["eps"], st(), rms=True)
         layer.run(b, 0, kc, state[0], step, {})
-        for r in (0, 1):
-            got[r].append(b.y[r * T:(r + 1) * T].clone())
+        for r, src in ((0, x), (1, z)):
+            got[r].append((b.x[r * T:(r + 1) * T, :d].cpu().double() - src[a:c].float().double()))
     Wd, eps, L = {k: v.double() for k, v in W.items()}, cfg["norm"]["eps"], cfg["layers"][0]
     for r, src in ((0, x), (1, z)):
         h = O.norm_one_plus(src, Wd["l0.norm1"], eps)
         want, _ = O.parallel_mixer(h, Wd, "l0.mix.", L["mixer"], torch.arange(n), eps)
         if L["mlp"]:
             want = want + O.dense_ff(h, Wd, "l0.mlp.")
+        # (read as the residual's change)
         assert relerr(torch.cat(got[r]), want) < TOL[dt] * 2, r
 
 
