@@ -33,7 +33,7 @@ struct GA {
   float* recw;             // their decay products [run][nseg][H][D]
   const int* runs;
   long ld, lda, ldo, ldg, ldout, sstride;
-  int H, D, V, nseg, fused, vec;
+  int H, D, V, nseg, fused, vec, vecq;
   float rs, eps;
 };
 
@@ -48,8 +48,9 @@ struct GC {
   static constexpr int LK = 20;                                     // scaled keys, transposed (f32),
   static constexpr int LKR = DP == 32 ? 40 : DP + 16;               // keys (in the place of the scaled ones),
   static constexpr int WC = 64 * NT, LV = WC + 8;                   // values (T)
-  static constexpr int OQ = 0, OK = OQ + SC * LQ * 4, OA = OK + NCH * DP * LK * 4, OG = OA + NCH * 16 * LK * 4,
-                       OS = OG + NCH * DP * 4, OR = OS + 4 * SC * 4, OV = OR + SC * LR * (int)sizeof(T),
+  static constexpr int LO = WC + 4;                                 // outputs (f32, in the place of queries and keys)
+  static constexpr int OQ = 0, OK = OQ + SC * LQ * 4, OE = OK + NCH * DP * LK * 4,
+                       OA = OE > SC * LO * 4 ? OE : SC * LO * 4, OG = OA + NCH * 16 * LK * 4, OS = OG + NCH * DP * 4, OR = OS + 4 * SC * 4, OV = OR + SC * LR * (int)sizeof(T),
                        LDS = OV + SC * LV * (int)sizeof(T);
   static_assert(16 * LKR <= DP * LK && LDS <= 160 * 1024, "LDS");
 };
@@ -100,56 +101,90 @@ __global__ __launch_bounds__(256, DP <= 64 ? 2 : 1) void gla_chunk_kernel(GA p) 
   const size_t seg = (size_t)blockIdx.y * p.nseg + z;
   float* st = p.state + (size_t)slot * p.sstride + hb * V;
 
+  // (loads below are never in a branch of their own: addresses are clamped and the value selected afterwards, so that they
+  // all are in flight together)
   f32x4 S[NTD][NT];                                                 // rows 16 t + 4 g + i, column wc + 16 c + r
   f32x4 pw[NTD];
+  if (LOCAL || (p.nseg == 1 && pos0 == 0)) {
 #pragma unroll
-  for (int t = 0; t < NTD; ++t) {
-    pw[t] = f32x4{1.f, 1.f, 1.f, 1.f};
+    for (int t = 0; t < NTD; ++t)
 #pragma unroll
-    for (int c = 0; c < NT; ++c)
+      for (int c = 0; c < NT; ++c) S[t][c] = f32x4{0.f, 0.f, 0.f, 0.f};
+  } else {
+    const float* src = p.nseg > 1 ? p.rec + seg * sst + hb * V : st;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int d = 16 * t + 4 * g + i, col = wc + 16 * c + r;
-        const bool in = d < D && col < V;
-        const float* src = p.nseg > 1 ? p.rec + seg * sst + hb * V : st;
-        S[t][c][i] = in && !LOCAL && (p.nseg > 1 || pos0 > 0) ? src[(size_t)d * V + col] : 0.f;
-      }
-  }
-
-  // loads of one round: chunk `wave`, a key channel per lane; values in groups of 4 columns
-  T fq[NDP][16], fk[NDP][16];
-  typedef T t4 __attribute__((ext_vector_type(4)));
-  float fa[NDP][16];
-  t4 fv[NVG];
-  auto fetch = [&](int base) __attribute__((always_inline)) {
-    if (wave < NCH)
+    for (int t = 0; t < NTD; ++t)
 #pragma unroll
-      for (int u = 0; u < NDP; ++u) {
-        const int d = lane + 64 * u;
+      for (int c = 0; c < NT; ++c)
 #pragma unroll
-        for (int t = 0; t < 16; ++t) {
-          const int tt = base + 16 * wave + t;
-          const bool in = tt < n && d < D;
-          const size_t row = (size_t)(t0 + min(tt, n - 1));
-          if (!LOCAL) fq[u][t] = in ? *((const T*)p.q + row * p.ld + hb + d) : (T)0.f;
-          fk[u][t] = in ? *((const T*)p.k + row * p.ld + hb + d) : (T)0.f;
-          fa[u][t] = in ? p.a[row * p.lda + hb + d] : 1.f;
+        for (int i = 0; i < 4; ++i) {
+          const int d = 16 * t + 4 * g + i, col = wc + 16 * c + r;
+          const float x = src[(size_t)min(d, D - 1) * V + min(col, V - 1)];
+          S[t][c][i] = d < D && col < V ? x : 0.f;
         }
-      }
+  }
 #pragma unroll
-    for (int e = 0; e < NVG; ++e) {
-      const int x = tid + 256 * e, tt = base + x / (WC / 4), col = c0 + (x % (WC / 4)) * 4;
-      const T* src = (const T*)p.v + (size_t)(t0 + min(tt, n - 1)) * p.ld + hv;
-      fv[e] = t4{(T)0.f, (T)0.f, (T)0.f, (T)0.f};
-      if (tt < n) {
-        if (p.vec) {
-          if (col < V) fv[e] = *reinterpret_cast<const t4*>(src + col);
+  for (int t = 0; t < NTD; ++t) pw[t] = f32x4{1.f, 1.f, 1.f, 1.f};
+
+  // loads of one round, in groups of 4 columns: a lane takes the channels 4 cg .. of TPL tokens of chunk `wave`
+  typedef T t4 __attribute__((ext_vector_type(4)));
+  constexpr int TPL = DP / 16;
+  const int cg = 4 * (lane % (DP / 4)), ts = TPL * (lane / (DP / 4));
+  t4 fq[TPL], fk[TPL], fv[NVG];
+  f32x4 fa[TPL];
+  auto fetch = [&](int base) __attribute__((always_inline)) {
+    if (wave < NCH) {
+      const T *qp = (const T*)p.q + hb, *kp = (const T*)p.k + hb;
+      const float* ap = p.a + hb;
+#pragma unroll
+      for (int e = 0; e < TPL; ++e) {
+        const size_t row = (size_t)(t0 + min(base + 16 * wave + ts + e, n - 1));
+        if (p.vecq) {
+          const int d = min(cg, D - 4);
+          if (!LOCAL) fq[e] = *reinterpret_cast<const t4*>(qp + row * p.ld + d);
+          fk[e] = *reinterpret_cast<const t4*>(kp + row * p.ld + d);
+          fa[e] = *reinterpret_cast<const f32x4*>(ap + row * p.lda + d);
         } else {
 #pragma unroll
-          for (int i = 0; i < 4; ++i)
-            if (col + i < V) fv[e][i] = src[col + i];
+          for (int i = 0; i < 4; ++i) {
+            const int d = min(cg + i, D - 1);
+            if (!LOCAL) fq[e][i] = qp[row * p.ld + d];
+            fk[e][i] = kp[row * p.ld + d];
+            fa[e][i] = ap[row * p.lda + d];
+          }
         }
       }
+#pragma unroll
+      for (int e = 0; e < TPL; ++e)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const bool in = base + 16 * wave + ts + e < n && cg + i < D;
+          if (!LOCAL) fq[e][i] = in ? fq[e][i] : (T)0.f;
+          fk[e][i] = in ? fk[e][i] : (T)0.f;
+          fa[e][i] = in ? fa[e][i] : 1.f;
+        }
+    }
+    const T* vp = (const T*)p.v + hv;
+    if (p.vec) {
+#pragma unroll
+      for (int e = 0; e < NVG; ++e) {
+        const int x = tid + 256 * e, col = c0 + (x % (WC / 4)) * 4;
+        fv[e] = *reinterpret_cast<const t4*>(vp + (size_t)(t0 + min(base + x / (WC / 4), n - 1)) * p.ld + min(col, V - 4));
+      }
+    } else {
+#pragma unroll
+      for (int e = 0; e < NVG; ++e) {
+        const int x = tid + 256 * e, col = c0 + (x % (WC / 4)) * 4;
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          fv[e][i] = vp[(size_t)(t0 + min(base + x / (WC / 4), n - 1)) * p.ld + min(col + i, V - 1)];
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < NVG; ++e) {
+      const int x = tid + 256 * e, col = c0 + (x % (WC / 4)) * 4;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) fv[e][i] = base + x / (WC / 4) < n && col + i < V ? fv[e][i] : (T)0.f;
     }
   };
   fetch(0);
@@ -157,18 +192,15 @@ __global__ __launch_bounds__(256, DP <= 64 ? 2 : 1) void gla_chunk_kernel(GA p) 
     // ---- this round's operands
     if (wave < NCH) {
       float* kr = kt + wave * DP * C::LK;
+      // as loaded: decays and keys (f32), queries
+#pragma unroll
+      for (int e = 0; e < TPL; ++e) {
+        *reinterpret_cast<f32x4*>(aq + (16 * wave + ts + e) * C::LQ + cg) = fa[e];
+        *reinterpret_cast<f32x4*>(kr + (ts + e) * C::LKR + cg) =
+            f32x4{(float)fk[e][0], (float)fk[e][1], (float)fk[e][2], (float)fk[e][3]};
+        if (!LOCAL) *reinterpret_cast<t4*>(rq + (16 * wave + ts + e) * C::LR + cg) = fq[e];
+      }
       if (!LOCAL) {
-#pragma unroll
-        for (int u = 0; u < NDP; ++u) {
-          const int d = lane + 64 * u;
-          if (DP >= 64 || d < DP)
-#pragma unroll
-            for (int t = 0; t < 16; ++t) {
-              aq[(16 * wave + t) * C::LQ + d] = fa[u][t];
-              rq[(16 * wave + t) * C::LR + d] = fq[u][t];
-              kr[t * C::LKR + d] = (float)fk[u][t];
-            }
-        }
         // A: lane = (key token j, channels 16 m + 4 dg ..), down the rows i = j, j + 1, ..; rows past the chunk clear the
         // part above the diagonal
         const int j = lane >> 2, dg = lane & 3;
@@ -179,6 +211,7 @@ __global__ __launch_bounds__(256, DP <= 64 ? 2 : 1) void gla_chunk_kernel(GA p) 
 #pragma unroll
           for (int e = 0; e < 4; ++e) uu[m][e] = x[e];
         }
+#pragma unroll 4
         for (int s = 0; s < 16; ++s) {
           const int i = j + s;
           const T* qr = rq + (16 * wave + min(i, 15)) * C::LR + 4 * dg;
@@ -199,27 +232,34 @@ __global__ __launch_bounds__(256, DP <= 64 ? 2 : 1) void gla_chunk_kernel(GA p) 
           if (dg == 0) am[(wave * 16 + (i & 15)) * C::LK + j] = i < 16 ? acc * p.rs : 0.f;
         }
       }
+      // the products: a lane per channel
+      float kx[NDP][16];
+#pragma unroll
+      for (int u = 0; u < NDP; ++u)
+#pragma unroll
+        for (int t = 0; t < 16; ++t) kx[u][t] = kr[t * C::LKR + min(lane + 64 * u, DP - 1)];
 #pragma unroll
       for (int u = 0; u < NDP; ++u) {
         const int d = lane + 64 * u;
         if (DP >= 64 || d < DP) {
-          float w = 1.f;
+          float ax[16], w = 1.f;
+#pragma unroll
+          for (int t = 0; t < 16; ++t) ax[t] = aq[(16 * wave + t) * C::LQ + d];
 #pragma unroll
           for (int t = 0; t < 16; ++t) {
-            w *= fa[u][t];
-            if (!LOCAL) aq[(16 * wave + t) * C::LQ + d] = (float)fq[u][t] * w * p.rs;
+            w *= ax[t];
+            if (!LOCAL) aq[(16 * wave + t) * C::LQ + d] = (float)rq[(16 * wave + t) * C::LR + d] * w * p.rs;
           }
           gm[wave * DP + d] = w;
           w = 1.f;
-          float x[16];
 #pragma unroll
           for (int t = 15; t >= 0; --t) {
-            x[t] = (float)fk[u][t] * w;
-            w *= fa[u][t];
+            kx[u][t] *= w;
+            w *= ax[t];
           }
 #pragma unroll
           for (int t = 0; t < 16; t += 4)
-            *reinterpret_cast<f32x4*>(kr + d * C::LK + t) = f32x4{x[t], x[t + 1], x[t + 2], x[t + 3]};
+            *reinterpret_cast<f32x4*>(kr + d * C::LK + t) = f32x4{kx[u][t], kx[u][t + 1], kx[u][t + 2], kx[u][t + 3]};
         }
       }
     }
@@ -287,6 +327,18 @@ __global__ __launch_bounds__(256, DP <= 64 ? 2 : 1) void gla_chunk_kernel(GA p) 
         }
     }
     if (!LOCAL && p.fused) {
+      // head norm, weight and gate: the outputs pass through LDS, so that rows are read and written in groups of 4 columns
+      float* ob = aq;                                               // [SC][LO]
+      t4 gt[NVG];
+#pragma unroll
+      for (int e = 0; e < NVG; ++e) {
+        const int x = tid + 256 * e, col = (x % (WC / 4)) * 4;
+        const T* gp = (const T*)p.gate + (size_t)(t0 + min(base + x / (WC / 4), n - 1)) * p.ldg + hv;
+        if (p.vec) gt[e] = *reinterpret_cast<const t4*>(gp + min(col, V - 4));
+        else
+#pragma unroll
+          for (int i = 0; i < 4; ++i) gt[e][i] = gp[min(col + i, V - 1)];
+      }
 #pragma unroll
       for (int ch = 0; ch < NCH; ++ch)
 #pragma unroll
@@ -298,22 +350,33 @@ __global__ __launch_bounds__(256, DP <= 64 ? 2 : 1) void gla_chunk_kernel(GA p) 
           if (r == 0) sq[wave * SC + 16 * ch + 4 * g + i] = s;
         }
       __syncthreads();
-      if (act)
 #pragma unroll
-        for (int ch = 0; ch < NCH; ++ch)
+      for (int ch = 0; ch < NCH; ++ch)
 #pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            const int tr = 16 * ch + 4 * g + i, tt = base + tr;
-            const float s = sq[tr] + sq[SC + tr] + sq[2 * SC + tr] + sq[3 * SC + tr];
-            const float inv = 1.f / sqrtf(s / (float)V + p.eps);
+        for (int c = 0; c < NT; ++c)
 #pragma unroll
-            for (int c = 0; c < NT; ++c) {
-              const int col = wc + 16 * c + r;
-              if (tt < n && col < V)
-                ((T*)p.out)[(size_t)(t0 + tt) * p.ldout + hv + col] =
-                    (T)(O[ch][c][i] * inv * p.norm[hv + col] * (float)((const T*)p.gate)[(size_t)(t0 + tt) * p.ldg + hv + col]);
-            }
+          for (int i = 0; i < 4; ++i) ob[(16 * ch + 4 * g + i) * C::LO + wave * 16 * NT + 16 * c + r] = O[ch][c][i];
+      __syncthreads();
+#pragma unroll
+      for (int e = 0; e < NVG; ++e) {
+        const int x = tid + 256 * e, tr = x / (WC / 4), col = (x % (WC / 4)) * 4, tt = base + tr;
+        const float s = sq[tr] + sq[SC + tr] + sq[2 * SC + tr] + sq[3 * SC + tr];
+        const float inv = 1.f / sqrtf(s / (float)V + p.eps);
+        const f32x4 o = *reinterpret_cast<const f32x4*>(ob + tr * C::LO + col);
+        T* op = (T*)p.out + (size_t)(t0 + tt) * p.ldout + hv + col;
+        if (tt >= n) continue;
+        if (p.vec) {
+          if (col < V) {
+            const f32x4 nw = *reinterpret_cast<const f32x4*>(p.norm + hv + col);
+            *reinterpret_cast<t4*>(op) = t4{(T)(o[0] * inv * nw[0] * (float)gt[e][0]), (T)(o[1] * inv * nw[1] * (float)gt[e][1]),
+                                            (T)(o[2] * inv * nw[2] * (float)gt[e][2]), (T)(o[3] * inv * nw[3] * (float)gt[e][3])};
           }
+        } else {
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            if (col + i < V) op[i] = (T)(o[i] * inv * p.norm[hv + col + i] * (float)gt[e][i]);
+        }
+      }
     }
     __syncthreads();
   }
@@ -396,9 +459,13 @@ int nls_gla_scan(const void* q, const void* k, const void* v, long ld, const flo
   const bool fused = norm && gate && out;
   if (nruns < 1 || H < 1 || D < 1 || V < 1 || nseg < 1 || nseg > 64 || (nseg > 1 && (!rec || !recw)) || (!fused && !o)) return -1;
   const long al = f32 ? 16 : 8;
-  const int vec = V % 4 == 0 && ld % 4 == 0 && (long)((uintptr_t)v % al) == 0;
+  const int vec = V % 4 == 0 && ld % 4 == 0 && (long)((uintptr_t)v % al) == 0 &&
+                  (!fused || (ldg % 4 == 0 && ldout % 4 == 0 && (long)(((uintptr_t)gate | (uintptr_t)out) % al) == 0 &&
+                              (uintptr_t)norm % 16 == 0));
+  const int vecq = D % 4 == 0 && ld % 4 == 0 && lda % 4 == 0 && (long)(((uintptr_t)q | (uintptr_t)k) % al) == 0 &&
+                   (uintptr_t)a % 16 == 0;
   const GA p{q, k, v, a, o, norm, gate, out, state, rec, recw, runs, ld, lda, ldo, ldg, ldout, sstride, H, D, V, nseg, fused, vec,
-             qscale, eps};
+             vecq, qscale, eps};
   return f32 ? chunk_d<float>(p, nruns, nt, (hipStream_t)stream) : chunk_d<__bf16>(p, nruns, nt, (hipStream_t)stream);
 }
 

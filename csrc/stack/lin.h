@@ -175,12 +175,12 @@ DEVI void lin_store4(const LinSeg& S, int grp, int ks, int n, int yr, f32x4 v) {
     case LE_DECAY:
 #pragma unroll
       for (int e = 0; e < 4; ++e)
-        if (n + e < S.N) v[e] = expf(-expf(v[e] + S.bias[n + e]));
+        v[e] = expf(-expf(v[e] + S.bias[min(n + e, S.N - 1)]));
       break;
     case LE_SIGPOW:
 #pragma unroll
       for (int e = 0; e < 4; ++e)
-        if (n + e < S.N) v[e] = lin_sigpow(v[e] + S.bias[n + e], S.alpha);
+        v[e] = lin_sigpow(v[e] + S.bias[min(n + e, S.N - 1)], S.alpha);
       break;
     case LE_SOFTCAP:
 #pragma unroll

@@ -448,11 +448,11 @@ def scan_out(o, norm, gate, out, H: int, D: int, T: int, eps: float, st: int):
 
 
 def gla_shape(T: int, nruns: int, H: int, V: int):
-    """(segments, groups of 64 value columns per workgroup) of a gla_scan launch: enough workgroups for the chip, segments of
-    at least 128 tokens."""
+    """(segments, groups of 64 value columns per workgroup) of a gla_scan launch: two workgroups per CU from segments of at
+    least 64 tokens, unless whole runs already give one."""
     nt = 1 if V <= 64 else 2
     wgs = H * -(-V // (64 * nt)) * nruns
-    return max(1, min(-(-512 // wgs), (T - nruns + 1) // 128, 16)), nt
+    return 1 if wgs >= 256 else max(1, min(-(-512 // wgs), (T - nruns + 1) // 64, 16)), nt
 
 
 def gla_scan(q, k, v, a, qscale: float, o, norm, gate, out, state, runs, nruns: int, H: int, D: int, V: int, eps: float, shape,

@@ -81,12 +81,12 @@ def test_registry(tmp_path):
 
 
 def test_launch_shapes():
-    """Segments of the recurrence: at least 128 tokens each, never more than the run, one for decoding."""
+    """Segments of the recurrence: at least 64 tokens each, none for decoding or for many runs."""
     from nats_llm_studio_amd.ops import stack as K
     for T, n, H, V in ((1, 1, 4, 64), (7, 7, 2, 20), (130, 3, 2, 64), (4096, 1, 32, 128), (4096, 4, 4, 512)):
         nseg, nt = K.gla_shape(T, n, H, V)
-        assert 1 <= nseg <= 16 and (nseg == 1 or (T - n + 1) // nseg >= 128) and nt == (1 if V <= 64 else 2)
-    assert K.gla_shape(4096, 1, 4, 64)[0] == 16
+        assert 1 <= nseg <= 16 and (nseg == 1 or (T - n + 1) // nseg >= 64) and nt == (1 if V <= 64 else 2)
+    assert K.gla_shape(4096, 1, 4, 64)[0] == 16 and K.gla_shape(4096, 8, 32, 128)[0] == 1
     assert K.head_pad(20) == (32, True) and K.head_pad(129) == (256, True) and K.head_pad(300) == (320, False)
     assert K.attn_groups(40, 2) == 4 and K.attn_groups(16, 1) == 1 and K.attn_groups(3, 3) == 3
 
