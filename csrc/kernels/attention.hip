@@ -1,5 +1,5 @@
 // Paged grouped-query attention for decode (and prefill expressed as per-token
-// causal decode), gfx950. SURVEY.md §2F attn_decode_paged.
+// causal decode), gfx950.
 //
 // KV cache (one layer): k/v [num_slots][Hkv][D] bf16, slot = block_table[seq][pos / BS] * BS + pos % BS.
 // Grid: (tokens, Hkv, n_split). A workgroup handles the G = Hq/Hkv query heads that

@@ -20,7 +20,7 @@ __device__ __forceinline__ int split_chunk(int chunk, int ctx, int n_split, int 
 }
 
 // ---------------------------------------------------------------------------------------------------
-// Decode attention on MFMA (large grids: batch x kv heads >= 1K workgroups). The VALU kernel above
+// Decode attention on MFMA (large grids: batch x kv heads >= 1K workgroups). The VALU kernel of attention.hip
 // spends ~170 vector instructions per 4 keys of a wave (dot products, cross-lane sums, the online
 // softmax and 32 FMAs of P.V per lane): at batch 512 it runs at ~3.5 TB/s of K/V, bound by issue, not
 // HBM (tools/attn_layout_probe.py: time linear in the context at every length). Here the G query heads
@@ -29,7 +29,7 @@ __device__ __forceinline__ int split_chunk(int chunk, int ctx, int n_split, int 
 //   S^T = K Q^T   A = K rows straight from HBM into registers (lane (g, r): key r, dims 8g..8g+7 of
 //                 each 32-dim k-step), B = Q^T (lane column r = head r, loaded once)
 //   O^T += V^T P^T  A = V^T through LDS: the 32-key V tile is stored row-major with a 16-byte chunk XOR
-//                 swizzle and read back transposed by ds_read_b64_tr_b16 (cdna_hip_programming.md T10);
+//                 swizzle and read back transposed by ds_read_b64_tr_b16;
 //                 B = P^T straight from the S^T accumulators (lane (g, r) holds keys 4g..4g+3 of each
 //                 16-key n-tile for head r: the MFMA's k order is free, so V^T's transposed reads take
 //                 rows {4g..4g+3} and {16+4g..16+4g+3} to match)
@@ -178,7 +178,7 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_mfma_kernel(
     return ((size_t)((long)blk * bs + pc % bs) * Hkv + kh) * D;
   };
   // swizzled byte offset of 16-byte chunk ch of V row `row` (2D-byte rows): D = 128 conflict-free for the
-  // transposed reads and the row writes (cdna_hip_programming.md T10, layout (b)); D = 64: chunk ^ (row & 7)
+  // transposed reads and the row writes; else the chunk ^ the row's low bits
   auto voff = [](int row, int ch) {
     if constexpr (D == 128) return row * 256 + 16 * (ch ^ (((row & 3) << 2) | ((row >> 2) & 3)));
     else return row * (2 * D) + 16 * (ch ^ (row & (NCH - 1)));

@@ -50,7 +50,8 @@ struct GC {
   static constexpr int WC = 64 * NT, LV = WC + 8;                   // values (T)
   static constexpr int LO = WC + 4;                                 // outputs (f32, in the place of queries and keys)
   static constexpr int OQ = 0, OK = OQ + SC * LQ * 4, OE = OK + NCH * DP * LK * 4,
-                       OA = OE > SC * LO * 4 ? OE : SC * LO * 4, OG = OA + NCH * 16 * LK * 4, OS = OG + NCH * DP * 4, OR = OS + 4 * SC * 4, OV = OR + SC * LR * (int)sizeof(T),
+                       OA = OE > SC * LO * 4 ? OE : SC * LO * 4, OG = OA + NCH * 16 * LK * 4,
+                       OS = OG + NCH * DP * 4, OR = OS + 4 * SC * 4, OV = OR + SC * LR * (int)sizeof(T),
                        LDS = OV + SC * LV * (int)sizeof(T);
   static_assert(16 * LKR <= DP * LK && LDS <= 160 * 1024, "LDS");
 };

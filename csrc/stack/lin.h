@@ -21,6 +21,7 @@
 namespace nls_lin {
 
 constexpr int LIN_SEGS = 6;
+constexpr int LIN_GM = 4;      // row tiles that are walked together down the weights (lin_tile)
 
 enum LinEpi : int {
   LE_NONE = 0, LE_SILU = 1, LE_TANH = 2, LE_SIGMOID = 3, LE_RELU2 = 4,
@@ -99,9 +100,15 @@ DEVI bool lin_tile(const LinArgs& a, int id, LinTile& t) {
   const LinSeg& S = a.s[s];
   int q = id - a.begin[s];
   const int nmt = a.nmt[s];
-  const int mi = q % nmt;
-  q /= nmt;
   const int nnt = (S.N + BN - 1) / BN;
+  int mi = q % nmt, ni = q / nmt;
+  if (nmt > LIN_GM && !S.rows && S.ng == 1 && S.ks == 1) {
+    // LIN_GM row tiles at a time: the workgroups that an XCD runs together share weight tiles and row tiles in its L2
+    const int first = q / (LIN_GM * nnt) * LIN_GM, gm = min(LIN_GM, nmt - first), r = q - first * nnt;
+    mi = first + r % gm;
+    ni = r / gm;
+  }
+  q = ni;
   t.seg = s;
   t.n0 = (q % nnt) * BN;
   t.ks = 0;

@@ -5,8 +5,8 @@
 // activation sub-tiles with the 16-byte chunks of a row permuted on the DMA source (chunk ^ swz(row)), so every
 // fragment is one conflict-free ds_read_b128. One raw barrier per step with a counted vmcnt leaves the later stages
 // in flight. Routed rows (experts) are gathered by the DMA's per-lane source addresses.
-// Tile ids are dealt to the 8 XCDs in contiguous ranges, m-tiles innermost: all row blocks of a weight tile read it
-// through one XCD's L2.
+// Tile ids are dealt to the 8 XCDs in contiguous ranges, a few m-tiles innermost (lin_tile): the workgroups that run
+// together on an XCD form a block of weight and row tiles and read both through its L2.
 #include "../kernels/lds_dma.h"
 #include "lin.h"
 
@@ -148,6 +148,7 @@ int gemm_d(LinArgs& a, int cfg, hipStream_t st) {
     case 3: return gemm_t<T, 256, 128, 4, 2, 3>(a, st);
     case 4: return gemm_t<T, 256, 256, 4, 2, 2>(a, st);
     case 5: return gemm_t<T, 64, 64, 2, 2, 8>(a, st);
+    case 6: return gemm_t<T, 192, 128, 4, 2, 3>(a, st);
   }
   return -1;
 }
@@ -157,7 +158,7 @@ int gemm_d(LinArgs& a, int cfg, hipStream_t st) {
 extern "C" {
 
 // cfg: tile of the launch (BN x BM): 0 = 64 x 64, 1 = 128 x 64, 2 = 128 x 128, 3 = 256 x 128, 4 = 256 x 256,
-// 5 = 64 x 64 with 8 stages in flight (launches of at most one workgroup per CU)
+// 5 = 64 x 64 with 8 stages in flight (launches of at most one workgroup per CU), 6 = 192 x 128
 int nls_lin_gemm(const void* args, int f32, int cfg, void* stream) {
   nls_lin::LinArgs a = *reinterpret_cast<const nls_lin::LinArgs*>(args);
   return f32 ? nls_lin::gemm_d<float>(a, cfg, (hipStream_t)stream)

@@ -64,9 +64,10 @@ __global__ __launch_bounds__(256) void embed_kernel(int* __restrict__ ids, const
   }
 }
 
-// ---- x[t] += norm(y) * w (w null: x[t] += y); y = one row (the sum of `nslab` slabs' rows), or (topk) sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t],
-// the shared expert); y null: x is only read. Optional second norm (the next sublayers' or the model's last one) of the
-// new x into `on`. norm: (v - mean) / sqrt(var + eps), or (rms) v / sqrt(mean(v^2) + eps).
+// ---- x[t] += norm(y) * w (w null: x[t] += y); y = one row (the sum of `nslab` slabs' rows), or (topk)
+// sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t], the shared expert); y null: x is only read. Optional second norm (the
+// next sublayers' or the model's last one) of the new x into `on`. norm: (v - mean) / sqrt(var + eps), or (rms)
+// v / sqrt(mean(v^2) + eps).
 // A workgroup per row (`rows`: gathered), 4 consecutive columns x NV per thread in registers.
 struct NormAdd {
   const float* y;

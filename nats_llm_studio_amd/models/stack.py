@@ -2,8 +2,9 @@
 
 A mixer or feed-forward is a class that loads its weights, adds its step buffers, and runs on the rows of a step; a layer
 class (OutputNormLayer, SharedNormLayer) places the norms and joins the sublayers. The per-token cache rows (paged) and the
-per-sequence states (slots) of all layers belong to the engine, which sees them as `kv_cache` / `state_pool`. Everything runs on the HIP kernels of csrc/stack (ops/stack.py): bf16 operands with an f32
-residual, or `dtype=torch.float32` for 32-bit throughout.
+per-sequence states (slots) of all layers belong to the engine, which sees them as `kv_cache` / `state_pool`. Everything
+runs on the HIP kernels of csrc/stack (ops/stack.py): bf16 operands with an f32 residual, or `dtype=torch.float32` for 32-bit
+throughout.
 
 Rows of a step are runs of consecutive tokens of one sequence (whole prompts, portions of any size, single decoded
 tokens), all in one batch:
@@ -451,7 +452,8 @@ class GlaPart(_SharedPart):
         if a is not None:
             e["decay"].run(T, st)
         if single:
-            K.gla_step(e["q"], e["k"], e["v"], a, (e["low"], self.a2r, self.a2b, 1.0 / c.tau), qs, S, b.runs, T, self.norm, e["g"], e["out"], H, D, V, eps, st)
+            K.gla_step(e["q"], e["k"], e["v"], a, (e["low"], self.a2r, self.a2b, 1.0 / c.tau), qs, S, b.runs, T, self.norm,
+                       e["g"], e["out"], H, D, V, eps, st)
             return
         n = step.nruns
         shape = K.gla_shape(T, n, H, V)

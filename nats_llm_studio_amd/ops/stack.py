@@ -176,11 +176,13 @@ class Seg:
         self.keep = (bias, gate, routed, rope, xmap)
 
 
-GEMM_TILES = ((64, 64), (128, 64), (128, 128), (256, 128), (256, 256), (64, 64))     # (weight rows, rows) of lin_gemm's cfg
+# (weight rows, rows) of lin_gemm's configs
+GEMM_TILES = ((64, 64), (128, 64), (128, 128), (256, 128), (256, 256), (64, 64), (192, 128))
 
 
 # relative multiply rates of the tiles: (up to so many workgroups, below, above); the small tiles run two or more to a CU
-GEMM_RATE = {4: (0, 0.96, 0.96), 3: (0, 1.0, 1.0), 2: (256, 0.47, 0.72), 1: (512, 0.5, 0.63), 0: (1024, 0.45, 0.55)}
+GEMM_RATE = {4: (0, 0.96, 0.96), 3: (0, 1.0, 1.0), 6: (0, 0.96, 0.96), 2: (256, 0.47, 0.72),
+             1: (512, 0.5, 0.63), 0: (1024, 0.45, 0.55)}
 
 
 class LinLaunch:
@@ -232,13 +234,18 @@ class LinLaunch:
             return True, (0 if M <= 2048 else 1)
         if n64 < 96 and n16 <= 1024:
             return False, 1, 16, 1
-        if M <= 512:
-            return True, (3 if self._tiles(256, 128, M) >= 120 else 5 if n64 <= 256 else 0)
-        # compute-bound: rounds of 256 workgroups times a tile's cost
+        if M > 512:
+            cand = GEMM_RATE
+        elif self._tiles(256, 128, M) >= 120:
+            cand = (3, 6)
+        else:
+            return True, (5 if n64 <= 256 else 0)
+
+        # rounds of 256 workgroups times a tile's cost
         def cost(c):
             n, (few, lo, hi) = self._tiles(*GEMM_TILES[c], M), GEMM_RATE[c]
             return -(-n // 256) * GEMM_TILES[c][0] * GEMM_TILES[c][1] / (lo if n <= few else hi)
-        return True, min(GEMM_RATE, key=cost)
+        return True, min(cand, key=cost)
 
     def split_config(self, M: int):
         """(config, K splits) of a launch that may split K: about 512 workgroups of 64 x 64 tiles, or 256 of 256 x 128."""
@@ -331,9 +338,9 @@ def embed(ids, table: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor],
 def norm_add(y: torch.Tensor, w: Optional[torch.Tensor], x: torch.Tensor, xb: Optional[torch.Tensor], T: int, eps: float,
              st: int, plan: Optional[MoePlan] = None, shared_row0: int = -1, out_norm: Optional[torch.Tensor] = None,
              out: Optional[torch.Tensor] = None, rms: bool = False, slabs: int = 1, slab_rows: int = 0):
-    """x[:T] += norm(y) * w, or += y without w (xb: its bf16 rounding); y may be the sum of `slabs` blocks of slab_rows rows. With `plan`, y holds the routed experts' rows
-    (token-major) and from row `shared_row0` on the shared expert's, combined first. out = norm(x) * out_norm (what the next
-    sublayers read, or the model's last norm). norm: layer norm, or RMS."""
+    """x[:T] += norm(y) * w, or += y without w (xb: its bf16 rounding); y may be the sum of `slabs` blocks of slab_rows rows.
+    With `plan`, y holds the routed experts' rows (token-major) and from row `shared_row0` on the shared expert's, combined
+    first. out = norm(x) * out_norm (what the next sublayers read, or the model's last norm). norm: layer norm, or RMS."""
     D = y.shape[1] if w is None else w.numel()
     _check(lib().nls_norm_add(y.data_ptr(), y.stride(0), _p(plan.topw) if plan else None, plan.top if plan else 0,
                               shared_row0, _p(w), x.data_ptr(), _p(xb), x.stride(0), _p(out_norm), _p(out),

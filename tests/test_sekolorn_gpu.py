@@ -44,7 +44,7 @@ def test_linear(K, dt, M, N, Kd):
 
 
 @pytest.mark.parametrize("dt", DT)
-@pytest.mark.parametrize("cfg", [(True, c) for c in range(6)] + [(False, m, w, r) for m, w, r in (
+@pytest.mark.parametrize("cfg", [(True, c) for c in range(7)] + [(False, m, w, r) for m, w, r in (
     (1, 4, 1), (1, 8, 1), (1, 16, 1), (1, 4, 2), (1, 8, 2), (2, 4, 1), (2, 8, 1), (2, 4, 2), (2, 8, 2), (2, 4, 4), (4, 4, 1),
     (4, 8, 1), (4, 4, 2), (4, 8, 2), (4, 4, 4))])
 def test_linear_every_tile(K, dt, cfg):
