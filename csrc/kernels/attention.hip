@@ -333,7 +333,7 @@ static int attn_decode_impl(const void* q, long ldq, const void* kc, const void*
 #define NLS_ATTN_M(KVT, W, DD)                                                                                 \
   hipLaunchKernelGGL((attn_decode_mfma_kernel<KVT, W, DD>), grid, dim3(64 * W), 0, st, (const __bf16*)q, ldq,   \
                      (const KVT*)kc, (const KVT*)vc, block_tables, bt_stride, tok_seq, ctx_len, Hkv, G, block_size, \
-                     scale, chunk, n_split, (act_t*)out, ldo, part_o, part_ml, cnt, (const float*)nullptr, 0L)
+                     scale, chunk, n_split, (act_t*)out, ldo, part_o, part_ml, cnt, (const float*)nullptr, 0L, AttnMask{})
 #define NLS_ATTN_MD(DD)                                                                                         \
     if (kv8) {                                                                                                  \
       if (big) NLS_ATTN_M(uint8_t, 1, DD); else if (mw == 4) NLS_ATTN_M(uint8_t, 4, DD); else NLS_ATTN_M(uint8_t, 8, DD); \

@@ -97,13 +97,21 @@ DEVI void merge_splits(const float* __restrict__ part_o, const float* __restrict
 // 16-byte chunks, XOR swizzled within the row), D / 8 lanes per V row on the loads.
 // Groups of more than 16 query heads take ceil(G / 16) workgroups (blockIdx.y = kv head * blocks + block of 16 heads).
 // gate (optional): [rows][ldg], one factor per token and query head on the output.
-template <typename KV, int WAVES, int D, typename OUT = act_t>
+// AttnMask: sink: the softmax's denominator holds one more, a score of 0 without a value (the state that the first wave of the
+// first split starts from). WIN: keys j < keep or j >= ctx - window only. The kernel then walks an index over the visible
+// keys (those of the kept ones' last group of 32 that are not kept are masked): the first `keep`, rounded up to a group, then
+// `gap` positions further on; splits and groups start at multiples of 32, so no group spans the gap.
+struct AttnMask {
+  int window = 0, keep = 0, sink = 0;
+};
+
+template <typename KV, int WAVES, int D, typename OUT = act_t, bool WIN = false>
 __global__ __launch_bounds__(64 * WAVES) void attn_decode_mfma_kernel(
     const __bf16* __restrict__ q, long ldq, const KV* __restrict__ kc, const KV* __restrict__ vc,
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ tok_seq,
     const int* __restrict__ ctx_len, int Hkv, int Gq, int bs, float scale, int chunk, int n_split,
     OUT* __restrict__ out, long ldo, float* __restrict__ part_o, float* __restrict__ part_ml,
-    int* __restrict__ cnt, const float* __restrict__ gate, long ldg) {
+    int* __restrict__ cnt, const float* __restrict__ gate, long ldg, AttnMask mask) {
   static_assert(D == 32 || D == 64 || D == 128 || (D == 256 && WAVES <= 2), "head dimension");
   constexpr int NKK = D / 32, NDT = D / 16, KG = 32;
   constexpr int NCH = D / 8, LPR = NCH, RPI = 64 / LPR, NVL = KG / RPI;   // V: chunks per row, lanes per row,
@@ -124,9 +132,12 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_mfma_kernel(
   const int wave = WAVES == 1 ? 0 : __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   uint8_t* Vs = Vsm + wave * KG * D * 2;
   const int Hq = Hkv * Gq;
-  const int ctx = ctx_len[t];
+  const int last_pos = ctx_len[t], kept = WIN ? (mask.keep + KG - 1) & ~(KG - 1) : 0;
+  const int gap = WIN ? max(0, last_pos - mask.window - kept) : 0;
+  const int ctx = last_pos - gap;
   // short contexts: at least one 32-key group per wave of the workgroup per split (>= 64 keys)
   chunk = split_chunk(chunk, ctx, n_split, bs, KG * WAVES > 64 ? KG * WAVES : 64);
+  if (WIN) chunk = (chunk + KG - 1) & ~(KG - 1);
   const int start = split * chunk;
   if (n_split > 1 && start >= ctx && ctx > 0) return;       // inactive split: combine skips it
   const int end = min(ctx, start + chunk);
@@ -145,7 +156,8 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_mfma_kernel(
   f32x4 o[NDT];
 #pragma unroll
   for (int c = 0; c < NDT; ++c) o[c] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m = -INFINITY, l = 0.f;
+  const bool sink = mask.sink && split == 0 && wave == 0;
+  float m = sink ? 0.f : -INFINITY, l = sink ? 1.f : 0.f;
 
   // Block-table entries come from a register window (lane i holds entry b0 + 64 * win + i, refreshed once
   // per 64 blocks), broadcast per 32-key group as wave-uniform values: the K/V loads of a group no
@@ -155,14 +167,16 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_mfma_kernel(
   const int b0 = start / bs;
   int btw = -1, btreg = 0;
   int gblk[NGB] = {0, 0, 0, 0};
-  auto group_blocks = [&](int base) __attribute__((always_inline)) {
+  auto shift = [&](int base) { return WIN && base >= kept ? gap : 0; };  // position of a group's keys, less their index
+  auto group_blocks = [&](int base0) __attribute__((always_inline)) {
+    const int sh = shift(base0), base = base0 + sh, end_p = end + sh;
     const int bi0 = base / bs - b0;
-    const int nbg = (min(base + KG, end) - 1) / bs - base / bs + 1;     // blocks this group touches
+    const int nbg = (min(base + KG, end_p) - 1) / bs - base / bs + 1;     // blocks this group touches
     const int win = bi0 >> 6;
     if (win != btw) {
       btw = win;
       const int e = b0 + win * 64 + lane;
-      btreg = e * bs < end ? bt[e] : 0;
+      btreg = e * bs < end_p ? bt[e] : 0;
     }
 #pragma unroll
     for (int i = 0; i < NGB; ++i) {
@@ -171,8 +185,8 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_mfma_kernel(
       if (i < nbg) gblk[i] = (bi >> 6) == win ? __builtin_amdgcn_readlane(btreg, bi & 63) : bt[b0 + bi];
     }
   };
-  auto kv_row = [&](int p, int base) -> size_t {       // element offset of key p's row for this kv head
-    const int pc = min(p, end - 1);
+  auto kv_row = [&](int p, int base0) -> size_t {      // element offset of key p's row for this kv head
+    const int base = base0 + shift(base0), pc = min(p, end - 1) - base0 + base;
     const int lb = pc / bs - base / bs;                // 0 .. NGB - 1
     const int blk = lb == 0 ? gblk[0] : (lb == 1 ? gblk[1] : (lb == 2 ? gblk[2] : gblk[3]));
     return ((size_t)((long)blk * bs + pc % bs) * Hkv + kh) * D;
@@ -229,7 +243,9 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_mfma_kernel(
     for (int nt = 0; nt < 2; ++nt)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const float v = base + 16 * nt + 4 * g + i < end ? s[nt][i] * sl2 : -INFINITY;
+        const int ki = base + 16 * nt + 4 * g + i, kp = ki + shift(base);
+        const bool see = ki < end && (!WIN || kp < mask.keep || kp >= last_pos - mask.window);
+        const float v = see ? s[nt][i] * sl2 : -INFINITY;
         s[nt][i] = v;
         mx = fmaxf(mx, v);
       }

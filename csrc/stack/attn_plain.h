@@ -22,6 +22,7 @@ struct PA {
   int bts, bs, gs;            // gs: query heads per key head
   int Dk, Dv;                 // columns (Dk a multiple of 4)
   float scale;
+  int window, keep, sink;     // window > 0: the newest `window` keys and the first `keep`; sink: one more in the denominator
 };
 
 template <typename T> DEVI f32x4 ld4(const T* p) {
@@ -42,9 +43,12 @@ __global__ __launch_bounds__(256) void attn_plain_kernel(PA p) {
   for (int i = threadIdx.x; i < p.Dk; i += 256) q[i] = (float)qr[i];
   __syncthreads();
   const int key = threadIdx.x >> 2, part = threadIdx.x & 3;
-  float m = -INFINITY, l = 0.f, acc[NC] = {0.f, 0.f, 0.f, 0.f};
+  float m = p.sink ? 0.f : -INFINITY, l = p.sink ? 1.f : 0.f, acc[NC] = {0.f, 0.f, 0.f, 0.f};
+  const int low = p.window > 0 ? ctx - p.window : 0;                  // first key of the window
   for (int k0 = 0; k0 < ctx; k0 += 64) {
+    if (k0 >= p.keep && k0 + 64 <= low) k0 = low & ~63;               // (none of the tiles between is seen)
     const int k = k0 + key;
+    const bool see = k < ctx && (k >= low || k < p.keep);
     float s = 0.f;
     if (k < ctx) {
       const T* c = kc + ((size_t)bt[k / p.bs] * p.bs + k % p.bs) * p.ldkv;
@@ -56,18 +60,18 @@ __global__ __launch_bounds__(256) void attn_plain_kernel(PA p) {
     }
     s += __shfl_xor(s, 1, 64);
     s += __shfl_xor(s, 2, 64);
-    if (part == 0) sc[key] = k < ctx ? s * p.scale : -INFINITY;
+    if (part == 0) sc[key] = see ? s * p.scale : -INFINITY;
     __syncthreads();
     float mn = m;
     for (int i = 0; i < 64; ++i) mn = fmaxf(mn, sc[i]);
-    const float alpha = m == -INFINITY ? 0.f : expf(m - mn);
+    const float alpha = m == -INFINITY ? 0.f : expf(m - mn), base = mn == -INFINITY ? 0.f : mn;
     l *= alpha;
 #pragma unroll
     for (int i = 0; i < NC; ++i) acc[i] *= alpha;
     m = mn;
     const int n = min(64, ctx - k0);
     for (int i = 0; i < n; ++i) {
-      const float e = expf(sc[i] - mn);
+      const float e = expf(sc[i] - base);
       l += e;
       const int kk = k0 + i;
       const T* c = vc + ((size_t)bt[kk / p.bs] * p.bs + kk % p.bs) * p.ldkv;

@@ -12,7 +12,7 @@
 //   closes with one lane exchange; P^T goes from those registers straight into O^T += V^T P^T (V^T by transposed LDS
 //   reads in the same key order), so a row's rescale is lane-local and skipped when no maximum grew.
 // The next tile's loads are in flight in registers while a tile computes (its cache slots one tile ahead of that); one
-// barrier per tile, two LDS buffers. Rows are padded in LDS (K: 16 bytes, V: 64) against bank conflicts. The epilogue applies
+// barrier per tile, two LDS buffers. Under a sliding window (with kept first keys) tiles that no row sees are left out. Rows are padded in LDS (K: 16 bytes, V: 64) against bank conflicts. The epilogue applies
 // the head's output gate.
 #include "../kernels/common.h"
 
@@ -41,13 +41,16 @@ struct FP {
   const __bf16* cache;    // latent: cache rows at their rotated part
   const int* xmap;        // cache slot of every context row
   const int* blocks;      // [n][8]: (first row, rows, sequence, first position, xoff, -, -, -), heaviest first
-  const float* gate;      // [T][H]
+  const float* gate;      // [T][H] (null: none)
   __bf16* out;            // [T][ldo], head stride vdim
   long ldqn, ldqr, ldc, ldo;
   int qns, qrs, H, vdim, ldg;
   int gs, nsub;           // grouped: query heads per key head; workgroups per block and key head
   float scale;
+  int window, keep, sink; // position i sees j <= i if i - j < window or j < keep; sink: one more in the denominator
 };
+constexpr int NO_WINDOW = 1 << 30;
+
 
 template <int NKU, int NKR, int NDB, int NWV>      // 32-column units: keys unrotated / rotated, values; waves
 __global__ __launch_bounds__(64 * NWV) void flash_prefill_kernel(FP p) {
@@ -76,7 +79,10 @@ __global__ __launch_bounds__(64 * NWV) void flash_prefill_kernel(FP p) {
   const int tw0 = row0 + 32 * wave;
   const int myrow = min(tw0 + tl, nrow - 1), mytok = myrow / gs, head = PAGED ? kh * gs + myrow - mytok * gs : kh;
   const float sl2 = p.scale * 1.4426950408889634f;
-  const int nkeys = pos0 + (min(row0 + 32 * NWV, nrow) - 1) / gs + 1, ntile = (nkeys + KT - 1) / KT;
+  const int nkeys = pos0 + (min(row0 + 32 * NWV, nrow) - 1) / gs + 1, lowt = max(pos0 + row0 / gs - p.window + 1, 0) / KT;
+  // tiles that no row sees are left out: `skip` of them behind the kept keys' `nkt`
+  const int nkt = min((p.keep + KT - 1) / KT, lowt), skip = lowt - nkt, ntile = (nkeys + KT - 1) / KT - skip;
+  auto tile = [&](int t) { return t < nkt ? t : t + skip; };
   const int wlast = pos0 + min(tw0 + 31, nrow - 1) / gs, wfirst = pos0 + tw0 / gs;
   const bool wact = tw0 < nrow;
   const int qpos = pos0 + mytok;
@@ -94,7 +100,7 @@ __global__ __launch_bounds__(64 * NWV) void flash_prefill_kernel(FP p) {
   auto load_slots = [&](int t) __attribute__((always_inline)) {
     if constexpr (PAGED) {
 #pragma unroll
-      for (int i = 0; i < NLK; ++i) sl[i] = p.xmap[xoff + min(t * KT + (tid + NT * i) / CU, nkeys - 1)];
+      for (int i = 0; i < NLK; ++i) sl[i] = p.xmap[xoff + min(tile(t) * KT + (tid + NT * i) / CU, nkeys - 1)];
     }
   };
   load_slots(0);
@@ -115,13 +121,13 @@ __global__ __launch_bounds__(64 * NWV) void flash_prefill_kernel(FP p) {
       const int e = tid + NT * i;
       u32x4 v = u32x4{0u, 0u, 0u, 0u};
       if (e < KT * CU) {
-        const int key = t * KT + e / CU;
+        const int key = tile(t) * KT + e / CU;
         if (key < nkeys) v = ld16(p.kx + ((size_t)(xoff + key) * p.H + kh) * DKU + (e % CU) * 8);
       } else if (e < KT * (CU + CR)) {
-        const int f = e - KT * CU, key = t * KT + f / max(CR, 1);
+        const int f = e - KT * CU, key = tile(t) * KT + f / max(CR, 1);
         if (key < nkeys) v = ld16(p.cache + (size_t)p.xmap[xoff + key] * p.ldc + (f % max(CR, 1)) * 8);
       } else if (e < KT * CPR) {
-        const int f = e - KT * (CU + CR), key = t * KT + f / CV;
+        const int f = e - KT * (CU + CR), key = tile(t) * KT + f / CV;
         if (key < nkeys) v = ld16(p.vx + ((size_t)(xoff + key) * p.H + kh) * DV + (f % CV) * 8);
       }
       st[i] = v;
@@ -155,19 +161,19 @@ __global__ __launch_bounds__(64 * NWV) void flash_prefill_kernel(FP p) {
   f32x16 o[NDB];
 #pragma unroll
   for (int i = 0; i < NDB; ++i) o[i] = f32x16{};
-  float m = -INFINITY, l = 0.f;
+  float m = p.sink ? 0.f : -INFINITY, l = p.sink && h == 0 ? 1.f : 0.f;       // (l: two lanes' shares of a row)
   load_tile(0);
   load_slots(1);
   store_tile(0);
   __syncthreads();
   const int vq = (lane & 15) >> 2, vp = lane & 3, vhalf = (lane >> 4) & 1;
   for (int t = 0; t < ntile; ++t) {
-    const int cur = t & 1, k0 = t * KT;
+    const int cur = t & 1, k0 = tile(t) * KT;
     if (t + 1 < ntile) {
       load_tile(t + 1);
       load_slots(t + 2);
     }
-    if (wact && k0 <= wlast) {
+    if (wact && k0 <= wlast && (k0 < p.keep || k0 + KT > wfirst - p.window + 1)) {
       const uint8_t* kb = lds + cur * TB;
       const uint8_t* vb = kb + KT * KROW;
       f32x16 s[2];
@@ -181,13 +187,13 @@ __global__ __launch_bounds__(64 * NWV) void flash_prefill_kernel(FP p) {
                                                          0, 0);
       }
       float mx = -INFINITY;
-      if (k0 + KT - 1 > wfirst) {
+      if (k0 + KT - 1 > wfirst || (k0 <= wlast - p.window && k0 + KT > p.keep)) {
 #pragma unroll
         for (int u = 0; u < 2; ++u)
 #pragma unroll
           for (int r = 0; r < 16; ++r) {
             const int key = k0 + 32 * u + (r & 3) + 8 * (r >> 2) + 4 * h;
-            s[u][r] = key <= qpos ? s[u][r] : -INFINITY;
+            s[u][r] = key <= qpos && (key > qpos - p.window || key < p.keep) ? s[u][r] : -INFINITY;
             mx = fmaxf(mx, s[u][r]);
           }
       } else {
@@ -235,7 +241,7 @@ __global__ __launch_bounds__(64 * NWV) void flash_prefill_kernel(FP p) {
   l += __shfl_xor(l, 32, 64);
   if (tw0 + tl >= nrow) return;
   // lane holds O[row][32 db + 8 g + 4 h + 0 .. 3] in o[db][4 g ..]
-  const float f = (l > 0.f ? 1.f / l : 0.f) * p.gate[(size_t)(t0 + mytok) * p.ldg + head];
+  const float f = (l > 0.f ? 1.f / l : 0.f) * (p.gate ? p.gate[(size_t)(t0 + mytok) * p.ldg + head] : 1.f);
   __bf16* y = p.out + (size_t)(t0 + mytok) * p.ldo + (size_t)head * p.vdim;
   const bool vec = (p.vdim & 3) == 0;
 #pragma unroll
@@ -291,7 +297,7 @@ int nls_latent_prefill(const void* qn, long ldqn, int qns, const void* qr, long 
                        int waves, float scale, void* stream) {
   if (nblocks < 1 || H < 1 || vdim < 1 || vdim > dv) return -1;
   FP p{(const __bf16*)qn, (const __bf16*)qr, (const __bf16*)kx, (const __bf16*)vx, (const __bf16*)cache, xmap, blocks,
-       gate, (__bf16*)out, ldqn, ldqr, ldc, ldo, qns, qrs, H, vdim, ldg, 1, 1, scale};
+       gate, (__bf16*)out, ldqn, ldqr, ldc, ldo, qns, qrs, H, vdim, ldg, 1, 1, scale, NO_WINDOW, 0, 0};
   hipStream_t st = (hipStream_t)stream;
 #define NLS_LP(U, R, V) \
   if (dku == 32 * U && dr == 32 * R && dv == 32 * V) \
@@ -303,13 +309,13 @@ int nls_latent_prefill(const void* qn, long ldqn, int qns, const void* qr, long 
   return -1;
 }
 
-// Dp: padded head width (32, 64, 128; 256 with 4 waves); k, v: paged [slots][G][Dp]; blocks of up to 32 * waves tokens
+// window > 0: sliding window with `keep` first keys. Dp: padded head width (32, 64, 128; 256 with 4 waves); k, v: paged [slots][G][Dp]; blocks of up to 32 * waves tokens
 int nls_gqa_prefill(const void* q, long ldq, const void* k, const void* v, const int* xmap, const int* blocks, int nblocks,
                     const float* gate, int ldg, void* out, long ldo, int H, int G, int Dp, int waves, float scale,
-                    void* stream) {
-  if (nblocks < 1 || G < 1 || H < 1 || H % G || !gate || (ldq & 7) || (ldo & 3)) return -1;
+                    int window, int keep, int sink, void* stream) {
+  if (nblocks < 1 || G < 1 || H < 1 || H % G || window < 0 || window > NO_WINDOW || keep < 0 || (ldq & 7) || (ldo & 3)) return -1;
   FP p{(const __bf16*)q, (const __bf16*)q, (const __bf16*)k, (const __bf16*)v, nullptr, xmap, blocks, gate, (__bf16*)out, ldq, ldq,
-       (long)G * Dp, ldo, Dp, Dp, H, Dp, ldg, H / G, H / G, scale};
+       (long)G * Dp, ldo, Dp, Dp, H, Dp, ldg, H / G, H / G, scale, window ? window : NO_WINDOW, keep, sink};
   hipStream_t st = (hipStream_t)stream;
   // (nsub = H / G workgroups of 32 * waves rows cover a block of 32 * waves tokens)
   if (waves == 8 && Dp == 256) {

@@ -5,7 +5,7 @@
 //   wkv: o_t[j] = sum_i r_t[i] (S[i][j] + u[i] k_t[i] v_t[j]);   S[i][j] = w_t[i] S[i][j] + k_t[i] v_t[j]
 //   gla: S[i][j] = w_t[i] S[i][j] + k_t[i] v_t[j];               o_t[j] = rs sum_i r_t[i] S[i][j]
 // A step of single tokens (decode) streams each head's state once with 16-byte accesses and ends with the head's norm and
-// gate (step_kernel).
+// gate, or (norm null) with the plain outputs (step_kernel).
 //
 // A run = (first row, tokens, state slot, first position): consecutive rows of one sequence. A run at position 0
 // starts from a zero state, any other from its slot; slot < 0 or 0 tokens: nothing to do (padded decode rows).
@@ -50,7 +50,7 @@ struct Scan {
 };
 
 // ---- one token per run: the state of (run, head) is read and written once, 4 value columns per thread; then
-// out = (o / rms(o)) * norm * gate. V is a multiple of 4, at most 1024; D at most 256.
+// out = (o / rms(o)) * norm * gate, or (norm null) p.o. V is a multiple of 4, at most 1024; D at most 256.
 template <typename T, int KIND>
 __global__ __launch_bounds__(256) void step_kernel(Scan p, const float* __restrict__ norm, const T* __restrict__ gate,
                                                    long ldg, T* __restrict__ out, long ldout, float eps) {
@@ -117,8 +117,10 @@ __global__ __launch_bounds__(256) void step_kernel(Scan p, const float* __restri
       for (int i = 0; i < G; ++i) o[q] += red[i * V + e];
       if (KIND == WKV) o[q] += ruk * vs[e];
       ss += o[q] * o[q];
+      if (KIND == GLA && !norm) p.o[(size_t)t * p.ldo + hv + e] = o[q];
     }
   }
+  if (KIND == GLA && !norm) return;
 #pragma unroll
   for (int q = 32; q > 0; q >>= 1) ss += __shfl_xor(ss, q, 64);
   if ((tid & 63) == 0) part[4 + (tid >> 6)] = ss;

@@ -27,54 +27,108 @@ DEVI float bsum(float v, float* sh) {
 template <typename T> DEVI float ldv(const T* p, long i) { return (float)p[i]; }
 template <typename T> DEVI void stv(T* p, long i, float v) { p[i] = (T)v; }
 
-// ---- x[t] = table[id] * scale, id from the host or (use_prev) the previous step's next_ids
-__global__ __launch_bounds__(256) void embed_kernel(int* __restrict__ ids, const int* __restrict__ next_ids,
-                                                    const int* __restrict__ use_prev, const __bf16* __restrict__ tab,
-                                                    int V, int D, float scale, float* __restrict__ x,
-                                                    __bf16* __restrict__ xb, long ldx) {
-  const int t = blockIdx.x;
-  int id = ids[t];
-  if (use_prev && use_prev[t]) id = next_ids[t];
-  id = min(max(id, 0), V - 1);
-  __syncthreads();
-  if (threadIdx.x == 0 && use_prev) ids[t] = id;
-  const __bf16* row = tab + (size_t)id * D;
-  if ((D & 7) == 0) {
-    for (int i = threadIdx.x * 8; i < D; i += 2048) {
-      const u32x4 v = ld16(row + i);
-      const bf16x8 b = __builtin_bit_cast(bf16x8, v);
-      float* o = x + (size_t)t * ldx + i;
-      const f32x4 lo = f32x4{(float)b[0], (float)b[1], (float)b[2], (float)b[3]} * scale;
-      const f32x4 hi = f32x4{(float)b[4], (float)b[5], (float)b[6], (float)b[7]} * scale;
-      *reinterpret_cast<f32x4*>(o) = lo;
-      *reinterpret_cast<f32x4*>(o + 4) = hi;
-      if (xb)
+// ---- x[t] = table[id] * scale (+ the row of the token pair, + the position's vector), id from the host or (use_prev) the
+// previous step's next_ids. The token ahead of a run's first is the slot's; the run's first row, which alone reads it,
+// leaves the run's last token there.
+struct Embed {
+  int* ids;
+  const int *next_ids, *use_prev;
+  const __bf16* tab;
+  float* x;
+  __bf16* xb;              // optional bf16 rounding, row stride ldx
+  void *c0, *c1;           // optional copies in the activation type (f32: float), row stride ldc
+  const __bf16* pairs;     // optional [buckets + 1][D]
+  int* prev;               // [slots]
+  const int *runs, *tok_seq;
+  const __bf16* ptab;      // optional [npos][D]
+  const int* pos;
+  long ldx, ldc;
+  int V, D, buckets, mul_prev, mul_cur, npos, f32;
+  float scale;
+};
+
+DEVI int token_of(const Embed& p, int t) {
+  return min(max(p.use_prev && p.use_prev[t] ? p.next_ids[t] : p.ids[t], 0), p.V - 1);
+}
+
+template <int N>
+DEVI void embed_cols(const Embed& p, int t, const __bf16* row, const __bf16* pair, const __bf16* pv) {
+  typedef __bf16 bfn __attribute__((ext_vector_type(N)));
+  for (int i = threadIdx.x * N; i < p.D; i += 256 * N) {
+    float v[N];
+    const bfn a = *reinterpret_cast<const bfn*>(row + i);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          xb[(size_t)t * ldx + i + e] = (__bf16)lo[e];
-          xb[(size_t)t * ldx + i + 4 + e] = (__bf16)hi[e];
-        }
+    for (int e = 0; e < N; ++e) v[e] = (float)a[e] * p.scale;
+    if (pair) {
+      const bfn b = *reinterpret_cast<const bfn*>(pair + i);
+#pragma unroll
+      for (int e = 0; e < N; ++e) v[e] += (float)b[e];
     }
-    return;
+    if (pv) {
+      const bfn b = *reinterpret_cast<const bfn*>(pv + i);
+#pragma unroll
+      for (int e = 0; e < N; ++e) v[e] += (float)b[e];
+    }
+#pragma unroll
+    for (int e = 0; e < N; ++e) {
+      const float y = v[e];
+      p.x[(size_t)t * p.ldx + i + e] = y;
+      if (p.xb) p.xb[(size_t)t * p.ldx + i + e] = (__bf16)y;
+      const size_t o = (size_t)t * p.ldc + i + e;
+      if (p.c0) {
+        if (p.f32) reinterpret_cast<float*>(p.c0)[o] = y;
+        else reinterpret_cast<__bf16*>(p.c0)[o] = (__bf16)y;
+      }
+      if (p.c1) {
+        if (p.f32) reinterpret_cast<float*>(p.c1)[o] = y;
+        else reinterpret_cast<__bf16*>(p.c1)[o] = (__bf16)y;
+      }
+    }
   }
-  for (int i = threadIdx.x; i < D; i += 256) {
-    const float v = (float)row[i] * scale;
-    x[(size_t)t * ldx + i] = v;
-    if (xb) xb[(size_t)t * ldx + i] = (__bf16)v;
+}
+
+__global__ __launch_bounds__(256) void embed_kernel(Embed p) {
+  const int t = blockIdx.x, id = token_of(p, t);
+  const __bf16 *pair = nullptr, *pv = nullptr;
+  int keep = -1, slot = -1;
+  if (p.pairs) {
+    const int* run = p.runs + 4 * p.tok_seq[t];
+    const int t0 = run[0], n = run[1], pos0 = run[3];
+    slot = run[2];
+    long r = p.buckets;
+    if (slot >= 0 && t >= t0 && t < t0 + n) {
+      if (t > t0 || pos0 > 0) {
+        const long before = t > t0 ? token_of(p, t - 1) : p.prev[slot];
+        r = (before * p.mul_prev + (long)id * p.mul_cur) % p.buckets;
+        if (r < 0) r += p.buckets;
+      }
+      if (t == t0) keep = token_of(p, t0 + n - 1);
+    }
+    pair = p.pairs + (size_t)r * p.D;
   }
+  if (p.ptab) pv = p.ptab + (size_t)min(max(p.pos[t], 0), p.npos - 1) * p.D;
+  __syncthreads();
+  if (threadIdx.x == 0) {
+    if (p.use_prev) p.ids[t] = id;
+    if (keep >= 0) p.prev[slot] = keep;
+  }
+  const __bf16* row = p.tab + (size_t)id * p.D;
+  if ((p.D & 7) == 0) embed_cols<8>(p, t, row, pair, pv);
+  else embed_cols<1>(p, t, row, pair, pv);
 }
 
 // ---- x[t] += norm(y) * w (w null: x[t] += y); y = one row (the sum of `nslab` slabs' rows), or (topk)
 // sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t], the shared expert); y null: x is only read. Optional second norm (the
 // next sublayers' or the model's last one) of the new x into `on`. norm: (v - mean) / sqrt(var + eps), or (rms)
-// v / sqrt(mean(v^2) + eps).
+// v / sqrt(mean(v^2) + eps). Without `keep` the new x is y (+ `add`, a vector) itself. The normed x may go out with two weights
+// (`ow` / `ow2`), and (gate) times a gate per column.
 // A workgroup per row (`rows`: gathered), 4 consecutive columns x NV per thread in registers.
 struct NormAdd {
   const float* y;
   const float* topw;
   const float* w;
   float* x;
-  __bf16* xb;
+  void* xb;             // optional copy of the new x, activation type
   const float* ow;      // optional output norm weight
   void* on;             // its output, activation type
   const int* rows;      // optional: row i of the launch is row rows[i] of x
@@ -84,6 +138,13 @@ struct NormAdd {
   float eps;
   int nslab;
   long slab;            // elements between slabs
+  long ldxb;
+  const float* add;     // optional [D], added to y
+  int keep;
+  const float* ow2;     // optional second weight of the output norm
+  void* on2;            // its output, row stride ldo
+  const void* gate;     // optional [rows][ldg], activation type: on *= gate
+  long ldg;
 };
 
 // 4 consecutive values, columns i .. i + 3 of a row of D (VEC: D and the row strides are multiples of 4)
@@ -96,6 +157,22 @@ DEVI f32x4 row4(const float* p, int i, int D) {
 #pragma unroll
     for (int e = 0; e < 4; ++e)
       if (i + e < D) v[e] = p[i + e];
+  }
+  return v;
+}
+template <bool VEC>
+DEVI f32x4 row4(const __bf16* p, int i, int D) {
+  typedef __bf16 bf4 __attribute__((ext_vector_type(4)));
+  f32x4 v = f32x4{0.f, 0.f, 0.f, 0.f};
+  if (VEC) {
+    if (i < D) {
+      const bf4 b = *reinterpret_cast<const bf4*>(p + i);
+      v = f32x4{(float)b[0], (float)b[1], (float)b[2], (float)b[3]};
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (i + e < D) v[e] = (float)p[i + e];
   }
   return v;
 }
@@ -151,7 +228,9 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
   float* xr = p.x + (size_t)t * p.ldx;
   f32x4 v[NV], x[NV], w[NV];
 #pragma unroll
-  for (int j = 0; j < NV; ++j) x[j] = row4<VEC>(xr, (threadIdx.x + j * NTH) * 4, D);
+  for (int j = 0; j < NV; ++j)
+    x[j] = p.keep ? row4<VEC>(xr, (threadIdx.x + j * NTH) * 4, D)
+                  : p.add ? row4<VEC>(p.add, (threadIdx.x + j * NTH) * 4, D) : f32x4{0.f, 0.f, 0.f, 0.f};
   if (p.y) {
 #pragma unroll
     for (int j = 0; j < NV; ++j)
@@ -182,7 +261,10 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
       const int i = (threadIdx.x + j * NTH) * 4;
       x[j] += v[j] * w[j];
       put4<VEC>(xr, i, D, x[j]);
-      if (p.xb) put4<VEC>(p.xb + (size_t)t * p.ldx, i, D, x[j]);
+      if (p.xb) {
+        if (p.f32) put4<VEC>(reinterpret_cast<float*>(p.xb) + (size_t)t * p.ldxb, i, D, x[j]);
+        else put4<VEC>(reinterpret_cast<__bf16*>(p.xb) + (size_t)t * p.ldxb, i, D, x[j]);
+      }
     }
   }
   if (!p.ow) return;
@@ -192,8 +274,20 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int i = (threadIdx.x + j * NTH) * 4;
-    if (p.f32) put4<VEC>(reinterpret_cast<float*>(p.on) + (size_t)blockIdx.x * p.ldo, i, D, x[j] * w[j]);
-    else put4<VEC>(reinterpret_cast<__bf16*>(p.on) + (size_t)blockIdx.x * p.ldo, i, D, x[j] * w[j]);
+    f32x4 y = x[j] * w[j];
+    if (p.gate)
+      y *= p.f32 ? row4<VEC>(reinterpret_cast<const float*>(p.gate) + (size_t)blockIdx.x * p.ldg, i, D)
+                 : row4<VEC>(reinterpret_cast<const __bf16*>(p.gate) + (size_t)blockIdx.x * p.ldg, i, D);
+    if (p.f32) put4<VEC>(reinterpret_cast<float*>(p.on) + (size_t)blockIdx.x * p.ldo, i, D, y);
+    else put4<VEC>(reinterpret_cast<__bf16*>(p.on) + (size_t)blockIdx.x * p.ldo, i, D, y);
+  }
+  if (!p.ow2) return;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int i = (threadIdx.x + j * NTH) * 4;
+    const f32x4 y = x[j] * row4<VEC>(p.ow2, i, D);
+    if (p.f32) put4<VEC>(reinterpret_cast<float*>(p.on2) + (size_t)blockIdx.x * p.ldo, i, D, y);
+    else put4<VEC>(reinterpret_cast<__bf16*>(p.on2) + (size_t)blockIdx.x * p.ldo, i, D, y);
   }
 }
 
@@ -213,7 +307,8 @@ int norm_add_v(const NormAdd& p, int n, hipStream_t st) {
 
 inline int norm_add(const NormAdd& p, int n, hipStream_t st) {
   if (n < 1 || p.D < 1) return -1;
-  const bool vec = !(p.D & 3) && !(p.ldx & 3) && !(p.ldy & 3) && !(p.ldo & 3);
+  const bool vec = !(p.D & 3) && !(p.ldx & 3) && !(p.ldy & 3) && !(p.ldo & 3) && !(p.ldxb & 3) && !(p.ldg & 3) &&
+                   !(((uintptr_t)p.gate | (uintptr_t)p.xb | (uintptr_t)p.add) & 15);
   return vec ? norm_add_v<true>(p, n, st) : norm_add_v<false>(p, n, st);
 }
 
@@ -262,7 +357,7 @@ struct AttnRows {
   const int *pos, *slot;
   void *qo, *kc, *vc;
   long ldq, ldqo, ldc;        // row strides: projections, qo, caches
-  int H, G, D, Dp, rot;
+  int H, G, D, Dp, rot, V;    // V: columns of a value head
   float eps;
 };
 
@@ -270,7 +365,7 @@ template <typename T>
 __global__ __launch_bounds__(256) void attn_rows_kernel(AttnRows p) {
   __shared__ float sh[4];
   const int t = blockIdx.x, D = p.D, slot = p.slot[t];
-  const float* f = p.cs + (size_t)p.pos[t] * p.rot;
+  const float* f = p.rot ? p.cs + (size_t)p.pos[t] * p.rot : nullptr;
   auto norm = [&](const float* a, int n) {
     float s = 0.f;
     for (int i = threadIdx.x; i < n; i += 256) s += a[i] * a[i];
@@ -301,7 +396,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnRows p) {
   if (slot < 0) return;
   put(k, p.kn, ik, p.G, (T*)p.kc + (size_t)slot * p.ldc);
   T* vo = (T*)p.vc + (size_t)slot * p.ldc;
-  for (int e = threadIdx.x; e < p.G * D; e += 256) vo[(size_t)(e / D) * p.Dp + e % D] = (T)v[e];
+  for (int e = threadIdx.x; e < p.G * p.V; e += 256) vo[(size_t)(e / p.V) * p.Dp + e % p.V] = (T)v[e];
 }
 
 // the same for heads of a multiple of 4 columns: the row's q and k stay in registers, NV groups of 4 columns per thread
@@ -311,7 +406,7 @@ __global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
   typedef T t4 __attribute__((ext_vector_type(4)));
   const int t = blockIdx.x, D4 = p.D >> 2, nq = p.H * D4, n = nq + p.G * D4, slot = p.slot[t];
   const float *q = p.q + (size_t)t * p.ldq, *k = p.k + (size_t)t * p.ldq, *v = p.v + (size_t)t * p.ldq;
-  const float* f = p.cs + (size_t)p.pos[t] * p.rot;
+  const float* f = p.rot ? p.cs + (size_t)p.pos[t] * p.rot : nullptr;
   f32x4 x[NV];
   float sq = 0.f, sk = 0.f;
 #pragma unroll
@@ -360,16 +455,23 @@ __global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
     } else {
       const size_t d = (size_t)slot * p.ldc + (size_t)h * p.Dp + c;
       *reinterpret_cast<t4*>((T*)p.kc + d) = o;
-      const f32x4 z = p.v == p.k ? x[j] : *reinterpret_cast<const f32x4*>(v + 4 * i);
-      *reinterpret_cast<t4*>((T*)p.vc + d) = t4{(T)z[0], (T)z[1], (T)z[2], (T)z[3]};
+      if (p.v == p.k) *reinterpret_cast<t4*>((T*)p.vc + d) = t4{(T)x[j][0], (T)x[j][1], (T)x[j][2], (T)x[j][3]};
     }
+  }
+  if (p.v == p.k || slot < 0) return;
+  const int V4 = p.V >> 2;
+  for (int e = threadIdx.x; e < p.G * V4; e += NTH) {
+    const int h = e / V4;
+    const f32x4 z = *reinterpret_cast<const f32x4*>(v + 4 * e);
+    *reinterpret_cast<t4*>((T*)p.vc + (size_t)slot * p.ldc + (size_t)h * p.Dp + 4 * (e - h * V4)) =
+        t4{(T)z[0], (T)z[1], (T)z[2], (T)z[3]};
   }
 }
 
 template <typename T>
 int attn_rows_t(const AttnRows& p, int n, hipStream_t st) {
   const int cols = (p.H + p.G) * p.D;
-  const bool vec = !(p.D & 3) && !(p.ldq & 3) && !(p.Dp & 3) && !(p.ldqo & 3) && !(p.ldc & 3) &&
+  const bool vec = !((p.D | p.V) & 3) && !(p.ldq & 3) && !(p.Dp & 3) && !(p.ldqo & 3) && !(p.ldc & 3) &&
                    !(((uintptr_t)p.q | (uintptr_t)p.k | (uintptr_t)p.v) & 15);
 #define NLS_AR(NV, NTH) \
   if (vec && cols <= 4 * NV * NTH) { \
@@ -551,28 +653,32 @@ __global__ __launch_bounds__(1024) void argmax_kernel(const float* __restrict__ 
 extern "C" {
 using namespace nls_stack;
 
+// pairs (optional): [buckets + 1][D] with the slots' previous tokens; ptab (optional): [npos][D]
 int nls_stack_embed(int* ids, const int* next_ids, const int* use_prev, const void* tab, int V, int D, float scale,
-                    float* x, void* xb, long ldx, int T, void* stream) {
-  if (T < 1 || D < 1 || V < 1) return -1;
-  hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, ids, next_ids, use_prev,
-                     (const __bf16*)tab, V, D, scale, x, (__bf16*)xb, ldx);
+                    float* x, void* xb, long ldx, int T, void* c0, void* c1, long ldc, int f32, const void* pairs, int buckets,
+                    int mul_prev, int mul_cur, int* prev, const int* runs, const int* tok_seq, const void* ptab, int npos,
+                    const int* pos, void* stream) {
+  if (T < 1 || D < 1 || V < 1 || (pairs && (buckets < 1 || !prev || !runs || !tok_seq)) || (ptab && (npos < 1 || !pos))) return -1;
+  const Embed p{ids, next_ids, use_prev, (const __bf16*)tab, x, (__bf16*)xb, c0, c1, (const __bf16*)pairs, prev, runs, tok_seq,
+                (const __bf16*)ptab, pos, ldx, ldc, V, D, buckets, mul_prev, mul_cur, npos, f32, scale};
+  hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
   return (int)hipGetLastError();
 }
 
-int nls_norm_add(const float* y, long ldy, const float* topw, int topk, long sh0, const float* w, float* x, void* xb,
-                 long ldx, const float* ow, void* on, long ldo, int D, int T, float eps, int f32, int rms, int nslab, long slab,
-                 void* stream) {
-  if (!y || nslab < 1 || (slab & 3)) return -1;
-  return norm_add(NormAdd{y, topw, w, x, (__bf16*)xb, ow, on, nullptr, ldy, ldx, ldo, sh0, D, topk, f32, rms, eps, nslab, slab},
-                  T,
-                  (hipStream_t)stream);
+int nls_norm_add(const float* y, long ldy, const float* topw, int topk, long sh0, const float* w, float* x, long ldx, void* xb,
+                 long ldxb, const float* ow, void* on, const float* ow2, void* on2, long ldo, const float* add, int keep, int D,
+                 int T, float eps, int f32, int rms, int nslab, long slab, void* stream) {
+  if (!y || nslab < 1 || (slab & 3) || (ow2 && (!ow || !on2)) || (keep && add)) return -1;
+  return norm_add(NormAdd{y, topw, w, x, xb, ow, on, nullptr, ldy, ldx, ldo, sh0, D, topk, f32, rms, eps, nslab, slab, ldxb, add,
+                          keep, ow2, on2, nullptr, 0}, T, (hipStream_t)stream);
 }
 
-// out[i] = norm(x[rows ? rows[i] : i]) * w
-int nls_row_norm(const float* x, long ldx, const int* rows, const float* w, void* out, long ldo, int D, int n,
-                 float eps, int f32, int rms, void* stream) {
+// out[i] = norm(x[rows ? rows[i] : i]) * w (* gate[i]); w2, out2: the same with another weight
+int nls_row_norm(const float* x, long ldx, const int* rows, const float* w, void* out, const float* w2, void* out2, long ldo,
+                 const void* gate, long ldg, int D, int n, float eps, int f32, int rms, void* stream) {
+  if (w2 && !out2) return -1;
   return norm_add(NormAdd{nullptr, nullptr, nullptr, const_cast<float*>(x), nullptr, w, out, rows, 0, ldx, ldo, -1, D, 0,
-                          f32, rms, eps, 1, 0}, n, (hipStream_t)stream);
+                          f32, rms, eps, 1, 0, 0, nullptr, 1, w2, out2, gate, ldg}, n, (hipStream_t)stream);
 }
 
 int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq, long ldcq, const float* dkv,
@@ -588,13 +694,13 @@ int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq
   return (int)hipGetLastError();
 }
 
-// heads of D columns, Dp apart in the outputs; rot even, at most D
+// heads of D columns (values: V), Dp apart in the outputs; rot even, at most D
 int nls_attn_rows(const float* q, const float* k, const float* v, long ldq, const float* qn, const float* kn, const float* cs,
                   const int* pos, const int* slot, void* qo, long ldqo, void* kc, void* vc, long ldc, int T, int H, int G,
-                  int D, int Dp, int rot, float eps, int f32, void* stream) {
-  if (T < 1 || H < 1 || G < 1 || D < 1 || Dp < D || (rot & 1) || rot < 0 || rot > D || (long)H * Dp > ldqo || (long)G * Dp > ldc)
+                  int D, int V, int Dp, int rot, float eps, int f32, void* stream) {
+  if (T < 1 || H < 1 || G < 1 || D < 1 || V < 1 || Dp < D || Dp < V || (v == k && V != D) || (rot && !cs) || (rot & 1) || rot < 0 || rot > D || (long)H * Dp > ldqo || (long)G * Dp > ldc)
     return -1;
-  AttnRows p{q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, ldq, ldqo, ldc, H, G, D, Dp, rot, eps};
+  AttnRows p{q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, ldq, ldqo, ldc, H, G, D, Dp, rot, V, eps};
   return f32 ? attn_rows_t<float>(p, T, (hipStream_t)stream) : attn_rows_t<__bf16>(p, T, (hipStream_t)stream);
 }
 

@@ -1,8 +1,9 @@
 """Decoder stacks assembled from a config: a list of layers, each a mixer plus an optional feed-forward.
 
 A mixer or feed-forward is a class that loads its weights, adds its step buffers, and runs on the rows of a step; a layer
-class (OutputNormLayer, SharedNormLayer) places the norms and joins the sublayers. The per-token cache rows (paged) and the
-per-sequence states (slots) of all layers belong to the engine, which sees them as `kv_cache` / `state_pool`. Everything
+class (OutputNormLayer, SharedNormLayer) places the norms and joins the sublayers. A looped model runs some layers several
+times with the same weights. The per-token cache rows (paged) and the per-sequence states (slots) of all layer runs belong to
+the engine, which sees them as `kv_cache` / `state_pool`. Everything
 runs on the HIP kernels of csrc/stack (ops/stack.py): bf16 operands with an f32 residual, or `dtype=torch.float32` for 32-bit
 throughout.
 
@@ -49,6 +50,8 @@ class StackBuffers:
     x: torch.Tensor                     # f32 residual
     xb: Optional[torch.Tensor]          # its bf16 rounding (None: 32-bit model, the residual itself is the operand)
     h: Optional[torch.Tensor]           # normed residual that the sublayers read (None: they read the residual)
+    h2: Optional[torch.Tensor]          # with its second norm: what the feed-forward reads (None: the same)
+    xx: Optional[torch.Tensor]          # looped models: [x | embedding output], the operand ahead of each pass
     y: Optional[torch.Tensor]           # f32 sublayer output (layers with a shared norm: the slabs of their output product)
     hn: torch.Tensor                    # normed rows of the head
     logits: torch.Tensor
@@ -330,31 +333,35 @@ class _SharedPart(_Part):
         """[width of the model, out_width]: the output projection, zero in the operand's padding columns."""
         raise NotImplementedError
 
-    def bind(self, b: StackBuffers, out: torch.Tensor) -> dict:
-        """Step buffers and launches; "inputs": the segments of the layer's input launch."""
+    def bind(self, b: StackBuffers, out: torch.Tensor, x: torch.Tensor) -> dict:
+        """Step buffers and launches; "inputs": the segments of the layer's input launch, which read x."""
         raise NotImplementedError
 
 
 class AttentionPart(_SharedPart):
     """Grouped-query softmax attention: queries and keys optionally RMS-normed over their whole projections, rotary positions
-    on the first columns of each head, values projected on their own or equal to the projected keys, a sigmoid gate per
-    head. The cache holds the finished keys and the values, [2][slots][kv_heads * padded head]."""
+    on the first columns of each head, values projected on their own or equal to the projected keys, optionally a sigmoid gate
+    per head, a sliding window with kept first keys, one more in the denominator. The cache holds the finished keys and the
+    values, [2][slots][kv_heads * padded head]."""
 
     def __init__(self, model, i, cfg, prefix, scale=1.0):
         super().__init__(model, i, cfg, prefix, scale)
         c, d, design = cfg, model.cfg.d_model, model.cfg.design
-        H, G, D = c.heads, c.kv_heads, c.dim
+        H, G, D, V = c.heads, c.kv_heads, c.dim, c.vdim
         self.attends = True
-        self.Dp, self.mfma = K.head_pad(D)
+        self.Dp, self.mfma = K.head_pad(max(D, V))
         self.mfma = self.mfma and not model.f32
         self.own_values = design.attn_values == "projection"
-        names = [("q", H), ("k", G)] + ([("v", G)] if self.own_values else [])
-        self.qkv = self.lin(torch.cat([self.mat(n, (h * D, d)) for n, h in names]))
+        names = [("q", H * D), ("k", G * D)] + ([("v", G * V)] if self.own_values else [])
+        self.qkv = self.lin(torch.cat([self.mat(n, (rows, d)) for n, rows in names]))
+        self.mask = dict(window=c.window, keep=c.keep_first, sink=design.attn_sink)
+        if not design.attn_gate and scale != 1.0:
+            raise ValueError("a weighted attention output needs its head gate")
         self.qn = self.kn = None
         if design.attn_qk_norm == "projection":
             self.qn, self.kn = self.vecn("q.norm", H * D), self.vecn("k.norm", G * D)
-        self.g = self.lin("g", (H, d))
-        self.cs = model.rope(c.rot_base, c.rot_dims)
+        self.g = self.lin("g", (H, d)) if design.attn_gate else None
+        self.cs = model.rope(c.rot_base, c.rot_dims) if c.rot_dims else None
         self.cache_width = 2 * G * self.Dp
         self.out_width = K.act_ld(H * self.Dp)
         self.groups = K.attn_groups(H, G)
@@ -368,15 +375,15 @@ class AttentionPart(_SharedPart):
 
     def out_weight(self):
         c, d = self.cfg, self.m.cfg.d_model
-        w = self.mat("o", (d, c.heads * c.dim)).view(d, c.heads, c.dim)
-        w = torch.nn.functional.pad(w, (0, self.Dp - c.dim)).reshape(d, c.heads * self.Dp)
+        w = self.mat("o", (d, c.heads * c.vdim)).view(d, c.heads, c.vdim)
+        w = torch.nn.functional.pad(w, (0, self.Dp - c.vdim)).reshape(d, c.heads * self.Dp)
         return torch.nn.functional.pad(w, (0, self.out_width - w.shape[1]))
 
-    def bind(self, b, out):
+    def bind(self, b, out, x):
         c, P, f = self.cfg, b.pad, torch.float32
         H, G, D = c.heads, c.kv_heads, c.dim
-        qkv = self.scratch(b, "attn.qkv", P, self.qkv.N, f)
-        gate = self.scratch(b, "attn.gate", P, H, f)
+        qkv = self.scratch(b, "attn.qkv", P, K.pad_to(self.qkv.N, 4), f)
+        gate = self.scratch(b, "attn.gate", P, H, f) if self.g is not None else None
         q = self.scratch(b, f"attn.q{D}", P, H * self.Dp)
         n = _SPLIT_WG // self.groups + 1                  # rows x splits
         part = (self.scratch(b, "attn.po", 1, n * H * self.Dp, f), self.scratch(b, "attn.pm", 1, n * H * 2, f),
@@ -384,22 +391,23 @@ class AttentionPart(_SharedPart):
         k0 = H * D
         return dict(q=q, gate=gate, out=out, part=part, qp=qkv, kp=qkv[:, k0:],
                     vp=qkv[:, k0 + G * D:] if self.own_values else qkv[:, k0:],
-                    inputs=[K.Seg(self.qkv, b.act, qkv), K.Seg(self.g, b.act, gate, "sigmoid", alpha=self.scale)])
+                    inputs=[K.Seg(self.qkv, x, qkv)] + ([K.Seg(self.g, x, gate, "sigmoid", alpha=self.scale)]
+                                                        if self.g is not None else []))
 
     def run(self, b, e, cache, state, step: "_Step"):
         c, st, T = self.cfg, step.st, step.T
         kc, vc = cache[0], cache[1]
         K.attn_rows(e["qp"], e["kp"], e["vp"], self.qn, self.kn, self.cs, b.pos, b.slot, e["q"], kc, vc, T, c.heads,
-                    c.kv_heads, c.dim, self.Dp, c.rot_dims, self.m.cfg.eps, st)
+                    c.kv_heads, c.dim, self.Dp, c.rot_dims, self.m.cfg.eps, st, V=c.vdim)
         plan = step.plan
         if plan is None or plan.rest:
             ns = max(1, min(_SPLIT_CAP, _SPLIT_WG // (T * self.groups))) if self.mfma else 1
             K.gqa_attention(e["q"], kc, vc, e["gate"], e["out"], e["part"], b.block_tables, step.block_size, b.tok_seq,
                             b.ctx_len if plan is None else plan.actx, T, c.heads, c.kv_heads, self.Dp, self.mfma, ns,
-                            c.scale, st)
+                            c.scale, st, **self.mask)
         if plan is not None:
             K.gqa_prefill(e["q"], kc, vc, plan.xmap, plan.blocks, plan.nblocks, plan.waves, e["gate"], e["out"], c.heads,
-                          c.kv_heads, self.Dp, c.scale, st)
+                          c.kv_heads, self.Dp, c.scale, st, **self.mask)
 
 
 class GlaPart(_SharedPart):
@@ -433,7 +441,7 @@ class GlaPart(_SharedPart):
         c, d = self.cfg, self.m.cfg.d_model
         return torch.nn.functional.pad(self.mat("o", (d, c.heads * c.vdim)), (0, self.out_width - c.heads * c.vdim))
 
-    def bind(self, b, out):
+    def bind(self, b, out, x):
         c, P, f = self.cfg, b.pad, torch.float32
         HD, HV = c.heads * c.dim, c.heads * c.vdim
         z = self.scratch(b, "gla.qkva", P, self.ld)
@@ -441,7 +449,7 @@ class GlaPart(_SharedPart):
         o = self.scratch(b, "gla.o", P, HV, f) if c.vdim > 128 else None
         g = self.scratch(b, "gla.g", P, HV)
         return dict(q=z, k=z[:, HD:], v=z[:, 2 * HD:], low=z[:, self.low:], a=a, o=o, g=g, out=out,
-                    inputs=[K.Seg(self.qkva, b.act, z), K.Seg(self.g, b.act, g, "silu")],
+                    inputs=[K.Seg(self.qkva, x, z), K.Seg(self.g, x, g, "silu")],
                     decay=K.LinLaunch([K.Seg(self.a2, z, a, "sigpow", xcol=self.low, bias=self.a2b, alpha=1.0 / c.tau)]))
 
     def run(self, b, e, cache, state, step: "_Step"):
@@ -468,9 +476,140 @@ class GlaPart(_SharedPart):
             K.scan_out(e["o"], self.norm, e["g"], e["out"], H, V, T, eps, st)
 
 
+class LightningPart(_SharedPart):
+    """Linear attention with one constant decay per head: silu on queries, keys and values, a recurrent state per head read
+    after each token's update; RMS norm over all heads' outputs together, sigmoid gate. Runs on the kernels of gated linear
+    attention, whose decays are a row that every token shares."""
+
+    def __init__(self, model, i, cfg, prefix, scale=1.0):
+        super().__init__(model, i, cfg, prefix, scale)
+        c, d = cfg, model.cfg.d_model
+        H, D, V = c.heads, c.dim, c.vdim
+        if D > 256 or H * V > 16384:
+            raise ValueError(f"lightning attention: key width {D} > 256 or {H} x {V} outputs > 16384")
+        self.qkv = self.lin(torch.cat([self.mat("q", (H * D, d)), self.mat("k", (H * D, d)), self.mat("v", (H * V, d))]))
+        self.g = self.lin("g", (H * V, d))
+        self.norm = (self.vecn("norm", H * V) * scale).contiguous()
+        self.a = torch.tensor(c.decay, dtype=torch.float32, device=model.device).repeat_interleave(D)[None].expand(2, -1)
+        self.out_width = K.act_ld(H * V)
+
+    def state_shapes(self):
+        c = self.cfg
+        return {"S": c.heads * c.dim * c.vdim}
+
+    def out_weight(self):
+        c, d = self.cfg, self.m.cfg.d_model
+        return torch.nn.functional.pad(self.mat("o", (d, c.heads * c.vdim)), (0, self.out_width - c.heads * c.vdim))
+
+    def bind(self, b, out, x):
+        c, P = self.cfg, b.pad
+        HD, HV = c.heads * c.dim, c.heads * c.vdim
+        z = self.scratch(b, "lightning.qkv", P, K.pad_to(2 * HD + HV, 8))
+        o = self.scratch(b, "lightning.o", P, K.pad_to(HV, 4), torch.float32)
+        g = self.scratch(b, "lightning.g", P, K.pad_to(HV, 8))
+        return dict(q=z, k=z[:, HD:], v=z[:, 2 * HD:], o=o, g=g, out=out,
+                    inputs=[K.Seg(self.qkv, x, z, "silu"), K.Seg(self.g, x, g, "sigmoid")])
+
+    def run(self, b, e, cache, state, step: "_Step"):
+        c, st, T, n, eps = self.cfg, step.st, step.T, step.nruns, self.m.cfg.eps
+        H, D, V, S = c.heads, c.dim, c.vdim, state["S"]
+        if T == n and V % 4 == 0 and V <= 1024:
+            K.gla_step(e["q"], e["k"], e["v"], self.a, None, 1.0, S, b.runs, T, None, None, None, H, D, V, eps, st, o=e["o"])
+        else:
+            shape = K.gla_shape(T, n, H, V)
+            seg = None
+            if shape[0] > 1:
+                seg = (self.m.grown(b, "gla.seg", n * shape[0], H * D * V, torch.float32),
+                       self.m.grown(b, "gla.segw", n * shape[0], H * D, torch.float32))
+            K.gla_scan(e["q"], e["k"], e["v"], self.a, 1.0, e["o"], None, None, None, S, b.runs, n, H, D, V, eps, shape, seg, st)
+        K.row_norm(e["o"], None, self.norm, e["out"], T, eps, st, rms=True, gate=e["g"])
+
+
+class DeltaPart(_SharedPart):
+    """Gated delta rule: queries, keys and values through a short causal convolution and silu, unit queries and keys, a recurrent
+    state per head with a low-rank decay per key channel, corrected by each token towards its value; per-head RMS norm, one
+    weight for all heads, a low-rank sigmoid gate."""
+
+    def __init__(self, model, i, cfg, prefix, scale=1.0):
+        super().__init__(model, i, cfg, prefix, scale)
+        c, d, dev = cfg, model.cfg.d_model, model.device
+        H, G, D, V = c.heads, c.kv_heads, c.dim, c.vdim
+        if D > 256:
+            raise ValueError(f"delta rule: key width {D} > 256")
+        a1, g1 = self.t("a1").to(dev), self.t("g1").to(dev)
+        self.ra, self.rg = a1.shape[0], g1.shape[0]
+        # one buffer [q | k | v | zeros | a1 | zeros | g1]: the low-rank inputs start at a linear layer's alignment
+        self.nch = 2 * G * D + H * V
+        self.low, qkv = K.act_ld(self.nch), [self.mat("q", (G * D, d)), self.mat("k", (G * D, d)), self.mat("v", (H * V, d))]
+        self.lowg = self.low + K.act_ld(self.ra)
+        gap = lambda n: a1.new_zeros(n, d)      # noqa: E731
+        self.zw = self.lin(torch.cat(qkv + [gap(self.low - self.nch), a1, gap(self.lowg - self.low - self.ra), g1]))
+        self.ld = self.lowg + K.act_ld(self.rg)
+        self.conv = torch.cat([self.mat(n + ".conv", (w, c.conv)) for n, w in (("q", G * D), ("k", G * D), ("v", H * V))])
+        self.conv = self.conv.to(torch.float32).contiguous()
+        self.b = self.lin("b", (H, d))
+        # exp(-A softplus(z)) = sigmoid(-z)^A
+        a2, g2 = -self.mat("a2", (H * D, self.ra)), self.mat("g2", (H * V, self.rg))
+        self.a2, self.g2 = self.lin(a2), self.lin(g2)
+        self.a2r, self.g2r = (w.to(model.dtype).contiguous() for w in (a2, g2))
+        self.dt = -self.vecn("dt_bias", H * D)
+        self.rate = self.vecn("A_log", H).exp().repeat_interleave(D).contiguous()
+        self.norm = (self.vecn("norm", V) * scale).repeat(H).contiguous()
+        self.out_width = K.act_ld(H * V)
+
+    def state_shapes(self):
+        c = self.cfg
+        s = {"S": c.heads * c.dim * c.vdim}
+        if c.conv > 1:
+            s["conv"] = (c.conv - 1) * self.nch
+        return s
+
+    def out_weight(self):
+        c, d = self.cfg, self.m.cfg.d_model
+        return torch.nn.functional.pad(self.mat("o", (d, c.heads * c.vdim)), (0, self.out_width - c.heads * c.vdim))
+
+    def bind(self, b, out, x):
+        c, P, f = self.cfg, b.pad, torch.float32
+        HD, HV, GD = c.heads * c.dim, c.heads * c.vdim, c.kv_heads * c.dim
+        z, y = self.scratch(b, "delta.z", P, self.ld), self.scratch(b, "delta.y", P, K.pad_to(self.nch, 8))
+        fac, beta = self.scratch(b, "delta.fac", P, 2 * c.kv_heads, f), self.scratch(b, "delta.beta", P, c.heads, f)
+        a, g = self.scratch(b, "delta.a", P, HD, f), self.scratch(b, "delta.g", P, K.pad_to(HV, 8))
+        o = self.scratch(b, "delta.o", P, HV, f) if c.vdim > 128 else None
+        return dict(z=z, q=y, k=y[:, GD:], v=y[:, 2 * GD:], fac=fac, beta=beta, a=a, g=g, o=o, out=out,
+                    low=z[:, self.low:], lowg=z[:, self.lowg:],
+                    inputs=[K.Seg(self.zw, x, z), K.Seg(self.b, x, beta, "sigmoid")],
+                    gates=K.LinLaunch([K.Seg(self.a2, z, a, "sigpow", xcol=self.low, bias=self.dt, gate=self.rate),
+                                       K.Seg(self.g2, z, g, "sigmoid", xcol=self.lowg)]))
+
+    def run(self, b, e, cache, state, step: "_Step"):
+        c, st, T, n, eps = self.cfg, step.st, step.T, step.nruns, self.m.cfg.eps
+        H, G, D, V, S = c.heads, c.kv_heads, c.dim, c.vdim, state["S"]
+        single = T == n and V % 4 == 0 and V <= 1024
+        rank = max(self.ra, self.rg)
+        own = single and (rank <= 64 or (T <= 16 and rank <= 256))    # the step makes its decays and gate itself
+        if not own:
+            e["gates"].run(T, st)
+        K.delta_conv(e["z"], self.conv, e["q"], e["fac"], state.get("conv"), b.runs, b.tok_seq, T, n, H, G, D, V, st)
+        qkv = (e["q"], e["k"], e["v"], e["fac"], e["beta"])
+        if single:
+            K.delta_step(*qkv, None if own else e["a"], (e["low"], self.a2r, self.dt, self.rate), None if own else e["g"],
+                         (e["lowg"], self.g2r), self.ld, S, b.runs, T, self.norm, e["out"], H, G, D, V, eps, st)
+            return
+        shape = K.delta_shape(T, n, H, D, V)
+        seg = None
+        if shape[0] > 1:
+            seg = (self.m.grown(b, "delta.seg", n * shape[0], H * D * V, torch.float32),
+                   self.m.grown(b, "delta.segm", n * shape[0], H * D * D, torch.float32))
+        fused = V <= 64 * shape[1]
+        K.delta_scan(*qkv, e["a"], e["o"], self.norm, e["g"], e["out"] if fused else None, S, b.runs, n, H, G, D, V, eps, shape, seg,
+                     st)
+        if not fused:
+            K.scan_out(e["o"], self.norm, e["g"], e["out"], H, V, T, eps, st)
+
+
 class DensePart(_SharedPart):
     """Gated dense feed-forward: down(act(gate h) * (up h)), the activation and product in the input launch's epilogue."""
-    EPI = {"gelu_tanh": "geglu"}
+    EPI = {"gelu_tanh": "geglu", "clamped_swiglu": "swiglu"}
 
     def __init__(self, model, i, cfg, prefix, scale=1.0):
         super().__init__(model, i, cfg, prefix, scale)
@@ -485,8 +624,8 @@ class DensePart(_SharedPart):
         ff = self.cfg.ff
         return torch.nn.functional.pad(self.mat("down", (self.m.cfg.d_model, ff)), (0, self.out_width - ff))
 
-    def bind(self, b, out):
-        return dict(inputs=[K.Seg(self.gu, b.act, out, self.EPI[self.m.cfg.design.glu_act])])
+    def bind(self, b, out, x):
+        return dict(inputs=[K.Seg(self.gu, x, out, self.EPI[self.m.cfg.design.glu_act], alpha=self.cfg.limit)])
 
     def run(self, b, e, cache, state, step):
         pass
@@ -525,17 +664,21 @@ class OutputNormLayer:
 
 
 class SharedNormLayer:
-    """h = norm1(x), x <- x + the sum of the sublayers' outputs on h. The sublayers' input projections are one launch (of up
-    to ops.stack.SEGS segments), their output projections one product over the columns of all their operands; the residual
-    add and the next layer's norm are one launch."""
+    """h = norm1(x), x <- x + the sum of the sublayers' outputs on h; or (norm_place "parallel") the feed-forward reads norm2(x).
+    The sublayers' input projections are one launch (of up to ops.stack.SEGS segments), their output projections one product
+    over the columns of all their operands; the residual add and the next layer's norms are one launch."""
 
     def __init__(self, model: "StackModel", i: int, L):
         p = f"l{i}."
         self.m = model
         self.norm1 = model.norm_weight(p + "norm1")
         self.parts = [PARTS[c.kind](model, i, c, p + "mix." + sub, scale) for c, sub, scale in mixer_parts(L.mixer)]
+        self.norm2 = None
+        self.mixers = len(self.parts)
         if L.mlp is not None:
             self.parts.append(PARTS[L.mlp.kind](model, i, L.mlp, p + "mlp."))
+            if model.cfg.design.norm_place == "parallel":
+                self.norm2 = model.norm_weight(p + "norm2")
         self.o = K.PackedLinear(torch.cat([q.out_weight() for q in self.parts], 1), model.f32, model.device)
         model.weight_bytes += self.o.nbytes
 
@@ -545,18 +688,14 @@ class SharedNormLayer:
         if cat is None:
             cat = b.shared["cat", sum(widths)] = torch.zeros(b.pad, sum(widths), dtype=self.m.dtype, device=self.m.device)
         e, c0, segs = [], 0, []
-        for q, w in zip(self.parts, widths):
-            e.append(q.bind(b, cat[:, c0:c0 + w]))
+        for j, (q, w) in enumerate(zip(self.parts, widths)):
+            e.append(q.bind(b, cat[:, c0:c0 + w], b.h2 if self.norm2 is not None and j >= self.mixers else b.act))
             segs += e[-1]["inputs"]
             c0 += w
         b.launches[key, "parts"] = e
         b.launches[key, "in"] = [K.LinLaunch(segs[o:o + K.SEGS]) for o in range(0, len(segs), K.SEGS)]
         # small steps may split K: slabs of up to 512 rows, added by the residual's launch
-        rows = max(b.pad, _SLABS * b.slab_rows)
-        y = b.shared.get("slabs")
-        if y is None:
-            y = b.shared["slabs"] = torch.zeros(rows, self.m.cfg.d_model, dtype=torch.float32, device=self.m.device)
-        b.launches[key, "out"] = K.LinLaunch([K.Seg(self.o, cat, y, slabs=_SLABS, slab_rows=b.slab_rows)])
+        b.launches[key, "out"] = K.LinLaunch([K.Seg(self.o, cat, self.m.slabs(b), slabs=_SLABS, slab_rows=b.slab_rows)])
 
     def new_caches(self, slots):
         return {j: q.new_cache(slots) for j, q in enumerate(self.parts) if q.cache_width}
@@ -568,8 +707,8 @@ class SharedNormLayer:
         for j, (q, e) in enumerate(zip(self.parts, b.launches[key, "parts"])):
             q.run(b, e, kc[step.layer].get(j), state, step)
         n = b.launches[key, "out"].run(step.T, step.st)
-        K.norm_add(b.shared["slabs"], None, b.x, None, step.T, cfg.eps, step.st, rms=cfg.design.norm == "rms", slabs=n,
-                   slab_rows=b.slab_rows, **fin)
+        K.norm_add(self.m.slabs(b), None, b.x, fin.pop("copy", None), step.T, cfg.eps, step.st, rms=cfg.design.norm == "rms",
+                   slabs=n, slab_rows=b.slab_rows, **fin)
 
 
 def mixer_parts(c) -> list:
@@ -581,8 +720,8 @@ def mixer_parts(c) -> list:
 
 MIXERS = {"wkv": WkvMixer, "latent_attention": LatentMixer}
 FEED_FORWARDS = {"moe": MoeFeedForward}
-PARTS = {"attention": AttentionPart, "gla": GlaPart, "dense": DensePart}
-LAYERS = {"output": OutputNormLayer, "shared": SharedNormLayer}
+PARTS = {"attention": AttentionPart, "gla": GlaPart, "lightning": LightningPart, "channel_delta": DeltaPart, "dense": DensePart}
+LAYERS = {"output": OutputNormLayer, "shared": SharedNormLayer, "parallel": SharedNormLayer}
 
 
 @dataclass
@@ -604,7 +743,7 @@ class _Step:
     block_size: int
     st: int
     plan: Optional[_ExpandPlan] = None
-    layer: int = 0              # the layer that runs: its cache and state (its parts may be another layer's)
+    layer: int = 0              # the layer run: its cache and state (its parts may be another run's)
 
 
 # runs of at least this many rows expand (below, the latent-space attention's extra products cost less than the expansion
@@ -636,7 +775,7 @@ class StackModel:
         self.reader = r = SafetensorsReader(os.path.join(path, "model.safetensors"))
         self.cfg = cfg = StackConfig.from_dir(path, lambda n: r.shape(n) if n in r else None)
         if ctx is not None:
-            cfg.ctx = int(ctx)
+            cfg.ctx = min(int(ctx), cfg.max_positions) if cfg.max_positions else int(ctx)
         if cfg.d_model > 16384:
             raise ValueError("stack models take widths up to 16384")
         if cfg.n_expert > 512:
@@ -646,15 +785,41 @@ class StackModel:
         dev = self.device
         self.embed = r.tensor("embed").to(device=dev, dtype=torch.bfloat16).contiguous()
         self.weight_bytes += self.embed.numel() * 2
-        # one layer object per set of weights; self.owners: the one each layer runs with
-        self.owners = [i if L.weights_of is None else L.weights_of for i, L in enumerate(cfg.layers)]
+        # one layer object per set of weights; self.owners: the one each layer run has; self.passes: the loop's pass that a run
+        # starts
+        self.owners = [i if cfg.layers[i].weights_of is None else cfg.layers[i].weights_of for i, _ in cfg.order]
+        self.passes = [t for _, t in cfg.order]
         layer = LAYERS[cfg.design.norm_place]
         own = {i: layer(self, i, cfg.layers[i]) for i in sorted(set(self.owners))}
         self.layers = [own[o] for o in self.owners]
         self.final_norm = self.norm_weight("final.norm")
-        self.head = K.PackedLinear(r.tensor("head"), self.f32, dev)
+        self.head = K.PackedLinear(r.tensor("embed" if cfg.design.tied_head else "head"), self.f32, dev)
         self.weight_bytes += self.head.nbytes
+        self.pairs = self.positions = self.loop_in = None
+        if cfg.bigram is not None:
+            self.pairs = self.table("bigram", cfg.bigram.buckets + 1)
+        if cfg.max_positions:
+            self.positions = self.table("pos", cfg.max_positions)
+        if cfg.loop is not None:
+            # operand [x | padding | embedding output | padding]
+            d, w, ld = cfg.d_model, r.tensor("loop.in").to(dev), K.act_ld(cfg.d_model)
+            if tuple(w.shape) != (d, 2 * d):
+                raise ValueError(f"loop.in: shape {tuple(w.shape)}, expected {(d, 2 * d)}")
+            w = torch.cat([torch.nn.functional.pad(v, (0, ld - d)) for v in (w[:, :d], w[:, d:])], 1)
+            self.loop_in = K.PackedLinear(w, self.f32, dev)
+            self.weight_bytes += self.loop_in.nbytes
+            self.loop_step = r.tensor("loop.step").to(device=dev, dtype=torch.float32).contiguous()
+            if tuple(self.loop_step.shape) != (cfg.loop.times, d):
+                raise ValueError(f"loop.step: shape {tuple(self.loop_step.shape)}, expected {(cfg.loop.times, d)}")
         self.vocab_lo, self.vocab_hi = 0, cfg.vocab
+
+    def table(self, name: str, rows: int) -> torch.Tensor:
+        """[rows, width] vectors that are added to the embedding."""
+        t = self.reader.tensor(name).to(device=self.device, dtype=torch.bfloat16).contiguous()
+        if tuple(t.shape) != (rows, self.cfg.d_model):
+            raise ValueError(f"{name}: shape {tuple(t.shape)}, expected {(rows, self.cfg.d_model)}")
+        self.weight_bytes += t.numel() * 2
+        return t
 
     def norm_weight(self, name: str) -> torch.Tensor:
         w = self.reader.tensor(name).to(device=self.device, dtype=torch.float32)
@@ -681,16 +846,18 @@ class StackModel:
         return self._rope[key]
 
     def kv_cache(self, num_blocks: int, block_size: int = 16):
-        """Paged rows of the layers that own a cache (a layer that shares another's weights has its own): {layer: rows}."""
+        """Paged rows of the layer runs that own a cache (one that shares another's weights has its own): {run: rows}."""
         slots = num_blocks * block_size
         return {i: c for i, c in ((i, L.new_caches(slots)) for i, L in enumerate(self.layers)) if c is not None}, None
 
     def state_pool(self, slots: int):
-        """Per-sequence states, f32: {layer: {name: [slots, n]}}. A sequence's first run (position 0) ignores what its
+        """Per-sequence states, f32: {layer run: {name: [slots, n]}} (and the previous token of each slot). A sequence's first run (position 0) ignores what its
         slot holds, so a reused slot needs no clearing."""
         out = {i: {k: torch.zeros(slots, n, dtype=torch.float32, device=self.device)
                    for q in L.parts for k, n in q.state_shapes().items()} for i, L in enumerate(self.layers)}
-        return {i: d for i, d in out.items() if d}
+        if self.pairs is not None:
+            out["token"] = torch.zeros(slots, dtype=torch.int32, device=self.device)       # the previous one
+        return {i: d for i, d in out.items() if len(d)}
 
     def step_buffers(self, cap: int, max_seqs: int, max_blocks: int, logit_rows: Optional[int] = None) -> StackBuffers:
         """Step metadata is ONE int32 tensor, as in LlamaModel.step_buffers, with the runs table behind the block tables:
@@ -703,19 +870,23 @@ class StackModel:
         f = dict(dtype=torch.float32, device=dev)
         ld = K.act_ld(cfg.d_model)
         nl = min(pad, max(64, max_seqs, logit_rows or 0))
-        shared = cfg.design.norm_place == "shared"
+        shared = cfg.design.norm_place in ("shared", "parallel")
         act = lambda: torch.zeros(pad, ld, dtype=self.dtype, device=dev)      # noqa: E731
         b = StackBuffers(
             cap=cap, pad=pad, meta=meta, ids=seg[0], pos=seg[1], slot=seg[2], tok_seq=seg[3], ctx_len=seg[4],
             use_prev=seg[5], block_tables=meta[6 * pad:6 * pad + nb].view(max_seqs, max_blocks),
             runs=meta[6 * pad + nb:].view(max_seqs, 4),
             x=torch.zeros(pad, ld, **f), xb=None if self.f32 or shared else act(), h=act() if shared else None,
+            h2=act() if cfg.design.norm_place == "parallel" else None,
+            xx=torch.zeros(pad, 2 * ld, dtype=self.dtype, device=dev) if self.loop_in is not None else None,
             y=None if shared else torch.zeros(pad, cfg.d_model, **f), hn=act(),
             logits=torch.zeros(nl, cfg.vocab, **f), next_ids=torch.zeros(pad, dtype=torch.int32, device=dev))
         b.slot.fill_(-1)
         b.runs[:, 2] = -1
         for o in sorted(set(self.owners)):
             self.layers[o].bind(b, o)
+        if b.xx is not None:
+            b.launches["pass"] = K.LinLaunch([K.Seg(self.loop_in, b.xx, self.slabs(b), slabs=_SLABS, slab_rows=b.slab_rows)])
         cap_epi = dict(epi="softcap", alpha=cfg.softcap) if cfg.softcap else {}
         b.launches["head"] = K.LinLaunch([K.Seg(self.head, b.hn, b.logits, **cap_epi)])
         return b
@@ -758,6 +929,13 @@ class StackModel:
         qb, info = self.row_blocks(b.tok_seq[:T].cpu().numpy(), b.pos[:T].cpu().numpy(), T)
         return {} if qb is None else dict(qblocks=torch.from_numpy(qb).to(self.device), nqb=len(qb), row_info=info)
 
+    def slabs(self, b: StackBuffers) -> torch.Tensor:
+        """f32 outputs of a product into the residual, in up to _SLABS blocks of slab_rows rows where K is split."""
+        if "slabs" not in b.shared:
+            rows = max(b.pad, _SLABS * b.slab_rows)
+            b.shared["slabs"] = torch.zeros(rows, self.cfg.d_model, dtype=torch.float32, device=self.device)
+        return b.shared["slabs"]
+
     def grown(self, b: StackBuffers, name: str, rows: int, cols: int, dtype=None) -> torch.Tensor:
         """A [>= rows, cols] scratch that grows (eager row batches only: captured graphs never use it)."""
         key = ("grown", name, cols)
@@ -778,6 +956,12 @@ class StackModel:
         return _ExpandPlan(info["nx"], xmap, qblocks[ns:], info["nblocks"], info["waves"], info["rest"], actx)
 
     # ---- forward
+    def _norms(self, b: StackBuffers, i: int) -> dict:
+        """What the launch ahead of layer run i leaves for its sublayers, as norm_add's arguments."""
+        L = self.layers[i]
+        n = dict(out_norm=L.norm1, out=b.h)
+        return n if getattr(L, "norm2", None) is None or b.h2 is None else dict(n, out_norm2=L.norm2, out2=b.h2)
+
     @torch.no_grad()
     def forward(self, b: StackBuffers, kc, vc, T: int, block_size: int, n_split: int = 1,
                 logit_rows: Optional[torch.Tensor] = None, n_logits: Optional[int] = None, qblocks=None, nqb: int = 0,
@@ -793,17 +977,33 @@ class StackModel:
         if row_info is not None and qblocks is not None:
             step.plan = self._expand_plan(b, qblocks, row_info, T, block_size, st)
         rms = cfg.design.norm == "rms"
-        K.embed(b.ids, self.embed, b.x, b.xb, T, st, prev=(b.next_ids, b.use_prev) if feed_prev else None,
-                scale=cfg.embed_scale)
-        if b.h is not None:
-            K.row_norm(b.x, None, self.layers[0].norm1, b.h, T, cfg.eps, st, rms=rms)
         last = len(self.layers) - 1
         direct = logit_rows is None
+        ld = K.act_ld(cfg.d_model)
+        more = {}
+        if b.xx is not None:                # (the first half ahead of a first pass that no layer precedes)
+            more["copies"] = (b.xx[:, ld:], b.xx if self.passes[0] is not None else None)
+        if self.pairs is not None:
+            bg = cfg.bigram
+            more["pairs"] = (self.pairs, bg.buckets, bg.mul_prev, bg.mul_cur, state["token"], b.runs, b.tok_seq)
+        if self.positions is not None:
+            more["positions"] = (self.positions, b.pos)
+        K.embed(b.ids, self.embed, b.x, b.xb, T, st, prev=(b.next_ids, b.use_prev) if feed_prev else None,
+                scale=cfg.embed_scale, **more)
+        if b.h is not None and self.passes[0] is None:
+            h = self._norms(b, 0)
+            K.row_norm(b.x, None, h["out_norm"], b.h, T, cfg.eps, st, rms=rms, w2=h.get("out_norm2"), out2=h.get("out2"))
         for i, layer in enumerate(self.layers):
+            if self.passes[i] is not None:
+                n = b.launches["pass"].run(T, st)
+                K.norm_add(self.slabs(b), None, b.x, None, T, cfg.eps, st, rms=rms, slabs=n, slab_rows=b.slab_rows, keep=False,
+                           add=self.loop_step[self.passes[i]], **self._norms(b, i))
             if i == last:
                 fin = dict(out_norm=self.final_norm, out=b.hn) if direct else {}
+            elif self.passes[i + 1] is not None:
+                fin = dict(copy=b.xx)
             else:
-                fin = dict(out_norm=self.layers[i + 1].norm1, out=b.h) if b.h is not None else {}
+                fin = self._norms(b, i + 1) if b.h is not None else {}
             step.layer = i
             layer.run(b, self.owners[i], kc, state.get(i) if state else None, step, fin)
             if taps is not None:

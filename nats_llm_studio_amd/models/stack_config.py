@@ -23,19 +23,28 @@ class Design:
     norm_one: bool = False             # the norm's weights are stored around zero: factor 1 + w
     norm_place: str = "output"         # output: x + norm(sublayer(x)), the sublayers read x itself
                                        # shared: h = norm(x), x + mixer(h) + feed-forward(h)
+                                       # parallel: x + mixer(norm1(x)) + feed-forward(norm2(x))
     mixers: tuple = ()
     feed_forwards: tuple = ()
     rotary: str = "interleaved"        # pairs (2i, 2i + 1)
     expert_act: str = "relu2"
     router_score: str = "sigmoid"
-    glu_act: str = "gelu_tanh"         # dense feed-forward: down(act(gate) * up)
-    attn_qk_norm: str = "projection"   # attention: one RMS norm over all heads of the queries, one over the keys'
-    attn_values: str = "keys"          # attention: the values are the projected keys, unnormed and unrotated
+    glu_act: str = "gelu_tanh"         # dense feed-forward: down(act(gate) * up), or clamped_swiglu: both clamped by the
+                                       # config's limit, down(gate sigmoid(1.702 gate) (up + 1))
+    attn_qk_norm: str = "projection"   # attention: one RMS norm over all heads of the queries, one over the keys'; none
+    attn_values: str = "keys"          # attention: the values are the projected keys, unnormed and unrotated; projection
+    attn_gate: bool = True             # attention: a sigmoid gate per head
+    attn_sink: bool = False            # attention: the softmax's denominator holds one more, a score of 0 without a value
+    tied_head: bool = False            # the logits are products with the (unscaled) embedding table
+    positions: bool = False            # a learned vector per position is added to the embedding
 
 
 DESIGNS = {
     "Sekolorn": Design(mixers=("wkv", "latent_attention"), feed_forwards=("moe",)),
     "Kolodra": Design(norm="rms", norm_one=True, norm_place="shared", mixers=("parallel",), feed_forwards=("dense",)),
+    "Bibapel": Design(norm="rms", norm_place="parallel", mixers=("channel_delta", "attention", "lightning"),
+                      feed_forwards=("dense",), glu_act="clamped_swiglu", attn_qk_norm="none", attn_values="projection",
+                      attn_gate=False, attn_sink=True, tied_head=True, positions=True),
 }
 
 
@@ -62,13 +71,17 @@ class LatentConfig:
 
 @dataclass
 class AttentionConfig:
-    """Grouped-query softmax attention with partial rotary positions and a gate per head."""
+    """Grouped-query softmax attention, optionally with partial rotary positions, or over a sliding window and the first
+    tokens: position i sees j <= i if i - j < window or j < keep_first."""
     heads: int
     kv_heads: int
-    dim: int                           # of queries, keys and values
+    dim: int                           # of queries and keys
     rot_dims: int
     rot_base: float
     scale: float
+    vdim: int = 0                      # of values
+    window: int = 0                    # 0: every earlier position is seen
+    keep_first: int = 0
     kind, recurrent = "attention", False
 
 
@@ -80,6 +93,28 @@ class GlaConfig:
     vdim: int
     tau: float
     kind, recurrent = "gla", True
+
+
+@dataclass
+class LightningConfig:
+    """Linear attention with one constant decay per head, a state [dim, vdim] per head."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: List[float]
+    kind, recurrent = "lightning", True
+
+
+@dataclass
+class DeltaConfig:
+    """Gated delta rule: a state [dim, vdim] per head, decayed per key channel, that each token corrects towards its value;
+    queries, keys and values pass a causal convolution of `conv` taps. Queries and keys have kv_heads heads."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    conv: int
+    kind, recurrent = "channel_delta", True
 
 
 @dataclass
@@ -107,6 +142,7 @@ class MoeConfig:
 @dataclass
 class DenseConfig:
     ff: int
+    limit: float = 0.0                 # clamped_swiglu: bound of gate (above) and up (both sides)
     kind = "dense"
     experts = top = 0
 
@@ -116,6 +152,23 @@ class LayerConfig:
     mixer: object
     mlp: object = None                 # MoeConfig, DenseConfig or None
     weights_of: Optional[int] = None   # the layer whose tensors this one uses (resolved: never itself such a layer)
+
+
+@dataclass
+class BigramConfig:
+    """A table row per pair of neighbouring tokens: (previous * mul_prev + current * mul_cur) mod buckets; the last row is that
+    of a sequence's first token."""
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+
+
+@dataclass
+class LoopConfig:
+    """Layers start .. stop - 1 run `times` times in a row with the same weights."""
+    start: int
+    stop: int
+    times: int
 
 
 @dataclass
@@ -129,10 +182,23 @@ class StackConfig:
     ctx: int = 32768
     embed_scale: float = 1.0
     softcap: float = 0.0               # logits: softcap * tanh(logits / softcap); 0: none
+    bigram: Optional[BigramConfig] = None
+    loop: Optional[LoopConfig] = None
+    max_positions: int = 0             # rows of the learned positions (0: none)
 
     @property
     def n_layer(self) -> int:
         return len(self.layers)
+
+    @property
+    def order(self) -> List[tuple]:
+        """The layer runs of a forward pass: (layer, the loop's pass that starts with this run or None)."""
+        n = len(self.layers)
+        if self.loop is None:
+            return [(i, None) for i in range(n)]
+        a, z = self.loop.start, self.loop.stop
+        passes = [(i, t if i == a else None) for t in range(self.loop.times) for i in range(a, z)]
+        return [(i, None) for i in range(a)] + passes + [(i, None) for i in range(z, n)]
 
     @property
     def n_expert(self) -> int:
@@ -144,8 +210,8 @@ class StackConfig:
 
     @property
     def recurrent(self) -> bool:
-        """Some layer carries per-sequence state besides the paged cache."""
-        return any(L.mixer.recurrent for L in self.layers)
+        """Sequences carry state besides the paged cache: some layer's, or the previous token."""
+        return self.bigram is not None or any(L.mixer.recurrent for L in self.layers)
 
     @classmethod
     def from_json(cls, cfg: dict, shape=None) -> "StackConfig":
@@ -169,6 +235,20 @@ class StackConfig:
                   eps=float(norm["eps"]), ctx=default_ctx(),
                   embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
                   softcap=float(cfg.get("logit_softcap") or 0.0))
+        if design.positions:
+            out.max_positions = size(cfg, "max_positions", "pos")
+            out.ctx = min(out.ctx, out.max_positions)
+        bg = (cfg.get("embedding") or {}).get("bigram")
+        if bg is not None:
+            rows = shape("bigram")
+            out.bigram = BigramConfig(int(bg["buckets"]) if "buckets" in bg else int(rows[0]) - 1, int(bg["mul_prev"]),
+                                      int(bg["mul_cur"]))
+            if out.bigram.buckets < 1 or max(abs(out.bigram.mul_prev), abs(out.bigram.mul_cur)) >= 1 << 31:
+                raise ValueError("config.json: embedding.bigram needs buckets >= 1 and 32-bit factors")
+        if cfg.get("loop"):
+            lp = out.loop = LoopConfig(*(int(cfg["loop"][k]) for k in ("start", "stop", "times")))
+            if not 0 <= lp.start < lp.stop <= len(cfg["layers"]) or lp.times < 1:
+                raise ValueError(f"config.json: loop {cfg['loop']} of {len(cfg['layers'])} layers")
 
         def wkv(i, m, p):
             u = shape(p + "u")
@@ -194,23 +274,45 @@ class StackConfig:
             return mix
 
         def attention(i, m, p):
-            H = size(m, "heads", p + "g")
+            own = design.attn_values == "projection"
+            H = int(m["heads"]) if not design.attn_gate else size(m, "heads", p + "g")
             D = size(m, "dim", p + "q", 0, H)
             G = size(m, "kv_heads", p + "k", 0, D)
+            V = size(m, "vdim", p + "v", 0, G) if own else int(m.get("vdim", D))
             rot = m.get("rot") or {"dims": 0, "base": 1.0}
             rd = int(rot.get("dims", D))
+            mask = m.get("mask") or {}
+            window, keep = int(mask.get("size") or 0), int(mask.get("keep_first") or 0)
             if H % G:
                 raise ValueError(f"layer {i}: {H} query heads do not divide into {G} key heads")
-            if int(m.get("vdim", D)) != D:
+            if not own and V != D:
                 raise ValueError(f"layer {i}: the values are the keys: vdim {m['vdim']} must be dim {D}")
             if rd % 2 or not 0 <= rd <= D:
                 raise ValueError(f"layer {i}: {rd} rotated dimensions of heads of {D}")
-            return AttentionConfig(heads=H, kv_heads=G, dim=D, rot_dims=rd, rot_base=float(rot["base"]), scale=float(m["scale"]))
+            if mask and (window < 1 or keep < 0):
+                raise ValueError(f"layer {i}: attention mask {mask}")
+            return AttentionConfig(heads=H, kv_heads=G, dim=D, rot_dims=rd, rot_base=float(rot["base"]), scale=float(m["scale"]),
+                                   vdim=V, window=window, keep_first=keep)
 
         def gla(i, m, p):
             V = size(m, "vdim", p + "norm")
             H = size(m, "heads", p + "v", 0, V)
             return GlaConfig(heads=H, dim=size(m, "dim", p + "k", 0, H), vdim=V, tau=float(m["tau"]))
+
+        def lightning(i, m, p):
+            decay = [float(a) for a in m["decay"]]
+            H = int(m.get("heads", len(decay)))
+            if len(decay) != H or not all(0.0 <= a <= 1.0 for a in decay):
+                raise ValueError(f"layer {i}: {H} heads need as many decays between 0 and 1")
+            return LightningConfig(heads=H, dim=size(m, "dim", p + "k", 0, H), vdim=size(m, "vdim", p + "v", 0, H), decay=decay)
+
+        def channel_delta(i, m, p):
+            H, V = size(m, "heads", p + "b"), size(m, "vdim", p + "norm")
+            D = size(m, "dim", p + "a2", 0, H)
+            G = size(m, "kv_heads", p + "k", 0, D)
+            if H % G:
+                raise ValueError(f"layer {i}: {H} heads do not divide into {G} query and key heads")
+            return DeltaConfig(heads=H, kv_heads=G, dim=D, vdim=V, conv=size(m, "conv", p + "q.conv", 1))
 
         def parallel(i, m, p):
             return ParallelConfig(left=attention(i, m["left"], p + "left."), right=gla(i, m["right"], p + "right."),
@@ -231,9 +333,11 @@ class StackConfig:
             return mlp
 
         def dense(i, f, p):
-            return DenseConfig(ff=size(f, "ff", p + "gate"))
+            return DenseConfig(ff=size(f, "ff", p + "gate"),
+                               limit=float(f["limit"]) if design.glu_act == "clamped_swiglu" else 0.0)
 
-        mixers = {"wkv": wkv, "latent_attention": latent, "parallel": parallel}
+        mixers = {"wkv": wkv, "latent_attention": latent, "parallel": parallel, "attention": attention,
+                  "lightning": lightning, "channel_delta": channel_delta}
         feed_forwards = {"moe": moe, "dense": dense}
         owners = weight_owners(cfg["layers"])
         for i, L in enumerate(cfg["layers"]):

@@ -16,7 +16,7 @@ LIB_PATH = os.environ.get("NLS_STACK_SO") or os.path.join(_PKG, "_stack.so")
 P, I, L, F = ctypes.c_void_p, ctypes.c_int, ctypes.c_long, ctypes.c_float
 SEGS = 6
 EPI = {"none": 0, "silu": 1, "tanh": 2, "sigmoid": 3, "relu2": 4, "decay": 5, "gate": 6, "rope": 7,
-       "geglu": 8, "sigpow": 9, "softcap": 10}
+       "geglu": 8, "sigpow": 9, "softcap": 10, "swiglu": 11}
 NO_BLOCK = 1 << 30       # LinSeg.cb: output columns are not blocked
 
 
@@ -38,14 +38,17 @@ _SIGS = {
     "nls_lin_args_size": [],
     "nls_lin_small": [P, I, I, I, I, P],
     "nls_lin_gemm": [P, I, I, P],
-    "nls_stack_embed": [P, P, P, P, I, I, F, P, P, L, I, P],
-    "nls_norm_add": [P, L, P, I, L, P, P, P, L, P, P, L, I, I, F, I, I, I, L, P],
-    "nls_row_norm": [P, L, P, P, P, L, I, I, F, I, I, P],
-    "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, F, I, P],
-    "nls_gqa_attn": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, P, L, P, L, P, P, P, I, I, P],
-    "nls_gqa_prefill": [P, L, P, P, P, P, I, P, I, P, L, I, I, I, I, F, P],
+    "nls_stack_embed": [P, P, P, P, I, I, F, P, P, L, I, P, P, L, I, P, I, I, I, P, P, P, P, I, P, P],
+    "nls_norm_add": [P, L, P, I, L, P, P, L, P, L, P, P, P, P, L, P, I, I, I, F, I, I, I, L, P],
+    "nls_row_norm": [P, L, P, P, P, P, P, L, P, L, I, I, F, I, I, P],
+    "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, I, F, I, P],
+    "nls_gqa_attn": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, P, L, P, L, P, P, P, I, I, I, I, I, P],
+    "nls_gqa_prefill": [P, L, P, P, P, P, I, P, I, P, L, I, I, I, I, F, I, I, I, P],
+    "nls_delta_conv": [P, L, P, P, L, P, L, P, L, P, P, I, I, I, I, I, I, I, I, P],
+    "nls_delta_scan": [P, P, P, L, P, L, P, L, P, L, P, L, P, P, L, P, L, F, P, L, P, I, I, I, I, I, I, P, P, I, I, P],
+    "nls_delta_step": [P, P, P, L, P, L, P, L, P, L, P, P, P, P, I, P, L, P, P, I, L, P, L, P, I, P, P, L, I, I, I, I, F, I, P],
     "nls_gla_scan": [P, P, P, L, P, L, F, P, L, P, P, L, P, L, F, P, L, P, I, I, I, I, I, P, P, I, I, P],
-    "nls_gla_step": [P, P, P, L, P, L, P, P, P, I, F, F, P, L, P, I, P, P, L, P, L, I, I, I, F, I, P],
+    "nls_gla_step": [P, P, P, L, P, L, P, P, P, I, F, F, P, L, P, I, P, P, L, P, L, P, L, I, I, I, F, I, P],
     "nls_latent_rows": [P, L, I, P, P, L, P, L, I, I, I, P, P, P, P, P, L, I, F, I, P],
     "nls_stack_argmax": [P, L, I, P, I, P],
     "nls_moe_plan": [P, L, I, I, I, I, I, F, P, P, I, P, P, P, I, P],
@@ -133,8 +136,8 @@ class Seg:
     """One segment of a LinLaunch. y / x: 2-D buffers (row stride = their stride(0)); ycol / xcol: first column.
     xgs / ygs: column step per group. block = (cb, cstep): output column n -> (n / cb) * cstep + n % cb.
     routed = (entry list, xdiv): the rows are routed entries (x row = entry / xdiv, y row = entry).
-    rope = (table, pos, pairs). alpha: constant of the epilogue (sigmoid, sigpow, softcap). geglu: the rows of w alternate
-    gate and up, y has half as many columns. slabs: K splits that launches of up to slab_rows rows may use; y holds that many
+    rope = (table, pos, pairs). alpha: constant of the epilogue (sigmoid, sigpow, softcap, swiglu); sigpow: `gate`,
+    a vector, gives an exponent per column instead. geglu, swiglu: the rows of w alternate gate and up, y has half as many columns. slabs: K splits that launches of up to slab_rows rows may use; y holds that many
     slabs of slab_rows rows, added by the caller (LinLaunch.run returns how many were written)."""
 
     def __init__(self, w: PackedLinear, x: torch.Tensor, y: torch.Tensor, epi: str = "none", ycol: int = 0,
@@ -329,31 +332,47 @@ class MoePlan:
 # ---------------------------------------------------------------------------
 
 def embed(ids, table: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor], T: int, st: int, prev=None,
-          scale: float = 1.0):
+          scale: float = 1.0, copies=(), pairs=None, positions=None):
+    """x = table[id] * scale (xb: its bf16 rounding). copies: up to two more of x in the activation type, of one row stride.
+    pairs = (table, buckets, mul_prev, mul_cur, previous token of each slot, runs, tok_seq): plus the row of the token pair, and
+    the slots' tokens move on. positions = (table, pos): plus the position's row."""
     nx, up = prev if prev is not None else (None, None)
+    c0, c1 = (tuple(copies) + (None, None))[:2]
+    pt, nb, mp, mc, pv, runs, seq = pairs if pairs is not None else (None, 0, 0, 0, None, None, None)
+    tab, pos = positions if positions is not None else (None, None)
     _check(lib().nls_stack_embed(ids.data_ptr(), _p(nx), _p(up), table.data_ptr(), table.shape[0], table.shape[1], scale,
-                                 x.data_ptr(), _p(xb), x.stride(0), T, st), "nls_stack_embed")
+                                 x.data_ptr(), _p(xb), x.stride(0), T, _p(c0), _p(c1), c0.stride(0) if c0 is not None else 0,
+                                 int(c0 is not None and c0.dtype == torch.float32), _p(pt), nb, mp, mc, _p(pv), _p(runs), _p(seq),
+                                 _p(tab), tab.shape[0] if tab is not None else 0, _p(pos), st), "nls_stack_embed")
 
 
 def norm_add(y: torch.Tensor, w: Optional[torch.Tensor], x: torch.Tensor, xb: Optional[torch.Tensor], T: int, eps: float,
              st: int, plan: Optional[MoePlan] = None, shared_row0: int = -1, out_norm: Optional[torch.Tensor] = None,
-             out: Optional[torch.Tensor] = None, rms: bool = False, slabs: int = 1, slab_rows: int = 0):
-    """x[:T] += norm(y) * w, or += y without w (xb: its bf16 rounding); y may be the sum of `slabs` blocks of slab_rows rows.
-    With `plan`, y holds the routed experts' rows (token-major) and from row `shared_row0` on the shared expert's, combined
-    first. out = norm(x) * out_norm (what the next sublayers read, or the model's last norm). norm: layer norm, or RMS."""
+             out: Optional[torch.Tensor] = None, rms: bool = False, slabs: int = 1, slab_rows: int = 0, out_norm2=None, out2=None,
+             keep: bool = True, add: Optional[torch.Tensor] = None):
+    """x[:T] += norm(y) * w, or += y without w (xb: a copy in the activation type); y may be the sum of `slabs` blocks of
+    slab_rows rows. With `plan`, y holds the routed experts' rows (token-major) and from row `shared_row0` on the shared
+    expert's, combined first. out = norm(x) * out_norm (what the next sublayers read, or the model's last norm), out2 the same
+    with out_norm2. norm: layer norm, or RMS. keep False: x becomes y (+ the vector `add`)."""
     D = y.shape[1] if w is None else w.numel()
+    typed = out if out is not None else xb
+    if out2 is not None and out2.stride(0) != out.stride(0):
+        raise ValueError("norm_add: equal row strides of the outputs")
     _check(lib().nls_norm_add(y.data_ptr(), y.stride(0), _p(plan.topw) if plan else None, plan.top if plan else 0,
-                              shared_row0, _p(w), x.data_ptr(), _p(xb), x.stride(0), _p(out_norm), _p(out),
-                              out.stride(0) if out is not None else 0, D, T, eps,
-                              int(out is not None and out.dtype == torch.float32), int(rms), slabs,
+                              shared_row0, _p(w), x.data_ptr(), x.stride(0), _p(xb), xb.stride(0) if xb is not None else 0,
+                              _p(out_norm), _p(out), _p(out_norm2), _p(out2), out.stride(0) if out is not None else 0, _p(add),
+                              int(keep), D, T, eps, int(typed is not None and typed.dtype == torch.float32), int(rms), slabs,
                               slab_rows * y.stride(0), st), "nls_norm_add")
 
 
 def row_norm(x: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor, out: torch.Tensor, n: int, eps: float,
-             st: int, rms: bool = False):
-    """out[i] = norm(x[rows[i]]) * w (rows None: row i): layer norm, or RMS."""
-    _check(lib().nls_row_norm(x.data_ptr(), x.stride(0), _p(rows), w.data_ptr(), out.data_ptr(), out.stride(0),
-                              w.numel(), n, eps, int(out.dtype == torch.float32), int(rms), st), "nls_row_norm")
+             st: int, rms: bool = False, w2=None, out2=None, gate: Optional[torch.Tensor] = None):
+    """out[i] = norm(x[rows[i]]) * w (rows None: row i) (* gate[i]): layer norm, or RMS. out2: the same with w2."""
+    if (out2 is not None and out2.stride(0) != out.stride(0)) or (gate is not None and gate.dtype != out.dtype):
+        raise ValueError("row_norm: equal row strides of the outputs, a gate of their type")
+    _check(lib().nls_row_norm(x.data_ptr(), x.stride(0), _p(rows), w.data_ptr(), out.data_ptr(), _p(w2), _p(out2), out.stride(0),
+                              _p(gate), gate.stride(0) if gate is not None else 0, w.numel(), n, eps,
+                              int(out.dtype == torch.float32), int(rms), st), "nls_row_norm")
 
 
 def argmax(logits: torch.Tensor, n: int, out: torch.Tensor, st: int):
@@ -481,14 +500,69 @@ def gla_scan(q, k, v, a, qscale: float, o, norm, gate, out, state, runs, nruns: 
 
 
 def gla_step(q, k, v, a, gate_in, qscale: float, state, runs, nruns: int, norm, gate, out, H: int, D: int, V: int, eps: float,
-             st: int):
-    """gla_scan of runs of one token each (V a multiple of 4), with the norm and gate. Decays `a`, or (None) from gate_in =
-    (low-rank gate input, a2, bias, exponent): sigmoid(a2 low + bias) ^ exponent."""
+             st: int, o=None):
+    """gla_scan of runs of one token each (V a multiple of 4), with the norm and gate, or (norm None) the plain outputs in `o`.
+    Decays `a`, or (None) from gate_in = (low-rank gate input, a2, bias, exponent): sigmoid(a2 low + bias) ^ exponent."""
     lo, a2, b, ia = gate_in if a is None else (None, None, None, 0.0)
+    y = out if norm is not None else o
     _check(lib().nls_gla_step(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), _p(a), a.stride(0) if a is not None else 0,
                               _p(lo), _p(a2), _p(b), a2.shape[1] if a2 is not None else 0, ia, qscale, state.data_ptr(),
-                              state.stride(0), runs.data_ptr(), nruns, norm.data_ptr(), gate.data_ptr(), gate.stride(0),
-                              out.data_ptr(), out.stride(0), H, D, V, eps, int(out.dtype == torch.float32), st), "nls_gla_step")
+                              state.stride(0), runs.data_ptr(), nruns, _p(norm), _p(gate),
+                              gate.stride(0) if gate is not None else 0, _p(out), out.stride(0) if out is not None else 0, _p(o),
+                              o.stride(0) if o is not None else 0, H, D, V, eps, int(q.dtype == torch.float32), st),
+           "nls_gla_step")
+
+
+# ---------------------------------------------------------------------------
+# Delta rule
+# ---------------------------------------------------------------------------
+
+def delta_conv(z, w, y, fac, state, runs, tok_seq, T: int, nruns: int, H: int, G: int, D: int, V: int, st: int):
+    """y = silu(causal convolution of z) per channel, [q: G * D | k: G * D | v: H * V]; w f32 [channels, taps]; the last taps - 1
+    inputs are carried in state [slots, (taps - 1) * channels] (None for one tap). fac [rows, 2 G]: what makes the heads of q
+    (times D^-1/2) and k unit vectors."""
+    _check(lib().nls_delta_conv(z.data_ptr(), z.stride(0), w.data_ptr(), y.data_ptr(), y.stride(0), fac.data_ptr(), fac.stride(0),
+                                _p(state), state.stride(0) if state is not None else 0, runs.data_ptr(), tok_seq.data_ptr(), T,
+                                nruns, H, G, D, V, w.shape[1], int(z.dtype == torch.float32), st), "nls_delta_conv")
+
+
+def delta_shape(T: int, nruns: int, H: int, D: int, V: int):
+    """(segments, groups of 64 value columns per workgroup) of a delta_scan launch. Segments cost a second pass over the tokens
+    with D more columns, so they start where whole runs fill less than half the CUs, and stay longer."""
+    nt = 1 if V <= 64 else 2
+    wgs = H * -(-V // (64 * nt)) * nruns
+    return 1 if wgs >= 128 else max(1, min(-(-256 // wgs), (T - nruns + 1) // 128, 16)), nt
+
+
+def delta_scan(q, k, v, fac, beta, a, o, norm, gate, out, state, runs, nruns: int, H: int, G: int, D: int, V: int, eps: float,
+               shape, seg, st: int):
+    """The delta rule over each run's tokens: q, k [rows, G * D], v [rows, H * V] of one buffer, the factors of delta_conv, beta
+    [rows, H], decays a [rows, H * D]; otherwise as gla_scan. seg: (states, matrices) scratch of the segments."""
+    nseg, nt = shape
+    if nseg > 1 and (seg[0].numel() < nruns * nseg * H * D * V or seg[1].numel() < nruns * nseg * H * D * D):
+        raise ValueError("delta_scan: segment scratch too small")
+    s0, s1 = seg if nseg > 1 else (None, None)
+    f = out is not None
+    _check(lib().nls_delta_scan(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), fac.data_ptr(), fac.stride(0),
+                                beta.data_ptr(), beta.stride(0), a.data_ptr(), a.stride(0), _p(o), o.stride(0) if o is not None else 0,
+                                norm.data_ptr() if f else None, gate.data_ptr() if f else None, gate.stride(0) if f else 0, _p(out),
+                                out.stride(0) if f else 0, eps, state.data_ptr(), state.stride(0), runs.data_ptr(), nruns, H, G, D,
+                                V, nseg, _p(s0), _p(s1), nt, int(q.dtype == torch.float32), st), "nls_delta_scan")
+
+
+def delta_step(q, k, v, fac, beta, a, decay_in, gate, gate_in, ldz: int, state, runs, nruns: int, norm, out, H: int, G: int, D: int,
+               V: int, eps: float, st: int):
+    """delta_scan of runs of one token each (V a multiple of 4), with the norm and gate. Decays a, or (None) from decay_in =
+    (low-rank input, a2, bias, exponent per channel): sigmoid(a2 low + bias) ^ exponent. The gate, or (None) from gate_in =
+    (low-rank input, g2): sigmoid(g2 low). ldz: row stride of the low-rank inputs."""
+    lo, a2, b, rate = decay_in if a is None else (None, None, None, None)
+    lg, g2 = gate_in if gate is None else (None, None)
+    _check(lib().nls_delta_step(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), fac.data_ptr(), fac.stride(0),
+                                beta.data_ptr(), beta.stride(0), _p(a), a.stride(0) if a is not None else 0, _p(lo), _p(a2), _p(b),
+                                _p(rate), a2.shape[1] if a2 is not None else 0, _p(gate),
+                                gate.stride(0) if gate is not None else 0, _p(lg), _p(g2), g2.shape[1] if g2 is not None else 0, ldz,
+                                state.data_ptr(), state.stride(0), runs.data_ptr(), nruns, norm.data_ptr(), out.data_ptr(),
+                                out.stride(0), H, G, D, V, eps, int(out.dtype == torch.float32), st), "nls_delta_step")
 
 
 # ---------------------------------------------------------------------------
@@ -513,29 +587,36 @@ def attn_groups(H: int, G: int) -> int:
     return G * -(-(H // G) // 16)
 
 
-def attn_rows(q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, T: int, H: int, G: int, D: int, Dp: int, rot: int, eps: float, st: int):
-    """Norm over the whole q and k projections (qn, kn: weights or None), rotation of the first `rot` columns of each head,
-    queries to qo, keys and (as projected) values to the tokens' cache rows. q, k, v: f32 with one row stride."""
-    _check(lib().nls_attn_rows(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), _p(qn), _p(kn), cs.data_ptr(),
+def attn_rows(q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, T: int, H: int, G: int, D: int, Dp: int, rot: int, eps: float, st: int,
+              V: Optional[int] = None):
+    """Norm over the whole q and k projections (qn, kn: weights or None), rotation of the first `rot` columns of each head (cs
+    None: none), queries to qo, keys and (as projected, V columns per head) values to the tokens' cache rows. q, k, v: f32
+    with one row stride."""
+    _check(lib().nls_attn_rows(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), _p(qn), _p(kn), _p(cs),
                                pos.data_ptr(), slot.data_ptr(), qo.data_ptr(), qo.stride(0), kc.data_ptr(), vc.data_ptr(),
-                               kc.stride(0), T, H, G, D, Dp, rot, eps, int(qo.dtype == torch.float32), st), "nls_attn_rows")
+                               kc.stride(0), T, H, G, D, D if V is None else V, Dp, rot, eps, int(qo.dtype == torch.float32), st),
+           "nls_attn_rows")
 
 
 def gqa_attention(q, kc, vc, gate, out, part, block_tables, block_size: int, tok_seq, ctx_len, T: int, H: int, G: int, Dp: int,
-                  mfma: bool, ns: int, scale: float, st: int):
-    """Row-by-row attention (decoded tokens, short runs); the head gate is applied to the output. part: (partial outputs,
-    (max, sum) pairs, ticket counters) of `ns` splits."""
+                  mfma: bool, ns: int, scale: float, st: int, window: int = 0, keep: int = 0, sink: bool = False):
+    """Row-by-row attention (decoded tokens, short runs); a head gate (or None) is applied to the output. part: (partial
+    outputs, (max, sum) pairs, ticket counters) of `ns` splits. window > 0: the newest `window` keys and the first `keep`;
+    sink: the softmax's denominator holds one more, a score of 0 without a value."""
     po, pm, cnt = part
     if ns > 1 and (po.numel() < T * H * ns * Dp or pm.numel() < T * H * ns * 2 or cnt.numel() < T * attn_groups(H, G)):
         raise ValueError("gqa_attention: split workspace too small")
     _check(lib().nls_gqa_attn(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), block_tables.data_ptr(),
                               block_tables.stride(0), block_size, tok_seq.data_ptr(), ctx_len.data_ptr(), T, H, G, Dp, ns,
-                              scale, gate.data_ptr(), gate.stride(0), out.data_ptr(), out.stride(0), po.data_ptr(),
-                              pm.data_ptr(), cnt.data_ptr(), int(not mfma), int(q.dtype == torch.float32), st), "nls_gqa_attn")
+                              scale, _p(gate), gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0),
+                              po.data_ptr(), pm.data_ptr(), cnt.data_ptr(), window, keep, int(sink), int(not mfma),
+                              int(q.dtype == torch.float32), st), "nls_gqa_attn")
 
 
-def gqa_prefill(q, kc, vc, xmap, blocks, nblocks: int, waves: int, gate, out, H: int, G: int, Dp: int, scale: float, st: int):
-    """Causal attention of query blocks over their sequences' paged keys and values."""
+def gqa_prefill(q, kc, vc, xmap, blocks, nblocks: int, waves: int, gate, out, H: int, G: int, Dp: int, scale: float, st: int,
+                window: int = 0, keep: int = 0, sink: bool = False):
+    """Causal attention of query blocks over their sequences' paged keys and values (gate, window, keep, sink: as
+    gqa_attention)."""
     _check(lib().nls_gqa_prefill(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), xmap.data_ptr(), blocks.data_ptr(),
-                                 nblocks, gate.data_ptr(), gate.stride(0), out.data_ptr(), out.stride(0), H, G, Dp, waves,
-                                 scale, st), "nls_gqa_prefill")
+                                 nblocks, _p(gate), gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), H, G,
+                                 Dp, waves, scale, window, keep, int(sink), st), "nls_gqa_prefill")
