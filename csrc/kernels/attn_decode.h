@@ -176,7 +176,7 @@ __global__ __launch_bounds__(64 * WAVES) void attn_decode_mfma_kernel(
     if (win != btw) {
       btw = win;
       const int e = b0 + win * 64 + lane;
-      btreg = e * bs < end_p ? bt[e] : 0;
+      btreg = e * bs < (WIN ? last_pos : end) ? bt[e] : 0;        // (WIN: the window may reach across the gap)
     }
 #pragma unroll
     for (int i = 0; i < NGB; ++i) {

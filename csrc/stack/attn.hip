@@ -52,9 +52,11 @@ extern "C" {
 // j <= i if i - j < window or j < keep. sink: one more in the denominator, a score of 0 without a value.
 int nls_gqa_attn(const void* q, long ldq, const void* k, const void* v, const int* bt, int bts, int bs, const int* tok_seq,
                  const int* ctx_len, int T, int H, int G, int Dp, int ns, float scale, const float* gate, long ldg, void* out,
-                 long ldo, float* part_o, float* part_ml, int* cnt, int window, int keep, int sink, int plain, int f32, void* stream) {
+                 long ldo, float* part_o, float* part_ml, int* cnt, int window, int keep, int sink, int plain, int f32,
+                 void* stream) {
   using namespace nls_gqa;
-  if (T < 1 || G < 1 || H < 1 || H % G || Dp < 1 || bs < 1 || ns < 1 || ns > 64 || window < 0 || keep < 0 || (ns > 1 && (!part_o || !part_ml || !cnt)))
+  if (T < 1 || G < 1 || H < 1 || H % G || Dp < 1 || bs < 1 || ns < 1 || ns > 64 || window < 0 || keep < 0 ||
+      (ns > 1 && (!part_o || !part_ml || !cnt)))
     return -1;
   hipStream_t st = (hipStream_t)stream;
   if (plain || f32) {

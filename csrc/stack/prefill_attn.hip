@@ -12,8 +12,8 @@
 //   closes with one lane exchange; P^T goes from those registers straight into O^T += V^T P^T (V^T by transposed LDS
 //   reads in the same key order), so a row's rescale is lane-local and skipped when no maximum grew.
 // The next tile's loads are in flight in registers while a tile computes (its cache slots one tile ahead of that); one
-// barrier per tile, two LDS buffers. Under a sliding window (with kept first keys) tiles that no row sees are left out. Rows are padded in LDS (K: 16 bytes, V: 64) against bank conflicts. The epilogue applies
-// the head's output gate.
+// barrier per tile, two LDS buffers. Rows are padded in LDS (K: 16 bytes, V: 64) against bank conflicts. Under a sliding window
+// (with kept first keys) tiles that no row sees are left out. The epilogue applies the head's output gate, if there is one.
 #include "../kernels/common.h"
 
 namespace nls_pfa {
@@ -50,7 +50,6 @@ struct FP {
   int window, keep, sink; // position i sees j <= i if i - j < window or j < keep; sink: one more in the denominator
 };
 constexpr int NO_WINDOW = 1 << 30;
-
 
 template <int NKU, int NKR, int NDB, int NWV>      // 32-column units: keys unrotated / rotated, values; waves
 __global__ __launch_bounds__(64 * NWV) void flash_prefill_kernel(FP p) {
@@ -309,11 +308,13 @@ int nls_latent_prefill(const void* qn, long ldqn, int qns, const void* qr, long 
   return -1;
 }
 
-// window > 0: sliding window with `keep` first keys. Dp: padded head width (32, 64, 128; 256 with 4 waves); k, v: paged [slots][G][Dp]; blocks of up to 32 * waves tokens
+// Dp: padded head width (32, 64, 128; 256 with 4 waves); k, v: paged [slots][G][Dp]; blocks of up to 32 * waves tokens. window > 0: a
+// sliding window with `keep` first keys
 int nls_gqa_prefill(const void* q, long ldq, const void* k, const void* v, const int* xmap, const int* blocks, int nblocks,
                     const float* gate, int ldg, void* out, long ldo, int H, int G, int Dp, int waves, float scale,
                     int window, int keep, int sink, void* stream) {
-  if (nblocks < 1 || G < 1 || H < 1 || H % G || window < 0 || window > NO_WINDOW || keep < 0 || (ldq & 7) || (ldo & 3)) return -1;
+  if (nblocks < 1 || G < 1 || H < 1 || H % G || window < 0 || window > NO_WINDOW || keep < 0 || (ldq & 7) || (ldo & 3))
+    return -1;
   FP p{(const __bf16*)q, (const __bf16*)q, (const __bf16*)k, (const __bf16*)v, nullptr, xmap, blocks, gate, (__bf16*)out, ldq, ldq,
        (long)G * Dp, ldo, Dp, Dp, H, Dp, ldg, H / G, H / G, scale, window ? window : NO_WINDOW, keep, sink};
   hipStream_t st = (hipStream_t)stream;

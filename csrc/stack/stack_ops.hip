@@ -698,7 +698,8 @@ int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq
 int nls_attn_rows(const float* q, const float* k, const float* v, long ldq, const float* qn, const float* kn, const float* cs,
                   const int* pos, const int* slot, void* qo, long ldqo, void* kc, void* vc, long ldc, int T, int H, int G,
                   int D, int V, int Dp, int rot, float eps, int f32, void* stream) {
-  if (T < 1 || H < 1 || G < 1 || D < 1 || V < 1 || Dp < D || Dp < V || (v == k && V != D) || (rot && !cs) || (rot & 1) || rot < 0 || rot > D || (long)H * Dp > ldqo || (long)G * Dp > ldc)
+  if (T < 1 || H < 1 || G < 1 || D < 1 || V < 1 || Dp < D || Dp < V || (v == k && V != D) || (rot && !cs) || (rot & 1) || rot < 0 ||
+      rot > D || (long)H * Dp > ldqo || (long)G * Dp > ldc)
     return -1;
   AttnRows p{q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, ldq, ldqo, ldc, H, G, D, Dp, rot, V, eps};
   return f32 ? attn_rows_t<float>(p, T, (hipStream_t)stream) : attn_rows_t<__bf16>(p, T, (hipStream_t)stream);

@@ -2,6 +2,8 @@
 GGUF families' closest model with the same width, layers and weights per layer, F16:
   sekolorn   Mixtral (attention + routed experts), the same experts
   kolodra    Llama (grouped-query attention + gated feed-forward), the feed-forward wider by the weights of the second mixer
+  bibapel    Llama, four layers beside four layer runs (the attention layer runs twice), the feed-forward wider by the weights that
+             the linear mixers and the passes' entries read
 
 Both run the engine's own loop: submit, chunked prefill, captured decode steps. Random weights; one JSON line per case."""
 from __future__ import annotations
@@ -29,8 +31,15 @@ SIZES = {
         "2k": dict(width=2048, left=(16, 4, 128), right=(16, 64, 128), ff=5632, closest=dict(n_head=16, n_kv_head=4, d_ff=8192)),
         "4k": dict(width=4096, left=(32, 8, 128), right=(32, 64, 128), ff=9216, closest=dict(n_head=32, n_kv_head=8, d_ff=14336)),
     },
+    # delta: heads, query and key heads, key and value width, rank of its gates; lightning: heads, key and value width
+    "bibapel": {
+        "2k": dict(width=2048, attention=(16, 4, 128), delta=(16, 8, 128, 128, 128), lightning=(16, 128, 128), ff=5632,
+                   closest=dict(n_head=16, n_kv_head=4, d_ff=6912)),
+        "4k": dict(width=4096, attention=(32, 8, 128), delta=(32, 16, 128, 128, 128), lightning=(32, 128, 128), ff=9216,
+                   closest=dict(n_head=32, n_kv_head=8, d_ff=11520)),
+    },
 }
-CLOSEST = {"sekolorn": "mixtral-8x7b", "kolodra": "llama-3-8b"}
+CLOSEST = {"sekolorn": "mixtral-8x7b", "kolodra": "llama-3-8b", "bibapel": "llama-3-8b"}
 DESIGNS = tuple(SIZES)
 
 
@@ -58,7 +67,21 @@ def kolodra_config(sz: dict) -> dict:
             "embedding": {"scale": 1.0}, "logit_softcap": 30.0}
 
 
-CONFIGS = {"sekolorn": sekolorn_config, "kolodra": kolodra_config}
+def bibapel_config(sz: dict) -> dict:
+    H, G, D = sz["attention"]
+    DH, DG, DD, DV, _ = sz["delta"]
+    LH, LD, LV = sz["lightning"]
+    mixers = [("channel_delta", {"heads": DH, "kv_heads": DG, "dim": DD, "vdim": DV, "conv": 4}),
+              ("attention", {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5,
+                             "mask": {"size": 1024, "keep_first": 16}}),
+              ("lightning", {"heads": LH, "dim": LD, "vdim": LV, "decay": [1.0 - 2.0 ** (-1 - 8 * h / LH) for h in range(LH)]})]
+    layers = [{"type": t, "mixer": m, "mlp": {"kind": "dense", "ff": sz["ff"], "limit": 7.0}} for t, m in mixers]
+    return {"architecture": "Bibapel", "width": sz["width"], "vocab": VOCAB, "norm": {"eps": 1e-5}, "layers": layers,
+            "embedding": {"scale": 1.0, "bigram": {"buckets": 8191, "mul_prev": 127, "mul_cur": 3}}, "max_positions": 8192,
+            "loop": {"start": 1, "stop": 2, "times": 2}, "rank": sz["delta"][4]}
+
+
+CONFIGS = {"sekolorn": sekolorn_config, "kolodra": kolodra_config, "bibapel": bibapel_config}
 
 
 def _sekolorn_layer(p: str, L: dict, d: int, lin, full):
@@ -121,6 +144,37 @@ def _kolodra_layer(p: str, L: dict, d: int, lin, full):
     lin(p + "mlp.down", d, ff)
 
 
+def _bibapel_layer(p: str, L: dict, d: int, lin, full, rank: int):
+    m, ff = L["mixer"], L["mlp"]["ff"]
+    H, D, V = m["heads"], m["dim"], m["vdim"]
+    full(p + "norm1", 1.0, d)
+    full(p + "norm2", 1.0, d)
+    q = p + "mix."
+    if L["type"] == "channel_delta":
+        for n, rows in (("q", m["kv_heads"] * D), ("k", m["kv_heads"] * D), ("v", H * V)):
+            lin(q + n, rows, d)
+            lin(q + n + ".conv", rows, m["conv"])
+        lin(q + "b", H, d)
+        full(q + "A_log", 0.0, H)
+        lin(q + "a1", rank, d)
+        lin(q + "a2", H * D, rank)
+        full(q + "dt_bias", -3.0, H * D)
+        full(q + "norm", 1.0, V)
+        lin(q + "g1", rank, d)
+        lin(q + "g2", H * V, rank)
+    elif L["type"] == "attention":
+        for n, rows in (("q", H * D), ("k", m["kv_heads"] * D), ("v", m["kv_heads"] * V)):
+            lin(q + n, rows, d)
+    else:
+        for n, rows in (("q", H * D), ("k", H * D), ("v", H * V), ("g", H * V)):
+            lin(q + n, rows, d)
+        full(q + "norm", 1.0, H * V)
+    lin(q + "o", d, H * V)
+    lin(p + "mlp.gate", ff, d)
+    lin(p + "mlp.up", ff, d)
+    lin(p + "mlp.down", d, ff)
+
+
 def write_stack(path: str, cfg: dict):
     """A checkpoint folder of `cfg` with random weights."""
     import torch
@@ -137,11 +191,19 @@ def write_stack(path: str, cfg: dict):
     def full(name, v, *shape):
         W[name] = torch.full(shape, v, dtype=torch.bfloat16)
     W["embed"] = torch.randn(cfg["vocab"], d, generator=g, device=dev).to(torch.bfloat16).cpu()
-    layer = {"Sekolorn": _sekolorn_layer, "Kolodra": _kolodra_layer}[cfg["architecture"]]
+    layer = {"Sekolorn": _sekolorn_layer, "Kolodra": _kolodra_layer, "Bibapel": _bibapel_layer}[cfg["architecture"]]
+    cfg = dict(cfg)
+    rank = cfg.pop("rank", None)                    # (of the delta rule's gates: a tensor shape, no part of the config)
     for i, L in enumerate(cfg["layers"]):
-        layer(f"l{i}.", L, d, lin, full)
-    full("final.norm", 1.0 if cfg["architecture"] == "Sekolorn" else 0.0, d)
-    lin("head", cfg["vocab"], d)
+        layer(f"l{i}.", L, d, lin, full, *([] if rank is None else [rank]))
+    full("final.norm", 0.0 if cfg["architecture"] == "Kolodra" else 1.0, d)
+    if cfg["architecture"] == "Bibapel":
+        lin("bigram", cfg["embedding"]["bigram"]["buckets"] + 1, d)
+        lin("pos", cfg["max_positions"], d)
+        lin("loop.in", d, 2 * d)
+        lin("loop.step", cfg["loop"]["times"], d)
+    else:
+        lin("head", cfg["vocab"], d)
     with open(os.path.join(path, "config.json"), "w") as fh:
         json.dump(cfg, fh)
     write_safetensors(os.path.join(path, "model.safetensors"), W)

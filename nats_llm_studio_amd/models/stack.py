@@ -3,9 +3,8 @@
 A mixer or feed-forward is a class that loads its weights, adds its step buffers, and runs on the rows of a step; a layer
 class (OutputNormLayer, SharedNormLayer) places the norms and joins the sublayers. A looped model runs some layers several
 times with the same weights. The per-token cache rows (paged) and the per-sequence states (slots) of all layer runs belong to
-the engine, which sees them as `kv_cache` / `state_pool`. Everything
-runs on the HIP kernels of csrc/stack (ops/stack.py): bf16 operands with an f32 residual, or `dtype=torch.float32` for 32-bit
-throughout.
+the engine, which sees them as `kv_cache` / `state_pool`. Everything runs on the HIP kernels of csrc/stack (ops/stack.py): bf16
+operands with an f32 residual, or `dtype=torch.float32` for 32-bit throughout.
 
 Rows of a step are runs of consecutive tokens of one sequence (whole prompts, portions of any size, single decoded
 tokens), all in one batch:
@@ -698,14 +697,15 @@ class SharedNormLayer:
         b.launches[key, "out"] = K.LinLaunch([K.Seg(self.o, cat, self.m.slabs(b), slabs=_SLABS, slab_rows=b.slab_rows)])
 
     def new_caches(self, slots):
-        return {j: q.new_cache(slots) for j, q in enumerate(self.parts) if q.cache_width}
+        return {j: q.new_cache(slots) for j, q in enumerate(self.parts) if q.cache_width} or None
 
     def run(self, b, key, kc, state, step: "_Step", fin: dict):
         cfg = self.m.cfg
         for launch in b.launches[key, "in"]:
             launch.run(step.T, step.st)
+        caches = kc.get(step.layer, {})
         for j, (q, e) in enumerate(zip(self.parts, b.launches[key, "parts"])):
-            q.run(b, e, kc[step.layer].get(j), state, step)
+            q.run(b, e, caches.get(j), state, step)
         n = b.launches[key, "out"].run(step.T, step.st)
         K.norm_add(self.m.slabs(b), None, b.x, fin.pop("copy", None), step.T, cfg.eps, step.st, rms=cfg.design.norm == "rms",
                    slabs=n, slab_rows=b.slab_rows, **fin)
@@ -851,12 +851,12 @@ class StackModel:
         return {i: c for i, c in ((i, L.new_caches(slots)) for i, L in enumerate(self.layers)) if c is not None}, None
 
     def state_pool(self, slots: int):
-        """Per-sequence states, f32: {layer run: {name: [slots, n]}} (and the previous token of each slot). A sequence's first run (position 0) ignores what its
-        slot holds, so a reused slot needs no clearing."""
+        """Per-sequence states, f32: {layer run: {name: [slots, n]}} (and "token": the previous token of each slot). A sequence's
+        first run (position 0) ignores what its slot holds, so a reused slot needs no clearing."""
         out = {i: {k: torch.zeros(slots, n, dtype=torch.float32, device=self.device)
                    for q in L.parts for k, n in q.state_shapes().items()} for i, L in enumerate(self.layers)}
         if self.pairs is not None:
-            out["token"] = torch.zeros(slots, dtype=torch.int32, device=self.device)       # the previous one
+            out["token"] = torch.zeros(slots, dtype=torch.int32, device=self.device)
         return {i: d for i, d in out.items() if len(d)}
 
     def step_buffers(self, cap: int, max_seqs: int, max_blocks: int, logit_rows: Optional[int] = None) -> StackBuffers:
@@ -883,8 +883,8 @@ class StackModel:
             logits=torch.zeros(nl, cfg.vocab, **f), next_ids=torch.zeros(pad, dtype=torch.int32, device=dev))
         b.slot.fill_(-1)
         b.runs[:, 2] = -1
-        for o in sorted(set(self.owners)):
-            self.layers[o].bind(b, o)
+        for o, layer in dict(zip(self.owners, self.layers)).items():
+            layer.bind(b, o)
         if b.xx is not None:
             b.launches["pass"] = K.LinLaunch([K.Seg(self.loop_in, b.xx, self.slabs(b), slabs=_SLABS, slab_rows=b.slab_rows)])
         cap_epi = dict(epi="softcap", alpha=cfg.softcap) if cfg.softcap else {}

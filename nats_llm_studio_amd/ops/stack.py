@@ -137,8 +137,9 @@ class Seg:
     xgs / ygs: column step per group. block = (cb, cstep): output column n -> (n / cb) * cstep + n % cb.
     routed = (entry list, xdiv): the rows are routed entries (x row = entry / xdiv, y row = entry).
     rope = (table, pos, pairs). alpha: constant of the epilogue (sigmoid, sigpow, softcap, swiglu); sigpow: `gate`,
-    a vector, gives an exponent per column instead. geglu, swiglu: the rows of w alternate gate and up, y has half as many columns. slabs: K splits that launches of up to slab_rows rows may use; y holds that many
-    slabs of slab_rows rows, added by the caller (LinLaunch.run returns how many were written)."""
+    a vector, gives an exponent per column instead. geglu, swiglu: the rows of w alternate gate and up, y has half as many
+    columns. slabs: K splits that launches of up to slab_rows rows may use; y holds that many slabs of slab_rows rows, added by
+    the caller (LinLaunch.run returns how many were written)."""
 
     def __init__(self, w: PackedLinear, x: torch.Tensor, y: torch.Tensor, epi: str = "none", ycol: int = 0,
                  xcol: int = 0, xgs: int = 0, ygs: int = 0, block=None, bias=None, gate=None, routed=None, rope=None,

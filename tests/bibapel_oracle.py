@@ -49,7 +49,8 @@ def embed(cfg, W, tokens, prev=None, first=0):
     e = cfg["embedding"]
     for i, t in enumerate(tokens):
         x = W["embed"][t] * e["scale"]
-        x = x + W["bigram"][bigram_row(prev, t, e["bigram"])]
+        if e.get("bigram"):
+            x = x + W["bigram"][bigram_row(prev, t, e["bigram"])]
         out.append(x + W["pos"][first + i])
         prev = t
     return torch.stack(out)
@@ -58,7 +59,10 @@ def embed(cfg, W, tokens, prev=None, first=0):
 # ---- attention
 
 def visible(i, j, mask):
-    return j <= i and (i - j < mask["size"] or j < mask["keep_first"])
+    """Whether position i sees position j (tensors of positions)."""
+    if not mask:
+        return j <= i
+    return (j <= i) & ((i - j < mask["size"]) | (j < mask["keep_first"]))
 
 
 def attend(q, k, v, positions, scale, mask):
@@ -66,14 +70,18 @@ def attend(q, k, v, positions, scale, mask):
     denominator."""
     H, G = q.shape[1], k.shape[1]
     out = torch.zeros(q.shape[0], H, v.shape[2], dtype=q.dtype)
-    see = torch.tensor([[visible(int(i), j, mask) for j in range(k.shape[0])] for i in positions])
+    see = visible(positions[:, None], torch.arange(k.shape[0])[None, :], mask)
     for h in range(H):
         g = h // (H // G)
         s = (q[:, h] @ k[:, g].T * scale).masked_fill(~see, -math.inf)
         m = torch.clamp(s.max(-1, keepdim=True).values, min=0.0)
-        e = torch.exp(s - m)
-        out[:, h] = (e / (torch.exp(-m) + e.sum(-1, keepdim=True))) @ v[:, g]
+        out[:, h] = sink_weights(torch.exp(s - m), torch.exp(-m)) @ v[:, g]
     return out
+
+
+def sink_weights(e, one):
+    """Softmax weights with one more in the denominator; both scaled by the same factor."""
+    return e / (one + e.sum(-1, keepdim=True))
 
 
 def attention_mixer(h, W, p, m, positions, eps, before=None):
@@ -84,7 +92,7 @@ def attention_mixer(h, W, p, m, positions, eps, before=None):
     v = (h @ W[p + "v"].T).reshape(-1, G, m["vdim"])
     if before is not None:
         k, v = torch.cat([before[0], k]), torch.cat([before[1], v])
-    o = attend(q, k, v, positions, m["scale"], m["mask"])
+    o = attend(q, k, v, positions, m["scale"], m.get("mask"))
     return o.reshape(h.shape[0], -1) @ W[p + "o"].T, (k, v)
 
 
