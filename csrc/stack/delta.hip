@@ -23,8 +23,10 @@ struct CV {
   int T, H, G, D, V, taps;
 };
 
-template <typename T, int TAPS, int TG>      // TAPS 0: any number, re-reading the inputs
+template <typename T, int TAPS, int TG, int VC>      // TAPS 0: any number, re-reading the inputs; VC: channels per lane
 __global__ __launch_bounds__(256) void conv_kernel(CV p) {
+  typedef T tv __attribute__((ext_vector_type(VC)));
+  typedef float fv __attribute__((ext_vector_type(VC)));
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int unit = blockIdx.y * 4 + wave, nqk = 2 * p.G;
   if (unit >= nqk + p.H) return;
@@ -34,13 +36,46 @@ __global__ __launch_bounds__(256) void conv_kernel(CV p) {
   float ss[TG];
 #pragma unroll
   for (int e = 0; e < TG; ++e) ss[e] = 0.f;
-  for (int c = lane; c < W; c += 64) {
+  for (int c = lane * VC; c < W; c += 64 * VC) {
     const int ch = ch0 + c;
     const T* zc = (const T*)p.z + ch;
-    float w[TAPS ? TAPS : 1], h[TAPS ? TAPS : 1];
+    auto row = [&](int u) { return __builtin_convertvector(*reinterpret_cast<const tv*>(zc + (size_t)u * p.ldz), fv); };
+    auto weight = [&](int j) {
+      fv v;
+#pragma unroll
+      for (int i = 0; i < VC; ++i) v[i] = p.w[(size_t)(ch + i) * taps + j];
+      return v;
+    };
+    fv w[TAPS ? TAPS : 1], h[TAPS ? TAPS : 1];
     if constexpr (TAPS > 0) {
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) w[j] = p.w[(size_t)ch * TAPS + j];
+      for (int j = 0; j < TAPS; ++j) w[j] = weight(j);
+    }
+    auto emit = [&](int e, const fv& acc) {
+      tv y;
+#pragma unroll
+      for (int i = 0; i < VC; ++i) {
+        y[i] = (T)(acc[i] * nls_lin::lin_sigmoid(acc[i]));
+        ss[e] = fmaf((float)y[i], (float)y[i], ss[e]);
+      }
+      *reinterpret_cast<tv*>((T*)p.y + (size_t)(r0 + e) * p.ldy + ch) = y;
+    };
+    if constexpr (TAPS > 0 && TG > 1) {      // rows inside a run, their inputs too: all loads in flight together
+      const int rn = p.tok_seq[r0];
+      const int* run = p.runs + 4 * rn;
+      if (r0 - (TAPS - 1) >= run[0] && r0 + TG <= run[0] + run[1] && run[2] >= 0) {
+        fv x[TG + TAPS - 1];
+#pragma unroll
+        for (int e = 0; e < TG + TAPS - 1; ++e) x[e] = row(r0 - (TAPS - 1) + e);
+#pragma unroll
+        for (int e = 0; e < TG; ++e) {
+          fv acc = w[TAPS - 1] * x[e + TAPS - 1];
+#pragma unroll
+          for (int j = 0; j + 1 < TAPS; ++j) acc += w[j] * x[e + j];
+          emit(e, acc);
+        }
+        continue;
+      }
     }
     int seen = -1;                           // run that h belongs to: its inputs at t - (taps - 1) .. t - 1
 #pragma unroll
@@ -52,13 +87,12 @@ __global__ __launch_bounds__(256) void conv_kernel(CV p) {
       const int t0 = run[0], n = run[1], slot = run[2], pos0 = run[3];
       if (slot < 0 || t < t0 || t >= t0 + n) continue;
       float* st = p.state + (size_t)slot * p.sstride + ch;
+      auto kept = [&](int j) -> fv& { return *reinterpret_cast<fv*>(st + (size_t)j * nch); };
       auto input = [&](int u) {              // input of row u of this run, or of the tokens ahead of it
-        if (u >= t0) return (float)zc[(size_t)u * p.ldz];
-        const int j = u - t0 + taps - 1;
-        return pos0 > 0 ? st[(size_t)j * nch] : 0.f;
+        return u >= t0 ? row(u) : pos0 > 0 ? kept(u - t0 + taps - 1) : (fv)(0.f);
       };
-      const float x = (float)zc[(size_t)t * p.ldz];
-      float acc;
+      const fv x = row(t);
+      fv acc;
       if constexpr (TAPS > 0) {
         if (rn != seen) {
 #pragma unroll
@@ -67,22 +101,20 @@ __global__ __launch_bounds__(256) void conv_kernel(CV p) {
         }
         acc = w[TAPS - 1] * x;
 #pragma unroll
-        for (int j = 0; j + 1 < TAPS; ++j) acc = fmaf(w[j], h[j], acc);
+        for (int j = 0; j + 1 < TAPS; ++j) acc += w[j] * h[j];
 #pragma unroll
         for (int j = 0; j + 2 < TAPS; ++j) h[j] = h[j + 1];
         if (TAPS > 1) h[TAPS > 1 ? TAPS - 2 : 0] = x;
         if (n == 1)
 #pragma unroll
-          for (int j = 0; j + 1 < TAPS; ++j) st[(size_t)j * nch] = h[j];
+          for (int j = 0; j + 1 < TAPS; ++j) kept(j) = h[j];
       } else {
-        acc = p.w[(size_t)ch * taps + taps - 1] * x;
-        for (int j = 0; j + 1 < taps; ++j) acc = fmaf(p.w[(size_t)ch * taps + j], input(t - (taps - 1) + j), acc);
+        acc = weight(taps - 1) * x;
+        for (int j = 0; j + 1 < taps; ++j) acc += weight(j) * input(t - (taps - 1) + j);
         if (n == 1)
-          for (int j = 0; j + 1 < taps; ++j) st[(size_t)j * nch] = j + 2 < taps ? (pos0 > 0 ? st[(size_t)(j + 1) * nch] : 0.f) : x;
+          for (int j = 0; j + 1 < taps; ++j) kept(j) = j + 2 < taps ? (pos0 > 0 ? kept(j + 1) : (fv)(0.f)) : x;
       }
-      const T y = (T)(acc * nls_lin::lin_sigmoid(acc));
-      ((T*)p.y)[(size_t)t * p.ldy + ch] = y;
-      ss[e] = fmaf((float)y, (float)y, ss[e]);
+      emit(e, acc);
     }
   }
   if (!qk) return;
@@ -110,12 +142,19 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(CV p) {
   }
 }
 
+template <typename T, int TAPS, int VC>
+int conv_v(const CV& p, hipStream_t st) {
+  const int units = 2 * p.G + p.H;
+  if (p.T <= 512) hipLaunchKernelGGL((conv_kernel<T, TAPS, 1, VC>), dim3(p.T, (units + 3) / 4), dim3(256), 0, st, p);
+  else hipLaunchKernelGGL((conv_kernel<T, TAPS, 8, VC>), dim3((p.T + 7) / 8, (units + 3) / 4), dim3(256), 0, st, p);
+  return (int)hipGetLastError();
+}
+
 template <typename T, int TAPS>
 int conv_t(const CV& p, hipStream_t st) {
-  const int units = 2 * p.G + p.H;
-  if (p.T <= 512) hipLaunchKernelGGL((conv_kernel<T, TAPS, 1>), dim3(p.T, (units + 3) / 4), dim3(256), 0, st, p);
-  else hipLaunchKernelGGL((conv_kernel<T, TAPS, 8>), dim3((p.T + 7) / 8, (units + 3) / 4), dim3(256), 0, st, p);
-  return (int)hipGetLastError();
+  const bool pair = !((p.D | p.V | p.ldz | p.ldy | p.sstride) & 1) && !((uintptr_t)p.state & 7) &&
+                    !(((uintptr_t)p.z | (uintptr_t)p.y) % (2 * sizeof(T)));
+  return pair ? conv_v<T, TAPS, 2>(p, st) : conv_v<T, TAPS, 1>(p, st);
 }
 
 template <typename T>
@@ -350,7 +389,8 @@ __global__ __launch_bounds__(256) void delta_step_kernel(DS p) {
     const int e = tid + 256 * x;
     if (e < V) {
       const float gt = p.gate ? (float)((const T*)p.gate)[(size_t)t * p.ldg + hv + e]
-                              : nls_lin::lin_sigmoid(low_dot((const T*)p.lowg + (size_t)t * p.ldz, (const T*)p.g2 + (hv + e) * p.rg, p.rg));
+                              : nls_lin::lin_sigmoid(low_dot((const T*)p.lowg + (size_t)t * p.ldz,
+                                                             (const T*)p.g2 + (hv + e) * p.rg, p.rg));
       ((T*)p.out)[(size_t)t * p.ldout + hv + e] = (T)(o[x] * inv * p.norm[hv + e] * gt);
     }
   }

@@ -43,46 +43,39 @@ struct Embed {
   const __bf16* ptab;      // optional [npos][D]
   const int* pos;
   long ldx, ldc;
-  int V, D, buckets, mul_prev, mul_cur, npos, f32;
+  int V, D, buckets, mul_prev, mul_cur, npos, f32, vec;
   float scale;
 };
 
 DEVI int token_of(const Embed& p, int t) {
-  return min(max(p.use_prev && p.use_prev[t] ? p.next_ids[t] : p.ids[t], 0), p.V - 1);
+  const int a = p.ids[t], n = p.use_prev ? p.next_ids[t] : 0, u = p.use_prev ? p.use_prev[t] : 0;       // (in flight together)
+  return min(max(u ? n : a, 0), p.V - 1);
 }
 
 template <int N>
 DEVI void embed_cols(const Embed& p, int t, const __bf16* row, const __bf16* pair, const __bf16* pv) {
   typedef __bf16 bfn __attribute__((ext_vector_type(N)));
+  typedef float fn __attribute__((ext_vector_type(N)));
   for (int i = threadIdx.x * N; i < p.D; i += 256 * N) {
-    float v[N];
-    const bfn a = *reinterpret_cast<const bfn*>(row + i);
-#pragma unroll
-    for (int e = 0; e < N; ++e) v[e] = (float)a[e] * p.scale;
-    if (pair) {
-      const bfn b = *reinterpret_cast<const bfn*>(pair + i);
-#pragma unroll
-      for (int e = 0; e < N; ++e) v[e] += (float)b[e];
-    }
-    if (pv) {
-      const bfn b = *reinterpret_cast<const bfn*>(pv + i);
-#pragma unroll
-      for (int e = 0; e < N; ++e) v[e] += (float)b[e];
-    }
+    const bfn none = (bfn)((__bf16)0.f);
+    const bfn a = *reinterpret_cast<const bfn*>(row + i), b = pair ? *reinterpret_cast<const bfn*>(pair + i) : none;
+    const bfn c = pv ? *reinterpret_cast<const bfn*>(pv + i) : none;
+    fn y;
+    bfn yb;
 #pragma unroll
     for (int e = 0; e < N; ++e) {
-      const float y = v[e];
-      p.x[(size_t)t * p.ldx + i + e] = y;
-      if (p.xb) p.xb[(size_t)t * p.ldx + i + e] = (__bf16)y;
-      const size_t o = (size_t)t * p.ldc + i + e;
-      if (p.c0) {
-        if (p.f32) reinterpret_cast<float*>(p.c0)[o] = y;
-        else reinterpret_cast<__bf16*>(p.c0)[o] = (__bf16)y;
-      }
-      if (p.c1) {
-        if (p.f32) reinterpret_cast<float*>(p.c1)[o] = y;
-        else reinterpret_cast<__bf16*>(p.c1)[o] = (__bf16)y;
-      }
+      y[e] = (float)a[e] * p.scale + (float)b[e] + (float)c[e];
+      yb[e] = (__bf16)y[e];
+    }
+    *reinterpret_cast<fn*>(p.x + (size_t)t * p.ldx + i) = y;
+    if (p.xb) *reinterpret_cast<bfn*>(p.xb + (size_t)t * p.ldx + i) = yb;
+    const size_t o = (size_t)t * p.ldc + i;
+#pragma unroll
+    for (int k = 0; k < 2; ++k) {
+      void* d = k ? p.c1 : p.c0;
+      if (!d) continue;
+      if (p.f32) *reinterpret_cast<fn*>(reinterpret_cast<float*>(d) + o) = y;
+      else *reinterpret_cast<bfn*>(reinterpret_cast<__bf16*>(d) + o) = yb;
     }
   }
 }
@@ -113,7 +106,7 @@ __global__ __launch_bounds__(256) void embed_kernel(Embed p) {
     if (keep >= 0) p.prev[slot] = keep;
   }
   const __bf16* row = p.tab + (size_t)id * p.D;
-  if ((p.D & 7) == 0) embed_cols<8>(p, t, row, pair, pv);
+  if (p.vec) embed_cols<8>(p, t, row, pair, pv);
   else embed_cols<1>(p, t, row, pair, pv);
 }
 
@@ -659,8 +652,11 @@ int nls_stack_embed(int* ids, const int* next_ids, const int* use_prev, const vo
                     int mul_prev, int mul_cur, int* prev, const int* runs, const int* tok_seq, const void* ptab, int npos,
                     const int* pos, void* stream) {
   if (T < 1 || D < 1 || V < 1 || (pairs && (buckets < 1 || !prev || !runs || !tok_seq)) || (ptab && (npos < 1 || !pos))) return -1;
+  const uintptr_t at = (uintptr_t)tab | (uintptr_t)x | (uintptr_t)xb | (uintptr_t)c0 | (uintptr_t)c1 | (uintptr_t)pairs |
+                       (uintptr_t)ptab;
+  const int vec = !((D | ldx | ldc) & 7) && !(at & 31);
   const Embed p{ids, next_ids, use_prev, (const __bf16*)tab, x, (__bf16*)xb, c0, c1, (const __bf16*)pairs, prev, runs, tok_seq,
-                (const __bf16*)ptab, pos, ldx, ldc, V, D, buckets, mul_prev, mul_cur, npos, f32, scale};
+                (const __bf16*)ptab, pos, ldx, ldc, V, D, buckets, mul_prev, mul_cur, npos, f32, vec, scale};
   hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
   return (int)hipGetLastError();
 }

@@ -36,7 +36,7 @@ SIZES = {
         "2k": dict(width=2048, attention=(16, 4, 128), delta=(16, 8, 128, 128, 128), lightning=(16, 128, 128), ff=5632,
                    closest=dict(n_head=16, n_kv_head=4, d_ff=6912)),
         "4k": dict(width=4096, attention=(32, 8, 128), delta=(32, 16, 128, 128, 128), lightning=(32, 128, 128), ff=9216,
-                   closest=dict(n_head=32, n_kv_head=8, d_ff=11520)),
+                   closest=dict(n_head=32, n_kv_head=8, d_ff=12288)),
     },
 }
 CLOSEST = {"sekolorn": "mixtral-8x7b", "kolodra": "llama-3-8b", "bibapel": "llama-3-8b"}

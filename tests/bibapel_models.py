@@ -34,7 +34,8 @@ def config(layers, width=136, vocab=203, eps=3e-5, scale=0.7, loop=None, buckets
 
 
 # name -> config: uneven sizes with a loop in the middle, one-of-everything sizes in one pass, sizes past the kernels' tiles with a
-# loop that ends the model, head widths without an MFMA kernel and odd sizes without a loop, no window, no recurrent mixer
+# loop that ends the model, head widths without an MFMA kernel and odd sizes without a loop, no window and no recurrent mixer,
+# products long enough to be split
 CONFIGS = {
     "uneven": config([layer(lightning(), 0), layer(delta()), layer(attention()), layer(lightning((0.8, 0.99), 33, 28), 50, 1.4),
                       layer(attention(3, 3, 34, 20, 0.25, 16, 0), 0), layer(delta(3, 3, 33, 16, 2), 40)], loop=(1, 4, 3)),
@@ -49,6 +50,8 @@ CONFIGS = {
                    layer(attention(5, 5, 33, 47, 0.2, 50, 17), 34), layer(lightning((0.2, 0.96), 7, 13), 6)], width=90, vocab=101),
     "attention only": config([layer(attention(4, 2, 24, 24, 0.3, 0)), layer(attention(4, 4, 16, 32, 0.4, 7, 40), 30)], width=64,
                              loop=(1, 2, 2)),
+    "split": config([layer(attention(2, 1, 32, 32, 0.2, 40, 4), 40), layer(lightning((0.9, 0.97), 16, 24), 2090, 2.0)], width=1030,
+                    vocab=101, loop=(0, 2, 2)),
 }
 
 
