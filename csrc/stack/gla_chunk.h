@@ -1,5 +1,5 @@
 // Linear recurrences with a decay per key channel over runs of tokens (gfx950), in chunks on f32 MFMA: gated linear attention
-// (gla.hip) and the delta rule (delta.hip). Keys and values may differ in width. First the form without the delta rule:
+// (gla.hip) and the delta rule (delta_chunk.h). Keys and values may differ in width. First the form without the delta rule:
 //
 // Per head, state S [D][V] in f32: S_t = diag(a_t) S_(t-1) + k_t v_t^T, o_t = rs S_t^T q_t. With the decays' products inside a
 // chunk of 16 tokens, P(j, i) = prod of a_t over j < t <= i (per key channel, P from the chunk's start with j = -1):
@@ -23,7 +23,7 @@
 // from 16 steps of substitution (a lane per column), and u takes the place of v above. The products' accumulators are again the
 // next product's operand. Queries and keys come with a 32-bit factor per token and head. A segment's effect on the state it
 // starts from is not diagonal: the first pass also runs the columns of the identity (without values), which end as the matrix M
-// of S_end = M S_start + S_local, and the chain multiplies by it (delta.hip).
+// of S_end = M S_start + S_local, and the chain multiplies by it (delta_chunk.h).
 #pragma once
 #include "scan.h"
 
