@@ -477,7 +477,7 @@ class LlamaModel:
         if n_split > 1 and b.attn_ws.numel() < need:
             # a larger explicit split than the policy's: grow, but keep the old buffer alive -- a graph
             # captured earlier still writes its partials there (freeing it let a later allocation, e.g.
-            # prefill metadata, land under a replaying graph: the 256 x 1K-context fault of this round)
+            # prefill metadata, land under a replaying graph: the 256 x 1K-context fault)
             _RETIRED.append(b.attn_ws)
             b.attn_ws = torch.zeros(need, dtype=torch.float32, device=self.device)
         fused = self.shard.size == 1            # row-parallel GEMM + residual + next RMSNorm in one pass
