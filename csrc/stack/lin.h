@@ -32,6 +32,7 @@ enum LinEpi : int {
   LE_SIGPOW = 9,    // sigmoid(v + bias[n]) ^ alpha, or (gate given) ^ gate[n]
   LE_SOFTCAP = 10,  // alpha * tanh(v / alpha)
   LE_SWIGLU = 11,   // g = min(v[n], alpha), u = v[n + 1] clamped to +- alpha: g sigmoid(1.702 g) (u + 1) -> column n / 2
+  LE_SILUGLU = 12,  // silu(v[n]) * v[n + 1] -> column n / 2
 };                  // LE_SIGMOID: alpha * sigmoid(v)
 
 struct LinSeg {
@@ -153,6 +154,10 @@ DEVI float lin_swiglu(float g, float u, float lim) {
   return g * lin_sigmoid(1.702f * g) * (fminf(fmaxf(u, -lim), lim) + 1.f);
 }
 
+DEVI float lin_glu(const LinSeg& S, float g, float u) {
+  return S.epi == LE_SWIGLU ? lin_swiglu(g, u, S.alpha) : (S.epi == LE_SILUGLU ? g * lin_sigmoid(g) : lin_gelu(g)) * u;
+}
+
 // sigmoid(z)^a = 2^(-a (max(-z, 0) log2(e) + log2(1 + u))), u = e^-|z|; log2(w) u / (w - 1) with w = fl(1 + u) keeps the
 // digits of a small u
 DEVI float lin_sigpow(float z, float a) {
@@ -201,11 +206,10 @@ DEVI void lin_store4(const LinSeg& S, int grp, int ks, int n, int yr, f32x4 v) {
       for (int e = 0; e < 4; ++e) v[e] = S.alpha * tanhf(v[e] / S.alpha);
       break;
     case LE_GEGLU:
-    case LE_SWIGLU: {                   // N is even: both pairs or the first one lie inside
+    case LE_SWIGLU:
+    case LE_SILUGLU: {                  // N is even: both pairs or the first one lie inside
       const size_t o = (size_t)yr * S.ldy + (size_t)grp * S.ygs + (n >> 1);
-      const bool sw = S.epi == LE_SWIGLU;
-      const float a = sw ? lin_swiglu(v[0], v[1], S.alpha) : lin_gelu(v[0]) * v[1];
-      const float b = sw ? lin_swiglu(v[2], v[3], S.alpha) : lin_gelu(v[2]) * v[3];
+      const float a = lin_glu(S, v[0], v[1]), b = lin_glu(S, v[2], v[3]);
       if (S.yact && sizeof(T) == 2) {
         __bf16* y = reinterpret_cast<__bf16*>(S.y) + o;
         typedef __bf16 bf2 __attribute__((ext_vector_type(2)));
@@ -274,7 +278,7 @@ inline int lin_count(LinArgs& a, int BN, int BM) {
     if (!S.w || !S.x || !S.y) return -1;
     if (S.epi == LE_ROPE && (!S.cs || !S.pos)) return -1;
     if ((S.epi == LE_DECAY || S.epi == LE_SIGPOW) && !S.bias) return -1;
-    if ((S.epi == LE_GEGLU || S.epi == LE_SWIGLU) && ((S.N & 1) || S.cb < S.N)) return -1;
+    if ((S.epi == LE_GEGLU || S.epi == LE_SWIGLU || S.epi == LE_SILUGLU) && ((S.N & 1) || S.cb < S.N)) return -1;
     if (S.epi == LE_GATE && !S.gate) return -1;
     if (S.ks < 1 || S.ks > S.nsub / 2 || (S.ks > 1 && (S.rows || S.yact || S.epi != LE_NONE))) return -1;
     if (S.rows && (!a.tiles || !a.ntiles || a.maxtiles < 1)) return -1;

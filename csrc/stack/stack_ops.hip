@@ -27,7 +27,7 @@ DEVI float bsum(float v, float* sh) {
 template <typename T> DEVI float ldv(const T* p, long i) { return (float)p[i]; }
 template <typename T> DEVI void stv(T* p, long i, float v) { p[i] = (T)v; }
 
-// ---- x[t] = table[id] * scale (+ the row of the token pair, + the position's vector), id from the host or (use_prev) the
+// ---- x[t] = table[id] * scale (+ the row of the token pair, + the position's vector, + a vector), id from the host or (use_prev) the
 // previous step's next_ids. The token ahead of a run's first is the slot's; the run's first row, which alone reads it,
 // leaves the run's last token there.
 struct Embed {
@@ -42,6 +42,7 @@ struct Embed {
   const int *runs, *tok_seq;
   const __bf16* ptab;      // optional [npos][D]
   const int* pos;
+  const float* add;        // optional [D]
   long ldx, ldc;
   int V, D, buckets, mul_prev, mul_cur, npos, f32, vec;
   float scale;
@@ -65,6 +66,7 @@ DEVI void embed_cols(const Embed& p, int t, const __bf16* row, const __bf16* pai
 #pragma unroll
     for (int e = 0; e < N; ++e) {
       y[e] = (float)a[e] * p.scale + (float)b[e] + (float)c[e];
+      if (p.add) y[e] += p.add[i + e];
       yb[e] = (__bf16)y[e];
     }
     *reinterpret_cast<fn*>(p.x + (size_t)t * p.ldx + i) = y;
@@ -113,8 +115,8 @@ __global__ __launch_bounds__(256) void embed_kernel(Embed p) {
 // ---- x[t] += norm(y) * w (w null: x[t] += y); y = one row (the sum of `nslab` slabs' rows), or (topk)
 // sum_j topw[t][j] * ye[t * topk + j] (+ ye[sh0 + t], the shared expert); y null: x is only read. Optional second norm (the
 // next sublayers' or the model's last one) of the new x into `on`. norm: (v - mean) / sqrt(var + eps), or (rms)
-// v / sqrt(mean(v^2) + eps). Without `keep` the new x is y (+ `add`, a vector) itself. The normed x may go out with two weights
-// (`ow` / `ow2`), and (gate) times a gate per column.
+// v / sqrt(mean(v^2) + eps), of `groups` equal parts of the row each on its own (rms). `add`, a vector, comes on top of the new x;
+// without `keep` the old x is left out. The normed x may go out with two weights (`ow` / `ow2`), and (gate) times a gate per column.
 // A workgroup per row (`rows`: gathered), 4 consecutive columns x NV per thread in registers.
 struct NormAdd {
   const float* y;
@@ -132,12 +134,13 @@ struct NormAdd {
   int nslab;
   long slab;            // elements between slabs
   long ldxb;
-  const float* add;     // optional [D], added to y
+  const float* add;     // optional [D], added to the new x
   int keep;
   const float* ow2;     // optional second weight of the output norm
   void* on2;            // its output, row stride ldo
   const void* gate;     // optional [rows][ldg], activation type: on *= gate
   long ldg;
+  int groups;           // parts of the row that are normed each on its own
 };
 
 // 4 consecutive values, columns i .. i + 3 of a row of D (VEC: D and the row strides are multiples of 4)
@@ -191,9 +194,62 @@ DEVI void put4(__bf16* p, int i, int D, const f32x4& v) {
       if (i + e < D) p[i + e] = b[e];
   }
 }
+// RMS norm of `groups` parts of the row each on its own. Parts of whole 256 columns are sums of the waves' sums, others are added up
+// from the squares in LDS (sh: D + groups floats).
+template <int NV, int NTH>
+DEVI void normalise_groups(f32x4 (&v)[NV], int D, float eps, int groups, float* sh) {
+  constexpr int NW = NTH / 64;
+  const int gs = D / groups, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  if (!(gs & 255)) {
+    const int per = gs >> 8;                       // 256-column slots of a part; slot j * NW + wave holds columns 256 slot ..
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const float s = wsum((v[j][0] * v[j][0] + v[j][1] * v[j][1]) + (v[j][2] * v[j][2] + v[j][3] * v[j][3]));
+      if (lane == 0) sh[j * NW + wave] = s;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int s0 = (j * NW + wave) / per * per;
+      if (s0 >= D >> 8) continue;
+      float s = 0.f;
+      for (int i = 0; i < per; ++i) s += sh[s0 + i];
+      v[j] *= 1.f / sqrtf(s / (float)gs + eps);
+    }
+    __syncthreads();
+    return;
+  }
+#pragma unroll
+  for (int j = 0; j < NV; ++j)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = (int)(threadIdx.x + j * NTH) * 4 + e;
+      if (i < D) sh[i] = v[j][e] * v[j][e];
+    }
+  __syncthreads();
+  for (int g = wave; g < groups; g += NW) {
+    float s = 0.f;
+    for (int i = lane; i < gs; i += 64) s += sh[g * gs + i];
+    s = wsum(s);
+    if (lane == 0) sh[D + g] = 1.f / sqrtf(s / (float)gs + eps);
+  }
+  __syncthreads();
+#pragma unroll
+  for (int j = 0; j < NV; ++j)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int i = (int)(threadIdx.x + j * NTH) * 4 + e;
+      if (i < D) v[j][e] *= sh[D + i / gs];
+    }
+}
+
 // the norm over the row's D columns (columns past D hold zeros)
 template <int NV, int NTH>
-DEVI void normalise(f32x4 (&v)[NV], int D, float eps, int rms, float* sh) {
+DEVI void normalise(f32x4 (&v)[NV], int D, float eps, int rms, int groups, float* sh) {
+  if (groups > 1) {
+    normalise_groups<NV, NTH>(v, D, eps, groups, sh);
+    return;
+  }
   float s = 0.f, mean = 0.f;
   if (!rms) {
 #pragma unroll
@@ -216,14 +272,15 @@ DEVI void normalise(f32x4 (&v)[NV], int D, float eps, int rms, float* sh) {
 
 template <int NV, int NTH, bool VEC>
 __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
-  __shared__ float sh[NTH / 64];
+  extern __shared__ float sh[];
   const int t = p.rows ? p.rows[blockIdx.x] : (int)blockIdx.x, D = p.D;
   float* xr = p.x + (size_t)t * p.ldx;
   f32x4 v[NV], x[NV], w[NV];
 #pragma unroll
-  for (int j = 0; j < NV; ++j)
-    x[j] = p.keep ? row4<VEC>(xr, (threadIdx.x + j * NTH) * 4, D)
-                  : p.add ? row4<VEC>(p.add, (threadIdx.x + j * NTH) * 4, D) : f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int j = 0; j < NV; ++j) {
+    x[j] = p.keep ? row4<VEC>(xr, (threadIdx.x + j * NTH) * 4, D) : f32x4{0.f, 0.f, 0.f, 0.f};
+    if (p.add) x[j] += row4<VEC>(p.add, (threadIdx.x + j * NTH) * 4, D);
+  }
   if (p.y) {
 #pragma unroll
     for (int j = 0; j < NV; ++j)
@@ -248,7 +305,7 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
 #pragma unroll
         for (int j = 0; j < NV; ++j) v[j] += row4<VEC>(p.y + s * p.slab + (size_t)t * p.ldy, (threadIdx.x + j * NTH) * 4, D);
     }
-    if (p.w) normalise<NV, NTH>(v, D, p.eps, p.rms, sh);
+    if (p.w) normalise<NV, NTH>(v, D, p.eps, p.rms, p.groups, sh);
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int i = (threadIdx.x + j * NTH) * 4;
@@ -263,7 +320,7 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
   if (!p.ow) return;
 #pragma unroll
   for (int j = 0; j < NV; ++j) w[j] = row4<VEC>(p.ow, (threadIdx.x + j * NTH) * 4, D);
-  normalise<NV, NTH>(x, D, p.eps, p.rms, sh);
+  normalise<NV, NTH>(x, D, p.eps, p.rms, p.groups, sh);
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int i = (threadIdx.x + j * NTH) * 4;
@@ -284,11 +341,16 @@ __global__ __launch_bounds__(NTH) void norm_add_kernel(NormAdd p) {
   }
 }
 
+// LDS of a row's sums: one float per wave and group of 4 columns per thread, or the squares of all columns
+inline size_t norm_lds(const NormAdd& p, int slots) {
+  return 4 * (size_t)(p.groups > 1 && (p.D / p.groups & 255) ? p.D + p.groups : slots);
+}
+
 template <bool VEC>
 int norm_add_v(const NormAdd& p, int n, hipStream_t st) {
 #define NLS_NA(LIM, NV, NTH) \
   if (p.D <= LIM) { \
-    hipLaunchKernelGGL((norm_add_kernel<NV, NTH, VEC>), dim3(n), dim3(NTH), 0, st, p); \
+    hipLaunchKernelGGL((norm_add_kernel<NV, NTH, VEC>), dim3(n), dim3(NTH), norm_lds(p, NV * NTH / 64), st, p); \
     return (int)hipGetLastError(); \
   }
   NLS_NA(1024, 1, 256) NLS_NA(2048, 2, 256)
@@ -299,7 +361,7 @@ int norm_add_v(const NormAdd& p, int n, hipStream_t st) {
 }
 
 inline int norm_add(const NormAdd& p, int n, hipStream_t st) {
-  if (n < 1 || p.D < 1) return -1;
+  if (n < 1 || p.D < 1 || p.groups < 1 || p.D % p.groups || (p.groups > 1 && !p.rms) || norm_lds(p, 0) > 65536) return -1;
   const bool vec = !(p.D & 3) && !(p.ldx & 3) && !(p.ldy & 3) && !(p.ldo & 3) && !(p.ldxb & 3) && !(p.ldg & 3) &&
                    !(((uintptr_t)p.gate | (uintptr_t)p.xb | (uintptr_t)p.add) & 15);
   return vec ? norm_add_v<true>(p, n, st) : norm_add_v<false>(p, n, st);
@@ -352,6 +414,7 @@ struct AttnRows {
   long ldq, ldqo, ldc;        // row strides: projections, qo, caches
   int H, G, D, Dp, rot, V;    // V: columns of a value head
   float eps;
+  int hnorm;                  // each rotated head of q and k is RMS-normed on its own, without weights
 };
 
 template <typename T>
@@ -461,8 +524,116 @@ __global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
   }
 }
 
+// the same with an RMS norm without weights of each rotated head of q and k: one wave per head
+template <typename T>
+__global__ __launch_bounds__(256) void attn_head_rows_kernel(AttnRows p) {
+  constexpr int NP = 8;                           // pairs of columns per lane: heads of up to 1024 columns
+  const int t = blockIdx.x, D = p.D, D2 = (D + 1) >> 1, lane = threadIdx.x & 63;
+  const int slot = p.slot[t], u = blockIdx.y * 4 + (threadIdx.x >> 6);          // a head of q, k or v
+  if (u >= p.H + 2 * p.G || (u >= p.H && slot < 0)) return;
+  if (u >= p.H + p.G) {
+    const int h = u - p.H - p.G;
+    const float* a = p.v + (size_t)t * p.ldq + (size_t)h * p.V;
+    T* o = (T*)p.vc + (size_t)slot * p.ldc + (size_t)h * p.Dp;
+    for (int c = lane; c < p.V; c += 64) o[c] = (T)a[c];
+    return;
+  }
+  const bool isq = u < p.H;
+  const int h = isq ? u : u - p.H;
+  const float* a = (isq ? p.q : p.k) + (size_t)t * p.ldq + (size_t)h * D;
+  T* o = isq ? (T*)p.qo + (size_t)t * p.ldqo + (size_t)h * p.Dp : (T*)p.kc + (size_t)slot * p.ldc + (size_t)h * p.Dp;
+  const float* f = p.rot ? p.cs + (size_t)p.pos[t] * p.rot : nullptr;
+  float x[NP], y[NP], s = 0.f;
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const int i = lane + 64 * j, c = 2 * i;
+    x[j] = y[j] = 0.f;
+    if (i >= D2) continue;
+    x[j] = a[c];
+    if (c + 1 < D) y[j] = a[c + 1];
+    if (c < p.rot) {
+      const float cc = f[c], ss = f[c + 1], v = x[j] * cc - y[j] * ss;
+      y[j] = y[j] * cc + x[j] * ss;
+      x[j] = v;
+    }
+    s += x[j] * x[j] + y[j] * y[j];
+  }
+  const float inv = 1.f / sqrtf(wsum(s) / (float)D + p.eps);
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const int i = lane + 64 * j, c = 2 * i;
+    if (i >= D2) continue;
+    o[c] = (T)(x[j] * inv);
+    if (c + 1 < D) o[c + 1] = (T)(y[j] * inv);
+  }
+}
+
+// ---- PolyNorm: out = a N(z) + b N(z^2) + c N(z^3) + e of each row, powers by element, N(v) = v / sqrt(mean(v^2) + eps)
+template <typename T, int NTH>
+__global__ __launch_bounds__(NTH) void poly_norm_kernel(const T* __restrict__ z, long ldz, const float* __restrict__ act,
+                                                        T* __restrict__ out, long ldo, int N, float eps) {
+  typedef T t8 __attribute__((ext_vector_type(8)));
+  __shared__ float sh[3][NTH / 64];
+  const T* a = z + (size_t)blockIdx.x * ldz;
+  T* o = out + (size_t)blockIdx.x * ldo;
+  float s1 = 0.f, s2 = 0.f, s3 = 0.f;
+  const int N8 = N & ~7;
+  auto add = [&](float v) {
+    const float q = v * v, q2 = q * q;
+    s1 += q;
+    s2 += q2;
+    s3 += q2 * q;
+  };
+  for (int i = threadIdx.x * 8; i < N8; i += NTH * 8) {
+    const t8 v = *reinterpret_cast<const t8*>(a + i);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) add((float)v[e]);
+  }
+  if (N8 + (int)threadIdx.x < N) add((float)a[N8 + threadIdx.x]);
+  s1 = wsum(s1);
+  s2 = wsum(s2);
+  s3 = wsum(s3);
+  if ((threadIdx.x & 63) == 0) {
+    sh[0][threadIdx.x >> 6] = s1;
+    sh[1][threadIdx.x >> 6] = s2;
+    sh[2][threadIdx.x >> 6] = s3;
+  }
+  __syncthreads();
+  s1 = s2 = s3 = 0.f;
+#pragma unroll
+  for (int i = 0; i < NTH / 64; ++i) {
+    s1 += sh[0][i];
+    s2 += sh[1][i];
+    s3 += sh[2][i];
+  }
+  const float n = (float)N, k1 = act[0] / sqrtf(s1 / n + eps), k2 = act[1] / sqrtf(s2 / n + eps), k3 = act[2] / sqrtf(s3 / n + eps);
+  const float k0 = act[3];
+  auto poly = [&](float v) { return fmaf(fmaf(fmaf(k3, v, k2), v, k1), v, k0); };
+  for (int i = threadIdx.x * 8; i < N8; i += NTH * 8) {
+    const t8 v = *reinterpret_cast<const t8*>(a + i);
+    t8 y;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) y[e] = (T)poly((float)v[e]);
+    *reinterpret_cast<t8*>(o + i) = y;
+  }
+  if (N8 + (int)threadIdx.x < N) o[N8 + threadIdx.x] = (T)poly((float)a[N8 + threadIdx.x]);
+}
+
+template <typename T>
+int poly_norm_t(const void* z, long ldz, const float* act, void* out, long ldo, int N, int n, float eps, hipStream_t st) {
+  if (N > 8192 || n <= 64)
+    hipLaunchKernelGGL((poly_norm_kernel<T, 1024>), dim3(n), dim3(1024), 0, st, (const T*)z, ldz, act, (T*)out, ldo, N, eps);
+  else
+    hipLaunchKernelGGL((poly_norm_kernel<T, 256>), dim3(n), dim3(256), 0, st, (const T*)z, ldz, act, (T*)out, ldo, N, eps);
+  return (int)hipGetLastError();
+}
+
 template <typename T>
 int attn_rows_t(const AttnRows& p, int n, hipStream_t st) {
+  if (p.hnorm) {
+    hipLaunchKernelGGL(attn_head_rows_kernel<T>, dim3(n, (p.H + 2 * p.G + 3) / 4), dim3(256), 0, st, p);
+    return (int)hipGetLastError();
+  }
   const int cols = (p.H + p.G) * p.D;
   const bool vec = !((p.D | p.V) & 3) && !(p.ldq & 3) && !(p.Dp & 3) && !(p.ldqo & 3) && !(p.ldc & 3) &&
                    !(((uintptr_t)p.q | (uintptr_t)p.k | (uintptr_t)p.v) & 15);
@@ -479,13 +650,38 @@ int attn_rows_t(const AttnRows& p, int n, hipStream_t st) {
   return (int)hipGetLastError();
 }
 
-// ---- expert choice of one token: sigmoid scores, the `keep` groups with the largest sum of their two best scores, the
-// `topk` best experts of those; weight = score * scale. Ties go to the lowest index. One wave per token; scores in LDS.
-DEVI void pick_experts(const float* __restrict__ z, int E, int topk, int groups, int keep, float scale, int lane,
-                       float* sc, float* gs, float* __restrict__ topw, int* __restrict__ sel) {
-  for (int e = lane; e < E; e += 64) {
-    const float s = 1.f / (1.f + expf(-z[e]));
-    sc[e] = s == s ? s : -1.f;
+// ---- expert choice of one token: scores (sigmoid, or a softmax over all experts), the `keep` groups with the largest sum of their
+// two best scores (gbest 2) or the largest score (1), the `topk` best experts of those; weight = score * scale. Ties go to the
+// lowest index. One wave per token; scores in LDS.
+struct Route {
+  int E, topk, groups, keep, softmax, gbest;
+  float scale;
+};
+
+DEVI void pick_experts(const float* __restrict__ z, const Route& R, int lane, float* sc, float* gs, float* __restrict__ topw,
+                       int* __restrict__ sel) {
+  const int E = R.E, topk = R.topk, groups = R.groups, keep = R.keep;
+  const float scale = R.scale;
+  if (R.softmax) {
+    float m = -INFINITY, l = 0.f;
+    for (int e = lane; e < E; e += 64) m = fmaxf(m, z[e]);
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) m = fmaxf(m, __shfl_xor(m, o, 64));
+    for (int e = lane; e < E; e += 64) {
+      const float s = expf(z[e] - m);
+      sc[e] = s;
+      l += s;
+    }
+    l = wsum(l);
+    for (int e = lane; e < E; e += 64) {
+      const float s = sc[e] / l;
+      sc[e] = s == s ? s : -1.f;
+    }
+  } else {
+    for (int e = lane; e < E; e += 64) {
+      const float s = 1.f / (1.f + expf(-z[e]));
+      sc[e] = s == s ? s : -1.f;
+    }
   }
   __builtin_amdgcn_wave_barrier();
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -497,7 +693,7 @@ DEVI void pick_experts(const float* __restrict__ z, int E, int topk, int groups,
       if (s > a) { b = a; a = s; }
       else if (s > b) b = s;
     }
-    gs[g] = per > 1 ? a + b : a;
+    gs[g] = per > 1 && R.gbest == 2 ? a + b : a;
   }
   __builtin_amdgcn_wave_barrier();
   asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -534,31 +730,28 @@ DEVI void pick_experts(const float* __restrict__ z, int E, int topk, int groups,
 constexpr int ME = 512;       // experts per layer
 constexpr int PW = 8;         // waves that choose experts in moe_plan_kernel<true>
 
-__global__ __launch_bounds__(64) void moe_pick_kernel(const float* __restrict__ z, long ldz, int E, int topk,
-                                                      int groups, int keep, float scale, float* __restrict__ topw,
+__global__ __launch_bounds__(64) void moe_pick_kernel(const float* __restrict__ z, long ldz, Route R, float* __restrict__ topw,
                                                       int* __restrict__ sel) {
   __shared__ float sc[ME], gs[ME];
   const int t = blockIdx.x;
-  pick_experts(z + (size_t)t * ldz, E, topk, groups, keep, scale, threadIdx.x, sc, gs, topw + (size_t)t * topk,
-               sel + (size_t)t * topk);
+  pick_experts(z + (size_t)t * ldz, R, threadIdx.x, sc, gs, topw + (size_t)t * R.topk, sel + (size_t)t * R.topk);
 }
 
 // ---- routed-entry lists of one step: entries (token t, choice j) = t * topk + j grouped by expert (entry order within
 // an expert is arbitrary: rows do not interact), and the (expert, <= bm entries) tiles of the grouped products.
 // One workgroup. PICK: also choose the experts (small steps: one launch less).
 template <bool PICK>
-__global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict__ z, long ldz, int T, int E, int topk,
-                                                        int groups, int keep, float scale, float* __restrict__ topw,
-                                                        int* __restrict__ sel, int bm, int* __restrict__ rows,
-                                                        int* __restrict__ tiles, int* __restrict__ ntiles, int maxtiles) {
+__global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict__ z, long ldz, int T, Route R,
+                                                        float* __restrict__ topw, int* __restrict__ sel, int bm,
+                                                        int* __restrict__ rows, int* __restrict__ tiles,
+                                                        int* __restrict__ ntiles, int maxtiles) {
   __shared__ int cnt[ME], off[ME], pos[ME];
   __shared__ float sc[PICK ? PW : 1][PICK ? ME : 1], gs[PICK ? PW : 1][PICK ? ME : 1];
-  const int n = T * topk;
+  const int E = R.E, topk = R.topk, n = T * topk;
   if constexpr (PICK) {
     const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
     for (int t = w; w < PW && t < T; t += PW)
-      pick_experts(z + (size_t)t * ldz, E, topk, groups, keep, scale, lane, sc[w], gs[w], topw + (size_t)t * topk,
-                   sel + (size_t)t * topk);
+      pick_experts(z + (size_t)t * ldz, R, lane, sc[w], gs[w], topw + (size_t)t * topk, sel + (size_t)t * topk);
     __threadfence_block();
   }
   for (int e = threadIdx.x; e < E; e += 1024) cnt[e] = 0;
@@ -650,31 +843,31 @@ using namespace nls_stack;
 int nls_stack_embed(int* ids, const int* next_ids, const int* use_prev, const void* tab, int V, int D, float scale,
                     float* x, void* xb, long ldx, int T, void* c0, void* c1, long ldc, int f32, const void* pairs, int buckets,
                     int mul_prev, int mul_cur, int* prev, const int* runs, const int* tok_seq, const void* ptab, int npos,
-                    const int* pos, void* stream) {
+                    const int* pos, const float* add, void* stream) {
   if (T < 1 || D < 1 || V < 1 || (pairs && (buckets < 1 || !prev || !runs || !tok_seq)) || (ptab && (npos < 1 || !pos))) return -1;
   const uintptr_t at = (uintptr_t)tab | (uintptr_t)x | (uintptr_t)xb | (uintptr_t)c0 | (uintptr_t)c1 | (uintptr_t)pairs |
                        (uintptr_t)ptab;
   const int vec = !((D | ldx | ldc) & 7) && !(at & 31);
   const Embed p{ids, next_ids, use_prev, (const __bf16*)tab, x, (__bf16*)xb, c0, c1, (const __bf16*)pairs, prev, runs, tok_seq,
-                (const __bf16*)ptab, pos, ldx, ldc, V, D, buckets, mul_prev, mul_cur, npos, f32, vec, scale};
+                (const __bf16*)ptab, pos, add, ldx, ldc, V, D, buckets, mul_prev, mul_cur, npos, f32, vec, scale};
   hipLaunchKernelGGL(embed_kernel, dim3(T), dim3(256), 0, (hipStream_t)stream, p);
   return (int)hipGetLastError();
 }
 
 int nls_norm_add(const float* y, long ldy, const float* topw, int topk, long sh0, const float* w, float* x, long ldx, void* xb,
                  long ldxb, const float* ow, void* on, const float* ow2, void* on2, long ldo, const float* add, int keep, int D,
-                 int T, float eps, int f32, int rms, int nslab, long slab, void* stream) {
-  if (!y || nslab < 1 || (slab & 3) || (ow2 && (!ow || !on2)) || (keep && add)) return -1;
+                 int T, float eps, int f32, int rms, int groups, int nslab, long slab, void* stream) {
+  if (!y || nslab < 1 || (slab & 3) || (ow2 && (!ow || !on2))) return -1;
   return norm_add(NormAdd{y, topw, w, x, xb, ow, on, nullptr, ldy, ldx, ldo, sh0, D, topk, f32, rms, eps, nslab, slab, ldxb, add,
-                          keep, ow2, on2, nullptr, 0}, T, (hipStream_t)stream);
+                          keep, ow2, on2, nullptr, 0, groups}, T, (hipStream_t)stream);
 }
 
 // out[i] = norm(x[rows ? rows[i] : i]) * w (* gate[i]); w2, out2: the same with another weight
 int nls_row_norm(const float* x, long ldx, const int* rows, const float* w, void* out, const float* w2, void* out2, long ldo,
-                 const void* gate, long ldg, int D, int n, float eps, int f32, int rms, void* stream) {
+                 const void* gate, long ldg, int D, int n, float eps, int f32, int rms, int groups, void* stream) {
   if (w2 && !out2) return -1;
   return norm_add(NormAdd{nullptr, nullptr, nullptr, const_cast<float*>(x), nullptr, w, out, rows, 0, ldx, ldo, -1, D, 0,
-                          f32, rms, eps, 1, 0, 0, nullptr, 1, w2, out2, gate, ldg}, n, (hipStream_t)stream);
+                          f32, rms, eps, 1, 0, 0, nullptr, 1, w2, out2, gate, ldg, groups}, n, (hipStream_t)stream);
 }
 
 int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq, long ldcq, const float* dkv,
@@ -690,15 +883,22 @@ int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq
   return (int)hipGetLastError();
 }
 
-// heads of D columns (values: V), Dp apart in the outputs; rot even, at most D
+// heads of D columns (values: V), Dp apart in the outputs; rot even, at most D; hnorm: no weights
 int nls_attn_rows(const float* q, const float* k, const float* v, long ldq, const float* qn, const float* kn, const float* cs,
                   const int* pos, const int* slot, void* qo, long ldqo, void* kc, void* vc, long ldc, int T, int H, int G,
-                  int D, int V, int Dp, int rot, float eps, int f32, void* stream) {
-  if (T < 1 || H < 1 || G < 1 || D < 1 || V < 1 || Dp < D || Dp < V || (v == k && V != D) || (rot && !cs) || (rot & 1) || rot < 0 ||
+                  int D, int V, int Dp, int rot, int hnorm, float eps, int f32, void* stream) {
+  if (T < 1 || (hnorm && (qn || kn || D > 1024)) || H < 1 || G < 1 || D < 1 || V < 1 || Dp < D || Dp < V || (v == k && V != D) || (rot && !cs) || (rot & 1) || rot < 0 ||
       rot > D || (long)H * Dp > ldqo || (long)G * Dp > ldc)
     return -1;
-  AttnRows p{q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, ldq, ldqo, ldc, H, G, D, Dp, rot, V, eps};
+  AttnRows p{q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, ldq, ldqo, ldc, H, G, D, Dp, rot, V, eps, hnorm};
   return f32 ? attn_rows_t<float>(p, T, (hipStream_t)stream) : attn_rows_t<__bf16>(p, T, (hipStream_t)stream);
+}
+
+// z, out: rows of N values, 16-byte aligned; act: a, b, c, e
+int nls_poly_norm(const void* z, long ldz, const float* act, void* out, long ldo, int N, int n, float eps, int f32, void* stream) {
+  if (n < 1 || N < 1 || ((ldz | ldo) & 7) || (((uintptr_t)z | (uintptr_t)out) & 15)) return -1;
+  return f32 ? poly_norm_t<float>(z, ldz, act, out, ldo, N, n, eps, (hipStream_t)stream)
+             : poly_norm_t<__bf16>(z, ldz, act, out, ldo, N, n, eps, (hipStream_t)stream);
 }
 
 int nls_stack_argmax(const float* z, long ldz, int V, int* out, int n, void* stream) {
@@ -708,20 +908,21 @@ int nls_stack_argmax(const float* z, long ldz, int V, int* out, int n, void* str
 }
 
 // rows: int [T * topk]; tiles: int [maxtiles][4], maxtiles >= min(T * topk, E + T * topk / bm)
-int nls_moe_plan(const float* z, long ldz, int T, int E, int topk, int groups, int keep, float scale, float* topw,
-                 int* sel, int bm, int* rows, int* tiles, int* ntiles, int maxtiles, void* stream) {
+int nls_moe_plan(const float* z, long ldz, int T, int E, int topk, int groups, int keep, int softmax, int gbest, float scale,
+                 float* topw, int* sel, int bm, int* rows, int* tiles, int* ntiles, int maxtiles, void* stream) {
   if (T < 1 || E < 1 || E > ME || topk < 1 || topk > E || groups < 1 || E % groups || keep < 1 || bm < 1 ||
-      (long)min(keep, groups) * (E / groups) < topk || maxtiles < 1)
+      (long)min(keep, groups) * (E / groups) < topk || maxtiles < 1 || gbest < 1 || gbest > 2)
     return -1;
+  const Route R{E, topk, groups, keep, softmax, gbest, scale};
   hipStream_t st = (hipStream_t)stream;
   if (T <= 32) {
-    hipLaunchKernelGGL(moe_plan_kernel<true>, dim3(1), dim3(1024), 0, st, z, ldz, T, E, topk, groups, keep, scale, topw,
-                       sel, bm, rows, tiles, ntiles, maxtiles);
+    hipLaunchKernelGGL(moe_plan_kernel<true>, dim3(1), dim3(1024), 0, st, z, ldz, T, R, topw, sel, bm,
+                       rows, tiles, ntiles, maxtiles);
     return (int)hipGetLastError();
   }
-  hipLaunchKernelGGL(moe_pick_kernel, dim3(T), dim3(64), 0, st, z, ldz, E, topk, groups, keep, scale, topw, sel);
-  hipLaunchKernelGGL(moe_plan_kernel<false>, dim3(1), dim3(1024), 0, st, z, ldz, T, E, topk, groups, keep, scale, topw,
-                     sel, bm, rows, tiles, ntiles, maxtiles);
+  hipLaunchKernelGGL(moe_pick_kernel, dim3(T), dim3(64), 0, st, z, ldz, R, topw, sel);
+  hipLaunchKernelGGL(moe_plan_kernel<false>, dim3(1), dim3(1024), 0, st, z, ldz, T, R, topw, sel, bm, rows,
+                     tiles, ntiles, maxtiles);
   return (int)hipGetLastError();
 }
 

@@ -1,7 +1,7 @@
 """Decoder stacks assembled from a config: a list of layers, each a mixer plus an optional feed-forward.
 
 A mixer or feed-forward is a class that loads its weights, adds its step buffers, and runs on the rows of a step; a layer
-class (OutputNormLayer, SharedNormLayer) places the norms and joins the sublayers. A looped model runs some layers several
+class (OutputNormLayer, SharedNormLayer, SandwichNormLayer) places the norms and joins the sublayers. A looped model runs some layers several
 times with the same weights. The per-token cache rows (paged) and the per-sequence states (slots) of all layer runs belong to
 the engine, which sees them as `kv_cache` / `state_pool`. Everything runs on the HIP kernels of csrc/stack (ops/stack.py): bf16
 operands with an f32 residual, or `dtype=torch.float32` for 32-bit throughout.
@@ -13,8 +13,9 @@ tokens), all in one batch:
 """
 from __future__ import annotations
 
+import math
 import os
-from dataclasses import dataclass, field
+from dataclasses import astuple, dataclass, field
 from typing import Dict, List, Optional
 
 import numpy as np
@@ -265,26 +266,36 @@ class LatentMixer(_Part):
 
 
 class MoeFeedForward(_Part):
-    """Routed experts (two matrices, squared-relu) chosen by group-limited sigmoid scores, plus a shared expert. Leaves
-    the experts' output rows in `ye`; the caller's output norm combines them."""
+    """Routed experts (two matrices with a squared relu, or three with a silu gate) chosen by group-limited scores, plus a shared
+    expert. Leaves the experts' output rows in `ye`; the caller's output norm combines them."""
+    EPI = {"relu2": "relu2", "silu_glu": "siluglu"}
 
     def __init__(self, model, i, cfg, prefix):
         super().__init__(model, i, cfg, prefix)
         d, E = model.cfg.d_model, cfg.experts
         self.router = self.lin("router", (E, d))
-        self.up = self.lin(torch.stack([self.t(f"e{j}.up") for j in range(E)]), (E, cfg.ff, d))
+        self.glu = model.cfg.design.expert_act == "silu_glu"
+        self.up = self.lin(torch.stack([self.first(f"e{j}.") for j in range(E)]), (E, cfg.ff * (1 + self.glu), d))
         self.down = self.lin(torch.stack([self.t(f"e{j}.down") for j in range(E)]), (E, d, cfg.ff))
         if cfg.shared_ff:
-            self.sup, self.sdown = self.lin("shared.up", (cfg.shared_ff, d)), self.lin("shared.down", (d, cfg.shared_ff))
+            self.sup = self.lin(self.first("shared."), (cfg.shared_ff * (1 + self.glu), d))
+            self.sdown = self.lin("shared.down", (d, cfg.shared_ff))
+
+    def first(self, name: str) -> torch.Tensor:
+        """The matrix ahead of the activation; gate and up rows alternate."""
+        up = self.t(name + "up")
+        return torch.stack([self.t(name + "gate"), up], 1).reshape(-1, up.shape[1]) if self.glu else up
 
     def bind(self, b: StackBuffers) -> dict:
         c, P = self.cfg, b.pad
         k = c.top
-        act = self.m.cfg.design.expert_act
+        design = self.m.cfg.design
+        act = self.EPI[design.expert_act]
         key = ("plan", c.experts, k, c.groups, c.keep, c.scale)
         plan = b.launches.get(key)
         if plan is None:
-            plan = b.launches[key] = K.MoePlan(P, c.experts, k, c.groups, c.keep, c.scale, self.m.device)
+            plan = b.launches[key] = K.MoePlan(P, c.experts, k, c.groups, c.keep, c.scale, self.m.device, design.router_score,
+                                               {"top2": 2, "max": 1}[design.router_group])
         z = self.scratch(b, "moe.z", P, c.experts, torch.float32)
         h = self.scratch(b, "moe.h", P * k, K.act_ld(c.ff))
         ye = self.scratch(b, "moe.y", P * (k + 1), self.m.cfg.d_model, torch.float32)
@@ -307,7 +318,7 @@ class MoeFeedForward(_Part):
 
 
 class _SharedPart(_Part):
-    """A part of a SharedNormLayer: reads the layer's normed input through segments of the layer's one input launch and leaves
+    """A part of a SharedNormLayer (or of a SandwichNormLayer, which has one in each half): reads the layer's normed input through segments of the layer's one input launch and leaves
     its operand of the layer's one output product in `out` (columns of a shared buffer). `scale` weights its output; it goes
     into a 32-bit factor that the operand is multiplied with anyway, so it costs no rounding."""
     out_width = 0                 # columns of the operand, a multiple of 64
@@ -338,10 +349,10 @@ class _SharedPart(_Part):
 
 
 class AttentionPart(_SharedPart):
-    """Grouped-query softmax attention: queries and keys optionally RMS-normed over their whole projections, rotary positions
-    on the first columns of each head, values projected on their own or equal to the projected keys, optionally a sigmoid gate
-    per head, a sliding window with kept first keys, one more in the denominator. The cache holds the finished keys and the
-    values, [2][slots][kv_heads * padded head]."""
+    """Grouped-query softmax attention: queries and keys optionally RMS-normed over their whole projections or (rotated) per
+    head, rotary positions on the first columns of each head, values projected on their own or equal to the projected keys,
+    optionally a sigmoid gate per head or per output column, a sliding window with kept first keys, one more in the denominator,
+    heads whose softmax weights are mixed. The cache holds the finished keys and the values, [2][slots][kv_heads * padded head]."""
 
     def __init__(self, model, i, cfg, prefix, scale=1.0):
         super().__init__(model, i, cfg, prefix, scale)
@@ -352,22 +363,35 @@ class AttentionPart(_SharedPart):
         self.mfma = self.mfma and not model.f32
         self.own_values = design.attn_values == "projection"
         names = [("q", H * D), ("k", G * D)] + ([("v", G * V)] if self.own_values else [])
-        self.qkv = self.lin(torch.cat([self.mat(n, (rows, d)) for n, rows in names]))
+        w = {n: self.mat(n, (rows, d)) for n, rows in names}
+        if design.rotary == "halves":
+            # columns i and i + dims / 2 of a head become neighbours: scores and norms do not see the order
+            half = torch.arange(c.rot_dims, device=model.device).view(2, -1).T.reshape(-1)
+            order = torch.cat([half, torch.arange(c.rot_dims, D, device=model.device)])
+            for n, heads in (("q", H), ("k", G)):
+                w[n] = w[n].view(heads, D, d)[:, order].reshape(heads * D, d)
+        self.qkv = self.lin(torch.cat([w[n] for n, _ in names]))
         self.mask = dict(window=c.window, keep=c.keep_first, sink=design.attn_sink)
-        if not design.attn_gate and scale != 1.0:
+        if design.attn_gate != "head" and scale != 1.0:
             raise ValueError("a weighted attention output needs its head gate")
+        if (design.attn_gate == "column") != design.attn_talk:
+            raise NotImplementedError("a gate per column and mixed heads come together")
         self.qn = self.kn = None
         if design.attn_qk_norm == "projection":
             self.qn, self.kn = self.vecn("q.norm", H * D), self.vecn("k.norm", G * D)
-        self.g = self.lin("g", (H, d)) if design.attn_gate else None
-        self.cs = model.rope(c.rot_base, c.rot_dims) if c.rot_dims else None
+        self.g = self.lin("g", (H if design.attn_gate == "head" else H * V, d)) if design.attn_gate else None
+        self.cs = model.rope(c.rot_base, c.rot_dims, c.rot_scaling) if c.rot_dims else None
+        self.talk = None
+        if design.attn_talk:
+            self.talk_plan = K.TalkPlan(H, G, self.Dp, c.window, model.cfg.ctx, model.f32, model.device)
+            self.talk = self.talk_plan.matrix(self.mat("talk", (H, H)))
         self.cache_width = 2 * G * self.Dp
         self.out_width = K.act_ld(H * self.Dp)
         self.groups = K.attn_groups(H, G)
 
     @property
     def plan_run(self):
-        return _FLASH_RUN if self.mfma else None
+        return _FLASH_RUN if (self.mfma if self.talk is None else self.talk_plan.prefill) else None
 
     def new_cache(self, slots):
         return torch.zeros(2, slots, self.cfg.kv_heads * self.Dp, dtype=self.m.dtype, device=self.m.device)
@@ -382,23 +406,42 @@ class AttentionPart(_SharedPart):
         c, P, f = self.cfg, b.pad, torch.float32
         H, G, D = c.heads, c.kv_heads, c.dim
         qkv = self.scratch(b, "attn.qkv", P, K.pad_to(self.qkv.N, 4), f)
-        gate = self.scratch(b, "attn.gate", P, H, f) if self.g is not None else None
+        gate = None
+        if self.g is not None:                            # per column: in the activation type, 16-byte rows
+            gate = self.scratch(b, "attn.gate", P, H, f) if self.talk is None else \
+                self.scratch(b, "attn.cgate", P, K.pad_to(self.g.N, 8))
         q = self.scratch(b, f"attn.q{D}", P, H * self.Dp)
-        n = _SPLIT_WG // self.groups + 1                  # rows x splits
-        part = (self.scratch(b, "attn.po", 1, n * H * self.Dp, f), self.scratch(b, "attn.pm", 1, n * H * 2, f),
-                self.scratch(b, "attn.cnt", 1, _SPLIT_WG + self.groups, torch.int32))
         k0 = H * D
-        return dict(q=q, gate=gate, out=out, part=part, qp=qkv, kp=qkv[:, k0:],
-                    vp=qkv[:, k0 + G * D:] if self.own_values else qkv[:, k0:],
-                    inputs=[K.Seg(self.qkv, x, qkv)] + ([K.Seg(self.g, x, gate, "sigmoid", alpha=self.scale)]
-                                                        if self.g is not None else []))
+        e = dict(q=q, gate=gate, out=out, qp=qkv, kp=qkv[:, k0:], vp=qkv[:, k0 + G * D:] if self.own_values else qkv[:, k0:],
+                 inputs=[K.Seg(self.qkv, x, qkv)] + ([K.Seg(self.g, x, gate, "sigmoid", alpha=self.scale)]
+                                                     if self.g is not None else []))
+        if self.talk is not None:
+            if self.talk_plan.mfma:
+                sizes = self.talk_plan.scratch(P)
+                names = ("talk.sc", "talk.st", "talk.po", "talk.cnt")
+                e["part"] = [self.scratch(b, n, 1, s, f if n != "talk.cnt" else torch.int32) for n, s in zip(names, sizes)]
+                e["part"] = [t.view(-1) for t in e["part"]]
+            return e
+        n = _SPLIT_WG // self.groups + 1                  # rows x splits
+        e["part"] = (self.scratch(b, "attn.po", 1, n * H * self.Dp, f), self.scratch(b, "attn.pm", 1, n * H * 2, f),
+                     self.scratch(b, "attn.cnt", 1, _SPLIT_WG + self.groups, torch.int32))
+        return e
 
     def run(self, b, e, cache, state, step: "_Step"):
         c, st, T = self.cfg, step.st, step.T
         kc, vc = cache[0], cache[1]
         K.attn_rows(e["qp"], e["kp"], e["vp"], self.qn, self.kn, self.cs, b.pos, b.slot, e["q"], kc, vc, T, c.heads,
-                    c.kv_heads, c.dim, self.Dp, c.rot_dims, self.m.cfg.eps, st, V=c.vdim)
+                    c.kv_heads, c.dim, self.Dp, c.rot_dims, self.m.cfg.eps, st, V=c.vdim,
+                    head_norm=self.m.cfg.design.attn_qk_norm == "head")
         plan = step.plan
+        if self.talk is not None:
+            args = (self.talk_plan, e["q"], kc, vc, self.talk, e["gate"], e["out"])
+            if plan is None or plan.rest:
+                K.talk_attention(*args, e.get("part"), b.block_tables, step.block_size, b.tok_seq,
+                                 b.ctx_len if plan is None else plan.actx, T, c.vdim, c.scale, st)
+            if plan is not None:
+                K.talk_prefill(*args, plan.xmap, plan.blocks, plan.nblocks, plan.waves, c.vdim, c.scale, st)
+            return
         if plan is None or plan.rest:
             ns = max(1, min(_SPLIT_CAP, _SPLIT_WG // (T * self.groups))) if self.mfma else 1
             K.gqa_attention(e["q"], kc, vc, e["gate"], e["out"], e["part"], b.block_tables, step.block_size, b.tok_seq,
@@ -630,6 +673,32 @@ class DensePart(_SharedPart):
         pass
 
 
+class PolyNormPart(_SharedPart):
+    """Dense feed-forward without a gate: down(a n(z) + b n(z^2) + c n(z^3) + e), z = up h, n an RMS norm over the token's values."""
+
+    def __init__(self, model, i, cfg, prefix, scale=1.0):
+        super().__init__(model, i, cfg, prefix, scale)
+        self.up = self.lin(self.mat("up", (cfg.ff, model.cfg.d_model)))
+        self.act = self.vecn("act", 4)
+        self.out_width = K.act_ld(cfg.ff)
+
+    def out_weight(self):
+        ff = self.cfg.ff
+        return torch.nn.functional.pad(self.mat("down", (self.m.cfg.d_model, ff)), (0, self.out_width - ff))
+
+    def bind(self, b, out, x):
+        z = self.scratch(b, "poly.z", b.pad, K.pad_to(self.cfg.ff, 8))
+        return dict(z=z, out=out, inputs=[K.Seg(self.up, x, z)])
+
+    def run(self, b, e, cache, state, step):
+        K.poly_norm(e["z"], self.act, e["out"], self.cfg.ff, step.T, self.m.cfg.eps, step.st)
+
+
+def dense_part(model, i, cfg, prefix, scale=1.0):
+    part = PolyNormPart if model.cfg.design.glu_act == "poly_norm" else DensePart
+    return part(model, i, cfg, prefix, scale)
+
+
 class OutputNormLayer:
     """x <- x + norm1(mixer(x)), then x <- x + norm2(feed-forward(x))."""
 
@@ -711,6 +780,58 @@ class SharedNormLayer:
                    slabs=n, slab_rows=b.slab_rows, **fin)
 
 
+class SandwichNormLayer:
+    """x <- x + norm1b(mixer(norm1(x))), then x <- x + norm2b(feed-forward(norm2(x))). The launch that adds a sublayer's output
+    (a product's slabs, or routed experts' rows) norms it, and the new residual for what comes next."""
+
+    def __init__(self, model: "StackModel", i: int, L):
+        p = f"l{i}."
+        self.m = model
+        if L.mixer.kind == "parallel":
+            raise NotImplementedError("mixers side by side between two norms")
+        self.parts = [PARTS[L.mixer.kind](model, i, L.mixer, p + "mix.")]
+        self.norm1, self.after = model.norm_weight(p + "norm1"), [model.norm_weight(p + "norm1b")]
+        self.norm_ff = None
+        if L.mlp is not None:
+            part = MoeFeedForward if L.mlp.kind == "moe" else PARTS[L.mlp.kind]
+            self.parts.append(part(model, i, L.mlp, p + "mlp."))
+            self.norm_ff = model.norm_weight(p + "norm2")
+            self.after.append(model.norm_weight(p + "norm2b"))
+        self.routed = [isinstance(q, MoeFeedForward) for q in self.parts]
+        self.o = [None if r else q.lin(q.out_weight()) for q, r in zip(self.parts, self.routed)]
+
+    def bind(self, b: StackBuffers, key):
+        halves = []
+        for q, routed, o in zip(self.parts, self.routed, self.o):
+            if routed:
+                halves.append((q.bind(b), None, None))
+                continue
+            x = q.scratch(b, "sandwich.out", b.pad, q.out_width)
+            e = q.bind(b, x, b.act)
+            halves.append((e, [K.LinLaunch(e["inputs"][j:j + K.SEGS]) for j in range(0, len(e["inputs"]), K.SEGS)],
+                           K.LinLaunch([K.Seg(o, x, self.m.slabs(b), slabs=_SLABS, slab_rows=b.slab_rows)])))
+        b.launches[key, "halves"] = halves
+
+    def new_caches(self, slots):
+        q = self.parts[0]
+        return q.new_cache(slots) if q.cache_width else None
+
+    def run(self, b, key, kc, state, step: "_Step", fin: dict):
+        cfg, T, st = self.m.cfg, step.T, step.st
+        for j, (q, (e, inputs, out)) in enumerate(zip(self.parts, b.launches[key, "halves"])):
+            if inputs is None:
+                q.run(b, e, step)
+                y = dict(y=e["ye"], plan=e["plan"], shared_row0=e["shared_row0"])
+            else:
+                for launch in inputs:
+                    launch.run(T, st)
+                q.run(b, e, kc.get(step.layer), state, step)
+                y = dict(y=self.m.slabs(b), slabs=out.run(T, st), slab_rows=b.slab_rows)
+            nxt = fin if j == len(self.parts) - 1 else dict(out_norm=self.norm_ff, out=b.h)
+            K.norm_add(w=self.after[j], x=b.x, xb=None, T=T, eps=cfg.eps, st=st, rms=cfg.design.norm == "rms", groups=cfg.norm_groups,
+                       **y, **nxt)
+
+
 def mixer_parts(c) -> list:
     """The parts of a mixer on a shared normed input: (config, tensor prefix, weight of the output)."""
     if c.kind == "parallel":
@@ -720,8 +841,18 @@ def mixer_parts(c) -> list:
 
 MIXERS = {"wkv": WkvMixer, "latent_attention": LatentMixer}
 FEED_FORWARDS = {"moe": MoeFeedForward}
-PARTS = {"attention": AttentionPart, "gla": GlaPart, "lightning": LightningPart, "channel_delta": DeltaPart, "dense": DensePart}
-LAYERS = {"output": OutputNormLayer, "shared": SharedNormLayer, "parallel": SharedNormLayer}
+PARTS = {"attention": AttentionPart, "gla": GlaPart, "lightning": LightningPart, "channel_delta": DeltaPart,
+         "dense": dense_part}
+LAYERS = {"output": OutputNormLayer, "shared": SharedNormLayer, "parallel": SharedNormLayer, "sandwich": SandwichNormLayer}
+
+
+def yarn(base: float, dims: int, s) -> tuple:
+    """(divisors of the rotation's frequencies, factor of sine and cosine) of a RotScaling."""
+    def pair(turns):                  # the (fractional) pair that turns so often over the original length
+        return dims * math.log(s.original / (2 * math.pi * turns)) / (2 * math.log(base))
+    lo, hi = max(math.floor(pair(s.fast)), 0), min(math.ceil(pair(s.slow)), dims - 1)
+    ramp = np.clip((np.arange(dims // 2) - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return 1.0 / (ramp / s.factor + (1.0 - ramp)), 0.1 * math.log(s.factor) + 1.0
 
 
 @dataclass
@@ -801,6 +932,10 @@ class StackModel:
         if cfg.max_positions:
             self.positions = self.table("pos", cfg.max_positions)
         if cfg.loop is not None:
+            self.loop_step = r.tensor("loop.step").to(device=dev, dtype=torch.float32).contiguous()
+            if tuple(self.loop_step.shape) != (cfg.loop.times, cfg.d_model):
+                raise ValueError(f"loop.step: shape {tuple(self.loop_step.shape)}, expected {(cfg.loop.times, cfg.d_model)}")
+        if cfg.loop is not None and cfg.design.loop_entry == "product":
             # operand [x | padding | embedding output | padding]
             d, w, ld = cfg.d_model, r.tensor("loop.in").to(dev), K.act_ld(cfg.d_model)
             if tuple(w.shape) != (d, 2 * d):
@@ -808,9 +943,6 @@ class StackModel:
             w = torch.cat([torch.nn.functional.pad(v, (0, ld - d)) for v in (w[:, :d], w[:, d:])], 1)
             self.loop_in = K.PackedLinear(w, self.f32, dev)
             self.weight_bytes += self.loop_in.nbytes
-            self.loop_step = r.tensor("loop.step").to(device=dev, dtype=torch.float32).contiguous()
-            if tuple(self.loop_step.shape) != (cfg.loop.times, d):
-                raise ValueError(f"loop.step: shape {tuple(self.loop_step.shape)}, expected {(cfg.loop.times, d)}")
         self.vocab_lo, self.vocab_hi = 0, cfg.vocab
 
     def table(self, name: str, rows: int) -> torch.Tensor:
@@ -839,10 +971,14 @@ class StackModel:
     def n_splits(self, T: int) -> int:
         return 1                      # (each attention layer sizes its own splits)
 
-    def rope(self, base: float, dims: int) -> torch.Tensor:
-        key = (base, dims)
+    def rope(self, base: float, dims: int, scaling=None) -> torch.Tensor:
+        key = (base, dims, None if scaling is None else astuple(scaling))
         if key not in self._rope:
-            self._rope[key] = rope_table(self.cfg.ctx, dims, base, self.device)
+            if scaling is None:
+                self._rope[key] = rope_table(self.cfg.ctx, dims, base, self.device)
+            else:
+                factors, gain = yarn(base, dims, scaling)
+                self._rope[key] = rope_table(self.cfg.ctx, dims, base, self.device, factors) * gain
         return self._rope[key]
 
     def kv_cache(self, num_blocks: int, block_size: int = 16):
@@ -870,7 +1006,7 @@ class StackModel:
         f = dict(dtype=torch.float32, device=dev)
         ld = K.act_ld(cfg.d_model)
         nl = min(pad, max(64, max_seqs, logit_rows or 0))
-        shared = cfg.design.norm_place in ("shared", "parallel")
+        shared = cfg.design.norm_place in ("shared", "parallel", "sandwich")
         act = lambda: torch.zeros(pad, ld, dtype=self.dtype, device=dev)      # noqa: E731
         b = StackBuffers(
             cap=cap, pad=pad, meta=meta, ids=seg[0], pos=seg[1], slot=seg[2], tok_seq=seg[3], ctx_len=seg[4],
@@ -976,8 +1112,9 @@ class StackModel:
         step = _Step(T, T if nruns is None else nruns, block_size, st)
         if row_info is not None and qblocks is not None:
             step.plan = self._expand_plan(b, qblocks, row_info, T, block_size, st)
-        rms = cfg.design.norm == "rms"
+        rms, groups = cfg.design.norm == "rms", cfg.norm_groups
         last = len(self.layers) - 1
+        steps = [None if t is None or self.loop_in is not None else self.loop_step[t] for t in self.passes]
         direct = logit_rows is None
         ld = K.act_ld(cfg.d_model)
         more = {}
@@ -988,32 +1125,38 @@ class StackModel:
             more["pairs"] = (self.pairs, bg.buckets, bg.mul_prev, bg.mul_cur, state["token"], b.runs, b.tok_seq)
         if self.positions is not None:
             more["positions"] = (self.positions, b.pos)
+        if steps[0] is not None:
+            more["add"] = steps[0]
         K.embed(b.ids, self.embed, b.x, b.xb, T, st, prev=(b.next_ids, b.use_prev) if feed_prev else None,
                 scale=cfg.embed_scale, **more)
-        if b.h is not None and self.passes[0] is None:
+        if b.h is not None and (self.passes[0] is None or steps[0] is not None):
             h = self._norms(b, 0)
-            K.row_norm(b.x, None, h["out_norm"], b.h, T, cfg.eps, st, rms=rms, w2=h.get("out_norm2"), out2=h.get("out2"))
+            K.row_norm(b.x, None, h["out_norm"], b.h, T, cfg.eps, st, rms=rms, w2=h.get("out_norm2"), out2=h.get("out2"),
+                       groups=groups)
         for i, layer in enumerate(self.layers):
-            if self.passes[i] is not None:
+            if self.passes[i] is not None and steps[i] is None:
                 n = b.launches["pass"].run(T, st)
                 K.norm_add(self.slabs(b), None, b.x, None, T, cfg.eps, st, rms=rms, slabs=n, slab_rows=b.slab_rows, keep=False,
                            add=self.loop_step[self.passes[i]], **self._norms(b, i))
             if i == last:
                 fin = dict(out_norm=self.final_norm, out=b.hn) if direct else {}
-            elif self.passes[i + 1] is not None:
+            elif self.passes[i + 1] is not None and steps[i + 1] is None:
                 fin = dict(copy=b.xx)
             else:
                 fin = self._norms(b, i + 1) if b.h is not None else {}
+                if steps[i + 1] is not None:
+                    fin["add"] = steps[i + 1]
             step.layer = i
             layer.run(b, self.owners[i], kc, state.get(i) if state else None, step, fin)
-            if taps is not None:
-                taps.append(b.x[:T, :cfg.d_model].clone())
+            if taps is not None:               # (without the next pass's step, which the layer's last launch adds)
+                x = b.x[:T, :cfg.d_model]
+                taps.append(x.clone() if i == last or steps[i + 1] is None else x - steps[i + 1])
         n = T
         if not direct:
             n = int(n_logits)
             if n == 0:
                 return 0
-            K.row_norm(b.x, logit_rows, self.final_norm, b.hn, n, cfg.eps, st, rms=rms)
+            K.row_norm(b.x, logit_rows, self.final_norm, b.hn, n, cfg.eps, st, rms=rms, groups=groups)
         if n > b.logits.shape[0]:
             raise ValueError(f"{n} logit rows, buffers hold {b.logits.shape[0]}")
         b.launches["head"].run(n, st)

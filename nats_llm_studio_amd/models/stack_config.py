@@ -24,19 +24,25 @@ class Design:
     norm_place: str = "output"         # output: x + norm(sublayer(x)), the sublayers read x itself
                                        # shared: h = norm(x), x + mixer(h) + feed-forward(h)
                                        # parallel: x + mixer(norm1(x)) + feed-forward(norm2(x))
+                                       # sandwich: x + norm1b(mixer(norm1(x))), then the same with norm2, norm2b
     mixers: tuple = ()
     feed_forwards: tuple = ()
-    rotary: str = "interleaved"        # pairs (2i, 2i + 1)
-    expert_act: str = "relu2"
-    router_score: str = "sigmoid"
+    rotary: str = "interleaved"        # pairs (2i, 2i + 1); halves: pairs (i, i + dims / 2)
+    expert_act: str = "relu2"          # down(relu(up)^2), or silu_glu: down(silu(gate) * up)
+    router_score: str = "sigmoid"      # or softmax, over all experts
+    router_group: str = "top2"         # score of a group of experts: the sum of its two best, or max
     glu_act: str = "gelu_tanh"         # dense feed-forward: down(act(gate) * up), or clamped_swiglu: both clamped by the
-                                       # config's limit, down(gate sigmoid(1.702 gate) (up + 1))
-    attn_qk_norm: str = "projection"   # attention: one RMS norm over all heads of the queries, one over the keys'; none
+                                       # config's limit, down(gate sigmoid(1.702 gate) (up + 1)); poly_norm: no gate,
+                                       # down(a n(z) + b n(z^2) + c n(z^3) + e) of z = up, n an RMS norm over the ff values
+    attn_qk_norm: str = "projection"   # attention: one RMS norm over all heads of the queries, one over the keys'; head: each
+                                       # rotated head on its own, without weights; none
     attn_values: str = "keys"          # attention: the values are the projected keys, unnormed and unrotated; projection
-    attn_gate: bool = True             # attention: a sigmoid gate per head
+    attn_gate: object = "head"         # attention: a sigmoid gate per head; column: per output column; None
+    attn_talk: bool = False            # attention: the heads' softmax weights are mixed by a matrix [heads, heads]
     attn_sink: bool = False            # attention: the softmax's denominator holds one more, a score of 0 without a value
     tied_head: bool = False            # the logits are products with the (unscaled) embedding table
     positions: bool = False            # a learned vector per position is added to the embedding
+    loop_entry: str = "product"        # looped layers, ahead of each pass: x = loop.in [x, embedding] + step; add: x + step
 
 
 DESIGNS = {
@@ -44,7 +50,11 @@ DESIGNS = {
     "Kolodra": Design(norm="rms", norm_one=True, norm_place="shared", mixers=("parallel",), feed_forwards=("dense",)),
     "Bibapel": Design(norm="rms", norm_place="parallel", mixers=("channel_delta", "attention", "lightning"),
                       feed_forwards=("dense",), glu_act="clamped_swiglu", attn_qk_norm="none", attn_values="projection",
-                      attn_gate=False, attn_sink=True, tied_head=True, positions=True),
+                      attn_gate=None, attn_sink=True, tied_head=True, positions=True),
+    "Pimodra": Design(norm="rms", norm_place="sandwich", mixers=("attention",), feed_forwards=("dense", "moe"), rotary="halves",
+                      expert_act="silu_glu", router_score="softmax", router_group="max", glu_act="poly_norm",
+                      attn_qk_norm="head", attn_values="projection", attn_gate="column", attn_talk=True, tied_head=True,
+                      loop_entry="add"),
 }
 
 
@@ -70,6 +80,16 @@ class LatentConfig:
 
 
 @dataclass
+class RotScaling:
+    """YaRN: wavelengths that turn at least `fast` times over the original length stay, those that turn at most `slow` times are
+    stretched by `factor`, with a ramp between them; sine and cosine grow by 0.1 ln(factor) + 1."""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass
 class AttentionConfig:
     """Grouped-query softmax attention, optionally with partial rotary positions, or over a sliding window and the first
     tokens: position i sees j <= i if i - j < window or j < keep_first."""
@@ -82,6 +102,7 @@ class AttentionConfig:
     vdim: int = 0                      # of values
     window: int = 0                    # 0: every earlier position is seen
     keep_first: int = 0
+    rot_scaling: Optional[RotScaling] = None
     kind, recurrent = "attention", False
 
 
@@ -185,6 +206,7 @@ class StackConfig:
     bigram: Optional[BigramConfig] = None
     loop: Optional[LoopConfig] = None
     max_positions: int = 0             # rows of the learned positions (0: none)
+    norm_groups: int = 1               # equal parts of the residual that the norms take each on its own
 
     @property
     def n_layer(self) -> int:
@@ -234,7 +256,9 @@ class StackConfig:
         out = cls(arch=arch, design=design, d_model=size(cfg, "width", "embed", 1), vocab=size(cfg, "vocab", "embed"),
                   eps=float(norm["eps"]), ctx=default_ctx(),
                   embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
-                  softcap=float(cfg.get("logit_softcap") or 0.0))
+                  softcap=float(cfg.get("logit_softcap") or 0.0), norm_groups=int(norm.get("groups", 1)))
+        if out.norm_groups < 1 or out.d_model % out.norm_groups or (out.norm_groups > 1 and design.norm != "rms"):
+            raise ValueError(f"config.json: {out.norm_groups} norm groups of {out.d_model} columns")
         if design.positions:
             out.max_positions = size(cfg, "max_positions", "pos")
             out.ctx = min(out.ctx, out.max_positions)
@@ -275,12 +299,18 @@ class StackConfig:
 
         def attention(i, m, p):
             own = design.attn_values == "projection"
-            H = int(m["heads"]) if not design.attn_gate else size(m, "heads", p + "g")
+            H = size(m, "heads", p + "g") if design.attn_gate == "head" else \
+                size(m, "heads", p + "talk") if design.attn_talk else int(m["heads"])
             D = size(m, "dim", p + "q", 0, H)
             G = size(m, "kv_heads", p + "k", 0, D)
             V = size(m, "vdim", p + "v", 0, G) if own else int(m.get("vdim", D))
             rot = m.get("rot") or {"dims": 0, "base": 1.0}
             rd = int(rot.get("dims", D))
+            sc = rot.get("scaling")
+            if sc is not None:
+                sc = RotScaling(*(float(sc[k]) for k in ("factor", "original", "fast", "slow")))
+                if min(sc.factor, sc.original, sc.fast, sc.slow) <= 0 or float(rot["base"]) <= 1:
+                    raise ValueError(f"layer {i}: rotation scaling {rot['scaling']} at base {rot['base']}")
             mask = m.get("mask") or {}
             window, keep = int(mask.get("size") or 0), int(mask.get("keep_first") or 0)
             if H % G:
@@ -291,8 +321,10 @@ class StackConfig:
                 raise ValueError(f"layer {i}: {rd} rotated dimensions of heads of {D}")
             if mask and (window < 1 or keep < 0):
                 raise ValueError(f"layer {i}: attention mask {mask}")
+            if design.attn_talk and (keep or design.attn_sink):
+                raise NotImplementedError(f"layer {i}: mixed heads with kept first tokens or a sink")
             return AttentionConfig(heads=H, kv_heads=G, dim=D, rot_dims=rd, rot_base=float(rot["base"]), scale=float(m["scale"]),
-                                   vdim=V, window=window, keep_first=keep)
+                                   vdim=V, window=window, keep_first=keep, rot_scaling=sc)
 
         def gla(i, m, p):
             V = size(m, "vdim", p + "norm")
@@ -333,7 +365,7 @@ class StackConfig:
             return mlp
 
         def dense(i, f, p):
-            return DenseConfig(ff=size(f, "ff", p + "gate"),
+            return DenseConfig(ff=size(f, "ff", p + "up"),
                                limit=float(f["limit"]) if design.glu_act == "clamped_swiglu" else 0.0)
 
         mixers = {"wkv": wkv, "latent_attention": latent, "parallel": parallel, "attention": attention,

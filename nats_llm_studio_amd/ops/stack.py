@@ -16,7 +16,7 @@ LIB_PATH = os.environ.get("NLS_STACK_SO") or os.path.join(_PKG, "_stack.so")
 P, I, L, F = ctypes.c_void_p, ctypes.c_int, ctypes.c_long, ctypes.c_float
 SEGS = 6
 EPI = {"none": 0, "silu": 1, "tanh": 2, "sigmoid": 3, "relu2": 4, "decay": 5, "gate": 6, "rope": 7,
-       "geglu": 8, "sigpow": 9, "softcap": 10, "swiglu": 11}
+       "geglu": 8, "sigpow": 9, "softcap": 10, "swiglu": 11, "siluglu": 12}
 NO_BLOCK = 1 << 30       # LinSeg.cb: output columns are not blocked
 
 
@@ -38,10 +38,14 @@ _SIGS = {
     "nls_lin_args_size": [],
     "nls_lin_small": [P, I, I, I, I, P],
     "nls_lin_gemm": [P, I, I, P],
-    "nls_stack_embed": [P, P, P, P, I, I, F, P, P, L, I, P, P, L, I, P, I, I, I, P, P, P, P, I, P, P],
-    "nls_norm_add": [P, L, P, I, L, P, P, L, P, L, P, P, P, P, L, P, I, I, I, F, I, I, I, L, P],
-    "nls_row_norm": [P, L, P, P, P, P, P, L, P, L, I, I, F, I, I, P],
-    "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, I, F, I, P],
+    "nls_stack_embed": [P, P, P, P, I, I, F, P, P, L, I, P, P, L, I, P, I, I, I, P, P, P, P, I, P, P, P],
+    "nls_norm_add": [P, L, P, I, L, P, P, L, P, L, P, P, P, P, L, P, I, I, I, F, I, I, I, I, L, P],
+    "nls_row_norm": [P, L, P, P, P, P, P, L, P, L, I, I, F, I, I, I, P],
+    "nls_poly_norm": [P, L, P, P, L, I, I, F, I, P],
+    "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, I, I, F, I, P],
+    "nls_talk_plain": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, I, P, P, L, P, L, I, P],
+    "nls_talk_decode": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, I, F, I, P, P, L, P, L, P, L, P, P, P, I, I, I, P],
+    "nls_talk_prefill": [P, L, P, P, P, P, I, I, I, I, I, I, F, I, P, P, L, P, L, P],
     "nls_gqa_attn": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, P, L, P, L, P, P, P, I, I, I, I, I, P],
     "nls_gqa_prefill": [P, L, P, P, P, P, I, P, I, P, L, I, I, I, I, F, I, I, I, P],
     "nls_delta_conv": [P, L, P, P, L, P, L, P, L, P, P, I, I, I, I, I, I, I, I, P],
@@ -51,7 +55,7 @@ _SIGS = {
     "nls_gla_step": [P, P, P, L, P, L, P, P, P, I, F, F, P, L, P, I, P, P, L, P, L, P, L, I, I, I, F, I, P],
     "nls_latent_rows": [P, L, I, P, P, L, P, L, I, I, I, P, P, P, P, P, L, I, F, I, P],
     "nls_stack_argmax": [P, L, I, P, I, P],
-    "nls_moe_plan": [P, L, I, I, I, I, I, F, P, P, I, P, P, P, I, P],
+    "nls_moe_plan": [P, L, I, I, I, I, I, I, I, F, P, P, I, P, P, P, I, P],
     "nls_shift_mix": [P, L, P, P, L, P, L, L, P, P, I, I, I, P],
     "nls_wkv_scan": [P, P, P, L, P, L, P, P, L, P, L, P, L, P, L, I, P, I, I, I, I, P],
     "nls_scan_out": [P, L, P, P, L, P, L, I, I, I, F, I, P],
@@ -137,7 +141,7 @@ class Seg:
     xgs / ygs: column step per group. block = (cb, cstep): output column n -> (n / cb) * cstep + n % cb.
     routed = (entry list, xdiv): the rows are routed entries (x row = entry / xdiv, y row = entry).
     rope = (table, pos, pairs). alpha: constant of the epilogue (sigmoid, sigpow, softcap, swiglu); sigpow: `gate`,
-    a vector, gives an exponent per column instead. geglu, swiglu: the rows of w alternate gate and up, y has half as many
+    a vector, gives an exponent per column instead. geglu, swiglu, siluglu: the rows of w alternate gate and up, y has half as many
     columns. slabs: K splits that launches of up to slab_rows rows may use; y holds that many slabs of slab_rows rows, added by
     the caller (LinLaunch.run returns how many were written)."""
 
@@ -294,10 +298,12 @@ class LinLaunch:
 
 class MoePlan:
     """Expert choice and routed-entry lists of one step (csrc/stack/stack_ops.hip moe_plan_kernel), shared by the layers
-    of a step. Scores: sigmoid of the router logits; the `keep` best of `groups` groups stay eligible; a chosen expert's
-    weight is score * scale."""
+    of a step. Scores: sigmoid of the router logits, or their softmax; the `keep` groups with the largest score (the sum of
+    their `group_best` best) of `groups` stay eligible; a chosen expert's weight is score * scale."""
 
-    def __init__(self, cap: int, experts: int, top: int, groups: int, keep: int, scale: float, device):
+    def __init__(self, cap: int, experts: int, top: int, groups: int, keep: int, scale: float, device, score: str = "sigmoid",
+                 group_best: int = 2):
+        self.softmax, self.group_best = {"sigmoid": 0, "softmax": 1}[score], group_best
         self.experts, self.top, self.groups, self.keep, self.scale = experts, top, groups, keep, scale
         i32 = dict(dtype=torch.int32, device=device)
         self.topw = torch.zeros(cap * top, dtype=torch.float32, device=device)
@@ -323,7 +329,7 @@ class MoePlan:
 
     def run(self, z: torch.Tensor, T: int, st: int):
         _check(lib().nls_moe_plan(z.data_ptr(), z.stride(0), T, self.experts, self.top, self.groups, self.keep,
-                                  self.scale, self.topw.data_ptr(), self.sel.data_ptr(), self.bm(T),
+                                  self.softmax, self.group_best, self.scale, self.topw.data_ptr(), self.sel.data_ptr(), self.bm(T),
                                   self.rows.data_ptr(), self.tiles.data_ptr(), self.ntiles.data_ptr(),
                                   self.max_tiles(T), st), "nls_moe_plan")
 
@@ -333,10 +339,10 @@ class MoePlan:
 # ---------------------------------------------------------------------------
 
 def embed(ids, table: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor], T: int, st: int, prev=None,
-          scale: float = 1.0, copies=(), pairs=None, positions=None):
+          scale: float = 1.0, copies=(), pairs=None, positions=None, add: Optional[torch.Tensor] = None):
     """x = table[id] * scale (xb: its bf16 rounding). copies: up to two more of x in the activation type, of one row stride.
     pairs = (table, buckets, mul_prev, mul_cur, previous token of each slot, runs, tok_seq): plus the row of the token pair, and
-    the slots' tokens move on. positions = (table, pos): plus the position's row."""
+    the slots' tokens move on. positions = (table, pos): plus the position's row. add: plus a vector."""
     nx, up = prev if prev is not None else (None, None)
     c0, c1 = (tuple(copies) + (None, None))[:2]
     pt, nb, mp, mc, pv, runs, seq = pairs if pairs is not None else (None, 0, 0, 0, None, None, None)
@@ -344,17 +350,18 @@ def embed(ids, table: torch.Tensor, x: torch.Tensor, xb: Optional[torch.Tensor],
     _check(lib().nls_stack_embed(ids.data_ptr(), _p(nx), _p(up), table.data_ptr(), table.shape[0], table.shape[1], scale,
                                  x.data_ptr(), _p(xb), x.stride(0), T, _p(c0), _p(c1), c0.stride(0) if c0 is not None else 0,
                                  int(c0 is not None and c0.dtype == torch.float32), _p(pt), nb, mp, mc, _p(pv), _p(runs), _p(seq),
-                                 _p(tab), tab.shape[0] if tab is not None else 0, _p(pos), st), "nls_stack_embed")
+                                 _p(tab), tab.shape[0] if tab is not None else 0, _p(pos), _p(add), st), "nls_stack_embed")
 
 
 def norm_add(y: torch.Tensor, w: Optional[torch.Tensor], x: torch.Tensor, xb: Optional[torch.Tensor], T: int, eps: float,
              st: int, plan: Optional[MoePlan] = None, shared_row0: int = -1, out_norm: Optional[torch.Tensor] = None,
              out: Optional[torch.Tensor] = None, rms: bool = False, slabs: int = 1, slab_rows: int = 0, out_norm2=None, out2=None,
-             keep: bool = True, add: Optional[torch.Tensor] = None):
+             keep: bool = True, add: Optional[torch.Tensor] = None, groups: int = 1):
     """x[:T] += norm(y) * w, or += y without w (xb: a copy in the activation type); y may be the sum of `slabs` blocks of
     slab_rows rows. With `plan`, y holds the routed experts' rows (token-major) and from row `shared_row0` on the shared
     expert's, combined first. out = norm(x) * out_norm (what the next sublayers read, or the model's last norm), out2 the same
-    with out_norm2. norm: layer norm, or RMS. keep False: x becomes y (+ the vector `add`)."""
+    with out_norm2. norm: layer norm, or RMS (of `groups` equal parts of a row each on its own). add: a vector that comes on top of
+    x; keep False: the old x is left out."""
     D = y.shape[1] if w is None else w.numel()
     typed = out if out is not None else xb
     if out2 is not None and out2.stride(0) != out.stride(0):
@@ -362,18 +369,27 @@ def norm_add(y: torch.Tensor, w: Optional[torch.Tensor], x: torch.Tensor, xb: Op
     _check(lib().nls_norm_add(y.data_ptr(), y.stride(0), _p(plan.topw) if plan else None, plan.top if plan else 0,
                               shared_row0, _p(w), x.data_ptr(), x.stride(0), _p(xb), xb.stride(0) if xb is not None else 0,
                               _p(out_norm), _p(out), _p(out_norm2), _p(out2), out.stride(0) if out is not None else 0, _p(add),
-                              int(keep), D, T, eps, int(typed is not None and typed.dtype == torch.float32), int(rms), slabs,
+                              int(keep), D, T, eps, int(typed is not None and typed.dtype == torch.float32), int(rms), groups, slabs,
                               slab_rows * y.stride(0), st), "nls_norm_add")
 
 
 def row_norm(x: torch.Tensor, rows: Optional[torch.Tensor], w: torch.Tensor, out: torch.Tensor, n: int, eps: float,
-             st: int, rms: bool = False, w2=None, out2=None, gate: Optional[torch.Tensor] = None):
-    """out[i] = norm(x[rows[i]]) * w (rows None: row i) (* gate[i]): layer norm, or RMS. out2: the same with w2."""
+             st: int, rms: bool = False, w2=None, out2=None, gate: Optional[torch.Tensor] = None, groups: int = 1):
+    """out[i] = norm(x[rows[i]]) * w (rows None: row i) (* gate[i]): layer norm, or RMS (of `groups` parts each on its own). out2: the
+    same with w2."""
     if (out2 is not None and out2.stride(0) != out.stride(0)) or (gate is not None and gate.dtype != out.dtype):
         raise ValueError("row_norm: equal row strides of the outputs, a gate of their type")
     _check(lib().nls_row_norm(x.data_ptr(), x.stride(0), _p(rows), w.data_ptr(), out.data_ptr(), _p(w2), _p(out2), out.stride(0),
                               _p(gate), gate.stride(0) if gate is not None else 0, w.numel(), n, eps,
-                              int(out.dtype == torch.float32), int(rms), st), "nls_row_norm")
+                              int(out.dtype == torch.float32), int(rms), groups, st), "nls_row_norm")
+
+
+def poly_norm(z: torch.Tensor, act: torch.Tensor, out: torch.Tensor, N: int, T: int, eps: float, st: int):
+    """out = a rms(z) + b rms(z^2) + c rms(z^3) + e over rows of N columns, powers by element; act: (a, b, c, e)."""
+    if z.dtype != out.dtype or act.numel() != 4 or N > min(z.stride(0), out.stride(0)):
+        raise ValueError("poly_norm: equal types, rows of N columns, four factors")
+    _check(lib().nls_poly_norm(z.data_ptr(), z.stride(0), act.data_ptr(), out.data_ptr(), out.stride(0), N, T, eps,
+                               int(out.dtype == torch.float32), st), "nls_poly_norm")
 
 
 def argmax(logits: torch.Tensor, n: int, out: torch.Tensor, st: int):
@@ -589,13 +605,14 @@ def attn_groups(H: int, G: int) -> int:
 
 
 def attn_rows(q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, T: int, H: int, G: int, D: int, Dp: int, rot: int, eps: float, st: int,
-              V: Optional[int] = None):
+              V: Optional[int] = None, head_norm: bool = False):
     """Norm over the whole q and k projections (qn, kn: weights or None), rotation of the first `rot` columns of each head (cs
-    None: none), queries to qo, keys and (as projected, V columns per head) values to the tokens' cache rows. q, k, v: f32
+    None: none), then (head_norm) an RMS norm of each head of queries and keys on its own; queries to qo, keys and (as projected, V columns per head) values to the tokens' cache rows. q, k, v: f32
     with one row stride."""
     _check(lib().nls_attn_rows(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), _p(qn), _p(kn), _p(cs),
                                pos.data_ptr(), slot.data_ptr(), qo.data_ptr(), qo.stride(0), kc.data_ptr(), vc.data_ptr(),
-                               kc.stride(0), T, H, G, D, D if V is None else V, Dp, rot, eps, int(qo.dtype == torch.float32), st),
+                               kc.stride(0), T, H, G, D, D if V is None else V, Dp, rot, int(head_norm), eps,
+                               int(qo.dtype == torch.float32), st),
            "nls_attn_rows")
 
 
@@ -621,3 +638,88 @@ def gqa_prefill(q, kc, vc, xmap, blocks, nblocks: int, waves: int, gate, out, H:
     _check(lib().nls_gqa_prefill(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), xmap.data_ptr(), blocks.data_ptr(),
                                  nblocks, _p(gate), gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), H, G,
                                  Dp, waves, scale, window, keep, int(sink), st), "nls_gqa_prefill")
+
+
+# ---------------------------------------------------------------------------
+# Attention with mixed heads
+# ---------------------------------------------------------------------------
+
+TALK_WIDTHS = (32, 64, 128)             # padded head widths of the prompt kernel, which takes up to 32 heads
+TALK_SCRATCH = 256 << 20                # bytes of scores that a decode launch may hold
+
+
+class TalkPlan:
+    """Kernels and scratch sizes of an attention whose heads' softmax weights are mixed, heads padded to Dp columns."""
+
+    def __init__(self, H: int, G: int, Dp: int, window: int, ctx: int, f32: bool, device):
+        self.H, self.G, self.Dp, self.window = H, G, Dp, window
+        self.mfma = not f32 and Dp in HEAD_WIDTHS and H <= 128
+        self.prefill = self.mfma and H <= 32 and Dp in TALK_WIDTHS
+        self.groups, self.hs = attn_groups(H, G), pad_to(H, 8)
+        self.ks = pad_to(min(window or ctx, ctx), 32) + 32              # keys of a row, from a multiple of 32 on
+        self.device = device
+
+    def matrix(self, talk: torch.Tensor) -> torch.Tensor:
+        """The [H, H] matrix as the kernels read it."""
+        if not self.mfma:
+            return talk.to(device=self.device, dtype=torch.float32).contiguous()
+        n = pad_to(self.H, 32) if self.H <= 64 else 128
+        out = torch.zeros(n, n, dtype=torch.bfloat16, device=self.device)
+        out[:self.H, :self.H] = talk.to(self.device)
+        return out
+
+    def rows(self, cap: int) -> int:
+        """Rows of a decode launch."""
+        return max(1, min(cap, TALK_SCRATCH // (4 * self.ks * self.hs)))
+
+    def splits(self, T: int):
+        """(splits of the scores, of the values, waves of a workgroup of the latter) at T rows."""
+        n = T * self.groups
+        ns1 = max(1, min(64, 2048 // n))
+        if n >= 1024 or self.Dp > 128:
+            return ns1, max(1, min(16, 1024 // n)), 1
+        return ns1, max(1, min(16, 512 // n)), 4
+
+    def scratch(self, cap: int):
+        """Element counts of (scores, score statistics, partial outputs, counters)."""
+        R = self.rows(cap)
+        part = max(T * self.splits(T)[1] for T in range(1, R + 1)) if R < 4096 else 16 * R
+        return (R * self.ks * self.hs, max(T * self.splits(T)[0] for T in range(1, R + 1)) * self.hs * 2, part * self.H * self.Dp,
+                R * self.groups)
+
+
+def talk_attention(plan: TalkPlan, q, kc, vc, talk, gate, out, scratch, block_tables, block_size: int, tok_seq, ctx_len, T: int,
+                   V: int, scale: float, st: int):
+    """Row-by-row attention with mixed heads (talk: TalkPlan.matrix); `gate`: a factor per output column, heads V columns apart."""
+    p = plan
+    ldg = gate.stride(0) if gate is not None else 0
+    if gate is not None and gate.dtype != out.dtype:
+        raise ValueError("talk_attention: a gate of the outputs' type")
+    if not p.mfma:
+        _check(lib().nls_talk_plain(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), block_tables.data_ptr(),
+                                    block_tables.stride(0), block_size, tok_seq.data_ptr(), ctx_len.data_ptr(), T, p.H, p.G, p.Dp, V,
+                                    scale, p.window, talk.data_ptr(), _p(gate), ldg, out.data_ptr(), out.stride(0),
+                                    int(q.dtype == torch.float32), st), "nls_talk_plain")
+        return
+    sc, ss, po, cnt = scratch
+    R = min(p.rows(T), sc.numel() // (p.ks * p.hs))
+    for t0 in range(0, T, R):
+        n = min(R, T - t0)
+        ns1, ns, waves = p.splits(n)
+        if (ss.numel() < n * ns1 * p.hs * 2 or cnt.numel() < n * p.groups or (ns > 1 and po.numel() < n * ns * p.H * p.Dp)):
+            raise ValueError("talk_attention: workspace too small")
+        _check(lib().nls_talk_decode(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), block_tables.data_ptr(),
+                                     block_tables.stride(0), block_size, tok_seq.data_ptr(), ctx_len.data_ptr(), t0, n, p.H, p.G,
+                                     p.Dp, V, scale, p.window, talk.data_ptr(), _p(gate), ldg, out.data_ptr(), out.stride(0),
+                                     sc.data_ptr(), p.ks, ss.data_ptr(), po.data_ptr(), cnt.data_ptr(), ns1, ns, waves, st),
+               "nls_talk_decode")
+
+
+def talk_prefill(plan: TalkPlan, q, kc, vc, talk, gate, out, xmap, blocks, nblocks: int, waves: int, V: int, scale: float, st: int):
+    """Attention with mixed heads of query blocks of up to 32 * waves tokens over their sequences' paged keys and values."""
+    p = plan
+    if not p.prefill or (gate is not None and gate.dtype != out.dtype):
+        raise ValueError("talk_prefill: a shape of the row-by-row kernels, or a gate of another type")
+    _check(lib().nls_talk_prefill(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), xmap.data_ptr(), blocks.data_ptr(),
+                                  nblocks, 2 * waves, p.H, p.G, p.Dp, V, scale, p.window, talk.data_ptr(), _p(gate),
+                                  gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), st), "nls_talk_prefill")
