@@ -72,10 +72,10 @@ def parse(argv=None):
     ap.add_argument("--stack", default=None, choices=("prefill", "decode", "all"),
                     help="instead of the headline workload: a config-driven stack design at sizes of real layers beside the "
                          "closest model of the GGUF families at equal size (nats_llm_studio_amd/bench_stack.py)")
-    ap.add_argument("--stack-design", default="sekolorn", choices=("sekolorn", "kolodra", "bibapel"),
+    ap.add_argument("--stack-design", default="sekolorn", choices=("sekolorn", "kolodra", "bibapel", "pimodra"),
                     help="with --stack: the design")
     ap.add_argument("--stack-sizes", default="2k,4k,4k-fine", help="with --stack: sizes to run")
-    ap.add_argument("--stack-only", default=None, choices=("sekolorn", "kolodra", "bibapel", "closest"),
+    ap.add_argument("--stack-only", default=None, choices=("sekolorn", "kolodra", "bibapel", "pimodra", "closest"),
                     help="with --stack: one of the two models")
     ap.add_argument("--stack-case", default=None, help="with --stack: one BATCHxPROMPT case")
     ap.add_argument("--step-breakdown", action="store_true",

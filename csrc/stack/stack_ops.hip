@@ -455,8 +455,10 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnRows p) {
   for (int e = threadIdx.x; e < p.G * p.V; e += 256) vo[(size_t)(e / p.V) * p.Dp + e % p.V] = (T)v[e];
 }
 
-// the same for heads of a multiple of 4 columns: the row's q and k stay in registers, NV groups of 4 columns per thread
-template <typename T, int NV, int NTH>
+// the same for heads of a multiple of 4 columns: the row's q and k stay in registers, NV groups of 4 columns per thread. HN (heads
+// of 4, 8, 16 .. 256 columns): no norm of the whole rows, but an RMS norm without weights of each rotated head on its own, whose
+// columns are lanes beside each other.
+template <typename T, int NV, int NTH, bool HN>
 __global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
   __shared__ float sh[2][NTH / 64];
   typedef T t4 __attribute__((ext_vector_type(4)));
@@ -470,24 +472,29 @@ __global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
     const int e = threadIdx.x + j * NTH;
     x[j] = f32x4{0.f, 0.f, 0.f, 0.f};
     if (e < n) x[j] = *reinterpret_cast<const f32x4*>(e < nq ? q + 4 * e : k + 4 * (e - nq));
+    if constexpr (HN) continue;
     const float s = (x[j][0] * x[j][0] + x[j][1] * x[j][1]) + (x[j][2] * x[j][2] + x[j][3] * x[j][3]);
     if (e < nq) sq += s;
     else sk += s;
   }
-  sq = wsum(sq);
-  sk = wsum(sk);
-  if ((threadIdx.x & 63) == 0) {
-    sh[0][threadIdx.x >> 6] = sq;
-    sh[1][threadIdx.x >> 6] = sk;
-  }
-  __syncthreads();
-  sq = sk = 0.f;
+  float iq = 1.f, ik = 1.f;
+  if constexpr (!HN) {
+    sq = wsum(sq);
+    sk = wsum(sk);
+    if ((threadIdx.x & 63) == 0) {
+      sh[0][threadIdx.x >> 6] = sq;
+      sh[1][threadIdx.x >> 6] = sk;
+    }
+    __syncthreads();
+    sq = sk = 0.f;
 #pragma unroll
-  for (int i = 0; i < NTH / 64; ++i) {
-    sq += sh[0][i];
-    sk += sh[1][i];
+    for (int i = 0; i < NTH / 64; ++i) {
+      sq += sh[0][i];
+      sk += sh[1][i];
+    }
+    iq = 1.f / sqrtf(sq / (float)(4 * nq) + p.eps);
+    ik = 1.f / sqrtf(sk / (float)(4 * (n - nq)) + p.eps);
   }
-  const float iq = 1.f / sqrtf(sq / (float)(4 * nq) + p.eps), ik = 1.f / sqrtf(sk / (float)(4 * (n - nq)) + p.eps);
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int e = threadIdx.x + j * NTH;
@@ -505,6 +512,11 @@ __global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
         y[u] = a * cc - b * ss;
         y[u + 1] = b * cc + a * ss;
       }
+    if constexpr (HN) {
+      float s = (y[0] * y[0] + y[1] * y[1]) + (y[2] * y[2] + y[3] * y[3]);
+      for (int m = D4 >> 1; m > 0; m >>= 1) s += __shfl_xor(s, m, 64);
+      y *= 1.f / sqrtf(s / (float)p.D + p.eps);
+    }
     const t4 o = {(T)y[0], (T)y[1], (T)y[2], (T)y[3]};
     if (isq) {
       *reinterpret_cast<t4*>((T*)p.qo + (size_t)t * p.ldqo + (size_t)h * p.Dp + c) = o;
@@ -630,22 +642,24 @@ int poly_norm_t(const void* z, long ldz, const float* act, void* out, long ldo, 
 
 template <typename T>
 int attn_rows_t(const AttnRows& p, int n, hipStream_t st) {
-  if (p.hnorm) {
-    hipLaunchKernelGGL(attn_head_rows_kernel<T>, dim3(n, (p.H + 2 * p.G + 3) / 4), dim3(256), 0, st, p);
-    return (int)hipGetLastError();
-  }
   const int cols = (p.H + p.G) * p.D;
   const bool vec = !((p.D | p.V) & 3) && !(p.ldq & 3) && !(p.Dp & 3) && !(p.ldqo & 3) && !(p.ldc & 3) &&
                    !(((uintptr_t)p.q | (uintptr_t)p.k | (uintptr_t)p.v) & 15);
+  const bool lanes = p.hnorm && p.D <= 256 && !(p.D & (p.D - 1));
 #define NLS_AR(NV, NTH) \
-  if (vec && cols <= 4 * NV * NTH) { \
-    hipLaunchKernelGGL((attn_rows4_kernel<T, NV, NTH>), dim3(n), dim3(NTH), 0, st, p); \
+  if (vec && (lanes || !p.hnorm) && cols <= 4 * NV * NTH) { \
+    if (lanes) hipLaunchKernelGGL((attn_rows4_kernel<T, NV, NTH, true>), dim3(n), dim3(NTH), 0, st, p); \
+    else hipLaunchKernelGGL((attn_rows4_kernel<T, NV, NTH, false>), dim3(n), dim3(NTH), 0, st, p); \
     return (int)hipGetLastError(); \
   }
   NLS_AR(1, 256)
   if (n <= 64) { NLS_AR(1, 1024) NLS_AR(2, 1024) }
   NLS_AR(2, 256) NLS_AR(5, 256) NLS_AR(8, 256) NLS_AR(8, 1024)
 #undef NLS_AR
+  if (p.hnorm) {
+    hipLaunchKernelGGL(attn_head_rows_kernel<T>, dim3(n, (p.H + 2 * p.G + 3) / 4), dim3(256), 0, st, p);
+    return (int)hipGetLastError();
+  }
   hipLaunchKernelGGL(attn_rows_kernel<T>, dim3(n), dim3(256), 0, st, p);
   return (int)hipGetLastError();
 }

@@ -9,6 +9,7 @@
 // exactly, and the sums are f32.
 #include "../kernels/lds_dma.h"
 #include "talk_plain.h"
+#include <type_traits>
 
 namespace nls_talk {
 using nls_dma::glds16;
@@ -26,34 +27,39 @@ DEVI f32x4 mma(const bf16x8& a, const bf16x8& b, const f32x4& c) { return __buil
 // byte offset of 16-byte chunk ch of row `row` in a tile of D-column bf16 rows, permuted against bank conflicts
 template <int D> DEVI int vswz(int row, int ch) {
   if constexpr (D == 128) return ch ^ (((row & 3) << 2) | ((row >> 2) & 3));
-  else return ch ^ (row & (D / 8 - 1));
+  else return ch ^ (row & (D == 256 ? 15 : D / 8 - 1));
 }
 template <int D> DEVI int voff(int row, int ch) { return row * (2 * D) + 16 * vswz<D>(row, ch); }
 
 // V^T fragment of columns 16 c .. 16 c + 15 from a 32-row tile: lane (g, r) gets column r of rows 4 g .. + 3 and 16 + 4 g .. + 3
-template <int D> DEVI bf16x8 vfrag(const uint8_t* vb, int c, int g, int r) {
-  const int qq = r >> 2, pp = r & 3, ch = 2 * c + (pp >> 1);
-  const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-      (__attribute__((address_space(3))) s16x4*)(vb + voff<D>(4 * g + qq, ch) + 8 * (pp & 1)));
-  const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-      (__attribute__((address_space(3))) s16x4*)(vb + voff<D>(16 + 4 * g + qq, ch) + 8 * (pp & 1)));
+// (at: vfrag_at(tile's LDS address); rows 16 apart are permuted alike, and tiles aligned to their rows, so the column is an xor)
+template <int D> DEVI uint32_t vfrag_at(uint32_t tile, int g, int r) {
+  const int qq = r >> 2, pp = r & 3;
+  return tile + voff<D>(4 * g + qq, pp >> 1) + 8 * (pp & 1);
+}
+template <int D> DEVI bf16x8 vfrag(uint32_t at, int c) {
+  typedef __attribute__((address_space(3))) s16x4* lp;
+  const uint32_t x = at ^ (32u * c);
+  const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lp)x);
+  const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lp)(x + 32 * D));
   return __builtin_bit_cast(bf16x8, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
 }
 
 // out[.. + 0 .. 3] = v * gate of columns d .. d + 3 of a head (V: its columns; the padding past them is not stored)
-DEVI void put_out(const TalkArgs& p, int t, int h, int d, const f32x4& v) {
+DEVI bool by_four(const TalkArgs& p) { return !((p.V | p.ldg) & 3); }
+template <bool FOUR> DEVI void put_out(const TalkArgs& p, int t, int h, int d, const f32x4& v) {
   const __bf16* ga = p.gate ? (const __bf16*)p.gate + (size_t)t * p.ldg + (size_t)h * p.V + d : nullptr;
   __bf16* y = (__bf16*)p.out + (size_t)t * p.ldo + (size_t)h * p.Dp + d;
-  if (!((p.V | p.ldg) & 3)) {
+  if constexpr (FOUR) {
     if (d >= p.V) return;
     const bf4 g4 = ga ? *reinterpret_cast<const bf4*>(ga) : bf4{(__bf16)1.f, (__bf16)1.f, (__bf16)1.f, (__bf16)1.f};
     *reinterpret_cast<bf4*>(y) = bf4{(__bf16)(v[0] * (float)g4[0]), (__bf16)(v[1] * (float)g4[1]), (__bf16)(v[2] * (float)g4[2]),
                                      (__bf16)(v[3] * (float)g4[3])};
-    return;
-  }
+  } else {
 #pragma unroll
-  for (int e = 0; e < 4; ++e)
-    if (d + e < p.V) y[e] = (__bf16)(v[e] * (ga ? (float)ga[e] : 1.f));
+    for (int e = 0; e < 4; ++e)
+      if (d + e < p.V) y[e] = (__bf16)(v[e] * (ga ? (float)ga[e] : 1.f));
+  }
 }
 
 // ---------------------------------------------------------------------------------------------------------------------
@@ -161,7 +167,7 @@ template <int D, int KK, int W>
 __global__ __launch_bounds__(64 * W) void talk_value_kernel(Decode p) {
   constexpr int NDT = D / 16, LPR = D / 8, RPI = 64 / LPR, NVL = KG / RPI;
   constexpr int HP = 32 * KK, VB = KG * D * 2, RB = W > 1 ? W * 16 * D * 4 : 0;
-  __shared__ __attribute__((aligned(16))) uint8_t smem[W * VB > RB ? W * VB : RB];
+  __shared__ __attribute__((aligned(512))) uint8_t smem[W * VB > RB ? W * VB : RB];
   __shared__ float lse[HP];
   __shared__ int last;
   const TalkArgs& a = p.a;
@@ -225,6 +231,7 @@ __global__ __launch_bounds__(64 * W) void talk_value_kernel(Decode p) {
   }
   __syncthreads();
   uint8_t* vs = smem + wave * VB;
+  const uint32_t vat = vfrag_at<D>(lds_addr(vs), g, r);
   auto store_v = [&](u32x4 (&V)[NVL]) __attribute__((always_inline)) {
 #pragma unroll
     for (int i = 0; i < NVL; ++i) *reinterpret_cast<u32x4*>(vs + voff<D>(RPI * i + lane / LPR, lane % LPR)) = V[i];
@@ -264,7 +271,7 @@ __global__ __launch_bounds__(64 * W) void talk_value_kernel(Decode p) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) pb[4 * nt + i] = (__bf16)mx[nt][i];
 #pragma unroll
-    for (int c = 0; c < NDT; ++c) o[c] = mma(vfrag<D>(vs, c, g, r), pb, o[c]);
+    for (int c = 0; c < NDT; ++c) o[c] = mma(vfrag<D>(vat, c), pb, o[c]);
     if (j + W < tb) {
       store_v(vn);
 #pragma unroll
@@ -278,7 +285,10 @@ __global__ __launch_bounds__(64 * W) void talk_value_kernel(Decode p) {
   }
   // lane (g, r): columns 16 c + 4 g + i of head r
   auto finish = [&](int h, int d, const f32x4& v) {                 // head of the workgroup, column
-    if (na == 1) put_out(a, t, h0 + h, d, v);
+    if (na == 1) {
+      if (by_four(a)) put_out<true>(a, t, h0 + h, d, v);
+      else put_out<false>(a, t, h0 + h, d, v);
+    }
     else *reinterpret_cast<f32x4*>(p.part + (((size_t)tr * a.H + h0 + h) * p.ns + split) * D + d) = v;
   };
   if constexpr (W > 1) {
@@ -322,7 +332,8 @@ __global__ __launch_bounds__(64 * W) void talk_value_kernel(Decode p) {
     f32x4 v = *reinterpret_cast<const f32x4*>(s);
 #pragma unroll 8
     for (int i = 1; i < na; ++i) v += *reinterpret_cast<const f32x4*>(s + (size_t)i * D);
-    put_out(a, t, h0 + h, d, v);
+    if (by_four(a)) put_out<true>(a, t, h0 + h, d, v);
+    else put_out<false>(a, t, h0 + h, d, v);
   }
 }
 
@@ -346,34 +357,48 @@ struct Prefill {
   TalkArgs a;
   const int* xmap;        // cache slot of every context row
   const int* blocks;      // [n][8]: (first row, rows, sequence, first position, xoff, -, -, -)
-  int nsub;               // workgroups of 16 tokens per block
+  int nblocks, nsub;      // blocks; workgroups of 16 tokens of each
 };
 
-// Eight waves of HW heads each, 16 tokens. Weights of a 32-key tile in LDS, [token][key][head] as two bf16 planes; wave w mixes
-// tokens 2 w and 2 w + 1 (rows: keys, columns: heads) and leaves the mixed weights, [token][head][key], where that token's first
-// plane was; then each wave multiplies its own heads with the values, whose tile it has fetched by LDS-DMA for itself.
-constexpr int PKS = 80, PTS = 32 * PKS + 16, PPL = 16 * PTS;     // bytes: key (head) row, token, plane
+// Eight waves of HW heads each, 16 tokens. Weights of a 32-key tile in LDS, [token][key][head][two bf16 parts]; wave w mixes
+// tokens 2 w and 2 w + 1 (rows: keys, columns: heads) and leaves the mixed weights, [token][head][key], in that token's space;
+// then each wave multiplies its own heads with the values, whose tile it has fetched by LDS-DMA for itself. Slots are read
+// two tiles ahead, keys one, values while the weights are mixed.
+constexpr int PKS = 144, PTS = 32 * PKS + 16, PW = 16 * PTS, PHS = 80;     // bytes: key row, token, all; row of a mixed head
+// behind the value tiles what the registers do not hold through the second walk: the matrix, the denominators, and at the largest
+// size some of the last head's queries
+template <int D, int HW> struct PL {
+  static constexpr int V = PW, T = V + 8 * KG * D * 2, L = T + 2048, Q = L + 2048, NQ = D == 128 && HW == 4 ? 2 : 0;
+  static constexpr int BYTES = Q + 8 * NQ * 1024;
+  static_assert(BYTES <= 160 * 1024, "LDS");
+};
 
-template <int D, int HW>
+// ONE: a wave's heads share a key head
+template <int D, int HW, bool ONE>
 __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
   constexpr int NKK = D / 32, NDT = D / 16, LPR = D / 8, RPI = 64 / LPR, NVL = KG / RPI, VB = KG * D * 2;
-  extern __shared__ __attribute__((aligned(16))) uint8_t lds[];      // [hi plane | lo plane | a value tile per wave]
+  typedef PL<D, HW> P;
+  extern __shared__ __attribute__((aligned(16))) uint8_t lds[];      // [weights | a value tile per wave | PL]
   const TalkArgs& a = p.a;
-  const int* blk = p.blocks + 8 * (blockIdx.x / p.nsub);
-  const int row0 = 16 * (p.nsub - 1 - blockIdx.x % p.nsub), n = min(16, blk[1] - row0);      // (later rows see more keys)
+  // a block's workgroups share most of their keys: they run on one XCD
+  const int unit = blockIdx.x >> 3, bi = unit / p.nsub * 8 + (blockIdx.x & 7);
+  if (bi >= p.nblocks) return;
+  const int* blk = p.blocks + 8 * bi;
+  const int row0 = 16 * (p.nsub - 1 - unit % p.nsub), n = min(16, blk[1] - row0);      // (later rows see more keys)
   if (n <= 0) return;
   const int t0 = blk[0] + row0, pos0 = blk[3] + row0, last = pos0 + n - 1;
   const int* xmap = p.xmap + blk[4];
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, r = lane & 15;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int hb = wave * HW, nh = min(HW, a.H - hb), gq = a.H / a.G;               // (nh <= 0: a wave without heads)
-  const bool one = nh > 0 && hb / gq == (hb + nh - 1) / gq;                       // its heads share a key head
+  const int hb = wave * HW, nh = min(HW, a.H - hb), gq = a.H / a.G;
+  // heads past nh (a wave may have none): queries of zeros, columns that the matrix leaves out, nothing stored. They run along: where
+  // paths with and without loads meet, the counted waits would become waits for everything.
   const int tok = t0 + min(r, n - 1), qpos = pos0 + min(r, n - 1);
   const int window = a.window > 0 ? a.window : 1 << 30;
-  const size_t ldkv = (size_t)a.G * D;
+  const uint32_t ldkv = (uint32_t)a.G * D;          // (slots and strides of 32 bits: one multiplication)
   const float sl2 = a.scale * LOG2E;
   const __bf16 *kc = (const __bf16*)a.k + 8 * g, *vc = (const __bf16*)a.v;
-  for (int i = tid; i < 2 * PPL / 16; i += 512) reinterpret_cast<u32x4*>(lds)[i] = u32x4{0u, 0u, 0u, 0u};
+  for (int i = tid; i < PW / 16; i += 512) reinterpret_cast<u32x4*>(lds)[i] = u32x4{0u, 0u, 0u, 0u};
 
   bf16x8 qf[HW][NKK];
 #pragma unroll
@@ -382,16 +407,16 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     for (int kk = 0; kk < NKK; ++kk)
       qf[i][kk] = i < nh ? *reinterpret_cast<const bf16x8*>((const __bf16*)a.q + (size_t)tok * a.ldq + (size_t)(hb + i) * D + 32 * kk + 8 * g)
                          : bf16x8{};
-  bf16x8 tf[2];
-#pragma unroll
-  for (int u = 0; u < 2; ++u) tf[u] = *reinterpret_cast<const bf16x8*>((const __bf16*)a.talk + (16 * u + r) * 32 + 8 * g);
 
   const int first = max(0, pos0 - window + 1) / KG, end = last / KG + 1;
   auto slots = [&](int t) { return xmap[min(t * KG + (lane & 31), last)]; };      // lane: slot of key lane % 32
   auto load_k = [&](int sl, int nt, int kh, u32x4 (&K)[NKK]) __attribute__((always_inline)) {
-    const __bf16* s = kc + (size_t)__shfl(sl, 16 * nt + r, 64) * ldkv + (size_t)kh * D;
+    const __bf16* s = kc + (uint64_t)(uint32_t)__shfl(sl, 16 * nt + r, 64) * ldkv + (size_t)kh * D;
 #pragma unroll
-    for (int kk = 0; kk < NKK; ++kk) K[kk] = ld16(s + 32 * kk);
+    for (int kk = 0; kk < NKK; ++kk) {
+      K[kk] = ld16(s + 32 * kk);
+      __builtin_amdgcn_sched_barrier(0);            // (in the order of their use, also ahead of the loops: the waits are counted)
+    }
   };
   auto score = [&](const u32x4 (&K)[NKK], const bf16x8 (&q)[NKK]) __attribute__((always_inline)) {
     f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
@@ -399,11 +424,13 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     for (int kk = 0; kk < NKK; ++kk) s = mma(__builtin_bit_cast(bf16x8, K[kk]), q[kk], s);
     return s;
   };
-  auto hide = [&](int k, float s) { return k <= qpos && k > qpos - window ? s : -INFINITY; };
+  // A tile that some token does not see whole is an edge; its body is another copy of the code, and selects without branches (a branch
+  // between a product and the first use of its result has been compiled without the wait that the matrix pipeline needs).
+  auto is_edge = [&](int t) { return t * KG + KG - 1 > pos0 || t * KG <= last - window; };
+  auto sees = [&](int k) { return (k <= qpos) & (k > qpos - window); };
   const int kh0 = min(hb / gq, a.G - 1);
 
   // ---- first walk: each head's log2 of the softmax's denominator (lane: token r, its own keys; joined at the end)
-  float lse[HW];
   {
     float m[HW], l[HW];
 #pragma unroll
@@ -411,49 +438,54 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
       m[i] = -1e30f;
       l[i] = 0.f;
     }
-    if (nh > 0) {
-      int sl = slots(first);
+    {
+      int sl = slots(first), s1 = slots(min(first + 1, end - 1));
+      asm volatile("" : "+v"(s1));
       u32x4 kf[2][NKK];
       load_k(sl, 0, kh0, kf[0]);
       load_k(sl, 1, kh0, kf[1]);
       for (int t = first; t < end; ++t) {
-        const bool edge = t * KG + KG - 1 > pos0 || t * KG <= last - window;
-        const int nx = slots(min(t + 1, end - 1));
-        u32x4 kn[2][NKK];
-        load_k(nx, 0, kh0, kn[0]);
-        load_k(nx, 1, kh0, kn[1]);
+        int s2 = slots(min(t + 2, end - 1));
+        __builtin_amdgcn_sched_barrier(0);
+        f32x4 s[HW][2];
 #pragma unroll
         for (int i = 0; i < HW; ++i) {
-          if (i >= nh) break;
-          if (!one && i > 0 && (hb + i) % gq == 0) {
+          if (!ONE && i > 0 && i < nh && (hb + i) % gq == 0) {
             load_k(sl, 0, (hb + i) / gq, kf[0]);
             load_k(sl, 1, (hb + i) / gq, kf[1]);
           }
-          f32x4 s[2] = {score(kf[0], qf[i]), score(kf[1], qf[i])};
-          if (edge) {
+#pragma unroll
+          for (int nt = 0; nt < 2; ++nt) s[i][nt] = score(kf[nt], qf[i]);
+        }
+        __builtin_amdgcn_sched_barrier(0);
+        asm volatile("" : "+v"(s2));                // (the next slots are waited for ahead of the next keys' loads, not behind them)
+        load_k(s1, 0, kh0, kf[0]);
+        load_k(s1, 1, kh0, kf[1]);
+        auto sum = [&](auto edge) __attribute__((always_inline)) {
+#pragma unroll
+          for (int i = 0; i < HW; ++i) {
+            float mn = m[i];                        // (of the scores as they are: sl2 >= 0)
 #pragma unroll
             for (int nt = 0; nt < 2; ++nt)
 #pragma unroll
-              for (int e = 0; e < 4; ++e) s[nt][e] = hide(t * KG + 16 * nt + 4 * g + e, s[nt][e]);
+              for (int e = 0; e < 4; ++e) {
+                if constexpr (decltype(edge)::value) s[i][nt][e] = sees(t * KG + 16 * nt + 4 * g + e) ? s[i][nt][e] : -INFINITY;
+                mn = fmaxf(mn, s[i][nt][e]);
+              }
+            const float nb = -mn * sl2;
+            float l2 = l[i] * __builtin_amdgcn_exp2f((m[i] - mn) * sl2);
+#pragma unroll
+            for (int nt = 0; nt < 2; ++nt)
+#pragma unroll
+              for (int e = 0; e < 4; ++e) l2 += __builtin_amdgcn_exp2f(fmaf(s[i][nt][e], sl2, nb));
+            l[i] = l2;
+            m[i] = mn;
           }
-          float mn = m[i];
-#pragma unroll
-          for (int nt = 0; nt < 2; ++nt)
-#pragma unroll
-            for (int e = 0; e < 4; ++e) mn = fmaxf(mn, s[nt][e] * sl2);
-          float sum = l[i] * __builtin_amdgcn_exp2f(m[i] - mn);
-#pragma unroll
-          for (int nt = 0; nt < 2; ++nt)
-#pragma unroll
-            for (int e = 0; e < 4; ++e) sum += __builtin_amdgcn_exp2f(fmaf(s[nt][e], sl2, -mn));
-          l[i] = sum;
-          m[i] = mn;
-        }
-        sl = nx;
-#pragma unroll
-        for (int nt = 0; nt < 2; ++nt)
-#pragma unroll
-          for (int kk = 0; kk < NKK; ++kk) kf[nt][kk] = kn[nt][kk];
+        };
+        if (is_edge(t)) sum(std::true_type{});
+        else sum(std::false_type{});
+        sl = s1;
+        s1 = s2;
       }
     }
 #pragma unroll
@@ -461,27 +493,40 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
 #pragma unroll
       for (int o = 16; o <= 32; o <<= 1) {
         const float mo = __shfl_xor(m[i], o, 64), lo = __shfl_xor(l[i], o, 64), M = fmaxf(m[i], mo);
-        l[i] = l[i] * __builtin_amdgcn_exp2f(m[i] - M) + lo * __builtin_amdgcn_exp2f(mo - M);
+        l[i] = l[i] * __builtin_amdgcn_exp2f((m[i] - M) * sl2) + lo * __builtin_amdgcn_exp2f((mo - M) * sl2);
         m[i] = M;
       }
-      lse[i] = m[i] + __builtin_amdgcn_logf(l[i]);
+      if (g == 0) reinterpret_cast<float*>(lds + P::L)[(hb + i) * 16 + r] = m[i] * sl2 + __builtin_amdgcn_logf(l[i]);
     }
   }
 
   // ---- second walk
+  bf4* tl = reinterpret_cast<bf4*>(lds + P::T) + lane;      // [4][64]: rows 16 u + r, columns 16 v + 4 g ..
+  if (wave < 4) tl[64 * wave] = *reinterpret_cast<const bf4*>((const __bf16*)a.talk + (16 * (wave >> 1) + r) * 32 + 16 * (wave & 1) + 4 * g);
+  bf16x8* ql = reinterpret_cast<bf16x8*>(lds + P::Q + wave * P::NQ * 1024) + lane;
+#pragma unroll
+  for (int j = 0; j < P::NQ; ++j) ql[64 * j] = qf[HW - 1][NKK - P::NQ + j];
   f32x4 o[HW][NDT];
 #pragma unroll
   for (int i = 0; i < HW; ++i)
 #pragma unroll
     for (int c = 0; c < NDT; ++c) o[i][c] = f32x4{0.f, 0.f, 0.f, 0.f};
-  const uint32_t vdst = __builtin_amdgcn_readfirstlane(lds_addr(lds)) + 2 * PPL + wave * VB;
-  const uint8_t* vs = lds + 2 * PPL + wave * VB;
+  const uint32_t vdst = __builtin_amdgcn_readfirstlane(lds_addr(lds)) + P::V + wave * VB;
+  // the lane's number anew: what follows from it need not live through the loop
+  auto again = [](int v) __attribute__((always_inline)) {
+    asm volatile("" : "+v"(v));
+    return v;
+  };
   auto fetch_v = [&](int sl, int kh) __attribute__((always_inline)) {
+    const int ln = again(lane);
+    int rs[NVL];
 #pragma unroll
-    for (int i = 0; i < NVL; ++i) {
-      const int row = RPI * i + lane / LPR;
-      glds16(vc + (size_t)__shfl(sl, row, 64) * ldkv + (size_t)kh * D + 8 * vswz<D>(row, lane % LPR), vdst + 1024 * i);
-    }
+    for (int i = 0; i < NVL; ++i) rs[i] = __shfl(sl, RPI * i + ln / LPR, 64);
+#pragma unroll
+    for (int i = 0; i < NVL; ++i) asm volatile("" : "+v"(rs[i]));               // (all of them in flight together)
+#pragma unroll
+    for (int i = 0; i < NVL; ++i)
+      glds16(vc + (uint64_t)(uint32_t)rs[i] * ldkv + (size_t)kh * D + 8 * vswz<D>(RPI * i + ln / LPR, ln % LPR), vdst + 1024 * i);
   };
   auto barrier = [&]() __attribute__((always_inline)) {
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -489,131 +534,154 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     asm volatile("" ::: "memory");
   };
   __syncthreads();
-  int sl = slots(first);
+  int sl = slots(first), s1 = slots(min(first + 1, end - 1));
+  asm volatile("" : "+v"(s1));                      // (waited for ahead of the keys: see below)
   u32x4 kf[2][NKK];
-  if (nh > 0) {
-    load_k(sl, 0, kh0, kf[0]);
-    load_k(sl, 1, kh0, kf[1]);
-  }
-  for (int t = first; t < end; ++t) {
-    const bool edge = t * KG + KG - 1 > pos0 || t * KG <= last - window;
-    const int nx = slots(min(t + 1, end - 1));
-    if (nh > 0) {
-      fetch_v(sl, kh0);
+  load_k(sl, 0, kh0, kf[0]);
+  load_k(sl, 1, kh0, kf[1]);
+  auto weigh = [&](auto edge, int t) __attribute__((always_inline)) {
+    const int ln = again(lane), g = ln >> 4, r = ln & 15;
+    const float* ll = reinterpret_cast<const float*>(lds + P::L) + hb * 16 + r;
+    const bf16x8* ql = reinterpret_cast<const bf16x8*>(lds + P::Q + wave * P::NQ * 1024) + ln;
+    auto product = [&](int u) __attribute__((always_inline)) {                  // keys 16 nt .., head i
+      const int nt = u / HW, i = u % HW;
+      if (!ONE && i > 0 && i < nh && (hb + i) % gq == 0) load_k(sl, nt, (hb + i) / gq, kf[nt]);
+      if (P::NQ && i == HW - 1) {
 #pragma unroll
-      for (int nt = 0; nt < 2; ++nt) {
-        __bf16 hi[4][HW], lo[4][HW];
-#pragma unroll
-        for (int i = 0; i < HW; ++i) {
-          if (!one && i > 0 && i < nh && (hb + i) % gq == 0) load_k(sl, nt, (hb + i) / gq, kf[nt]);
-          f32x4 s = score(kf[nt], qf[i]);
-#pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            if (edge) s[e] = hide(t * KG + 16 * nt + 4 * g + e, s[e]);
-            const float w = i < nh ? __builtin_amdgcn_exp2f(fmaf(s[e], sl2, -lse[i])) : 0.f;
-            hi[e][i] = (__bf16)w;
-            lo[e][i] = (__bf16)(w - (float)hi[e][i]);
-          }
-        }
-        load_k(nx, nt, kh0, kf[nt]);
-        typedef __bf16 bfw __attribute__((ext_vector_type(HW)));
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          bfw a1, a2;
-#pragma unroll
-          for (int i = 0; i < HW; ++i) {
-            if constexpr (HW == 1) {
-              a1 = hi[e][i];
-              a2 = lo[e][i];
-            } else {
-              a1[i] = hi[e][i];
-              a2[i] = lo[e][i];
-            }
-          }
-          uint8_t* d = lds + r * PTS + (16 * nt + 4 * g + e) * PKS + hb * 2;
-          *reinterpret_cast<bfw*>(d) = a1;
-          *reinterpret_cast<bfw*>(d + PPL) = a2;
-        }
+        for (int j = 0; j < P::NQ; ++j) qf[i][NKK - P::NQ + j] = ql[64 * j];
       }
+      return score(kf[nt], qf[i]);
+    };
+    f32x4 s = product(0);
+    float lse = ll[0];
+    uint32_t held[4];
+#pragma unroll
+    for (int u = 0; u < 2 * HW; ++u) {                                          // a product is on its way while the last one's weights are made
+      const int nt = u / HW, i = u % HW;
+      f32x4 sn = s;
+      if (u + 1 < 2 * HW) sn = product(u + 1);
+      const float lsen = ll[16 * ((u + 1) % HW)];
+      constexpr int PAIR = HW > 1 ? 2 : 1;          // heads per store
+      uint8_t* d = lds + r * PTS + (16 * nt + 4 * g) * PKS + (hb + i / PAIR * PAIR) * 4;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        if constexpr (decltype(edge)::value) s[e] = sees(t * KG + 16 * nt + 4 * g + e) ? s[e] : -INFINITY;
+        const float w = __builtin_amdgcn_exp2f(fmaf(s[e], sl2, -lse));
+        // the upper half of w, and of what that leaves: 16 bits of it
+        const uint32_t up = __builtin_bit_cast(uint32_t, w) & 0xffff0000u;
+        const uint32_t low = __builtin_bit_cast(uint32_t, w - __builtin_bit_cast(float, up));
+        const uint32_t both = __builtin_amdgcn_perm(low, up, 0x07060302);
+        if constexpr (PAIR == 1) *reinterpret_cast<uint32_t*>(d + e * PKS) = both;
+        else if (i & 1) *reinterpret_cast<uint2*>(d + e * PKS) = uint2{held[e], both};
+        else held[e] = both;
+      }
+      s = sn;
+      lse = lsen;
+      __builtin_amdgcn_sched_barrier(0);            // (heads one by one: registers)
     }
+  };
+  for (int t = first; t < end; ++t) {
+    int s2 = slots(min(t + 2, end - 1));
+    __builtin_amdgcn_sched_barrier(0);
+    if (is_edge(t)) weigh(std::true_type{}, t);
+    else weigh(std::false_type{}, t);
+    fetch_v(sl, kh0);
     barrier();
+    const int ln = again(lane), g = ln >> 4, r = ln & 15;
+    bf4 tf[2][2];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) tf[u >> 1][u & 1] = reinterpret_cast<const bf4*>(lds + P::T)[64 * u + ln];
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
       uint8_t* tw = lds + (2 * wave + u) * PTS;
-      bf16x8 w[2][2];
+      bf16x8 w[2][2];                              // keys 16 nt + r, both parts of heads 16 v + 4 g ..
 #pragma unroll
       for (int nt = 0; nt < 2; ++nt)
 #pragma unroll
-        for (int pl = 0; pl < 2; ++pl)
-          w[nt][pl] = *reinterpret_cast<const bf16x8*>(tw + pl * PPL + (16 * nt + r) * PKS + 16 * g);
+        for (int v = 0; v < 2; ++v)
+          w[nt][v] = *reinterpret_cast<const bf16x8*>(tw + (16 * nt + r) * PKS + 64 * v + 16 * g);
 #pragma unroll
       for (int ht = 0; ht < 2; ++ht) {
-        if (16 * ht >= a.H) break;
         bf16x8 pb;
 #pragma unroll
         for (int nt = 0; nt < 2; ++nt) {
           f32x4 mx = f32x4{0.f, 0.f, 0.f, 0.f};
-          mx = mma(w[nt][0], tf[ht], mx);
-          mx = mma(w[nt][1], tf[ht], mx);
+#pragma unroll
+          for (int v = 0; v < 2; ++v) mx = mma(w[nt][v], __builtin_shufflevector(tf[ht][v], tf[ht][v], 0, 0, 1, 1, 2, 2, 3, 3), mx);
 #pragma unroll
           for (int e = 0; e < 4; ++e) pb[4 * nt + e] = (__bf16)mx[e];
         }
-        *reinterpret_cast<bf16x8*>(tw + (16 * ht + r) * PKS + 16 * g) = pb;      // keys 4 g .., 16 + 4 g .. of head 16 ht + r
+        *reinterpret_cast<bf16x8*>(tw + (16 * ht + r) * PHS + 16 * g) = pb;      // keys 4 g .., 16 + 4 g .. of head 16 ht + r
       }
+      __builtin_amdgcn_sched_barrier(0);
     }
     barrier();
-    if (nh > 0) {
-      wait_vm_lgkm0<0>();
-      const uint8_t* pw = lds + r * PTS + hb * PKS + 16 * g;
-      if (one) {
-        bf16x8 pb[HW];
+    wait_vm_lgkm0<0>();                             // the values
+    asm volatile("" : "+v"(s2));                    // (and the slots: no wait for them behind the loads of the next keys)
+    load_k(s1, 0, kh0, kf[0]);
+    const uint32_t vat = vfrag_at<D>(vdst, g, r);
+    const uint8_t* pw = lds + r * PTS + hb * PHS + 16 * g;
+    if constexpr (ONE) {
+      bf16x8 pb[HW];
 #pragma unroll
-        for (int i = 0; i < HW; ++i) pb[i] = *reinterpret_cast<const bf16x8*>(pw + (i < nh ? i : 0) * PKS);
+      for (int i = 0; i < HW; ++i) pb[i] = *reinterpret_cast<const bf16x8*>(pw + i * PHS);
+      bf16x8 vf = vfrag<D>(vat, 0);
 #pragma unroll
-        for (int c = 0; c < NDT; ++c) {
-          const bf16x8 vf = vfrag<D>(vs, c, g, r);
+      for (int c = 0; c < NDT; ++c) {
+        const bf16x8 vn = c + 1 < NDT ? vfrag<D>(vat, c + 1) : vf;
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-          for (int i = 0; i < HW; ++i) o[i][c] = mma(vf, pb[i], o[i][c]);
+        for (int i = 0; i < HW; ++i) o[i][c] = mma(vf, pb[i], o[i][c]);
+        vf = vn;
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < HW; ++i) {
+        if (i > 0 && i < nh && (hb + i) % gq == 0) {
+          asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");                   // the last head's reads are done
+          fetch_v(sl, (hb + i) / gq);
+          wait_vm_lgkm0<0>();
         }
-      } else {
+        const bf16x8 pb = *reinterpret_cast<const bf16x8*>(pw + i * PHS);
 #pragma unroll
-        for (int i = 0; i < HW; ++i) {
-          if (i >= nh) break;
-          if (i > 0 && (hb + i) % gq == 0) {
-            asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");                   // the last head's reads are done
-            fetch_v(sl, (hb + i) / gq);
-            wait_vm_lgkm0<0>();
-          }
-          const bf16x8 pb = *reinterpret_cast<const bf16x8*>(pw + i * PKS);
-#pragma unroll
-          for (int c = 0; c < NDT; ++c) o[i][c] = mma(vfrag<D>(vs, c, g, r), pb, o[i][c]);
-        }
+        for (int c = 0; c < NDT; ++c) o[i][c] = mma(vfrag<D>(vat, c), pb, o[i][c]);
       }
     }
+    __builtin_amdgcn_sched_barrier(0);
+    load_k(s1, 1, kh0, kf[1]);
     barrier();
-    sl = nx;
+    sl = s1;
+    s1 = s2;
   }
   if (r >= n) return;
+  auto store = [&](auto four) {
 #pragma unroll
-  for (int i = 0; i < HW; ++i) {
-    if (i >= nh) break;
+    for (int i = 0; i < HW; ++i)
+      if (i < nh) {
 #pragma unroll
-    for (int c = 0; c < NDT; ++c) put_out(a, tok, hb + i, 16 * c + 4 * g, o[i][c]);
+        for (int c = 0; c < NDT; ++c) put_out<decltype(four)::value>(a, tok, hb + i, 16 * c + 4 * g, o[i][c]);
+      }
+  };
+  if (by_four(a)) store(std::true_type{});
+  else store(std::false_type{});
+}
+
+template <int D, int HW, bool ONE>
+int prefill_o(const Prefill& p, int n, hipStream_t st) {
+  constexpr int LDS = PL<D, HW>::BYTES;
+  static bool attr = false;
+  if (!attr) {
+    if (hipFuncSetAttribute((const void*)talk_prefill_kernel<D, HW, ONE>, hipFuncAttributeMaxDynamicSharedMemorySize, LDS) != hipSuccess)
+      return -1;
+    attr = true;
   }
+  hipLaunchKernelGGL((talk_prefill_kernel<D, HW, ONE>), dim3((n + 7) / 8 * 8 * p.nsub), dim3(512), LDS, st, p);
+  return (int)hipGetLastError();
 }
 
 template <int D, int HW>
 int prefill_t(const Prefill& p, int n, hipStream_t st) {
-  constexpr int LDS = 2 * PPL + 8 * KG * D * 2;
-  static_assert(LDS <= 160 * 1024, "LDS");
-  static bool attr = false;
-  if (!attr) {
-    if (hipFuncSetAttribute((const void*)talk_prefill_kernel<D, HW>, hipFuncAttributeMaxDynamicSharedMemorySize, LDS) != hipSuccess)
-      return -1;
-    attr = true;
-  }
-  hipLaunchKernelGGL((talk_prefill_kernel<D, HW>), dim3(n * p.nsub), dim3(512), LDS, st, p);
-  return (int)hipGetLastError();
+  return p.a.H / p.a.G % HW == 0 ? prefill_o<D, HW, true>(p, n, st) : prefill_o<D, HW, false>(p, n, st);
 }
 
 inline bool valid(const TalkArgs& a) {
@@ -662,14 +730,13 @@ int nls_talk_decode(const void* q, long ldq, const void* k, const void* v, const
   return rc;
 }
 
-// query blocks of up to 16 * nsub tokens, bf16; H <= 32, Dp 32, 64 or 128, ceil(H / 8) heads of Dp columns at most 512 columns. talk:
-// bf16 [32][32]
+// query blocks of up to 16 * nsub tokens, bf16; H <= 32, Dp 32, 64 or 128, scale > 0. talk: bf16 [32][32]
 int nls_talk_prefill(const void* q, long ldq, const void* k, const void* v, const int* xmap, const int* blocks, int nblocks, int nsub,
                      int H, int G, int Dp, int V, float scale, int window, const void* talk, const void* gate, long ldg, void* out,
                      long ldo, void* stream) {
   const TalkArgs a{q, k, v, out, gate, talk, nullptr, nullptr, nullptr, ldq, ldo, ldg, 0, 0, H, G, Dp, V, scale, window};
-  if (nblocks < 1 || nsub < 1 || !valid(a) || H > 32 || (ldq & 7) || (ldo & 3) || !xmap || !blocks) return -1;
-  const Prefill p{a, xmap, blocks, nsub};
+  if (nblocks < 1 || nsub < 1 || !valid(a) || H > 32 || !(scale > 0.f) || (ldq & 7) || (ldo & 3) || !xmap || !blocks) return -1;
+  const Prefill p{a, xmap, blocks, nblocks, nsub};
   const int hw = (H + 7) / 8;
   hipStream_t s = (hipStream_t)stream;
 #define NLS_TP(D) \

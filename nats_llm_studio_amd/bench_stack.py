@@ -4,6 +4,8 @@ GGUF families' closest model with the same width, layers and weights per layer, 
   kolodra    Llama (grouped-query attention + gated feed-forward), the feed-forward wider by the weights of the second mixer
   bibapel    Llama, four layers beside four layer runs (the attention layer runs twice), the feed-forward wider by the weights that
              the linear mixers and the passes' entries read
+  pimodra    Mixtral, four layers beside four layer runs (one with a dense feed-forward of a token's expert weights, then experts,
+             one of these layers twice), the same experts
 
 Both run the engine's own loop: submit, chunked prefill, captured decode steps. Random weights; one JSON line per case."""
 from __future__ import annotations
@@ -38,10 +40,15 @@ SIZES = {
         "4k": dict(width=4096, attention=(32, 8, 128), delta=(32, 16, 128, 128, 128), lightning=(32, 128, 128), ff=9216,
                    closest=dict(n_head=32, n_kv_head=8, d_ff=12288)),
     },
+    # dense ff: 2 matrices = the 3 matrices of a token's experts
+    "pimodra": {
+        "2k": dict(width=2048, attention=(16, 4, 128), ff=12288, moe=(8, 2, 4096), closest=dict(n_head=16, n_kv_head=4, d_ff=4096)),
+        "4k": dict(width=4096, attention=(32, 8, 128), ff=12288, moe=(8, 2, 4096), closest=dict(n_head=32, n_kv_head=8, d_ff=4096)),
+        # many small experts, group-limited choice (no GGUF family has this shape)
+        "4k-fine": dict(width=4096, attention=(32, 8, 128), ff=12288, moe=(64, 6, 1024), groups=(8, 4), closest=None),
+    },
 }
-CLOSEST = {"sekolorn": "mixtral-8x7b", "kolodra": "llama-3-8b", "bibapel": "llama-3-8b"}
-DESIGNS = tuple(SIZES)
-
+CLOSEST = {"sekolorn": "mixtral-8x7b", "kolodra": "llama-3-8b", "bibapel": "llama-3-8b", "pimodra": "mixtral-8x7b"}
 
 def sekolorn_config(sz: dict) -> dict:
     H, D = sz["wkv"]
@@ -81,7 +88,20 @@ def bibapel_config(sz: dict) -> dict:
             "loop": {"start": 1, "stop": 2, "times": 2}, "rank": sz["delta"][4]}
 
 
-CONFIGS = {"sekolorn": sekolorn_config, "kolodra": kolodra_config, "bibapel": bibapel_config}
+def pimodra_config(sz: dict) -> dict:
+    H, G, D = sz["attention"]
+    E, top, ff = sz["moe"]
+    mixer = {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "mask": {"size": 1024},
+             "rot": {"base": 10000.0, "dims": D, "scaling": {"factor": 4.0, "original": 2048, "fast": 32.0, "slow": 1.0}}}
+    moe = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": E, "top": top}}
+    if "groups" in sz:
+        moe["router"]["groups"] = {"count": sz["groups"][0], "keep": sz["groups"][1]}
+    layers = [{"type": "attention", "mixer": mixer, "mlp": f} for f in ({"kind": "dense", "ff": sz["ff"]}, moe, moe)]
+    return {"architecture": "Pimodra", "width": sz["width"], "vocab": VOCAB, "norm": {"eps": 1e-5, "groups": 2}, "layers": layers,
+            "loop": {"start": 1, "stop": 2, "times": 2}}
+
+
+CONFIGS = {"sekolorn": sekolorn_config, "kolodra": kolodra_config, "bibapel": bibapel_config, "pimodra": pimodra_config}
 
 
 def _sekolorn_layer(p: str, L: dict, d: int, lin, full):
@@ -175,10 +195,32 @@ def _bibapel_layer(p: str, L: dict, d: int, lin, full, rank: int):
     lin(p + "mlp.down", d, ff)
 
 
+def _pimodra_layer(p: str, L: dict, d: int, lin, full):
+    m, f = L["mixer"], L["mlp"]
+    for n in ("norm1", "norm1b", "norm2", "norm2b"):
+        full(p + n, 1.0, d)
+    H, G, D, V = (m[k] for k in ("heads", "kv_heads", "dim", "vdim"))
+    for n, rows in (("q", H * D), ("k", G * D), ("v", G * V), ("g", H * V)):
+        lin(p + "mix." + n, rows, d)
+    lin(p + "mix.talk", H, H)
+    lin(p + "mix.o", d, H * V)
+    if f["kind"] == "dense":
+        lin(p + "mlp.up", f["ff"], d)
+        lin(p + "mlp.down", d, f["ff"])
+        full(p + "mlp.act", 0.5, 4)
+        return
+    lin(p + "mlp.router", f["router"]["experts"], d)
+    for e in range(f["router"]["experts"]):
+        for n in ("gate", "up"):
+            lin(f"{p}mlp.e{e}.{n}", f["expert"]["ff"], d)
+        lin(f"{p}mlp.e{e}.down", d, f["expert"]["ff"])
+
+
 def write_stack(path: str, cfg: dict):
     """A checkpoint folder of `cfg` with random weights."""
     import torch
 
+    from .models.stack_config import DESIGNS
     from .safetensors_io import write_safetensors
     os.makedirs(path, exist_ok=True)
     W, d = {}, cfg["width"]
@@ -191,7 +233,8 @@ def write_stack(path: str, cfg: dict):
     def full(name, v, *shape):
         W[name] = torch.full(shape, v, dtype=torch.bfloat16)
     W["embed"] = torch.randn(cfg["vocab"], d, generator=g, device=dev).to(torch.bfloat16).cpu()
-    layer = {"Sekolorn": _sekolorn_layer, "Kolodra": _kolodra_layer, "Bibapel": _bibapel_layer}[cfg["architecture"]]
+    layer = {"Sekolorn": _sekolorn_layer, "Kolodra": _kolodra_layer, "Bibapel": _bibapel_layer,
+             "Pimodra": _pimodra_layer}[cfg["architecture"]]
     cfg = dict(cfg)
     rank = cfg.pop("rank", None)                    # (of the delta rule's gates: a tensor shape, no part of the config)
     for i, L in enumerate(cfg["layers"]):
@@ -201,8 +244,9 @@ def write_stack(path: str, cfg: dict):
         lin("bigram", cfg["embedding"]["bigram"]["buckets"] + 1, d)
         lin("pos", cfg["max_positions"], d)
         lin("loop.in", d, 2 * d)
+    if cfg.get("loop"):
         lin("loop.step", cfg["loop"]["times"], d)
-    else:
+    if not DESIGNS[cfg["architecture"]].tied_head:
         lin("head", cfg["vocab"], d)
     with open(os.path.join(path, "config.json"), "w") as fh:
         json.dump(cfg, fh)

@@ -383,7 +383,7 @@ class AttentionPart(_SharedPart):
         self.cs = model.rope(c.rot_base, c.rot_dims, c.rot_scaling) if c.rot_dims else None
         self.talk = None
         if design.attn_talk:
-            self.talk_plan = K.TalkPlan(H, G, self.Dp, c.window, model.cfg.ctx, model.f32, model.device)
+            self.talk_plan = K.TalkPlan(H, G, self.Dp, c.window, model.cfg.ctx, model.f32, model.device, c.scale)
             self.talk = self.talk_plan.matrix(self.mat("talk", (H, H)))
         self.cache_width = 2 * G * self.Dp
         self.out_width = K.act_ld(H * self.Dp)

@@ -651,10 +651,10 @@ TALK_SCRATCH = 256 << 20                # bytes of scores that a decode launch m
 class TalkPlan:
     """Kernels and scratch sizes of an attention whose heads' softmax weights are mixed, heads padded to Dp columns."""
 
-    def __init__(self, H: int, G: int, Dp: int, window: int, ctx: int, f32: bool, device):
+    def __init__(self, H: int, G: int, Dp: int, window: int, ctx: int, f32: bool, device, scale: float = 1.0):
         self.H, self.G, self.Dp, self.window = H, G, Dp, window
         self.mfma = not f32 and Dp in HEAD_WIDTHS and H <= 128
-        self.prefill = self.mfma and H <= 32 and Dp in TALK_WIDTHS
+        self.prefill = self.mfma and H <= 32 and Dp in TALK_WIDTHS and scale > 0
         self.groups, self.hs = attn_groups(H, G), pad_to(H, 8)
         self.ks = pad_to(min(window or ctx, ctx), 32) + 32              # keys of a row, from a multiple of 32 on
         self.device = device
@@ -678,7 +678,7 @@ class TalkPlan:
         ns1 = max(1, min(64, 2048 // n))
         if n >= 1024 or self.Dp > 128:
             return ns1, max(1, min(16, 1024 // n)), 1
-        return ns1, max(1, min(16, 512 // n)), 4
+        return ns1, max(1, min(16, 256 // n)), 4
 
     def scratch(self, cap: int):
         """Element counts of (scores, score statistics, partial outputs, counters)."""
