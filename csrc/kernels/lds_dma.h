@@ -17,6 +17,14 @@ DEVI void glds16(const void* gsrc, uint32_t lds_dst) {
                : "v"(gsrc), "s"(lds_dst)
                : "memory");
 }
+// the same from a wave-uniform base and a byte offset per lane
+DEVI void glds16(const void* base, uint32_t offset, uint32_t lds_dst) {
+  uint32_t keep;
+  asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2\n\ts_mov_b32 m0, %0"
+               : "=&s"(keep)
+               : "v"(offset), "s"(base), "s"(lds_dst)
+               : "memory");
+}
 template <int N>
 DEVI void wait_vm_lgkm0() {
   asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" ::"i"(N) : "memory");

@@ -355,15 +355,16 @@ int decode_value(const Decode& p, int rows, int groups, int waves, hipStream_t s
 // ---------------------------------------------------------------------------------------------------------------------
 struct Prefill {
   TalkArgs a;
-  const int* xmap;        // cache slot of every context row
-  const int* blocks;      // [n][8]: (first row, rows, sequence, first position, xoff, -, -, -)
+  const int* blocks;      // [n][8]: (first row, rows, sequence, first position, -, -, -, -)
+  int bshift;             // pages of 1 << bshift >= 16 keys
   int nblocks, nsub;      // blocks; workgroups of 16 tokens of each
 };
 
 // Eight waves of HW heads each, 16 tokens. Weights of a 32-key tile in LDS, [token][key][head][two bf16 parts]; wave w mixes
 // tokens 2 w and 2 w + 1 (rows: keys, columns: heads) and leaves the mixed weights, [token][head][key], in that token's space;
-// then each wave multiplies its own heads with the values, whose tile it has fetched by LDS-DMA for itself. Slots are read
-// two tiles ahead, keys one, values while the weights are mixed.
+// then each wave multiplies its own heads with the values, whose tile it has fetched by LDS-DMA for itself. Keys are read a tile
+// ahead, values while the weights are mixed. 16 keys beside each other lie in one page, so addresses are a wave-uniform base and a
+// constant offset per lane.
 constexpr int PKS = 144, PTS = 32 * PKS + 16, PW = 16 * PTS, PHS = 80;     // bytes: key row, token, all; row of a mixed head
 // behind the value tiles what the registers do not hold through the second walk: the matrix, the denominators, and at the largest
 // size some of the last head's queries
@@ -387,7 +388,6 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
   const int row0 = 16 * (p.nsub - 1 - unit % p.nsub), n = min(16, blk[1] - row0);      // (later rows see more keys)
   if (n <= 0) return;
   const int t0 = blk[0] + row0, pos0 = blk[3] + row0, last = pos0 + n - 1;
-  const int* xmap = p.xmap + blk[4];
   const int tid = threadIdx.x, lane = tid & 63, g = lane >> 4, r = lane & 15;
   const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int hb = wave * HW, nh = min(HW, a.H - hb), gq = a.H / a.G;
@@ -395,9 +395,8 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
   // paths with and without loads meet, the counted waits would become waits for everything.
   const int tok = t0 + min(r, n - 1), qpos = pos0 + min(r, n - 1);
   const int window = a.window > 0 ? a.window : 1 << 30;
-  const uint32_t ldkv = (uint32_t)a.G * D;          // (slots and strides of 32 bits: one multiplication)
+  const long ldkv = (long)a.G * D;
   const float sl2 = a.scale * LOG2E;
-  const __bf16 *kc = (const __bf16*)a.k + 8 * g, *vc = (const __bf16*)a.v;
   for (int i = tid; i < PW / 16; i += 512) reinterpret_cast<u32x4*>(lds)[i] = u32x4{0u, 0u, 0u, 0u};
 
   bf16x8 qf[HW][NKK];
@@ -409,12 +408,33 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
                          : bf16x8{};
 
   const int first = max(0, pos0 - window + 1) / KG, end = last / KG + 1;
-  auto slots = [&](int t) { return xmap[min(t * KG + (lane & 31), last)]; };      // lane: slot of key lane % 32
-  auto load_k = [&](int sl, int nt, int kh, u32x4 (&K)[NKK]) __attribute__((always_inline)) {
-    const __bf16* s = kc + (uint64_t)(uint32_t)__shfl(sl, 16 * nt + r, 64) * ldkv + (size_t)kh * D;
+  // cache rows of the two groups of 16 keys of a tile (past the last key: its group again, masked): table entries come from a
+  // register window of 64
+  const int* bt = a.bt + (size_t)__builtin_amdgcn_readfirstlane(blk[2]) * a.bts;
+  const int e0 = first * KG >> p.bshift, elast = last >> p.bshift;
+  int btwin = -1, btreg = 0;
+  struct Rows { long at[2]; };
+  auto rows = [&](int t) __attribute__((always_inline)) {
+    Rows s;
+#pragma unroll
+    for (int nt = 0; nt < 2; ++nt) {
+      const int k = min(t * KG + 16 * nt, last & ~15), e = (k >> p.bshift) - e0;
+      if (nt == 0 && e >> 6 != btwin) {             // (both groups lie in one window: it starts with a tile)
+        btwin = e >> 6;
+        const int i = e0 + 64 * btwin + lane;
+        btreg = i <= elast ? bt[i] : 0;
+        asm volatile("" : "+v"(btreg));             // waited for here, not where the paths meet: there other loads are on their way
+      }
+      s.at[nt] = (((long)__builtin_amdgcn_readlane(btreg, e & 63) << p.bshift) + (k & ((1 << p.bshift) - 1))) * ldkv;
+    }
+    return s;
+  };
+  const uint32_t koff = r * (uint32_t)ldkv + 8 * g;
+  auto load_k = [&](const Rows& s, int nt, int kh, u32x4 (&K)[NKK]) __attribute__((always_inline)) {
+    const __bf16* base = (const __bf16*)a.k + s.at[nt] + kh * D;
 #pragma unroll
     for (int kk = 0; kk < NKK; ++kk) {
-      K[kk] = ld16(s + 32 * kk);
+      K[kk] = ld16(base + (koff + 32 * kk));
       __builtin_amdgcn_sched_barrier(0);            // (in the order of their use, also ahead of the loops: the waits are counted)
     }
   };
@@ -439,14 +459,12 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
       l[i] = 0.f;
     }
     {
-      int sl = slots(first), s1 = slots(min(first + 1, end - 1));
-      asm volatile("" : "+v"(s1));
+      Rows sl = rows(first);
       u32x4 kf[2][NKK];
       load_k(sl, 0, kh0, kf[0]);
       load_k(sl, 1, kh0, kf[1]);
       for (int t = first; t < end; ++t) {
-        int s2 = slots(min(t + 2, end - 1));
-        __builtin_amdgcn_sched_barrier(0);
+        const Rows s1 = rows(min(t + 1, end - 1));
         f32x4 s[HW][2];
 #pragma unroll
         for (int i = 0; i < HW; ++i) {
@@ -458,7 +476,6 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
           for (int nt = 0; nt < 2; ++nt) s[i][nt] = score(kf[nt], qf[i]);
         }
         __builtin_amdgcn_sched_barrier(0);
-        asm volatile("" : "+v"(s2));                // (the next slots are waited for ahead of the next keys' loads, not behind them)
         load_k(s1, 0, kh0, kf[0]);
         load_k(s1, 1, kh0, kf[1]);
         auto sum = [&](auto edge) __attribute__((always_inline)) {
@@ -485,7 +502,6 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
         if (is_edge(t)) sum(std::true_type{});
         else sum(std::false_type{});
         sl = s1;
-        s1 = s2;
       }
     }
 #pragma unroll
@@ -511,22 +527,21 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
   for (int i = 0; i < HW; ++i)
 #pragma unroll
     for (int c = 0; c < NDT; ++c) o[i][c] = f32x4{0.f, 0.f, 0.f, 0.f};
+  btwin = -1;
   const uint32_t vdst = __builtin_amdgcn_readfirstlane(lds_addr(lds)) + P::V + wave * VB;
   // the lane's number anew: what follows from it need not live through the loop
   auto again = [](int v) __attribute__((always_inline)) {
     asm volatile("" : "+v"(v));
     return v;
   };
-  auto fetch_v = [&](int sl, int kh) __attribute__((always_inline)) {
+  auto fetch_v = [&](const Rows& s, int kh) __attribute__((always_inline)) {
     const int ln = again(lane);
-    int rs[NVL];
 #pragma unroll
-    for (int i = 0; i < NVL; ++i) rs[i] = __shfl(sl, RPI * i + ln / LPR, 64);
-#pragma unroll
-    for (int i = 0; i < NVL; ++i) asm volatile("" : "+v"(rs[i]));               // (all of them in flight together)
-#pragma unroll
-    for (int i = 0; i < NVL; ++i)
-      glds16(vc + (uint64_t)(uint32_t)rs[i] * ldkv + (size_t)kh * D + 8 * vswz<D>(RPI * i + ln / LPR, ln % LPR), vdst + 1024 * i);
+    for (int i = 0; i < NVL; ++i) {
+      const int row = RPI * i;
+      glds16((const __bf16*)a.v + s.at[row >> 4] + (row & 15) * ldkv + kh * D,
+             2 * ((ln / LPR) * (uint32_t)ldkv + 8 * vswz<D>(row + ln / LPR, ln % LPR)), vdst + 1024 * i);
+    }
   };
   auto barrier = [&]() __attribute__((always_inline)) {
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -534,8 +549,7 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     asm volatile("" ::: "memory");
   };
   __syncthreads();
-  int sl = slots(first), s1 = slots(min(first + 1, end - 1));
-  asm volatile("" : "+v"(s1));                      // (waited for ahead of the keys: see below)
+  Rows sl = rows(first);
   u32x4 kf[2][NKK];
   load_k(sl, 0, kh0, kf[0]);
   load_k(sl, 1, kh0, kf[1]);
@@ -581,8 +595,7 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     }
   };
   for (int t = first; t < end; ++t) {
-    int s2 = slots(min(t + 2, end - 1));
-    __builtin_amdgcn_sched_barrier(0);
+    const Rows s1 = rows(min(t + 1, end - 1));
     if (is_edge(t)) weigh(std::true_type{}, t);
     else weigh(std::false_type{}, t);
     fetch_v(sl, kh0);
@@ -617,7 +630,6 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     }
     barrier();
     wait_vm_lgkm0<0>();                             // the values
-    asm volatile("" : "+v"(s2));                    // (and the slots: no wait for them behind the loads of the next keys)
     load_k(s1, 0, kh0, kf[0]);
     const uint32_t vat = vfrag_at<D>(vdst, g, r);
     const uint8_t* pw = lds + r * PTS + hb * PHS + 16 * g;
@@ -651,7 +663,6 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     load_k(s1, 1, kh0, kf[1]);
     barrier();
     sl = s1;
-    s1 = s2;
   }
   if (r >= n) return;
   auto store = [&](auto four) {
@@ -730,13 +741,15 @@ int nls_talk_decode(const void* q, long ldq, const void* k, const void* v, const
   return rc;
 }
 
-// query blocks of up to 16 * nsub tokens, bf16; H <= 32, Dp 32, 64 or 128, scale > 0. talk: bf16 [32][32]
-int nls_talk_prefill(const void* q, long ldq, const void* k, const void* v, const int* xmap, const int* blocks, int nblocks, int nsub,
-                     int H, int G, int Dp, int V, float scale, int window, const void* talk, const void* gate, long ldg, void* out,
-                     long ldo, void* stream) {
-  const TalkArgs a{q, k, v, out, gate, talk, nullptr, nullptr, nullptr, ldq, ldo, ldg, 0, 0, H, G, Dp, V, scale, window};
-  if (nblocks < 1 || nsub < 1 || !valid(a) || H > 32 || !(scale > 0.f) || (ldq & 7) || (ldo & 3) || !xmap || !blocks) return -1;
-  const Prefill p{a, xmap, blocks, nblocks, nsub};
+// query blocks of up to 16 * nsub tokens, bf16; H <= 32, Dp 32, 64 or 128, scale > 0, bs a power of two >= 16. talk: bf16 [32][32]
+int nls_talk_prefill(const void* q, long ldq, const void* k, const void* v, const int* bt, int bts, int bs, const int* blocks,
+                     int nblocks, int nsub, int H, int G, int Dp, int V, float scale, int window, const void* talk, const void* gate,
+                     long ldg, void* out, long ldo, void* stream) {
+  const TalkArgs a{q, k, v, out, gate, talk, bt, nullptr, nullptr, ldq, ldo, ldg, bts, bs, H, G, Dp, V, scale, window};
+  if (nblocks < 1 || nsub < 1 || !valid(a) || H > 32 || !(scale > 0.f) || (ldq & 7) || (ldo & 3) || !bt || !blocks || bs < 16 ||
+      (bs & (bs - 1)))
+    return -1;
+  const Prefill p{a, blocks, __builtin_ctz((unsigned)bs), nblocks, nsub};
   const int hw = (H + 7) / 8;
   hipStream_t s = (hipStream_t)stream;
 #define NLS_TP(D) \

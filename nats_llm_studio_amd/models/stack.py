@@ -440,7 +440,7 @@ class AttentionPart(_SharedPart):
                 K.talk_attention(*args, e.get("part"), b.block_tables, step.block_size, b.tok_seq,
                                  b.ctx_len if plan is None else plan.actx, T, c.vdim, c.scale, st)
             if plan is not None:
-                K.talk_prefill(*args, plan.xmap, plan.blocks, plan.nblocks, plan.waves, c.vdim, c.scale, st)
+                K.talk_prefill(*args, b.block_tables, step.block_size, plan.blocks, plan.nblocks, plan.waves, c.vdim, c.scale, st)
             return
         if plan is None or plan.rest:
             ns = max(1, min(_SPLIT_CAP, _SPLIT_WG // (T * self.groups))) if self.mfma else 1

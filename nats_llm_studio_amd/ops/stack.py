@@ -45,7 +45,7 @@ _SIGS = {
     "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, I, I, F, I, P],
     "nls_talk_plain": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, I, P, P, L, P, L, I, P],
     "nls_talk_decode": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, I, F, I, P, P, L, P, L, P, L, P, P, P, I, I, I, P],
-    "nls_talk_prefill": [P, L, P, P, P, P, I, I, I, I, I, I, F, I, P, P, L, P, L, P],
+    "nls_talk_prefill": [P, L, P, P, P, I, I, P, I, I, I, I, I, I, F, I, P, P, L, P, L, P],
     "nls_gqa_attn": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, P, L, P, L, P, P, P, I, I, I, I, I, P],
     "nls_gqa_prefill": [P, L, P, P, P, P, I, P, I, P, L, I, I, I, I, F, I, I, I, P],
     "nls_delta_conv": [P, L, P, P, L, P, L, P, L, P, P, I, I, I, I, I, I, I, I, P],
@@ -715,11 +715,12 @@ def talk_attention(plan: TalkPlan, q, kc, vc, talk, gate, out, scratch, block_ta
                "nls_talk_decode")
 
 
-def talk_prefill(plan: TalkPlan, q, kc, vc, talk, gate, out, xmap, blocks, nblocks: int, waves: int, V: int, scale: float, st: int):
+def talk_prefill(plan: TalkPlan, q, kc, vc, talk, gate, out, block_tables, block_size: int, blocks, nblocks: int, waves: int, V: int,
+                 scale: float, st: int):
     """Attention with mixed heads of query blocks of up to 32 * waves tokens over their sequences' paged keys and values."""
     p = plan
     if not p.prefill or (gate is not None and gate.dtype != out.dtype):
         raise ValueError("talk_prefill: a shape of the row-by-row kernels, or a gate of another type")
-    _check(lib().nls_talk_prefill(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), xmap.data_ptr(), blocks.data_ptr(),
-                                  nblocks, 2 * waves, p.H, p.G, p.Dp, V, scale, p.window, talk.data_ptr(), _p(gate),
+    _check(lib().nls_talk_prefill(q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(), block_tables.data_ptr(),
+                                  block_tables.stride(0), block_size, blocks.data_ptr(), nblocks, 2 * waves, p.H, p.G, p.Dp, V, scale, p.window, talk.data_ptr(), _p(gate),
                                   gate.stride(0) if gate is not None else 0, out.data_ptr(), out.stride(0), st), "nls_talk_prefill")
