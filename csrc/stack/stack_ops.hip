@@ -404,7 +404,8 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const float* __restric
 // ---- attention rows: one workgroup per token. q and k are RMS-normed over all their heads together (norm weights optional),
 // rotated on the first `rot` columns of each head (pairs 2i, 2i + 1) and stored in the activation type, heads Dp columns
 // apart: q to `qo`, k and v (unnormed, unrotated) to the token's rows of the paged caches. The columns past D of a head
-// are never written (zero from the start); slot < 0: no cache row.
+// are never written (zero from the start); slot < 0: no cache row. ktile: 16 slots of the key cache are a tile [G][Dp / 8][16][8]
+// instead of rows, in which the 16 keys of an MFMA operand lie side by side.
 struct AttnRows {
   const float *q, *k, *v;     // projections, f32
   const float *qn, *kn;       // norm weights (null: no norm)
@@ -415,19 +416,30 @@ struct AttnRows {
   int H, G, D, Dp, rot, V;    // V: columns of a value head
   float eps;
   int hnorm;                  // each rotated head of q and k is RMS-normed on its own, without weights
+  int ktile;
+  // 16 tokens beside each other, which fill the same lines of a key tile, run on one XCD
+  DEVI int token() const {
+    const int b = blockIdx.x;
+    return ktile && b < ((int)gridDim.x & ~127) ? (b & ~127) | (b & 7) << 4 | (b >> 3 & 15) : b;
+  }
+  // where column c of a slot's key head h goes
+  DEVI size_t key(int slot, int h, int c) const {
+    return ktile ? (size_t)(slot & ~15) * ldc + (size_t)h * 16 * Dp + (c >> 3) * 128 + (slot & 15) * 8 + (c & 7)
+                 : (size_t)slot * ldc + (size_t)h * Dp + c;
+  }
 };
 
 template <typename T>
 __global__ __launch_bounds__(256) void attn_rows_kernel(AttnRows p) {
   __shared__ float sh[4];
-  const int t = blockIdx.x, D = p.D, slot = p.slot[t];
+  const int t = p.token(), D = p.D, slot = p.slot[t];
   const float* f = p.rot ? p.cs + (size_t)p.pos[t] * p.rot : nullptr;
   auto norm = [&](const float* a, int n) {
     float s = 0.f;
     for (int i = threadIdx.x; i < n; i += 256) s += a[i] * a[i];
     return 1.f / sqrtf(bsum<4>(s, sh) / (float)n + p.eps);
   };
-  auto put = [&](const float* a, const float* w, float inv, int heads, T* o) {
+  auto put = [&](const float* a, const float* w, float inv, int heads, auto at) {
     const int D2 = (D + 1) >> 1;
     for (int e = threadIdx.x; e < heads * D2; e += 256) {
       const int h = e / D2, c = 2 * (e - h * D2), i = h * D + c;
@@ -442,15 +454,17 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(AttnRows p) {
         v = v * cc + u * ss;
         u = r;
       }
-      o[(size_t)h * p.Dp + c] = (T)u;
-      if (two) o[(size_t)h * p.Dp + c + 1] = (T)v;
+      T* o = at(h, c);                              // (columns c and c + 1, c even, are beside each other)
+      o[0] = (T)u;
+      if (two) o[1] = (T)v;
     }
   };
   const float *q = p.q + (size_t)t * p.ldq, *k = p.k + (size_t)t * p.ldq, *v = p.v + (size_t)t * p.ldq;
-  put(q, p.qn, p.qn ? norm(q, p.H * D) : 1.f, p.H, (T*)p.qo + (size_t)t * p.ldqo);
+  put(q, p.qn, p.qn ? norm(q, p.H * D) : 1.f, p.H,
+      [&](int h, int c) { return (T*)p.qo + (size_t)t * p.ldqo + (size_t)h * p.Dp + c; });
   const float ik = p.kn ? norm(k, p.G * D) : 1.f;
   if (slot < 0) return;
-  put(k, p.kn, ik, p.G, (T*)p.kc + (size_t)slot * p.ldc);
+  put(k, p.kn, ik, p.G, [&](int h, int c) { return (T*)p.kc + p.key(slot, h, c); });
   T* vo = (T*)p.vc + (size_t)slot * p.ldc;
   for (int e = threadIdx.x; e < p.G * p.V; e += 256) vo[(size_t)(e / p.V) * p.Dp + e % p.V] = (T)v[e];
 }
@@ -462,7 +476,7 @@ template <typename T, int NV, int NTH, bool HN>
 __global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
   __shared__ float sh[2][NTH / 64];
   typedef T t4 __attribute__((ext_vector_type(4)));
-  const int t = blockIdx.x, D4 = p.D >> 2, nq = p.H * D4, n = nq + p.G * D4, slot = p.slot[t];
+  const int t = p.token(), D4 = p.D >> 2, nq = p.H * D4, n = nq + p.G * D4, slot = p.slot[t];
   const float *q = p.q + (size_t)t * p.ldq, *k = p.k + (size_t)t * p.ldq, *v = p.v + (size_t)t * p.ldq;
   const float* f = p.rot ? p.cs + (size_t)p.pos[t] * p.rot : nullptr;
   f32x4 x[NV];
@@ -521,9 +535,8 @@ __global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
     if (isq) {
       *reinterpret_cast<t4*>((T*)p.qo + (size_t)t * p.ldqo + (size_t)h * p.Dp + c) = o;
     } else {
-      const size_t d = (size_t)slot * p.ldc + (size_t)h * p.Dp + c;
-      *reinterpret_cast<t4*>((T*)p.kc + d) = o;
-      if (p.v == p.k) *reinterpret_cast<t4*>((T*)p.vc + d) = t4{(T)x[j][0], (T)x[j][1], (T)x[j][2], (T)x[j][3]};
+      *reinterpret_cast<t4*>((T*)p.kc + p.key(slot, h, c)) = o;
+      if (p.v == p.k) *reinterpret_cast<t4*>((T*)p.vc + (size_t)slot * p.ldc + (size_t)h * p.Dp + c) = t4{(T)x[j][0], (T)x[j][1], (T)x[j][2], (T)x[j][3]};
     }
   }
   if (p.v == p.k || slot < 0) return;
@@ -540,7 +553,7 @@ __global__ __launch_bounds__(NTH) void attn_rows4_kernel(AttnRows p) {
 template <typename T>
 __global__ __launch_bounds__(256) void attn_head_rows_kernel(AttnRows p) {
   constexpr int NP = 8;                           // pairs of columns per lane: heads of up to 1024 columns
-  const int t = blockIdx.x, D = p.D, D2 = (D + 1) >> 1, lane = threadIdx.x & 63;
+  const int t = p.token(), D = p.D, D2 = (D + 1) >> 1, lane = threadIdx.x & 63;
   const int slot = p.slot[t], u = blockIdx.y * 4 + (threadIdx.x >> 6);          // a head of q, k or v
   if (u >= p.H + 2 * p.G || (u >= p.H && slot < 0)) return;
   if (u >= p.H + p.G) {
@@ -553,7 +566,7 @@ __global__ __launch_bounds__(256) void attn_head_rows_kernel(AttnRows p) {
   const bool isq = u < p.H;
   const int h = isq ? u : u - p.H;
   const float* a = (isq ? p.q : p.k) + (size_t)t * p.ldq + (size_t)h * D;
-  T* o = isq ? (T*)p.qo + (size_t)t * p.ldqo + (size_t)h * p.Dp : (T*)p.kc + (size_t)slot * p.ldc + (size_t)h * p.Dp;
+  auto at = [&](int c) { return isq ? (T*)p.qo + (size_t)t * p.ldqo + (size_t)h * p.Dp + c : (T*)p.kc + p.key(slot, h, c); };
   const float* f = p.rot ? p.cs + (size_t)p.pos[t] * p.rot : nullptr;
   float x[NP], y[NP], s = 0.f;
 #pragma unroll
@@ -575,8 +588,9 @@ __global__ __launch_bounds__(256) void attn_head_rows_kernel(AttnRows p) {
   for (int j = 0; j < NP; ++j) {
     const int i = lane + 64 * j, c = 2 * i;
     if (i >= D2) continue;
-    o[c] = (T)(x[j] * inv);
-    if (c + 1 < D) o[c + 1] = (T)(y[j] * inv);
+    T* o = at(c);                                   // (columns c and c + 1, c even, are beside each other)
+    o[0] = (T)(x[j] * inv);
+    if (c + 1 < D) o[1] = (T)(y[j] * inv);
   }
 }
 
@@ -900,11 +914,11 @@ int nls_latent_rows(const float* dq, long lddq, int Q, const float* wq, void* cq
 // heads of D columns (values: V), Dp apart in the outputs; rot even, at most D; hnorm: no weights
 int nls_attn_rows(const float* q, const float* k, const float* v, long ldq, const float* qn, const float* kn, const float* cs,
                   const int* pos, const int* slot, void* qo, long ldqo, void* kc, void* vc, long ldc, int T, int H, int G,
-                  int D, int V, int Dp, int rot, int hnorm, float eps, int f32, void* stream) {
-  if (T < 1 || (hnorm && (qn || kn || D > 1024)) || H < 1 || G < 1 || D < 1 || V < 1 || Dp < D || Dp < V || (v == k && V != D) || (rot && !cs) || (rot & 1) || rot < 0 ||
+                  int D, int V, int Dp, int rot, int hnorm, int ktile, float eps, int f32, void* stream) {
+  if (T < 1 || (ktile && ((Dp & 7) || ldc != (long)G * Dp)) || (hnorm && (qn || kn || D > 1024)) || H < 1 || G < 1 || D < 1 || V < 1 || Dp < D || Dp < V || (v == k && V != D) || (rot && !cs) || (rot & 1) || rot < 0 ||
       rot > D || (long)H * Dp > ldqo || (long)G * Dp > ldc)
     return -1;
-  AttnRows p{q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, ldq, ldqo, ldc, H, G, D, Dp, rot, V, eps, hnorm};
+  AttnRows p{q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, ldq, ldqo, ldc, H, G, D, Dp, rot, V, eps, hnorm, ktile};
   return f32 ? attn_rows_t<float>(p, T, (hipStream_t)stream) : attn_rows_t<__bf16>(p, T, (hipStream_t)stream);
 }
 

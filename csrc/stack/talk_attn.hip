@@ -5,6 +5,8 @@
 //                               gate. Splits of normalised weights add up without a rescale.
 //   prompts                     one workgroup per 16 tokens and all heads, two walks over the keys: the first leaves each head's
 //                               log-sum-exp in registers, the second scores again, mixes and multiplies with the values.
+// Keys come in tiles of 16 slots, [slots / 16][G][Dp / 8][16][8]: the 16 keys of an MFMA operand lie side by side, and a wave's load of
+// 32 of their columns is 1 KB in a row. Values are rows.
 // The mix itself is on MFMA: a softmax weight goes in as two bf16 parts (16 bits of it), the matrix, which is stored in bf16,
 // exactly, and the sums are f32.
 #include "../kernels/lds_dma.h"
@@ -98,7 +100,7 @@ __global__ __launch_bounds__(64) void talk_score_kernel(Decode p) {
   const int tps = (key.ntile + p.ns1 - 1) / p.ns1, ta = split * tps, tb = min(ta + tps, key.ntile);
   if (ta >= tb) return;
   const int* bt = a.bt + (size_t)a.tok_seq[t] * a.bts;
-  const __bf16* kc = (const __bf16*)a.k + (size_t)kh * D + 8 * g;
+  const __bf16* kc = (const __bf16*)a.k + (size_t)kh * 16 * D + 128 * g;
   const size_t ldkv = (size_t)a.G * D;
   bf16x8 qf[NKK];
 #pragma unroll
@@ -110,9 +112,10 @@ __global__ __launch_bounds__(64) void talk_score_kernel(Decode p) {
 #pragma unroll
     for (int nt = 0; nt < 2; ++nt) {
       const int k = min(key.first + tile * KG + 16 * nt + r, key.ctx - 1);
-      const size_t o = (((size_t)bt[k >> p.bshift] << p.bshift) + (k & ((1 << p.bshift) - 1))) * ldkv;
+      const size_t slot = ((size_t)bt[k >> p.bshift] << p.bshift) + (k & ((1 << p.bshift) - 1));
+      const size_t o = (slot & ~(size_t)15) * ldkv + (slot & 15) * 8;
 #pragma unroll
-      for (int kk = 0; kk < NKK; ++kk) K[nt][kk] = ld16(kc + o + 32 * kk);
+      for (int kk = 0; kk < NKK; ++kk) K[nt][kk] = ld16(kc + o + 512 * kk);
     }
   };
   u32x4 kr[2][NKK], kn[2][NKK];
@@ -429,25 +432,27 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     }
     return s;
   };
-  const uint32_t koff = r * (uint32_t)ldkv + 8 * g;
   auto load_k = [&](const Rows& s, int nt, int kh, u32x4 (&K)[NKK]) __attribute__((always_inline)) {
-    const __bf16* base = (const __bf16*)a.k + s.at[nt] + kh * D;
+    const __bf16* base = (const __bf16*)a.k + s.at[nt] + kh * 16 * D;
 #pragma unroll
     for (int kk = 0; kk < NKK; ++kk) {
-      K[kk] = ld16(base + (koff + 32 * kk));
+      K[kk] = ld16(base + (8u * lane + 512 * kk));
       __builtin_amdgcn_sched_barrier(0);            // (in the order of their use, also ahead of the loops: the waits are counted)
     }
   };
-  auto score = [&](const u32x4 (&K)[NKK], const bf16x8 (&q)[NKK]) __attribute__((always_inline)) {
-    f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
+  // The scores' sums start from what hides the keys 4 g .. of a group that the lane's token does not see. No branch over whole and
+  // partly seen tiles: where its paths meet, the counted waits would become waits for everything.
+  auto hidden = [&](int k0, int g) __attribute__((always_inline)) {
+    f32x4 c;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) c[e] = (uint32_t)(qpos - (k0 + 4 * g + e)) < (uint32_t)window ? 0.f : -INFINITY;
+    return c;
+  };
+  auto score = [&](const u32x4 (&K)[NKK], const bf16x8 (&q)[NKK], f32x4 s) __attribute__((always_inline)) {
 #pragma unroll
     for (int kk = 0; kk < NKK; ++kk) s = mma(__builtin_bit_cast(bf16x8, K[kk]), q[kk], s);
     return s;
   };
-  // A tile that some token does not see whole is an edge; its body is another copy of the code, and selects without branches (a branch
-  // between a product and the first use of its result has been compiled without the wait that the matrix pipeline needs).
-  auto is_edge = [&](int t) { return t * KG + KG - 1 > pos0 || t * KG <= last - window; };
-  auto sees = [&](int k) { return (k <= qpos) & (k > qpos - window); };
   const int kh0 = min(hb / gq, a.G - 1);
 
   // ---- first walk: each head's log2 of the softmax's denominator (lane: token r, its own keys; joined at the end)
@@ -466,6 +471,7 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
       for (int t = first; t < end; ++t) {
         const Rows s1 = rows(min(t + 1, end - 1));
         f32x4 s[HW][2];
+        const f32x4 c[2] = {hidden(t * KG, g), hidden(t * KG + 16, g)};
 #pragma unroll
         for (int i = 0; i < HW; ++i) {
           if (!ONE && i > 0 && i < nh && (hb + i) % gq == 0) {
@@ -473,34 +479,27 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
             load_k(sl, 1, (hb + i) / gq, kf[1]);
           }
 #pragma unroll
-          for (int nt = 0; nt < 2; ++nt) s[i][nt] = score(kf[nt], qf[i]);
+          for (int nt = 0; nt < 2; ++nt) s[i][nt] = score(kf[nt], qf[i], c[nt]);
         }
         __builtin_amdgcn_sched_barrier(0);
         load_k(s1, 0, kh0, kf[0]);
         load_k(s1, 1, kh0, kf[1]);
-        auto sum = [&](auto edge) __attribute__((always_inline)) {
 #pragma unroll
-          for (int i = 0; i < HW; ++i) {
-            float mn = m[i];                        // (of the scores as they are: sl2 >= 0)
+        for (int i = 0; i < HW; ++i) {
+          float mn = m[i];                          // (of the scores as they are: sl2 >= 0)
 #pragma unroll
-            for (int nt = 0; nt < 2; ++nt)
+          for (int nt = 0; nt < 2; ++nt)
 #pragma unroll
-              for (int e = 0; e < 4; ++e) {
-                if constexpr (decltype(edge)::value) s[i][nt][e] = sees(t * KG + 16 * nt + 4 * g + e) ? s[i][nt][e] : -INFINITY;
-                mn = fmaxf(mn, s[i][nt][e]);
-              }
-            const float nb = -mn * sl2;
-            float l2 = l[i] * __builtin_amdgcn_exp2f((m[i] - mn) * sl2);
+            for (int e = 0; e < 4; ++e) mn = fmaxf(mn, s[i][nt][e]);
+          const float nb = -mn * sl2;
+          float l2 = l[i] * __builtin_amdgcn_exp2f((m[i] - mn) * sl2);
 #pragma unroll
-            for (int nt = 0; nt < 2; ++nt)
+          for (int nt = 0; nt < 2; ++nt)
 #pragma unroll
-              for (int e = 0; e < 4; ++e) l2 += __builtin_amdgcn_exp2f(fmaf(s[i][nt][e], sl2, nb));
-            l[i] = l2;
-            m[i] = mn;
-          }
-        };
-        if (is_edge(t)) sum(std::true_type{});
-        else sum(std::false_type{});
+            for (int e = 0; e < 4; ++e) l2 += __builtin_amdgcn_exp2f(fmaf(s[i][nt][e], sl2, nb));
+          l[i] = l2;
+          m[i] = mn;
+        }
         sl = s1;
       }
     }
@@ -553,10 +552,11 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
   u32x4 kf[2][NKK];
   load_k(sl, 0, kh0, kf[0]);
   load_k(sl, 1, kh0, kf[1]);
-  auto weigh = [&](auto edge, int t) __attribute__((always_inline)) {
+  auto weigh = [&](int t, const Rows& sl) __attribute__((always_inline)) {
     const int ln = again(lane), g = ln >> 4, r = ln & 15;
     const float* ll = reinterpret_cast<const float*>(lds + P::L) + hb * 16 + r;
     const bf16x8* ql = reinterpret_cast<const bf16x8*>(lds + P::Q + wave * P::NQ * 1024) + ln;
+    f32x4 c;
     auto product = [&](int u) __attribute__((always_inline)) {                  // keys 16 nt .., head i
       const int nt = u / HW, i = u % HW;
       if (!ONE && i > 0 && i < nh && (hb + i) % gq == 0) load_k(sl, nt, (hb + i) / gq, kf[nt]);
@@ -564,7 +564,8 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
 #pragma unroll
         for (int j = 0; j < P::NQ; ++j) qf[i][NKK - P::NQ + j] = ql[64 * j];
       }
-      return score(kf[nt], qf[i]);
+      if (i == 0) c = hidden(t * KG + 16 * nt, g);
+      return score(kf[nt], qf[i], c);
     };
     f32x4 s = product(0);
     float lse = ll[0];
@@ -573,13 +574,13 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     for (int u = 0; u < 2 * HW; ++u) {                                          // a product is on its way while the last one's weights are made
       const int nt = u / HW, i = u % HW;
       f32x4 sn = s;
+      if (u == HW) fetch_v(sl, kh0);                // (the tile's keys are there: nothing else waits for it)
       if (u + 1 < 2 * HW) sn = product(u + 1);
       const float lsen = ll[16 * ((u + 1) % HW)];
       constexpr int PAIR = HW > 1 ? 2 : 1;          // heads per store
       uint8_t* d = lds + r * PTS + (16 * nt + 4 * g) * PKS + (hb + i / PAIR * PAIR) * 4;
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        if constexpr (decltype(edge)::value) s[e] = sees(t * KG + 16 * nt + 4 * g + e) ? s[e] : -INFINITY;
         const float w = __builtin_amdgcn_exp2f(fmaf(s[e], sl2, -lse));
         // the upper half of w, and of what that leaves: 16 bits of it
         const uint32_t up = __builtin_bit_cast(uint32_t, w) & 0xffff0000u;
@@ -596,9 +597,7 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
   };
   for (int t = first; t < end; ++t) {
     const Rows s1 = rows(min(t + 1, end - 1));
-    if (is_edge(t)) weigh(std::true_type{}, t);
-    else weigh(std::false_type{}, t);
-    fetch_v(sl, kh0);
+    weigh(t, sl);
     barrier();
     const int ln = again(lane), g = ln >> 4, r = ln & 15;
     bf4 tf[2][2];
@@ -629,14 +628,15 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
       __builtin_amdgcn_sched_barrier(0);
     }
     barrier();
-    wait_vm_lgkm0<0>();                             // the values
-    load_k(s1, 0, kh0, kf[0]);
     const uint32_t vat = vfrag_at<D>(vdst, g, r);
     const uint8_t* pw = lds + r * PTS + hb * PHS + 16 * g;
     if constexpr (ONE) {
       bf16x8 pb[HW];
 #pragma unroll
       for (int i = 0; i < HW; ++i) pb[i] = *reinterpret_cast<const bf16x8*>(pw + i * PHS);
+      barrier();                                    // the next tile's weights may come: waves go on at their own pace until they mix
+      wait_vm_lgkm0<0>();                           // the values
+      load_k(s1, 0, kh0, kf[0]);
       bf16x8 vf = vfrag<D>(vat, 0);
 #pragma unroll
       for (int c = 0; c < NDT; ++c) {
@@ -647,6 +647,8 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
         vf = vn;
       }
     } else {
+      wait_vm_lgkm0<0>();
+      load_k(s1, 0, kh0, kf[0]);
 #pragma unroll
       for (int i = 0; i < HW; ++i) {
         if (i > 0 && i < nh && (hb + i) % gq == 0) {
@@ -661,7 +663,7 @@ __global__ __launch_bounds__(512) void talk_prefill_kernel(Prefill p) {
     }
     __builtin_amdgcn_sched_barrier(0);
     load_k(s1, 1, kh0, kf[1]);
-    barrier();
+    if constexpr (!ONE) barrier();
     sl = s1;
   }
   if (r >= n) return;

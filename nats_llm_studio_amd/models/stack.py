@@ -394,7 +394,7 @@ class AttentionPart(_SharedPart):
         return _FLASH_RUN if (self.mfma if self.talk is None else self.talk_plan.prefill) else None
 
     def new_cache(self, slots):
-        return torch.zeros(2, slots, self.cfg.kv_heads * self.Dp, dtype=self.m.dtype, device=self.m.device)
+        return torch.zeros(2, K.pad_to(slots, K.KEY_TILE), self.cfg.kv_heads * self.Dp, dtype=self.m.dtype, device=self.m.device)
 
     def out_weight(self):
         c, d = self.cfg, self.m.cfg.d_model
@@ -432,7 +432,7 @@ class AttentionPart(_SharedPart):
         kc, vc = cache[0], cache[1]
         K.attn_rows(e["qp"], e["kp"], e["vp"], self.qn, self.kn, self.cs, b.pos, b.slot, e["q"], kc, vc, T, c.heads,
                     c.kv_heads, c.dim, self.Dp, c.rot_dims, self.m.cfg.eps, st, V=c.vdim,
-                    head_norm=self.m.cfg.design.attn_qk_norm == "head")
+                    head_norm=self.m.cfg.design.attn_qk_norm == "head", key_tiles=self.talk is not None and self.talk_plan.mfma)
         plan = step.plan
         if self.talk is not None:
             args = (self.talk_plan, e["q"], kc, vc, self.talk, e["gate"], e["out"])

@@ -42,7 +42,7 @@ _SIGS = {
     "nls_norm_add": [P, L, P, I, L, P, P, L, P, L, P, P, P, P, L, P, I, I, I, F, I, I, I, I, L, P],
     "nls_row_norm": [P, L, P, P, P, P, P, L, P, L, I, I, F, I, I, I, P],
     "nls_poly_norm": [P, L, P, P, L, I, I, F, I, P],
-    "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, I, I, F, I, P],
+    "nls_attn_rows": [P, P, P, L, P, P, P, P, P, P, L, P, P, L, I, I, I, I, I, I, I, I, I, F, I, P],
     "nls_talk_plain": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, F, I, P, P, L, P, L, I, P],
     "nls_talk_decode": [P, L, P, P, P, I, I, P, P, I, I, I, I, I, I, F, I, P, P, L, P, L, P, L, P, P, P, I, I, I, P],
     "nls_talk_prefill": [P, L, P, P, P, I, I, P, I, I, I, I, I, I, F, I, P, P, L, P, L, P],
@@ -605,13 +605,17 @@ def attn_groups(H: int, G: int) -> int:
 
 
 def attn_rows(q, k, v, qn, kn, cs, pos, slot, qo, kc, vc, T: int, H: int, G: int, D: int, Dp: int, rot: int, eps: float, st: int,
-              V: Optional[int] = None, head_norm: bool = False):
+              V: Optional[int] = None, head_norm: bool = False, key_tiles: bool = False):
     """Norm over the whole q and k projections (qn, kn: weights or None), rotation of the first `rot` columns of each head (cs
-    None: none), then (head_norm) an RMS norm of each head of queries and keys on its own; queries to qo, keys and (as projected, V columns per head) values to the tokens' cache rows. q, k, v: f32
-    with one row stride."""
+    None: none), then (head_norm) an RMS norm of each head of queries and keys on its own; queries to qo, keys and (as projected, V
+    columns per head) values to the tokens' cache rows. q, k, v: f32 with one row stride. key_tiles: 16 slots of the key cache are a
+    tile [G][Dp / 8][16][8] (slots in whole tiles)."""
+    if key_tiles and kc.shape[0] % KEY_TILE:
+        raise ValueError("attn_rows: a key cache of whole tiles")
     _check(lib().nls_attn_rows(q.data_ptr(), k.data_ptr(), v.data_ptr(), q.stride(0), _p(qn), _p(kn), _p(cs),
                                pos.data_ptr(), slot.data_ptr(), qo.data_ptr(), qo.stride(0), kc.data_ptr(), vc.data_ptr(),
-                               kc.stride(0), T, H, G, D, D if V is None else V, Dp, rot, int(head_norm), eps,
+                               kc.stride(0), T, H, G, D, D if V is None else V, Dp, rot, int(head_norm),
+                               int(key_tiles), eps,
                                int(qo.dtype == torch.float32), st),
            "nls_attn_rows")
 
@@ -644,12 +648,14 @@ def gqa_prefill(q, kc, vc, xmap, blocks, nblocks: int, waves: int, gate, out, H:
 # Attention with mixed heads
 # ---------------------------------------------------------------------------
 
+KEY_TILE = 16                           # slots of a key tile
 TALK_WIDTHS = (32, 64, 128)             # padded head widths of the prompt kernel, which takes up to 32 heads
 TALK_SCRATCH = 256 << 20                # bytes of scores that a decode launch may hold
 
 
 class TalkPlan:
-    """Kernels and scratch sizes of an attention whose heads' softmax weights are mixed, heads padded to Dp columns."""
+    """Kernels and scratch sizes of an attention whose heads' softmax weights are mixed, heads padded to Dp columns. The MFMA kernels
+    read keys in tiles of 16 slots (attn_rows: key_tiles), the plain one rows."""
 
     def __init__(self, H: int, G: int, Dp: int, window: int, ctx: int, f32: bool, device, scale: float = 1.0):
         self.H, self.G, self.Dp, self.window = H, G, Dp, window

@@ -64,6 +64,15 @@ def paged(d, ctxs, G, D, V, Dp, nb, bs, spikes):
     return kc.view(-1, G * Dp).cuda(), vc.view(-1, G * Dp).cuda(), bt.int().cuda(), rows
 
 
+def key_tiles(kc, G):
+    """Rows of keys [slots][G * Dp] as tiles of 16 slots."""
+    return kc.view(kc.shape[0] // 16, 16, G, -1, 8).permute(0, 2, 3, 1, 4).reshape(kc.shape)
+
+
+def key_rows(kc, G):
+    return kc.view(kc.shape[0] // 16, G, -1, 16, 8).permute(0, 3, 1, 2, 4).reshape(kc.shape)
+
+
 def loud(q, scale):
     """A key whose score with q is 9."""
     q = q.double()
@@ -100,6 +109,8 @@ def test_decode_attention(K, dt, H, G, D, V, window):
                         for t, c in enumerate(ctxs)]) * gate.double().view(T, H, V)
     plan = K.TalkPlan(H, G, Dp, window, 480, dt == "f32", "cuda")
     assert plan.mfma == (dt == "bf16" and Dp <= 256)
+    if plan.mfma:
+        kc = key_tiles(kc, G)
     m = plan.matrix(talk)
     ld = H * V + 5
     for rep, rows_at_once in ((1, None), (1, 7), (1 + 1024 // (T * plan.groups), None)) if plan.mfma else ((1, None),):
@@ -149,7 +160,7 @@ def test_prompt_attention(K, H, G, D, V, waves, window):
     mask = {"size": window} if window else None
     plan = K.TalkPlan(H, G, Dp, window, 480, False, "cuda")
     assert plan.prefill
-    K.talk_prefill(plan, q.view(T, -1).cuda(), kc, vc, plan.matrix(talk), gate.cuda(), out, bt, bs, i32(blocks), len(blocks), waves, V,
+    K.talk_prefill(plan, q.view(T, -1).cuda(), key_tiles(kc, G), vc, plan.matrix(talk), gate.cuda(), out, bt, bs, i32(blocks), len(blocks), waves, V,
                    scale, st())
     o = out[:T].view(T, H, Dp).cpu()
     assert (out[T] == 7).all() and (o[..., V:] == 7).all()
@@ -178,14 +189,15 @@ def test_attention_far_pages(K, dt):
         want = torch.cat([O.attend(q[16 * t:16 * t + 16].double(), *rows[t], torch.arange(c - 16, c), scale, mask, talk.double())
                           for t, c in enumerate(ctxs)]) * gate.double().view(-1, H, D)
         part = [torch.zeros(s, device="cuda") for s in plan.scratch(T)[:3]] + [i32([0] * T * G)] if plan.mfma else ()
+        keys = key_tiles(kc, G) if plan.mfma else kc
         out = torch.zeros(16 * T, H * D, dtype=d, device="cuda")
-        K.talk_attention(plan, q[last].reshape(T, -1).cuda(), kc, vc, m, gate[last].cuda(), out, part, bt, bs, i32(list(range(T))),
+        K.talk_attention(plan, q[last].reshape(T, -1).cuda(), keys, vc, m, gate[last].cuda(), out, part, bt, bs, i32(list(range(T))),
                          i32(ctxs), T, D, scale, st())
         for t in range(T):
             assert relerr(out[t].view(H, D), want[last[t]]) < TOL[dt], (window, t)
         if plan.prefill:
             blocks = i32([(16 * t, 16, t, c - 16, 0, 0, 0, 0) for t, c in enumerate(ctxs)])
-            K.talk_prefill(plan, q.view(16 * T, -1).cuda(), kc, vc, m, gate.cuda(), out, bt, bs, blocks, T, 4, D, scale, st())
+            K.talk_prefill(plan, q.view(16 * T, -1).cuda(), keys, vc, m, gate.cuda(), out, bt, bs, blocks, T, 4, D, scale, st())
             for t in range(16 * T):
                 assert relerr(out[t].view(H, D), want[t]) < TOL[dt], (window, t)
 
@@ -194,12 +206,15 @@ def test_attention_far_pages(K, dt):
 @pytest.mark.parametrize("H,G,D,V", [(1, 1, 8, 4), (6, 2, 20, 36), (5, 5, 33, 21), (4, 2, 64, 128), (2, 1, 128, 7), (3, 1, 256, 256),
                                      (2, 2, 300, 16), (40, 8, 128, 128)])
 @pytest.mark.parametrize("rot", ["none", "some", "all"])
-def test_attention_rows(K, dt, H, G, D, V, rot):
-    """Rotation with a factor, then a norm per head of queries and keys; values as projected; rows without a cache row."""
+@pytest.mark.parametrize("tiles", [False, True])
+@pytest.mark.parametrize("T", [70, 300])
+def test_attention_rows(K, dt, H, G, D, V, rot, tiles, T):
+    """Rotation with a factor, then a norm per head of queries and keys; values as projected; rows without a cache row; keys in rows
+    and in tiles."""
     from nats_llm_studio_amd.models.stack import yarn
     from nats_llm_studio_amd.models.stack_config import RotScaling
     from nats_llm_studio_amd.ops import rope_table
-    d, T, eps = DT[dt], 70, 1e-3
+    d, eps, S = DT[dt], 1e-3, 304
     Dp, _ = K.head_pad(max(D, V))
     dims = {"none": 0, "some": D // 4 * 2, "all": D // 2 * 2}[rot]
     z = rnd(T, -(-((H + G) * D + G * V) // 4) * 4, seed=1).float()
@@ -210,12 +225,14 @@ def test_attention_rows(K, dt, H, G, D, V, rot):
     if dims:
         f, gain = yarn(700.0, dims, RotScaling(5.0, 100, 4.0, 0.5))
         cs = rope_table(1000, dims, 700.0, "cuda", f) * gain
-    slot = [(3 * t) % T if t != 5 else -1 for t in range(T)]
+    slot = [(5 * t) % 301 if t != 5 else -1 for t in range(T)]
     qo = torch.zeros(T, H * Dp, dtype=d, device="cuda")
-    kc, vc = (torch.full((T, G * Dp), 7.0, dtype=d, device="cuda") for _ in range(2))
+    kc, vc = (torch.full((S, G * Dp), 7.0, dtype=d, device="cuda") for _ in range(2))
     zc = z.cuda()
     K.attn_rows(zc, zc[:, H * D:], zc[:, (H + G) * D:], None, None, cs, pos.int().cuda(), i32(slot), qo, kc, vc, T, H, G, D, Dp, dims,
-                eps, st(), V=V, head_norm=True)
+                eps, st(), V=V, head_norm=True, key_tiles=tiles)
+    if tiles:
+        kc = key_rows(kc, G)
     # (columns 2 i, 2 i + 1 of a head are the pair that the plain implementation has at i, i + dims / 2)
     order = torch.cat([torch.arange(dims).view(-1, 2).T.reshape(-1), torch.arange(dims, D)])
 
@@ -225,11 +242,11 @@ def test_attention_rows(K, dt, H, G, D, V, rot):
     tol = 2e-6 if dt == "f32" else 5e-3
     live = [t for t in range(T) if slot[t] >= 0]
     s = torch.tensor(slot)[live]
-    qo, kc, vc = qo.cpu().view(T, H, Dp), kc.cpu().view(T, G, Dp), vc.cpu().view(T, G, Dp)
+    qo, kc, vc = qo.cpu().view(T, H, Dp), kc.cpu().view(S, G, Dp), vc.cpu().view(S, G, Dp)
     assert relerr(qo[..., :D][..., order], plain(z[:, :H * D], H)) < tol and (qo[..., D:] == 0).all()
     assert relerr(kc[s][..., :D][..., order], plain(z[:, H * D:(H + G) * D], G)[live]) < tol
     assert torch.equal(vc[s][..., :V], z[live, (H + G) * D:(H + G) * D + G * V].view(len(live), G, V).to(d))
-    assert (kc[slot[4]][..., D:] == 7).all() and (kc[3 * 5] == 7).all() and (vc[3 * 5] == 7).all()
+    assert (kc[slot[4]][..., D:] == 7).all() and (kc[5 * 5] == 7).all() and (vc[5 * 5] == 7).all()
 
 
 # ---------------------------------------------------------------- embedding, norms, feed-forwards
